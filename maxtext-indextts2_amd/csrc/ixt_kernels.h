@@ -1686,7 +1686,7 @@ __global__ __launch_bounds__(256) void k_attn_decode_w(DecAttnArgs a, int npairs
 //      key order, l in page order, P = bf16(e / l), PV page chains -> super-blocks of 4 pages in order -> super-blocks in order.
 //      Scores: the query operand of the chains is wave-uniform, so it comes by scalar loads (bf16 pairs expanded on the scalar unit, the
 //      next 32 d of both queries in flight while the current 32 are multiplied) -- no LDS traffic, no vector registers -- and two query
-//      vectors run as the two halves of packed f32 fmas.  Softmax: one wave per four query vectors, their phases interleaved.
+//      vectors run side by side.  Softmax: one wave per four query vectors, their phases interleaved.
 //      PV: lane = (page, 4 d), page chains for all NQ vectors in registers; the page sums meet in LDS, where the thread that owns
 //      (vector, d) adds them up four pages at a time and in order.  Rows of a tile that sit in different page groups (a tile across the
 //      border of two packed prompts) are worked off group by group.  grid = (nkv, ceil(R / TQ)), block 256;
@@ -1776,7 +1776,7 @@ __global__ __launch_bounds__(256, 2) void k_attn_tile(TileAttnArgs a) {
 #define IXT_QPTR(QV_) ((ixt_cq16p)(a.qbuf + ((size_t)min(r0 + (QV_) / GQ, a.R - 1) * g.nq + kvh * GQ + (QV_) % GQ) * HD))
 #pragma unroll
       for (int hh = 0; hh < NH; ++hh) {
-        ixt_f32x2 kf[HDH / 2];                           // (k[2c], k[2c+1]): one packed fma takes either half for both of its lanes (op_sel)
+        ixt_f32x2 kf[HDH / 2];                           // (k[2c], k[2c+1])
         if (j < kv_all) {
           const bf16_t* kp = a.kpages + kpage_off(g, prow[j / g.P], kvh, hh * (HDH / 8), j % g.P);
 #pragma unroll
@@ -1802,11 +1802,10 @@ __global__ __launch_bounds__(256, 2) void k_attn_tile(TileAttnArgs a) {
             __builtin_amdgcn_sched_barrier(0);                   // the loads are issued here, ahead of the 32 fmas that hide them
 #pragma unroll
             for (int k = 0; k < 16; ++k) {
-              // acc.x += qa[d] k[d], acc.y += qb[d] k[d] for d = 2k (first) and 2k + 1 (second): the key operand is one half of the
-              // register pair for both lanes of the packed fma -- the compiler would copy it into a second register instead
-              const ixt_f32x2 qlo = {bflo(ca[k]), bflo(cb[k])}, qhi = {bfhi(ca[k]), bfhi(cb[k])};
-              asm("v_pk_fma_f32 %0, %1, %2, %0 op_sel:[0,0,0] op_sel_hi:[1,0,1]" : "+v"(acc) : "s"(qlo), "v"(kf[part * 16 + k]));
-              asm("v_pk_fma_f32 %0, %1, %2, %0 op_sel:[0,1,0] op_sel_hi:[1,1,1]" : "+v"(acc) : "s"(qhi), "v"(kf[part * 16 + k]));
+              // acc.x += qa[d] k[d], acc.y += qb[d] k[d] for d = 2k (first) and 2k + 1 (second): the query operand is a scalar register
+              const ixt_f32x2 kd = kf[part * 16 + k];
+              acc.x = __builtin_fmaf(bflo(ca[k]), kd.x, acc.x); acc.y = __builtin_fmaf(bflo(cb[k]), kd.x, acc.y);
+              acc.x = __builtin_fmaf(bfhi(ca[k]), kd.y, acc.x); acc.y = __builtin_fmaf(bfhi(cb[k]), kd.y, acc.y);
             }
             ca = na; cb = nb;
           }
