@@ -30,6 +30,29 @@ typedef enum ixt_status {
 
 typedef enum ixt_dtype { IXT_BF16 = 0, IXT_F32 = 1 } ixt_dtype;
 
+/* One layer of an IXT_BLOCK_HYBRID decoder: a sequence mixer, then a feed-forward, each with a norm on its output only:
+ *   x <- x + norm1(mixer(x)), x <- x + norm2(ff(x)), norm(t) = t / sqrt(mean(t^2) + eps) (1 + w), the residual x in f32. */
+typedef struct ixt_layer {
+  int32_t mixer;                   /* IXT_MIX_LATENT_ATTENTION | IXT_MIX_GATED_DELTA */
+  int32_t weights_of;              /* -1, or the layer whose parameters this one shares (it keeps a cache or state of its own) */
+  int32_t heads, dim, vdim;        /* heads; query / key dims (latent attention: the unrotated ones) and value dims per head */
+  /* latent attention: keys and values are up-projections of one cached latent per token plus one rotated key part shared by all heads */
+  int32_t rot_dim, kv_rank;        /* rotated dims per head (even), latent size (<= 1024) */
+  int32_t window;                  /* position i sees i - window + 1 .. i; <= 0: everything up to i */
+  float rope_base, attn_scale;     /* neighbouring pairs (2 i, 2 i + 1) turn by p base^(-2 i / rot_dim); score factor */
+  /* gated delta rule with one decay per head and key channel: S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q */
+  int32_t kv_heads;                /* query / key heads (heads % kv_heads == 0) */
+  int32_t conv;                    /* taps of the causal convolutions in front of q, k, v */
+  int32_t decay_rank, gate_rank;   /* ranks of the decay and output-gate projections */
+  /* feed-forward */
+  int32_t ffn;                     /* IXT_FFN_NONE | IXT_FFN_DENSE | IXT_FFN_MOE */
+  int32_t ff;                      /* hidden size (MoE: of one expert) */
+  float glu_limit;                 /* y = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit) */
+  int32_t experts, top;            /* MoE: softmax over all router logits, the `top` largest, weights not renormalized */
+} ixt_layer;
+enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1 };
+enum { IXT_FFN_NONE = 0, IXT_FFN_DENSE = 1, IXT_FFN_MOE = 2 };
+
 /* Derived hyper-parameters of MaxText/pyconfig.py:551-644 that shape the path. */
 typedef struct ixt_config {
   int32_t vocab_size;              /* base.yml:430 */
@@ -93,9 +116,15 @@ typedef struct ixt_config {
    * (2 i, 2 i + 1), sin / cos are f32 and the result rounds to bf16 once; rope_use_scale applies the llama-3.1 frequency scaling
    * (factor 8, low / high frequency factors 1 / 4, original context 8192; :417-443).  0: the default RotaryEmbedding (:216-351).  llama2 block only. */
   int32_t rope_llama31, rope_use_scale;
+  /* IXT_BLOCK_HYBRID: the layers one by one (HOST array of num_decoder_layers entries, copied by ixt_create).  vocab_size, emb_dim, the page, slot and
+   * length fields and normalization_layer_epsilon are read as for the other blocks; head and MLP fields are not.  Any sizes: the library pads
+   * what its kernels need padded.  float32 != 0: activations, caches and products in f32 throughout (no matrix instruction of lower precision). */
+  const ixt_layer* layers;
+  float embedding_scale;           /* x = embedding[token] * scale */
+  int32_t float32;
 } ixt_config;
 
-enum { IXT_BLOCK_LLAMA2 = 0, IXT_BLOCK_GEMMA2 = 1, IXT_BLOCK_GEMMA3 = 2, IXT_BLOCK_MIXTRAL = 3 };
+enum { IXT_BLOCK_LLAMA2 = 0, IXT_BLOCK_GEMMA2 = 1, IXT_BLOCK_GEMMA3 = 2, IXT_BLOCK_MIXTRAL = 3, IXT_BLOCK_HYBRID = 4 };
 
 typedef struct ixt_ctx ixt_ctx;
 
@@ -115,6 +144,7 @@ int ixt_destroy(ixt_ctx* ctx);
  * pointer to a dense row-major array of `shape[ndim]`; IXT_F32 sources are rounded to bf16
  * (round-to-nearest-even) as linears.py:216 / embeddings.py:154 do at use.  Projection kernels are re-tiled into the
  * matrix-fragment order of the GEMM kernels while they are copied (the caller's array is not kept). */
+/* IXT_BLOCK_HYBRID: the names are `embed`, `final.norm`, `head` and `l<i>.{norm1,norm2}`, `l<i>.mix.*`, `l<i>.mlp.*`; linear weights are [out, in]. */
 int ixt_load_weight(ixt_ctx* ctx, const char* maxtext_path, const void* dev_ptr, int dtype, const int64_t* shape, int ndim, void* stream);
 /* 1 when every parameter of the configured model has been loaded. */
 int ixt_weights_complete(ixt_ctx* ctx);
@@ -158,6 +188,12 @@ int ixt_pages_status_async(ixt_ctx* ctx, int32_t* host_out4, void* stream);
  * reset (the affected step's numbers are then wrong -- the reference has no counterpart: its generate step, maxengine.py:838-935, is one XLA
  * program), 0 otherwise.  Synchronises `stream`; reset != 0 re-arms the exchange. */
 int ixt_exchange_status(ixt_ctx* ctx, int32_t* out1, int reset, void* stream);
+/* Recurrent layers (IXT_BLOCK_HYBRID): rows that did not start where their group's state stands (nor at position 0), or a second run of rows of one
+ * group in one call, are left idle and counted; out1 (HOST) = their number of runs since the last reset.  Synchronises `stream`. */
+int ixt_state_status(ixt_ctx* ctx, int32_t* out1, int reset, void* stream);
+/* IXT_BLOCK_HYBRID: every following pass also copies its residual stream after each layer to `dev` (device, f32 [layers][rows][emb]); NULL stops it.
+ * Passes replayed from a captured graph do not copy. */
+int ixt_set_residual_tap(ixt_ctx* ctx, float* dev, int64_t floats);
 /* Copy the seven PageState fields to HOST arrays (synchronises `stream`); the decode slots' groups only:
  * page_status[num_pages], page_map[max_slots*max_pages_per_group], num_pages_used[max_slots],
  * sequence_lengths[max_slots], active_page[max_slots], has_active_page[max_slots] (0/1),
@@ -184,7 +220,9 @@ int ixt_prefill_chunk(ixt_ctx* ctx, int slot, const int32_t* tokens_dev, int n_t
  * rows of different groups never see each other.  first_tokens_dev[j] = argmax of the logits of row logits_rows_dev[j] (the last row of
  * prompt j, :797-812), logits_dev f32[n_logits][vocab] may be NULL.  All arrays are device arrays.  max_len: the caller's bound on
  * position + 1 over the rows (the longest prompt end; it sizes the on-chip score rows of the tiled attention; <= 0: max_target_length);
- * a row at or beyond it is left idle and counted in ixt_pages_status()[3]. */
+ * a row at or beyond it is left idle and counted in ixt_pages_status()[3].
+ * Rows may be portions of prompts and single decoded tokens of running sequences in any mix (a group's rows are consecutive and start where its
+ * sequence stands).  IXT_BLOCK_HYBRID: n_logits may be anything from 0 to n_rows. */
 int ixt_prefill_rows(ixt_ctx* ctx, int n_rows, const int32_t* tokens_dev, const int32_t* row_group_dev, const int32_t* row_pos_dev, int max_len,
                      int n_logits, const int32_t* logits_rows_dev, int32_t* first_tokens_dev, float* logits_dev, void* stream);
 /* MaxEngine._generate_jit model step (maxengine.py:868-936) for all slots: row b = token tokens_dev[b] at

@@ -20,6 +20,13 @@ c_f64p = ctypes.POINTER(ctypes.c_double)
 vp = ctypes.c_void_p
 
 
+class IxtLayer(ctypes.Structure):
+  _fields_ = [(n, ctypes.c_int32) for n in ("mixer", "weights_of", "heads", "dim", "vdim", "rot_dim", "kv_rank", "window")] + [
+      ("rope_base", ctypes.c_float), ("attn_scale", ctypes.c_float)] + [
+      (n, ctypes.c_int32) for n in ("kv_heads", "conv", "decay_rank", "gate_rank", "ffn", "ff")] + [
+      ("glu_limit", ctypes.c_float), ("experts", ctypes.c_int32), ("top", ctypes.c_int32)]
+
+
 class IxtConfig(ctypes.Structure):
   _fields_ = [
       ("vocab_size", ctypes.c_int32), ("emb_dim", ctypes.c_int32), ("num_query_heads", ctypes.c_int32),
@@ -37,9 +44,10 @@ class IxtConfig(ctypes.Structure):
       ("num_experts", ctypes.c_int32), ("num_experts_per_tok", ctypes.c_int32),
       ("ep_rank", ctypes.c_int32), ("ep_size", ctypes.c_int32), ("fp8_weights", ctypes.c_int32),
       ("rope_llama31", ctypes.c_int32), ("rope_use_scale", ctypes.c_int32),
+      ("layers", ctypes.POINTER(IxtLayer)), ("embedding_scale", ctypes.c_float), ("float32", ctypes.c_int32),
   ]
 
-BLOCK_LLAMA2, BLOCK_GEMMA2, BLOCK_GEMMA3, BLOCK_MIXTRAL = 0, 1, 2, 3
+BLOCK_LLAMA2, BLOCK_GEMMA2, BLOCK_GEMMA3, BLOCK_MIXTRAL, BLOCK_HYBRID = 0, 1, 2, 3, 4
 
 
 # name -> (restype, argtypes); every symbol include/ixt.h declares
@@ -61,6 +69,8 @@ SIGNATURES = {
     "ixt_pages_status": (ctypes.c_int, [vp, c_i32p, ctypes.c_int, vp]),
     "ixt_pages_status_async": (ctypes.c_int, [vp, vp, vp]),
     "ixt_exchange_status": (ctypes.c_int, [vp, c_i32p, ctypes.c_int, vp]),
+    "ixt_state_status": (ctypes.c_int, [vp, c_i32p, ctypes.c_int, vp]),
+    "ixt_set_residual_tap": (ctypes.c_int, [vp, vp, ctypes.c_int64]),
     "ixt_prefill_prompt_logp": (ctypes.c_int, [vp, vp, ctypes.c_int, vp, vp]),
     "ixt_build_id": (ctypes.c_char_p, []),
     "ixt_prefill_rows": (ctypes.c_int, [vp, ctypes.c_int, vp, vp, vp, ctypes.c_int, ctypes.c_int, vp, vp, vp, vp]),

@@ -1,0 +1,152 @@
+"""Model folders (config.json + model.safetensors) -> the engine's configuration keys.
+
+`read_model_dir` looks the folder's `architecture` up in ARCHITECTURES; a reader turns config.json (and, for sizes that only a tensor's shape
+tells, the safetensors header) into config keys: vocabulary and width, `decoder_block: hybrid` and one HybridLayer per layer (include/ixt.h,
+ixt_layer).  A new design of known mechanisms needs a reader here and nothing else."""
+from __future__ import annotations
+
+import dataclasses
+import json
+import os
+import struct
+from typing import Any, Callable, Dict, Mapping, Tuple
+
+MIX_LATENT_ATTENTION, MIX_GATED_DELTA = 0, 1
+FFN_NONE, FFN_DENSE, FFN_MOE = 0, 1, 2
+
+
+@dataclasses.dataclass(frozen=True)
+class HybridLayer:
+  """One layer of a hybrid decoder; the fields of ixt_layer."""
+  mixer: int
+  weights_of: int = -1
+  heads: int = 1
+  dim: int = 1
+  vdim: int = 1
+  rot_dim: int = 0
+  kv_rank: int = 0
+  window: int = 0
+  rope_base: float = 10000.0
+  attn_scale: float = 1.0
+  kv_heads: int = 1
+  conv: int = 1
+  decay_rank: int = 1
+  gate_rank: int = 1
+  ffn: int = FFN_NONE
+  ff: int = 0
+  glu_limit: float = 0.0
+  experts: int = 0
+  top: int = 0
+
+
+Shapes = Mapping[str, Tuple[int, ...]]
+
+
+def safetensors_shapes(path: str) -> Dict[str, Tuple[int, ...]]:
+  """{tensor name: shape} from the header of a safetensors file (8-byte little-endian length, then JSON)."""
+  with open(path, "rb") as f:
+    (n,) = struct.unpack("<Q", f.read(8))
+    header = json.loads(f.read(n))
+  return {k: tuple(v["shape"]) for k, v in header.items() if k != "__metadata__"}
+
+
+def _vilepel_feed_forward(mlp: Any) -> Dict[str, Any]:
+  if mlp is None:
+    return {"ffn": FFN_NONE}
+  if mlp["kind"] == "dense":
+    return {"ffn": FFN_DENSE, "ff": int(mlp["ff"]), "glu_limit": float(mlp["limit"])}
+  if mlp["kind"] == "moe":
+    return {"ffn": FFN_MOE, "ff": int(mlp["expert"]["ff"]), "glu_limit": float(mlp["expert"]["limit"]),
+            "experts": int(mlp["router"]["experts"]), "top": int(mlp["router"]["top"])}
+  raise ValueError(f"Vilepel: feed-forward kind {mlp['kind']!r}")
+
+
+def _vilepel_latent(m: Mapping[str, Any], name: Callable[[str], str], shapes: Shapes) -> Dict[str, Any]:
+  del name, shapes
+  rot = m["rot"]
+  if int(rot["dims"]) != int(m["rot_dim"]):
+    raise ValueError(f"Vilepel: rot.dims ({rot['dims']}) must equal rot_dim ({m['rot_dim']})")
+  return {"mixer": MIX_LATENT_ATTENTION, "heads": int(m["heads"]), "dim": int(m["dim"]), "vdim": int(m["vdim"]), "rot_dim": int(m["rot_dim"]),
+          "kv_rank": int(m["kv_rank"]), "window": int((m.get("mask") or {}).get("size") or 0), "rope_base": float(rot["base"]), "attn_scale": float(m["scale"])}
+
+
+def _vilepel_delta(m: Mapping[str, Any], name: Callable[[str], str], shapes: Shapes) -> Dict[str, Any]:
+  # config.json does not give the two ranks: a1 is [decay rank, width], g1 [gate rank, width].  Without weights (synthetic ones): the key dims.
+  rank = lambda t: int(shapes[name(t)][0]) if name(t) in shapes else int(m["dim"])
+  return {"mixer": MIX_GATED_DELTA, "heads": int(m["heads"]), "kv_heads": int(m["kv_heads"]), "dim": int(m["dim"]), "vdim": int(m["vdim"]), "conv": int(m["conv"]),
+          "decay_rank": rank("a1"), "gate_rank": rank("g1")}
+
+
+_VILEPEL_MIXERS = {"latent_attention": _vilepel_latent, "channel_delta": _vilepel_delta}
+
+
+def vilepel_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
+  """Vilepel: layers of latent attention and of a gated delta rule with per-channel decay in any order, RMS norms (stored around zero) on the
+  sublayers' outputs, clamped gated units (dense or routed)."""
+  layers = []
+  for i, entry in enumerate(cfg["layers"]):
+    src = entry.get("weights_of")
+    src = -1 if src is None else int(src)
+    if entry["type"] not in _VILEPEL_MIXERS:
+      raise ValueError(f"Vilepel: layer {i} has type {entry['type']!r}")
+    own = i if src < 0 else src
+    spec = _VILEPEL_MIXERS[entry["type"]](entry["mixer"], lambda t, own=own: f"l{own}.mix.{t}", shapes)
+    layers.append(HybridLayer(weights_of=src, **spec, **_vilepel_feed_forward(entry.get("mlp"))))
+  return {
+      "decoder_block": "hybrid",
+      "vocab_size": int(cfg["vocab"]),
+      "base_emb_dim": int(cfg["width"]),
+      "base_num_decoder_layers": len(layers),
+      "normalization_layer_epsilon": float(cfg["norm"]["eps"]),
+      "embedding_scale": float(cfg["embedding"]["scale"]),
+      "hybrid_layers": tuple(layers),
+  }
+
+
+ARCHITECTURES: Dict[str, Callable[[Mapping[str, Any], Shapes], Dict[str, Any]]] = {
+    "Vilepel": vilepel_keys,
+}
+
+
+def read_model_dir(path: str) -> Dict[str, Any]:
+  """Config keys of the model in `path`; `load_parameters_path` names its weights when they are there."""
+  with open(os.path.join(path, "config.json"), "r", encoding="utf-8") as f:
+    cfg = json.load(f)
+  name = cfg.get("architecture")
+  if name not in ARCHITECTURES:
+    raise ValueError(f"{path}: architecture {name!r} is not built (built: {sorted(ARCHITECTURES)})")
+  weights = os.path.join(path, "model.safetensors")
+  have = os.path.isfile(weights)
+  keys = ARCHITECTURES[name](cfg, safetensors_shapes(weights) if have else {})
+  if have:
+    keys["load_parameters_path"] = weights
+  return keys
+
+
+def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
+  """{tensor name: shape} of a hybrid decoder; linear weights are [out, in]."""
+  E, V = int(config.emb_dim), int(config.vocab_size)
+  out: Dict[str, Tuple[int, ...]] = {"embed": (V, E), "final.norm": (E,), "head": (V, E)}
+  for i, l in enumerate(config.hybrid_layers):
+    if l.weights_of >= 0:
+      continue
+    p = f"l{i}."
+    out[p + "norm1"] = (E,)
+    if l.mixer == MIX_LATENT_ATTENTION:
+      out.update({p + "mix.q": (l.heads * (l.dim + l.rot_dim), E), p + "mix.dkv": (l.kv_rank + l.rot_dim, E), p + "mix.dkv.norm": (l.kv_rank,),
+                  p + "mix.uk": (l.heads * l.dim, l.kv_rank), p + "mix.uv": (l.heads * l.vdim, l.kv_rank), p + "mix.o": (E, l.heads * l.vdim)})
+    else:
+      kq, v = l.kv_heads * l.dim, l.heads * l.vdim
+      for t, n in (("q", kq), ("k", kq), ("v", v)):
+        out[p + f"mix.{t}"], out[p + f"mix.{t}.conv"] = (n, E), (n, l.conv)
+      out.update({p + "mix.b": (l.heads, E), p + "mix.A_log": (l.heads,), p + "mix.norm": (l.vdim,), p + "mix.a1": (l.decay_rank, E),
+                  p + "mix.a2": (l.heads * l.dim, l.decay_rank), p + "mix.dt_bias": (l.heads * l.dim,), p + "mix.g1": (l.gate_rank, E),
+                  p + "mix.g2": (v, l.gate_rank), p + "mix.o": (E, v)})
+    if l.ffn == FFN_NONE:
+      continue
+    out[p + "norm2"] = (E,)
+    for q in ([f"mlp.e{e}." for e in range(l.experts)] if l.ffn == FFN_MOE else ["mlp."]):
+      out[p + q + "gate"], out[p + q + "up"], out[p + q + "down"] = (l.ff, E), (l.ff, E), (E, l.ff)
+    if l.ffn == FFN_MOE:
+      out[p + "mlp.router"] = (l.experts, E)
+  return out

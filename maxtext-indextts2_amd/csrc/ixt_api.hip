@@ -6,6 +6,7 @@
 #include "ixt_moe_kernels.h"
 #include "ixt_small.h"
 #include "ixt_fp8.h"
+#include "ixt_hybrid_kernels.h"
 
 #include <hip/hip_runtime.h>
 #include <math.h>
@@ -15,6 +16,7 @@
 #include <string.h>
 
 #include <algorithm>
+#include <functional>
 #include <map>
 #include <string>
 #include <vector>
@@ -52,8 +54,21 @@ struct GraphEntry {
   hipGraphExec_t exec;
 };
 
+struct HybridModel;           // IXT_BLOCK_HYBRID (ixt_hybrid.h)
+static int hybrid_check(const ixt_config& c);
+static int hybrid_init(ixt_ctx* c);
+static int hybrid_load_weight(ixt_ctx* c, const std::string& name, const void* src, int dtype, const int64_t* shape, int ndim, hipStream_t st);
+static bool hybrid_complete(const ixt_ctx* c);
+static void hybrid_free(ixt_ctx* c);
+static HybridModel* hybrid_new();
+static int hybrid_copy_group(ixt_ctx* c, int src, int dst, int npages, hipStream_t st);
+static int hybrid_prompt_logits(ixt_ctx* c, int row0, int n, hipStream_t st);
+static int forward_rows_hybrid(ixt_ctx* c, int R, const int32_t* tokens, int len_hint, int lrow0, int nl, const int32_t* lrows, int32_t* argmax_out, float* logits_out, bool decode,
+                               hipStream_t st);
+
 struct ixt_ctx {
   ixt_config cfg;
+  HybridModel* hy = nullptr;
   int E, Q, KV, D, F, V, L, P, B, Rmax, NQKV, QN, KN, Tmax, mpg, nsb_max, GQ;
   int G = 0, S = 0;            // page groups = B decode slots + S staging groups of packed prefill
   int NLmax = 1;               // rows that can be unembedded in one call (decode slots / prompts of a packed prefill)
@@ -247,11 +262,16 @@ static int sdot_set_attributes();
 extern "C" int ixt_create(const ixt_config* cfg, ixt_ctx** out) {
   if (!cfg || !out) return set_err(IXT_ERR_INVALID, "null argument");
   const ixt_config& c = *cfg;
+  const bool hybrid = c.decoder_block == IXT_BLOCK_HYBRID;
   const bool gemma3 = c.decoder_block == IXT_BLOCK_GEMMA3;
   const bool gemma = c.decoder_block == IXT_BLOCK_GEMMA2 || gemma3;
+  const bool moe = c.decoder_block == IXT_BLOCK_MIXTRAL;
+  int gq = 1;
+  if (hybrid) {
+    TRY(hybrid_check(c));
+  } else {
   if (c.head_dim != 64 && c.head_dim != 128 && !(c.head_dim == 256 && gemma))
     return set_err(IXT_ERR_UNSUPPORTED, "head_dim %d (64 and 128 built; 256 for decoder_block gemma2 / gemma3)", c.head_dim);
-  const bool moe = c.decoder_block == IXT_BLOCK_MIXTRAL;
   if (c.decoder_block != IXT_BLOCK_LLAMA2 && !gemma && !moe) return set_err(IXT_ERR_UNSUPPORTED, "decoder_block %d (llama2, gemma2, gemma3 and mixtral built)", c.decoder_block);
   if (moe && (c.num_experts < 1 || c.num_experts > IXT_MOE_MAX_EXPERTS || c.num_experts_per_tok < 1 || c.num_experts_per_tok > IXT_MOE_MAX_TOPK ||
               c.num_experts_per_tok > c.num_experts))
@@ -269,11 +289,12 @@ extern "C" int ixt_create(const ixt_config* cfg, ixt_ctx** out) {
   if (c.emb_dim % IXT_KALIGN || c.mlp_dim % IXT_KALIGN || (c.num_query_heads * c.head_dim) % IXT_KALIGN)
     return set_err(IXT_ERR_UNSUPPORTED, "emb_dim, mlp_dim and num_query_heads*head_dim must be multiples of %d", IXT_KALIGN);
   if (c.num_kv_heads <= 0 || c.num_query_heads % c.num_kv_heads) return set_err(IXT_ERR_INVALID, "num_query_heads %% num_kv_heads != 0");
-  const int gq = c.num_query_heads / c.num_kv_heads;
+  gq = c.num_query_heads / c.num_kv_heads;
   if (gq != 1 && gq != 2 && gq != 4) return set_err(IXT_ERR_UNSUPPORTED, "query heads per kv head = %d (1, 2, 4 built)", gq);
+  if (c.vocab_size % 16) return set_err(IXT_ERR_UNSUPPORTED, "vocab_size must be a multiple of 16");
+  }
   if (!is_pow2(c.pagedattn_tokens_per_page) || c.pagedattn_tokens_per_page < 8 || c.pagedattn_tokens_per_page > 64)
     return set_err(IXT_ERR_UNSUPPORTED, "pagedattn_tokens_per_page must be a power of two in [8, 64]");
-  if (c.vocab_size % 16) return set_err(IXT_ERR_UNSUPPORTED, "vocab_size must be a multiple of 16");
   if (c.staging_groups < 0 || c.max_packed_rows < 0) return set_err(IXT_ERR_INVALID, "staging_groups / max_packed_rows must be >= 0");
   if (c.max_slots + c.staging_groups > IXT_MAX_GROUPS || c.pagedattn_max_pages_per_group > IXT_MAX_GROUPS)
     return set_err(IXT_ERR_UNSUPPORTED, "more than %d page groups or pages per group", IXT_MAX_GROUPS);
@@ -300,16 +321,18 @@ extern "C" int ixt_create(const ixt_config* cfg, ixt_ctx** out) {
   x->S = c.staging_groups; x->G = x->B + x->S;
   x->NLmax = x->B > x->S ? x->B : x->S;
   if (x->NLmax < 1) x->NLmax = 1;
+  if (hybrid) { x->L = 0; x->Q = x->KV = 1; x->D = 0; x->F = 0; x->QN = x->KN = x->NQKV = 0; }
   const int E = x->E, F = x->F, V = x->V, L = x->L, R = x->Rmax;
   *out = nullptr;
   int rc = IXT_OK;
   auto fail = [&](int code) { ixt_destroy(x); return code; };
 #define A(expr) do { rc = (expr); if (rc != IXT_OK) return fail(rc); } while (0)
+  x->loaded.assign(L + 1, 0);
+  if (!hybrid) {
   A(dmalloc(x, &x->embedding, (size_t)V * E));
   A(dmalloc(x, &x->final_norm, (size_t)E));
   A(dmalloc(x, &x->logits_w, (size_t)E * V));
   x->layers.resize(L);
-  x->loaded.assign(L + 1, 0);
   for (int i = 0; i < L; ++i) {
     LayerW& w = x->layers[i];
     A(dmalloc(x, &w.ln1, (size_t)E));
@@ -391,6 +414,7 @@ extern "C" int ixt_create(const ixt_config* cfg, ixt_ctx** out) {
   }
   if (!zero_ok)
     return fail(set_err(IXT_ERR_HIP, "page pool memset failed"));
+  }
   // page state
   PageStateDev& s = x->ps;
   s.num_pages = c.pagedattn_num_pages; s.groups = x->G; s.decode_groups = x->B; s.mpg = x->mpg; s.P = x->P;
@@ -403,6 +427,12 @@ extern "C" int ixt_create(const ixt_config* cfg, ixt_ctx** out) {
   A(dmalloc(x, &s.active_page, (size_t)s.groups));
   A(dmalloc(x, &s.has_active_page, (size_t)s.groups));
   A(dmalloc(x, &s.active_page_position, (size_t)s.groups));
+  if (hybrid) {
+    x->hy = hybrid_new();
+    A(dmalloc(x, &x->split_cnt, (size_t)128));
+    HIPCHK(hipMemset(x->split_cnt, 0, sizeof(int32_t) * 128));
+    A(hybrid_init(x));
+  } else {
   // workspaces
   A(dmalloc(x, &x->h_a, (size_t)R * E));
   A(dmalloc(x, &x->h_b, (size_t)R * E));
@@ -478,6 +508,7 @@ extern "C" int ixt_create(const ixt_config* cfg, ixt_ctx** out) {
       }
     }
   }
+  }
   A(dmalloc(x, &x->row_slot, (size_t)R));
   A(dmalloc(x, &x->row_pos, (size_t)R));
   A(dmalloc(x, &x->row_active, (size_t)R));
@@ -486,7 +517,7 @@ extern "C" int ixt_create(const ixt_config* cfg, ixt_ctx** out) {
   A(dmalloc(x, &x->lrows, (size_t)x->NLmax));
   A(dmalloc(x, &x->kptrs_d, (size_t)L));
   A(dmalloc(x, &x->vptrs_d, (size_t)L));
-  if (hipMemcpy(x->kptrs_d, x->kpages_l.data(), sizeof(bf16_t*) * L, hipMemcpyHostToDevice) != hipSuccess ||
+  if (L > 0) if (hipMemcpy(x->kptrs_d, x->kpages_l.data(), sizeof(bf16_t*) * L, hipMemcpyHostToDevice) != hipSuccess ||
       hipMemcpy(x->vptrs_d, x->vpages_l.data(), sizeof(bf16_t*) * L, hipMemcpyHostToDevice) != hipSuccess)
     return fail(set_err(IXT_ERR_HIP, "page pointer upload failed"));
 #undef A
@@ -507,6 +538,7 @@ extern "C" int ixt_destroy(ixt_ctx* c) {
   for (auto& t : c->tpairs) { (void)hipEventDestroy(t.a); (void)hipEventDestroy(t.b); }
   for (void* p : c->allocs) (void)hipFree(p);
   if (c->wt_op) (void)hipFree(c->wt_op);
+  hybrid_free(c);
   delete c;
   return IXT_OK;
 }
@@ -539,6 +571,7 @@ extern "C" int ixt_load_weight(ixt_ctx* c, const char* path, const void* dev_ptr
   hipStream_t st = (hipStream_t)stream;
   c->fp8_ready = false;          // the e4m3 twins are made from the bf16 copies on the next forward pass
   std::string p(path);
+  if (c->hy) return hybrid_load_weight(c, p, dev_ptr, dtype, shape, ndim, st);
   if (p.rfind("params/", 0) == 0) p = p.substr(7);
   int64_t numel = 1;
   for (int i = 0; i < ndim; ++i) numel *= shape[i];
@@ -638,6 +671,7 @@ extern "C" int ixt_load_weight(ixt_ctx* c, const char* path, const void* dev_ptr
 
 extern "C" int ixt_weights_complete(ixt_ctx* c) {
   if (!c) return 0;
+  if (c->hy) return hybrid_complete(c) ? 1 : 0;
   for (int i = 0; i < c->L; ++i) {
     uint32_t want = (1u << W_PER_LAYER) - 1;
     if (c->layers[i].pan) want |= 1u << W_PAN;
@@ -716,6 +750,7 @@ extern "C" int ixt_pages_move(ixt_ctx* c, int src_group, int dst_slot, void* str
   if (src_group == dst_slot) return IXT_OK;
   hipLaunchKernelGGL(k_pages_move, dim3(1), dim3(64), 0, (hipStream_t)stream, c->ps, src_group, dst_slot);
   LAUNCHCHK();
+  if (c->hy) return hybrid_copy_group(c, src_group, dst_slot, 0, (hipStream_t)stream);   // recurrent state does not live in pages
   return IXT_OK;
 }
 extern "C" int ixt_pages_copy(ixt_ctx* c, int src_group, int dst_slot, int length, void* stream) {
@@ -727,6 +762,7 @@ extern "C" int ixt_pages_copy(ixt_ctx* c, int src_group, int dst_slot, int lengt
   hipStream_t st = (hipStream_t)stream;
   hipLaunchKernelGGL(k_pages_reserve, dim3(1), dim3(64), 0, st, c->ps, dst_slot, length, 0);
   const int npages = (length + c->P - 1) / c->P;
+  if (c->hy) return hybrid_copy_group(c, src_group, dst_slot, npages, st);
   hipLaunchKernelGGL(k_pages_copy, dim3(npages, c->L), dim3(256), 0, st, c->ps, src_group, dst_slot, c->kptrs_d, c->vptrs_d,
                      (size_t)c->KV * c->P * c->D);
   LAUNCHCHK();
@@ -1639,7 +1675,7 @@ static int moe_experts_routed(ixt_ctx* c, const LayerW& w, const bf16_t* x, cons
       const int ti = timing_begin(c, st, (double)K * N * 2.0 * c->NEL + (double)rows_g * K * 2.0 + out_bytes);
       dim3 grid((((nwaves + 3) / 4 + 7) / 8) * 8 * zblocks, 1, 1);
       hipLaunchKernelGGL(kern, grid, dim3(256), (size_t)64 * 1024, st, reinterpret_cast<const u32x4*>(xin), reinterpret_cast<const u32x4*>(wbase), K, N, rows_g, out, nwaves, zblocks,
-                         c->moe_rbexp, wstride);
+                         c->moe_rbexp, wstride, 0, 0.0f);
       timing_end(c, st, ti);
     };
     if ((size_t)rows_g * E > c->part_floats) return set_err(IXT_ERR_INVALID, "moe: output workspace too small");
@@ -1772,6 +1808,7 @@ static int forward_rows_small(ixt_ctx* c, int R, const int32_t* tokens, int len_
 static int forward_rows(ixt_ctx* c, int R, const int32_t* tokens, int len_hint, int lrow0, int nl, const int32_t* lrows, int32_t* argmax_out,
                         float* logits_out, bool decode, hipStream_t st) {
   if (!ixt_weights_complete(c)) return set_err(IXT_ERR_NOT_LOADED, "weights incomplete");
+  if (c->hy) return forward_rows_hybrid(c, R, tokens, len_hint, lrow0, nl, lrows, argmax_out, logits_out, decode, st);
   TRY(fp8_prepare(c, st));
   if (c->gemma) return forward_rows_gemma2(c, R, tokens, len_hint, lrow0, nl, lrows, argmax_out, logits_out, st);
   if (c->moe && c->NEL != c->NE) return set_err(IXT_ERR_UNSUPPORTED, "this context holds experts %d..%d of %d: the fused engine needs every expert (expert-parallel contexts serve ixt_op_moe_route / ixt_op_moe_experts)", c->E0, c->E0 + c->NEL - 1, c->NE);
@@ -1944,7 +1981,7 @@ extern "C" int ixt_prefill_chunk(ixt_ctx* c, int slot, const int32_t* tokens_dev
 // 256-row chunk at V = 264 192 are 270 MB: they never exist as a whole).
 extern "C" int ixt_prefill_prompt_logp(ixt_ctx* c, const int32_t* tokens_dev, int n_tokens, float* prompt_logp_dev, void* stream) {
   if (!c || !tokens_dev || !prompt_logp_dev) return set_err(IXT_ERR_INVALID, "null argument");
-  if (c->h_final == nullptr || n_tokens <= 0 || n_tokens != c->h_final_rows)
+  if ((c->h_final == nullptr && c->hy == nullptr) || n_tokens <= 0 || n_tokens != c->h_final_rows)
     return set_err(IXT_ERR_INVALID, "prompt log-probabilities: call right after ixt_prefill_chunk with the same n_tokens (%d rows are held)", c->h_final_rows);
   hipStream_t st = (hipStream_t)stream;
   if (c->plogits == nullptr) {
@@ -1954,6 +1991,11 @@ extern "C" int ixt_prefill_prompt_logp(ixt_ctx* c, const int32_t* tokens_dev, in
   const ixt_config& cf = c->cfg;
   for (int row0 = 0; row0 < n_tokens; row0 += c->NLmax) {
     const int g = n_tokens - row0 < c->NLmax ? n_tokens - row0 : c->NLmax;
+    if (c->hy) {
+      TRY(hybrid_prompt_logits(c, row0, g, st));
+      TRY(ixt_op_logprob(c, c->plogits, g, tokens_dev + row0, prompt_logp_dev + row0, stream));
+      continue;
+    }
     TRY(launch_rownorm(c, 2, g, nullptr, nullptr, c->h_final + (size_t)row0 * c->E, nullptr, c->final_norm, c->xn, st));
     TRY(launch_unembed(c, c->xn, g, c->plogits, c->pargmax, st));
     if (c->gemma) {   // decoders.py:552-565
@@ -1968,14 +2010,15 @@ extern "C" int ixt_prefill_prompt_logp(ixt_ctx* c, const int32_t* tokens_dev, in
 
 extern "C" int ixt_prefill_rows(ixt_ctx* c, int n_rows, const int32_t* tokens_dev, const int32_t* row_group_dev, const int32_t* row_pos_dev, int max_len,
                                 int n_logits, const int32_t* logits_rows_dev, int32_t* first_tokens_dev, float* logits_dev, void* stream) {
-  if (!c || !tokens_dev || !row_group_dev || !row_pos_dev || !logits_rows_dev || !first_tokens_dev) return set_err(IXT_ERR_INVALID, "null argument");
+  if (!c || !tokens_dev || !row_group_dev || !row_pos_dev || (n_logits > 0 && (!logits_rows_dev || !first_tokens_dev))) return set_err(IXT_ERR_INVALID, "null argument");
   if (n_rows <= 0 || n_rows > c->Rmax) return set_err(IXT_ERR_RANGE, "packed prefill of %d rows (max %d: ixt_config.max_packed_rows)", n_rows, c->Rmax);
-  if (n_logits <= 0 || n_logits > c->NLmax || n_logits > n_rows) return set_err(IXT_ERR_RANGE, "packed prefill with %d prompts (max %d)", n_logits, c->NLmax);
+  if (c->hy ? (n_logits < 0 || n_logits > n_rows) : (n_logits <= 0 || n_logits > c->NLmax || n_logits > n_rows)) return set_err(IXT_ERR_RANGE, "packed prefill with %d prompts (max %d)", n_logits, c->NLmax);
   if (max_len <= 0 || max_len > c->Tmax) max_len = c->Tmax;
   hipStream_t st = (hipStream_t)stream;
   hipLaunchKernelGGL(k_rows_packed, dim3((n_rows + 255) / 256), dim3(256), 0, st, c->row_slot, c->row_pos, c->row_active, row_group_dev, row_pos_dev, n_rows,
                      c->ps.num_pages_used, c->P, c->G, c->Tmax, max_len, c->ps.status);
   LAUNCHCHK();
+  if (c->hy) return forward_rows(c, n_rows, tokens_dev, max_len, 0, n_logits, logits_rows_dev, first_tokens_dev, logits_dev, false, st);
   HIPCHK(hipMemcpyAsync(c->lrows, logits_rows_dev, sizeof(int32_t) * n_logits, hipMemcpyDeviceToDevice, st));
   return forward_rows(c, n_rows, tokens_dev, max_len, 0, n_logits, c->lrows, first_tokens_dev, logits_dev, false, st);
 }
@@ -2043,6 +2086,8 @@ extern "C" int ixt_generate(ixt_ctx* c, int32_t* tokens_dev, int32_t* next_pos_d
   HIPCHK(hipGraphLaunch(it->second.exec, st));
   return IXT_OK;
 }
+
+#include "ixt_hybrid.h"
 
 // --------------------------------------------------------------------------------------- op-level
 __global__ void k_sum_slices(const float* part, int slices, size_t stride, float* out, size_t n) {
@@ -2170,6 +2215,7 @@ extern "C" int ixt_op_rmsnorm(ixt_ctx* c, const uint16_t* x, const uint16_t* sca
 
 extern "C" int ixt_op_rope(ixt_ctx* c, uint16_t* x, const int32_t* pos, int R, int nheads, void* stream) {
   if (!c || !x || !pos || R <= 0) return set_err(IXT_ERR_INVALID, "bad argument");
+  if (c->hy) return set_err(IXT_ERR_UNSUPPORTED, "a hybrid decoder's layers have rotation tables of their own");
   hipLaunchKernelGGL(k_rope, dim3(R, nheads), dim3(c->D / 2), 0, (hipStream_t)stream, x, pos, c->rope_sin, c->rope_cos, nheads, c->D, c->rope32 ? 1 : 0);
   LAUNCHCHK();
   return IXT_OK;

@@ -108,6 +108,12 @@ __device__ __forceinline__ bf16_t ixt_geglu(float a, float b) {
   return f2bf(g * b);
 }
 
+// clamped gated unit: g = min(a, limit), u = clamp(b, -limit, limit), g sigmoid(1.702 g) (u + 1), in f32
+__device__ __forceinline__ float ixt_glu_clamped(float a, float b, float limit) {
+  const float g = fminf(a, limit), u = fminf(fmaxf(b, -limit), limit);
+  return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
+
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
 // agent-scope (L1-bypassing) accesses for state one wave re-reads after writing it

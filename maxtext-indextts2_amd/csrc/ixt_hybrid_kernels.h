@@ -1,0 +1,1008 @@
+// ixt_hybrid_kernels.h -- kernels of decoders whose layers are listed one by one (ixt_config.layers): each layer has a sequence mixer (latent
+// attention over a paged latent cache, or a gated delta rule with a recurrent state per page group), a feed-forward (a clamped gated unit, dense or
+// as a routed mixture) and norms on the sublayers' outputs only.
+//
+// Every kernel is a template over T, the storage of activations and cached keys: bf16_t (activations in the dot kernels' fragment order, xidx) or
+// float (row-major; the 32-bit mode).  The residual stream, norms, rotations, scores, routers and the recurrence are f32 in both.
+//
+//   act(T)      an activation matrix [rows][Kp], Kp a multiple of 128 with zeros behind the real columns, in the order the dot of T reads
+//   "slices"    a dot's output: f32 [slices][rows][ncols], to be added up by the reader
+#pragma once
+#include "ixt_kernels.h"
+#include "ixt_moe_kernels.h"
+
+// ---------------------------------------------------------------------------------------------------- activation storage
+__device__ __forceinline__ void act_store1(bf16_t* b, int r, int k, int Kp, float v) { b[xidx(r, k, Kp)] = f2bf(v); }
+__device__ __forceinline__ void act_store1(float* b, int r, int k, int Kp, float v) { b[(size_t)r * Kp + k] = v; }
+__device__ __forceinline__ void act_store4(bf16_t* b, int r, int k0, int Kp, const float* v) {      // k0 % 4 == 0
+  uint2 o;
+  o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3]));
+  *reinterpret_cast<uint2*>(b + xidx(r, k0, Kp)) = o;
+}
+__device__ __forceinline__ void act_store4(float* b, int r, int k0, int Kp, const float* v) {
+  *reinterpret_cast<float4*>(b + (size_t)r * Kp + k0) = make_float4(v[0], v[1], v[2], v[3]);
+}
+__device__ __forceinline__ void act_store8(bf16_t* b, int r, int k0, int Kp, const float* v) {      // k0 % 8 == 0
+  u32x4 o;
+  o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3])); o.z = pack2(f2bf(v[4]), f2bf(v[5])); o.w = pack2(f2bf(v[6]), f2bf(v[7]));
+  *reinterpret_cast<u32x4*>(b + xidx(r, k0, Kp)) = o;
+}
+__device__ __forceinline__ void act_store8(float* b, int r, int k0, int Kp, const float* v) {
+  act_store4(b, r, k0, Kp, v); act_store4(b, r, k0 + 4, Kp, v + 4);
+}
+__device__ __forceinline__ float to_f(bf16_t v) { return bf2f(v); }
+__device__ __forceinline__ float to_f(float v) { return v; }
+template <typename T> __device__ __forceinline__ T from_f(float v);
+template <> __device__ __forceinline__ bf16_t from_f<bf16_t>(float v) { return f2bf(v); }
+template <> __device__ __forceinline__ float from_f<float>(float v) { return v; }
+
+struct Slices {             // a dot's output
+  const float* p; int n; size_t stride; int ncols;
+  __device__ __forceinline__ float at(int r, int c) const {
+    const float* q = p + (size_t)r * ncols + c;
+    float t = q[0];
+    for (int s = 1; s < n; ++s) t += q[(size_t)s * stride];
+    return t;
+  }
+  __device__ __forceinline__ void at4(int r, int c, float* o) const {       // c % 4 == 0
+    const float* q = p + (size_t)r * ncols + c;
+    float4 t = *reinterpret_cast<const float4*>(q);
+    for (int s = 1; s < n; ++s) {
+      const float4 u = *reinterpret_cast<const float4*>(q + (size_t)s * stride);
+      t.x += u.x; t.y += u.y; t.z += u.z; t.w += u.w;
+    }
+    o[0] = t.x; o[1] = t.y; o[2] = t.z; o[3] = t.w;
+  }
+};
+
+__device__ __forceinline__ float wave_sum(float v) {
+#pragma unroll
+  for (int off = 1; off < 64; off <<= 1) v += __shfl_xor(v, off, 64);
+  return v;
+}
+__device__ __forceinline__ float block_sum256(float v, float* red /*[4] LDS*/) {
+  v = wave_sum(v);
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return (red[0] + red[1]) + (red[2] + red[3]);
+}
+__device__ __forceinline__ float f32_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float f32_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+
+// ---------------------------------------------------------------------------------------------------- f32 dot
+// out[r][n] = sum_k x[r][k] w[n][k], k ascending by fma.  x [R][Kp], w [Np][Kp] row-major f32, Kp % 32 == 0, Np % 16 == 0.  Grouped: 16-row block rb
+// uses the matrix of group rb_exp[rb] (-1: none), wstride floats apart.  grid (ceil(Np / 64), ceil(R / 16)), block 256 (16 rows x 16 column lanes).
+__global__ __launch_bounds__(256) void k_dot32(const float* __restrict__ x, const float* __restrict__ w, int Kp, int Np, int R, float* __restrict__ out,
+                                               const int32_t* __restrict__ rb_exp, size_t wstride) {
+  __shared__ float xs[16][33], ws[64][33];
+  const int tid = threadIdx.x, n0 = blockIdx.x * 64, r0 = blockIdx.y * 16;
+  if (rb_exp != nullptr) {
+    const int ex = rb_exp[blockIdx.y];
+    if (ex < 0) return;
+    w += (size_t)ex * wstride;
+  }
+  const int tr = tid >> 4, tc = tid & 15;
+  float acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int k0 = 0; k0 < Kp; k0 += 32) {
+    for (int i = tid; i < 16 * 32; i += 256) xs[i >> 5][i & 31] = (r0 + (i >> 5) < R) ? x[(size_t)(r0 + (i >> 5)) * Kp + k0 + (i & 31)] : 0.0f;
+    for (int i = tid; i < 64 * 32; i += 256) ws[i >> 5][i & 31] = (n0 + (i >> 5) < Np) ? w[(size_t)(n0 + (i >> 5)) * Kp + k0 + (i & 31)] : 0.0f;
+    __syncthreads();
+#pragma unroll 8
+    for (int k = 0; k < 32; ++k) {
+      const float xv = xs[tr][k];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[j] = fmaf(xv, ws[tc + 16 * j][k], acc[j]);
+    }
+    __syncthreads();
+  }
+  if (r0 + tr < R) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (n0 + tc + 16 * j < Np) out[(size_t)(r0 + tr) * Np + n0 + tc + 16 * j] = acc[j];
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------- weights
+// src [n][k] row-major ([out, in] linear weights) -> rows n of a dot operand of Kp k-columns, at (column n_off + n, k k_off + k).  inter: 16-column
+// tile j goes to tile 2 j + n_off (the two matrices of a gated unit side by side).  trans: src is [k][n].
+template <typename S, typename T>
+__global__ void k_load_nk(const S* __restrict__ src, T* __restrict__ dst, int n, int k, int Kp, int n_off, int k_off, int inter, int trans) {
+  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= (int64_t)n * k) return;
+  const int nn = trans ? (int)(i % n) : (int)(i / k), kk = trans ? (int)(i / n) : (int)(i % k);
+  const int col = inter ? ((nn >> 4) * 2 + n_off) * 16 + (nn & 15) : n_off + nn;
+  const float v = to_f(src[i]);
+  if constexpr (sizeof(T) == 2) dst[widx(k_off + kk, col, Kp)] = f2bf(v);
+  else dst[(size_t)col * Kp + k_off + kk] = v;
+}
+template <typename S, typename T>
+__global__ void k_load_vec(const S* __restrict__ src, T* __restrict__ dst, int64_t n) {
+  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) dst[i] = from_f<T>(to_f(src[i]));
+}
+
+// ---------------------------------------------------------------------------------------------------- row segments
+// A segment = consecutive rows of one page group at consecutive positions: what a recurrence walks through.  One block of 1024 threads.
+//   row_seg[r], row_j[r]   segment of row r and its place in it (row_seg -1: idle)
+//   seg[s] = {first row, rows, page group, first position, parity of the convolution tail to read, 0, 0, 0}
+// recurrent != 0: a segment must start at position 0 (the state counts as zero) or where its group's state stands (state_len); anything else, and a
+// second segment of a group in one call, idles and is counted in err[0].  The tails of short convolutions are double-buffered: a pass reads parity
+// p and writes 1 - p, so no row waits for another one's tail.
+// head_rb: 16-row block b of a head-major activation matrix (rbh blocks per head) belongs to head b / rbh.
+__global__ __launch_bounds__(1024) void k_segments(int R, int32_t* row_active, const int32_t* row_slot, const int32_t* row_pos, int32_t* row_seg, int32_t* row_j,
+                                                   int32_t* seg /*[.][8]*/, int32_t* nseg_out, int32_t* state_len, int32_t* parity, int32_t* claim, int groups,
+                                                   int recurrent, int32_t* err, int32_t* head_rb, int nhead_rb, int rbh) {
+  __shared__ int s_last[1024];
+  __shared__ int s_cnt;
+  const int tid = threadIdx.x;
+  for (int i = tid; i < groups; i += 1024) claim[i] = 0;
+  for (int i = tid; i < nhead_rb; i += 1024) head_rb[i] = i / rbh;
+  if (tid == 0) s_cnt = 0;
+  const int per = (R + 1023) / 1024, lo = min(tid * per, R), hi = min(lo + per, R);
+  auto starts = [&](int r) { return r == 0 || !row_active[r - 1] || row_slot[r - 1] != row_slot[r] || row_pos[r - 1] + 1 != row_pos[r]; };
+  int last = -1;
+  for (int r = lo; r < hi; ++r)
+    if (row_active[r] && starts(r)) last = r;
+  s_last[tid] = last;
+  __syncthreads();
+  for (int off = 1; off < 1024; off <<= 1) {               // inclusive maximum over the threads before and at this one
+    const int v = tid >= off ? s_last[tid - off] : -1;
+    __syncthreads();
+    s_last[tid] = max(s_last[tid], v);
+    __syncthreads();
+  }
+  int cur = tid > 0 ? s_last[tid - 1] : -1;                // start of the segment that reaches into this thread's rows
+  const int cur0 = cur;
+  for (int r = lo; r < hi; ++r) {
+    if (!row_active[r]) { row_seg[r] = -1; row_j[r] = 0; continue; }
+    if (starts(r)) {
+      cur = r;
+      const int s = atomicAdd(&s_cnt, 1);
+      row_seg[r] = s;
+    }
+    row_j[r] = r - cur;
+  }
+  __syncthreads();
+  cur = cur0;
+  for (int r = lo; r < hi; ++r) {                          // the last row of a segment writes its descriptor
+    if (!row_active[r]) continue;
+    if (row_j[r] == 0) cur = r;
+    const bool ends = r == R - 1 || !row_active[r + 1] || row_j[r + 1] == 0;
+    if (!ends) continue;
+    const int s = row_seg[cur], g = row_slot[r], start = row_pos[cur], n = r - cur + 1;
+    bool ok = true;
+    int par = 0;
+    if (recurrent) {
+      ok = atomicAdd(&claim[g], 1) == 0 && (start == 0 || start == state_len[g]);
+      if (ok) { par = parity[g]; parity[g] = par ^ 1; state_len[g] = start + n; }
+      else atomicAdd(err, 1);
+    }
+    int32_t* d = seg + (size_t)s * 8;
+    d[0] = cur; d[1] = ok ? n : 0; d[2] = g; d[3] = start; d[4] = par;
+  }
+  __syncthreads();
+  cur = cur0;
+  for (int r = lo; r < hi; ++r) {
+    if (!row_active[r]) continue;
+    if (row_j[r] == 0) cur = r;
+    const int s = row_seg[cur];
+    const bool ok = seg[(size_t)s * 8 + 1] > 0;
+    if (r != cur) row_seg[r] = s;
+    if (!ok) row_seg[r] = -1;
+  }
+  __syncthreads();
+  for (int r = lo; r < hi; ++r)
+    if (row_seg[r] < 0) row_active[r] = 0;
+  if (tid == 0) *nseg_out = s_cnt;
+}
+
+// state of group src -> group dst (both tail buffers, the recurrent matrices, the length).  grid (chunks), block 256; n0, n1: floats per group
+__global__ __launch_bounds__(256) void k_state_copy(float* const* bases, const int64_t* per_group, int nbuf, int src, int dst, int32_t* state_len, int32_t* parity) {
+  for (int b = 0; b < nbuf; ++b) {
+    float* p = bases[b];
+    const int64_t n = per_group[b];
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) p[dst * n + i] = p[src * n + i];
+  }
+  if (blockIdx.x == 0 && threadIdx.x == 0) { state_len[dst] = state_len[src]; parity[dst] = parity[src]; }
+}
+__global__ __launch_bounds__(256) void k_latent_pages_copy(PageStateDev s, int src, int dst, char* const* pools, const int64_t* page_bytes, int P) {
+  const int i = blockIdx.x, l = blockIdx.y;
+  if (i >= s.num_pages_used[dst] || i >= s.num_pages_used[src]) return;
+  const int64_t n = page_bytes[l];
+  const u32x4* a = reinterpret_cast<const u32x4*>(pools[l] + (size_t)s.page_map[(size_t)src * s.mpg + i] * n);
+  u32x4* b = reinterpret_cast<u32x4*>(pools[l] + (size_t)s.page_map[(size_t)dst * s.mpg + i] * n);
+  for (int64_t e = threadIdx.x; e < n / 16; e += 256) b[e] = a[e];
+}
+
+// ---------------------------------------------------------------------------------------------------- embedding, norms
+// x[r] = table[token] * scale (f32) and its copy as the first dot's operand.  grid R, block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ table, const int32_t* __restrict__ ids, float scale, int E, int Ep, int V, float* __restrict__ x,
+                                                      T* __restrict__ xb) {
+  const int r = blockIdx.x;
+  const int id = min(max(ids[r], 0), V - 1);
+  for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
+    float v[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      v[j] = k0 + j < E ? to_f(table[(size_t)id * E + k0 + j]) * scale : 0.0f;
+      if (k0 + j < E) x[(size_t)r * E + k0 + j] = v[j];
+    }
+    act_store8(xb, r, k0, Ep, v);
+  }
+}
+
+// A sublayer's output t (slices, or the weighted sum of a row's expert outputs) -> RMS norm with a zero-centred weight -> residual:
+//   x <- x + t / sqrt(mean(t^2) + eps) * (1 + w);  xb = the new x as the next dot's operand.
+// pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  grid R, block 256, LDS E floats.
+template <typename T>
+__global__ __launch_bounds__(256) void k_post_norm(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, const float* __restrict__ w, float eps,
+                                                   int E, int Ep, float* __restrict__ x, T* __restrict__ xb) {
+  extern __shared__ __attribute__((aligned(16))) float tb[];
+  __shared__ float red[4];
+  const int r = blockIdx.x;
+  float ss = 0.0f;
+  for (int k0 = threadIdx.x * 4; k0 < E; k0 += 1024) {
+    float v[4];
+    if (pos == nullptr) {
+      t.at4(r, k0, v);
+    } else {
+      v[0] = v[1] = v[2] = v[3] = 0.0f;
+      for (int j = 0; j < top; ++j) {
+        float u[4];
+        t.at4(pos[(size_t)r * top + j], k0, u);
+        const float wj = wts[(size_t)r * top + j];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = fmaf(wj, u[i], v[i]);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (k0 + i < E) { ss = fmaf(v[i], v[i], ss); tb[k0 + i] = v[i]; }
+  }
+  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+  for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
+    float v[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int k = k0 + j;
+      v[j] = 0.0f;
+      if (k < E) {
+        v[j] = x[(size_t)r * E + k] + tb[k] * rs * (1.0f + w[k]);
+        x[(size_t)r * E + k] = v[j];
+      }
+    }
+    act_store8(xb, r, k0, Ep, v);
+  }
+}
+
+// rows lrows[i] (or lrow0 + i) of x -> zero-centred RMS norm -> the head's operand.  grid nl, block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_final_norm(const float* __restrict__ x, const int32_t* __restrict__ lrows, int lrow0, int nrows, const float* __restrict__ w, float eps,
+                                                    int E, int Ep, T* __restrict__ xn) {
+  __shared__ float red[4];
+  const int i = blockIdx.x;
+  const int r = min(max(lrows != nullptr ? lrows[i] : lrow0 + i, 0), nrows - 1);
+  float ss = 0.0f;
+  for (int k = threadIdx.x; k < E; k += 256) { const float v = x[(size_t)r * E + k]; ss = fmaf(v, v, ss); }
+  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+  for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
+    float v[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = k0 + j < E ? x[(size_t)r * E + k0 + j] * rs * (1.0f + w[k0 + j]) : 0.0f;
+    act_store8(xn, i, k0, Ep, v);
+  }
+}
+
+// logits = the head's slices; (max, first index) per block of 1024 columns over the allowed ones.  grid (ceil(V / 1024), nl), block 256.
+__global__ __launch_bounds__(256) void k_head_post(Slices t, int V, ColRanges cr, float* __restrict__ logits /*[nl][V] or nullptr*/, float* __restrict__ amax_val,
+                                                   int32_t* __restrict__ amax_idx) {
+  __shared__ float bv[4];
+  __shared__ int bi[4];
+  const int r = blockIdx.y, lane = threadIdx.x & 63;
+  float best = -INFINITY;
+  int idx = 0x7fffffff;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = blockIdx.x * 1024 + i * 256 + threadIdx.x;
+    if (c >= V) continue;
+    const float v = t.at(r, c);
+    if (logits != nullptr) logits[(size_t)r * V + c] = v;
+    if (v > best && col_allowed(cr, c)) { best = v; idx = c; }
+  }
+#pragma unroll
+  for (int off = 1; off < 64; off <<= 1) {
+    const float ov = __shfl_xor(best, off, 64);
+    const int oi = __shfl_xor(idx, off, 64);
+    if (ov > best || (ov == best && oi < idx)) { best = ov; idx = oi; }
+  }
+  if (lane == 0) { bv[threadIdx.x >> 6] = best; bi[threadIdx.x >> 6] = idx; }
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    for (int w = 1; w < 4; ++w)
+      if (bv[w] > best || (bv[w] == best && bi[w] < idx)) { best = bv[w]; idx = bi[w]; }
+    amax_val[(size_t)r * gridDim.x + blockIdx.x] = best;
+    amax_idx[(size_t)r * gridDim.x + blockIdx.x] = idx;
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------- latent attention
+struct LatentGeom {
+  int H, dn, dr, rank, P, mpg, window;      // heads, unrotated / rotated query dims, latent size, page size, pages per group, window (<= 0: none)
+  int rankp, rotp;                          // padded sizes: cached row = [rankp latent | rotp rotated key part], DK = rankp + rotp elements
+  float scale;
+};
+
+// The input projection's slices ([q heads of dn + dr | d_off: latent, rotated key part]) -> the row's cache entry (normed latent, rotated key part)
+// and the queries: unrotated parts head-major as the operand of the key up-projection (row h Rp + r), rotated parts qr [R][H][rotp].
+// rope: f32 [position][dr / 2] cos, sin.  grid (R, 1 + ceil(H / 4)), block 256: y = 0 the cache entry, y > 0 four heads (a wave each).
+template <typename T>
+__global__ __launch_bounds__(256) void k_latent_prep(Slices t, int d_off, LatentGeom g, const float* __restrict__ cnorm, float eps, const float* __restrict__ rope_cos,
+                                                     const float* __restrict__ rope_sin, const int32_t* __restrict__ row_slot, const int32_t* __restrict__ row_pos,
+                                                     const int32_t* __restrict__ row_active, const int32_t* __restrict__ page_map, T* __restrict__ pages, T* __restrict__ qx,
+                                                     int dnp, int Rp, T* __restrict__ qr) {
+  __shared__ float red[4];
+  const int r = blockIdx.x, half = g.dr >> 1;
+  const bool act = row_active[r] != 0;
+  const int pos = act ? row_pos[r] : 0;
+  if (blockIdx.y == 0) {
+    if (!act) return;
+    float ss = 0.0f;
+    for (int k = threadIdx.x; k < g.rank; k += 256) { const float v = t.at(r, d_off + k); ss = fmaf(v, v, ss); }
+    const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)g.rank + eps);
+    const int page = page_map[(size_t)row_slot[r] * g.mpg + pos / g.P];
+    T* row = pages + ((size_t)page * g.P + pos % g.P) * (g.rankp + g.rotp);
+    for (int k = threadIdx.x; k < g.rank; k += 256) row[k] = from_f<T>(t.at(r, d_off + k) * rs * cnorm[k]);
+    for (int i = threadIdx.x; i < half; i += 256) {
+      const float u = t.at(r, d_off + g.rank + 2 * i), v = t.at(r, d_off + g.rank + 2 * i + 1);
+      const float c = rope_cos[(size_t)pos * half + i], s = rope_sin[(size_t)pos * half + i];
+      row[g.rankp + 2 * i] = from_f<T>(u * c - v * s);
+      row[g.rankp + 2 * i + 1] = from_f<T>(v * c + u * s);
+    }
+    return;
+  }
+  const int h = (blockIdx.y - 1) * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (h >= g.H) return;
+  const int c0 = h * (g.dn + g.dr);
+  for (int k = lane; k < dnp; k += 64) act_store1(qx, h * Rp + r, k, dnp, k < g.dn ? t.at(r, c0 + k) : 0.0f);
+  T* qo = qr + ((size_t)r * g.H + h) * g.rotp;
+  for (int i = lane; i < g.rotp / 2; i += 64) {
+    float a = 0.0f, b = 0.0f;
+    if (i < half) {
+      const float u = t.at(r, c0 + g.dn + 2 * i), v = t.at(r, c0 + g.dn + 2 * i + 1);
+      const float c = rope_cos[(size_t)pos * half + i], s = rope_sin[(size_t)pos * half + i];
+      a = u * c - v * s; b = v * c + u * s;
+    }
+    qo[2 * i] = from_f<T>(a); qo[2 * i + 1] = from_f<T>(b);
+  }
+}
+
+// Any sizes (rank <= 1024), any T: block = (row, head); thread = key for the scores (tiles of 256 keys, running maximum and sum), thread = latent
+// column for the weighted sum.  qa: slices of the queries in latent space (row h Rp + r); out: act(T), row h Rp + r.  grid (R, H), block 256,
+// LDS = (rankp + rotp + 256) floats.
+template <typename T>
+__global__ __launch_bounds__(256) void k_latent_attn_any(Slices qa, const T* __restrict__ qr, LatentGeom g, const int32_t* __restrict__ row_slot, const int32_t* __restrict__ row_pos,
+                                                         const int32_t* __restrict__ row_active, const int32_t* __restrict__ page_map, const T* __restrict__ pages, int Rp,
+                                                         T* __restrict__ out, int Kp) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  __shared__ float red[4];
+  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, DK = g.rankp + g.rotp;
+  if (!row_active[r]) return;
+  float* q = sm;
+  float* p = sm + DK;
+  for (int k = tid; k < DK; k += 256) {
+    float v = 0.0f;
+    if (k < g.rank) v = qa.at(h * Rp + r, k);
+    else if (k >= g.rankp) v = to_f(qr[((size_t)r * g.H + h) * g.rotp + k - g.rankp]);
+    q[k] = to_f(from_f<T>(v));
+  }
+  __syncthreads();
+  const int pos = row_pos[r], k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
+  const int32_t* prow = page_map + (size_t)row_slot[r] * g.mpg;
+  float m = -INFINITY, l = 0.0f, acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int j0 = k_lo; j0 <= pos; j0 += 256) {
+    const int j = j0 + tid;
+    float s = -INFINITY;
+    if (j <= pos) {
+      const T* kp = pages + ((size_t)prow[j / g.P] * g.P + j % g.P) * DK;
+      float a = 0.0f;
+      for (int k = 0; k < g.rank; ++k) a = fmaf(q[k], to_f(kp[k]), a);
+      float b = 0.0f;
+      for (int k = g.rankp; k < g.rankp + g.dr; ++k) b = fmaf(q[k], to_f(kp[k]), b);
+      s = (a + b) * g.scale;
+    }
+    float tm = s;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) tm = fmaxf(tm, __shfl_xor(tm, off, 64));
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = tm;
+    __syncthreads();
+    const float mn = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), m);
+    const float e = j <= pos ? expf(s - mn) : 0.0f;
+    p[tid] = e;
+    const float al = expf(m - mn);
+    const float ls = block_sum256(e, red);                  // (its barriers also publish p)
+    l = l * al + ls;
+    m = mn;
+    const int nk = min(256, pos - j0 + 1);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] *= al;
+    for (int kk = 0; kk < nk; ++kk) {
+      const T* kp = pages + ((size_t)prow[(j0 + kk) / g.P] * g.P + (j0 + kk) % g.P) * DK;
+      const float w = p[kk];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (tid + 256 * i < g.rank) acc[i] = fmaf(w, to_f(kp[tid + 256 * i]), acc[i]);
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (tid + 256 * i < Kp) act_store1(out, h * Rp + r, tid + 256 * i, Kp, tid + 256 * i < g.rank ? acc[i] / l : 0.0f);
+}
+
+// The bf16 matrix-core form.  All heads of a row share the cached latent, so the tile's M side is (row, head) pairs: WM = 4 (prompts): 64 pairs = up
+// to 64 / HB consecutive rows x HB heads, a wave owns 16 pairs, the four waves share every 32-key tile; WM = 1 (decode): 16 pairs = the heads of one
+// row, the four waves take different key tiles (and blockIdx.z splits them further) and merge at the end.
+//   scores   D[key][pair] = mfma(A = cached rows, B = queries [latent | rotated]): a lane holds 4 + 4 keys of one pair
+//   weights  running maximum / sum per pair in f32, exp2; P packs to bf16 in registers -- the lane's own 8 keys ARE its operand of the next product
+//            when the cached rows are read with the same key order (4q .. 4q + 3, 16 + 4q .. 16 + 4q + 3 for lane group q)
+//   output   D[column][pair] = mfma(A = cached latent read column-wise (ds_read_b64_tr_b16), B = P)
+// RT = 16-column tiles of the padded latent, RS = 32-wide steps of the padded rotated part.
+// grid (ceil(R / NQ), ceil(H / HB), WM == 1 ? splits : 1), block 256.
+struct LatentAttnArgs {
+  Slices qa; const bf16_t* qr; LatentGeom g;
+  const int32_t *row_slot, *row_pos, *row_active, *page_map;
+  const bf16_t* pages;
+  int R, Rp, NQ, HB;
+  bf16_t* out; int Kp;                     // act, row h Rp + r
+  float *part_o, *part_ml;                 // splits > 1: [R H][splits][rankp], [R H][splits][2]
+};
+template <int RT, int RS> constexpr int latent_pitch() { return RT * 16 + RS * 32 + 8; }
+template <int RT, int RS, int WM>
+__global__ __launch_bounds__(256, 1) void k_latent_attn(LatentAttnArgs a) {
+  constexpr int DK = RT * 16 + RS * 32, PITCH = latent_pitch<RT, RS>(), CPR = DK / 8;
+  constexpr int NTH = WM == 4 ? 256 : 64;                 // threads that stage one tile
+  constexpr int NC = (32 * CPR + NTH - 1) / NTH;          // 16-byte pieces per thread
+  constexpr int NKS = RT / 2 + RS;                        // k-steps of the scores
+  extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
+  __shared__ float s_m[4][16], s_l[4][16];
+  const LatentGeom& g = a.g;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
+  const int r0 = blockIdx.x * a.NQ, nr = min(a.NQ, a.R - r0), h0 = blockIdx.y * a.HB, hb = min(a.HB, g.H - h0);
+  bf16_t* tile = WM == 4 ? lds : lds + (size_t)wave * 32 * PITCH;
+  const int pair = (WM == 4 ? wave * 16 : 0) + r_in;
+  const int qi = pair / a.HB, hh = pair % a.HB;
+  const bool pair_ok = qi < nr && hh < hb;
+  const int row = r0 + (pair_ok ? qi : 0), head = h0 + (pair_ok ? hh : 0);
+  const bool live = pair_ok && a.row_active[row] != 0;
+  const int pos = live ? a.row_pos[row] : -1;
+  // queries: lane = pair r_in, 8 consecutive features per step
+  bf16x8 qf[NKS];
+#pragma unroll
+  for (int ks = 0; ks < RT / 2; ++ks) {
+    float v[8];
+    a.qa.at4(head * a.Rp + row, ks * 32 + cq * 8, v);
+    a.qa.at4(head * a.Rp + row, ks * 32 + cq * 8 + 4, v + 4);
+    u32x4 o;
+    o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3])); o.z = pack2(f2bf(v[4]), f2bf(v[5])); o.w = pack2(f2bf(v[6]), f2bf(v[7]));
+    qf[ks] = __builtin_bit_cast(bf16x8, o);
+  }
+#pragma unroll
+  for (int ks = 0; ks < RS; ++ks)
+    qf[RT / 2 + ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.qr + ((size_t)row * g.H + head) * g.rotp + ks * 32 + cq * 8));
+  f32x4 o[RT];
+#pragma unroll
+  for (int i = 0; i < RT; ++i) o[i] = f32x4(0.0f);
+  float m = -INFINITY, l = 0.0f;
+  const float sc = g.scale * 1.44269504088896340736f;
+
+  u32x4 stg[NC];
+  for (int ra = 0; ra < nr;) {                            // runs of rows that share a page group
+    if (!a.row_active[r0 + ra]) { ++ra; continue; }
+    const int slot = a.row_slot[r0 + ra];
+    int lo = a.row_pos[r0 + ra], hi = lo, rb = ra + 1;
+    while (rb < nr && a.row_active[r0 + rb] && a.row_slot[r0 + rb] == slot) { const int p = a.row_pos[r0 + rb]; lo = min(lo, p); hi = max(hi, p); ++rb; }
+    const bool mine = live && qi >= ra && qi < rb;
+    ra = rb;
+    const int k_lo = g.window > 0 ? max(0, lo - g.window + 1) : 0;
+    const int ntile = (hi - k_lo) / 32 + 1;
+    const int32_t* prow = a.page_map + (size_t)slot * g.mpg;
+    const int my_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
+    const int t0 = WM == 4 ? 0 : (int)blockIdx.z * 4 + wave, tstep = WM == 4 ? 1 : 4 * (int)gridDim.z;
+    auto fetch = [&](int t) {
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        const int c = (WM == 4 ? tid : lane) + i * NTH;
+        if ((32 * CPR) % NTH == 0 || c < 32 * CPR) {
+          const int key = min(k_lo + t * 32 + c / CPR, hi), pc = c % CPR;
+          stg[i] = *reinterpret_cast<const u32x4*>(a.pages + ((size_t)prow[key / g.P] * g.P + key % g.P) * DK + pc * 8);
+        }
+      }
+    };
+    if (t0 < ntile) fetch(t0);
+    for (int t = t0; t < ntile; t += tstep) {
+      if constexpr (WM == 4) __syncthreads();              // every wave is done with the previous tile
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        const int c = (WM == 4 ? tid : lane) + i * NTH;
+        if ((32 * CPR) % NTH == 0 || c < 32 * CPR) *reinterpret_cast<u32x4*>(tile + (c / CPR) * PITCH + (c % CPR) * 8) = stg[i];
+      }
+      if constexpr (WM == 4) __syncthreads();
+      else __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      if (t + tstep < ntile) fetch(t + tstep);
+      f32x4 s0 = f32x4(0.0f), s1 = f32x4(0.0f);
+#pragma unroll
+      for (int ks = 0; ks < NKS; ++ks) {
+        const bf16x8 k0 = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + r_in * PITCH + ks * 32 + cq * 8));
+        const bf16x8 k1 = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + (16 + r_in) * PITCH + ks * 32 + cq * 8));
+        s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[ks], s0, 0, 0, 0);
+        s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[ks], s1, 0, 0, 0);
+      }
+      float sv[8];
+      float tm = -INFINITY;
+      const int kb = k_lo + t * 32 + cq * 4;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int key = kb + (j < 4 ? j : 12 + j);
+        const float v = (j < 4 ? s0[j & 3] : s1[j & 3]) * sc;
+        sv[j] = (mine && key <= pos && key >= my_lo) ? v : -INFINITY;
+        tm = fmaxf(tm, sv[j]);
+      }
+      tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+      tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+      const float mn = fmaxf(m, tm);
+      const float al = mn == -INFINITY ? 1.0f : exp2f(m - mn);
+      float ls = 0.0f, pv[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) { pv[j] = sv[j] == -INFINITY ? 0.0f : exp2f(sv[j] - mn); ls += pv[j]; }
+      ls += __shfl_xor(ls, 16, 64);
+      ls += __shfl_xor(ls, 32, 64);
+      l = l * al + ls;
+      m = mn;
+      u32x4 pk;
+      pk.x = pack2(f2bf(pv[0]), f2bf(pv[1])); pk.y = pack2(f2bf(pv[2]), f2bf(pv[3])); pk.z = pack2(f2bf(pv[4]), f2bf(pv[5])); pk.w = pack2(f2bf(pv[6]), f2bf(pv[7]));
+      const bf16x8 pf = __builtin_bit_cast(bf16x8, pk);
+      if (__any(al != 1.0f)) {
+#pragma unroll
+        for (int i = 0; i < RT; ++i) o[i] *= al;
+      }
+      // lane 4 a + p of a 16-lane group addresses row 4 q + a, columns 4 p .. 4 p + 3, and receives its column of the 4 rows
+      const bf16_t* vb = tile + (4 * cq + (r_in >> 2)) * PITCH + 4 * (r_in & 3);
+      const uint32_t va = (uint32_t)(uintptr_t)((const __attribute__((address_space(3))) void*)(vb));
+      constexpr int VG = RT < 8 ? RT : 8;                  // tiles whose reads are in flight together
+#pragma unroll
+      for (int i0 = 0; i0 < RT; i0 += VG) {
+        uint2 f[VG][2];
+#pragma unroll
+        for (int i = 0; i < VG; ++i) {
+          asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[i][0]) : "v"(va), "n"((i0 + i) * 32) : "memory");
+          asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[i][1]) : "v"(va), "n"((i0 + i) * 32 + 16 * PITCH * 2) : "memory");
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int i = 0; i < VG; ++i) asm volatile("" : "+v"(f[i][0]), "+v"(f[i][1]));     // the products read what the wait has delivered
+#pragma unroll
+        for (int i = 0; i < VG; ++i) {
+          u32x4 v; v.x = f[i][0].x; v.y = f[i][0].y; v.z = f[i][1].x; v.w = f[i][1].y;
+          o[i0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), pf, o[i0 + i], 0, 0, 0);
+        }
+      }
+    }
+  }
+  if constexpr (WM == 4) {
+    if (!live) return;
+    const float inv = l > 0.0f ? 1.0f / l : 0.0f;
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+      const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+      act_store4(a.out, head * a.Rp + row, i * 16 + cq * 4, a.Kp, v);
+    }
+    const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    for (int c = RT * 16 + cq * 4; c < a.Kp; c += 16) act_store4(a.out, head * a.Rp + row, c, a.Kp, z);
+  } else {
+    float* ob = reinterpret_cast<float*>(tile);            // [16 pairs][RT * 16]: the wave's own tile region
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+#pragma unroll
+    for (int i = 0; i < RT; ++i) *reinterpret_cast<float4*>(ob + r_in * (RT * 16) + i * 16 + cq * 4) = make_float4(o[i][0], o[i][1], o[i][2], o[i][3]);
+    if (cq == 0) { s_m[wave][r_in] = m; s_l[wave][r_in] = l; }
+    __syncthreads();
+    if (!a.row_active[r0]) return;
+    const int nsplit = gridDim.z;
+    for (int e = tid; e < hb * RT * 4; e += 256) {
+      const int pr = e / (RT * 4), c = (e % (RT * 4)) * 4;
+      float mm = -INFINITY;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) mm = fmaxf(mm, s_m[w][pr]);
+      float ll = 0.0f, v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+      for (int w = 0; w < 4; ++w) {
+        const float f = s_m[w][pr] == -INFINITY ? 0.0f : exp2f(s_m[w][pr] - mm);
+        ll = fmaf(s_l[w][pr], f, ll);
+        const float4 u = *reinterpret_cast<const float4*>(reinterpret_cast<const float*>(lds + (size_t)w * 32 * PITCH) + pr * (RT * 16) + c);
+        v[0] = fmaf(u.x, f, v[0]); v[1] = fmaf(u.y, f, v[1]); v[2] = fmaf(u.z, f, v[2]); v[3] = fmaf(u.w, f, v[3]);
+      }
+      if (nsplit == 1) {
+        const float inv = ll > 0.0f ? 1.0f / ll : 0.0f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] *= inv;
+        act_store4(a.out, (h0 + pr) * a.Rp + r0, c, a.Kp, v);
+      } else {
+        const size_t pi = ((size_t)r0 * g.H + h0 + pr) * nsplit + blockIdx.z;
+        *reinterpret_cast<float4*>(a.part_o + pi * (RT * 16) + c) = make_float4(v[0], v[1], v[2], v[3]);
+        if (c == 0) { a.part_ml[pi * 2] = mm; a.part_ml[pi * 2 + 1] = ll; }
+      }
+    }
+    if (nsplit == 1) {
+      const int pad4 = (a.Kp - RT * 16) / 4;
+      const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+      for (int e = tid; e < hb * pad4; e += 256) act_store4(a.out, (h0 + e / pad4) * a.Rp + r0, RT * 16 + (e % pad4) * 4, a.Kp, z);
+    }
+  }
+}
+// the key splits of a row's heads put together.  grid (R, H), block 64.
+__global__ __launch_bounds__(64) void k_latent_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int cols, int H, int Rp,
+                                                       const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
+  const int r = blockIdx.x, h = blockIdx.y;
+  if (!row_active[r]) return;
+  const size_t p0 = ((size_t)r * H + h) * nsplit;
+  float mm = -INFINITY;
+  for (int s = 0; s < nsplit; ++s) mm = fmaxf(mm, part_ml[(p0 + s) * 2]);
+  float ll = 0.0f;
+  for (int s = 0; s < nsplit; ++s) { const float ms = part_ml[(p0 + s) * 2]; if (ms != -INFINITY) ll = fmaf(part_ml[(p0 + s) * 2 + 1], exp2f(ms - mm), ll); }
+  const float inv = 1.0f / ll;
+  for (int c = threadIdx.x * 4; c < Kp; c += 256) {
+    float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    if (c < cols) {
+      for (int s = 0; s < nsplit; ++s) {
+        const float ms = part_ml[(p0 + s) * 2];
+        if (ms == -INFINITY) continue;
+        const float f = exp2f(ms - mm) * inv;
+        const float4 u = *reinterpret_cast<const float4*>(part_o + (p0 + s) * cols + c);
+        v[0] = fmaf(u.x, f, v[0]); v[1] = fmaf(u.y, f, v[1]); v[2] = fmaf(u.z, f, v[2]); v[3] = fmaf(u.w, f, v[3]);
+      }
+    }
+    act_store4(out, h * Rp + r, c, Kp, v);
+  }
+}
+// head-major slices (row h Rp + r, n columns each) -> act of the output projection: column h n + c.  grid (R, ceil(Kp / 256)), block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_heads_x(Slices t, int H, int n, int Rp, T* __restrict__ out, int Kp) {
+  const int r = blockIdx.x, k = blockIdx.y * 256 + threadIdx.x;
+  if (k >= Kp) return;
+  act_store1(out, r, k, Kp, k < H * n ? t.at((k / n) * Rp + r, k % n) : 0.0f);
+}
+
+// ---------------------------------------------------------------------------------------------------- gated delta rule
+struct DeltaGeom {
+  int H, KH, d, dv, dp, taps;               // heads, query/key heads, key dims, value dims, padded key dims (16 RP), convolution taps
+  int oq, ok, ov, ob, oa, og, ra, rg;       // columns of the input projection: q, k, v, beta, decay rank, gate rank; the two ranks
+  int og2;                                  // column of the output gate in the second low-rank product (decays start at 0)
+  int C;                                    // convolution channels = 2 KH d + H dv (q, k, v)
+};
+// the two low-rank activations side by side as ONE operand (the second matrices form a block diagonal).  grid R, block 128.
+template <typename T>
+__global__ __launch_bounds__(128) void k_lowrank_x(Slices t, DeltaGeom g, T* __restrict__ out, int Kp) {
+  const int r = blockIdx.x;
+  for (int k = threadIdx.x; k < Kp; k += 128) {
+    float v = 0.0f;
+    if (k < g.ra) v = t.at(r, g.oa + k);
+    else if (k < g.ra + g.rg) v = t.at(r, g.og + k - g.ra);
+    act_store1(out, r, k, Kp, v);
+  }
+}
+
+// one channel of a short causal convolution: taps[0 .. n-1], the last for the row itself.  Earlier inputs come from the segment's rows or, before
+// its start, from the group's tail (oldest first).  Returns the convolution and leaves the channel's next tail (rows among the segment's last
+// n - 1 write their input; the last row carries older entries over when the segment is shorter than the tail).
+struct ConvCtx { const float* tail_in; float* tail_out; int j, n, start; };
+__device__ __forceinline__ float conv_channel(const Slices& t, int r, int col, const float* __restrict__ tp, int taps, int ch, int C, const ConvCtx& cc) {
+  const float x0 = t.at(r, col);
+  float acc = x0 * tp[taps - 1];
+  for (int b = 1; b < taps; ++b) {
+    float v = 0.0f;
+    if (cc.j - b >= 0) v = t.at(r - b, col);
+    else if (cc.start > 0) v = cc.tail_in[(size_t)(taps - 1 - (b - cc.j)) * C + ch];
+    acc = fmaf(v, tp[taps - 1 - b], acc);
+  }
+  const int dist = cc.n - 1 - cc.j;
+  if (dist < taps - 1) cc.tail_out[(size_t)(taps - 2 - dist) * C + ch] = x0;
+  if (dist == 0)
+    for (int e = cc.n; e < taps - 1; ++e)      // entries that are still older than the segment
+      cc.tail_out[(size_t)(taps - 2 - e) * C + ch] = cc.start > 0 ? cc.tail_in[(size_t)(taps - 2 - (e - cc.n)) * C + ch] : 0.0f;
+  return acc;
+}
+
+// Everything the recurrence takes in: convolutions, silu, unit vectors, step sizes, decays (f32).  wave = one query/key head, or one value head with
+// its beta and decays.  grid (R, ceil((KH + H) / 4)), block 256.
+struct DeltaPrepArgs {
+  Slices t, t2; DeltaGeom g;
+  const float *cq, *ck, *cv, *a_log, *dt_bias;
+  const int32_t *row_seg, *row_j, *seg;
+  float* tails;                             // [group][2][taps - 1][C]
+  float *q, *k, *kq, *v, *dec, *beta;       // [R][KH][dp], .., [R][KH], [R][H][dv], [R][H][dp], [R][H]
+};
+__global__ __launch_bounds__(256) void k_delta_prep(DeltaPrepArgs a) {
+  const DeltaGeom& g = a.g;
+  const int r = blockIdx.x, lane = threadIdx.x & 63, vi = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const int s = a.row_seg[r];
+  if (s < 0 || vi >= g.KH + g.H) return;
+  const int32_t* sg = a.seg + (size_t)s * 8;
+  const size_t tsz = (size_t)(g.taps - 1) * g.C;
+  float* tb = a.tails + (size_t)sg[2] * 2 * tsz;
+  const ConvCtx cc{tb + (size_t)sg[4] * tsz, tb + (size_t)(sg[4] ^ 1) * tsz, a.row_j[r], sg[1], sg[3]};
+  if (vi < g.KH) {
+    float* qo = a.q + ((size_t)r * g.KH + vi) * g.dp;
+    float* ko = a.k + ((size_t)r * g.KH + vi) * g.dp;
+    float qq = 0.0f, kk = 0.0f, qk = 0.0f;
+    float qv[8], kv[8];                     // dims up to 512, eight per lane
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int c = lane + 64 * i;
+      qv[i] = kv[i] = 0.0f;
+      if (c < g.d) {
+        const int ch = vi * g.d + c;
+        const float x = conv_channel(a.t, r, g.oq + ch, a.cq + (size_t)ch * g.taps, g.taps, ch, g.C, cc);
+        const float y = conv_channel(a.t, r, g.ok + ch, a.ck + (size_t)ch * g.taps, g.taps, g.KH * g.d + ch, g.C, cc);
+        qv[i] = x * f32_sigmoid(x); kv[i] = y * f32_sigmoid(y);
+        qq = fmaf(qv[i], qv[i], qq); kk = fmaf(kv[i], kv[i], kk);
+      }
+    }
+    qq = wave_sum(qq); kk = wave_sum(kk);
+    const float qs = 1.0f / sqrtf(qq + 1e-6f) * (1.0f / sqrtf((float)g.d)), ks = 1.0f / sqrtf(kk + 1e-6f);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int c = lane + 64 * i;
+      if (c < g.dp) { qo[c] = qv[i] * qs; ko[c] = kv[i] * ks; qk = fmaf(qv[i] * qs, kv[i] * ks, qk); }
+    }
+    qk = wave_sum(qk);
+    if (lane == 0) a.kq[(size_t)r * g.KH + vi] = qk;
+    return;
+  }
+  const int h = vi - g.KH;
+  for (int c = lane; c < g.dv; c += 64) {
+    const int ch = h * g.dv + c;
+    const float x = conv_channel(a.t, r, g.ov + ch, a.cv + (size_t)ch * g.taps, g.taps, 2 * g.KH * g.d + ch, g.C, cc);
+    a.v[((size_t)r * g.H + h) * g.dv + c] = x * f32_sigmoid(x);
+  }
+  const float ea = expf(a.a_log[h]);
+  float* go = a.dec + ((size_t)r * g.H + h) * g.dp;
+  for (int c = lane; c < g.dp; c += 64)
+    go[c] = c < g.d ? expf(-ea * f32_softplus(a.t2.at(r, h * g.d + c) + a.dt_bias[h * g.d + c])) : 0.0f;
+  if (lane == 0) a.beta[(size_t)r * g.H + h] = f32_sigmoid(a.t.at(r, g.ob + h));
+}
+
+// sum over the 16 lanes of a DPP row, every lane ends up with it
+__device__ __forceinline__ float row16_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, false));   // row_ror:8
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, false));   // row_ror:4
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, false));   // row_ror:2
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, false));   // row_ror:1
+  return v;
+}
+
+// The recurrence, per head:  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q, all f32.  The columns of S (value dims) never meet, so a
+// block owns 16 of them for one (segment, head): a wave four, 16 lanes per column with RP key rows each in registers.  o = (g S)^T q + (k . q) u: both
+// sums over the key rows are taken from the decayed state and run side by side.  Tokens come through LDS, TT at a time, the next ones already in
+// registers.  State [group][H][dv][dp]; a segment at position 0 starts from zero.  grid (segments, H, ceil(dv / 16)), block 256.
+struct DeltaScanArgs {
+  DeltaGeom g;
+  const int32_t *seg, *nseg;
+  const float *q, *k, *kq, *v, *dec, *beta;
+  float* state;
+  float* o;                                 // [R][H][dv]
+};
+template <int RP>
+__global__ __launch_bounds__(256) void k_delta_scan(DeltaScanArgs a) {
+  constexpr int DP = 16 * RP, TT = RP <= 8 ? 16 : 128 / RP;
+  constexpr int NL = (3 * TT * DP / 4 + 255) / 256;        // float4 loads per thread and token tile (q, k, decays)
+  __shared__ __attribute__((aligned(16))) float sm[3][TT][DP];
+  __shared__ float sv[TT][16], sb[TT], skq[TT];
+  const DeltaGeom& g = a.g;
+  const int s = blockIdx.x;
+  if (s >= *a.nseg) return;
+  const int first = a.seg[s * 8], n = a.seg[s * 8 + 1], grp = a.seg[s * 8 + 2], start = a.seg[s * 8 + 3];
+  if (n <= 0) return;
+  const int h = blockIdx.y, kh = h / (g.H / g.KH), tid = threadIdx.x, lane = tid & 63, sub = lane & 15;
+  const int cb = blockIdx.z * 16, cl = (tid >> 6) * 4 + (lane >> 4), col = cb + cl;
+  const bool col_ok = col < g.dv;
+  float S[RP];
+  float* sp = a.state + (((size_t)grp * g.H + h) * g.dv + (col_ok ? col : 0)) * DP + sub * RP;
+#pragma unroll
+  for (int i = 0; i < RP; ++i) S[i] = 0.0f;
+  if (start > 0 && col_ok) {
+    if constexpr (RP % 4 == 0) {
+#pragma unroll
+      for (int i = 0; i < RP; i += 4) { const float4 x = *reinterpret_cast<const float4*>(sp + i); S[i] = x.x; S[i + 1] = x.y; S[i + 2] = x.z; S[i + 3] = x.w; }
+    } else {
+#pragma unroll
+      for (int i = 0; i < RP; ++i) S[i] = sp[i];
+    }
+  }
+  float4 pf[NL];
+  float pv = 0.0f, pb = 0.0f;
+  auto fetch = [&](int t0) {                               // tokens t0 .. t0 + TT - 1 (past the end: the last one again, never used)
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = tid + i * 256;
+      if ((3 * TT * DP / 4) % 256 == 0 || e < 3 * TT * DP / 4) {
+        const int w = e / (TT * DP / 4), t = (e / (DP / 4)) % TT, c = (e % (DP / 4)) * 4, r = first + min(t0 + t, n - 1);
+        const float* src = w == 0 ? a.q + ((size_t)r * g.KH + kh) * DP : (w == 1 ? a.k + ((size_t)r * g.KH + kh) * DP : a.dec + ((size_t)r * g.H + h) * DP);
+        pf[i] = *reinterpret_cast<const float4*>(src + c);
+      }
+    }
+    if (tid < TT * 16) {
+      const int t = tid >> 4, c = cb + (tid & 15), r = first + min(t0 + t, n - 1);
+      pv = c < g.dv ? a.v[((size_t)r * g.H + h) * g.dv + c] : 0.0f;
+    }
+    if (tid < 2 * TT) {
+      const int r = first + min(t0 + (tid % TT), n - 1);
+      pb = tid < TT ? a.beta[(size_t)r * g.H + h] : a.kq[(size_t)r * g.KH + kh];
+    }
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < n; t0 += TT) {
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = tid + i * 256;
+      if ((3 * TT * DP / 4) % 256 == 0 || e < 3 * TT * DP / 4) *reinterpret_cast<float4*>(&sm[0][0][0] + (size_t)e * 4) = pf[i];
+    }
+    if (tid < TT * 16) sv[tid >> 4][tid & 15] = pv;
+    if (tid < 2 * TT) { if (tid < TT) sb[tid] = pb; else skq[tid - TT] = pb; }
+    __syncthreads();
+    if (t0 + TT < n) fetch(t0 + TT);
+    const int nt = min(TT, n - t0);
+    for (int t = 0; t < nt; ++t) {
+      float kv[RP], ax = 0.0f, bx = 0.0f;
+#pragma unroll
+      for (int i = 0; i < RP; ++i) {
+        kv[i] = sm[1][t][sub * RP + i];
+        S[i] *= sm[2][t][sub * RP + i];
+        ax = fmaf(kv[i], S[i], ax);
+        bx = fmaf(sm[0][t][sub * RP + i], S[i], bx);
+      }
+      ax = row16_sum(ax);
+      bx = row16_sum(bx);
+      const float u = sb[t] * (sv[t][cl] - ax);
+#pragma unroll
+      for (int i = 0; i < RP; ++i) S[i] = fmaf(kv[i], u, S[i]);
+      if (sub == 0 && col_ok) a.o[((size_t)(first + t0 + t) * g.H + h) * g.dv + col] = fmaf(skq[t], u, bx);
+    }
+  }
+  if (col_ok) {
+    if constexpr (RP % 4 == 0) {
+#pragma unroll
+      for (int i = 0; i < RP; i += 4) *reinterpret_cast<float4*>(sp + i) = make_float4(S[i], S[i + 1], S[i + 2], S[i + 3]);
+    } else {
+#pragma unroll
+      for (int i = 0; i < RP; ++i) sp[i] = S[i];
+    }
+  }
+}
+
+// read-out: o / rms(o) * norm * sigmoid(gate) per head -> the output projection's operand (column h dv + c).  grid (R, ceil(H / 4)), block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_delta_out(const float* __restrict__ o, Slices t2, DeltaGeom g, const float* __restrict__ nw, float eps, const int32_t* __restrict__ row_seg,
+                                                   T* __restrict__ out, int Kp) {
+  const int r = blockIdx.x, h = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (h >= g.H) return;
+  const bool live = row_seg[r] >= 0;
+  const float* oh = o + ((size_t)r * g.H + h) * g.dv;
+  float ss = 0.0f;
+  if (live)
+    for (int c = lane; c < g.dv; c += 64) ss = fmaf(oh[c], oh[c], ss);
+  const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)g.dv + eps);
+  for (int c = lane; c < g.dv; c += 64)
+    act_store1(out, r, h * g.dv + c, Kp, live ? oh[c] * rs * nw[c] * f32_sigmoid(t2.at(r, g.og2 + h * g.dv + c)) : 0.0f);
+  if (h == g.H - 1)
+    for (int k = g.H * g.dv + lane; k < Kp; k += 64) act_store1(out, r, k, Kp, 0.0f);
+}
+
+// ---------------------------------------------------------------------------------------------------- feed-forward
+// clamped gated unit from interleaved slices (tile 2 j gate, 2 j + 1 up): y = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up).
+// grid (ceil(Fp / 256), rows), block 256; rb_exp: rows of blocks without an expert are skipped.
+template <typename T>
+__global__ __launch_bounds__(256) void k_glu_clamped(Slices t, int Fp, float limit, T* __restrict__ out, const int32_t* __restrict__ rb_exp) {
+  const int f = blockIdx.x * 256 + threadIdx.x, r = blockIdx.y;
+  if (f >= Fp || (rb_exp != nullptr && rb_exp[r >> 4] < 0)) return;
+  const int c = (f >> 4) * 32 + (f & 15);
+  act_store1(out, r, f, Fp, ixt_glu_clamped(t.at(r, c), t.at(r, c + 16), limit));
+}
+
+// softmax over all n logits of a row in f32, the `top` largest (first index on a tie), their scores as they are.  One wave; z in LDS or HBM.
+__device__ __forceinline__ void route_top(const float* z, int n, int top, int lane, int32_t* idx, float* wts) {
+  float v[16];
+  float mx = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < 16; ++i) { v[i] = lane + 64 * i < n ? z[lane + 64 * i] : -INFINITY; mx = fmaxf(mx, v[i]); }
+#pragma unroll
+  for (int off = 1; off < 64; off <<= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
+  float sum = 0.0f;
+#pragma unroll
+  for (int i = 0; i < 16; ++i) if (lane + 64 * i < n) sum += expf(v[i] - mx);
+  sum = wave_sum(sum);
+  for (int j = 0; j < top; ++j) {
+    float b = -INFINITY;
+    int bi = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < 16; ++i)
+      if (v[i] > b) { b = v[i]; bi = lane + 64 * i; }
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float ob = __shfl_xor(b, off, 64);
+      const int oi = __shfl_xor(bi, off, 64);
+      if (ob > b || (ob == b && oi < bi)) { b = ob; bi = oi; }
+    }
+    if (bi >= n) bi = 0;                                   // only a row without finite logits gets here: any expert will do
+#pragma unroll
+    for (int i = 0; i < 16; ++i) if (lane + 64 * i == bi) v[i] = -INFINITY;
+    if (lane == 0) { idx[j] = bi; wts[j] = expf(b - mx) / sum; }
+  }
+}
+// few rows: logits and choice in one launch, f32 residual x f32 router weights.  grid R, block 256, LDS n floats.
+__global__ __launch_bounds__(256) void k_route_row(const float* __restrict__ x, const float* __restrict__ w /*[n][Ep]*/, int E, int Ep, int n, int top, int32_t* __restrict__ idx,
+                                                   float* __restrict__ wts) {
+  extern __shared__ __attribute__((aligned(16))) float z[];
+  const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const float* xr = x + (size_t)r * E;
+  for (int e = wave; e < n; e += 4) {
+    float a = 0.0f;
+    for (int k = lane; k < E; k += 64) a = fmaf(xr[k], w[(size_t)e * Ep + k], a);
+    a = wave_sum(a);
+    if (lane == 0) z[e] = a;
+  }
+  __syncthreads();
+  if (wave == 0) route_top(z, n, top, lane, idx + (size_t)r * top, wts + (size_t)r * top);
+}
+// many rows: 8 rows x 32 experts per block, x and w through LDS in steps of 32 k; z [R][n].  grid (ceil(n / 32), ceil(R / 8)), block 256.
+__global__ __launch_bounds__(256) void k_route_logits(const float* __restrict__ x, const float* __restrict__ w, int E, int Ep, int n, int R, float* __restrict__ z) {
+  __shared__ float xs[8][65], ws[32][65];
+  const int tid = threadIdx.x, e0 = blockIdx.x * 32, r0 = blockIdx.y * 8, tr = tid >> 5, te = tid & 31;
+  float a = 0.0f;
+  for (int k0 = 0; k0 < E; k0 += 64) {
+    for (int i = tid; i < 8 * 64; i += 256) xs[i >> 6][i & 63] = (r0 + (i >> 6) < R && k0 + (i & 63) < E) ? x[(size_t)(r0 + (i >> 6)) * E + k0 + (i & 63)] : 0.0f;
+    for (int i = tid; i < 32 * 64; i += 256) ws[i >> 6][i & 63] = (e0 + (i >> 6) < n && k0 + (i & 63) < E) ? w[(size_t)(e0 + (i >> 6)) * Ep + k0 + (i & 63)] : 0.0f;
+    __syncthreads();
+#pragma unroll 8
+    for (int k = 0; k < 64; ++k) a = fmaf(xs[tr][k], ws[te][k], a);
+    __syncthreads();
+  }
+  if (r0 + tr < R && e0 + te < n) z[(size_t)(r0 + tr) * n + e0 + te] = a;
+}
+__global__ __launch_bounds__(256) void k_route_pick(const float* __restrict__ z, int n, int top, int R, int32_t* __restrict__ idx, float* __restrict__ wts) {
+  const int r = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (r < R) route_top(z + (size_t)r * n, n, top, threadIdx.x & 63, idx + (size_t)r * top, wts + (size_t)r * top);
+}
+// any number of experts (<= 1024): destination row of every copy by one pass of counters; the order inside an expert is free.  One block of 1024.
+__global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __restrict__ idx, int npairs, int n, int align, int nrb_cap, int32_t* __restrict__ pos, int32_t* __restrict__ rb_exp) {
+  __shared__ int cnt[1024], off[1024];
+  const int tid = threadIdx.x;
+  cnt[tid] = 0;
+  for (int i = tid; i < nrb_cap; i += 1024) rb_exp[i] = -1;
+  __syncthreads();
+  for (int p = tid; p < npairs; p += 1024) pos[p] = atomicAdd(&cnt[idx[p]], 1);
+  __syncthreads();
+  const int padded = tid < n ? (cnt[tid] + align - 1) / align * align : 0;
+  off[tid] = padded;
+  __syncthreads();
+  for (int o = 1; o < 1024; o <<= 1) {
+    const int v = tid >= o ? off[tid - o] : 0;
+    __syncthreads();
+    off[tid] += v;
+    __syncthreads();
+  }
+  const int base = off[tid] - padded;
+  __syncthreads();
+  off[tid] = base;
+  __syncthreads();
+  if (tid < n)
+    for (int i = 0; i < (cnt[tid] + 15) / 16; ++i) rb_exp[base / 16 + i] = tid;
+  for (int p = tid; p < npairs; p += 1024) pos[p] += off[idx[p]];
+}
+__global__ __launch_bounds__(256) void k_gather32(const float* __restrict__ x, const int32_t* __restrict__ pos, int top, int Ep, float* __restrict__ xg) {
+  const int k = blockIdx.x * 256 + threadIdx.x, p = blockIdx.y;
+  if (k < Ep) xg[(size_t)pos[p] * Ep + k] = x[(size_t)(p / top) * Ep + k];
+}

@@ -23,6 +23,7 @@ import torch
 from . import _lib
 from . import engine_api
 from . import synth as _synth
+from . import architectures as _architectures
 from .inference.page_manager import PageManager, PageState
 
 Params = Any
@@ -101,7 +102,16 @@ class MaxEngine(engine_api.Engine):
       c.rope_llama31, c.rope_use_scale = 1, 1 if config.rope_use_scale else 0
     elif rope_type != "default":
       raise NotImplementedError(f"rope_type {config.rope_type}: 'default' and 'llama3.1' are built")
-    if config.decoder_block in ("gemma2", "gemma3"):   # layers/gemma2.py:69-236, layers/gemma3.py:35-200
+    if config.decoder_block == "hybrid":               # the layers are listed one by one (architectures.py)
+      c.decoder_block = _lib.BLOCK_HYBRID
+      fields = [f.name for f in dataclasses.fields(_architectures.HybridLayer)]
+      self._hybrid_layers = (_lib.IxtLayer * len(config.hybrid_layers))(
+          *[_lib.IxtLayer(**{n: getattr(l, n) for n in fields}) for l in config.hybrid_layers])
+      c.layers, c.num_decoder_layers = self._hybrid_layers, len(config.hybrid_layers)
+      c.embedding_scale, c.float32 = float(config.embedding_scale), 1 if config.dtype == "float32" else 0
+    elif config.dtype != "bfloat16":
+      raise NotImplementedError(f"dtype {config.dtype}: only decoder_block hybrid runs in float32")
+    elif config.decoder_block in ("gemma2", "gemma3"):   # layers/gemma2.py:69-236, layers/gemma3.py:35-200
       if tuple(config.mlp_activations) != ("gelu", "linear"):
         raise ValueError(f"decoder_block {config.decoder_block} is built with mlp_activations ['gelu', 'linear']")
       c.decoder_block = _lib.BLOCK_GEMMA2 if config.decoder_block == "gemma2" else _lib.BLOCK_GEMMA3
@@ -134,6 +144,7 @@ class MaxEngine(engine_api.Engine):
     self._result = torch.zeros((B, 3), dtype=torch.int32, device=self.device)
     self._first = torch.zeros((1,), dtype=torch.int32, device=self.device)
     self._page_failures = 0
+    self._recurrent = any(l.mixer == _architectures.MIX_GATED_DELTA for l in config.hybrid_layers) if config.decoder_block == "hybrid" else False
     self._status_host = torch.zeros((4,), dtype=torch.int32).pin_memory()   # deferred reservation check of the packed prefill
     self._status_event = None
     self._status_what = ""
@@ -184,6 +195,15 @@ class MaxEngine(engine_api.Engine):
     out = (ctypes.c_int32 * 1)()
     _lib.check(self.lib.ixt_exchange_status(self._ctx, out, 1 if reset else 0, ctypes.c_void_p(_stream_ptr())))
     return int(out[0])
+
+  def _check_state(self, what: str) -> None:
+    """Layers that carry a state: a run of tokens must continue where its slot's state stands (a state cannot be rewound the way pages can)."""
+    if not self._recurrent:
+      return
+    out = (ctypes.c_int32 * 1)()
+    _lib.check(self.lib.ixt_state_status(self._ctx, out, 1, ctypes.c_void_p(_stream_ptr())))
+    if out[0]:
+      raise ValueError(f"{what}: the tokens do not continue where the recurrent state of their slot stands; they were not computed")
 
   def close(self) -> None:
     """Give the engine's HBM (weights copy, page pools, workspaces) back now; the engine cannot be used afterwards.  Handles returned by
@@ -282,6 +302,8 @@ class MaxEngine(engine_api.Engine):
     first = torch.empty((1, 1), dtype=torch.int32, device=self.device)
     _lib.check(self.lib.ixt_prefill_chunk(self._ctx, slot, ctypes.c_void_p(toks.data_ptr()), true_length, start,
                                           ctypes.c_void_p(first.data_ptr()), ctypes.c_void_p(logits.data_ptr()), ctypes.c_void_p(_stream_ptr())))
+    if start > 0:
+      self._check_state("prefill")
     prompt_logp = None
     if return_prompt_logp:     # maxengine.py:477-478: log_softmax(logits[t])[tokens[t]] per position; positions past true_length (padding) hold 0
       prompt_logp = torch.zeros((1, toks.numel()), dtype=torch.float32, device=self.device)
@@ -379,6 +401,66 @@ class MaxEngine(engine_api.Engine):
     cache = PagedCacheHandle(self, None, 0, groups=[B + i for i in range(n)], lengths=lens)
     return cache, prefill_results, results
 
+  # ------------------------------------------------------------------ mixed batches
+  def step(self, entries, want_logits: bool = True):
+    """One batch of portions of prompts and single decoded tokens (no counterpart in the reference engine, whose prefill and generate are separate
+    programs, maxengine.py:400-936).  entries: [(slot, tokens already in the slot, next tokens, places among them whose logits are wanted)].
+    A slot that holds nothing gets fresh pages, otherwise its pages grow.  -> (logits f32 [wanted, vocab] or None, greedy tokens int32 [wanted])."""
+    self._settle_pages()
+    rows, wanted = [], 0
+    for slot, start, tokens, want in entries:
+      n = len(tokens)
+      if slot < 0 or slot >= self._B or n <= 0 or any(w < 0 or w >= n for w in want):
+        raise ValueError(f"step: slot {slot} (of {self._B}), {n} tokens, wanted places {list(want)}")
+      if start == 0:
+        self.page_state = self.page_manager.update_prefill_pages(page_state=self.page_state, page_group_id=slot, true_length=n)
+      else:
+        self.page_state = self.page_manager.extend_prefill_pages(page_state=self.page_state, page_group_id=slot, total_length=start + n)
+      rows.append((slot, start, np.asarray(tokens, np.int32), list(want), wanted))
+      wanted += len(want)
+    self._check_pages("step")
+    V = self.config.vocab_size
+    out_tok = torch.empty((wanted,), dtype=torch.int32, device=self.device)
+    out_lg = torch.empty((wanted, V), dtype=torch.float32, device=self.device) if want_logits else None
+    # passes of at most _packed_rows rows; an entry that does not fit is cut like any other portion
+    passes, room = [], 0
+    for slot, start, toks, want, w0 in rows:
+      done = 0
+      while done < len(toks):
+        if room == 0:
+          passes.append([])
+          room = self._packed_rows
+        n = min(room, len(toks) - done)
+        passes[-1].append((slot, start + done, toks[done:done + n], [(w - done, w0 + i) for i, w in enumerate(want) if done <= w < done + n]))
+        done += n
+        room -= n
+    for part in passes:
+      tok = np.concatenate([p[2] for p in part])
+      grp = np.concatenate([np.full(len(p[2]), p[0], np.int32) for p in part])
+      pos = np.concatenate([np.arange(p[1], p[1] + len(p[2]), dtype=np.int32) for p in part])
+      base, lrows, dest = 0, [], []
+      for p in part:
+        lrows += [base + w for w, _ in p[3]]
+        dest += [d for _, d in p[3]]
+        base += len(p[2])
+      n_want = len(lrows)
+      if n_want == 0 and self.config.decoder_block != "hybrid":
+        lrows = [base - 1]                                       # the other blocks always unembed a row
+      desc = torch.from_numpy(np.concatenate([tok, grp, pos, np.asarray(lrows, np.int32)])).to(self.device)
+      n = len(tok)
+      first = torch.empty((max(len(lrows), 1),), dtype=torch.int32, device=self.device)
+      lg = torch.empty((len(lrows), V), dtype=torch.float32, device=self.device) if want_logits and lrows else None
+      at = lambda k: ctypes.c_void_p(desc.data_ptr() + 4 * k)
+      _lib.check(self.lib.ixt_prefill_rows(self._ctx, n, at(0), at(n), at(2 * n), int(pos.max()) + 1, len(lrows), at(3 * n), ctypes.c_void_p(first.data_ptr()),
+                                           ctypes.c_void_p(lg.data_ptr()) if lg is not None else None, ctypes.c_void_p(_stream_ptr())))
+      if n_want:
+        d = torch.tensor(dest, dtype=torch.int64, device=self.device)
+        out_tok[d] = first[:n_want]
+        if lg is not None:
+          out_lg[d] = lg[:n_want]
+    self._check_state("step")
+    return out_lg, out_tok
+
   # ------------------------------------------------------------------ generate
   def generate(self, params: Params, decode_state: DecodeState, sampler: Any = None, rng: Any = None) -> Tuple[DecodeState, engine_api.ResultTokens]:
     """maxengine.py:838-936: page advance + one token for all slots + state update, in one library call."""
@@ -411,6 +493,7 @@ class MaxEngine(engine_api.Engine):
       if handle.slot != slot:
         _lib.check(self.lib.ixt_pages_copy(self._ctx, handle.slot, slot, handle.length, st))
         self._check_pages("insert")
+        self._check_state("insert")
       _lib.check(self.lib.ixt_pages_resync(self._ctx, slot, handle.length, st))
     decode_state["next_pos"][slot] = prefix["next_pos"][0]
     decode_state["generated_tokens"][slot] = prefix["generated_tokens"][0]
@@ -468,6 +551,8 @@ class MaxEngine(engine_api.Engine):
 
   def gather_kv(self, layer: int, slot: int, length: int):
     c = self.config
+    if c.decoder_block == "hybrid":
+      raise NotImplementedError("gather_kv: a hybrid decoder caches latents and states, not keys and values per head")
     k = torch.empty((length, c.num_kv_heads, c.head_dim), dtype=torch.bfloat16, device=self.device)
     v = torch.empty_like(k)
     _lib.check(self.lib.ixt_kv_gather(self._ctx, layer, slot, length, ctypes.c_void_p(k.data_ptr()), ctypes.c_void_p(v.data_ptr()),

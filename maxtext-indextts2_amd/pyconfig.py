@@ -168,8 +168,12 @@ def _derive(keys: Dict[str, Any]) -> None:
     keys["pagedattn_max_pages_per_group"] = -(-keys["max_target_length"] // keys["pagedattn_tokens_per_page"])
   if keys["attention"] not in VALID_ATTENTION:
     raise ValueError(f"Invalid attention {keys['attention']}; valid: {VALID_ATTENTION}")
-  if keys["decoder_block"] not in ("llama2", "default", "gemma2", "gemma3", "mixtral"):
-    raise ValueError(f"decoder_block {keys['decoder_block']} is outside this build's hot path (llama2, gemma2, gemma3 and mixtral are built)")
+  if keys["decoder_block"] not in ("llama2", "default", "gemma2", "gemma3", "mixtral", "hybrid"):
+    raise ValueError(f"decoder_block {keys['decoder_block']} is outside this build's hot path (llama2, gemma2, gemma3, mixtral and hybrid are built)")
+  if keys["decoder_block"] == "hybrid" and not keys["hybrid_layers"]:
+    raise ValueError("decoder_block hybrid: the layers come from a model folder (ixt_model_dir)")
+  if keys["dtype"] not in ("bfloat16", "float32"):
+    raise ValueError(f"dtype {keys['dtype']}: bfloat16 and (decoder_block hybrid) float32 are built")
   if keys["decoder_block"] == "mixtral":
     if not 1 <= keys["num_experts_per_tok"] <= min(keys["num_experts"], 8) or keys["num_experts"] > 32:
       raise ValueError("mixtral: 1 <= num_experts_per_tok <= min(num_experts, 8) and num_experts <= 32")
@@ -202,6 +206,15 @@ def _resolve(argv: List[str], kwargs: Mapping[str, Any]) -> Dict[str, Any]:
       if twice:
         raise ValueError(f"Keys {twice} are overwritten from both the model and the environment/command line. This isn't allowed.")
     validate_and_update_keys(keys, model_keys, config_name=argv[1])
+  if keys["ixt_model_dir"]:                                 # a model folder: its config.json decides (architectures.py)
+    if name != "default":
+      raise ValueError(f"both model_name={name} and ixt_model_dir={keys['ixt_model_dir']} are given")
+    from . import architectures  # pylint: disable=import-outside-toplevel
+    found = architectures.read_model_dir(str(keys["ixt_model_dir"]))
+    twice = [k for k in found if k in overrides and k != "load_parameters_path"]
+    if twice:
+      raise ValueError(f"Keys {twice} are overwritten from both the model folder and the environment/command line. This isn't allowed.")
+    keys.update({k: v for k, v in found.items() if k not in overrides})
   _derive(keys)
   return keys
 
