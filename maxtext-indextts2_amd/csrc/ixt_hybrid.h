@@ -17,7 +17,7 @@ struct HLayer {
   void* pages = nullptr;                         // latent layer: [page][token][rankp + rotp]
   float *state = nullptr, *tails = nullptr;      // delta layer: [group][H][dv][dp], [group][2][taps - 1][C]
 };
-struct HTensor { std::vector<int64_t> shape; std::function<int(const void*, int, hipStream_t)> load; bool done = false; };
+struct HTensor { std::vector<int64_t> shape; std::function<int(const void*, int, hipStream_t)> load; bool done = false; };   // load empty: accepted, unused
 struct HybridModel {
   bool f32 = false, recurrent = false;
   size_t esz = 2;                                // bytes per activation / weight element
@@ -172,7 +172,9 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     TRY(h_mat(c, &L.o, g.H * g.dv, E));
     mat("mix.o", L.o, E, g.H * g.dv, 0);
   }
-  if (l.ffn != IXT_FFN_NONE) {
+  if (l.ffn == IXT_FFN_NONE) {
+    m->tensors[p + "norm2"] = HTensor{{E}, nullptr, true};       // a layer without a feed-forward has no use for its norm
+  } else {
     TRY(vec("norm2", &L.n2, E, {E}));
     const int Fp = up_to(l.ff, IXT_KALIGN), n = l.ffn == IXT_FFN_MOE ? l.experts : 1;
     TRY(h_mat(c, &L.gu, E, 2 * Fp, n));
@@ -289,7 +291,8 @@ static int hybrid_init(ixt_ctx* c) {
   }
   for (int i = 0; i < n; ++i)
     if (m->layers[i].src == i) TRY(hybrid_layer_params(c, i));
-  m->missing = m->tensors.size();
+  m->missing = 0;
+  for (auto& kv : m->tensors) m->missing += kv.second.done ? 0 : 1;
   upd(part, (size_t)c->NLmax * m->head.Np * (c->NLmax < 128 ? (m->head.Kp + IXT_CHAIN - 1) / IXT_CHAIN : 1));
   c->part_floats = part; TRY(h_allocf(c, &c->part, part));
   m->part2_floats = part2; TRY(h_allocf(c, &m->part2, part2 + 4));
@@ -335,7 +338,7 @@ static int hybrid_load_weight(ixt_ctx* c, const std::string& name, const void* s
     for (int64_t v : t.shape) want += (want.empty() ? "" : " x ") + std::to_string(v);
     return set_err(IXT_ERR_INVALID, "%s: expected %s", name.c_str(), want.c_str());
   }
-  TRY(t.load(src, dtype, st));
+  if (t.load) TRY(t.load(src, dtype, st));
   if (!t.done) { t.done = true; --m->missing; }
   return IXT_OK;
 }

@@ -183,8 +183,37 @@ def synth_weights_mixtral(cfg, seed: int = 0) -> Dict[str, np.ndarray]:
   return w
 
 
+def synth_weights_hybrid(cfg, seed: int = 0) -> Dict[str, np.ndarray]:
+  """Random parameters of a hybrid decoder (architectures.parameter_shapes): linear weights N(0, 1 / fan_in), norms around their neutral value,
+  decays between about exp(-4) and 1."""
+  from . import architectures  # pylint: disable=import-outside-toplevel
+  rng = np.random.Generator(np.random.PCG64(seed))
+  w: Dict[str, np.ndarray] = {}
+  for name, shape in architectures.parameter_shapes(cfg).items():
+    z = rng.standard_normal(int(np.prod(shape)), dtype=np.float32).reshape(shape)
+    leaf = name.rsplit(".", 1)[-1]
+    if name == "embed":
+      z = z * np.float32(1.0 / cfg.embedding_scale)
+    elif leaf == "A_log":
+      z = np.float32(0.5) * z
+    elif leaf == "dt_bias":
+      z = z - np.float32(1.0)
+    elif leaf == "conv":
+      z = z * np.float32(1.0 / math.sqrt(shape[1]))
+    elif leaf in ("norm1", "norm2") or name == "final.norm":      # stored around zero
+      z = np.float32(0.1) * z
+    elif leaf == "norm":                                          # plain
+      z = np.float32(1.0) + np.float32(0.1) * z
+    else:
+      z = z * np.float32(1.0 / math.sqrt(shape[-1]))
+    w[name] = f32_to_bf16_bits(z).reshape(shape)
+  return w
+
+
 def synth_weights(cfg, seed: int = 0) -> Dict[str, np.ndarray]:
   """cfg needs vocab_size, emb_dim, num_query_heads, num_kv_heads, head_dim, mlp_dim, num_decoder_layers."""
+  if getattr(cfg, "decoder_block", "llama2") == "hybrid":
+    return synth_weights_hybrid(cfg, seed)
   if getattr(cfg, "decoder_block", "llama2") == "mixtral":
     return synth_weights_mixtral(cfg, seed)
   if getattr(cfg, "decoder_block", "llama2") == "gemma2":
