@@ -69,6 +69,7 @@ static int forward_rows_hybrid(ixt_ctx* c, int R, const int32_t* tokens, int len
 struct ixt_ctx {
   ixt_config cfg;
   HybridModel* hy = nullptr;
+  bool one_segment = false;    // the rows of the running call belong to one page group (ixt_prefill_chunk)
   int E, Q, KV, D, F, V, L, P, B, Rmax, NQKV, QN, KN, Tmax, mpg, nsb_max, GQ;
   int G = 0, S = 0;            // page groups = B decode slots + S staging groups of packed prefill
   int NLmax = 1;               // rows that can be unembedded in one call (decode slots / prompts of a packed prefill)
@@ -1973,7 +1974,10 @@ extern "C" int ixt_prefill_chunk(ixt_ctx* c, int slot, const int32_t* tokens_dev
   hipLaunchKernelGGL(k_rows_prefill, dim3((n_tokens + 255) / 256), dim3(256), 0, st, c->row_slot, c->row_pos, c->row_active, slot, start_pos, n_tokens,
                      c->ps.num_pages_used, c->P);
   LAUNCHCHK();
-  return forward_rows(c, n_tokens, tokens_dev, start_pos + n_tokens, n_tokens - 1, 1, nullptr, first_token_dev, last_logits_dev, false, st);
+  c->one_segment = true;
+  const int rc = forward_rows(c, n_tokens, tokens_dev, start_pos + n_tokens, n_tokens - 1, 1, nullptr, first_token_dev, last_logits_dev, false, st);
+  c->one_segment = false;
+  return rc;
 }
 
 // maxengine.py:477-478 (`return_prompt_logp`): log_softmax(logits[t])[tokens[t]] of every row t of the chunk the last ixt_prefill_chunk call

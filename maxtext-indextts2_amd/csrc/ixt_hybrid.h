@@ -256,7 +256,7 @@ static int hybrid_init(ixt_ctx* c) {
       dotsz(up_to(g.H * l.vdim, IXT_KALIGN), up_to(m->E, 16));
       upd(act_k, up_to(g.H * l.vdim, IXT_KALIGN));
       upd(qx_e, (size_t)g.H * Rp * dnp); upd(qr_e, (size_t)R * g.H * g.rotp); upd(olat_e, (size_t)g.H * Rp * kp);
-      upd(po, (size_t)(512 + g.H) * 16 * g.rankp);
+      upd(po, (size_t)(1024 + g.H) * 16 * g.rankp);
     } else {
       m->recurrent = true;
       DeltaGeom& g = L.dg;
@@ -307,7 +307,7 @@ static int hybrid_init(ixt_ctx* c) {
   TRY(h_allocf(c, &m->dec, s_dec + 4)); TRY(h_allocf(c, &m->beta, s_b + 4)); TRY(h_allocf(c, &m->dout, s_v + 4));
   TRY(h_allocf(c, &m->zlog, z_e + 4)); TRY(h_allocf(c, &m->mw, mi + 4)); TRY(h_allocf(c, &m->midx, mi + 4)); TRY(h_allocf(c, &m->mpos, mi + 4));
   TRY(h_allocf(c, &m->mrb, (size_t)m->moe_cap / 16 + 16));
-  TRY(h_allocf(c, &m->po, po + 4)); TRY(h_allocf(c, &m->pml, (size_t)(512 + m->maxH) * 16 * 2 + 4));
+  TRY(h_allocf(c, &m->po, po + 4)); TRY(h_allocf(c, &m->pml, (size_t)(1024 + m->maxH) * 16 * 2 + 4));
   TRY(h_allocf(c, &m->row_seg, (size_t)R)); TRY(h_allocf(c, &m->row_j, (size_t)R)); TRY(h_allocf(c, &m->seg, (size_t)R * 8)); TRY(h_allocf(c, &m->nseg, 4));
   TRY(h_allocf(c, &m->state_len, (size_t)c->G)); TRY(h_allocf(c, &m->parity, (size_t)c->G)); TRY(h_allocf(c, &m->claim, (size_t)c->G)); TRY(h_allocf(c, &m->err, 4));
   TRY(h_allocf(c, &m->head_rb, (size_t)m->maxH * Rp / 16 + 16));
@@ -355,6 +355,13 @@ static int hybrid_copy_group(ixt_ctx* c, int src, int dst, int npages, hipStream
 // ---------------------------------------------------------------------------------------------------- the forward pass
 template <typename T> static int hdot(ixt_ctx* c, const T* x, const HMat& w, int R, float* out, size_t out_floats, hipStream_t st, Slices* res);
 template <> int hdot<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, int R, float* out, size_t out_floats, hipStream_t st, Slices* res) {
+  if (R <= c->small_rows && (size_t)R * w.Np <= out_floats && w.Np <= 65536 && sdot_plan(c, GEPI_F32, false, w.Kp, w.Np, R).ok) {     // few rows: one slice
+    GemmEpi e{};
+    e.out = out;
+    TRY(launch_sdot(c, GEPI_F32, false, x, nullptr, (const bf16_t*)w.w, w.Kp, w.Np, R, e, st));
+    *res = Slices{out, 1, (size_t)R * w.Np, w.Np};
+    return IXT_OK;
+  }
   DotResult dr;
   TRY(launch_dot(c, x, (const bf16_t*)w.w, w.Kp, w.Np, R, out, out_floats, false, st, &dr));
   *res = Slices{out, dr.slices, dr.slice_stride, w.Np};
@@ -402,6 +409,11 @@ template <> int hglu<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, size_t 
     e.act = out; e.glu = 1; e.glu_limit = limit; e.rb_exp = rb; e.wstride = stride / 8;
     return launch_ring(c, GEPI_SWIGLU, x, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, false, st);
   }
+  if (!rb && rows <= c->small_rows && sdot_plan(c, GEPI_SWIGLU, false, w.Kp, w.Np, rows).ok) {
+    GemmEpi e{};
+    e.act = out; e.glu = 1; e.glu_limit = limit;
+    return launch_sdot(c, GEPI_SWIGLU, false, x, nullptr, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, st);
+  }
   const int rowblocks = (rows + 15) / 16, nrb = rb ? 1 : (rowblocks >= 3 ? 4 : rowblocks), zblocks = (rowblocks + nrb - 1) / nrb, ntile = w.Np / 16;
   dim3 grid((((ntile + 3) / 4 + 7) / 8) * 8 * zblocks, 1, 1);
   const u32x4 *xp = reinterpret_cast<const u32x4*>(x), *wp = reinterpret_cast<const u32x4*>(w.w);
@@ -424,19 +436,20 @@ template <> int hglu<float>(ixt_ctx* c, const float* x, const HMat& w, size_t st
 
 template <int RT, int RS>
 static int latent_launch(bool tall, int H, int splits, LatentAttnArgs a, hipStream_t st) {
-  constexpr size_t one = (size_t)32 * latent_pitch<RT, RS>() * 2;
+  constexpr size_t tile = LatentTile<RT, RS>::BYTES;
+  static bool attr_done = false;
+  if (!attr_done) {
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RT, RS>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)(2 * tile)));
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_decode<RT, RS>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)tile));
+    attr_done = true;
+  }
   if (tall) {
     a.HB = std::min(H, 64); a.NQ = std::max(1, 64 / a.HB);
-    hipLaunchKernelGGL((k_latent_attn<RT, RS, 4>), dim3((a.R + a.NQ - 1) / a.NQ, (H + a.HB - 1) / a.HB), dim3(256), one, st, a);
+    hipLaunchKernelGGL((k_latent_attn<RT, RS>), dim3((a.R + a.NQ - 1) / a.NQ, (H + a.HB - 1) / a.HB), dim3(256), 2 * tile, st, a);
   } else {
-    static bool attr_done = false;
-    if (!attr_done) {
-      HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<RT, RS, 1>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)(4 * one)));
-      attr_done = true;
-    }
     const int hg = (H + 15) / 16;
     a.HB = (H + hg - 1) / hg; a.NQ = 1;
-    hipLaunchKernelGGL((k_latent_attn<RT, RS, 1>), dim3(a.R, (H + a.HB - 1) / a.HB, splits), dim3(256), 4 * one, st, a);
+    hipLaunchKernelGGL((k_latent_decode<RT, RS>), dim3(a.R, (H + a.HB - 1) / a.HB, splits), dim3(256), tile, st, a);
   }
   LAUNCHCHK();
   return IXT_OK;
@@ -452,10 +465,8 @@ static int latent_attention(ixt_ctx* c, const HLayer& L, const Slices& qa, int R
       const bool tall = !decode && R > 32;
       const int hg = (g.H + 15) / 16, span = g.window > 0 ? std::min(g.window, len_hint) : len_hint;
       int splits = 1;
-      if (!tall) {                                         // a block per CU and at least a tile per wave
-        splits = std::min(std::min(16, std::max(1, 256 / (R * hg))), std::max(1, (span + 127) / 128));
-      }
-      LatentAttnArgs a{qa, (const bf16_t*)m->qr, g, c->row_slot, c->row_pos, c->row_active, c->ps.page_map, (const bf16_t*)L.pages, R, Rp, 1, 1, (bf16_t*)m->olat, Kp, m->po, m->pml};
+      if (!tall) splits = std::min(std::min(16, std::max(1, 512 / (R * hg))), std::max(1, (span + 63) / 64));     // two blocks per CU, at least a tile each
+      LatentAttnArgs a{qa, (const bf16_t*)m->qr, g, c->row_slot, c->row_pos, c->row_active, c->ps.page_map, (const bf16_t*)L.pages, R, Rp, 1, 1, __builtin_ctz(c->P), (bf16_t*)m->olat, Kp, m->po, m->pml};
       int rc = IXT_ERR_UNSUPPORTED;
       if (g.rotp == 32) {
         if (g.rankp == 64) rc = latent_launch<4, 1>(tall, g.H, splits, a, st);
@@ -500,7 +511,7 @@ static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int
 }
 
 template <typename T>
-static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, hipStream_t st, Slices* out) {
+static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st, Slices* out) {
   HybridModel* m = c->hy;
   const DeltaGeom& g = L.dg;
   Slices t, t2;
@@ -508,20 +519,24 @@ static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int 
   hipLaunchKernelGGL((k_lowrank_x<T>), dim3(R), dim3(128), 0, st, t, g, (T*)m->act, W.low.Kp);
   LAUNCHCHK();
   TRY(hdot<T>(c, (const T*)m->act, W.low, R, m->part2, m->part2_floats, st, &t2));
+  if (single) {            // every row is a segment of one token
+    DeltaStepArgs da{t, t2, g, W.cq, W.ck, W.cv, W.a_log, W.dt_bias, W.onorm, m->eps, m->row_seg, m->row_j, m->seg, L.tails, L.state};
+    const dim3 grid(R, g.H);
+    const size_t lds = sizeof(float) * (3 * g.dp + 2 * g.dv);
+#define HSTEP(RP_) case RP_: hipLaunchKernelGGL((k_delta_step<T, RP_>), grid, dim3(256), lds, st, da, (T*)m->act, W.o.Kp); break
+    switch (g.dp / 16) { HSTEP(1); HSTEP(2); HSTEP(4); HSTEP(8); HSTEP(16); HSTEP(32); default: return set_err(IXT_ERR_UNSUPPORTED, "delta rule: %d key dims", g.d); }
+#undef HSTEP
+    LAUNCHCHK();
+    return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
+  }
   DeltaPrepArgs pa{t, t2, g, W.cq, W.ck, W.cv, W.a_log, W.dt_bias, m->row_seg, m->row_j, m->seg, L.tails, m->dq, m->dk, m->dkq, m->dv, m->dec, m->beta};
   hipLaunchKernelGGL(k_delta_prep, dim3(R, (g.KH + g.H + 3) / 4), dim3(256), 0, st, pa);
   LAUNCHCHK();
   DeltaScanArgs sa{g, m->seg, m->nseg, m->dq, m->dk, m->dkq, m->dv, m->dec, m->beta, L.state, m->dout};
   const dim3 grid(nseg_max, g.H, (g.dv + 15) / 16);
-  switch (g.dp / 16) {
-    case 1: hipLaunchKernelGGL((k_delta_scan<1>), grid, dim3(256), 0, st, sa); break;
-    case 2: hipLaunchKernelGGL((k_delta_scan<2>), grid, dim3(256), 0, st, sa); break;
-    case 4: hipLaunchKernelGGL((k_delta_scan<4>), grid, dim3(256), 0, st, sa); break;
-    case 8: hipLaunchKernelGGL((k_delta_scan<8>), grid, dim3(256), 0, st, sa); break;
-    case 16: hipLaunchKernelGGL((k_delta_scan<16>), grid, dim3(256), 0, st, sa); break;
-    case 32: hipLaunchKernelGGL((k_delta_scan<32>), grid, dim3(256), 0, st, sa); break;
-    default: return set_err(IXT_ERR_UNSUPPORTED, "delta rule: %d key dims", g.d);
-  }
+#define HSCAN(RP_) case RP_: hipLaunchKernelGGL((k_delta_scan<RP_>), grid, dim3(256), sizeof(float) * 6 * scan_tokens<RP_>() * 16 * RP_, st, sa); break
+  switch (g.dp / 16) { HSCAN(1); HSCAN(2); HSCAN(4); HSCAN(8); HSCAN(16); HSCAN(32); default: return set_err(IXT_ERR_UNSUPPORTED, "delta rule: %d key dims", g.d); }
+#undef HSCAN
   LAUNCHCHK();
   hipLaunchKernelGGL((k_delta_out<T>), dim3(R, (g.H + 3) / 4), dim3(256), 0, st, m->dout, t2, g, W.onorm, m->eps, m->row_seg, (T*)m->act, W.o.Kp);
   LAUNCHCHK();
@@ -571,6 +586,16 @@ static int hybrid_logits(ixt_ctx* c, int R, int lrow0, int nl, const int32_t* lr
 }
 
 template <typename T>
+static int hybrid_norm(ixt_ctx* c, const Slices& t, const int32_t* pos, const float* wts, int top, const float* w, int R, hipStream_t st) {
+  HybridModel* m = c->hy;
+#define HNORM(NI_) hipLaunchKernelGGL((k_post_norm<T, NI_>), dim3(R), dim3(256), 0, st, t, pos, wts, top, w, m->eps, m->E, m->Ep, m->x, (T*)m->xb)
+  if (m->Ep <= 2048) HNORM(1); else if (m->Ep <= 4096) HNORM(2); else if (m->Ep <= 8192) HNORM(4); else HNORM(6);
+#undef HNORM
+  LAUNCHCHK();
+  return IXT_OK;
+}
+
+template <typename T>
 static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int len_hint, int lrow0, int nl, const int32_t* lrows, int32_t* argmax_out, float* logits_out, bool decode,
                                  int nseg_max, hipStream_t st) {
   HybridModel* m = c->hy;
@@ -579,24 +604,21 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
                      m->recurrent ? 1 : 0, m->err, m->head_rb, m->maxH * (Rp / 16), Rp / 16);
   hipLaunchKernelGGL((k_embed_scaled<T>), dim3(R), dim3(256), 0, st, (const T*)m->embed, tokens, m->emb_scale, m->E, m->Ep, m->V, m->x, (T*)m->xb);
   LAUNCHCHK();
-  const size_t nlds = sizeof(float) * m->E;
   for (size_t i = 0; i < m->layers.size(); ++i) {
     const HLayer& L = m->layers[i];
     const HLayer& W = m->layers[L.src];
     Slices t;
     if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) TRY((hybrid_mixer_latent<T>(c, L, W, R, Rp, decode, len_hint, st, &t)));
-    else TRY((hybrid_mixer_delta<T>(c, L, W, R, nseg_max, st, &t)));
-    hipLaunchKernelGGL((k_post_norm<T>), dim3(R), dim3(256), nlds, st, t, (const int32_t*)nullptr, (const float*)nullptr, 0, W.n1, m->eps, m->E, m->Ep, m->x, (T*)m->xb);
-    LAUNCHCHK();
+    else TRY((hybrid_mixer_delta<T>(c, L, W, R, nseg_max, decode, st, &t)));
+    TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n1, R, st)));
     if (L.c.ffn == IXT_FFN_DENSE) {
       TRY(hglu<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu_limit, (T*)m->hact, st));
       TRY(hdot<T>(c, (const T*)m->hact, W.down, R, c->part, c->part_floats, st, &t));
-      hipLaunchKernelGGL((k_post_norm<T>), dim3(R), dim3(256), nlds, st, t, (const int32_t*)nullptr, (const float*)nullptr, 0, W.n2, m->eps, m->E, m->Ep, m->x, (T*)m->xb);
+      TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n2, R, st)));
     } else if (L.c.ffn == IXT_FFN_MOE) {
       TRY(hybrid_moe<T>(c, L, W, R, st, &t));
-      hipLaunchKernelGGL((k_post_norm<T>), dim3(R), dim3(256), nlds, st, t, m->mpos, m->mw, L.c.top, W.n2, m->eps, m->E, m->Ep, m->x, (T*)m->xb);
+      TRY((hybrid_norm<T>(c, t, m->mpos, m->mw, L.c.top, W.n2, R, st)));
     }
-    LAUNCHCHK();
     if (m->tap && !c->capturing) {
       if ((i + 1) * (size_t)R * m->E > m->tap_floats) return set_err(IXT_ERR_INVALID, "residual tap: buffer too small");
       HIPCHK(hipMemcpyAsync(m->tap + i * (size_t)R * m->E, m->x, sizeof(float) * (size_t)R * m->E, hipMemcpyDeviceToDevice, st));
@@ -608,7 +630,7 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
 }
 static int forward_rows_hybrid(ixt_ctx* c, int R, const int32_t* tokens, int len_hint, int lrow0, int nl, const int32_t* lrows, int32_t* argmax_out, float* logits_out, bool decode,
                                hipStream_t st) {
-  const int nseg_max = decode ? R : std::min(R, c->G);     // a page group has at most one run of rows in a call
+  const int nseg_max = decode ? R : std::min(R, c->one_segment ? 1 : c->G);     // a page group has at most one run of rows in a call
   if (c->hy->f32) return forward_rows_hybrid_t<float>(c, R, tokens, len_hint, lrow0, nl, lrows, argmax_out, logits_out, decode, nseg_max, st);
   return forward_rows_hybrid_t<bf16_t>(c, R, tokens, len_hint, lrow0, nl, lrows, argmax_out, logits_out, decode, nseg_max, st);
 }

@@ -235,45 +235,65 @@ __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ tabl
 
 // A sublayer's output t (slices, or the weighted sum of a row's expert outputs) -> RMS norm with a zero-centred weight -> residual:
 //   x <- x + t / sqrt(mean(t^2) + eps) * (1 + w);  xb = the new x as the next dot's operand.
-// pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  grid R, block 256, LDS E floats.
-template <typename T>
+// pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  A thread owns 8 consecutive features of every 2048 (NI times).  grid R, block 256.
+template <typename T, int NI>
 __global__ __launch_bounds__(256) void k_post_norm(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, const float* __restrict__ w, float eps,
                                                    int E, int Ep, float* __restrict__ x, T* __restrict__ xb) {
-  extern __shared__ __attribute__((aligned(16))) float tb[];
   __shared__ float red[4];
   const int r = blockIdx.x;
+  const bool vec = (E & 3) == 0;
+  float v[NI][8], xv[NI][8];
   float ss = 0.0f;
-  for (int k0 = threadIdx.x * 4; k0 < E; k0 += 1024) {
-    float v[4];
-    if (pos == nullptr) {
-      t.at4(r, k0, v);
-    } else {
-      v[0] = v[1] = v[2] = v[3] = 0.0f;
-      for (int j = 0; j < top; ++j) {
-        float u[4];
-        t.at4(pos[(size_t)r * top + j], k0, u);
-        const float wj = wts[(size_t)r * top + j];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = fmaf(wj, u[i], v[i]);
+  for (int i = 0; i < NI; ++i) {
+    const int k0 = i * 2048 + threadIdx.x * 8;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[i][j] = xv[i][j] = 0.0f;
+#pragma unroll
+    for (int q = 0; q < 8; q += 4) {
+      if (k0 + q >= E) continue;
+      if (pos == nullptr) {
+        t.at4(r, k0 + q, v[i] + q);
+      } else {
+        for (int j = 0; j < top; ++j) {
+          float u[4];
+          t.at4(pos[(size_t)r * top + j], k0 + q, u);
+          const float wj = wts[(size_t)r * top + j];
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[i][q + e] = fmaf(wj, u[e], v[i][q + e]);
+        }
+      }
+      if (vec) {
+        const float4 xx = *reinterpret_cast<const float4*>(x + (size_t)r * E + k0 + q);
+        xv[i][q] = xx.x; xv[i][q + 1] = xx.y; xv[i][q + 2] = xx.z; xv[i][q + 3] = xx.w;
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (k0 + q + e < E) xv[i][q + e] = x[(size_t)r * E + k0 + q + e];
       }
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (k0 + i < E) { ss = fmaf(v[i], v[i], ss); tb[k0 + i] = v[i]; }
+    for (int j = 0; j < 8; ++j)
+      if (k0 + j < E) ss = fmaf(v[i][j], v[i][j], ss);
   }
   const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
-  for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
-    float v[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int k = k0 + j;
-      v[j] = 0.0f;
-      if (k < E) {
-        v[j] = x[(size_t)r * E + k] + tb[k] * rs * (1.0f + w[k]);
-        x[(size_t)r * E + k] = v[j];
-      }
+  for (int i = 0; i < NI; ++i) {
+    const int k0 = i * 2048 + threadIdx.x * 8;
+    if (k0 >= Ep) continue;
+    float y[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) y[j] = k0 + j < E ? xv[i][j] + v[i][j] * rs * (1.0f + w[k0 + j]) : 0.0f;
+    if (vec) {
+#pragma unroll
+      for (int q = 0; q < 8; q += 4)
+        if (k0 + q < E) *reinterpret_cast<float4*>(x + (size_t)r * E + k0 + q) = make_float4(y[q], y[q + 1], y[q + 2], y[q + 3]);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        if (k0 + j < E) x[(size_t)r * E + k0 + j] = y[j];
     }
-    act_store8(xb, r, k0, Ep, v);
+    act_store8(xb, r, k0, Ep, y);
   }
 }
 
@@ -442,53 +462,118 @@ __global__ __launch_bounds__(256) void k_latent_attn_any(Slices qa, const T* __r
     if (tid + 256 * i < Kp) act_store1(out, h * Rp + r, tid + 256 * i, Kp, tid + 256 * i < g.rank ? acc[i] / l : 0.0f);
 }
 
-// The bf16 matrix-core form.  All heads of a row share the cached latent, so the tile's M side is (row, head) pairs: WM = 4 (prompts): 64 pairs = up
-// to 64 / HB consecutive rows x HB heads, a wave owns 16 pairs, the four waves share every 32-key tile; WM = 1 (decode): 16 pairs = the heads of one
-// row, the four waves take different key tiles (and blockIdx.z splits them further) and merge at the end.
-//   scores   D[key][pair] = mfma(A = cached rows, B = queries [latent | rotated]): a lane holds 4 + 4 keys of one pair
-//   weights  running maximum / sum per pair in f32, exp2; P packs to bf16 in registers -- the lane's own 8 keys ARE its operand of the next product
-//            when the cached rows are read with the same key order (4q .. 4q + 3, 16 + 4q .. 16 + 4q + 3 for lane group q)
-//   output   D[column][pair] = mfma(A = cached latent read column-wise (ds_read_b64_tr_b16), B = P)
+// The bf16 matrix-core forms.  All heads of a row share the cached latent, so the M side of the products is (row, head) pairs and every cached row is
+// read once for all of them.  Keys come in tiles of 64 by LDS-DMA (no registers in between); inside a group of 8 pieces of 16 bytes a row's pieces
+// are XORed with the row number, so that neither the score operand (16 rows x 16 bytes) nor the column-wise reads of the value operand
+// (ds_read_b64_tr_b16: 4 rows x 16 columns) pile up on a bank.
+//   scores   D[key][pair] = mfma(A = cached rows, B = queries [latent | rotated]): a lane holds 4 keys of one pair per product
+//   weights  running maximum / sum per pair in f32, exp2; P goes to bf16
+//   output   D[column][pair] = mfma(A = cached latent read column-wise, B = P)
 // RT = 16-column tiles of the padded latent, RS = 32-wide steps of the padded rotated part.
-// grid (ceil(R / NQ), ceil(H / HB), WM == 1 ? splits : 1), block 256.
 struct LatentAttnArgs {
   Slices qa; const bf16_t* qr; LatentGeom g;
   const int32_t *row_slot, *row_pos, *row_active, *page_map;
   const bf16_t* pages;
-  int R, Rp, NQ, HB;
+  int R, Rp, NQ, HB, pshift;
   bf16_t* out; int Kp;                     // act, row h Rp + r
   float *part_o, *part_ml;                 // splits > 1: [R H][splits][rankp], [R H][splits][2]
 };
-template <int RT, int RS> constexpr int latent_pitch() { return RT * 16 + RS * 32 + 8; }
-template <int RT, int RS, int WM>
+// A tile in LDS: groups of 8 pieces (64 features), each [64 rows][8 pieces]; piece c of row r lies at place c ^ (r & 7).  RS odd: a last group of 4 pieces,
+// [64 rows][4 pieces], place c ^ (r & 3).  A wave load (1 KiB) is 8 rows of a group (16 of the last), so all its addresses are two (three) row pointers
+// plus constants.
+template <int RT, int RS> struct LatentTile {
+  static_assert(RT % 4 == 0 && (RS == 1 || RS == 2), "whole groups of the latent; one group or half a group of the rotated part");
+  static constexpr int DK = RT * 16 + RS * 32, NKS = RT / 2 + RS, NG = DK / 64;                 // elements per row, score steps, full groups
+  static constexpr int BYTES = 64 * DK * 2;
+};
+// 64 cached rows -> LDS: `off` = the row that this lane's key (key lane of the tile) occupies in the pool
+template <int RT, int RS>
+__device__ __forceinline__ void latent_dma(const bf16_t* __restrict__ pages, int off, bf16_t* tile, int wave, int lane) {
+  typedef LatentTile<RT, RS> T;
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int o = __shfl(off, (wave + 4 * j) * 8 + (lane >> 3), 64);
+    const bf16_t* src = pages + (size_t)o * T::DK + ((lane & 7) ^ (lane >> 3)) * 8;
+#pragma unroll
+    for (int gr = 0; gr < T::NG; ++gr)
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + gr * 64),
+                                       (__attribute__((address_space(3))) void*)(tile + gr * 4096 + (wave + 4 * j) * 512), 16, 0, 0);
+  }
+  if constexpr (RS == 1) {
+    const int o = __shfl(off, wave * 16 + (lane >> 2), 64);
+    const bf16_t* src = pages + (size_t)o * T::DK + T::NG * 64 + ((lane & 3) ^ ((lane >> 2) & 3)) * 8;
+    __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src, (__attribute__((address_space(3))) void*)(tile + T::NG * 4096 + wave * 512), 16, 0, 0);
+  }
+}
+__device__ __forceinline__ int latent_row(const int32_t* __restrict__ prow, int key, int pshift) { return (prow[key >> pshift] << pshift) + (key & ((1 << pshift) - 1)); }
+__device__ __forceinline__ bf16x8 latent_q8(const LatentAttnArgs& a, int qrow, int c) {
+  float v[8];
+  a.qa.at4(qrow, c, v);
+  a.qa.at4(qrow, c + 4, v + 4);
+  u32x4 o;
+  o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3])); o.z = pack2(f2bf(v[4]), f2bf(v[5])); o.w = pack2(f2bf(v[6]), f2bf(v[7]));
+  return __builtin_bit_cast(bf16x8, o);
+}
+// where a lane reads in a tile (byte offsets; the rest of every address is a constant)
+struct LatentLane {
+  uint32_t k0, k1, kh;      // score operand: row r_in, even / odd steps of a full group, the half group
+  uint32_t v[4];            // value operand: row 4 q + a, column tiles 0 .. 3 of a group (lane 4 a + p of a 16-lane group: columns 4 p .. 4 p + 3)
+};
+__device__ __forceinline__ LatentLane latent_lane(int r_in, int cq) {
+  LatentLane L;
+  L.k0 = r_in * 128 + ((cq ^ (r_in & 7)) * 16);
+  L.k1 = r_in * 128 + (((4 + cq) ^ (r_in & 7)) * 16);
+  L.kh = r_in * 64 + ((cq ^ (r_in & 3)) * 16);
+  const int row = 4 * cq + (r_in >> 2), p = r_in & 3;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) L.v[i] = row * 128 + (((2 * i + (p >> 1)) ^ (row & 7)) * 16) + (p & 1) * 8;
+  return L;
+}
+// score operand of step ks, rows 16 n .. 16 n + 15
+template <int RT, int RS>
+__device__ __forceinline__ bf16x8 latent_kf(const char* tile, const LatentLane& L, int ks, int n) {
+  if (RS == 1 && ks == RT / 2) return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + L.kh + LatentTile<RT, RS>::NG * 8192 + n * 1024));
+  return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + ((ks & 1) ? L.k1 : L.k0) + (ks >> 1) * 8192 + n * 2048));
+}
+// value operand of column tiles 4 G .. 4 G + 3 (group G), keys 32 U + 4 q .. + 3 and 32 U + 16 + 4 q .. + 3 for lane group q; tb = LDS address of the tile
+#define IXT_LATENT_VT(F_, TB_, L_, G_, U_)                                                                                                                    \
+  do {                                                                                                                                                        \
+    _Pragma("unroll") for (int i_ = 0; i_ < 4; ++i_) {                                                                                                        \
+      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][0]) : "v"((TB_) + (L_).v[i_]), "n"((G_) * 8192 + (U_) * 4096) : "memory");              \
+      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][1]) : "v"((TB_) + (L_).v[i_]), "n"((G_) * 8192 + (U_) * 4096 + 2048) : "memory");       \
+    }                                                                                                                                                         \
+  } while (0)
+// all but the youngest N_ reads have been delivered: everything that uses F_ comes behind this
+#define IXT_LATENT_VWAIT(F_, N_)                                                                                                                                \
+  do {                                                                                                                                                        \
+    asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(N_) : "memory");                                                                                               \
+    __builtin_amdgcn_sched_barrier(0);                                                                                                                        \
+    _Pragma("unroll") for (int i_ = 0; i_ < 4; ++i_) asm volatile("" : "+v"(F_[i_][0]), "+v"(F_[i_][1]));                                                      \
+  } while (0)
+__device__ __forceinline__ uint32_t lds_addr(const void* p) { return (uint32_t)(uintptr_t)((const __attribute__((address_space(3))) void*)(p)); }
+__device__ __forceinline__ bf16x8 latent_vfrag(const uint2 (&f)[2]) {
+  u32x4 v; v.x = f[0].x; v.y = f[0].y; v.z = f[1].x; v.w = f[1].y;
+  return __builtin_bit_cast(bf16x8, v);
+}
+
+// Prompts: a block owns 64 pairs = up to 64 / HB consecutive rows x HB heads (a wave 16 of them), all waves walk the same key tiles, the next tile
+// arriving while the current one is used.  P stays in registers: with the key order 4q .. 4q + 3, 16 + 4q .. 16 + 4q + 3 per lane group q of 32
+// keys, the lane's own scores ARE its operand of the next product.  grid (ceil(R / NQ), ceil(H / HB)), block 256, LDS two tiles.
+template <int RT, int RS>
 __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentAttnArgs a) {
-  constexpr int DK = RT * 16 + RS * 32, PITCH = latent_pitch<RT, RS>(), CPR = DK / 8;
-  constexpr int NTH = WM == 4 ? 256 : 64;                 // threads that stage one tile
-  constexpr int NC = (32 * CPR + NTH - 1) / NTH;          // 16-byte pieces per thread
-  constexpr int NKS = RT / 2 + RS;                        // k-steps of the scores
+  typedef LatentTile<RT, RS> T;
   extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
-  __shared__ float s_m[4][16], s_l[4][16];
   const LatentGeom& g = a.g;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
   const int r0 = blockIdx.x * a.NQ, nr = min(a.NQ, a.R - r0), h0 = blockIdx.y * a.HB, hb = min(a.HB, g.H - h0);
-  bf16_t* tile = WM == 4 ? lds : lds + (size_t)wave * 32 * PITCH;
-  const int pair = (WM == 4 ? wave * 16 : 0) + r_in;
-  const int qi = pair / a.HB, hh = pair % a.HB;
+  const int pair = wave * 16 + r_in, qi = pair / a.HB, hh = pair % a.HB;
   const bool pair_ok = qi < nr && hh < hb;
   const int row = r0 + (pair_ok ? qi : 0), head = h0 + (pair_ok ? hh : 0);
   const bool live = pair_ok && a.row_active[row] != 0;
   const int pos = live ? a.row_pos[row] : -1;
-  // queries: lane = pair r_in, 8 consecutive features per step
-  bf16x8 qf[NKS];
+  bf16x8 qf[T::NKS];                                      // queries: lane = pair r_in, 8 consecutive features per step
 #pragma unroll
-  for (int ks = 0; ks < RT / 2; ++ks) {
-    float v[8];
-    a.qa.at4(head * a.Rp + row, ks * 32 + cq * 8, v);
-    a.qa.at4(head * a.Rp + row, ks * 32 + cq * 8 + 4, v + 4);
-    u32x4 o;
-    o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3])); o.z = pack2(f2bf(v[4]), f2bf(v[5])); o.w = pack2(f2bf(v[6]), f2bf(v[7]));
-    qf[ks] = __builtin_bit_cast(bf16x8, o);
-  }
+  for (int ks = 0; ks < RT / 2; ++ks) qf[ks] = latent_q8(a, head * a.Rp + row, ks * 32 + cq * 8);
 #pragma unroll
   for (int ks = 0; ks < RS; ++ks)
     qf[RT / 2 + ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.qr + ((size_t)row * g.H + head) * g.rotp + ks * 32 + cq * 8));
@@ -497,8 +582,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentAttnArgs a) {
   for (int i = 0; i < RT; ++i) o[i] = f32x4(0.0f);
   float m = -INFINITY, l = 0.0f;
   const float sc = g.scale * 1.44269504088896340736f;
-
-  u32x4 stg[NC];
+  const LatentLane L = latent_lane(r_in, cq);
   for (int ra = 0; ra < nr;) {                            // runs of rows that share a page group
     if (!a.row_active[r0 + ra]) { ++ra; continue; }
     const int slot = a.row_slot[r0 + ra];
@@ -507,139 +591,229 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentAttnArgs a) {
     const bool mine = live && qi >= ra && qi < rb;
     ra = rb;
     const int k_lo = g.window > 0 ? max(0, lo - g.window + 1) : 0;
-    const int ntile = (hi - k_lo) / 32 + 1;
+    const int ntile = (hi - k_lo) / 64 + 1;
     const int32_t* prow = a.page_map + (size_t)slot * g.mpg;
     const int my_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
-    const int t0 = WM == 4 ? 0 : (int)blockIdx.z * 4 + wave, tstep = WM == 4 ? 1 : 4 * (int)gridDim.z;
-    auto fetch = [&](int t) {
+    __syncthreads();                                      // the previous run's last tile has been read
+    int off = latent_row(prow, min(k_lo + lane, hi), a.pshift);
+    latent_dma<RT, RS>(a.pages, off, lds, wave, lane);
+    off = latent_row(prow, min(k_lo + 64 + lane, hi), a.pshift);
+    for (int t = 0; t < ntile; ++t) {
+      const bf16_t* tile = lds + (size_t)(t & 1) * 64 * T::DK;
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      __syncthreads();                                    // the tile is there; every wave is done with the other one
+      if (t + 1 < ntile) {
+        latent_dma<RT, RS>(a.pages, off, lds + (size_t)((t + 1) & 1) * 64 * T::DK, wave, lane);
+        off = latent_row(prow, min(k_lo + (t + 2) * 64 + lane, hi), a.pshift);
+      }
+      f32x4 s[4];
 #pragma unroll
-      for (int i = 0; i < NC; ++i) {
-        const int c = (WM == 4 ? tid : lane) + i * NTH;
-        if ((32 * CPR) % NTH == 0 || c < 32 * CPR) {
-          const int key = min(k_lo + t * 32 + c / CPR, hi), pc = c % CPR;
-          stg[i] = *reinterpret_cast<const u32x4*>(a.pages + ((size_t)prow[key / g.P] * g.P + key % g.P) * DK + pc * 8);
+      for (int n = 0; n < 4; ++n) s[n] = f32x4(0.0f);
+      bf16x8 kf[2][4];                                    // operands one step ahead of the products
+#pragma unroll
+      for (int n = 0; n < 4; ++n) kf[0][n] = latent_kf<RT, RS>(reinterpret_cast<const char*>(tile), L, 0, n);
+#pragma unroll
+      for (int ks = 0; ks < T::NKS; ++ks) {
+        if (ks + 1 < T::NKS) {
+#pragma unroll
+          for (int n = 0; n < 4; ++n) kf[(ks + 1) & 1][n] = latent_kf<RT, RS>(reinterpret_cast<const char*>(tile), L, ks + 1, n);
         }
-      }
-    };
-    if (t0 < ntile) fetch(t0);
-    for (int t = t0; t < ntile; t += tstep) {
-      if constexpr (WM == 4) __syncthreads();              // every wave is done with the previous tile
 #pragma unroll
-      for (int i = 0; i < NC; ++i) {
-        const int c = (WM == 4 ? tid : lane) + i * NTH;
-        if ((32 * CPR) % NTH == 0 || c < 32 * CPR) *reinterpret_cast<u32x4*>(tile + (c / CPR) * PITCH + (c % CPR) * 8) = stg[i];
+        for (int n = 0; n < 4; ++n) s[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][n], qf[ks], s[n], 0, 0, 0);
+        __builtin_amdgcn_sched_barrier(0);
       }
-      if constexpr (WM == 4) __syncthreads();
-      else __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-      if (t + tstep < ntile) fetch(t + tstep);
-      f32x4 s0 = f32x4(0.0f), s1 = f32x4(0.0f);
-#pragma unroll
-      for (int ks = 0; ks < NKS; ++ks) {
-        const bf16x8 k0 = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + r_in * PITCH + ks * 32 + cq * 8));
-        const bf16x8 k1 = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + (16 + r_in) * PITCH + ks * 32 + cq * 8));
-        s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[ks], s0, 0, 0, 0);
-        s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[ks], s1, 0, 0, 0);
-      }
-      float sv[8];
       float tm = -INFINITY;
-      const int kb = k_lo + t * 32 + cq * 4;
+      const int kb = k_lo + t * 64 + cq * 4;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int key = kb + (j < 4 ? j : 12 + j);
-        const float v = (j < 4 ? s0[j & 3] : s1[j & 3]) * sc;
-        sv[j] = (mine && key <= pos && key >= my_lo) ? v : -INFINITY;
-        tm = fmaxf(tm, sv[j]);
-      }
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int key = kb + n * 16 + j;
+          s[n][j] = (mine && key <= pos && key >= my_lo) ? s[n][j] * sc : -INFINITY;
+          tm = fmaxf(tm, s[n][j]);
+        }
       tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
       tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
       const float mn = fmaxf(m, tm);
       const float al = mn == -INFINITY ? 1.0f : exp2f(m - mn);
-      float ls = 0.0f, pv[8];
+      float ls = 0.0f;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) { pv[j] = sv[j] == -INFINITY ? 0.0f : exp2f(sv[j] - mn); ls += pv[j]; }
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { s[n][j] = s[n][j] == -INFINITY ? 0.0f : exp2f(s[n][j] - mn); ls += s[n][j]; }
       ls += __shfl_xor(ls, 16, 64);
       ls += __shfl_xor(ls, 32, 64);
       l = l * al + ls;
       m = mn;
-      u32x4 pk;
-      pk.x = pack2(f2bf(pv[0]), f2bf(pv[1])); pk.y = pack2(f2bf(pv[2]), f2bf(pv[3])); pk.z = pack2(f2bf(pv[4]), f2bf(pv[5])); pk.w = pack2(f2bf(pv[6]), f2bf(pv[7]));
-      const bf16x8 pf = __builtin_bit_cast(bf16x8, pk);
       if (__any(al != 1.0f)) {
 #pragma unroll
-        for (int i = 0; i < RT; ++i) o[i] *= al;
+        for (int i = 0; i < RT; ++i) { o[i][0] *= al; o[i][1] *= al; o[i][2] *= al; o[i][3] *= al; }
       }
-      // lane 4 a + p of a 16-lane group addresses row 4 q + a, columns 4 p .. 4 p + 3, and receives its column of the 4 rows
-      const bf16_t* vb = tile + (4 * cq + (r_in >> 2)) * PITCH + 4 * (r_in & 3);
-      const uint32_t va = (uint32_t)(uintptr_t)((const __attribute__((address_space(3))) void*)(vb));
-      constexpr int VG = RT < 8 ? RT : 8;                  // tiles whose reads are in flight together
+      const uint32_t tb = lds_addr(tile);
 #pragma unroll
-      for (int i0 = 0; i0 < RT; i0 += VG) {
-        uint2 f[VG][2];
+      for (int u = 0; u < 2; ++u) {                       // 32 keys each
+        u32x4 pk;
+        pk.x = pack2(f2bf(s[2 * u][0]), f2bf(s[2 * u][1])); pk.y = pack2(f2bf(s[2 * u][2]), f2bf(s[2 * u][3]));
+        pk.z = pack2(f2bf(s[2 * u + 1][0]), f2bf(s[2 * u + 1][1])); pk.w = pack2(f2bf(s[2 * u + 1][2]), f2bf(s[2 * u + 1][3]));
+        const bf16x8 pf = __builtin_bit_cast(bf16x8, pk);
+        uint2 f[2][4][2];
+        IXT_LATENT_VT(f[0], tb, L, 0, u);
 #pragma unroll
-        for (int i = 0; i < VG; ++i) {
-          asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[i][0]) : "v"(va), "n"((i0 + i) * 32) : "memory");
-          asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[i][1]) : "v"(va), "n"((i0 + i) * 32 + 16 * PITCH * 2) : "memory");
-        }
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-        __builtin_amdgcn_sched_barrier(0);
+        for (int gr = 0; gr < RT / 4; ++gr) {             // the next group's reads travel under this one's products
+          if (gr + 1 < RT / 4) {
+            IXT_LATENT_VT(f[(gr + 1) & 1], tb, L, gr + 1, u);
+            IXT_LATENT_VWAIT(f[gr & 1], 8);
+          } else {
+            IXT_LATENT_VWAIT(f[gr & 1], 0);
+          }
 #pragma unroll
-        for (int i = 0; i < VG; ++i) asm volatile("" : "+v"(f[i][0]), "+v"(f[i][1]));     // the products read what the wait has delivered
-#pragma unroll
-        for (int i = 0; i < VG; ++i) {
-          u32x4 v; v.x = f[i][0].x; v.y = f[i][0].y; v.z = f[i][1].x; v.w = f[i][1].y;
-          o[i0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), pf, o[i0 + i], 0, 0, 0);
+          for (int i = 0; i < 4; ++i) o[gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_vfrag(f[gr & 1][i]), pf, o[gr * 4 + i], 0, 0, 0);
         }
       }
     }
   }
-  if constexpr (WM == 4) {
-    if (!live) return;
-    const float inv = l > 0.0f ? 1.0f / l : 0.0f;
+  if (!live) return;
+  const float inv = l > 0.0f ? 1.0f / l : 0.0f;
 #pragma unroll
-    for (int i = 0; i < RT; ++i) {
+  for (int i = 0; i < RT; ++i) {
+    const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+    act_store4(a.out, head * a.Rp + row, i * 16 + cq * 4, a.Kp, v);
+  }
+  const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int c = RT * 16 + cq * 4; c < a.Kp; c += 16) act_store4(a.out, head * a.Rp + row, c, a.Kp, z);
+}
+
+// Few rows (decode): a block owns the (at most 16) heads of ONE row and every gridDim.z-th key tile of its window.  Scores: a wave takes 16 of the 64
+// keys; P and the tile maxima meet in LDS; output: a wave takes a quarter of the latent columns.  One tile of LDS: two blocks share a CU and one's
+// loads run under the other's products.  grid (R, ceil(H / HB), splits), block 256.
+template <int RT, int RS>
+__global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
+  typedef LatentTile<RT, RS> T;
+  constexpr int OT = RT / 4;                              // column tiles per wave
+  extern __shared__ __attribute__((aligned(16))) bf16_t tile[];
+  __shared__ __attribute__((aligned(16))) bf16_t ps[16][72];
+  __shared__ float s_m[4][16], s_l[4][16];
+  const LatentGeom& g = a.g;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
+  const int row = blockIdx.x, h0 = blockIdx.y * a.HB, hb = min(a.HB, g.H - h0), nsplit = gridDim.z;
+  if (!a.row_active[row]) return;
+  const bool pair_ok = r_in < hb;
+  const int head = h0 + (pair_ok ? r_in : 0), pos = a.row_pos[row];
+  const int32_t* prow = a.page_map + (size_t)a.row_slot[row] * g.mpg;
+  const int k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0, ntile = (pos - k_lo) / 64 + 1;
+  int t = blockIdx.z;
+  if (t < ntile) latent_dma<RT, RS>(a.pages, latent_row(prow, min(k_lo + t * 64 + lane, pos), a.pshift), tile, wave, lane);
+  bf16x8 qf[T::NKS];
+#pragma unroll
+  for (int ks = 0; ks < RT / 2; ++ks) qf[ks] = latent_q8(a, head * a.Rp + row, ks * 32 + cq * 8);
+#pragma unroll
+  for (int ks = 0; ks < RS; ++ks)
+    qf[RT / 2 + ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.qr + ((size_t)row * g.H + head) * g.rotp + ks * 32 + cq * 8));
+  f32x4 o[OT];
+#pragma unroll
+  for (int i = 0; i < OT; ++i) o[i] = f32x4(0.0f);
+  float m = -INFINITY, l = 0.0f;                          // l: this lane's keys only
+  const float sc = g.scale * 1.44269504088896340736f;
+  const LatentLane L = latent_lane(r_in, cq);
+  [[maybe_unused]] const uint32_t tb = lds_addr(tile) + wave * (OT / 4) * 8192;                              // the wave's first column group
+  [[maybe_unused]] const uint32_t tg = lds_addr(tile) + (wave * OT / 4) * 8192;                              // fewer than 4 tiles per wave: the group they are in
+  for (; t < ntile; t += nsplit) {
+    int off = 0;
+    if (t + nsplit < ntile) off = latent_row(prow, min(k_lo + (t + nsplit) * 64 + lane, pos), a.pshift);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    f32x4 s = f32x4(0.0f);
+#pragma unroll
+    for (int ks = 0; ks < T::NKS; ++ks) {
+      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_kf<RT, RS>(reinterpret_cast<const char*>(tile) + wave * (RS == 1 && ks == RT / 2 ? 1024 : 2048), L, ks, 0), qf[ks], s, 0, 0, 0);
+    }
+    float tm = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      s[j] = k_lo + t * 64 + wave * 16 + cq * 4 + j <= pos ? s[j] * sc : -INFINITY;
+      tm = fmaxf(tm, s[j]);
+    }
+    tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+    tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+    if (cq == 0) s_m[wave][r_in] = tm;
+    __syncthreads();
+    const float mn = fmaxf(m, fmaxf(fmaxf(s_m[0][r_in], s_m[1][r_in]), fmaxf(s_m[2][r_in], s_m[3][r_in])));   // (a tile has at least one visible key: finite)
+    const float al = exp2f(m - mn);
+    float p[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) p[j] = exp2f(s[j] - mn);
+    l = l * al + ((p[0] + p[1]) + (p[2] + p[3]));
+    m = mn;
+    uint2 pk;
+    pk.x = pack2(f2bf(p[0]), f2bf(p[1])); pk.y = pack2(f2bf(p[2]), f2bf(p[3]));
+    *reinterpret_cast<uint2*>(&ps[r_in][wave * 16 + cq * 4]) = pk;
+    if (__any(al != 1.0f)) {
+#pragma unroll
+      for (int i = 0; i < OT; ++i) { o[i][0] *= al; o[i][1] *= al; o[i][2] *= al; o[i][3] *= al; }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {                         // lane group q holds keys 32 u + 4 q .. + 3 and 32 u + 16 + 4 q .. + 3 (as in k_latent_attn)
+      const uint2 p0 = *reinterpret_cast<const uint2*>(&ps[r_in][u * 32 + 4 * cq]), p1 = *reinterpret_cast<const uint2*>(&ps[r_in][u * 32 + 16 + 4 * cq]);
+      u32x4 pv; pv.x = p0.x; pv.y = p0.y; pv.z = p1.x; pv.w = p1.y;
+      const bf16x8 pf = __builtin_bit_cast(bf16x8, pv);
+      if constexpr (OT >= 4) {                            // whole column groups
+        uint2 f[2][4][2];
+        IXT_LATENT_VT(f[0], tb, L, 0, u);
+#pragma unroll
+        for (int gr = 0; gr < OT / 4; ++gr) {
+          if (gr + 1 < OT / 4) {
+            IXT_LATENT_VT(f[(gr + 1) & 1], tb, L, gr + 1, u);
+            IXT_LATENT_VWAIT(f[gr & 1], 8);
+          } else {
+            IXT_LATENT_VWAIT(f[gr & 1], 0);
+          }
+#pragma unroll
+          for (int i = 0; i < 4; ++i) o[gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_vfrag(f[gr & 1][i]), pf, o[gr * 4 + i], 0, 0, 0);
+        }
+      } else {                                            // OT column tiles, from place (wave OT) % 4 of one group on
+        uint2 f[4][2];
+        IXT_LATENT_VT(f, tg, L, 0, u);
+        IXT_LATENT_VWAIT(f, 0);
+        const int at = (wave * OT) & 3;
+#pragma unroll
+        for (int i = 0; i < OT; ++i) {
+          uint2 x = f[i][0], y = f[i][1];
+#pragma unroll
+          for (int k = 1; k + i < 4; ++k) {
+            const bool take = at == k;
+            x.x = take ? f[k + i][0].x : x.x; x.y = take ? f[k + i][0].y : x.y; y.x = take ? f[k + i][1].x : y.x; y.y = take ? f[k + i][1].y : y.y;
+          }
+          const uint2 xy[2] = {x, y};
+          o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_vfrag(xy), pf, o[i], 0, 0, 0);
+        }
+      }
+    }
+    __syncthreads();                                      // the tile has been read by every wave
+    if (t + nsplit < ntile) latent_dma<RT, RS>(a.pages, off, tile, wave, lane);
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (cq == 0) s_l[wave][r_in] = l;
+  __syncthreads();
+  l = (s_l[0][r_in] + s_l[1][r_in]) + (s_l[2][r_in] + s_l[3][r_in]);
+  if (!pair_ok) return;
+  if (nsplit == 1) {
+    const float inv = 1.0f / l;
+#pragma unroll
+    for (int i = 0; i < OT; ++i) {
       const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
-      act_store4(a.out, head * a.Rp + row, i * 16 + cq * 4, a.Kp, v);
+      act_store4(a.out, head * a.Rp + row, (wave * OT + i) * 16 + cq * 4, a.Kp, v);
     }
     const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-    for (int c = RT * 16 + cq * 4; c < a.Kp; c += 16) act_store4(a.out, head * a.Rp + row, c, a.Kp, z);
+    if (wave == 0)
+      for (int c = RT * 16 + cq * 4; c < a.Kp; c += 16) act_store4(a.out, head * a.Rp + row, c, a.Kp, z);
   } else {
-    float* ob = reinterpret_cast<float*>(tile);            // [16 pairs][RT * 16]: the wave's own tile region
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    const size_t pi = ((size_t)row * g.H + head) * nsplit + blockIdx.z;
 #pragma unroll
-    for (int i = 0; i < RT; ++i) *reinterpret_cast<float4*>(ob + r_in * (RT * 16) + i * 16 + cq * 4) = make_float4(o[i][0], o[i][1], o[i][2], o[i][3]);
-    if (cq == 0) { s_m[wave][r_in] = m; s_l[wave][r_in] = l; }
-    __syncthreads();
-    if (!a.row_active[r0]) return;
-    const int nsplit = gridDim.z;
-    for (int e = tid; e < hb * RT * 4; e += 256) {
-      const int pr = e / (RT * 4), c = (e % (RT * 4)) * 4;
-      float mm = -INFINITY;
-#pragma unroll
-      for (int w = 0; w < 4; ++w) mm = fmaxf(mm, s_m[w][pr]);
-      float ll = 0.0f, v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll
-      for (int w = 0; w < 4; ++w) {
-        const float f = s_m[w][pr] == -INFINITY ? 0.0f : exp2f(s_m[w][pr] - mm);
-        ll = fmaf(s_l[w][pr], f, ll);
-        const float4 u = *reinterpret_cast<const float4*>(reinterpret_cast<const float*>(lds + (size_t)w * 32 * PITCH) + pr * (RT * 16) + c);
-        v[0] = fmaf(u.x, f, v[0]); v[1] = fmaf(u.y, f, v[1]); v[2] = fmaf(u.z, f, v[2]); v[3] = fmaf(u.w, f, v[3]);
-      }
-      if (nsplit == 1) {
-        const float inv = ll > 0.0f ? 1.0f / ll : 0.0f;
-#pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] *= inv;
-        act_store4(a.out, (h0 + pr) * a.Rp + r0, c, a.Kp, v);
-      } else {
-        const size_t pi = ((size_t)r0 * g.H + h0 + pr) * nsplit + blockIdx.z;
-        *reinterpret_cast<float4*>(a.part_o + pi * (RT * 16) + c) = make_float4(v[0], v[1], v[2], v[3]);
-        if (c == 0) { a.part_ml[pi * 2] = mm; a.part_ml[pi * 2 + 1] = ll; }
-      }
-    }
-    if (nsplit == 1) {
-      const int pad4 = (a.Kp - RT * 16) / 4;
-      const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-      for (int e = tid; e < hb * pad4; e += 256) act_store4(a.out, (h0 + e / pad4) * a.Rp + r0, RT * 16 + (e % pad4) * 4, a.Kp, z);
-    }
+    for (int i = 0; i < OT; ++i)
+      *reinterpret_cast<float4*>(a.part_o + pi * (RT * 16) + (wave * OT + i) * 16 + cq * 4) = make_float4(o[i][0], o[i][1], o[i][2], o[i][3]);
+    if (wave == 0 && cq == 0) { a.part_ml[pi * 2] = m; a.part_ml[pi * 2 + 1] = l; }
   }
 }
 // the key splits of a row's heads put together.  grid (R, H), block 64.
@@ -697,7 +871,7 @@ __global__ __launch_bounds__(128) void k_lowrank_x(Slices t, DeltaGeom g, T* __r
 // one channel of a short causal convolution: taps[0 .. n-1], the last for the row itself.  Earlier inputs come from the segment's rows or, before
 // its start, from the group's tail (oldest first).  Returns the convolution and leaves the channel's next tail (rows among the segment's last
 // n - 1 write their input; the last row carries older entries over when the segment is shorter than the tail).
-struct ConvCtx { const float* tail_in; float* tail_out; int j, n, start; };
+struct ConvCtx { const float* tail_in; float* tail_out; int j, n, start; };      // tail_out nullptr: another block leaves the tail
 __device__ __forceinline__ float conv_channel(const Slices& t, int r, int col, const float* __restrict__ tp, int taps, int ch, int C, const ConvCtx& cc) {
   const float x0 = t.at(r, col);
   float acc = x0 * tp[taps - 1];
@@ -707,6 +881,7 @@ __device__ __forceinline__ float conv_channel(const Slices& t, int r, int col, c
     else if (cc.start > 0) v = cc.tail_in[(size_t)(taps - 1 - (b - cc.j)) * C + ch];
     acc = fmaf(v, tp[taps - 1 - b], acc);
   }
+  if (cc.tail_out == nullptr) return acc;
   const int dist = cc.n - 1 - cc.j;
   if (dist < taps - 1) cc.tail_out[(size_t)(taps - 2 - dist) * C + ch] = x0;
   if (dist == 0)
@@ -785,8 +960,9 @@ __device__ __forceinline__ float row16_sum(float v) {
 
 // The recurrence, per head:  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q, all f32.  The columns of S (value dims) never meet, so a
 // block owns 16 of them for one (segment, head): a wave four, 16 lanes per column with RP key rows each in registers.  o = (g S)^T q + (k . q) u: both
-// sums over the key rows are taken from the decayed state and run side by side.  Tokens come through LDS, TT at a time, the next ones already in
-// registers.  State [group][H][dv][dp]; a segment at position 0 starts from zero.  grid (segments, H, ceil(dv / 16)), block 256.
+// sums over the key rows are taken from the decayed state and run side by side.  q, k and the decays of TT tokens at a time come by LDS-DMA into one of
+// two buffers while the other is used; a token's operands are read into registers one token ahead.
+// State [group][H][dv][dp]; a segment at position 0 starts from zero.  grid (segments, H, ceil(dv / 16)), block 256, LDS 2 x 3 x TT x DP floats.
 struct DeltaScanArgs {
   DeltaGeom g;
   const int32_t *seg, *nseg;
@@ -794,93 +970,196 @@ struct DeltaScanArgs {
   float* state;
   float* o;                                 // [R][H][dv]
 };
+template <int RP> constexpr int scan_tokens() { return RP <= 8 ? 16 : 128 / RP; }
 template <int RP>
 __global__ __launch_bounds__(256) void k_delta_scan(DeltaScanArgs a) {
-  constexpr int DP = 16 * RP, TT = RP <= 8 ? 16 : 128 / RP;
-  constexpr int NL = (3 * TT * DP / 4 + 255) / 256;        // float4 loads per thread and token tile (q, k, decays)
-  __shared__ __attribute__((aligned(16))) float sm[3][TT][DP];
-  __shared__ float sv[TT][16], sb[TT], skq[TT];
+  constexpr int DP = 16 * RP, TT = scan_tokens<RP>(), TILE = 3 * TT * DP, NW = TILE / 256;      // floats of a token tile; wave loads (64 x 16 bytes) in it
+  static_assert(TILE % 256 == 0, "whole wave loads");
+  extern __shared__ __attribute__((aligned(16))) float sm[];            // [2][q, k, decay][TT][DP]
+  __shared__ float sv[2][TT][16], sb[2][TT], skq[2][TT], so[TT][16];
   const DeltaGeom& g = a.g;
   const int s = blockIdx.x;
   if (s >= *a.nseg) return;
   const int first = a.seg[s * 8], n = a.seg[s * 8 + 1], grp = a.seg[s * 8 + 2], start = a.seg[s * 8 + 3];
   if (n <= 0) return;
-  const int h = blockIdx.y, kh = h / (g.H / g.KH), tid = threadIdx.x, lane = tid & 63, sub = lane & 15;
-  const int cb = blockIdx.z * 16, cl = (tid >> 6) * 4 + (lane >> 4), col = cb + cl;
+  const int h = blockIdx.y, kh = h / (g.H / g.KH), tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, sub = lane & 15;
+  const int cb = blockIdx.z * 16, cl = wave * 4 + (lane >> 4), col = cb + cl;
   const bool col_ok = col < g.dv;
   float S[RP];
   float* sp = a.state + (((size_t)grp * g.H + h) * g.dv + (col_ok ? col : 0)) * DP + sub * RP;
 #pragma unroll
   for (int i = 0; i < RP; ++i) S[i] = 0.0f;
   if (start > 0 && col_ok) {
-    if constexpr (RP % 4 == 0) {
 #pragma unroll
-      for (int i = 0; i < RP; i += 4) { const float4 x = *reinterpret_cast<const float4*>(sp + i); S[i] = x.x; S[i + 1] = x.y; S[i + 2] = x.z; S[i + 3] = x.w; }
-    } else {
-#pragma unroll
-      for (int i = 0; i < RP; ++i) S[i] = sp[i];
-    }
+    for (int i = 0; i < RP; ++i) S[i] = sp[i];
   }
-  float4 pf[NL];
   float pv = 0.0f, pb = 0.0f;
-  auto fetch = [&](int t0) {                               // tokens t0 .. t0 + TT - 1 (past the end: the last one again, never used)
-#pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int e = tid + i * 256;
-      if ((3 * TT * DP / 4) % 256 == 0 || e < 3 * TT * DP / 4) {
-        const int w = e / (TT * DP / 4), t = (e / (DP / 4)) % TT, c = (e % (DP / 4)) * 4, r = first + min(t0 + t, n - 1);
-        const float* src = w == 0 ? a.q + ((size_t)r * g.KH + kh) * DP : (w == 1 ? a.k + ((size_t)r * g.KH + kh) * DP : a.dec + ((size_t)r * g.H + h) * DP);
-        pf[i] = *reinterpret_cast<const float4*>(src + c);
-      }
-    }
-    if (tid < TT * 16) {
-      const int t = tid >> 4, c = cb + (tid & 15), r = first + min(t0 + t, n - 1);
-      pv = c < g.dv ? a.v[((size_t)r * g.H + h) * g.dv + c] : 0.0f;
-    }
-    if (tid < 2 * TT) {
-      const int r = first + min(t0 + (tid % TT), n - 1);
-      pb = tid < TT ? a.beta[(size_t)r * g.H + h] : a.kq[(size_t)r * g.KH + kh];
-    }
-  };
-  fetch(0);
-  for (int t0 = 0; t0 < n; t0 += TT) {
-    __syncthreads();
-#pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int e = tid + i * 256;
-      if ((3 * TT * DP / 4) % 256 == 0 || e < 3 * TT * DP / 4) *reinterpret_cast<float4*>(&sm[0][0][0] + (size_t)e * 4) = pf[i];
-    }
-    if (tid < TT * 16) sv[tid >> 4][tid & 15] = pv;
-    if (tid < 2 * TT) { if (tid < TT) sb[tid] = pb; else skq[tid - TT] = pb; }
-    __syncthreads();
-    if (t0 + TT < n) fetch(t0 + TT);
+  const int vt = tid >> 4, vc = cb + (tid & 15);
+  // tokens T0_ .. T0_ + TT - 1 (past the end: the last one again, never used): vectors into buffer B_, scalars into registers
+#define IXT_SCAN_FETCH(T0_, B_)                                                                                                         \
+  do {                                                                                                                                  \
+    _Pragma("unroll") for (int i_ = 0; i_ < (NW + 3) / 4; ++i_) {                                                                       \
+      const int w_ = i_ * 4 + wave;                                                                                                     \
+      if (NW % 4 == 0 || w_ < NW) {                                                                                                     \
+        const int e_ = w_ * 256 + lane * 4, x_ = e_ / (TT * DP), t_ = (e_ / DP) % TT, c_ = e_ % DP, r_ = first + min((T0_) + t_, n - 1); \
+        const float* src_ = x_ == 0 ? a.q + ((size_t)r_ * g.KH + kh) * DP : (x_ == 1 ? a.k + ((size_t)r_ * g.KH + kh) * DP : a.dec + ((size_t)r_ * g.H + h) * DP); \
+        __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src_ + c_),                                    \
+                                         (__attribute__((address_space(3))) void*)(sm + (B_) * TILE + w_ * 256), 16, 0, 0);              \
+      }                                                                                                                                 \
+    }                                                                                                                                   \
+    if (vt < TT) pv = vc < g.dv ? a.v[((size_t)(first + min((T0_) + vt, n - 1)) * g.H + h) * g.dv + vc] : 0.0f;                         \
+    if (tid < TT) pb = a.beta[(size_t)(first + min((T0_) + tid, n - 1)) * g.H + h];                                                     \
+    else if (tid < 2 * TT) pb = a.kq[(size_t)(first + min((T0_) + tid - TT, n - 1)) * g.KH + kh];                                       \
+  } while (0)
+  IXT_SCAN_FETCH(0, 0);
+  int buf = 0;
+  for (int t0 = 0; t0 < n; t0 += TT, buf ^= 1) {
+    if (vt < TT) sv[buf][vt][tid & 15] = pv;
+    if (tid < TT) sb[buf][tid] = pb;
+    else if (tid < 2 * TT) skq[buf][tid - TT] = pb;
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();                                        // this tile is in LDS; the read-outs of the one before have left
+    if (t0 + TT < n) IXT_SCAN_FETCH(t0 + TT, buf ^ 1);
     const int nt = min(TT, n - t0);
+    const float* qb = sm + buf * TILE + sub * RP;
+    float kv[RP], qv[RP], gv[RP], vv, bb, kk;
+#define IXT_SCAN_LOAD(T_)                                                                      \
+  do {                                                                                         \
+    _Pragma("unroll") for (int i_ = 0; i_ < RP; ++i_) {                                        \
+      nq[i_] = qb[(T_) * DP + i_]; nk[i_] = qb[(TT + (T_)) * DP + i_]; ng[i_] = qb[(2 * TT + (T_)) * DP + i_]; \
+    }                                                                                          \
+    nv = sv[buf][T_][cl]; nb = sb[buf][T_]; nkk = skq[buf][T_];                                 \
+  } while (0)
+    float nq[RP], nk[RP], ng[RP], nv, nb, nkk;
+    IXT_SCAN_LOAD(0);
+#pragma unroll 2
     for (int t = 0; t < nt; ++t) {
-      float kv[RP], ax = 0.0f, bx = 0.0f;
+#pragma unroll
+      for (int i = 0; i < RP; ++i) { qv[i] = nq[i]; kv[i] = nk[i]; gv[i] = ng[i]; }
+      vv = nv; bb = nb; kk = nkk;
+      { const int tn = min(t + 1, TT - 1); IXT_SCAN_LOAD(tn); }
+      float a0 = 0.0f, a1 = 0.0f, b0 = 0.0f, b1 = 0.0f;
 #pragma unroll
       for (int i = 0; i < RP; ++i) {
-        kv[i] = sm[1][t][sub * RP + i];
-        S[i] *= sm[2][t][sub * RP + i];
-        ax = fmaf(kv[i], S[i], ax);
-        bx = fmaf(sm[0][t][sub * RP + i], S[i], bx);
+        S[i] *= gv[i];
+        if (i & 1) { a1 = fmaf(kv[i], S[i], a1); b1 = fmaf(qv[i], S[i], b1); }
+        else { a0 = fmaf(kv[i], S[i], a0); b0 = fmaf(qv[i], S[i], b0); }
       }
-      ax = row16_sum(ax);
-      bx = row16_sum(bx);
-      const float u = sb[t] * (sv[t][cl] - ax);
+      const float ax = row16_sum(a0 + a1), bx = row16_sum(b0 + b1);
+      const float u = bb * (vv - ax);
 #pragma unroll
       for (int i = 0; i < RP; ++i) S[i] = fmaf(kv[i], u, S[i]);
-      if (sub == 0 && col_ok) a.o[((size_t)(first + t0 + t) * g.H + h) * g.dv + col] = fmaf(skq[t], u, bx);
+      if (sub == 0) so[t][cl] = fmaf(kk, u, bx);
     }
+#undef IXT_SCAN_LOAD
+    __syncthreads();                                        // read-outs of the tile -> HBM, 16 consecutive columns per token
+    if (vt < nt && vc < g.dv) a.o[((size_t)(first + t0 + vt) * g.H + h) * g.dv + vc] = so[vt][tid & 15];
   }
+#undef IXT_SCAN_FETCH
   if (col_ok) {
-    if constexpr (RP % 4 == 0) {
 #pragma unroll
-      for (int i = 0; i < RP; i += 4) *reinterpret_cast<float4*>(sp + i) = make_float4(S[i], S[i + 1], S[i + 2], S[i + 3]);
-    } else {
+    for (int i = 0; i < RP; ++i) sp[i] = S[i];
+  }
+}
+
+// One token per row (decode): everything between the projections of a gated-delta layer in one launch.  Block = (row, head): its whole state matrix is
+// requested first and travels while the convolutions, unit vectors, decays and the step size are computed; then the recurrence on 16 columns at a
+// time, the head's norm and output gate.  A query / key head that several heads share is computed by each of them; the first one keeps its tail.
+// grid (R, H), block 256, dynamic LDS = (3 dp + 2 dv) floats.
+struct DeltaStepArgs {
+  Slices t, t2; DeltaGeom g;
+  const float *cq, *ck, *cv, *a_log, *dt_bias, *nw;
+  float eps;
+  const int32_t *row_seg, *row_j, *seg;
+  float *tails, *state;
+};
+template <typename T, int RP>
+__global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restrict__ out, int Kp) {
+  constexpr int DP = 16 * RP, NJ = RP <= 8 ? 8 : (RP == 16 ? 4 : 2);      // columns in flight per lane
+  extern __shared__ __attribute__((aligned(16))) float lm[];
+  __shared__ float red[4];
+  float *qs = lm, *ks = lm + DP, *gs = lm + 2 * DP, *vs = lm + 3 * DP, *os = vs + a.g.dv;
+  const DeltaGeom& g = a.g;
+  const int r = blockIdx.x, h = blockIdx.y, kh = h / (g.H / g.KH), tid = threadIdx.x, lane = tid & 63, sub = lane & 15, cl = (tid >> 6) * 4 + (lane >> 4);
+  const int s = a.row_seg[r];
+  if (s < 0) return;
+  const int32_t* sg = a.seg + (size_t)s * 8;
+  const int start = sg[3];
+  float* sp = a.state + ((size_t)sg[2] * g.H + h) * g.dv * DP + sub * RP;
+  float S[NJ][RP];
 #pragma unroll
-      for (int i = 0; i < RP; ++i) sp[i] = S[i];
+  for (int j = 0; j < NJ; ++j) {
+    const int col = cl + 16 * j;
+#pragma unroll
+    for (int i = 0; i < RP; ++i) S[j][i] = (start > 0 && col < g.dv) ? sp[(size_t)col * DP + i] : 0.0f;
+  }
+  const size_t tsz = (size_t)(g.taps - 1) * g.C;
+  float* tb = a.tails + (size_t)sg[2] * 2 * tsz;
+  ConvCtx cc{tb + (size_t)sg[4] * tsz, tb + (size_t)(sg[4] ^ 1) * tsz, 0, 1, start};
+  const bool owner = h % (g.H / g.KH) == 0;
+  ConvCtx ck = cc;
+  if (!owner) ck.tail_out = nullptr;
+  float qq = 0.0f, kk = 0.0f;
+  const float ea = expf(a.a_log[h]);
+  for (int c = tid; c < DP; c += 256) {
+    float x = 0.0f, y = 0.0f, dg = 0.0f;
+    if (c < g.d) {
+      const int ch = kh * g.d + c;
+      x = conv_channel(a.t, r, g.oq + ch, a.cq + (size_t)ch * g.taps, g.taps, ch, g.C, ck);
+      y = conv_channel(a.t, r, g.ok + ch, a.ck + (size_t)ch * g.taps, g.taps, g.KH * g.d + ch, g.C, ck);
+      x *= f32_sigmoid(x); y *= f32_sigmoid(y);
+      dg = expf(-ea * f32_softplus(a.t2.at(r, h * g.d + c) + a.dt_bias[h * g.d + c]));
+    }
+    qs[c] = x; ks[c] = y; gs[c] = dg;
+    qq = fmaf(x, x, qq); kk = fmaf(y, y, kk);
+  }
+  for (int c = tid; c < g.dv; c += 256) {
+    const int ch = h * g.dv + c;
+    const float x = conv_channel(a.t, r, g.ov + ch, a.cv + (size_t)ch * g.taps, g.taps, 2 * g.KH * g.d + ch, g.C, cc);
+    vs[c] = x * f32_sigmoid(x);
+  }
+  const float beta = f32_sigmoid(a.t.at(r, g.ob + h));
+  const float qsum = block_sum256(qq, red), ksum = block_sum256(kk, red);       // (their barriers publish the vectors)
+  const float qn = 1.0f / sqrtf(qsum + 1e-6f) * (1.0f / sqrtf((float)g.d)), kn = 1.0f / sqrtf(ksum + 1e-6f);
+  float qv[RP], kv[RP], gv[RP], qk = 0.0f;
+#pragma unroll
+  for (int i = 0; i < RP; ++i) {
+    qv[i] = qs[sub * RP + i] * qn; kv[i] = ks[sub * RP + i] * kn; gv[i] = gs[sub * RP + i];
+    qk = fmaf(qv[i], kv[i], qk);
+  }
+  qk = row16_sum(qk);
+  for (int c0 = 0; c0 < g.dv; c0 += 16 * NJ) {
+    if (c0 > 0) {
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) {
+        const int col = c0 + cl + 16 * j;
+#pragma unroll
+        for (int i = 0; i < RP; ++i) S[j][i] = (start > 0 && col < g.dv) ? sp[(size_t)col * DP + i] : 0.0f;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const int col = c0 + cl + 16 * j;
+      float ax = 0.0f, bx = 0.0f;
+#pragma unroll
+      for (int i = 0; i < RP; ++i) { S[j][i] *= gv[i]; ax = fmaf(kv[i], S[j][i], ax); bx = fmaf(qv[i], S[j][i], bx); }
+      ax = row16_sum(ax);
+      bx = row16_sum(bx);
+      if (col < g.dv) {
+        const float u = beta * (vs[col] - ax);
+#pragma unroll
+        for (int i = 0; i < RP; ++i) sp[(size_t)col * DP + i] = fmaf(kv[i], u, S[j][i]);
+        if (sub == 0) os[col] = fmaf(qk, u, bx);
+      }
     }
   }
+  __syncthreads();
+  float ss = 0.0f;
+  for (int c = tid; c < g.dv; c += 256) ss = fmaf(os[c], os[c], ss);
+  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)g.dv + a.eps);
+  for (int c = tid; c < g.dv; c += 256) act_store1(out, r, h * g.dv + c, Kp, os[c] * rs * a.nw[c] * f32_sigmoid(a.t2.at(r, g.og2 + h * g.dv + c)));
+  if (h == g.H - 1)
+    for (int k = g.H * g.dv + tid; k < Kp; k += 256) act_store1(out, r, k, Kp, 0.0f);
 }
 
 // read-out: o / rms(o) * norm * sigmoid(gate) per head -> the output projection's operand (column h dv + c).  grid (R, ceil(H / 4)), block 256.

@@ -288,7 +288,11 @@ class DeviceTree:
 
 
 def device_tree_spec(cfg):
-  """[(tree path, shape, std or None for a norm scale)] of the configured block (llama2, gemma2, mixtral)."""
+  """[(tree path, shape, std or None for a norm scale)] of the configured block (llama2, gemma2, mixtral, hybrid)."""
+  if getattr(cfg, "decoder_block", "llama2") == "hybrid":
+    from . import architectures  # pylint: disable=import-outside-toplevel
+    std = lambda name, shape: (1 / cfg.embedding_scale if name == "embed" else 0.1 if "norm" in name else 0.5 if len(shape) == 1 else 1 / math.sqrt(shape[-1]))
+    return [(name, shape, std(name, shape)) for name, shape in architectures.parameter_shapes(cfg).items()]
   E, Q, KV, D, F, V = cfg.emb_dim, cfg.num_query_heads, cfg.num_kv_heads, cfg.head_dim, cfg.mlp_dim, cfg.vocab_size
   block = getattr(cfg, "decoder_block", "llama2")
   spec = [("params/token_embedder/embedding", (V, E), 1.0)]
