@@ -481,7 +481,7 @@ static int latent_attention(ixt_ctx* c, const HLayer& L, const Slices& qa, int R
       }
       TRY(rc);
       if (splits > 1) {
-        hipLaunchKernelGGL(k_latent_combine, dim3(R, g.H), dim3(64), 0, st, m->po, m->pml, splits, g.rankp, g.H, Rp, c->row_active, (bf16_t*)m->olat, Kp);
+        hipLaunchKernelGGL(k_latent_combine, dim3(R, g.H), dim3(128), 0, st, m->po, m->pml, splits, g.rankp, g.H, Rp, c->row_active, (bf16_t*)m->olat, Kp);
         LAUNCHCHK();
       }
       return IXT_OK;

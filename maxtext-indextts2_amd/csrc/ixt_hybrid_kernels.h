@@ -60,6 +60,14 @@ __device__ __forceinline__ float wave_sum(float v) {
   for (int off = 1; off < 64; off <<= 1) v += __shfl_xor(v, off, 64);
   return v;
 }
+// sum over the 16 lanes of a DPP row, every lane ends up with it
+__device__ __forceinline__ float row16_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, false));   // row_ror:8
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, false));   // row_ror:4
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, false));   // row_ror:2
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, false));   // row_ror:1
+  return v;
+}
 __device__ __forceinline__ float block_sum256(float v, float* red /*[4] LDS*/) {
   v = wave_sum(v);
   __syncthreads();
@@ -816,26 +824,36 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
     if (wave == 0 && cq == 0) { a.part_ml[pi * 2] = m; a.part_ml[pi * 2 + 1] = l; }
   }
 }
-// the key splits of a row's heads put together.  grid (R, H), block 64.
-__global__ __launch_bounds__(64) void k_latent_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int cols, int H, int Rp,
-                                                       const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
-  const int r = blockIdx.x, h = blockIdx.y;
+// the key splits of a row's heads put together.  grid (R, H), block 128; nsplit <= 16.
+__global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int cols, int H, int Rp,
+                                                        const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
+  __shared__ float fac[16];
+  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   if (!row_active[r]) return;
   const size_t p0 = ((size_t)r * H + h) * nsplit;
-  float mm = -INFINITY;
-  for (int s = 0; s < nsplit; ++s) mm = fmaxf(mm, part_ml[(p0 + s) * 2]);
-  float ll = 0.0f;
-  for (int s = 0; s < nsplit; ++s) { const float ms = part_ml[(p0 + s) * 2]; if (ms != -INFINITY) ll = fmaf(part_ml[(p0 + s) * 2 + 1], exp2f(ms - mm), ll); }
-  const float inv = 1.0f / ll;
-  for (int c = threadIdx.x * 4; c < Kp; c += 256) {
+  if (tid < 64) {
+    const int s = tid & 15;
+    const float ms = s < nsplit ? part_ml[(p0 + s) * 2] : -INFINITY, ls = s < nsplit ? part_ml[(p0 + s) * 2 + 1] : 0.0f;
+    float mm = ms;
+#pragma unroll
+    for (int off = 1; off < 16; off <<= 1) mm = fmaxf(mm, __shfl_xor(mm, off, 64));
+    const float f = ms == -INFINITY ? 0.0f : exp2f(ms - mm);      // a split without a key of its own
+    const float ll = row16_sum(ls * f);
+    if (tid < 16) fac[s] = f / ll;
+  }
+  __syncthreads();
+  for (int c = tid * 4; c < Kp; c += 512) {
     float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
     if (c < cols) {
-      for (int s = 0; s < nsplit; ++s) {
-        const float ms = part_ml[(p0 + s) * 2];
-        if (ms == -INFINITY) continue;
-        const float f = exp2f(ms - mm) * inv;
-        const float4 u = *reinterpret_cast<const float4*>(part_o + (p0 + s) * cols + c);
-        v[0] = fmaf(u.x, f, v[0]); v[1] = fmaf(u.y, f, v[1]); v[2] = fmaf(u.z, f, v[2]); v[3] = fmaf(u.w, f, v[3]);
+      for (int s0 = 0; s0 < nsplit; s0 += 4) {
+        float4 u[4];
+#pragma unroll
+        for (int s = 0; s < 4; ++s) u[s] = *reinterpret_cast<const float4*>(part_o + (p0 + min(s0 + s, nsplit - 1)) * cols + c);
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          const float f = s0 + s < nsplit ? fac[s0 + s] : 0.0f;
+          if (f != 0.0f) { v[0] = fmaf(u[s].x, f, v[0]); v[1] = fmaf(u[s].y, f, v[1]); v[2] = fmaf(u[s].z, f, v[2]); v[3] = fmaf(u[s].w, f, v[3]); }
+        }
       }
     }
     act_store4(out, h * Rp + r, c, Kp, v);
@@ -949,15 +967,6 @@ __global__ __launch_bounds__(256) void k_delta_prep(DeltaPrepArgs a) {
   if (lane == 0) a.beta[(size_t)r * g.H + h] = f32_sigmoid(a.t.at(r, g.ob + h));
 }
 
-// sum over the 16 lanes of a DPP row, every lane ends up with it
-__device__ __forceinline__ float row16_sum(float v) {
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, false));   // row_ror:8
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, false));   // row_ror:4
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, false));   // row_ror:2
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, false));   // row_ror:1
-  return v;
-}
-
 // The recurrence, per head:  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q, all f32.  The columns of S (value dims) never meet, so a
 // block owns 16 of them for one (segment, head): a wave four, 16 lanes per column with RP key rows each in registers.  o = (g S)^T q + (k . q) u: both
 // sums over the key rows are taken from the decayed state and run side by side.  q, k and the decays of TT tokens at a time come by LDS-DMA into one of
@@ -970,6 +979,8 @@ struct DeltaScanArgs {
   float* state;
   float* o;                                 // [R][H][dv]
 };
+// key row of register i of lane `sub`: 16 lanes x 4 rows per access, so that 16 lanes read and write 256 contiguous bytes
+template <int RP> __device__ __forceinline__ int delta_row(int sub, int i) { return RP >= 4 ? (i >> 2) * 64 + sub * 4 + (i & 3) : sub * RP + i; }
 template <int RP> constexpr int scan_tokens() { return RP <= 8 ? 16 : 128 / RP; }
 template <int RP>
 __global__ __launch_bounds__(256) void k_delta_scan(DeltaScanArgs a) {
@@ -986,13 +997,15 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaScanArgs a) {
   const int cb = blockIdx.z * 16, cl = wave * 4 + (lane >> 4), col = cb + cl;
   const bool col_ok = col < g.dv;
   float S[RP];
-  float* sp = a.state + (((size_t)grp * g.H + h) * g.dv + (col_ok ? col : 0)) * DP + sub * RP;
+  float* sp = a.state + (((size_t)grp * g.H + h) * g.dv + (col_ok ? col : 0)) * DP;
 #pragma unroll
   for (int i = 0; i < RP; ++i) S[i] = 0.0f;
   if (start > 0 && col_ok) {
 #pragma unroll
-    for (int i = 0; i < RP; ++i) S[i] = sp[i];
+    for (int i = 0; i < RP; ++i) S[i] = sp[delta_row<RP>(sub, i)];
   }
+#pragma unroll
+  for (int i = 0; i < RP; ++i) asm volatile("" : "+v"(S[i]));        // arrived before the loop: nothing in it waits for HBM
   float pv = 0.0f, pb = 0.0f;
   const int vt = tid >> 4, vc = cb + (tid & 15);
   // tokens T0_ .. T0_ + TT - 1 (past the end: the last one again, never used): vectors into buffer B_, scalars into registers
@@ -1021,44 +1034,47 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaScanArgs a) {
     __syncthreads();                                        // this tile is in LDS; the read-outs of the one before have left
     if (t0 + TT < n) IXT_SCAN_FETCH(t0 + TT, buf ^ 1);
     const int nt = min(TT, n - t0);
-    const float* qb = sm + buf * TILE + sub * RP;
-    float kv[RP], qv[RP], gv[RP], vv, bb, kk;
-#define IXT_SCAN_LOAD(T_)                                                                      \
-  do {                                                                                         \
-    _Pragma("unroll") for (int i_ = 0; i_ < RP; ++i_) {                                        \
-      nq[i_] = qb[(T_) * DP + i_]; nk[i_] = qb[(TT + (T_)) * DP + i_]; ng[i_] = qb[(2 * TT + (T_)) * DP + i_]; \
-    }                                                                                          \
-    nv = sv[buf][T_][cl]; nb = sb[buf][T_]; nkk = skq[buf][T_];                                 \
+    const float* qb = sm + buf * TILE;
+#define IXT_SCAN_LOAD(X_, T_)                                                                                                       \
+  do {                                                                                                                              \
+    const int tt_ = min((T_), TT - 1);                                                                                              \
+    _Pragma("unroll") for (int i_ = 0; i_ < RP; ++i_) {                                                                             \
+      const int e_ = tt_ * DP + delta_row<RP>(sub, i_);                                                                             \
+      q##X_[i_] = qb[e_]; k##X_[i_] = qb[TT * DP + e_]; g##X_[i_] = qb[2 * TT * DP + e_];                                           \
+    }                                                                                                                               \
+    v##X_ = sv[buf][tt_][cl]; b##X_ = sb[buf][tt_]; d##X_ = skq[buf][tt_];                                                          \
   } while (0)
-    float nq[RP], nk[RP], ng[RP], nv, nb, nkk;
-    IXT_SCAN_LOAD(0);
-#pragma unroll 2
-    for (int t = 0; t < nt; ++t) {
-#pragma unroll
-      for (int i = 0; i < RP; ++i) { qv[i] = nq[i]; kv[i] = nk[i]; gv[i] = ng[i]; }
-      vv = nv; bb = nb; kk = nkk;
-      { const int tn = min(t + 1, TT - 1); IXT_SCAN_LOAD(tn); }
-      float a0 = 0.0f, a1 = 0.0f, b0 = 0.0f, b1 = 0.0f;
-#pragma unroll
-      for (int i = 0; i < RP; ++i) {
-        S[i] *= gv[i];
-        if (i & 1) { a1 = fmaf(kv[i], S[i], a1); b1 = fmaf(qv[i], S[i], b1); }
-        else { a0 = fmaf(kv[i], S[i], a0); b0 = fmaf(qv[i], S[i], b0); }
+#define IXT_SCAN_STEP(X_, T_)                                                                                                       \
+  do {                                                                                                                              \
+    float a0_ = 0.0f, a1_ = 0.0f, b0_ = 0.0f, b1_ = 0.0f;                                                                           \
+    _Pragma("unroll") for (int i_ = 0; i_ < RP; ++i_) {                                                                             \
+      S[i_] *= g##X_[i_];                                                                                                           \
+      if (i_ & 1) { a1_ = fmaf(k##X_[i_], S[i_], a1_); b1_ = fmaf(q##X_[i_], S[i_], b1_); }                                         \
+      else { a0_ = fmaf(k##X_[i_], S[i_], a0_); b0_ = fmaf(q##X_[i_], S[i_], b0_); }                                                \
+    }                                                                                                                               \
+    const float ax_ = row16_sum(a0_ + a1_), bx_ = row16_sum(b0_ + b1_), u_ = b##X_ * (v##X_ - ax_);                                 \
+    _Pragma("unroll") for (int i_ = 0; i_ < RP; ++i_) S[i_] = fmaf(k##X_[i_], u_, S[i_]);                                           \
+    if (sub == 0) so[T_][cl] = fmaf(d##X_, u_, bx_);                                                                                \
+  } while (0)
+    float qA[RP], kA[RP], gA[RP], vA, bA, dA, qB[RP], kB[RP], gB[RP], vB, bB, dB;
+    IXT_SCAN_LOAD(A, 0);
+    for (int t = 0; t < nt; t += 2) {
+      IXT_SCAN_LOAD(B, t + 1);
+      IXT_SCAN_STEP(A, t);
+      if (t + 1 < nt) {
+        IXT_SCAN_LOAD(A, t + 2);
+        IXT_SCAN_STEP(B, t + 1);
       }
-      const float ax = row16_sum(a0 + a1), bx = row16_sum(b0 + b1);
-      const float u = bb * (vv - ax);
-#pragma unroll
-      for (int i = 0; i < RP; ++i) S[i] = fmaf(kv[i], u, S[i]);
-      if (sub == 0) so[t][cl] = fmaf(kk, u, bx);
     }
 #undef IXT_SCAN_LOAD
+#undef IXT_SCAN_STEP
     __syncthreads();                                        // read-outs of the tile -> HBM, 16 consecutive columns per token
     if (vt < nt && vc < g.dv) a.o[((size_t)(first + t0 + vt) * g.H + h) * g.dv + vc] = so[vt][tid & 15];
   }
 #undef IXT_SCAN_FETCH
   if (col_ok) {
 #pragma unroll
-    for (int i = 0; i < RP; ++i) sp[i] = S[i];
+    for (int i = 0; i < RP; ++i) sp[delta_row<RP>(sub, i)] = S[i];
   }
 }
 
@@ -1077,7 +1093,7 @@ template <typename T, int RP>
 __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restrict__ out, int Kp) {
   constexpr int DP = 16 * RP, NJ = RP <= 8 ? 8 : (RP == 16 ? 4 : 2);      // columns in flight per lane
   extern __shared__ __attribute__((aligned(16))) float lm[];
-  __shared__ float red[4];
+  __shared__ float red[4], red2[4];
   float *qs = lm, *ks = lm + DP, *gs = lm + 2 * DP, *vs = lm + 3 * DP, *os = vs + a.g.dv;
   const DeltaGeom& g = a.g;
   const int r = blockIdx.x, h = blockIdx.y, kh = h / (g.H / g.KH), tid = threadIdx.x, lane = tid & 63, sub = lane & 15, cl = (tid >> 6) * 4 + (lane >> 4);
@@ -1085,46 +1101,46 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
   if (s < 0) return;
   const int32_t* sg = a.seg + (size_t)s * 8;
   const int start = sg[3];
-  float* sp = a.state + ((size_t)sg[2] * g.H + h) * g.dv * DP + sub * RP;
+  float* sp = a.state + ((size_t)sg[2] * g.H + h) * g.dv * DP;
   float S[NJ][RP];
 #pragma unroll
   for (int j = 0; j < NJ; ++j) {
     const int col = cl + 16 * j;
 #pragma unroll
-    for (int i = 0; i < RP; ++i) S[j][i] = (start > 0 && col < g.dv) ? sp[(size_t)col * DP + i] : 0.0f;
+    for (int i = 0; i < RP; ++i) S[j][i] = (start > 0 && col < g.dv) ? sp[(size_t)col * DP + delta_row<RP>(sub, i)] : 0.0f;
   }
   const size_t tsz = (size_t)(g.taps - 1) * g.C;
   float* tb = a.tails + (size_t)sg[2] * 2 * tsz;
-  ConvCtx cc{tb + (size_t)sg[4] * tsz, tb + (size_t)(sg[4] ^ 1) * tsz, 0, 1, start};
-  const bool owner = h % (g.H / g.KH) == 0;
-  ConvCtx ck = cc;
-  if (!owner) ck.tail_out = nullptr;
+  const float* tail_in = tb + (size_t)sg[4] * tsz;
+  float* tail_out = tb + (size_t)(sg[4] ^ 1) * tsz;
+  const bool first = h % (g.H / g.KH) == 0;          // of the heads that share a query / key head
   float qq = 0.0f, kk = 0.0f;
-  const float ea = expf(a.a_log[h]);
-  for (int c = tid; c < DP; c += 256) {
-    float x = 0.0f, y = 0.0f, dg = 0.0f;
-    if (c < g.d) {
-      const int ch = kh * g.d + c;
-      x = conv_channel(a.t, r, g.oq + ch, a.cq + (size_t)ch * g.taps, g.taps, ch, g.C, ck);
-      y = conv_channel(a.t, r, g.ok + ch, a.ck + (size_t)ch * g.taps, g.taps, g.KH * g.d + ch, g.C, ck);
-      x *= f32_sigmoid(x); y *= f32_sigmoid(y);
-      dg = expf(-ea * f32_softplus(a.t2.at(r, h * g.d + c) + a.dt_bias[h * g.d + c]));
+  // one channel per thread and round: queries, keys, decays, values side by side
+  for (int i = tid; i < 3 * DP + g.dv; i += 256) {
+    const int kind = i < DP ? 0 : (i < 2 * DP ? 1 : (i < 3 * DP ? 2 : 3)), c = i - kind * DP;
+    float x = 0.0f;
+    if (kind == 2) {
+      if (c < g.d) x = expf(-expf(a.a_log[h]) * f32_softplus(a.t2.at(r, h * g.d + c) + a.dt_bias[h * g.d + c]));
+    } else if (kind == 3 || c < g.d) {
+      const int ch = kind == 3 ? h * g.dv + c : kh * g.d + c, col = (kind == 0 ? g.oq : (kind == 1 ? g.ok : g.ov)) + ch;
+      x = conv_channel(a.t, r, col, (kind == 0 ? a.cq : (kind == 1 ? a.ck : a.cv)) + (size_t)ch * g.taps, g.taps, kind == 3 ? 2 * g.KH * g.d + ch : kind * g.KH * g.d + ch, g.C,
+                       ConvCtx{tail_in, kind == 3 || first ? tail_out : nullptr, 0, 1, start});
+      x *= f32_sigmoid(x);
+      if (kind == 0) qq = fmaf(x, x, qq);
+      else if (kind == 1) kk = fmaf(x, x, kk);
     }
-    qs[c] = x; ks[c] = y; gs[c] = dg;
-    qq = fmaf(x, x, qq); kk = fmaf(y, y, kk);
-  }
-  for (int c = tid; c < g.dv; c += 256) {
-    const int ch = h * g.dv + c;
-    const float x = conv_channel(a.t, r, g.ov + ch, a.cv + (size_t)ch * g.taps, g.taps, 2 * g.KH * g.d + ch, g.C, cc);
-    vs[c] = x * f32_sigmoid(x);
+    lm[i] = x;                              // [q | k | decay | v]
   }
   const float beta = f32_sigmoid(a.t.at(r, g.ob + h));
-  const float qsum = block_sum256(qq, red), ksum = block_sum256(kk, red);       // (their barriers publish the vectors)
-  const float qn = 1.0f / sqrtf(qsum + 1e-6f) * (1.0f / sqrtf((float)g.d)), kn = 1.0f / sqrtf(ksum + 1e-6f);
+  qq = wave_sum(qq); kk = wave_sum(kk);
+  if (lane == 0) { red[tid >> 6] = qq; red2[tid >> 6] = kk; }
+  __syncthreads();
+  const float qn = 1.0f / sqrtf((red[0] + red[1]) + (red[2] + red[3]) + 1e-6f) * (1.0f / sqrtf((float)g.d)), kn = 1.0f / sqrtf((red2[0] + red2[1]) + (red2[2] + red2[3]) + 1e-6f);
   float qv[RP], kv[RP], gv[RP], qk = 0.0f;
 #pragma unroll
   for (int i = 0; i < RP; ++i) {
-    qv[i] = qs[sub * RP + i] * qn; kv[i] = ks[sub * RP + i] * kn; gv[i] = gs[sub * RP + i];
+    const int e = delta_row<RP>(sub, i);
+    qv[i] = qs[e] * qn; kv[i] = ks[e] * kn; gv[i] = gs[e];
     qk = fmaf(qv[i], kv[i], qk);
   }
   qk = row16_sum(qk);
@@ -1134,7 +1150,7 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
       for (int j = 0; j < NJ; ++j) {
         const int col = c0 + cl + 16 * j;
 #pragma unroll
-        for (int i = 0; i < RP; ++i) S[j][i] = (start > 0 && col < g.dv) ? sp[(size_t)col * DP + i] : 0.0f;
+        for (int i = 0; i < RP; ++i) S[j][i] = (start > 0 && col < g.dv) ? sp[(size_t)col * DP + delta_row<RP>(sub, i)] : 0.0f;
       }
     }
 #pragma unroll
@@ -1148,7 +1164,7 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
       if (col < g.dv) {
         const float u = beta * (vs[col] - ax);
 #pragma unroll
-        for (int i = 0; i < RP; ++i) sp[(size_t)col * DP + i] = fmaf(kv[i], u, S[j][i]);
+        for (int i = 0; i < RP; ++i) sp[(size_t)col * DP + delta_row<RP>(sub, i)] = fmaf(kv[i], u, S[j][i]);
         if (sub == 0) os[col] = fmaf(qk, u, bx);
       }
     }
