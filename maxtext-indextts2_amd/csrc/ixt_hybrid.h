@@ -33,7 +33,7 @@ struct HybridModel {
   float *x = nullptr, *part2 = nullptr;
   size_t part2_floats = 0;
   void *xb = nullptr, *act = nullptr, *hact = nullptr, *xn = nullptr, *qx = nullptr, *qr = nullptr, *olat = nullptr, *xg = nullptr, *mhact = nullptr;
-  float *dq = nullptr, *dk = nullptr, *dkq = nullptr, *dv = nullptr, *dec = nullptr, *beta = nullptr, *dout = nullptr, *zlog = nullptr, *mw = nullptr, *po = nullptr, *pml = nullptr;
+  float *dq = nullptr, *dk = nullptr, *dkq = nullptr, *dv = nullptr, *dec = nullptr, *beta = nullptr, *dout = nullptr, *mw = nullptr, *msum = nullptr, *po = nullptr, *pml = nullptr;
   int32_t *midx = nullptr, *mpos = nullptr, *mrb = nullptr;
   int moe_cap = 0;
   int32_t *row_seg = nullptr, *row_j = nullptr, *seg = nullptr, *nseg = nullptr, *state_len = nullptr, *parity = nullptr, *claim = nullptr, *err = nullptr, *head_rb = nullptr;
@@ -214,7 +214,7 @@ static int hybrid_init(ixt_ctx* c) {
   { float* d = m->fnorm; const int E = m->E;
     m->tensors["final.norm"] = HTensor{{E}, [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, d, E, st); }, false}; }
   std::map<std::pair<int, float>, std::pair<float*, float*>> ropes;
-  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, z_e = 0, mi = 0, po = 0;
+  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0;
   auto upd = [](size_t& a, size_t v) { if (v > a) a = v; };
   // f32 slices of a dot over at most R rows (split-K only below 128 rows; launch_dot keeps to one slice when the slices do not fit)
   auto dotsz = [&](int K, int N) { upd(part, std::max((size_t)R * N, (size_t)std::min(R, 128) * N * ((K + IXT_CHAIN - 1) / IXT_CHAIN))); };
@@ -283,7 +283,7 @@ static int hybrid_init(ixt_ctx* c) {
       const int Fp = up_to(l.ff, IXT_KALIGN), pairs = R * l.top;
       const int cap = std::max(up_to(pairs, 128) + 128 * std::min(l.experts, pairs), 64 + 16 * l.experts);
       m->moe_cap = std::max(m->moe_cap, cap);
-      upd(xg_e, (size_t)cap * m->Ep); upd(mh_e, (size_t)cap * Fp); upd(z_e, (size_t)R * l.experts); upd(mi, (size_t)pairs);
+      upd(xg_e, (size_t)cap * m->Ep); upd(mh_e, (size_t)cap * Fp); upd(mi, (size_t)pairs);
       upd(part, (size_t)cap * up_to(m->E, 16));
       upd(part, (size_t)(64 + 16 * std::min(l.experts, 64)) * up_to(m->E, 16) * ((Fp + IXT_CHAIN - 1) / IXT_CHAIN));
       if (m->f32) upd(part, (size_t)cap * 2 * Fp);
@@ -305,8 +305,9 @@ static int hybrid_init(ixt_ctx* c) {
   TRY(h_alloc(c, &m->xg, (xg_e + 8) * m->esz)); TRY(h_alloc(c, &m->mhact, (mh_e + 8) * m->esz));
   TRY(h_allocf(c, &m->dq, s_q + 4)); TRY(h_allocf(c, &m->dk, s_q + 4)); TRY(h_allocf(c, &m->dkq, s_kq + 4)); TRY(h_allocf(c, &m->dv, s_v + 4));
   TRY(h_allocf(c, &m->dec, s_dec + 4)); TRY(h_allocf(c, &m->beta, s_b + 4)); TRY(h_allocf(c, &m->dout, s_v + 4));
-  TRY(h_allocf(c, &m->zlog, z_e + 4)); TRY(h_allocf(c, &m->mw, mi + 4)); TRY(h_allocf(c, &m->midx, mi + 4)); TRY(h_allocf(c, &m->mpos, mi + 4));
+  TRY(h_allocf(c, &m->mw, mi + 4)); TRY(h_allocf(c, &m->midx, mi + 4)); TRY(h_allocf(c, &m->mpos, mi + 4));
   TRY(h_allocf(c, &m->mrb, (size_t)m->moe_cap / 16 + 16));
+  TRY(h_allocf(c, &m->msum, (size_t)64 * up_to(m->E, 16)));
   TRY(h_allocf(c, &m->po, po + 4)); TRY(h_allocf(c, &m->pml, (size_t)(1024 + m->maxH) * 16 * 2 + 4));
   TRY(h_allocf(c, &m->row_seg, (size_t)R)); TRY(h_allocf(c, &m->row_j, (size_t)R)); TRY(h_allocf(c, &m->seg, (size_t)R * 8)); TRY(h_allocf(c, &m->nseg, 4));
   TRY(h_allocf(c, &m->state_len, (size_t)c->G)); TRY(h_allocf(c, &m->parity, (size_t)c->G)); TRY(h_allocf(c, &m->claim, (size_t)c->G)); TRY(h_allocf(c, &m->err, 4));
@@ -549,12 +550,8 @@ static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipSt
   HybridModel* m = c->hy;
   const ixt_layer& l = L.c;
   const int pairs = R * l.top;
-  if (R <= 64) {
-    hipLaunchKernelGGL(k_route_row, dim3(R), dim3(256), sizeof(float) * l.experts, st, m->x, W.router, m->E, m->Ep, l.experts, l.top, m->midx, m->mw);
-  } else {
-    hipLaunchKernelGGL(k_route_logits, dim3((l.experts + 31) / 32, (R + 7) / 8), dim3(256), 0, st, m->x, W.router, m->E, m->Ep, l.experts, R, m->zlog);
-    hipLaunchKernelGGL(k_route_pick, dim3((R + 3) / 4), dim3(256), 0, st, m->zlog, l.experts, l.top, R, m->midx, m->mw);
-  }
+  if (R <= 256) hipLaunchKernelGGL((k_route<1>), dim3(R), dim3(256), sizeof(float) * l.experts, st, m->x, W.router, m->E, m->Ep, l.experts, l.top, R, m->midx, m->mw);
+  else hipLaunchKernelGGL((k_route<4>), dim3((R + 3) / 4), dim3(256), sizeof(float) * 4 * l.experts, st, m->x, W.router, m->E, m->Ep, l.experts, l.top, R, m->midx, m->mw);
   LAUNCHCHK();
   const int align = (m->f32 || pairs <= 64) ? 16 : 128;
   const int rows_g = up_to(pairs, align) + align * std::min(l.experts, pairs);     // every expert with a copy may waste up to align - 1 rows
@@ -617,7 +614,13 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
       TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n2, R, st)));
     } else if (L.c.ffn == IXT_FFN_MOE) {
       TRY(hybrid_moe<T>(c, L, W, R, st, &t));
-      TRY((hybrid_norm<T>(c, t, m->mpos, m->mw, L.c.top, W.n2, R, st)));
+      if (t.n > 2 && R <= 64) {
+        hipLaunchKernelGGL(k_moe_sum, dim3((t.ncols + 255) / 256, R), dim3(64), 0, st, t, m->mpos, m->mw, L.c.top, m->msum);
+        LAUNCHCHK();
+        TRY((hybrid_norm<T>(c, Slices{m->msum, 1, 0, t.ncols}, nullptr, nullptr, 0, W.n2, R, st)));
+      } else {
+        TRY((hybrid_norm<T>(c, t, m->mpos, m->mw, L.c.top, W.n2, R, st)));
+      }
     }
     if (m->tap && !c->capturing) {
       if ((i + 1) * (size_t)R * m->E > m->tap_floats) return set_err(IXT_ERR_INVALID, "residual tap: buffer too small");

@@ -47,9 +47,13 @@ struct Slices {             // a dot's output
   __device__ __forceinline__ void at4(int r, int c, float* o) const {       // c % 4 == 0
     const float* q = p + (size_t)r * ncols + c;
     float4 t = *reinterpret_cast<const float4*>(q);
-    for (int s = 1; s < n; ++s) {
-      const float4 u = *reinterpret_cast<const float4*>(q + (size_t)s * stride);
-      t.x += u.x; t.y += u.y; t.z += u.z; t.w += u.w;
+    for (int s = 1; s < n; s += 4) {                                        // four slices in flight
+      float4 u[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) u[i] = *reinterpret_cast<const float4*>(q + (size_t)min(s + i, n - 1) * stride);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (s + i < n) { t.x += u[i].x; t.y += u[i].y; t.z += u[i].z; t.w += u[i].w; }
     }
     o[0] = t.x; o[1] = t.y; o[2] = t.z; o[3] = t.w;
   }
@@ -1237,39 +1241,51 @@ __device__ __forceinline__ void route_top(const float* z, int n, int top, int la
     if (lane == 0) { idx[j] = bi; wts[j] = expf(b - mx) / sum; }
   }
 }
-// few rows: logits and choice in one launch, f32 residual x f32 router weights.  grid R, block 256, LDS n floats.
-__global__ __launch_bounds__(256) void k_route_row(const float* __restrict__ x, const float* __restrict__ w /*[n][Ep]*/, int E, int Ep, int n, int top, int32_t* __restrict__ idx,
-                                                   float* __restrict__ wts) {
-  extern __shared__ __attribute__((aligned(16))) float z[];
-  const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const float* xr = x + (size_t)r * E;
-  for (int e = wave; e < n; e += 4) {
-    float a = 0.0f;
-    for (int k = lane; k < E; k += 64) a = fmaf(xr[k], w[(size_t)e * Ep + k], a);
-    a = wave_sum(a);
-    if (lane == 0) z[e] = a;
-  }
-  __syncthreads();
-  if (wave == 0) route_top(z, n, top, lane, idx + (size_t)r * top, wts + (size_t)r * top);
-}
-// many rows: 8 rows x 32 experts per block, x and w through LDS in steps of 32 k; z [R][n].  grid (ceil(n / 32), ceil(R / 8)), block 256.
-__global__ __launch_bounds__(256) void k_route_logits(const float* __restrict__ x, const float* __restrict__ w, int E, int Ep, int n, int R, float* __restrict__ z) {
-  __shared__ float xs[8][65], ws[32][65];
-  const int tid = threadIdx.x, e0 = blockIdx.x * 32, r0 = blockIdx.y * 8, tr = tid >> 5, te = tid & 31;
-  float a = 0.0f;
-  for (int k0 = 0; k0 < E; k0 += 64) {
-    for (int i = tid; i < 8 * 64; i += 256) xs[i >> 6][i & 63] = (r0 + (i >> 6) < R && k0 + (i & 63) < E) ? x[(size_t)(r0 + (i >> 6)) * E + k0 + (i & 63)] : 0.0f;
-    for (int i = tid; i < 32 * 64; i += 256) ws[i >> 6][i & 63] = (e0 + (i >> 6) < n && k0 + (i & 63) < E) ? w[(size_t)(e0 + (i >> 6)) * Ep + k0 + (i & 63)] : 0.0f;
+// router: logits (f32 residual x f32 weights) and choice of RB rows in one block, eight experts at a time: a thread takes every 256th feature of the RB
+// rows and the eight weight rows.  w [n][Ep]; grid ceil(R / RB), block 256, LDS RB n floats.
+template <int RB>
+__global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, const float* __restrict__ w, int E, int Ep, int n, int top, int R, int32_t* __restrict__ idx,
+                                               float* __restrict__ wts) {
+  extern __shared__ __attribute__((aligned(16))) float z[];            // [RB][n]
+  __shared__ float red[4][RB * 8];
+  const int r0 = blockIdx.x * RB, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const float* xr[RB];
+#pragma unroll
+  for (int i = 0; i < RB; ++i) xr[i] = x + (size_t)min(r0 + i, R - 1) * E;
+  for (int e0 = 0; e0 < n; e0 += 8) {
+    float acc[RB][8];
+#pragma unroll
+    for (int i = 0; i < RB; ++i)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[i][e] = 0.0f;
+    const float* wr[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) wr[e] = w + (size_t)min(e0 + e, n - 1) * Ep;
+#pragma unroll 2
+    for (int k = tid; k < E; k += 256) {
+      float xv[RB], wv[8];
+#pragma unroll
+      for (int i = 0; i < RB; ++i) xv[i] = xr[i][k];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) wv[e] = wr[e][k];
+#pragma unroll
+      for (int i = 0; i < RB; ++i)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[i][e] = fmaf(xv[i], wv[e], acc[i][e]);
+    }
+#pragma unroll
+    for (int i = 0; i < RB; ++i)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float t = wave_sum(acc[i][e]);
+        if (lane == 0) red[wave][i * 8 + e] = t;
+      }
     __syncthreads();
-#pragma unroll 8
-    for (int k = 0; k < 64; ++k) a = fmaf(xs[tr][k], ws[te][k], a);
+    if (tid < RB * 8 && e0 + (tid & 7) < n) z[(tid >> 3) * n + e0 + (tid & 7)] = (red[0][tid] + red[1][tid]) + (red[2][tid] + red[3][tid]);
     __syncthreads();
   }
-  if (r0 + tr < R && e0 + te < n) z[(size_t)(r0 + tr) * n + e0 + te] = a;
-}
-__global__ __launch_bounds__(256) void k_route_pick(const float* __restrict__ z, int n, int top, int R, int32_t* __restrict__ idx, float* __restrict__ wts) {
-  const int r = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (r < R) route_top(z + (size_t)r * n, n, top, threadIdx.x & 63, idx + (size_t)r * top, wts + (size_t)r * top);
+  for (int i = wave; i < RB; i += 4)
+    if (r0 + i < R) route_top(z + (size_t)i * n, n, top, lane, idx + (size_t)(r0 + i) * top, wts + (size_t)(r0 + i) * top);
 }
 // any number of experts (<= 1024): destination row of every copy by one pass of counters; the order inside an expert is free.  One block of 1024.
 __global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __restrict__ idx, int npairs, int n, int align, int nrb_cap, int32_t* __restrict__ pos, int32_t* __restrict__ rb_exp) {
@@ -1300,4 +1316,18 @@ __global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __restrict
 __global__ __launch_bounds__(256) void k_gather32(const float* __restrict__ x, const int32_t* __restrict__ pos, int top, int Ep, float* __restrict__ xg) {
   const int k = blockIdx.x * 256 + threadIdx.x, p = blockIdx.y;
   if (k < Ep) xg[(size_t)pos[p] * Ep + k] = x[(size_t)(p / top) * Ep + k];
+}
+// few rows whose expert outputs lie in many split-K slices: the weighted sum of a row's copies as one slice.  grid (ceil(ncols / 256), R), block 64.
+__global__ __launch_bounds__(64) void k_moe_sum(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, float* __restrict__ out) {
+  const int c = (blockIdx.x * 64 + threadIdx.x) * 4, r = blockIdx.y;
+  if (c >= t.ncols) return;
+  float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int j = 0; j < top; ++j) {
+    float u[4];
+    t.at4(pos[(size_t)r * top + j], c, u);
+    const float w = wts[(size_t)r * top + j];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = fmaf(w, u[i], v[i]);
+  }
+  *reinterpret_cast<float4*>(out + (size_t)r * t.ncols + c) = make_float4(v[0], v[1], v[2], v[3]);
 }
