@@ -281,6 +281,7 @@ static int hybrid_init(ixt_ctx* c) {
       dotsz(Fp, up_to(m->E, 16));
     } else if (l.ffn == IXT_FFN_MOE) {
       const int Fp = up_to(l.ff, IXT_KALIGN), pairs = R * l.top;
+      if (pairs > 60000) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d rows x %d experts per token exceed one launch (60000 copies): smaller max_packed_rows / max_prefill_predict_length", i, R, l.top);
       const int cap = std::max(up_to(pairs, 128) + 128 * std::min(l.experts, pairs), 64 + 16 * l.experts);
       m->moe_cap = std::max(m->moe_cap, cap);
       upd(xg_e, (size_t)cap * m->Ep); upd(mh_e, (size_t)cap * Fp); upd(mi, (size_t)pairs);
@@ -521,7 +522,7 @@ static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int 
   LAUNCHCHK();
   TRY(hdot<T>(c, (const T*)m->act, W.low, R, m->part2, m->part2_floats, st, &t2));
   if (single) {            // every row is a segment of one token
-    DeltaStepArgs da{t, t2, g, W.cq, W.ck, W.cv, W.a_log, W.dt_bias, W.onorm, m->eps, m->row_seg, m->row_j, m->seg, L.tails, L.state};
+    DeltaStepArgs da{t, t2, g, W.cq, W.ck, W.cv, W.a_log, W.dt_bias, W.onorm, m->eps, c->row_active, c->row_slot, c->row_pos, m->parity, L.tails, L.state};
     const dim3 grid(R, g.H);
     const size_t lds = sizeof(float) * (3 * g.dp + 2 * g.dv);
 #define HSTEP(RP_) case RP_: hipLaunchKernelGGL((k_delta_step<T, RP_>), grid, dim3(256), lds, st, da, (T*)m->act, W.o.Kp); break

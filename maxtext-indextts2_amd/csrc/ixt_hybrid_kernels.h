@@ -708,10 +708,11 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
   const LatentGeom& g = a.g;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
   const int row = blockIdx.x, h0 = blockIdx.y * a.HB, hb = min(a.HB, g.H - h0), nsplit = gridDim.z;
-  if (!a.row_active[row]) return;
+  const int active = a.row_active[row], pos = a.row_pos[row], slot = a.row_slot[row];     // (requested together)
+  if (!active) return;
   const bool pair_ok = r_in < hb;
-  const int head = h0 + (pair_ok ? r_in : 0), pos = a.row_pos[row];
-  const int32_t* prow = a.page_map + (size_t)a.row_slot[row] * g.mpg;
+  const int head = h0 + (pair_ok ? r_in : 0);
+  const int32_t* prow = a.page_map + (size_t)slot * g.mpg;
   const int k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0, ntile = (pos - k_lo) / 64 + 1;
   int t = blockIdx.z;
   if (t < ntile) latent_dma<RT, RS>(a.pages, latent_row(prow, min(k_lo + t * 64 + lane, pos), a.pshift), tile, wave, lane);
@@ -897,11 +898,20 @@ struct ConvCtx { const float* tail_in; float* tail_out; int j, n, start; };     
 __device__ __forceinline__ float conv_channel(const Slices& t, int r, int col, const float* __restrict__ tp, int taps, int ch, int C, const ConvCtx& cc) {
   const float x0 = t.at(r, col);
   float acc = x0 * tp[taps - 1];
-  for (int b = 1; b < taps; ++b) {
-    float v = 0.0f;
-    if (cc.j - b >= 0) v = t.at(r - b, col);
-    else if (cc.start > 0) v = cc.tail_in[(size_t)(taps - 1 - (b - cc.j)) * C + ch];
-    acc = fmaf(v, tp[taps - 1 - b], acc);
+  for (int b0 = 1; b0 < taps; b0 += 4) {                   // four earlier inputs in flight
+    float v[4], w[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int b = min(b0 + i, taps - 1);
+      const bool mine = cc.j - b >= 0;
+      const float* src = mine ? t.p + (size_t)(r - b) * t.ncols + col : cc.tail_in + (size_t)(taps - 1 - (b - cc.j)) * C + ch;
+      v[i] = mine || cc.start > 0 ? *src : 0.0f;
+      w[i] = b0 + i < taps ? tp[taps - 1 - b] : 0.0f;
+      if (mine)
+        for (int s = 1; s < t.n; ++s) v[i] += src[(size_t)s * t.stride];
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc = fmaf(v[i], w[i], acc);
   }
   if (cc.tail_out == nullptr) return acc;
   const int dist = cc.n - 1 - cc.j;
@@ -1090,7 +1100,7 @@ struct DeltaStepArgs {
   Slices t, t2; DeltaGeom g;
   const float *cq, *ck, *cv, *a_log, *dt_bias, *nw;
   float eps;
-  const int32_t *row_seg, *row_j, *seg;
+  const int32_t *row_active, *row_slot, *row_pos, *parity;     // parity: as k_segments has left it for the NEXT pass
   float *tails, *state;
 };
 template <typename T, int RP>
@@ -1101,11 +1111,10 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
   float *qs = lm, *ks = lm + DP, *gs = lm + 2 * DP, *vs = lm + 3 * DP, *os = vs + a.g.dv;
   const DeltaGeom& g = a.g;
   const int r = blockIdx.x, h = blockIdx.y, kh = h / (g.H / g.KH), tid = threadIdx.x, lane = tid & 63, sub = lane & 15, cl = (tid >> 6) * 4 + (lane >> 4);
-  const int s = a.row_seg[r];
-  if (s < 0) return;
-  const int32_t* sg = a.seg + (size_t)s * 8;
-  const int start = sg[3];
-  float* sp = a.state + ((size_t)sg[2] * g.H + h) * g.dv * DP;
+  const int active = a.row_active[r], grp = a.row_slot[r], start = a.row_pos[r];      // (requested together)
+  if (!active) return;
+  const int par = a.parity[grp] ^ 1;
+  float* sp = a.state + ((size_t)grp * g.H + h) * g.dv * DP;
   float S[NJ][RP];
 #pragma unroll
   for (int j = 0; j < NJ; ++j) {
@@ -1114,9 +1123,10 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
     for (int i = 0; i < RP; ++i) S[j][i] = (start > 0 && col < g.dv) ? sp[(size_t)col * DP + delta_row<RP>(sub, i)] : 0.0f;
   }
   const size_t tsz = (size_t)(g.taps - 1) * g.C;
-  float* tb = a.tails + (size_t)sg[2] * 2 * tsz;
-  const float* tail_in = tb + (size_t)sg[4] * tsz;
-  float* tail_out = tb + (size_t)(sg[4] ^ 1) * tsz;
+  float* tb = a.tails + (size_t)grp * 2 * tsz;
+  const float* tail_in = tb + (size_t)par * tsz;
+  float* tail_out = tb + (size_t)(par ^ 1) * tsz;
+  const float gate0 = tid < g.dv ? a.t2.at(r, g.og2 + h * g.dv + tid) : 0.0f, beta_z = a.t.at(r, g.ob + h), ea = expf(a.a_log[h]);
   const bool first = h % (g.H / g.KH) == 0;          // of the heads that share a query / key head
   float qq = 0.0f, kk = 0.0f;
   // one channel per thread and round: queries, keys, decays, values side by side
@@ -1124,7 +1134,7 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
     const int kind = i < DP ? 0 : (i < 2 * DP ? 1 : (i < 3 * DP ? 2 : 3)), c = i - kind * DP;
     float x = 0.0f;
     if (kind == 2) {
-      if (c < g.d) x = expf(-expf(a.a_log[h]) * f32_softplus(a.t2.at(r, h * g.d + c) + a.dt_bias[h * g.d + c]));
+      if (c < g.d) x = expf(-ea * f32_softplus(a.t2.at(r, h * g.d + c) + a.dt_bias[h * g.d + c]));
     } else if (kind == 3 || c < g.d) {
       const int ch = kind == 3 ? h * g.dv + c : kh * g.d + c, col = (kind == 0 ? g.oq : (kind == 1 ? g.ok : g.ov)) + ch;
       x = conv_channel(a.t, r, col, (kind == 0 ? a.cq : (kind == 1 ? a.ck : a.cv)) + (size_t)ch * g.taps, g.taps, kind == 3 ? 2 * g.KH * g.d + ch : kind * g.KH * g.d + ch, g.C,
@@ -1135,7 +1145,7 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
     }
     lm[i] = x;                              // [q | k | decay | v]
   }
-  const float beta = f32_sigmoid(a.t.at(r, g.ob + h));
+  const float beta = f32_sigmoid(beta_z);
   qq = wave_sum(qq); kk = wave_sum(kk);
   if (lane == 0) { red[tid >> 6] = qq; red2[tid >> 6] = kk; }
   __syncthreads();
@@ -1177,7 +1187,7 @@ __global__ __launch_bounds__(256) void k_delta_step(DeltaStepArgs a, T* __restri
   float ss = 0.0f;
   for (int c = tid; c < g.dv; c += 256) ss = fmaf(os[c], os[c], ss);
   const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)g.dv + a.eps);
-  for (int c = tid; c < g.dv; c += 256) act_store1(out, r, h * g.dv + c, Kp, os[c] * rs * a.nw[c] * f32_sigmoid(a.t2.at(r, g.og2 + h * g.dv + c)));
+  for (int c = tid; c < g.dv; c += 256) act_store1(out, r, h * g.dv + c, Kp, os[c] * rs * a.nw[c] * f32_sigmoid(c < 256 ? gate0 : a.t2.at(r, g.og2 + h * g.dv + c)));
   if (h == g.H - 1)
     for (int k = g.H * g.dv + tid; k < Kp; k += 256) act_store1(out, r, k, Kp, 0.0f);
 }

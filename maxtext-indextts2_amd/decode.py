@@ -9,7 +9,8 @@ range(max_prefill_predict_length, max_target_length) -> tokens of each stream.  
 (the reference tokenizes `prompt` with a sentencepiece / HF tokenizer that is not part of this path): the prompt ids come from
 `ixt_prompt_tokens` (comma-separated ids) or, when that is empty, from the seeded synthetic prompt the tests and the bench use
 (text-like ids followed by audio-code rows).  `ixt_audio_only_sampling=true` restricts greedy sampling to the audio rows of
-`audio_token_mapping_path` and prints the audio codes next to the rows.
+`audio_token_mapping_path` and prints the audio codes next to the rows.  `ixt_model_dir=DIR` (instead of model_name) runs the model of a folder with
+config.json and model.safetensors (architectures.py), `dtype=float32` in 32-bit where the decoder block has it.
 """
 from __future__ import annotations
 

@@ -137,11 +137,9 @@ def run(args) -> int:
       with open(os.path.join(d, "config.json"), "w", encoding="utf-8") as f:
         json.dump(cfg_json, f)
       mine = _measure(lambda slots: pyconfig.initialize(["bench", base], ixt_model_dir=d, **common(slots)), slots_list, args.opt, lambda m: log(f"{name} vilepel {m}"))
-    row = {"vilepel": mine}
-    if args.batch >= 0:
-      row["closest"] = _measure(lambda slots: pyconfig.initialize(["bench", base], vocab_size=32000, head_dim=128, **like, **common(slots)), slots_list, args.opt, lambda m: log(f"{name} closest {m}"))
-      row["closest_model"] = like.get("decoder_block", "llama2")
-      row["time_ratio"] = {k: mine[k].get("ms", mine[k].get("ms_per_step")) / row["closest"][k].get("ms", row["closest"][k].get("ms_per_step")) for k in mine}
-    rows[name] = row
+    closest = _measure(lambda slots: pyconfig.initialize(["bench", base], vocab_size=32000, head_dim=128, **like, **common(slots)), slots_list, args.opt,
+                       lambda m: log(f"{name} closest {m}"))
+    time_of = lambda r: r.get("ms", r.get("ms_per_step"))
+    rows[name] = {"vilepel": mine, "closest": closest, "closest_model": like.get("decoder_block", "llama2"), "time_ratio": {k: time_of(mine[k]) / time_of(closest[k]) for k in mine}}
   print(json.dumps({"metric": "hybrid_decoder_rates", "data": "synthetic", "dtype": "bf16", "build_id": build.source_hash(), "rows": rows}), flush=True)
   return 0

@@ -15,7 +15,7 @@ from typing import List
 
 SLOTS = 4            # requests that may be live at a time
 PAGE = 64
-MAX_ROWS = 8192      # rows of one pass; longer steps run as several
+MAX_ROWS = 4096      # rows of one pass; longer steps run as several
 
 
 def main(argv: List[str] | None = None) -> int:
