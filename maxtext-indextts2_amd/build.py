@@ -5,18 +5,19 @@ import hashlib
 import os
 import subprocess
 import sys
+import tempfile
 
 PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(PKG_DIR, "csrc")
 LIB = os.path.join(PKG_DIR, "libixt.so")
-SOURCES = ["ixt_api.hip"]
-HEADERS = ["ixt_device.h", "ixt_kernels.h", "ixt_gemma_kernels.h", "ixt_moe_kernels.h", "ixt_gemm.h", "ixt_small.h", "ixt_fp8.h", "ixt_hybrid_kernels.h", "ixt_hybrid.h", "ixt_train_kernels.h", "ixt_train.hip", os.path.join("..", "..", "include", "ixt.h"),
+SOURCES = ["ixt_api.hip", "ixt_hybrid.hip", "ixt_train.hip"]
+HEADERS = ["ixt_device.h", "ixt_kernels.h", "ixt_gemma_kernels.h", "ixt_moe_kernels.h", "ixt_gemm.h", "ixt_small.h", "ixt_fp8.h", "ixt_hybrid_kernels.h", "ixt_internal.h", "ixt_train_kernels.h", os.path.join("..", "..", "include", "ixt.h"),
            os.path.join("..", "..", "include", "ixt_train.h")]
 
 # -ffp-contract=off: the numerics contract allows fused multiply-adds only where the source
 # says fmaf; correctly rounded f32 divide/sqrt and IEEE denormals are hipcc defaults and are stated explicitly.
 HIPCC_FLAGS = [
-    "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared", "-ffp-contract=off", "-fno-fast-math",
+    "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fno-fast-math",
     "-fhip-fp32-correctly-rounded-divide-sqrt", "-fno-gpu-flush-denormals-to-zero", "-Wall", "-Wno-unused-function",
     # no packed-f32 instructions: some of their forms give wrong results on this hardware now and then
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
@@ -58,10 +59,18 @@ def build(force: bool = False, verbose: bool = False) -> str:
   if not force and not needs_build():
     return LIB
   h = source_hash()
-  cmd = [hipcc()] + HIPCC_FLAGS + [f'-DIXT_SOURCE_HASH="{h}"'] + [os.path.join(CSRC, s) for s in SOURCES] + ["-o", LIB]
-  if verbose:
-    print(" ".join(cmd), flush=True)
-  subprocess.check_call(cmd)
+  with tempfile.TemporaryDirectory(prefix="ixt_build_") as tmp:       # one object per source, side by side
+    jobs, objects = [], []
+    for s in SOURCES:
+      objects.append(os.path.join(tmp, s + ".o"))
+      cmd = [hipcc()] + HIPCC_FLAGS + ["-c", f'-DIXT_SOURCE_HASH="{h}"', os.path.join(CSRC, s), "-o", objects[-1]]
+      if verbose:
+        print(" ".join(cmd), flush=True)
+      jobs.append((cmd, subprocess.Popen(cmd)))
+    failed = [cmd for cmd, p in jobs if p.wait() != 0]
+    if failed:
+      raise subprocess.CalledProcessError(1, failed[0])
+    subprocess.check_call([hipcc(), "--offload-arch=gfx950", "-fPIC", "-shared"] + objects + ["-o", LIB])
   with open(LIB + ".hash", "w", encoding="utf-8") as f:
     f.write(h + "\n")
   return LIB

@@ -30,7 +30,7 @@ __device__ __forceinline__ uint32_t f8pack(float a, float b, uint32_t old, bool 
 
 // ---- weights: bf16 kernel in the dot kernels' fragment order (widx, final column order) -> e4m3 fragments + one scale per column.
 //      grid = N (one block per column), block 256.
-__global__ __launch_bounds__(256) void k_f8_quant_w(const bf16_t* __restrict__ w /*widx*/, int K, int N, uint8_t* __restrict__ w8, float* __restrict__ wscale) {
+static __global__ __launch_bounds__(256) void k_f8_quant_w(const bf16_t* __restrict__ w /*widx*/, int K, int N, uint8_t* __restrict__ w8, float* __restrict__ wscale) {
   __shared__ float red[4];
   const int n = blockIdx.x, tid = threadIdx.x;
   float m = 0.0f;
@@ -50,7 +50,7 @@ __global__ __launch_bounds__(256) void k_f8_quant_w(const bf16_t* __restrict__ w
 
 // ---- activations: bf16 rows in the dot kernels' x layout (xidx) -> e4m3 fragments + one scale per (row, 512-k block).
 //      grid = (chains, row blocks), block 64: lane (r = lane % 16, kq = lane / 16) holds its row's 8 k of every 32-k step of the block.
-__global__ __launch_bounds__(64) void k_f8_quant_x(const bf16_t* __restrict__ x /*xidx*/, int K, int R, uint8_t* __restrict__ x8, float* __restrict__ xscale /*[rows16][chains]*/) {
+static __global__ __launch_bounds__(64) void k_f8_quant_x(const bf16_t* __restrict__ x /*xidx*/, int K, int R, uint8_t* __restrict__ x8, float* __restrict__ xscale /*[rows16][chains]*/) {
   const int c = blockIdx.x, rb = blockIdx.y, lane = threadIdx.x;
   const int nsteps = K >> 5, chains = gridDim.x;
   const int s0 = c * 16, cs = min(16, nsteps - s0);
@@ -158,7 +158,7 @@ __global__ __launch_bounds__(256, 2) void k_dotb8(const u32x4* __restrict__ x8, 
 }
 
 // f32 -> e4m3 -> f32 (tests: the conversion against the numpy restatement of OCP e4m3 rounding)
-__global__ void k_f8_roundtrip(const float* in, float* out, int64_t n) {
+static __global__ void k_f8_roundtrip(const float* in, float* out, int64_t n) {
   const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (i >= n) return;
   const uint32_t p = f8pack(in[i], 0.0f, 0, false);

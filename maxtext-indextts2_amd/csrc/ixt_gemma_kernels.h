@@ -21,7 +21,7 @@ struct GNormArgs {
   int E; float eps;
 };
 
-__global__ __launch_bounds__(256) void k_gnorm(GNormArgs a) {
+static __global__ __launch_bounds__(256) void k_gnorm(GNormArgs a) {
   extern __shared__ __attribute__((aligned(16))) float smem[];
   float* row = smem;             // [E] o, then h
   float* blk = smem + a.E;       // [<=64] block sums of o^2
@@ -117,7 +117,7 @@ __global__ __launch_bounds__(256) void k_gnorm(GNormArgs a) {
 // =====================================================================================================
 // GELU(tanh) gate from partial slices: k_swiglu_part with ixt_geglu (linears.py:449-464 with mlp_activations ["gelu", "linear"]).
 // =====================================================================================================
-__global__ __launch_bounds__(256) void k_geglu_part(const float* part, int slices, size_t slice_stride, int F, bf16_t* out /*[R][F] in xidx layout*/) {
+static __global__ __launch_bounds__(256) void k_geglu_part(const float* part, int slices, size_t slice_stride, int F, bf16_t* out /*[R][F] in xidx layout*/) {
   const int f0 = (blockIdx.x * 256 + threadIdx.x) * 8, r = blockIdx.y;
   if (f0 >= F) return;
   const float* p = part + (size_t)r * 2 * F;
@@ -142,7 +142,7 @@ __global__ __launch_bounds__(256) void k_geglu_part(const float* part, int slice
   *reinterpret_cast<u32x4*>(out + xidx(r, f0, F)) = ov;
 }
 
-__global__ __launch_bounds__(256) void k_geglu(const bf16_t* a, const bf16_t* b, bf16_t* out, int64_t n) {
+static __global__ __launch_bounds__(256) void k_geglu(const bf16_t* a, const bf16_t* b, bf16_t* out, int64_t n) {
   const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (i < n) out[i] = ixt_geglu(bf2f(a[i]), bf2f(b[i]));
 }
@@ -166,7 +166,7 @@ __device__ __forceinline__ float ixt_logit_post(float v, int normalize, float sq
 // (maximum, first index) over the allowed columns in amax_val / amax_idx [row][block] for k_argmax_final (one block per row took 0.48 ms at
 // 258 176 columns: 9 % of a Gemma-2 2B decode step).
 #define IXT_LPOST_COLS 4096
-__global__ __launch_bounds__(256) void k_logits_post(float* logits, int vocab, int normalize, float sqrt_emb, float cap, ColRanges cols, float* amax_val,
+static __global__ __launch_bounds__(256) void k_logits_post(float* logits, int vocab, int normalize, float sqrt_emb, float cap, ColRanges cols, float* amax_val,
                                                      int32_t* amax_idx) {
   __shared__ float bv[256];
   __shared__ int bi[256];
@@ -198,7 +198,7 @@ __global__ __launch_bounds__(256) void k_logits_post(float* logits, int vocab, i
 }
 
 // embedding table [V][E] -> [E][V] (the logits kernel of the tied head before it is re-tiled).  grid = (ceil(V/32), ceil(E/32)), block (32, 8).
-__global__ void k_transpose_ve(const bf16_t* __restrict__ src, bf16_t* __restrict__ dst, int V, int E) {
+static __global__ void k_transpose_ve(const bf16_t* __restrict__ src, bf16_t* __restrict__ dst, int V, int E) {
   __shared__ bf16_t tile[32][33];
   const int v0 = blockIdx.x * 32, e0 = blockIdx.y * 32;
   for (int i = threadIdx.y; i < 32; i += 8) {

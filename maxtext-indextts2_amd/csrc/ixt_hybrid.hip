@@ -1,6 +1,7 @@
-// ixt_hybrid.h -- host side of IXT_BLOCK_HYBRID (included by ixt_api.hip behind the launch helpers): layer plans, weight loading, caches and states,
-// and the forward pass over rows that every engine entry point (prefill chunk, packed rows, decode step) ends in.
-#pragma once
+// ixt_hybrid.hip -- host side of IXT_BLOCK_HYBRID: layer plans, weight loading, caches and states, and the forward pass over rows that every engine
+// entry point (prefill chunk, packed rows, decode step) ends in.
+#include "ixt_internal.h"
+#include "ixt_hybrid_kernels.h"
 
 struct HMat { void* w = nullptr; int K = 0, N = 0, Kp = 0, Np = 0; };       // a dot operand of the ctx's storage type, zero-padded
 struct HLayer {
@@ -84,7 +85,7 @@ static int h_load_mat(const HybridModel* m, const void* src, int dtype, void* ds
   return h_load_nk(src, dtype, (bf16_t*)dst, n, k, Kp, n_off, k_off, inter, trans, st);
 }
 
-static int hybrid_check(const ixt_config& c) {
+int hybrid_check(const ixt_config& c) {
   if (!c.layers || c.num_decoder_layers < 1) return set_err(IXT_ERR_INVALID, "hybrid decoder: no layers");
   if (c.emb_dim < 1 || c.emb_dim > 12288 || c.vocab_size < 1) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: emb_dim %d (1 .. 12288), vocab_size %d", c.emb_dim, c.vocab_size);
   if (c.fp8_weights) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: fp8 weights are not built");
@@ -197,7 +198,7 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
 }
 
 // everything a hybrid ctx owns besides the page state and the row descriptors (which all contexts share)
-static int hybrid_init(ixt_ctx* c) {
+int hybrid_init(ixt_ctx* c) {
   const ixt_config& cf = c->cfg;
   HybridModel* m = c->hy;
   m->f32 = cf.float32 != 0; m->esz = m->f32 ? 4 : 2;
@@ -328,7 +329,7 @@ static int hybrid_init(ixt_ctx* c) {
   return IXT_OK;
 }
 
-static int hybrid_load_weight(ixt_ctx* c, const std::string& name, const void* src, int dtype, const int64_t* shape, int ndim, hipStream_t st) {
+int hybrid_load_weight(ixt_ctx* c, const std::string& name, const void* src, int dtype, const int64_t* shape, int ndim, hipStream_t st) {
   HybridModel* m = c->hy;
   auto it = m->tensors.find(name);
   if (it == m->tensors.end()) return set_err(IXT_ERR_INVALID, "unknown parameter %s", name.c_str());
@@ -346,7 +347,7 @@ static int hybrid_load_weight(ixt_ctx* c, const std::string& name, const void* s
 }
 
 // pages and state of group src -> group dst (dst's pages reserved for `length` tokens) / state only (the page list moves elsewhere)
-static int hybrid_copy_group(ixt_ctx* c, int src, int dst, int npages, hipStream_t st) {
+int hybrid_copy_group(ixt_ctx* c, int src, int dst, int npages, hipStream_t st) {
   HybridModel* m = c->hy;
   if (npages > 0 && m->pg_n > 0) hipLaunchKernelGGL(k_latent_pages_copy, dim3(npages, m->pg_n), dim3(256), 0, st, c->ps, src, dst, m->pg_pools, m->pg_bytes, c->P);
   if (m->st_n > 0) hipLaunchKernelGGL(k_state_copy, dim3(256), dim3(256), 0, st, m->st_bases, m->st_per, m->st_n, src, dst, m->state_len, m->parity);
@@ -632,17 +633,17 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
   if (nl > 0) TRY((hybrid_logits<T>(c, R, lrow0, nl, lrows, argmax_out, logits_out, st)));
   return IXT_OK;
 }
-static int forward_rows_hybrid(ixt_ctx* c, int R, const int32_t* tokens, int len_hint, int lrow0, int nl, const int32_t* lrows, int32_t* argmax_out, float* logits_out, bool decode,
+int forward_rows_hybrid(ixt_ctx* c, int R, const int32_t* tokens, int len_hint, int lrow0, int nl, const int32_t* lrows, int32_t* argmax_out, float* logits_out, bool decode,
                                hipStream_t st) {
   const int nseg_max = decode ? R : std::min(R, c->one_segment ? 1 : c->G);     // a page group has at most one run of rows in a call
   if (c->hy->f32) return forward_rows_hybrid_t<float>(c, R, tokens, len_hint, lrow0, nl, lrows, argmax_out, logits_out, decode, nseg_max, st);
   return forward_rows_hybrid_t<bf16_t>(c, R, tokens, len_hint, lrow0, nl, lrows, argmax_out, logits_out, decode, nseg_max, st);
 }
 
-static HybridModel* hybrid_new() { return new HybridModel(); }
-static void hybrid_free(ixt_ctx* c) { delete c->hy; c->hy = nullptr; }
-static bool hybrid_complete(const ixt_ctx* c) { return c->hy->missing == 0; }
-static int hybrid_prompt_logits(ixt_ctx* c, int row0, int n, hipStream_t st) {       // rows of the last pass's residual stream -> c->plogits
+HybridModel* hybrid_new() { return new HybridModel(); }
+void hybrid_free(ixt_ctx* c) { delete c->hy; c->hy = nullptr; }
+bool hybrid_complete(const ixt_ctx* c) { return c->hy->missing == 0; }
+int hybrid_prompt_logits(ixt_ctx* c, int row0, int n, hipStream_t st) {       // rows of the last pass's residual stream -> c->plogits
   if (c->hy->f32) return hybrid_logits<float>(c, c->h_final_rows, row0, n, nullptr, c->pargmax, c->plogits, st);
   return hybrid_logits<bf16_t>(c, c->h_final_rows, row0, n, nullptr, c->pargmax, c->plogits, st);
 }

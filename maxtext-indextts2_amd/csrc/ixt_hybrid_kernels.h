@@ -85,7 +85,7 @@ __device__ __forceinline__ float f32_softplus(float z) { return z > 20.0f ? z : 
 // ---------------------------------------------------------------------------------------------------- f32 dot
 // out[r][n] = sum_k x[r][k] w[n][k], k ascending by fma.  x [R][Kp], w [Np][Kp] row-major f32, Kp % 32 == 0, Np % 16 == 0.  Grouped: 16-row block rb
 // uses the matrix of group rb_exp[rb] (-1: none), wstride floats apart.  grid (ceil(Np / 64), ceil(R / 16)), block 256 (16 rows x 16 column lanes).
-__global__ __launch_bounds__(256) void k_dot32(const float* __restrict__ x, const float* __restrict__ w, int Kp, int Np, int R, float* __restrict__ out,
+static __global__ __launch_bounds__(256) void k_dot32(const float* __restrict__ x, const float* __restrict__ w, int Kp, int Np, int R, float* __restrict__ out,
                                                const int32_t* __restrict__ rb_exp, size_t wstride) {
   __shared__ float xs[16][33], ws[64][33];
   const int tid = threadIdx.x, n0 = blockIdx.x * 64, r0 = blockIdx.y * 16;
@@ -142,7 +142,7 @@ __global__ void k_load_vec(const S* __restrict__ src, T* __restrict__ dst, int64
 // second segment of a group in one call, idles and is counted in err[0].  The tails of short convolutions are double-buffered: a pass reads parity
 // p and writes 1 - p, so no row waits for another one's tail.
 // head_rb: 16-row block b of a head-major activation matrix (rbh blocks per head) belongs to head b / rbh.
-__global__ __launch_bounds__(1024) void k_segments(int R, int32_t* row_active, const int32_t* row_slot, const int32_t* row_pos, int32_t* row_seg, int32_t* row_j,
+static __global__ __launch_bounds__(1024) void k_segments(int R, int32_t* row_active, const int32_t* row_slot, const int32_t* row_pos, int32_t* row_seg, int32_t* row_j,
                                                    int32_t* seg /*[.][8]*/, int32_t* nseg_out, int32_t* state_len, int32_t* parity, int32_t* claim, int groups,
                                                    int recurrent, int32_t* err, int32_t* head_rb, int nhead_rb, int rbh) {
   __shared__ int s_last[1024];
@@ -210,7 +210,7 @@ __global__ __launch_bounds__(1024) void k_segments(int R, int32_t* row_active, c
 }
 
 // state of group src -> group dst (both tail buffers, the recurrent matrices, the length).  grid (chunks), block 256; n0, n1: floats per group
-__global__ __launch_bounds__(256) void k_state_copy(float* const* bases, const int64_t* per_group, int nbuf, int src, int dst, int32_t* state_len, int32_t* parity) {
+static __global__ __launch_bounds__(256) void k_state_copy(float* const* bases, const int64_t* per_group, int nbuf, int src, int dst, int32_t* state_len, int32_t* parity) {
   for (int b = 0; b < nbuf; ++b) {
     float* p = bases[b];
     const int64_t n = per_group[b];
@@ -218,7 +218,7 @@ __global__ __launch_bounds__(256) void k_state_copy(float* const* bases, const i
   }
   if (blockIdx.x == 0 && threadIdx.x == 0) { state_len[dst] = state_len[src]; parity[dst] = parity[src]; }
 }
-__global__ __launch_bounds__(256) void k_latent_pages_copy(PageStateDev s, int src, int dst, char* const* pools, const int64_t* page_bytes, int P) {
+static __global__ __launch_bounds__(256) void k_latent_pages_copy(PageStateDev s, int src, int dst, char* const* pools, const int64_t* page_bytes, int P) {
   const int i = blockIdx.x, l = blockIdx.y;
   if (i >= s.num_pages_used[dst] || i >= s.num_pages_used[src]) return;
   const int64_t n = page_bytes[l];
@@ -328,7 +328,7 @@ __global__ __launch_bounds__(256) void k_final_norm(const float* __restrict__ x,
 }
 
 // logits = the head's slices; (max, first index) per block of 1024 columns over the allowed ones.  grid (ceil(V / 1024), nl), block 256.
-__global__ __launch_bounds__(256) void k_head_post(Slices t, int V, ColRanges cr, float* __restrict__ logits /*[nl][V] or nullptr*/, float* __restrict__ amax_val,
+static __global__ __launch_bounds__(256) void k_head_post(Slices t, int V, ColRanges cr, float* __restrict__ logits /*[nl][V] or nullptr*/, float* __restrict__ amax_val,
                                                    int32_t* __restrict__ amax_idx) {
   __shared__ float bv[4];
   __shared__ int bi[4];
@@ -830,7 +830,7 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
   }
 }
 // the key splits of a row's heads put together.  grid (R, H), block 128; nsplit <= 16.
-__global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int cols, int H, int Rp,
+static __global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int cols, int H, int Rp,
                                                         const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
   __shared__ float fac[16];
   const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
@@ -931,7 +931,7 @@ struct DeltaPrepArgs {
   float* tails;                             // [group][2][taps - 1][C]
   float *q, *k, *kq, *v, *dec, *beta;       // [R][KH][dp], .., [R][KH], [R][H][dv], [R][H][dp], [R][H]
 };
-__global__ __launch_bounds__(256) void k_delta_prep(DeltaPrepArgs a) {
+static __global__ __launch_bounds__(256) void k_delta_prep(DeltaPrepArgs a) {
   const DeltaGeom& g = a.g;
   const int r = blockIdx.x, lane = threadIdx.x & 63, vi = blockIdx.y * 4 + (threadIdx.x >> 6);
   const int s = a.row_seg[r];
@@ -1298,7 +1298,7 @@ __global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, cons
     if (r0 + i < R) route_top(z + (size_t)i * n, n, top, lane, idx + (size_t)(r0 + i) * top, wts + (size_t)(r0 + i) * top);
 }
 // any number of experts (<= 1024): destination row of every copy by one pass of counters; the order inside an expert is free.  One block of 1024.
-__global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __restrict__ idx, int npairs, int n, int align, int nrb_cap, int32_t* __restrict__ pos, int32_t* __restrict__ rb_exp) {
+static __global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __restrict__ idx, int npairs, int n, int align, int nrb_cap, int32_t* __restrict__ pos, int32_t* __restrict__ rb_exp) {
   __shared__ int cnt[1024], off[1024];
   const int tid = threadIdx.x;
   cnt[tid] = 0;
@@ -1323,12 +1323,12 @@ __global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __restrict
     for (int i = 0; i < (cnt[tid] + 15) / 16; ++i) rb_exp[base / 16 + i] = tid;
   for (int p = tid; p < npairs; p += 1024) pos[p] += off[idx[p]];
 }
-__global__ __launch_bounds__(256) void k_gather32(const float* __restrict__ x, const int32_t* __restrict__ pos, int top, int Ep, float* __restrict__ xg) {
+static __global__ __launch_bounds__(256) void k_gather32(const float* __restrict__ x, const int32_t* __restrict__ pos, int top, int Ep, float* __restrict__ xg) {
   const int k = blockIdx.x * 256 + threadIdx.x, p = blockIdx.y;
   if (k < Ep) xg[(size_t)pos[p] * Ep + k] = x[(size_t)(p / top) * Ep + k];
 }
 // few rows whose expert outputs lie in many split-K slices: the weighted sum of a row's copies as one slice.  grid (ceil(ncols / 256), R), block 64.
-__global__ __launch_bounds__(64) void k_moe_sum(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, float* __restrict__ out) {
+static __global__ __launch_bounds__(64) void k_moe_sum(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, float* __restrict__ out) {
   const int c = (blockIdx.x * 64 + threadIdx.x) * 4, r = blockIdx.y;
   if (c >= t.ncols) return;
   float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};

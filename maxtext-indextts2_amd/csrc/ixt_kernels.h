@@ -550,13 +550,13 @@ __global__ void k_tile_w(const T* __restrict__ src, bf16_t* __restrict__ dst, in
 }
 
 // x [R][K] row-major bf16 -> the dot kernel's x layout (op-level entry point only; the model's producers write it directly)
-__global__ void k_transpose_x(const bf16_t* x, bf16_t* xT, int R, int K) {
+static __global__ void k_transpose_x(const bf16_t* x, bf16_t* xT, int R, int K) {
   const int k = blockIdx.x * blockDim.x + threadIdx.x, r = blockIdx.y;
   if (k < K) xT[xidx(r, k, K)] = x[(size_t)r * K + k];
 }
 
 // final (max, first index) over the per-tile pairs.  grid = R, block 256.
-__global__ __launch_bounds__(256) void k_argmax_final(const float* amax_val, const int32_t* amax_idx, int ntiles, int32_t* out_idx) {
+static __global__ __launch_bounds__(256) void k_argmax_final(const float* amax_val, const int32_t* amax_idx, int ntiles, int32_t* out_idx) {
   __shared__ float bv[256];
   __shared__ int bi[256];
   const int r = blockIdx.x, tid = threadIdx.x;
@@ -580,7 +580,7 @@ __global__ __launch_bounds__(256) void k_argmax_final(const float* amax_val, con
 }
 
 // h_out = bf16(h_in + bf16(sum of slices))  (llama2.py:127, :157).  grid = (ceil(E/256), R), block 128, 2 columns per thread.
-__global__ __launch_bounds__(128) void k_sumres(const float* part, int slices, size_t slice_stride, const bf16_t* h_in, bf16_t* h_out, int E) {
+static __global__ __launch_bounds__(128) void k_sumres(const float* part, int slices, size_t slice_stride, const bf16_t* h_in, bf16_t* h_out, int E) {
   const int c = (blockIdx.x * 128 + threadIdx.x) * 2, r = blockIdx.y;
   if (c >= E) return;
   const float2 o = sum_slices2<16>(part + (size_t)r * E + c, slice_stride, slices);
@@ -695,7 +695,7 @@ __global__ __launch_bounds__(256) void k_rownorm(RowNormArgs a) {
 // grid = (ceil(F/2048), R), block 256: a thread owns 8 consecutive features (two 16-byte loads per slice and operand, one
 // 16-byte store: 8 consecutive features of a row are one lane's fragment bytes in the dot kernel's x layout).
 // =====================================================================================================
-__global__ __launch_bounds__(256) void k_swiglu_part(const float* part, int slices, size_t slice_stride, int F,
+static __global__ __launch_bounds__(256) void k_swiglu_part(const float* part, int slices, size_t slice_stride, int F,
                                                       bf16_t* out /*[R][F] in xidx layout*/, const int32_t* rb_exp = nullptr) {
   const int f0 = (blockIdx.x * 256 + threadIdx.x) * 8, r = blockIdx.y;
   if (f0 >= F) return;
@@ -724,11 +724,11 @@ __global__ __launch_bounds__(256) void k_swiglu_part(const float* part, int slic
 
 // op-level helpers of the layers.* module surface: residual add bf16(a + b) (llama2.py:127, :157) and the embedding gather
 // (embeddings.py:154).  Elementwise, 8 elements per thread where the size allows.
-__global__ __launch_bounds__(256) void k_residual(const bf16_t* a, const bf16_t* b, bf16_t* out, int64_t n) {
+static __global__ __launch_bounds__(256) void k_residual(const bf16_t* a, const bf16_t* b, bf16_t* out, int64_t n) {
   const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (i < n) out[i] = f2bf(bf2f(a[i]) + bf2f(b[i]));
 }
-__global__ __launch_bounds__(256) void k_embed(const bf16_t* table, const int32_t* ids, bf16_t* out, int E, int V) {
+static __global__ __launch_bounds__(256) void k_embed(const bf16_t* table, const int32_t* ids, bf16_t* out, int E, int V) {
   const int r = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 8;
   if (c >= E) return;
   int id = ids[r];
@@ -736,7 +736,7 @@ __global__ __launch_bounds__(256) void k_embed(const bf16_t* table, const int32_
   *reinterpret_cast<u32x4*>(out + (size_t)r * E + c) = *reinterpret_cast<const u32x4*>(table + (size_t)id * E + c);
 }
 
-__global__ __launch_bounds__(256) void k_swiglu(const bf16_t* a, const bf16_t* b, bf16_t* out, int64_t n) {
+static __global__ __launch_bounds__(256) void k_swiglu(const bf16_t* a, const bf16_t* b, bf16_t* out, int64_t n) {
   const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (i < n) out[i] = ixt_swiglu(bf2f(a[i]), bf2f(b[i]));
 }
@@ -796,7 +796,7 @@ struct QkvArgs {
   float eps = 0.0f, q_scalar = 0.0f;
 };
 
-__global__ __launch_bounds__(64) void k_qkv_finalize(QkvArgs a) {
+static __global__ __launch_bounds__(64) void k_qkv_finalize(QkvArgs a) {
   const int r = blockIdx.x, hh = blockIdx.y;
   const AttnGeom& g = a.g;
   const int half = g.hd / 2;
@@ -872,7 +872,7 @@ __global__ __launch_bounds__(64) void k_qkv_finalize(QkvArgs a) {
 }
 
 // ---- dense k/v bf16 [R][nkv][hd] -> pages (op-level entry point).  grid = (R, nkv), block = hd.
-__global__ void k_kv_write(const bf16_t* k, const bf16_t* v, const int32_t* row_slot, const int32_t* row_pos,
+static __global__ void k_kv_write(const bf16_t* k, const bf16_t* v, const int32_t* row_slot, const int32_t* row_pos,
                            const int32_t* row_active, const int32_t* page_map, bf16_t* kpages, bf16_t* vpages, AttnGeom g) {
   const int r = blockIdx.x, kvh = blockIdx.y, d = threadIdx.x;
   if (!row_active[r] || d >= g.hd) return;
@@ -885,7 +885,7 @@ __global__ void k_kv_write(const bf16_t* k, const bf16_t* v, const int32_t* row_
 }
 
 // ---- pages -> dense [len][nkv][hd] (cache export).  grid = (len, nkv), block = hd.
-__global__ void k_kv_gather(const bf16_t* kpages, const bf16_t* vpages, const int32_t* page_map, int slot, AttnGeom g,
+static __global__ void k_kv_gather(const bf16_t* kpages, const bf16_t* vpages, const int32_t* page_map, int slot, AttnGeom g,
                             bf16_t* k_out, bf16_t* v_out) {
   const int j = blockIdx.x, kvh = blockIdx.y, d = threadIdx.x;
   if (d >= g.hd) return;
@@ -2001,7 +2001,7 @@ __global__ __launch_bounds__(256, 2) void k_attn_tile(TileAttnArgs a) {
 }
 
 // ---- step 4: out = bf16(sum over super-blocks, in order).  grid = R, block 256.
-__global__ __launch_bounds__(256) void k_attn_combine(const float* pvpart, const int32_t* row_pos, const int32_t* row_active,
+static __global__ __launch_bounds__(256) void k_attn_combine(const float* pvpart, const int32_t* row_pos, const int32_t* row_active,
                                                       bf16_t* out, AttnGeom g, int kmajor) {
   const int r = blockIdx.x;
   const int kv_len = row_active[r] ? row_pos[r] + 1 : 0;
@@ -2020,7 +2020,7 @@ __global__ __launch_bounds__(256) void k_attn_combine(const float* pvpart, const
 // inference_utils.log_prob_of_chosen_token (inference_utils.py:56-63) on rows of f32 logits: (x[chosen] - max) - log(sum exp(x - max)); the sum
 // in blocks of 1024 consecutive columns (one thread each, left to right), block sums added left to right.  grid = rows, block 256.
 // =====================================================================================================
-__global__ __launch_bounds__(256) void k_logprob(const float* __restrict__ logits, int vocab, const int32_t* __restrict__ chosen, float* __restrict__ out) {
+static __global__ __launch_bounds__(256) void k_logprob(const float* __restrict__ logits, int vocab, const int32_t* __restrict__ chosen, float* __restrict__ out) {
   extern __shared__ float lp_sm[];              // [ceil(vocab / 1024)] block sums
   __shared__ float wred[4];
   const int r = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
@@ -2051,7 +2051,7 @@ __global__ __launch_bounds__(256) void k_logprob(const float* __restrict__ logit
 // RoPE on dense rows (op-level).  grid = (R, nheads), block = hd/2.
 // =====================================================================================================
 // rope32 (rope_type "llama3.1"): the pair of table index i is the NEIGHBOURING features (2 i, 2 i + 1) of the caller's row (embeddings.py:446-458).
-__global__ void k_rope(bf16_t* x, const int32_t* pos, const bf16_t* rope_sin, const bf16_t* rope_cos, int nheads, int hd, int rope32) {
+static __global__ void k_rope(bf16_t* x, const int32_t* pos, const bf16_t* rope_sin, const bf16_t* rope_cos, int nheads, int hd, int rope32) {
   const int r = blockIdx.x, h = blockIdx.y, i = threadIdx.x, half = hd / 2;
   if (i >= half) return;
   bf16_t* p = x + ((size_t)r * nheads + h) * hd;
@@ -2067,7 +2067,7 @@ __global__ void k_rope(bf16_t* x, const int32_t* pos, const bf16_t* rope_sin, co
 // =====================================================================================================
 // A row is computed (K/V written, keys attended) only where the page manager has granted the page of its position: a reservation that
 // found no room leaves the group without pages (page_manager.py:305-311), and such rows must not write through stale page_map entries.
-__global__ void k_rows_prefill(int32_t* row_slot, int32_t* row_pos, int32_t* row_active, int slot, int start, int n,
+static __global__ void k_rows_prefill(int32_t* row_slot, int32_t* row_pos, int32_t* row_active, int slot, int start, int n,
                                const int32_t* num_pages_used, int P) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) { row_slot[i] = slot; row_pos[i] = start + i; row_active[i] = (start + i) / P < num_pages_used[slot] ? 1 : 0; }
@@ -2075,7 +2075,7 @@ __global__ void k_rows_prefill(int32_t* row_slot, int32_t* row_pos, int32_t* row
 // caller-described rows (packed prefill): slot and position per row, same page guard; out-of-range descriptors make the row inactive
 // max_len: the caller's bound on position + 1 (it sizes the tiled attention's score rows); a row at or beyond it is idle and counted in
 // status[3] instead of being computed against a bound the caller did not mean.
-__global__ void k_rows_packed(int32_t* row_slot, int32_t* row_pos, int32_t* row_active, const int32_t* slot_in, const int32_t* pos_in, int n,
+static __global__ void k_rows_packed(int32_t* row_slot, int32_t* row_pos, int32_t* row_active, const int32_t* slot_in, const int32_t* pos_in, int n,
                               const int32_t* num_pages_used, int P, int groups, int Tmax, int max_len, int32_t* status) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) {
@@ -2090,7 +2090,7 @@ __global__ void k_rows_packed(int32_t* row_slot, int32_t* row_pos, int32_t* row_
 // deactivates the row instead of letting it write through a stale page_map entry), and -- check_len, ixt_generate -- the position is
 // the one the page manager has just advanced to (sequence_lengths - 1): a slot that was prefilled but not inserted yet carries the
 // previous occupant's next_pos and stays idle until MaxEngine.insert.
-__global__ void k_rows_decode(int32_t* row_slot, int32_t* row_pos, int32_t* row_active, int32_t* row_tok,
+static __global__ void k_rows_decode(int32_t* row_slot, int32_t* row_pos, int32_t* row_active, int32_t* row_tok,
                               const int32_t* tokens, const int32_t* pos, const int32_t* has_active, const int32_t* num_pages_used,
                               const int32_t* sequence_lengths, int check_len, int P, int Tmax, int B) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
@@ -2102,7 +2102,7 @@ __global__ void k_rows_decode(int32_t* row_slot, int32_t* row_pos, int32_t* row_
   }
 }
 // maxengine.py:913-935
-__global__ void k_generate_epilogue(const int32_t* new_tok, int32_t* tokens, int32_t* next_pos, int32_t* generated,
+static __global__ void k_generate_epilogue(const int32_t* new_tok, int32_t* tokens, int32_t* next_pos, int32_t* generated,
                                     int32_t* result, int B) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i < B) {
@@ -2137,7 +2137,7 @@ struct PageStateDev {
 // same wave re-reads words that its lane 0 has just written.
 __device__ __forceinline__ void wave_drain() { __builtin_amdgcn_fence(__ATOMIC_SEQ_CST, "workgroup"); }
 
-__device__ void wave_release_group(PageStateDev s, int g, int lane) {
+static __device__ void wave_release_group(PageStateDev s, int g, int lane) {
   const int nvalid = ldg_i32(s.num_pages_used + g);
   int nrel = 0, lowest = 0x7fffffff;
   for (int i = lane; i < s.mpg; i += 64) {
@@ -2159,7 +2159,7 @@ __device__ void wave_release_group(PageStateDev s, int g, int lane) {
   wave_drain();
 }
 
-__global__ __launch_bounds__(64) void k_pages_reset(PageStateDev s) {
+static __global__ __launch_bounds__(64) void k_pages_reset(PageStateDev s) {
   const int lane = threadIdx.x;
   for (int i = lane; i < s.num_pages; i += 64) s.page_status[i] = (i == 0) ? 1 : 0;
   for (int i = lane; i < s.groups * s.mpg; i += 64) s.page_map[i] = 0;
@@ -2171,7 +2171,7 @@ __global__ __launch_bounds__(64) void k_pages_reset(PageStateDev s) {
   if (lane == 0) { s.meta[0] = s.num_pages - 1; s.meta[1] = 1; }
 }
 // page_status written from outside (tests): count the free pages and find the lowest one again
-__global__ __launch_bounds__(64) void k_pages_recount(PageStateDev s) {
+static __global__ __launch_bounds__(64) void k_pages_recount(PageStateDev s) {
   const int lane = threadIdx.x;
   int c = 0, lowest = s.num_pages;
   for (int i = 1 + lane; i < s.num_pages; i += 64)
@@ -2180,7 +2180,7 @@ __global__ __launch_bounds__(64) void k_pages_recount(PageStateDev s) {
   for (int off = 1; off < 64; off <<= 1) { c += __shfl_xor(c, off, 64); lowest = min(lowest, __shfl_xor(lowest, off, 64)); }
   if (lane == 0) { s.meta[0] = c; s.meta[1] = lowest; }
 }
-__global__ __launch_bounds__(64) void k_pages_release(PageStateDev s, int g) { wave_release_group(s, g, threadIdx.x); }
+static __global__ __launch_bounds__(64) void k_pages_release(PageStateDev s, int g) { wave_release_group(s, g, threadIdx.x); }
 
 // The m lowest free pages (index >= 1) in ascending order -> out[0..m) (LDS), each marked used; returns how many exist (<= m).
 // Sequential first-fit (page_manager.py:268-283, :373-395: "next free page" for one request after the other, nothing freed in
@@ -2189,7 +2189,7 @@ __global__ __launch_bounds__(64) void k_pages_release(PageStateDev s, int g) { w
 // The scan starts at meta[1] (no page below it is free: releases lower it, and the m lowest free pages having been taken, everything up to
 // the last of them is in use) and meta[0] counts the free pages -- the pool of a 1024-slot engine has 41 000 status words, and a scan from
 // index 0 per reservation cost 117 us.
-__device__ int wave_take_free(PageStateDev s, int lane, int m, int32_t* out) {
+static __device__ int wave_take_free(PageStateDev s, int lane, int m, int32_t* out) {
   int32_t* status = s.page_status;
   const int num_pages = s.num_pages;
   int cnt = 0, last = -1;
@@ -2226,7 +2226,7 @@ __device__ int wave_take_free(PageStateDev s, int lane, int m, int32_t* out) {
 #define IXT_MAX_GROUPS 4096
 
 // release + reserve (page_manager.py:208-328); extend != 0: keep pages, grow to `length` tokens (build extension)
-__global__ __launch_bounds__(64) void k_pages_reserve(PageStateDev s, int g, int length, int extend) {
+static __global__ __launch_bounds__(64) void k_pages_reserve(PageStateDev s, int g, int length, int extend) {
   __shared__ int32_t got[IXT_MAX_GROUPS];
   const int lane = threadIdx.x;
   if (!extend) {
@@ -2257,7 +2257,7 @@ __global__ __launch_bounds__(64) void k_pages_reserve(PageStateDev s, int g, int
 
 // page_manager.py:331-412: every active group advances one token; groups that cross a page boundary take the next free page,
 // in group order
-__global__ __launch_bounds__(64) void k_pages_advance(PageStateDev s) {
+static __global__ __launch_bounds__(64) void k_pages_advance(PageStateDev s) {
   __shared__ int32_t need[IXT_MAX_GROUPS];
   __shared__ int32_t got[IXT_MAX_GROUPS];
   const int lane = threadIdx.x;
@@ -2290,12 +2290,12 @@ __global__ __launch_bounds__(64) void k_pages_advance(PageStateDev s) {
     s.active_page[gg] = nf;
   }
 }
-__global__ void k_pages_set_active(PageStateDev s, int g, int v) { s.has_active_page[g] = v; }
+static __global__ void k_pages_set_active(PageStateDev s, int g, int v) { s.has_active_page[g] = v; }
 
 // ---- build extensions around MaxEngine.insert (no reference counterpart) ----------------------------------
 // insert of a prefix of `length` tokens into the slot that already holds its pages: has_active_page = 1 (maxengine.py:1189-1191) and the
 // length fields back to their post-prefill values -- a generate() between prefill(slot) and insert(slot) has advanced them.
-__global__ void k_pages_resync(PageStateDev s, int g, int length) {
+static __global__ void k_pages_resync(PageStateDev s, int g, int length) {
   const int need = (length + s.P - 1) / s.P;
   if (need > s.num_pages_used[g] || need < 1) return;           // the reservation failed: leave the (empty) group alone
   s.sequence_lengths[g] = length;
@@ -2305,7 +2305,7 @@ __global__ void k_pages_resync(PageStateDev s, int g, int length) {
 }
 // hand the pages of group `src` (a staging group filled by a packed prefill) to slot `dst`: dst's old pages are released, the page list
 // moves (no K/V byte is copied), src ends empty.  One wave.
-__global__ __launch_bounds__(64) void k_pages_move(PageStateDev s, int src, int dst) {
+static __global__ __launch_bounds__(64) void k_pages_move(PageStateDev s, int src, int dst) {
   const int lane = threadIdx.x;
   wave_release_group(s, dst, lane);
   __syncthreads();
@@ -2320,7 +2320,7 @@ __global__ __launch_bounds__(64) void k_pages_move(PageStateDev s, int src, int 
 }
 // copy the K and V pages of group `src` (first `npages` logical pages) into the pages of group `dst`, all layers (the reference's page
 // copy loop, maxengine.py:1106-1125).  grid = (npages, layers), block 256; kp / vp: per-layer pool pointers.
-__global__ __launch_bounds__(256) void k_pages_copy(PageStateDev s, int src, int dst, bf16_t* const* kp, bf16_t* const* vp, size_t page_elems) {
+static __global__ __launch_bounds__(256) void k_pages_copy(PageStateDev s, int src, int dst, bf16_t* const* kp, bf16_t* const* vp, size_t page_elems) {
   const int i = blockIdx.x, l = blockIdx.y;
   if (i >= s.num_pages_used[dst] || i >= s.num_pages_used[src]) return;
   const size_t so = (size_t)s.page_map[(size_t)src * s.mpg + i] * page_elems, d_o = (size_t)s.page_map[(size_t)dst * s.mpg + i] * page_elems;

@@ -11,7 +11,7 @@
 
 // grid = R, block = 64 n_exp (one wave per expert: the n_exp dot products of a row run side by side, each wave's loads of a block of 512 k
 // issued together).  xn: the dot kernels' x layout (xidx); gate: row-major bf16 [E][n_exp].
-__global__ __launch_bounds__(1024) void k_moe_route(const bf16_t* xn, const bf16_t* gate, int E, int n_exp, int top_k, int32_t* idx_out /*[R][top_k]*/,
+static __global__ __launch_bounds__(1024) void k_moe_route(const bf16_t* xn, const bf16_t* gate, int E, int n_exp, int top_k, int32_t* idx_out /*[R][top_k]*/,
                                                    float* w_out /*[R][top_k]*/) {
   __shared__ float gl[IXT_MOE_MAX_EXPERTS];
   const int r = blockIdx.x, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
@@ -135,7 +135,7 @@ __global__ __launch_bounds__(1024) void k_moe_route_blocks(const bf16_t* xn, con
 }
 
 // Expert e's down-projection slices -> bf16 -> the (row, j) slots that selected e.  grid = ((E + 255) / 256, R), block 256.
-__global__ __launch_bounds__(256) void k_moe_scatter(const float* part, int slices, size_t slice_stride, int E, int e, int top_k, const int32_t* idx,
+static __global__ __launch_bounds__(256) void k_moe_scatter(const float* part, int slices, size_t slice_stride, int E, int e, int top_k, const int32_t* idx,
                                                      bf16_t* ybuf /*[R][top_k][E]*/) {
   const int c = blockIdx.x * 256 + threadIdx.x, r = blockIdx.y;
   if (c >= E) return;
@@ -147,7 +147,7 @@ __global__ __launch_bounds__(256) void k_moe_scatter(const float* part, int slic
 }
 
 // out[r][c] = bf16(fma chain over j of y_j * weight_j) as one f32 "slice" (the residual / norm kernels take it from there).
-__global__ __launch_bounds__(256) void k_moe_combine(const bf16_t* ybuf, const float* w, int E, int top_k, float* out /*[R][E]*/, bf16_t* out16 = nullptr) {
+static __global__ __launch_bounds__(256) void k_moe_combine(const bf16_t* ybuf, const float* w, int E, int top_k, float* out /*[R][E]*/, bf16_t* out16 = nullptr) {
   const int c = blockIdx.x * 256 + threadIdx.x, r = blockIdx.y;
   if (c >= E) return;
   float t = 0.0f;
@@ -157,7 +157,7 @@ __global__ __launch_bounds__(256) void k_moe_combine(const bf16_t* ybuf, const f
 }
 
 // bf16(sum of slices) of a [R][N] projection (op-level entry points)
-__global__ __launch_bounds__(256) void k_slices_to_bf16(const float* part, int slices, size_t slice_stride, size_t n, bf16_t* out) {
+static __global__ __launch_bounds__(256) void k_slices_to_bf16(const float* part, int slices, size_t slice_stride, size_t n, bf16_t* out) {
   const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
   if (i >= n) return;
   out[i] = f2bf(sum_slices<16>(part + i, slice_stride, slices));
@@ -173,7 +173,7 @@ __global__ __launch_bounds__(256) void k_slices_to_bf16(const float* part, int s
 //   k_moe_gather  xg[pos[p]] = xn[r] in the dot kernels' x layout.
 // The order of the copies inside an expert changes nothing: a row's result does not depend on its neighbours in a launch.
 // =====================================================================================================
-__global__ __launch_bounds__(1024) void k_moe_plan(const int32_t* idx /*[npairs]*/, int npairs, int e0, int n_exp, int align, int nrb_cap, int32_t* pos /*[npairs]*/,
+static __global__ __launch_bounds__(1024) void k_moe_plan(const int32_t* idx /*[npairs]*/, int npairs, int e0, int n_exp, int align, int nrb_cap, int32_t* pos /*[npairs]*/,
                                                    int32_t* rb_exp /*[nrb_cap]*/, int32_t* cnt_off /*[2 n_exp]: counts, then offsets*/) {
   __shared__ int wsum[16];
   __shared__ int s_base, s_off;
@@ -215,7 +215,7 @@ __global__ __launch_bounds__(1024) void k_moe_plan(const int32_t* idx /*[npairs]
 }
 
 // grid = (ceil(E / 2048), npairs), block 256: 8 consecutive features per thread.
-__global__ __launch_bounds__(256) void k_moe_gather(const bf16_t* xn /*xidx, [R][E]*/, const int32_t* pos, int top_k, int E, bf16_t* xg /*xidx*/) {
+static __global__ __launch_bounds__(256) void k_moe_gather(const bf16_t* xn /*xidx, [R][E]*/, const int32_t* pos, int top_k, int E, bf16_t* xg /*xidx*/) {
   const int k0 = (blockIdx.x * 256 + threadIdx.x) * 8, p = blockIdx.y;
   if (k0 >= E || pos[p] < 0) return;
   *reinterpret_cast<u32x4*>(xg + xidx(pos[p], k0, E)) = *reinterpret_cast<const u32x4*>(xn + xidx(p / top_k, k0, E));
@@ -223,7 +223,7 @@ __global__ __launch_bounds__(256) void k_moe_gather(const bf16_t* xn /*xidx, [R]
 
 // The mixture from the experts' down-projection slices in copy-row order: y_j = bf16(sum of slices of row pos[r top_k + j]),
 // out[r][c] = bf16(fma chain over j of y_j weight_j) as one f32 slice (k_moe_combine's arithmetic).  grid = ((E + 255) / 256, R), block 256.
-__global__ __launch_bounds__(256) void k_moe_combine_rows(const float* part, int slices, size_t slice_stride, const int32_t* pos, const float* w, int E, int top_k,
+static __global__ __launch_bounds__(256) void k_moe_combine_rows(const float* part, int slices, size_t slice_stride, const int32_t* pos, const float* w, int E, int top_k,
                                                           float* out /*[R][E]*/) {
   const int c = blockIdx.x * 256 + threadIdx.x, r = blockIdx.y;
   if (c >= E) return;
@@ -236,7 +236,7 @@ __global__ __launch_bounds__(256) void k_moe_combine_rows(const float* part, int
 }
 
 // op-level form of the routed evaluation (ixt_op_moe_experts): out[p] = bf16(sum of slices of row pos[p]).  grid = ((E + 255) / 256, npairs).
-__global__ __launch_bounds__(256) void k_moe_rows_out(const float* part, int slices, size_t slice_stride, const int32_t* pos, int E, bf16_t* out /*[npairs][E]*/) {
+static __global__ __launch_bounds__(256) void k_moe_rows_out(const float* part, int slices, size_t slice_stride, const int32_t* pos, int E, bf16_t* out /*[npairs][E]*/) {
   const int c = blockIdx.x * 256 + threadIdx.x, p = blockIdx.y;
   if (c >= E) return;
   out[(size_t)p * E + c] = pos[p] < 0 ? (bf16_t)0 : f2bf(sum_slices<16>(part + (size_t)pos[p] * E + c, slice_stride, slices));

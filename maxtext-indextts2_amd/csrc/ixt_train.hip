@@ -5,7 +5,6 @@
 #include "../../include/ixt_train.h"
 #include "ixt_kernels.h"
 #include "ixt_train_kernels.h"
-// (compiled as part of ixt_api.hip: one translation unit, one libixt.so)
 
 #include <hip/hip_runtime.h>
 #include <math.h>

@@ -157,7 +157,7 @@ __global__ __launch_bounds__(256) void k_tgemm(TGemm g) {
 }
 
 // ---------------------------------------------------------------------------------------------------------------- elementwise / rows
-__global__ void k_t_cast_bf16(const float* __restrict__ src, bf16_t* __restrict__ dst, long n) {
+static __global__ void k_t_cast_bf16(const float* __restrict__ src, bf16_t* __restrict__ dst, long n) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) dst[i] = f2bf(src[i]);
 }
@@ -172,7 +172,7 @@ __device__ __forceinline__ float t_block_sum(float v, float* red) {   // 256 thr
 }
 
 // RMSNorm forward (normalizations.py:57-70): y = bf16(bf16(x r) scale), r = rsqrt(mean(x^2) + eps) saved per row.  grid = T, block 256.
-__global__ __launch_bounds__(256) void k_t_rmsnorm_fwd(const bf16_t* __restrict__ x, const bf16_t* __restrict__ scale, bf16_t* __restrict__ y,
+static __global__ __launch_bounds__(256) void k_t_rmsnorm_fwd(const bf16_t* __restrict__ x, const bf16_t* __restrict__ scale, bf16_t* __restrict__ y,
                                                        float* __restrict__ rstd, int E, float eps) {
   __shared__ float red[4];
   const long row = blockIdx.x;
@@ -188,7 +188,7 @@ __global__ __launch_bounds__(256) void k_t_rmsnorm_fwd(const bf16_t* __restrict_
 // and row took 466 us per launch at 16384 x 2048: 2048 addresses under 33 M atomics).  grid = ceil(T / TN_RPB), block 256, E <= 256 TN_FPT.
 #define TN_RPB 16
 #define TN_FPT 16
-__global__ __launch_bounds__(256) void k_t_rmsnorm_bwd(const float* __restrict__ dy, const bf16_t* __restrict__ x, const bf16_t* __restrict__ scale,
+static __global__ __launch_bounds__(256) void k_t_rmsnorm_bwd(const float* __restrict__ dy, const bf16_t* __restrict__ x, const bf16_t* __restrict__ scale,
                                                        const float* __restrict__ rstd, float* __restrict__ dh, float* __restrict__ dscale, int E, long T) {
   __shared__ float red[4];
   float ds[TN_FPT];
@@ -220,7 +220,7 @@ __global__ __launch_bounds__(256) void k_t_rmsnorm_bwd(const float* __restrict__
   }
 }
 // out[i] = parts[0][i] + parts[1][i] + ... (split-K partial products, in order)
-__global__ void k_t_sum_parts(const float* __restrict__ parts, int nparts, long n, float* __restrict__ out) {
+static __global__ void k_t_sum_parts(const float* __restrict__ parts, int nparts, long n, float* __restrict__ out) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n) return;
   float t = parts[i];
@@ -243,7 +243,7 @@ __global__ void k_t_rope(bf16_t* __restrict__ x, const int32_t* __restrict__ pos
 
 // Attention softmax over scores f32 [BH][S][S] with the train-mode mask (attentions.py:586-618: same segment AND col <= row), P bf16 out.
 // grid = (S, BH), block 256; one row per block.
-__global__ __launch_bounds__(256) void k_t_softmax_fwd(const float* __restrict__ sc, const int32_t* __restrict__ seg, bf16_t* __restrict__ P, int S, int H) {
+static __global__ __launch_bounds__(256) void k_t_softmax_fwd(const float* __restrict__ sc, const int32_t* __restrict__ seg, bf16_t* __restrict__ P, int S, int H) {
   __shared__ float red[4];
   const int row = blockIdx.x;
   const long bh = blockIdx.y, b = bh / H;
@@ -271,7 +271,7 @@ __global__ __launch_bounds__(256) void k_t_softmax_fwd(const float* __restrict__
 // The same row in ONE pass over memory (S <= 256 TS_MAXV): a thread's scores and segment tests stay in registers, every exponential is taken once.
 // Same values as the three-pass form bit for bit (same per-thread order of the partial sums); 1.70 -> see DESIGN.md section 9.
 #define TS_MAXV 16
-__global__ __launch_bounds__(256) void k_t_softmax_fwd_reg(const float* __restrict__ sc, const int32_t* __restrict__ seg, bf16_t* __restrict__ P, int S, int H) {
+static __global__ __launch_bounds__(256) void k_t_softmax_fwd_reg(const float* __restrict__ sc, const int32_t* __restrict__ seg, bf16_t* __restrict__ P, int S, int H) {
   __shared__ float red[4];
   const int row = blockIdx.x;
   const long bh = blockIdx.y, b = bh / H;
@@ -307,7 +307,7 @@ __global__ __launch_bounds__(256) void k_t_softmax_fwd_reg(const float* __restri
   }
 }
 // dS = P o (dP - sum_j dP P), bf16 out (in place of nothing: separate buffer).  grid = (S, BH), block 256.
-__global__ __launch_bounds__(256) void k_t_softmax_bwd(const float* __restrict__ dP, const bf16_t* __restrict__ P, bf16_t* __restrict__ dS, int S) {
+static __global__ __launch_bounds__(256) void k_t_softmax_bwd(const float* __restrict__ dP, const bf16_t* __restrict__ P, bf16_t* __restrict__ dS, int S) {
   __shared__ float red[4];
   const long base = ((long)blockIdx.y * S + blockIdx.x) * S;
   float s = 0.0f;
@@ -316,7 +316,7 @@ __global__ __launch_bounds__(256) void k_t_softmax_bwd(const float* __restrict__
   for (int j = threadIdx.x; j < S; j += 256) { const float p = bf2f(P[base + j]); dS[base + j] = f2bf(p * (dP[base + j] - dot)); }
 }
 // one pass (S <= 256 TS_MAXV); columns beyond the row hold P = 0 (the causal mask): their dP is not read
-__global__ __launch_bounds__(256) void k_t_softmax_bwd_reg(const float* __restrict__ dP, const bf16_t* __restrict__ P, bf16_t* __restrict__ dS, int S) {
+static __global__ __launch_bounds__(256) void k_t_softmax_bwd_reg(const float* __restrict__ dP, const bf16_t* __restrict__ P, bf16_t* __restrict__ dS, int S) {
   __shared__ float red[4];
   const int row = blockIdx.x;
   const long base = ((long)blockIdx.y * S + row) * S;
@@ -339,11 +339,11 @@ __global__ __launch_bounds__(256) void k_t_softmax_bwd_reg(const float* __restri
 }
 
 // SwiGLU (linears.py:449-464) forward: act = bf16(bf16(a sg) b), sg = bf16(sigmoid(a)); backward through the unrounded formula.
-__global__ void k_t_swiglu_fwd(const bf16_t* __restrict__ a, const bf16_t* __restrict__ b, bf16_t* __restrict__ act, long n) {
+static __global__ void k_t_swiglu_fwd(const bf16_t* __restrict__ a, const bf16_t* __restrict__ b, bf16_t* __restrict__ act, long n) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) act[i] = ixt_swiglu(bf2f(a[i]), bf2f(b[i]));
 }
-__global__ void k_t_swiglu_bwd(const bf16_t* __restrict__ dact, const bf16_t* __restrict__ a, const bf16_t* __restrict__ b, bf16_t* __restrict__ da,
+static __global__ void k_t_swiglu_bwd(const bf16_t* __restrict__ dact, const bf16_t* __restrict__ a, const bf16_t* __restrict__ b, bf16_t* __restrict__ da,
                                bf16_t* __restrict__ db, long n) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n) return;
@@ -354,21 +354,21 @@ __global__ void k_t_swiglu_bwd(const bf16_t* __restrict__ dact, const bf16_t* __
 }
 
 // residual stream: h_out = bf16(h + y) (llama2.py:127, :157); gradient helpers
-__global__ void k_t_add_bf16(const bf16_t* __restrict__ a, const bf16_t* __restrict__ b, bf16_t* __restrict__ out, long n) {
+static __global__ void k_t_add_bf16(const bf16_t* __restrict__ a, const bf16_t* __restrict__ b, bf16_t* __restrict__ out, long n) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) out[i] = f2bf(bf2f(a[i]) + bf2f(b[i]));
 }
-__global__ void k_t_f32_to_bf16(const float* __restrict__ a, bf16_t* __restrict__ out, long n) {
+static __global__ void k_t_f32_to_bf16(const float* __restrict__ a, bf16_t* __restrict__ out, long n) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) out[i] = f2bf(a[i]);
 }
-__global__ void k_t_bf16_to_f32(const bf16_t* __restrict__ a, float* __restrict__ out, long n, int add) {
+static __global__ void k_t_bf16_to_f32(const bf16_t* __restrict__ a, float* __restrict__ out, long n, int add) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) out[i] = (add ? out[i] : 0.0f) + bf2f(a[i]);
 }
 
 // embedding: forward gather (embeddings.py:154) = k_embed of ixt_kernels.h; backward scatter-add of dh f32 [T][E] into dE f32 [V][E]
-__global__ void k_t_embed_bwd(const float* __restrict__ dh, const int32_t* __restrict__ ids, float* __restrict__ dE, int E, int V) {
+static __global__ void k_t_embed_bwd(const float* __restrict__ dh, const int32_t* __restrict__ ids, float* __restrict__ dE, int E, int V) {
   const long t = blockIdx.y;
   const int e = blockIdx.x * blockDim.x + threadIdx.x;
   if (e >= E) return;
@@ -379,7 +379,7 @@ __global__ void k_t_embed_bwd(const float* __restrict__ dh, const int32_t* __res
 
 // cross entropy with the reference's VJP (max_utils.py:563-654, z_loss = 0) on a chunk of f32 logits [Tc][V] (already bf16-rounded values,
 // decoders.py:570,586): loss_row = log(sum exp(l - max)) + max - l[target]; dlogits = (softmax - onehot) * weight, bf16.  grid = Tc, block 256.
-__global__ __launch_bounds__(256) void k_t_xent(const float* __restrict__ logits, const int32_t* __restrict__ targets, const int32_t* __restrict__ tseg,
+static __global__ __launch_bounds__(256) void k_t_xent(const float* __restrict__ logits, const int32_t* __restrict__ targets, const int32_t* __restrict__ tseg,
                                                 bf16_t* __restrict__ dlogits, float* __restrict__ row_loss, int V) {
   __shared__ float red[4];
   const long row = blockIdx.x;
@@ -403,13 +403,13 @@ __global__ __launch_bounds__(256) void k_t_xent(const float* __restrict__ logits
 }
 
 // out[i] = 1 where s[i] != 0 (the weight of a target position, train.py:308-309)
-__global__ void k_t_nonzero(const int32_t* __restrict__ s, float* __restrict__ out, long n) {
+static __global__ void k_t_nonzero(const int32_t* __restrict__ s, float* __restrict__ out, long n) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i < n) out[i] = s[i] != 0 ? 1.0f : 0.0f;
 }
 
 // fixed-order sum of n floats by one block (deterministic), optionally of squares; out[0] (+)= sum
-__global__ __launch_bounds__(256) void k_t_reduce(const float* __restrict__ x, long n, int squares, float* __restrict__ out, int accumulate) {
+static __global__ __launch_bounds__(256) void k_t_reduce(const float* __restrict__ x, long n, int squares, float* __restrict__ out, int accumulate) {
   __shared__ float red[4];
   double s = 0.0;
   for (long i = threadIdx.x; i < n; i += 256) { const float v = x[i]; s += squares ? (double)v * v : (double)v; }
@@ -418,7 +418,7 @@ __global__ __launch_bounds__(256) void k_t_reduce(const float* __restrict__ x, l
   if (threadIdx.x == 0) out[0] = (accumulate ? out[0] : 0.0f) + f;
 }
 // sum of squares of a large buffer: one partial per block, then k_t_reduce over the partials.  grid = nblk, block 256.
-__global__ __launch_bounds__(256) void k_t_sumsq_partial(const float* __restrict__ x, long n, float* __restrict__ part) {
+static __global__ __launch_bounds__(256) void k_t_sumsq_partial(const float* __restrict__ x, long n, float* __restrict__ part) {
   __shared__ float red[4];
   float s = 0.0f;
   for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) { const float v = x[i]; s += v * v; }
@@ -429,7 +429,7 @@ __global__ __launch_bounds__(256) void k_t_sumsq_partial(const float* __restrict
 // optax.clip_by_global_norm + optax.adamw (optimizers.py:28-38): g <- g * gscale (1 / total_weights and the clip factor), mu, nu, bias
 // correction with `count` (1 at the first step), decoupled weight decay, p -= lr * update; the bf16 copy of the parameter is refreshed.
 struct AdamArgs { float lr, b1, b2, eps, eps_root, wd, bc1, bc2; };
-__global__ void k_t_adamw(float* __restrict__ p, const float* __restrict__ g, float* __restrict__ mu, float* __restrict__ nu, bf16_t* __restrict__ pb,
+static __global__ void k_t_adamw(float* __restrict__ p, const float* __restrict__ g, float* __restrict__ mu, float* __restrict__ nu, bf16_t* __restrict__ pb,
                           const float* __restrict__ gscale, long n, AdamArgs a) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n) return;
@@ -443,7 +443,7 @@ __global__ void k_t_adamw(float* __restrict__ p, const float* __restrict__ g, fl
   pb[i] = f2bf(np_);
 }
 // gscale[0] = (1 / denom) * min(1, clip / (norm / denom)) with norm = sqrt(sumsq[0]); norms_out = {raw grad norm, clipped grad norm}
-__global__ void k_t_clip_scale(const float* __restrict__ sumsq, float denom, float clip, float* __restrict__ gscale, float* __restrict__ norms_out) {
+static __global__ void k_t_clip_scale(const float* __restrict__ sumsq, float denom, float clip, float* __restrict__ gscale, float* __restrict__ norms_out) {
   const float raw = sqrtf(sumsq[0]) / denom;
   const float f = (clip > 0.0f && raw >= clip) ? clip / raw : 1.0f;
   gscale[0] = f / denom;
