@@ -453,3 +453,23 @@ def test_trace_runner(tmp_path, dtype):
   VH.check(load(0), wa[[0, 63]], dtype)
   VH.check(load(2), np.stack([wa[69], wb[11]]), dtype)
   VH.check(load(3), wb[11:12], dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_large_mixed_steps(tmp_path, dtype):
+  """Steps of some hundred rows made of long portions beside single tokens: the prompt kernels with several requests per tile and per launch."""
+  cfg = VH.mixed_model()
+  w = VH.random_weights(cfg, 18)      # (no routing decision that bf16 inputs alone turn over in the first tokens)
+  eng, _ = VH.engine(VH.write_model(tmp_path, cfg, w), dtype=dtype, slots=4, pages=110, target=256, rows=512)
+  toks = {k: VH.tokens(cfg, n, 100 + n) for k, n in (("a", 250), ("b", 131), ("c", 9), ("d", 200))}
+  s, at, got = VH.scheduler(eng), dict.fromkeys(toks, 0), {k: [] for k in toks}
+  for sizes in ((("a", 1), ("c", 5), ("b", 130)), (("a", 150), ("b", 1), ("d", 129), ("c", 1)), (("d", 70), ("c", 3), ("a", 98)), (("a", 1), ("d", 1))):
+    lg, _ = s.step([(k, toks[k][at[k]:at[k] + n], list(range(n))) for k, n in sizes])
+    lg = lg.cpu().numpy()
+    for k, n in sizes:
+      got[k].append(lg[:n])
+      lg, at[k] = lg[n:], at[k] + n
+  for k in toks:
+    assert at[k] == len(toks[k])
+    VH.check(np.concatenate(got[k]), V.forward(cfg, w, toks[k]), dtype, k)
+  eng.close()
