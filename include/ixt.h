@@ -48,7 +48,7 @@ typedef struct ixt_layer {
   int32_t ffn;                     /* IXT_FFN_NONE | IXT_FFN_DENSE | IXT_FFN_MOE */
   int32_t ff;                      /* hidden size (MoE: of one expert) */
   float glu_limit;                 /* y = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit) */
-  int32_t experts, top;            /* MoE: softmax over all router logits, the `top` largest, weights not renormalized */
+  int32_t experts, top;            /* MoE: weight of a picked expert = its softmax probability among all of them */
 } ixt_layer;
 enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1 };
 enum { IXT_FFN_NONE = 0, IXT_FFN_DENSE = 1, IXT_FFN_MOE = 2 };

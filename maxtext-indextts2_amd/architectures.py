@@ -81,8 +81,7 @@ _VILEPEL_MIXERS = {"latent_attention": _vilepel_latent, "channel_delta": _vilepe
 
 
 def vilepel_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
-  """Vilepel: layers of latent attention and of a gated delta rule with per-channel decay in any order, RMS norms (stored around zero) on the
-  sublayers' outputs, clamped gated units (dense or routed)."""
+  """Vilepel: latent-attention and gated-delta layers in any order, zero-centred RMS norms behind every sublayer, clamped gated units (dense or routed)."""
   layers = []
   for i, entry in enumerate(cfg["layers"]):
     src = entry.get("weights_of")

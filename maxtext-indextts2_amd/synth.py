@@ -200,7 +200,7 @@ def synth_weights_hybrid(cfg, seed: int = 0) -> Dict[str, np.ndarray]:
       z = z - np.float32(1.0)
     elif leaf == "conv":
       z = z * np.float32(1.0 / math.sqrt(shape[1]))
-    elif leaf in ("norm1", "norm2") or name == "final.norm":      # stored around zero
+    elif leaf in ("norm1", "norm2") or name == "final.norm":      # zero-centred
       z = np.float32(0.1) * z
     elif leaf == "norm":                                          # plain
       z = np.float32(1.0) + np.float32(0.1) * z

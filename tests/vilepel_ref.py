@@ -16,7 +16,7 @@ def rms(x, eps):
 
 
 def zero_centred_norm(x, w, eps):
-  """RMS norm with a weight stored around zero: rms(x) (1 + w)."""
+  """rms(x) (1 + w)."""
   return rms(x, eps) * (1.0 + w)
 
 
@@ -33,7 +33,7 @@ def softplus(z):
 
 
 def rotate_pairs(x, pos, base):
-  """x [..., T, dims] with positions pos [T]: neighbouring pairs (2i, 2i + 1) turn by p * base^(-2i/dims)."""
+  """x [..., T, dims], positions pos [T]: features 2i and 2i + 1 form a plane that turns by p base^(-2i/dims)."""
   dims = x.shape[-1]
   f = base ** (-np.arange(0, dims, 2) / dims)
   a = pos[:, None] * f[None, :]
@@ -46,7 +46,7 @@ def rotate_pairs(x, pos, base):
 
 
 def window_softmax(scores, window):
-  """scores [T, T] -> weights: row i sees j with 0 <= i - j < window."""
+  """scores [T, T] -> softmax weights of row i over columns i - window + 1 .. i."""
   T = scores.shape[0]
   i, j = np.arange(T)[:, None], np.arange(T)[None, :]
   s = np.where((i - j >= 0) & (i - j < window), scores, -np.inf)
@@ -74,7 +74,7 @@ def latent_attention(h, w, m, eps):
 
 
 def short_conv(x, taps):
-  """x [T, channels], taps [channels, n], last column the current token's: causal convolution per channel, zeros before the start."""
+  """x [T, channels], taps [channels, n] -> y_t = sum_b taps[:, n - 1 - b] x_{t - b}, with x_{<0} = 0."""
   n = taps.shape[1]
   padded = np.concatenate([np.zeros((n - 1, x.shape[1])), x])
   return sum(padded[j:j + x.shape[0]] * taps[:, j] for j in range(n))
@@ -122,7 +122,7 @@ def clamped_glu(h, wg, wu, wd, limit):
 
 
 def route(h, router, top):
-  """-> (chosen experts [T, top], their softmax scores over ALL experts, not renormalized)."""
+  """-> (experts [T, top] by descending softmax probability, those probabilities)."""
   z = linear(router, h)
   e = np.exp(z - z.max(axis=1, keepdims=True))
   s = e / e.sum(axis=1, keepdims=True)
