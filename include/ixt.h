@@ -30,10 +30,10 @@ typedef enum ixt_status {
 
 typedef enum ixt_dtype { IXT_BF16 = 0, IXT_F32 = 1 } ixt_dtype;
 
-/* One layer of an IXT_BLOCK_HYBRID decoder: a sequence mixer, then a feed-forward, each with a norm on its output only:
- *   x <- x + norm1(mixer(x)), x <- x + norm2(ff(x)), norm(t) = t / sqrt(mean(t^2) + eps) (1 + w), the residual x in f32. */
+/* One layer of an IXT_BLOCK_HYBRID decoder: a sequence mixer, then a feed-forward, each with a norm in front, behind, or both (ixt_config.norm_places):
+ *   x <- x + after(mixer(before(x))), x <- x + after(ff(before(x))), the residual x in f32. */
 typedef struct ixt_layer {
-  int32_t mixer;                   /* IXT_MIX_LATENT_ATTENTION | IXT_MIX_GATED_DELTA */
+  int32_t mixer;                   /* IXT_MIX_* */
   int32_t weights_of;              /* -1, or the layer whose parameters this one shares (it keeps a cache or state of its own) */
   int32_t heads, dim, vdim;        /* heads; query / key dims (latent attention: the unrotated ones) and value dims per head */
   /* latent attention: keys and values are up-projections of one cached latent per token plus one rotated key part shared by all heads */
@@ -41,17 +41,35 @@ typedef struct ixt_layer {
   int32_t window;                  /* position i sees i - window + 1 .. i; <= 0: everything up to i */
   float rope_base, attn_scale;     /* neighbouring pairs (2 i, 2 i + 1) turn by p base^(-2 i / rot_dim); score factor */
   /* gated delta rule with one decay per head and key channel: S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q */
-  int32_t kv_heads;                /* query / key heads (heads % kv_heads == 0) */
+  int32_t kv_heads;                /* query / key heads (heads % kv_heads == 0); IXT_MIX_ATTENTION: key / value heads */
   int32_t conv;                    /* taps of the causal convolutions in front of q, k, v */
   int32_t decay_rank, gate_rank;   /* ranks of the decay and output-gate projections */
   /* feed-forward */
   int32_t ffn;                     /* IXT_FFN_NONE | IXT_FFN_DENSE | IXT_FFN_MOE */
   int32_t ff;                      /* hidden size (MoE: of one expert) */
-  float glu_limit;                 /* y = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit) */
-  int32_t experts, top;            /* MoE: weight of a picked expert = its softmax probability among all of them */
+  float glu_limit;                 /* IXT_GLU_CLAMPED: the limit */
+  int32_t experts, top;            /* MoE */
+  /* attention over keys and values per head (heads / kv_heads query heads share one; rot_dim <= dim: the first rot_dim features of a head turn) */
+  int32_t qk_norm;                 /* != 0: every query and key head is RMS-normed with a plain weight before the rotation */
+  int32_t sink;                    /* != 0: the softmax denominator of head h also holds exp(sink_h) */
+  float rope_factor, rope_low, rope_high, rope_original;   /* rope_factor > 0: a pair of wavelength l = 2 pi / f turns at f where l < original / high, at
+                                      f / factor where l > original / low, in between at the mixture linear in original / l */
+  int32_t glu;                     /* IXT_GLU_*: the gated unit of the feed-forward (MoE: of every expert) */
+  int32_t router;                  /* IXT_ROUTE_SOFTMAX: weight of a picked expert = its softmax probability among all; IXT_ROUTE_SIGMOID: its sigmoid */
+  int32_t router_correction;       /* != 0: a per-expert number joins the scores for the choice only */
+  int32_t groups, groups_keep;     /* > 1: equal groups of neighbours, a group scores the sum of its two best choice scores, the best groups_keep are open */
+  int32_t router_norm;             /* != 0: weights divided by (their sum + 1e-20) */
+  float router_scale;              /* then multiplied by this */
+  int32_t shared_ff;               /* > 0: hidden size of a gated unit of the same form that every token runs through, added to the mixture */
 } ixt_layer;
-enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1 };
+enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1, IXT_MIX_ATTENTION = 2 };
 enum { IXT_FFN_NONE = 0, IXT_FFN_DENSE = 1, IXT_FFN_MOE = 2 };
+/* gated units of g = gate, u = up: min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u, -limit, limit) + 1); gelu(g) u (tanh form); silu(g) u */
+enum { IXT_GLU_CLAMPED = 1, IXT_GLU_GELU_TANH = 2, IXT_GLU_SILU = 3 };
+enum { IXT_ROUTE_SOFTMAX = 0, IXT_ROUTE_SIGMOID = 1 };
+/* norms around the sublayers and in front of the head: t / sqrt(mean(t^2) + eps) (1 + w); tanh(alpha t) w + b */
+enum { IXT_NORM_RMS = 0, IXT_NORM_TANH = 1 };
+enum { IXT_NORM_BEFORE = 1, IXT_NORM_AFTER = 2 };
 
 /* Derived hyper-parameters of MaxText/pyconfig.py:551-644 that shape the path. */
 typedef struct ixt_config {
@@ -122,6 +140,7 @@ typedef struct ixt_config {
   const ixt_layer* layers;
   float embedding_scale;           /* x = embedding[token] * scale */
   int32_t float32;
+  int32_t norm_kind, norm_places;  /* IXT_NORM_RMS | IXT_NORM_TANH; sum of IXT_NORM_BEFORE, IXT_NORM_AFTER */
 } ixt_config;
 
 enum { IXT_BLOCK_LLAMA2 = 0, IXT_BLOCK_GEMMA2 = 1, IXT_BLOCK_GEMMA3 = 2, IXT_BLOCK_MIXTRAL = 3, IXT_BLOCK_HYBRID = 4 };
@@ -144,7 +163,8 @@ int ixt_destroy(ixt_ctx* ctx);
  * pointer to a dense row-major array of `shape[ndim]`; IXT_F32 sources are rounded to bf16
  * (round-to-nearest-even) as linears.py:216 / embeddings.py:154 do at use.  Projection kernels are re-tiled into the
  * matrix-fragment order of the GEMM kernels while they are copied (the caller's array is not kept). */
-/* IXT_BLOCK_HYBRID: the names are `embed`, `final.norm`, `head` and `l<i>.{norm1,norm2}`, `l<i>.mix.*`, `l<i>.mlp.*`; linear weights are [out, in]. */
+/* IXT_BLOCK_HYBRID: the names are `embed`, `final.norm`, `head` and `l<i>.{norm1,norm2}` (norms on both sides: the ones behind are `norm1b`, `norm2b`; tanh
+ * norms add `.alpha` and `.b`), `l<i>.mix.*`, `l<i>.mlp.*`; linear weights are [out, in]. */
 int ixt_load_weight(ixt_ctx* ctx, const char* maxtext_path, const void* dev_ptr, int dtype, const int64_t* shape, int ndim, void* stream);
 /* 1 when every parameter of the configured model has been loaded. */
 int ixt_weights_complete(ixt_ctx* ctx);

@@ -24,7 +24,10 @@ class IxtLayer(ctypes.Structure):
   _fields_ = [(n, ctypes.c_int32) for n in ("mixer", "weights_of", "heads", "dim", "vdim", "rot_dim", "kv_rank", "window")] + [
       ("rope_base", ctypes.c_float), ("attn_scale", ctypes.c_float)] + [
       (n, ctypes.c_int32) for n in ("kv_heads", "conv", "decay_rank", "gate_rank", "ffn", "ff")] + [
-      ("glu_limit", ctypes.c_float), ("experts", ctypes.c_int32), ("top", ctypes.c_int32)]
+      ("glu_limit", ctypes.c_float), ("experts", ctypes.c_int32), ("top", ctypes.c_int32), ("qk_norm", ctypes.c_int32), ("sink", ctypes.c_int32)] + [
+      (n, ctypes.c_float) for n in ("rope_factor", "rope_low", "rope_high", "rope_original")] + [
+      (n, ctypes.c_int32) for n in ("glu", "router", "router_correction", "groups", "groups_keep", "router_norm")] + [
+      ("router_scale", ctypes.c_float), ("shared_ff", ctypes.c_int32)]
 
 
 class IxtConfig(ctypes.Structure):
@@ -45,6 +48,7 @@ class IxtConfig(ctypes.Structure):
       ("ep_rank", ctypes.c_int32), ("ep_size", ctypes.c_int32), ("fp8_weights", ctypes.c_int32),
       ("rope_llama31", ctypes.c_int32), ("rope_use_scale", ctypes.c_int32),
       ("layers", ctypes.POINTER(IxtLayer)), ("embedding_scale", ctypes.c_float), ("float32", ctypes.c_int32),
+      ("norm_kind", ctypes.c_int32), ("norm_places", ctypes.c_int32),
   ]
 
 BLOCK_LLAMA2, BLOCK_GEMMA2, BLOCK_GEMMA3, BLOCK_MIXTRAL, BLOCK_HYBRID = 0, 1, 2, 3, 4

@@ -11,8 +11,12 @@ import os
 import struct
 from typing import Any, Callable, Dict, Mapping, Tuple
 
-MIX_LATENT_ATTENTION, MIX_GATED_DELTA = 0, 1
+MIX_LATENT_ATTENTION, MIX_GATED_DELTA, MIX_ATTENTION = 0, 1, 2
 FFN_NONE, FFN_DENSE, FFN_MOE = 0, 1, 2
+GLU_CLAMPED, GLU_GELU_TANH, GLU_SILU = 1, 2, 3
+ROUTE_SOFTMAX, ROUTE_SIGMOID = 0, 1
+NORM_RMS, NORM_TANH = 0, 1
+NORM_BEFORE, NORM_AFTER = 1, 2
 
 
 @dataclasses.dataclass(frozen=True)
@@ -37,6 +41,20 @@ class HybridLayer:
   glu_limit: float = 0.0
   experts: int = 0
   top: int = 0
+  qk_norm: int = 0
+  sink: int = 0
+  rope_factor: float = 0.0
+  rope_low: float = 1.0
+  rope_high: float = 1.0
+  rope_original: float = 1.0
+  glu: int = GLU_CLAMPED
+  router: int = ROUTE_SOFTMAX
+  router_correction: int = 0
+  groups: int = 1
+  groups_keep: int = 1
+  router_norm: int = 0
+  router_scale: float = 1.0
+  shared_ff: int = 0
 
 
 Shapes = Mapping[str, Tuple[int, ...]]
@@ -102,7 +120,55 @@ def vilepel_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
   }
 
 
+def _vazilorn_mixer(m: Mapping[str, Any]) -> Dict[str, Any]:
+  rot = m["rot"]
+  heads, kv_heads, dim, dims = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(rot["dims"])
+  if heads % kv_heads or dims % 2 or dims > dim:
+    raise ValueError(f"Vazilorn: {heads} heads over {kv_heads} key heads, {dims} of {dim} dims rotated")
+  out = {"mixer": MIX_ATTENTION, "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": int(m["vdim"]), "rot_dim": dims, "rope_base": float(rot["base"]),
+         "window": int((m.get("mask") or {}).get("size") or 0), "attn_scale": float(m["scale"]), "qk_norm": 1, "sink": 1}
+  scaling = rot.get("scaling")
+  if scaling:
+    out.update(rope_factor=float(scaling["factor"]), rope_low=float(scaling["low"]), rope_high=float(scaling["high"]), rope_original=float(scaling["original"]))
+  return out
+
+
+def _vazilorn_feed_forward(mlp: Any) -> Dict[str, Any]:
+  if mlp is None:
+    return {"ffn": FFN_NONE}
+  if mlp["kind"] == "dense":
+    return {"ffn": FFN_DENSE, "ff": int(mlp["ff"]), "glu": GLU_GELU_TANH}
+  if mlp["kind"] == "moe":
+    r, groups, shared = mlp["router"], mlp["router"].get("groups") or {}, mlp.get("shared") or {}
+    return {"ffn": FFN_MOE, "ff": int(mlp["expert"]["ff"]), "glu": GLU_SILU, "experts": int(r["experts"]), "top": int(r["top"]), "router": ROUTE_SIGMOID,
+            "router_correction": 1, "groups": int(groups.get("count") or 1), "groups_keep": int(groups.get("keep") or 1), "router_norm": 1,
+            "router_scale": float(r["scale"]), "shared_ff": int(shared.get("ff") or 0)}
+  raise ValueError(f"Vazilorn: feed-forward kind {mlp['kind']!r}")
+
+
+def vazilorn_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
+  """Vazilorn: windowed attention with sinks, normed queries and keys and scaled rotations; tanh norms on both sides of every sublayer; gelu units or a
+  routed mixture of silu units (sigmoid scores, groups, a shared unit)."""
+  del shapes
+  layers = []
+  for i, entry in enumerate(cfg["layers"]):
+    if entry["type"] != "attention":
+      raise ValueError(f"Vazilorn: layer {i} has type {entry['type']!r}")
+    layers.append(HybridLayer(**_vazilorn_mixer(entry["mixer"]), **_vazilorn_feed_forward(entry.get("mlp"))))
+  return {
+      "decoder_block": "hybrid",
+      "vocab_size": int(cfg["vocab"]),
+      "base_emb_dim": int(cfg["width"]),
+      "base_num_decoder_layers": len(layers),
+      "normalization_layer_epsilon": float(cfg["norm"]["eps"]),
+      "hybrid_norm_kind": NORM_TANH,
+      "hybrid_norm_places": NORM_BEFORE | NORM_AFTER,
+      "hybrid_layers": tuple(layers),
+  }
+
+
 ARCHITECTURES: Dict[str, Callable[[Mapping[str, Any], Shapes], Dict[str, Any]]] = {
+    "Vazilorn": vazilorn_keys,
     "Vilepel": vilepel_keys,
 }
 
@@ -125,15 +191,33 @@ def read_model_dir(path: str) -> Dict[str, Any]:
 def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
   """{tensor name: shape} of a hybrid decoder; linear weights are [out, in]."""
   E, V = int(config.emb_dim), int(config.vocab_size)
-  out: Dict[str, Tuple[int, ...]] = {"embed": (V, E), "final.norm": (E,), "head": (V, E)}
+  out: Dict[str, Tuple[int, ...]] = {"embed": (V, E), "head": (V, E)}
+
+  def norm(name: str) -> None:
+    out[name] = (E,)
+    if config.hybrid_norm_kind == NORM_TANH:
+      out[name + ".alpha"], out[name + ".b"] = (), (E,)
+
+  def gated(name: str, ff: int) -> None:
+    out[name + "gate"], out[name + "up"], out[name + "down"] = (ff, E), (ff, E), (E, ff)
+
+  both = config.hybrid_norm_places == NORM_BEFORE | NORM_AFTER
+  norm("final.norm")
   for i, l in enumerate(config.hybrid_layers):
     if l.weights_of >= 0:
       continue
     p = f"l{i}."
-    out[p + "norm1"] = (E,)
+    for n in ("norm1", "norm1b")[:1 + both] + (() if l.ffn == FFN_NONE else ("norm2", "norm2b")[:1 + both]):
+      norm(p + n)
     if l.mixer == MIX_LATENT_ATTENTION:
       out.update({p + "mix.q": (l.heads * (l.dim + l.rot_dim), E), p + "mix.dkv": (l.kv_rank + l.rot_dim, E), p + "mix.dkv.norm": (l.kv_rank,),
                   p + "mix.uk": (l.heads * l.dim, l.kv_rank), p + "mix.uv": (l.heads * l.vdim, l.kv_rank), p + "mix.o": (E, l.heads * l.vdim)})
+    elif l.mixer == MIX_ATTENTION:
+      out.update({p + "mix.q": (l.heads * l.dim, E), p + "mix.k": (l.kv_heads * l.dim, E), p + "mix.v": (l.kv_heads * l.vdim, E), p + "mix.o": (E, l.heads * l.vdim)})
+      if l.qk_norm:
+        out[p + "mix.q.norm"] = out[p + "mix.k.norm"] = (l.dim,)
+      if l.sink:
+        out[p + "mix.sink"] = (l.heads,)
     else:
       kq, v = l.kv_heads * l.dim, l.heads * l.vdim
       for t, n in (("q", kq), ("k", kq), ("v", v)):
@@ -141,11 +225,14 @@ def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
       out.update({p + "mix.b": (l.heads, E), p + "mix.A_log": (l.heads,), p + "mix.norm": (l.vdim,), p + "mix.a1": (l.decay_rank, E),
                   p + "mix.a2": (l.heads * l.dim, l.decay_rank), p + "mix.dt_bias": (l.heads * l.dim,), p + "mix.g1": (l.gate_rank, E),
                   p + "mix.g2": (v, l.gate_rank), p + "mix.o": (E, v)})
-    if l.ffn == FFN_NONE:
-      continue
-    out[p + "norm2"] = (E,)
-    for q in ([f"mlp.e{e}." for e in range(l.experts)] if l.ffn == FFN_MOE else ["mlp."]):
-      out[p + q + "gate"], out[p + q + "up"], out[p + q + "down"] = (l.ff, E), (l.ff, E), (E, l.ff)
-    if l.ffn == FFN_MOE:
+    if l.ffn == FFN_DENSE:
+      gated(p + "mlp.", l.ff)
+    elif l.ffn == FFN_MOE:
+      for e in range(l.experts):
+        gated(p + f"mlp.e{e}.", l.ff)
       out[p + "mlp.router"] = (l.experts, E)
+      if l.router_correction:
+        out[p + "mlp.correction"] = (l.experts,)
+      if l.shared_ff > 0:
+        gated(p + "mlp.shared.", l.shared_ff)
   return out

@@ -1462,7 +1462,7 @@ static int moe_experts_routed(ixt_ctx* c, const LayerW& w, const bf16_t* x, cons
   const int rows_g = (npairs + align - 1) / align * align + align * c->NEL;
   if (rows_g > c->moe_rows_cap) return set_err(IXT_ERR_INVALID, "moe: %d copies exceed the routed workspaces (%d rows)", npairs, c->moe_rows_cap);
   hipLaunchKernelGGL(k_moe_plan, dim3(1), dim3(1024), 0, st, idx, npairs, c->E0, c->NEL, align, rows_g / 16, c->moe_pos, c->moe_rbexp, c->moe_cnt);
-  hipLaunchKernelGGL(k_moe_gather, dim3((E + 2047) / 2048, npairs), dim3(256), 0, st, x, c->moe_pos, top_k, E, c->moe_xg);
+  hipLaunchKernelGGL(k_moe_gather, dim3(npairs, (E + 2047) / 2048), dim3(256), 0, st, x, c->moe_pos, top_k, E, c->moe_xg);
   LAUNCHCHK();
   const size_t wi_stride = c->moe_wi_stride / 8, wo_stride = c->moe_wo_stride / 8;   // 16-byte units
   if (c->fp8) {   // IXT-FP8-v1: the experts' e4m3 twins (contiguous per layer), activations quantised per copy row and 512-k block

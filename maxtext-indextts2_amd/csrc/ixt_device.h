@@ -108,10 +108,16 @@ __device__ __forceinline__ bf16_t ixt_geglu(float a, float b) {
   return f2bf(g * b);
 }
 
-// clamped gated unit: g = min(a, limit), u = clamp(b, -limit, limit), g sigmoid(1.702 g) (u + 1), in f32
+// gated units in f32, by kind (IXT_GLU_*).  1: g = min(a, limit), u = clamp(b, -limit, limit), g sigmoid(1.702 g) (u + 1); 2: tanh form of gelu, as
+// a sigmoid(2 sqrt(2 / pi) (a + 0.044715 a^3)) b; 3: a sigmoid(a) b
 __device__ __forceinline__ float ixt_glu_clamped(float a, float b, float limit) {
   const float g = fminf(a, limit), u = fminf(fmaxf(b, -limit), limit);
   return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
+__device__ __forceinline__ float ixt_glu(int kind, float a, float b, float limit) {
+  if (kind == 1) return ixt_glu_clamped(a, b, limit);
+  const float z = kind == 2 ? 1.59576912160573071176f * fmaf(0.044715f * a * a, a, a) : a;
+  return a / (1.0f + expf(-z)) * b;
 }
 
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));

@@ -40,7 +40,7 @@ struct GemmEpi {
   AttnGeom g;
   const float* xscale; const float* wscale;             // F8: activation scales [rows][chains], column scales [N] (ixt_fp8.h)
   size_t sstride;                                       // F8 + routed experts: floats between two experts' column scales
-  int glu; float glu_limit;                             // SWIGLU: glu != 0 takes the clamped gated unit of the f32 totals instead (ixt_glu_clamped)
+  int glu; float glu_limit;                             // SWIGLU: glu != 0 takes that gated unit of the f32 totals instead (ixt_glu)
   const int32_t* rb_exp; size_t wstride;                // routed experts: expert of every 16-row block (-1: none), 16-byte units between experts' kernels
 };
 
@@ -282,7 +282,7 @@ __global__ __launch_bounds__(WR * WC * 64, 2) void k_gemm_ring(const u32x4* __re
           bf16_t o[4];
 #pragma unroll
           for (int j = 0; j < 4; ++j)
-            o[j] = e.glu ? f2bf(ixt_glu_clamped(tot[i][b][j], tot[i + 1][b][j], e.glu_limit)) : ixt_swiglu(rbf(tot[i][b][j]), rbf(tot[i + 1][b][j]));
+            o[j] = e.glu ? f2bf(ixt_glu(e.glu, tot[i][b][j], tot[i + 1][b][j], e.glu_limit)) : ixt_swiglu(rbf(tot[i][b][j]), rbf(tot[i + 1][b][j]));
           uint2 ov;
           ov.x = pack2(o[0], o[1]); ov.y = pack2(o[2], o[3]);
           *reinterpret_cast<uint2*>(e.act + xidx(row, f0, F)) = ov;

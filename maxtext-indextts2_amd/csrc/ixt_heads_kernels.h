@@ -1,0 +1,455 @@
+// ixt_heads_kernels.h -- attention of hybrid decoders over keys and values per head (IXT_MIX_ATTENTION): query heads in equal groups on one key / value
+// head each, optional norm of query and key heads, rotation of a head's first features, optional window, optional sink (a number per head that joins the
+// softmax denominator without a key or a value).  Sizes of keys and values are independent.
+//
+//   k_heads_prep     projection slices -> queries [R][H][dkp], the row's keys and values in their pages
+//   k_heads_prompt   many rows, bf16, matrix cores
+//   k_heads_decode   few rows, bf16, matrix cores, keys split over blocks (+ k_heads_combine)
+//   k_heads_any      any sizes, any T
+//
+// Pages: [page][kv head][token][dkp] and [page][kv head][token][dvp]; what lies behind the real features is zero from the pool's creation on.
+#pragma once
+#include "ixt_hybrid_kernels.h"
+
+struct HeadsGeom {
+  int H, G, d, dv, rot, P, mpg, window;     // query heads, key / value heads, key and value dims, rotated dims, page size, pages per group, window (<= 0: none)
+  int dkp, dvp;                             // padded key / value rows
+  int hs, vs, ok, ov;                       // projection columns: a query / key head takes hs, a value head vs; keys from ok on, values from ov on
+  float scale;
+};
+struct RowsArgs { const int32_t *slot, *pos, *active, *page_map; };      // the rows of a pass
+
+// A wave per head: queries and keys are normed (qn / kn; null: not) and rotated in f32, values copied.  rope: f32 [position][rot / 2] cos, sin.
+// grid (R, ceil((H + 2 G) / 4)), block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_heads_prep(Slices t, HeadsGeom g, const float* __restrict__ qn, const float* __restrict__ kn, float eps, const float* __restrict__ rope_cos,
+                                                    const float* __restrict__ rope_sin, RowsArgs rows, T* __restrict__ kpages, T* __restrict__ vpages, T* __restrict__ q) {
+  const int r = blockIdx.x, j = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (j >= g.H + 2 * g.G) return;
+  const bool act = rows.active[r] != 0;
+  if (!act && j >= g.H) return;
+  const int pos = act ? rows.pos[r] : 0;
+  const int page = act ? rows.page_map[(size_t)rows.slot[r] * g.mpg + pos / g.P] : 0;
+  const bool is_q = j < g.H;
+  const int kh = is_q ? 0 : (j - g.H) % g.G;
+  const size_t at = ((size_t)page * g.G + kh) * g.P + pos % g.P;          // row of the key / value pools
+  if (j >= g.H + g.G) {
+    T* v = vpages + at * g.dvp;
+    for (int c = lane; c < g.dv; c += 64) v[c] = from_f<T>(t.at(r, g.ov + kh * g.vs + c));
+    return;
+  }
+  const int c0 = is_q ? j * g.hs : g.ok + kh * g.hs;
+  const float* w = is_q ? qn : kn;
+  float rs = 1.0f;
+  if (w != nullptr) {
+    float ss = 0.0f;
+    for (int c = lane; c < g.d; c += 64) { const float v = t.at(r, c0 + c); ss = fmaf(v, v, ss); }
+    rs = 1.0f / sqrtf(wave_sum(ss) / (float)g.d + eps);
+  }
+  T* o = is_q ? q + ((size_t)r * g.H + j) * g.dkp : kpages + at * g.dkp;
+  const int half = g.rot >> 1;
+  for (int i = lane; i < g.dkp / 2; i += 64) {
+    float u = 2 * i < g.d ? t.at(r, c0 + 2 * i) * rs : 0.0f, v = 2 * i + 1 < g.d ? t.at(r, c0 + 2 * i + 1) * rs : 0.0f;
+    if (w != nullptr) { u *= 2 * i < g.d ? w[2 * i] : 0.0f; v *= 2 * i + 1 < g.d ? w[2 * i + 1] : 0.0f; }
+    if (i < half) {
+      const float c = rope_cos[(size_t)pos * half + i], s = rope_sin[(size_t)pos * half + i], a = u;
+      u = a * c - v * s; v = v * c + a * s;
+    }
+    if constexpr (sizeof(T) == 2) *reinterpret_cast<uint32_t*>(o + 2 * i) = pack2(f2bf(u), f2bf(v));
+    else *reinterpret_cast<float2*>(o + 2 * i) = make_float2(u, v);
+  }
+}
+
+// Any sizes (dv <= 1024), any T: block = (row, head); thread = key for the scores (tiles of 256 keys, running maximum and sum, the sink as their start),
+// thread = value column for the weighted sum.  out: act(T), column h vs + c.  grid (R, H), block 256, LDS = (dkp + 256) floats.
+template <typename T>
+__global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, HeadsGeom g, const float* __restrict__ sink, RowsArgs rows, const T* __restrict__ kpages,
+                                                   const T* __restrict__ vpages, T* __restrict__ out, int Kp) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  __shared__ float red[4];
+  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, kh = h / (g.H / g.G);
+  if (!rows.active[r]) return;
+  float* q = sm;
+  float* p = sm + g.dkp;
+  for (int k = tid; k < g.dkp; k += 256) q[k] = to_f(qb[((size_t)r * g.H + h) * g.dkp + k]);
+  __syncthreads();
+  const int pos = rows.pos[r], k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
+  const int32_t* prow = rows.page_map + (size_t)rows.slot[r] * g.mpg;
+  float m = sink != nullptr ? sink[h] : -INFINITY, l = sink != nullptr ? 1.0f : 0.0f, acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int j0 = k_lo; j0 <= pos; j0 += 256) {
+    const int j = j0 + tid;
+    float s = -INFINITY;
+    if (j <= pos) {
+      const T* kp = kpages + (((size_t)prow[j / g.P] * g.G + kh) * g.P + j % g.P) * g.dkp;
+      float a = 0.0f;
+      for (int k = 0; k < g.d; ++k) a = fmaf(q[k], to_f(kp[k]), a);
+      s = a * g.scale;
+    }
+    float tm = s;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) tm = fmaxf(tm, __shfl_xor(tm, off, 64));
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = tm;
+    __syncthreads();
+    const float mn = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), m);
+    const float e = j <= pos ? expf(s - mn) : 0.0f;
+    p[tid] = e;
+    const float al = expf(m - mn);
+    const float ls = block_sum256(e, red);                  // (its barriers also publish p)
+    l = l * al + ls;
+    m = mn;
+    const int nk = min(256, pos - j0 + 1);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] *= al;
+    for (int kk = 0; kk < nk; ++kk) {
+      const T* vp = vpages + (((size_t)prow[(j0 + kk) / g.P] * g.G + kh) * g.P + (j0 + kk) % g.P) * g.dvp;
+      const float w = p[kk];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (tid + 256 * i < g.dv) acc[i] = fmaf(w, to_f(vp[tid + 256 * i]), acc[i]);
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (tid + 256 * i < g.vs) act_store1(out, r, h * g.vs + tid + 256 * i, Kp, tid + 256 * i < g.dv ? acc[i] / l : 0.0f);
+  if (h == g.H - 1)
+    for (int k = g.H * g.vs + tid; k < Kp; k += 256) act_store1(out, r, k, Kp, 0.0f);
+}
+
+// ---------------------------------------------------------------------------------------------------- matrix-core forms
+// The M side of the products is (row, query head) pairs of one key / value head.  Per tile of 64 keys:
+//   scores   D[key][pair] = mfma(A = keys, B = queries): a lane holds 4 keys of one pair per product
+//   weights  running maximum / sum per pair in f32 (they start at the sink), exp2; P goes to bf16
+//   output   D[column][pair] = mfma(A = values read column-wise, B = P)
+struct HeadsAttnArgs {
+  const bf16_t* q; HeadsGeom g; const float* sink;
+  RowsArgs rows;
+  const bf16_t *kpages, *vpages;
+  int R, NQ, HB, hchunks, pshift;           // rows per block, query heads per block, blocks of query heads per key / value head
+  bf16_t* out; int Kp;                      // act, column h vs + c
+  float *part_o, *part_ml;                  // splits > 1: [R H][splits][dvp], [R H][splits][2]
+};
+__device__ __forceinline__ float heads_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+// the pool row of a key: page (G heads) -> head -> token
+__device__ __forceinline__ int heads_row(const int32_t* __restrict__ prow, int key, int pshift, int G, int kh) {
+  return ((prow[key >> pshift] * G + kh) << pshift) + (key & ((1 << pshift) - 1));
+}
+
+// Prompts: a block owns 64 MP pairs = up to 64 MP / HB consecutive rows x HB query heads of one key / value head (a wave 16 MP of them); all waves walk
+// the same key tiles, the next tile arriving while the current one is used.  P stays in registers: with the key order 4q .. 4q + 3, 16 + 4q ..
+// 16 + 4q + 3 per lane group q of 32 keys, the lane's own scores ARE its operand of the next product.  Consecutive blocks are different heads: with
+// 8 heads or a multiple of them, a head's keys and values stay in one XCD's L2.  grid (G hchunks, ceil(R / NQ)), block 256, LDS two tiles.
+template <int DK, int DV, int MP>
+__global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(HeadsAttnArgs a) {
+  constexpr int NKS = DK / 32, NT = DV / 16, NGV = DV / 64, TILE = 64 * (DK + DV);
+  extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
+  const HeadsGeom& g = a.g;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
+  const int kh = blockIdx.x % g.G, hc = blockIdx.x / g.G, GQ = g.H / g.G;
+  const int r0 = blockIdx.y * a.NQ, nr = min(a.NQ, a.R - r0), h0 = kh * GQ + hc * a.HB, hb = min(a.HB, GQ - hc * a.HB);
+  int qi[MP], head[MP], row[MP], pos[MP];
+  bool live[MP];
+  bf16x8 qf[MP][NKS];                                     // queries: lane = pair r_in, 8 consecutive features per step
+  float m[MP], l[MP];
+  f32x4 o[MP][NT];
+#pragma unroll
+  for (int p = 0; p < MP; ++p) {
+    const int pair = (wave * MP + p) * 16 + r_in, hh = pair % a.HB;
+    qi[p] = pair / a.HB;
+    const bool ok = qi[p] < nr && hh < hb;
+    row[p] = r0 + (ok ? qi[p] : 0); head[p] = h0 + (ok ? hh : 0);
+    live[p] = ok && a.rows.active[row[p]] != 0;
+    pos[p] = live[p] ? a.rows.pos[row[p]] : -1;
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks)
+      qf[p][ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.q + ((size_t)row[p] * g.H + head[p]) * DK + ks * 32 + cq * 8));
+    m[p] = a.sink != nullptr ? a.sink[head[p]] * 1.44269504088896340736f : -INFINITY;
+    l[p] = a.sink != nullptr ? 1.0f : 0.0f;
+#pragma unroll
+    for (int i = 0; i < NT; ++i) o[p][i] = f32x4(0.0f);
+  }
+  const float sc = g.scale * 1.44269504088896340736f;
+  const TileLane L = tile_lane(r_in, cq);
+  for (int ra = 0; ra < nr;) {                            // runs of rows that share a page group
+    if (!a.rows.active[r0 + ra]) { ++ra; continue; }
+    const int slot = a.rows.slot[r0 + ra];
+    int lo = a.rows.pos[r0 + ra], hi = lo, rb = ra + 1;
+    while (rb < nr && a.rows.active[r0 + rb] && a.rows.slot[r0 + rb] == slot) { const int p = a.rows.pos[r0 + rb]; lo = min(lo, p); hi = max(hi, p); ++rb; }
+    const bool whole = ra == 0 && rb == nr;               // no other run in this block: only the keys decide what is masked
+    bool mine[MP];
+    int my_lo[MP];
+#pragma unroll
+    for (int p = 0; p < MP; ++p) {
+      mine[p] = live[p] && qi[p] >= ra && qi[p] < rb;
+      my_lo[p] = g.window > 0 ? max(0, pos[p] - g.window + 1) : 0;
+    }
+    ra = rb;
+    const int k_lo = g.window > 0 ? max(0, lo - g.window + 1) : 0, k_all = g.window > 0 ? max(0, hi - g.window + 1) : 0;    // (k_all .. lo: seen by every row)
+    const int ntile = (hi - k_lo) / 64 + 1;
+    const int32_t* prow = a.rows.page_map + (size_t)slot * g.mpg;
+    __syncthreads();                                      // the previous run's last tile has been read
+    int off = heads_row(prow, min(k_lo + lane, hi), a.pshift, g.G, kh);
+    tile_dma<DK>(a.kpages, off, lds, wave, lane);
+    tile_dma<DV>(a.vpages, off, lds + 64 * DK, wave, lane);
+    off = heads_row(prow, min(k_lo + 64 + lane, hi), a.pshift, g.G, kh);
+    for (int t = 0; t < ntile; ++t) {
+      const bf16_t* tile = lds + (size_t)(t & 1) * TILE;
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      __syncthreads();                                    // the tile is there; every wave is done with the other one
+      if (t + 1 < ntile) {
+        bf16_t* next = lds + (size_t)((t + 1) & 1) * TILE;
+        tile_dma<DK>(a.kpages, off, next, wave, lane);
+        tile_dma<DV>(a.vpages, off, next + 64 * DK, wave, lane);
+        off = heads_row(prow, min(k_lo + (t + 2) * 64 + lane, hi), a.pshift, g.G, kh);
+      }
+      f32x4 s[MP][4];
+#pragma unroll
+      for (int p = 0; p < MP; ++p)
+#pragma unroll
+        for (int n = 0; n < 4; ++n) s[p][n] = f32x4(0.0f);
+      bf16x8 kf[2][4];                                    // operands one step ahead of the products
+#pragma unroll
+      for (int n = 0; n < 4; ++n) kf[0][n] = tile_kf<DK>(reinterpret_cast<const char*>(tile), L, 0, n);
+#pragma unroll
+      for (int ks = 0; ks < NKS; ++ks) {
+        if (ks + 1 < NKS) {
+#pragma unroll
+          for (int n = 0; n < 4; ++n) kf[(ks + 1) & 1][n] = tile_kf<DK>(reinterpret_cast<const char*>(tile), L, ks + 1, n);
+        }
+#pragma unroll
+        for (int n = 0; n < 4; ++n)
+#pragma unroll
+          for (int p = 0; p < MP; ++p) s[p][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][n], qf[p][ks], s[p][n], 0, 0, 0);
+        __builtin_amdgcn_sched_barrier(0);
+      }
+      const int t0 = k_lo + t * 64;
+      const bool inside = whole && t0 >= k_all && t0 + 63 <= lo;
+      bf16x8 pf[MP][2];
+#pragma unroll
+      for (int p = 0; p < MP; ++p) {
+        float tm = -INFINITY;
+        if (inside) {
+#pragma unroll
+          for (int n = 0; n < 4; ++n)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) tm = fmaxf(tm, s[p][n][j]);
+        } else {
+#pragma unroll
+          for (int n = 0; n < 4; ++n)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+              const int key = t0 + n * 16 + cq * 4 + j;
+              const bool seen = mine[p] && key <= pos[p] && key >= my_lo[p];
+              s[p][n][j] = seen ? s[p][n][j] : -INFINITY;
+              tm = fmaxf(tm, s[p][n][j]);
+            }
+        }
+        tm *= sc;                                         // (a positive factor keeps the order)
+        tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+        tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+        const float mn = fmaxf(m[p], tm), mz = mn == -INFINITY ? 0.0f : mn;
+        const float al = heads_exp2(m[p] - mz);           // (nothing seen so far: exp2(-inf) = 0, and l and o are 0)
+        float ls = 0.0f;
+#pragma unroll
+        for (int n = 0; n < 4; ++n)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) { s[p][n][j] = heads_exp2(fmaf(s[p][n][j], sc, -mz)); ls += s[p][n][j]; }
+        ls += __shfl_xor(ls, 16, 64);
+        ls += __shfl_xor(ls, 32, 64);
+        l[p] = l[p] * al + ls;
+        m[p] = mn;
+        if (__any(al != 1.0f)) {
+#pragma unroll
+          for (int i = 0; i < NT; ++i) { o[p][i][0] *= al; o[p][i][1] *= al; o[p][i][2] *= al; o[p][i][3] *= al; }
+        }
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {                     // 32 keys each
+          u32x4 pk;
+          pk.x = pack2(f2bf(s[p][2 * u][0]), f2bf(s[p][2 * u][1])); pk.y = pack2(f2bf(s[p][2 * u][2]), f2bf(s[p][2 * u][3]));
+          pk.z = pack2(f2bf(s[p][2 * u + 1][0]), f2bf(s[p][2 * u + 1][1])); pk.w = pack2(f2bf(s[p][2 * u + 1][2]), f2bf(s[p][2 * u + 1][3]));
+          pf[p][u] = __builtin_bit_cast(bf16x8, pk);
+        }
+      }
+      const uint32_t tb = lds_addr(tile) + 64 * DK * 2;
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        [[maybe_unused]] uint2 f[2][4][2];
+        if constexpr (NGV > 0) IXT_TILE_VT(f[0], tb, L, 0, u);
+#pragma unroll
+        for (int gr = 0; gr < NGV; ++gr) {                // the next group's reads travel under this one's products
+          if (gr + 1 < NGV) {
+            IXT_TILE_VT(f[(gr + 1) & 1], tb, L, gr + 1, u);
+            IXT_TILE_VWAIT(f[gr & 1], 8);
+          } else {
+            IXT_TILE_VWAIT(f[gr & 1], 0);
+          }
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int p = 0; p < MP; ++p) o[p][gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(f[gr & 1][i]), pf[p][u], o[p][gr * 4 + i], 0, 0, 0);
+        }
+        if constexpr (DV % 64 != 0) {
+          uint2 fh[2][2];
+          IXT_TILE_VTH(fh, tb, L, NGV, u);
+          IXT_TILE_VWAITN(fh, 2, 0);
+#pragma unroll
+          for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int p = 0; p < MP; ++p) o[p][NGV * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(fh[i]), pf[p][u], o[p][NGV * 4 + i], 0, 0, 0);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int p = 0; p < MP; ++p) {
+    if (!live[p]) continue;
+    const float inv = 1.0f / l[p];
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const float v[4] = {o[p][i][0] * inv, o[p][i][1] * inv, o[p][i][2] * inv, o[p][i][3] * inv};
+      if (i * 16 + cq * 4 < g.vs) act_store4(a.out, row[p], head[p] * g.vs + i * 16 + cq * 4, a.Kp, v);      // (columns dv .. vs - 1 are zero: so are the values there)
+    }
+    const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    if (head[p] == g.H - 1)
+      for (int c = g.H * g.vs + cq * 4; c < a.Kp; c += 16) act_store4(a.out, row[p], c, a.Kp, z);
+  }
+}
+
+// Few rows (decode): a block owns up to 16 query heads of one key / value head of ONE row and every gridDim.z-th key tile of its window.  Scores: a wave
+// takes 16 of the 64 keys; P and the tile maxima meet in LDS; output: a wave takes every fourth column tile.  One tile of LDS: several blocks share a
+// CU and one's loads run under the other's products.  grid (R, G hchunks, splits), block 256.
+template <int DK, int DV>
+__global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
+  constexpr int NKS = DK / 32, NGV = DV / 64, NH = DV % 64 != 0 ? 1 : 0, OT = NGV + NH;     // column tiles per wave: one of every full group, waves 0 and 1 one of the half group
+  extern __shared__ __attribute__((aligned(16))) bf16_t tile[];
+  __shared__ __attribute__((aligned(16))) bf16_t ps[16][72];
+  __shared__ float s_m[4][16], s_l[4][16];
+  const HeadsGeom& g = a.g;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
+  const int row = blockIdx.x, kh = blockIdx.y % g.G, hc = blockIdx.y / g.G, GQ = g.H / g.G, nsplit = gridDim.z;
+  const int h0 = kh * GQ + hc * a.HB, hb = min(a.HB, GQ - hc * a.HB);
+  const int active = a.rows.active[row], pos = a.rows.pos[row], slot = a.rows.slot[row];     // (requested together)
+  if (!active) return;
+  const bool pair_ok = r_in < hb;
+  const int head = h0 + (pair_ok ? r_in : 0);
+  const int32_t* prow = a.rows.page_map + (size_t)slot * g.mpg;
+  const int k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0, ntile = (pos - k_lo) / 64 + 1;
+  int t = blockIdx.z;
+  if (t < ntile) {
+    const int off = heads_row(prow, min(k_lo + t * 64 + lane, pos), a.pshift, g.G, kh);
+    tile_dma<DK>(a.kpages, off, tile, wave, lane);
+    tile_dma<DV>(a.vpages, off, tile + 64 * DK, wave, lane);
+  }
+  bf16x8 qf[NKS];
+#pragma unroll
+  for (int ks = 0; ks < NKS; ++ks) qf[ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.q + ((size_t)row * g.H + head) * DK + ks * 32 + cq * 8));
+  f32x4 o[OT];
+#pragma unroll
+  for (int i = 0; i < OT; ++i) o[i] = f32x4(0.0f);
+  const bool sink = a.sink != nullptr && blockIdx.z == 0;          // counted once
+  float m = sink ? a.sink[head] * 1.44269504088896340736f : -INFINITY, l = sink && wave == 0 && cq == 0 ? 1.0f : 0.0f;      // l: this lane's keys only
+  const float sc = g.scale * 1.44269504088896340736f;
+  const TileLane L = tile_lane(r_in, cq);
+  const uint32_t vl = wave == 0 ? L.v[0] : (wave == 1 ? L.v[1] : (wave == 2 ? L.v[2] : L.v[3]));
+  [[maybe_unused]] const uint32_t vh = (wave & 1) ? L.vh[1] : L.vh[0];
+  const uint32_t tb = lds_addr(tile) + 64 * DK * 2;
+  for (; t < ntile; t += nsplit) {
+    int off = 0;
+    if (t + nsplit < ntile) off = heads_row(prow, min(k_lo + (t + nsplit) * 64 + lane, pos), a.pshift, g.G, kh);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    f32x4 s = f32x4(0.0f);
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks)
+      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_kf<DK>(reinterpret_cast<const char*>(tile) + wave * (DK % 64 != 0 && ks == DK / 64 * 2 ? 1024 : 2048), L, ks, 0), qf[ks], s, 0, 0, 0);
+    float tm = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      s[j] = k_lo + t * 64 + wave * 16 + cq * 4 + j <= pos ? s[j] * sc : -INFINITY;
+      tm = fmaxf(tm, s[j]);
+    }
+    tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+    tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+    if (cq == 0) s_m[wave][r_in] = tm;
+    __syncthreads();
+    const float mn = fmaxf(m, fmaxf(fmaxf(s_m[0][r_in], s_m[1][r_in]), fmaxf(s_m[2][r_in], s_m[3][r_in])));   // (a tile has at least one visible key: finite)
+    const float al = heads_exp2(m - mn);
+    float p[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) p[j] = heads_exp2(s[j] - mn);
+    l = l * al + ((p[0] + p[1]) + (p[2] + p[3]));
+    m = mn;
+    uint2 pk;
+    pk.x = pack2(f2bf(p[0]), f2bf(p[1])); pk.y = pack2(f2bf(p[2]), f2bf(p[3]));
+    *reinterpret_cast<uint2*>(&ps[r_in][wave * 16 + cq * 4]) = pk;
+    if (__any(al != 1.0f)) {
+#pragma unroll
+      for (int i = 0; i < OT; ++i) { o[i][0] *= al; o[i][1] *= al; o[i][2] *= al; o[i][3] *= al; }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {                         // lane group q holds keys 32 u + 4 q .. + 3 and 32 u + 16 + 4 q .. + 3 (as in k_heads_prompt)
+      uint2 f[OT][2];
+#pragma unroll
+      for (int i = 0; i < NGV; ++i) {
+        asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[i][0]) : "v"(tb + vl), "n"(i * 8192 + u * 4096) : "memory");
+        asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[i][1]) : "v"(tb + vl), "n"(i * 8192 + u * 4096 + 2048) : "memory");
+      }
+      if constexpr (NH == 1) {
+        asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[NGV][0]) : "v"(tb + vh), "n"(NGV * 8192 + u * 2048) : "memory");
+        asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(f[NGV][1]) : "v"(tb + vh), "n"(NGV * 8192 + u * 2048 + 1024) : "memory");
+      }
+      const uint2 p0 = *reinterpret_cast<const uint2*>(&ps[r_in][u * 32 + 4 * cq]), p1 = *reinterpret_cast<const uint2*>(&ps[r_in][u * 32 + 16 + 4 * cq]);
+      u32x4 pv; pv.x = p0.x; pv.y = p0.y; pv.z = p1.x; pv.w = p1.y;
+      const bf16x8 pf = __builtin_bit_cast(bf16x8, pv);
+      IXT_TILE_VWAITN(f, OT, 0);
+#pragma unroll
+      for (int i = 0; i < OT; ++i) o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(f[i]), pf, o[i], 0, 0, 0);
+    }
+    __syncthreads();                                      // the tile has been read by every wave
+    if (t + nsplit < ntile) {
+      tile_dma<DK>(a.kpages, off, tile, wave, lane);
+      tile_dma<DV>(a.vpages, off, tile + 64 * DK, wave, lane);
+    }
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (cq == 0) s_l[wave][r_in] = l;
+  __syncthreads();
+  l = (s_l[0][r_in] + s_l[1][r_in]) + (s_l[2][r_in] + s_l[3][r_in]);
+  if (!pair_ok) return;
+  const size_t pi = ((size_t)row * g.H + head) * nsplit + blockIdx.z;
+  const float inv = nsplit == 1 ? 1.0f / l : 1.0f;
+#pragma unroll
+  for (int i = 0; i < OT; ++i) {
+    if (i == NGV && wave > 1) continue;                   // the half group has two column tiles
+    const int c = i * 64 + wave * 16 + cq * 4;
+    const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+    if (nsplit == 1) { if (c < g.vs) act_store4(a.out, row, head * g.vs + c, a.Kp, v); }
+    else *reinterpret_cast<float4*>(a.part_o + pi * DV + c) = make_float4(v[0], v[1], v[2], v[3]);
+  }
+  if (nsplit > 1) {
+    if (wave == 0 && cq == 0) { a.part_ml[pi * 2] = m; a.part_ml[pi * 2 + 1] = l; }
+  } else if (head == g.H - 1 && wave == 0) {
+    const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    for (int c = g.H * g.vs + cq * 4; c < a.Kp; c += 16) act_store4(a.out, row, c, a.Kp, z);
+  }
+}
+// the key splits of a row's heads put together.  grid (R, H), block 64; nsplit <= 16.
+static __global__ __launch_bounds__(64) void k_heads_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int dvp, int H, int vs,
+                                                      const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
+  __shared__ float fac[16];
+  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  if (!row_active[r]) return;
+  const size_t p0 = ((size_t)r * H + h) * nsplit;
+  split_factors(part_ml + p0 * 2, nsplit, tid, fac);
+  for (int c = tid * 4; c < vs; c += 256) {
+    float v[4];
+    split_sum4(part_o + p0 * dvp + c, dvp, nsplit, fac, v);
+    act_store4(out, r, h * vs + c, Kp, v);
+  }
+  const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  if (h == H - 1)
+    for (int c = H * vs + tid * 4; c < Kp; c += 256) act_store4(out, r, c, Kp, z);
+}

@@ -1,6 +1,7 @@
 // ixt_hybrid.hip -- host side of IXT_BLOCK_HYBRID: layer plans, weight loading, caches and states, and the forward pass over rows that every engine
 // entry point (prefill chunk, packed rows, decode step) ends in.
 #include "ixt_internal.h"
+#include "ixt_heads_kernels.h"
 #include "ixt_hybrid_kernels.h"
 
 struct HMat { void* w = nullptr; int K = 0, N = 0, Kp = 0, Np = 0; };       // a dot operand of the ctx's storage type, zero-padded
@@ -9,29 +10,34 @@ struct HLayer {
   int src = 0;                                   // the layer whose parameters are used
   LatentGeom lg{};
   DeltaGeom dg{};
+  HeadsGeom hg{};
   HMat in, low, o, gu, down;                     // input projection, second low-rank product, output projection, gate | up, down
   HMat uk, uv;                                   // per-head matrices of a latent layer (heads * wstride elements apart): d -> rank, rank -> v
   int d_off = 0;                                 // latent layer: column of the latent in the input projection
   size_t uk_stride = 0, uv_stride = 0, gu_stride = 0, down_stride = 0;
-  float *n1 = nullptr, *n2 = nullptr, *cnorm = nullptr, *cq = nullptr, *ck = nullptr, *cv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *onorm = nullptr, *router = nullptr;
+  NormW n1{}, n1b{}, n2{}, n2b{};                // in front of / behind the mixer, in front of / behind the feed-forward
+  int moe_n = 0, moe_top = 0, moe_shared = 0;    // experts and picks per token with the shared unit counted as moe_shared experts that are always picked
+  float *qn = nullptr, *kn = nullptr, *sink = nullptr, *corr = nullptr;
+  float *cnorm = nullptr, *cq = nullptr, *ck = nullptr, *cv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *onorm = nullptr, *router = nullptr;
   const float *rope_cos = nullptr, *rope_sin = nullptr;
-  void* pages = nullptr;                         // latent layer: [page][token][rankp + rotp]
+  void* pages = nullptr;                         // latent layer: [page][token][rankp + rotp]; attention layer: keys [page][kv head][token][dkp]
+  void* vpages = nullptr;                        // attention layer: values [page][kv head][token][dvp]
   float *state = nullptr, *tails = nullptr;      // delta layer: [group][H][dv][dp], [group][2][taps - 1][C]
 };
 struct HTensor { std::vector<int64_t> shape; std::function<int(const void*, int, hipStream_t)> load; bool done = false; };   // load empty: accepted, unused
 struct HybridModel {
   bool f32 = false, recurrent = false;
   size_t esz = 2;                                // bytes per activation / weight element
-  int E = 0, Ep = 0, V = 0, maxH = 0, kmax_pad = 0;
+  int E = 0, Ep = 0, V = 0, maxH = 0, kmax_pad = 0, norm_kind = 0, norm_places = 0;      // maxH: most heads of a latent layer
   float emb_scale = 1.0f, eps = 1e-5f;
   std::vector<HLayer> layers;
   std::map<std::string, HTensor> tensors;
   size_t missing = 0;
   void* embed = nullptr;
   HMat head;
-  float* fnorm = nullptr;
+  NormW fnorm{};
   // workspaces
-  float *x = nullptr, *part2 = nullptr;
+  float *x = nullptr, *part2 = nullptr, *h32 = nullptr;      // h32: a routed layer's normed input in f32
   size_t part2_floats = 0;
   void *xb = nullptr, *act = nullptr, *hact = nullptr, *xn = nullptr, *qx = nullptr, *qr = nullptr, *olat = nullptr, *xg = nullptr, *mhact = nullptr;
   float *dq = nullptr, *dk = nullptr, *dkq = nullptr, *dv = nullptr, *dec = nullptr, *beta = nullptr, *dout = nullptr, *mw = nullptr, *msum = nullptr, *po = nullptr, *pml = nullptr;
@@ -48,6 +54,16 @@ static int up_to(int v, int m) { return (v + m - 1) / m * m; }
 // what one latent row is padded to: the matrix-core kernel's sizes, beyond them multiples of 32 (k_latent_attn_any)
 static int latent_rankp(int rank) { return rank <= 64 ? 64 : rank <= 128 ? 128 : rank <= 256 ? 256 : rank <= 512 ? 512 : up_to(rank, 32); }
 static int latent_rotp(int rot) { return rot <= 32 ? 32 : rot <= 64 ? 64 : up_to(rot, 32); }
+// k_heads_prompt / k_heads_decode: the padded (key, value) sizes they are built for, cheapest first; none fits: k_heads_any
+#define IXT_HEADS_SIZES(X) X(32, 32) X(64, 64) X(64, 128) X(128, 64) X(96, 96) X(128, 128) X(192, 128) X(192, 192) X(256, 256)
+#define IXT_HEADS_SPLIT_BLOCKS 1024              // few rows: blocks that the keys of a launch are split into (four per CU)
+static bool heads_mfma_sizes(int d, int dv, bool f32, int* dkp, int* dvp) {
+  if (f32) return false;
+#define X(DK_, DV_) if (d <= DK_ && dv <= DV_) { *dkp = DK_; *dvp = DV_; return true; }
+  IXT_HEADS_SIZES(X)
+#undef X
+  return false;
+}
 static bool latent_mfma_fits(const HybridModel& m, const LatentGeom& g) { return !m.f32 && g.rankp <= 512 && g.rotp <= 64; }
 
 static int h_alloc(ixt_ctx* c, void** p, size_t bytes) {      // zero-filled: padding behind real columns is never written and must read as zero
@@ -62,11 +78,17 @@ static int h_mat(ixt_ctx* c, HMat* m, int K, int N, size_t copies = 1) {
   m->K = K; m->N = N; m->Kp = up_to(K, IXT_KALIGN); m->Np = up_to(N, 16);
   return h_alloc(c, &m->w, (size_t)m->Kp * m->Np * copies * c->hy->esz);
 }
+// where `k_load_nk` puts a matrix of n columns and k inputs; the other fields of LoadMap by name
+static LoadMap load_map(int n, int k, int Kp, int n_off = 0, int k_off = 0) {
+  LoadMap m{};
+  m.n = n; m.k = k; m.ld = k; m.Kp = Kp; m.n_off = n_off; m.k_off = k_off;
+  return m;
+}
 template <typename T>
-static int h_load_nk(const void* src, int dtype, T* dst, int n, int k, int Kp, int n_off, int k_off, int inter, int trans, hipStream_t st) {
-  const unsigned blocks = (unsigned)(((int64_t)n * k + 255) / 256);
-  if (dtype == IXT_BF16) hipLaunchKernelGGL((k_load_nk<bf16_t, T>), dim3(blocks), dim3(256), 0, st, (const bf16_t*)src, dst, n, k, Kp, n_off, k_off, inter, trans);
-  else if (dtype == IXT_F32) hipLaunchKernelGGL((k_load_nk<float, T>), dim3(blocks), dim3(256), 0, st, (const float*)src, dst, n, k, Kp, n_off, k_off, inter, trans);
+static int h_load_nk(const void* src, int dtype, T* dst, const LoadMap& lm, hipStream_t st) {
+  const unsigned blocks = (unsigned)(((int64_t)lm.n * lm.k + 255) / 256);
+  if (dtype == IXT_BF16) hipLaunchKernelGGL((k_load_nk<bf16_t, T>), dim3(blocks), dim3(256), 0, st, (const bf16_t*)src, dst, lm);
+  else if (dtype == IXT_F32) hipLaunchKernelGGL((k_load_nk<float, T>), dim3(blocks), dim3(256), 0, st, (const float*)src, dst, lm);
   else return set_err(IXT_ERR_INVALID, "dtype %d", dtype);
   LAUNCHCHK();
   return IXT_OK;
@@ -80,15 +102,20 @@ static int h_load_vec(const void* src, int dtype, T* dst, int64_t n, hipStream_t
   LAUNCHCHK();
   return IXT_OK;
 }
-static int h_load_mat(const HybridModel* m, const void* src, int dtype, void* dst, int n, int k, int Kp, int n_off, int k_off, int inter, int trans, hipStream_t st) {
-  if (m->f32) return h_load_nk(src, dtype, (float*)dst, n, k, Kp, n_off, k_off, inter, trans, st);
-  return h_load_nk(src, dtype, (bf16_t*)dst, n, k, Kp, n_off, k_off, inter, trans, st);
+static int h_load_mat(const HybridModel* m, const void* src, int dtype, void* dst, const LoadMap& lm, hipStream_t st) {
+  return m->f32 ? h_load_nk(src, dtype, (float*)dst, lm, st) : h_load_nk(src, dtype, (bf16_t*)dst, lm, st);
 }
+
+// The shared unit of a mixture is the sum of units over parts of its hidden features: it runs as further experts of the common padded size.
+static int moe_shared_parts(const ixt_layer& l) { return l.shared_ff > 0 ? (l.shared_ff + up_to(l.ff, IXT_KALIGN) - 1) / up_to(l.ff, IXT_KALIGN) : 0; }
+static int moe_experts(const ixt_layer& l) { return l.experts + moe_shared_parts(l); }
 
 int hybrid_check(const ixt_config& c) {
   if (!c.layers || c.num_decoder_layers < 1) return set_err(IXT_ERR_INVALID, "hybrid decoder: no layers");
   if (c.emb_dim < 1 || c.emb_dim > 12288 || c.vocab_size < 1) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: emb_dim %d (1 .. 12288), vocab_size %d", c.emb_dim, c.vocab_size);
   if (c.fp8_weights) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: fp8 weights are not built");
+  if ((c.norm_kind != IXT_NORM_RMS && c.norm_kind != IXT_NORM_TANH) || c.norm_places < IXT_NORM_BEFORE || c.norm_places > (IXT_NORM_BEFORE | IXT_NORM_AFTER))
+    return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: norm kind %d, places %d", c.norm_kind, c.norm_places);
   for (int i = 0; i < c.num_decoder_layers; ++i) {
     const ixt_layer& l = c.layers[i];
     if (l.weights_of >= c.num_decoder_layers || (l.weights_of >= 0 && c.layers[l.weights_of].weights_of >= 0) || l.weights_of == i)
@@ -99,12 +126,41 @@ int hybrid_check(const ixt_config& c) {
     } else if (l.mixer == IXT_MIX_GATED_DELTA) {
       if (l.kv_heads < 1 || l.heads % l.kv_heads || l.conv < 1 || l.decay_rank < 1 || l.gate_rank < 1) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / conv / ranks", i);
       if (l.dim > 512) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: delta rule key dims %d (at most 512)", i, l.dim);
+    } else if (l.mixer == IXT_MIX_ATTENTION) {
+      if (l.kv_heads < 1 || l.heads % l.kv_heads || l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > l.dim) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / rot_dim", i);
+      if (l.dim > 4096 || l.vdim > 1024) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d key dims (at most 4096), %d value dims (at most 1024)", i, l.dim, l.vdim);
+      if (!(l.attn_scale > 0.0f)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: score factor %g (positive)", i, l.attn_scale);
+      if (l.rope_factor > 0.0f && !(l.rope_low > 0.0f && l.rope_high > l.rope_low && l.rope_original > 0.0f)) return set_err(IXT_ERR_INVALID, "layer %d: rotation scaling", i);
     } else return set_err(IXT_ERR_UNSUPPORTED, "layer %d: mixer %d", i, l.mixer);
+    if (l.ffn != IXT_FFN_NONE && (l.glu < IXT_GLU_CLAMPED || l.glu > IXT_GLU_SILU)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: gated unit %d", i, l.glu);
     if (l.ffn == IXT_FFN_MOE) {
-      if (l.experts < 1 || l.experts > 1024 || l.top < 1 || l.top > l.experts || l.ff < 1) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: experts %d (1 .. 1024), top %d", i, l.experts, l.top);
+      if (l.experts < 1 || l.top < 1 || l.top > l.experts || l.ff < 1 || l.shared_ff < 0 || moe_experts(l) > 1024)
+        return set_err(IXT_ERR_UNSUPPORTED, "layer %d: experts %d (with the shared unit's share 1 .. 1024), top %d", i, l.experts, l.top);
+      if (l.router != IXT_ROUTE_SOFTMAX && l.router != IXT_ROUTE_SIGMOID) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: router %d", i, l.router);
+      if (l.groups > 1 && (l.experts % l.groups || l.groups_keep < 1 || l.groups_keep > l.groups || l.top > l.experts / l.groups * l.groups_keep))
+        return set_err(IXT_ERR_INVALID, "layer %d: %d of %d groups of experts, top %d", i, l.groups_keep, l.groups, l.top);
     } else if (l.ffn == IXT_FFN_DENSE) {
       if (l.ff < 1) return set_err(IXT_ERR_INVALID, "layer %d: ff", i);
     } else if (l.ffn != IXT_FFN_NONE) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: ffn %d", i, l.ffn);
+  }
+  return IXT_OK;
+}
+
+// a norm's tensors: `name`, and for a tanh norm name.alpha (a scalar) and name.b; zeros behind the E features
+static int hybrid_norm_params(ixt_ctx* c, const std::string& name, NormW* w) {
+  HybridModel* m = c->hy;
+  const int E = m->E;
+  auto one = [&](const std::string& t, const float** dst, int64_t n, std::vector<int64_t> shape) -> int {
+    float* d = nullptr;
+    TRY(h_allocf(c, &d, (size_t)m->Ep));
+    *dst = d;
+    m->tensors[t] = HTensor{std::move(shape), [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, d, n, st); }, false};
+    return IXT_OK;
+  };
+  TRY(one(name, &w->w, E, {E}));
+  if (m->norm_kind == IXT_NORM_TANH) {
+    TRY(one(name + ".alpha", &w->alpha, 1, {}));
+    TRY(one(name + ".b", &w->b, E, {E}));
   }
   return IXT_OK;
 }
@@ -123,12 +179,15 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     add(name, std::move(shape), [d, n](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, d, n, st); });
     return IXT_OK;
   };
-  auto mat = [&](const std::string& name, const HMat& M, int n, int k, int n_off, int k_off = 0, int inter = 0, size_t elem_off = 0) {
+  auto mat_as = [&](const std::string& name, const HMat& M, const LoadMap& lm, size_t elem_off = 0) {
     char* d = (char*)M.w + elem_off * m->esz;
-    const int Kp = M.Kp;
-    add(name, {n, k}, [=](const void* s, int dt, hipStream_t st) { return h_load_mat(m, s, dt, d, n, k, Kp, n_off, k_off, inter, 0, st); });
+    add(name, {lm.n, lm.k}, [=](const void* s, int dt, hipStream_t st) { return h_load_mat(m, s, dt, d, lm, st); });
   };
-  TRY(vec("norm1", &L.n1, E, {E}));
+  auto mat = [&](const std::string& name, const HMat& M, int n, int k, int n_off, int k_off = 0) { mat_as(name, M, load_map(n, k, M.Kp, n_off, k_off)); };
+  auto norm = [&](const std::string& name, NormW* w) -> int { return hybrid_norm_params(c, p + name, w); };
+  const bool both = m->norm_places == (IXT_NORM_BEFORE | IXT_NORM_AFTER);
+  TRY(norm("norm1", m->norm_places & IXT_NORM_BEFORE ? &L.n1 : &L.n1b));
+  if (both) TRY(norm("norm1b", &L.n1b));
   if (l.mixer == IXT_MIX_LATENT_ATTENTION) {
     const LatentGeom& g = L.lg;
     const int NQ = g.H * (g.dn + g.dr);
@@ -141,17 +200,33 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     L.uk_stride = (size_t)L.uk.Kp * L.uk.Np; L.uv_stride = (size_t)L.uv.Kp * L.uv.Np;
     const HLayer* Lp = &L;
     add("mix.uk", {(int64_t)g.H * g.dn, g.rank}, [=](const void* s, int dt, hipStream_t st) {     // [h dn + i][c] -> per head (k = i, n = c): queries into latent space
+      LoadMap uk = load_map(Lp->lg.rank, Lp->lg.dn, Lp->uk.Kp);
+      uk.trans = 1; uk.ld = uk.n;
       for (int h = 0; h < Lp->lg.H; ++h)
-        TRY(h_load_mat(m, (const char*)s + (size_t)h * Lp->lg.dn * Lp->lg.rank * (dt == IXT_F32 ? 4 : 2), dt, (char*)Lp->uk.w + h * Lp->uk_stride * m->esz, Lp->lg.rank, Lp->lg.dn, Lp->uk.Kp, 0, 0, 0, 1, st));
+        TRY(h_load_mat(m, (const char*)s + (size_t)h * Lp->lg.dn * Lp->lg.rank * (dt == IXT_F32 ? 4 : 2), dt, (char*)Lp->uk.w + h * Lp->uk_stride * m->esz, uk, st));
       return (int)IXT_OK;
     });
     add("mix.uv", {(int64_t)g.H * l.vdim, g.rank}, [=](const void* s, int dt, hipStream_t st) {
       for (int h = 0; h < Lp->lg.H; ++h)
-        TRY(h_load_mat(m, (const char*)s + (size_t)h * Lp->c.vdim * Lp->lg.rank * (dt == IXT_F32 ? 4 : 2), dt, (char*)Lp->uv.w + h * Lp->uv_stride * m->esz, Lp->c.vdim, Lp->lg.rank, Lp->uv.Kp, 0, 0, 0, 0, st));
+        TRY(h_load_mat(m, (const char*)s + (size_t)h * Lp->c.vdim * Lp->lg.rank * (dt == IXT_F32 ? 4 : 2), dt, (char*)Lp->uv.w + h * Lp->uv_stride * m->esz, load_map(Lp->c.vdim, Lp->lg.rank, Lp->uv.Kp), st));
       return (int)IXT_OK;
     });
     TRY(h_mat(c, &L.o, g.H * l.vdim, E));
     mat("mix.o", L.o, E, g.H * l.vdim, 0);
+  } else if (l.mixer == IXT_MIX_ATTENTION) {
+    const HeadsGeom& g = L.hg;
+    TRY(h_mat(c, &L.in, E, g.ov + g.G * g.vs));
+    LoadMap q = load_map(g.H * g.d, E, L.in.Kp), k = load_map(g.G * g.d, E, L.in.Kp, g.ok), v = load_map(g.G * g.dv, E, L.in.Kp, g.ov);
+    q.ng = k.ng = g.d; q.ngp = k.ngp = g.hs; v.ng = g.dv; v.ngp = g.vs;
+    mat_as("mix.q", L.in, q);
+    mat_as("mix.k", L.in, k);
+    mat_as("mix.v", L.in, v);
+    if (l.qk_norm) { TRY(vec("mix.q.norm", &L.qn, g.d, {g.d})); TRY(vec("mix.k.norm", &L.kn, g.d, {g.d})); }
+    if (l.sink) TRY(vec("mix.sink", &L.sink, g.H, {g.H}));
+    TRY(h_mat(c, &L.o, g.H * g.vs, E));
+    LoadMap o = load_map(E, g.H * g.dv, L.o.Kp);
+    o.kg = g.dv; o.kgp = g.vs;
+    mat_as("mix.o", L.o, o);
   } else {
     const DeltaGeom& g = L.dg;
     TRY(h_mat(c, &L.in, E, g.og + g.rg));
@@ -173,27 +248,78 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     TRY(h_mat(c, &L.o, g.H * g.dv, E));
     mat("mix.o", L.o, E, g.H * g.dv, 0);
   }
-  if (l.ffn == IXT_FFN_NONE) {
-    m->tensors[p + "norm2"] = HTensor{{E}, nullptr, true};       // a layer without a feed-forward has no use for its norm
-  } else {
-    TRY(vec("norm2", &L.n2, E, {E}));
-    const int Fp = up_to(l.ff, IXT_KALIGN), n = l.ffn == IXT_FFN_MOE ? l.experts : 1;
-    TRY(h_mat(c, &L.gu, E, 2 * Fp, n));
-    TRY(h_mat(c, &L.down, l.ff, E, n));
-    L.gu_stride = (size_t)L.gu.Kp * L.gu.Np; L.down_stride = (size_t)L.down.Kp * L.down.Np;
-    for (int e = 0; e < n; ++e) {
-      const std::string q = l.ffn == IXT_FFN_MOE ? "mlp.e" + std::to_string(e) + "." : "mlp.";
-      mat(q + "gate", L.gu, l.ff, E, 0, 0, 1, e * L.gu_stride);
-      mat(q + "up", L.gu, l.ff, E, 1, 0, 1, e * L.gu_stride);
-      mat(q + "down", L.down, E, l.ff, 0, 0, 0, e * L.down_stride);
+  if (l.ffn == IXT_FFN_NONE) {                                   // a layer without a feed-forward has no use for its norms
+    for (const char* n : {"norm2", "norm2b"}) {
+      if (!both && std::string(n) == "norm2b") continue;
+      m->tensors[p + n] = HTensor{{E}, nullptr, true};
+      if (m->norm_kind == IXT_NORM_TANH) { m->tensors[p + n + ".alpha"] = HTensor{{}, nullptr, true}; m->tensors[p + n + ".b"] = HTensor{{E}, nullptr, true}; }
     }
-    if (l.ffn == IXT_FFN_MOE) {
-      TRY(h_allocf(c, &L.router, (size_t)l.experts * m->Ep));
-      float* d = L.router;
-      const int n_ = l.experts, E_ = E, Ep_ = m->Ep;
-      add("mlp.router", {l.experts, E}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, n_, E_, Ep_, 0, 0, 0, 0, st); });
-    }
+    return IXT_OK;
   }
+  TRY(norm("norm2", m->norm_places & IXT_NORM_BEFORE ? &L.n2 : &L.n2b));
+  if (both) TRY(norm("norm2b", &L.n2b));
+  const int Fp = up_to(l.ff, IXT_KALIGN), n = l.ffn == IXT_FFN_MOE ? L.moe_n : 1;
+  TRY(h_mat(c, &L.gu, E, 2 * Fp, n));
+  TRY(h_mat(c, &L.down, Fp, E, n));
+  L.gu_stride = (size_t)L.gu.Kp * L.gu.Np; L.down_stride = (size_t)L.down.Kp * L.down.Np;
+  LoadMap gate = load_map(l.ff, E, L.gu.Kp), up = load_map(l.ff, E, L.gu.Kp, 1);
+  gate.inter = up.inter = 1;
+  for (int e = 0; e < (l.ffn == IXT_FFN_MOE ? l.experts : 1); ++e) {
+    const std::string q = l.ffn == IXT_FFN_MOE ? "mlp.e" + std::to_string(e) + "." : "mlp.";
+    mat_as(q + "gate", L.gu, gate, e * L.gu_stride);
+    mat_as(q + "up", L.gu, up, e * L.gu_stride);
+    mat_as(q + "down", L.down, load_map(E, l.ff, L.down.Kp), e * L.down_stride);
+  }
+  if (l.ffn != IXT_FFN_MOE) return IXT_OK;
+  if (L.moe_shared > 0) {                                        // Fp hidden features per part
+    const HLayer* Lp = &L;
+    auto part = [&](const char* name, bool down, int n_off) {
+      std::vector<int64_t> shape = down ? std::vector<int64_t>{E, l.shared_ff} : std::vector<int64_t>{l.shared_ff, E};
+      add(std::string("mlp.shared.") + name, shape, [=](const void* s, int dt, hipStream_t st) {
+        const int ff = Lp->c.shared_ff;
+        for (int j = 0; j < Lp->moe_shared; ++j) {
+          const int w = std::min(Fp, ff - j * Fp), e = Lp->c.experts + j;
+          LoadMap lm = down ? load_map(E, w, Lp->down.Kp) : load_map(w, E, Lp->gu.Kp, n_off);
+          if (down) lm.ld = ff; else lm.inter = 1;
+          const size_t at = (size_t)j * Fp * (down ? 1 : E) * (dt == IXT_F32 ? 4 : 2);
+          TRY(h_load_mat(m, (const char*)s + at, dt, (char*)(down ? Lp->down.w : Lp->gu.w) + e * (down ? Lp->down_stride : Lp->gu_stride) * m->esz, lm, st));
+        }
+        return (int)IXT_OK;
+      });
+    };
+    part("gate", false, 0); part("up", false, 1); part("down", true, 0);
+  }
+  TRY(h_allocf(c, &L.router, (size_t)l.experts * m->Ep));
+  float* d = L.router;
+  const LoadMap lm = load_map(l.experts, E, m->Ep);
+  add("mlp.router", {l.experts, E}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, lm, st); });
+  if (l.router_correction) TRY(vec("mlp.correction", &L.corr, l.experts, {l.experts}));
+  return IXT_OK;
+}
+
+// rotation tables of a layer, f32 [position][rot_dim / 2] cos and sin of angles in f64; layers with the same rotation share them
+static int hybrid_rope(ixt_ctx* c, const ixt_layer& l, std::map<std::vector<float>, std::pair<float*, float*>>* ropes, HLayer* L) {
+  const std::vector<float> key = {(float)l.rot_dim, l.rope_base, l.rope_factor, l.rope_low, l.rope_high, l.rope_original};
+  auto it = ropes->find(key);
+  if (it == ropes->end()) {
+    const int half = l.rot_dim / 2;
+    std::vector<float> cs((size_t)c->Tmax * half + 1), sn((size_t)c->Tmax * half + 1);
+    for (int j = 0; j < half; ++j) {
+      double f = pow((double)l.rope_base, -2.0 * j / l.rot_dim);
+      if (l.rope_factor > 0.0f) {
+        const double turns = l.rope_original * f / (2.0 * M_PI);            // of this pair over the original context
+        if (turns < l.rope_low) f /= l.rope_factor;
+        else if (turns <= l.rope_high) { const double s = (turns - l.rope_low) / ((double)l.rope_high - l.rope_low); f = (1.0 - s) * f / l.rope_factor + s * f; }
+      }
+      for (int p = 0; p < c->Tmax; ++p) { cs[(size_t)p * half + j] = (float)cos(p * f); sn[(size_t)p * half + j] = (float)sin(p * f); }
+    }
+    float *dc = nullptr, *ds = nullptr;
+    TRY(h_allocf(c, &dc, cs.size())); TRY(h_allocf(c, &ds, sn.size()));
+    HIPCHK(hipMemcpy(dc, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
+    HIPCHK(hipMemcpy(ds, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
+    it = ropes->emplace(key, std::make_pair(dc, ds)).first;
+  }
+  L->rope_cos = it->second.first; L->rope_sin = it->second.second;
   return IXT_OK;
 }
 
@@ -203,18 +329,17 @@ int hybrid_init(ixt_ctx* c) {
   HybridModel* m = c->hy;
   m->f32 = cf.float32 != 0; m->esz = m->f32 ? 4 : 2;
   m->E = cf.emb_dim; m->Ep = up_to(m->E, IXT_KALIGN); m->V = cf.vocab_size; m->emb_scale = cf.embedding_scale; m->eps = cf.normalization_layer_epsilon;
+  m->norm_kind = cf.norm_kind; m->norm_places = cf.norm_places;
   const int n = cf.num_decoder_layers, R = c->Rmax, Rp = up_to(R, 128);
   m->layers.resize(n);
   TRY(h_alloc(c, &m->embed, (size_t)m->V * m->E * m->esz));
   { void* d = m->embed; const int64_t ne = (int64_t)m->V * m->E; const bool f = m->f32;
     m->tensors["embed"] = HTensor{{m->V, m->E}, [=](const void* s, int dt, hipStream_t st) { return f ? h_load_vec(s, dt, (float*)d, ne, st) : h_load_vec(s, dt, (bf16_t*)d, ne, st); }, false}; }
   TRY(h_mat(c, &m->head, m->E, m->V));
-  { void* d = m->head.w; const int V = m->V, E = m->E, Kp = m->head.Kp;
-    m->tensors["head"] = HTensor{{V, E}, [=](const void* s, int dt, hipStream_t st) { return h_load_mat(m, s, dt, d, V, E, Kp, 0, 0, 0, 0, st); }, false}; }
-  TRY(h_allocf(c, &m->fnorm, (size_t)m->E));
-  { float* d = m->fnorm; const int E = m->E;
-    m->tensors["final.norm"] = HTensor{{E}, [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, d, E, st); }, false}; }
-  std::map<std::pair<int, float>, std::pair<float*, float*>> ropes;
+  { void* d = m->head.w; const LoadMap lm = load_map(m->V, m->E, m->head.Kp);
+    m->tensors["head"] = HTensor{{m->V, m->E}, [=](const void* s, int dt, hipStream_t st) { return h_load_mat(m, s, dt, d, lm, st); }, false}; }
+  TRY(hybrid_norm_params(c, "final.norm", &m->fnorm));
+  std::map<std::vector<float>, std::pair<float*, float*>> ropes;
   size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0;
   auto upd = [](size_t& a, size_t v) { if (v > a) a = v; };
   // f32 slices of a dot over at most R rows (split-K only below 128 rows; launch_dot keeps to one slice when the slices do not fit)
@@ -230,23 +355,7 @@ int hybrid_init(ixt_ctx* c) {
       g.rankp = latent_rankp(l.kv_rank); g.rotp = latent_rotp(l.rot_dim);
       L.d_off = up_to(g.H * (g.dn + g.dr), 16);
       TRY(h_alloc(c, &L.pages, (size_t)cf.pagedattn_num_pages * c->P * (g.rankp + g.rotp) * m->esz));
-      auto key = std::make_pair(l.rot_dim, l.rope_base);
-      auto it = ropes.find(key);
-      if (it == ropes.end()) {
-        const int half = l.rot_dim / 2;
-        std::vector<float> cs((size_t)c->Tmax * half + 1), sn((size_t)c->Tmax * half + 1);
-        for (int p = 0; p < c->Tmax; ++p)
-          for (int j = 0; j < half; ++j) {
-            const double a = (double)p * pow((double)l.rope_base, -2.0 * j / l.rot_dim);
-            cs[(size_t)p * half + j] = (float)cos(a); sn[(size_t)p * half + j] = (float)sin(a);
-          }
-        float *dc = nullptr, *ds = nullptr;
-        TRY(h_allocf(c, &dc, cs.size())); TRY(h_allocf(c, &ds, sn.size()));
-        HIPCHK(hipMemcpy(dc, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
-        HIPCHK(hipMemcpy(ds, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
-        it = ropes.emplace(key, std::make_pair(dc, ds)).first;
-      }
-      L.rope_cos = it->second.first; L.rope_sin = it->second.second;
+      TRY(hybrid_rope(c, l, &ropes, &L));
       m->maxH = std::max(m->maxH, g.H);
       const int dnp = up_to(g.dn, IXT_KALIGN), ukn = up_to(g.rankp, 16), kp = up_to(g.rankp, IXT_KALIGN), uvn = up_to(l.vdim, 16);
       dotsz(m->Ep, up_to(L.d_off + g.rank + g.dr, 16));
@@ -258,6 +367,21 @@ int hybrid_init(ixt_ctx* c) {
       upd(act_k, up_to(g.H * l.vdim, IXT_KALIGN));
       upd(qx_e, (size_t)g.H * Rp * dnp); upd(qr_e, (size_t)R * g.H * g.rotp); upd(olat_e, (size_t)g.H * Rp * kp);
       upd(po, (size_t)(1024 + g.H) * 16 * g.rankp);
+    } else if (l.mixer == IXT_MIX_ATTENTION) {
+      HeadsGeom& g = L.hg;
+      g.H = l.heads; g.G = l.kv_heads; g.d = l.dim; g.dv = l.vdim; g.rot = l.rot_dim; g.P = c->P; g.mpg = c->mpg; g.window = l.window; g.scale = l.attn_scale;
+      if (!heads_mfma_sizes(l.dim, l.vdim, m->f32, &g.dkp, &g.dvp)) { g.dkp = up_to(l.dim, 32); g.dvp = up_to(l.vdim, 32); }
+      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4); g.ok = up_to(g.H * g.hs, 16); g.ov = g.ok + up_to(g.G * g.hs, 16);
+      const size_t tokens = (size_t)cf.pagedattn_num_pages * c->P * g.G;
+      if (tokens > (size_t)INT32_MAX) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %zu cached heads in the page pool", i, tokens);
+      TRY(h_alloc(c, &L.pages, tokens * g.dkp * m->esz));
+      TRY(h_alloc(c, &L.vpages, tokens * g.dvp * m->esz));
+      TRY(hybrid_rope(c, l, &ropes, &L));
+      dotsz(m->Ep, up_to(g.ov + g.G * g.vs, 16));
+      dotsz(up_to(g.H * g.vs, IXT_KALIGN), up_to(m->E, 16));
+      upd(act_k, up_to(g.H * g.vs, IXT_KALIGN));
+      upd(qx_e, (size_t)R * g.H * g.dkp);
+      upd(po, (size_t)IXT_HEADS_SPLIT_BLOCKS * 16 * g.dvp);
     } else {
       m->recurrent = true;
       DeltaGeom& g = L.dg;
@@ -281,14 +405,16 @@ int hybrid_init(ixt_ctx* c) {
       if (m->f32) upd(part, (size_t)R * 2 * Fp);
       dotsz(Fp, up_to(m->E, 16));
     } else if (l.ffn == IXT_FFN_MOE) {
-      const int Fp = up_to(l.ff, IXT_KALIGN), pairs = R * l.top;
-      if (pairs > 60000) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d rows x %d experts per token exceed one launch (60000 copies): smaller max_packed_rows / max_prefill_predict_length", i, R, l.top);
-      const int cap = std::max(up_to(pairs, 128) + 128 * std::min(l.experts, pairs), 64 + 16 * l.experts);
+      L.moe_shared = moe_shared_parts(l); L.moe_n = moe_experts(l); L.moe_top = l.top + L.moe_shared;
+      const int Fp = up_to(l.ff, IXT_KALIGN);
+      if ((int64_t)R * L.moe_top > (1 << 24)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d rows x %d experts per token: smaller max_packed_rows / max_prefill_predict_length", i, R, L.moe_top);
+      const int pairs = R * L.moe_top, cap = std::max(up_to(pairs, 128) + 128 * std::min(L.moe_n, pairs), 64 + 16 * L.moe_n);
       m->moe_cap = std::max(m->moe_cap, cap);
       upd(xg_e, (size_t)cap * m->Ep); upd(mh_e, (size_t)cap * Fp); upd(mi, (size_t)pairs);
       upd(part, (size_t)cap * up_to(m->E, 16));
-      upd(part, (size_t)(64 + 16 * std::min(l.experts, 64)) * up_to(m->E, 16) * ((Fp + IXT_CHAIN - 1) / IXT_CHAIN));
+      upd(part, (size_t)(64 + 16 * std::min(L.moe_n, 64)) * up_to(m->E, 16) * ((Fp + IXT_CHAIN - 1) / IXT_CHAIN));
       if (m->f32) upd(part, (size_t)cap * 2 * Fp);
+      if (!m->h32 && (m->norm_places & IXT_NORM_BEFORE)) TRY(h_allocf(c, &m->h32, (size_t)R * m->E));
     }
   }
   for (int i = 0; i < n; ++i)
@@ -310,7 +436,7 @@ int hybrid_init(ixt_ctx* c) {
   TRY(h_allocf(c, &m->mw, mi + 4)); TRY(h_allocf(c, &m->midx, mi + 4)); TRY(h_allocf(c, &m->mpos, mi + 4));
   TRY(h_allocf(c, &m->mrb, (size_t)m->moe_cap / 16 + 16));
   TRY(h_allocf(c, &m->msum, (size_t)64 * up_to(m->E, 16)));
-  TRY(h_allocf(c, &m->po, po + 4)); TRY(h_allocf(c, &m->pml, (size_t)(1024 + m->maxH) * 16 * 2 + 4));
+  TRY(h_allocf(c, &m->po, po + 4)); TRY(h_allocf(c, &m->pml, (size_t)(IXT_HEADS_SPLIT_BLOCKS + m->maxH) * 16 * 2 + 4));
   TRY(h_allocf(c, &m->row_seg, (size_t)R)); TRY(h_allocf(c, &m->row_j, (size_t)R)); TRY(h_allocf(c, &m->seg, (size_t)R * 8)); TRY(h_allocf(c, &m->nseg, 4));
   TRY(h_allocf(c, &m->state_len, (size_t)c->G)); TRY(h_allocf(c, &m->parity, (size_t)c->G)); TRY(h_allocf(c, &m->claim, (size_t)c->G)); TRY(h_allocf(c, &m->err, 4));
   TRY(h_allocf(c, &m->head_rb, (size_t)m->maxH * Rp / 16 + 16));
@@ -319,7 +445,10 @@ int hybrid_init(ixt_ctx* c) {
   // what a copy of a whole page group moves
   std::vector<float*> sb; std::vector<int64_t> sp, pb; std::vector<char*> pp;
   for (HLayer& L : m->layers) {
-    if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) { pp.push_back((char*)L.pages); pb.push_back((int64_t)c->P * (L.lg.rankp + L.lg.rotp) * (int64_t)m->esz); }
+    if (L.c.mixer == IXT_MIX_ATTENTION) {
+      pp.push_back((char*)L.pages); pb.push_back((int64_t)c->P * L.hg.G * L.hg.dkp * (int64_t)m->esz);
+      pp.push_back((char*)L.vpages); pb.push_back((int64_t)c->P * L.hg.G * L.hg.dvp * (int64_t)m->esz);
+    } else if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) { pp.push_back((char*)L.pages); pb.push_back((int64_t)c->P * (L.lg.rankp + L.lg.rotp) * (int64_t)m->esz); }
     else { sb.push_back(L.state); sp.push_back((int64_t)L.dg.H * L.dg.dv * L.dg.dp); sb.push_back(L.tails); sp.push_back((int64_t)2 * (L.dg.taps - 1) * L.dg.C); }
   }
   m->st_n = (int)sb.size(); m->pg_n = (int)pp.size();
@@ -404,24 +533,24 @@ template <> int hdot_grouped<float>(ixt_ctx*, const float* x, const HMat& w, siz
   *res = Slices{out, 1, (size_t)rows * w.Np, w.Np};
   return IXT_OK;
 }
-// gate | up product with the clamped unit behind it -> act(T) of the down product
-template <typename T> static int hglu(ixt_ctx* c, const T* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, float limit, T* out, hipStream_t st);
-template <> int hglu<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, float limit, bf16_t* out, hipStream_t st) {
+// gate | up product with the gated unit (IXT_GLU_*) behind it -> act(T) of the down product
+template <typename T> static int hglu(ixt_ctx* c, const T* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, float limit, T* out, hipStream_t st);
+template <> int hglu<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, float limit, bf16_t* out, hipStream_t st) {
   if (rb ? group_rows % 128 == 0 : rows >= c->ring_min_rows) {
     GemmEpi e{};
-    e.act = out; e.glu = 1; e.glu_limit = limit; e.rb_exp = rb; e.wstride = stride / 8;
+    e.act = out; e.glu = kind; e.glu_limit = limit; e.rb_exp = rb; e.wstride = stride / 8;
     return launch_ring(c, GEPI_SWIGLU, x, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, false, st);
   }
   if (!rb && rows <= c->small_rows && sdot_plan(c, GEPI_SWIGLU, false, w.Kp, w.Np, rows).ok) {
     GemmEpi e{};
-    e.act = out; e.glu = 1; e.glu_limit = limit;
+    e.act = out; e.glu = kind; e.glu_limit = limit;
     return launch_sdot(c, GEPI_SWIGLU, false, x, nullptr, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, st);
   }
   const int rowblocks = (rows + 15) / 16, nrb = rb ? 1 : (rowblocks >= 3 ? 4 : rowblocks), zblocks = (rowblocks + nrb - 1) / nrb, ntile = w.Np / 16;
   dim3 grid((((ntile + 3) / 4 + 7) / 8) * 8 * zblocks, 1, 1);
   const u32x4 *xp = reinterpret_cast<const u32x4*>(x), *wp = reinterpret_cast<const u32x4*>(w.w);
   float* o = reinterpret_cast<float*>(out);
-#define HGLU(B_, NT_) hipLaunchKernelGGL((k_dotb<B_, false, NT_, 1>), grid, dim3(256), (size_t)(B_) * 16 * 1024, st, xp, wp, w.Kp, w.Np, rows, o, ntile, zblocks, rb, stride / 8, 1, limit)
+#define HGLU(B_, NT_) hipLaunchKernelGGL((k_dotb<B_, false, NT_, 1>), grid, dim3(256), (size_t)(B_) * 16 * 1024, st, xp, wp, w.Kp, w.Np, rows, o, ntile, zblocks, rb, stride / 8, kind, limit)
   if (nrb == 4) { if (zblocks == 1) HGLU(4, true); else HGLU(4, false); }
   else if (nrb == 2) HGLU(2, true);
   else HGLU(1, true);
@@ -429,10 +558,10 @@ template <> int hglu<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, size_t 
   LAUNCHCHK();
   return IXT_OK;
 }
-template <> int hglu<float>(ixt_ctx* c, const float* x, const HMat& w, size_t stride, int rows, int, const int32_t* rb, float limit, float* out, hipStream_t st) {
+template <> int hglu<float>(ixt_ctx* c, const float* x, const HMat& w, size_t stride, int rows, int, const int32_t* rb, int kind, float limit, float* out, hipStream_t st) {
   Slices t;
   TRY(hdot_grouped<float>(c, x, w, stride, rows, 16, rb, c->part, c->part_floats, st, &t));
-  hipLaunchKernelGGL((k_glu_clamped<float>), dim3((w.Np / 2 + 255) / 256, rows), dim3(256), 0, st, t, w.Np / 2, limit, out, rb);
+  hipLaunchKernelGGL((k_glu_slices<float>), dim3(rows, (w.Np / 2 + 255) / 256), dim3(256), 0, st, t, w.Np / 2, kind, limit, out, rb);
   LAUNCHCHK();
   return IXT_OK;
 }
@@ -513,6 +642,71 @@ static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int
   return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
 }
 
+template <int DK, int DV, int MP>
+static int heads_prompt_launch(HeadsAttnArgs a, hipStream_t st) {
+  constexpr int lds = 2 * 64 * (DK + DV) * 2;
+  static bool attr_done = false;
+  if (!attr_done) {
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_prompt<DK, DV, MP>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    attr_done = true;
+  }
+  const int GQ = a.g.H / a.g.G;
+  a.HB = std::min(GQ, 64 * MP); a.NQ = 64 * MP / a.HB; a.hchunks = (GQ + a.HB - 1) / a.HB;
+  hipLaunchKernelGGL((k_heads_prompt<DK, DV, MP>), dim3(a.g.G * a.hchunks, (a.R + a.NQ - 1) / a.NQ), dim3(256), lds, st, a);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <int DK, int DV>
+static int heads_launch(bool tall, int splits, HeadsAttnArgs a, hipStream_t st) {
+  if (tall) return heads_prompt_launch<DK, DV, 1>(a, st);
+  hipLaunchKernelGGL((k_heads_decode<DK, DV>), dim3(a.R, a.g.G * a.hchunks, splits), dim3(256), 64 * (DK + DV) * 2, st, a);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+// queries over the paged keys and values -> act(T) of the output projection
+template <typename T>
+static int heads_attention(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, bool decode, int len_hint, hipStream_t st) {
+  HybridModel* m = c->hy;
+  const HeadsGeom& g = L.hg;
+  const RowsArgs rows{c->row_slot, c->row_pos, c->row_active, c->ps.page_map};
+  int dkp = 0, dvp = 0;
+  if constexpr (sizeof(T) == 2) {
+    if (heads_mfma_sizes(g.d, g.dv, m->f32, &dkp, &dvp)) {
+      const bool tall = !decode && R > 32;
+      const int GQ = g.H / g.G, hchunks = (GQ + 15) / 16, blocks = R * g.G * hchunks, span = g.window > 0 ? std::min(g.window, len_hint) : len_hint;
+      int splits = 1;
+      if (!tall) splits = std::min(std::min(16, std::max(1, IXT_HEADS_SPLIT_BLOCKS / blocks)), std::max(1, (span + 63) / 64));     // at least a tile each
+      HeadsAttnArgs a{(const bf16_t*)m->qx, g, W.sink, rows, (const bf16_t*)L.pages, (const bf16_t*)L.vpages, R, 1, (GQ + hchunks - 1) / hchunks, hchunks, __builtin_ctz(c->P),
+                      (bf16_t*)m->act, W.o.Kp, m->po, m->pml};
+      int rc = IXT_ERR_UNSUPPORTED;
+#define X(DK_, DV_) if (dkp == DK_ && dvp == DV_) rc = heads_launch<DK_, DV_>(tall, splits, a, st);
+      IXT_HEADS_SIZES(X)
+#undef X
+      TRY(rc);
+      if (splits > 1) {
+        hipLaunchKernelGGL(k_heads_combine, dim3(R, g.H), dim3(64), 0, st, m->po, m->pml, splits, g.dvp, g.H, g.vs, c->row_active, (bf16_t*)m->act, W.o.Kp);
+        LAUNCHCHK();
+      }
+      return IXT_OK;
+    }
+  }
+  hipLaunchKernelGGL((k_heads_any<T>), dim3(R, g.H), dim3(256), sizeof(float) * (g.dkp + 256), st, (const T*)m->qx, g, W.sink, rows, (const T*)L.pages, (const T*)L.vpages, (T*)m->act, W.o.Kp);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <typename T>
+static int hybrid_mixer_heads(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, bool decode, int len_hint, hipStream_t st, Slices* out) {
+  HybridModel* m = c->hy;
+  const HeadsGeom& g = L.hg;
+  Slices t;
+  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &t));
+  hipLaunchKernelGGL((k_heads_prep<T>), dim3(R, (g.H + 2 * g.G + 3) / 4), dim3(256), 0, st, t, g, W.qn, W.kn, m->eps, L.rope_cos, L.rope_sin,
+                     RowsArgs{c->row_slot, c->row_pos, c->row_active, c->ps.page_map}, (T*)L.pages, (T*)L.vpages, (T*)m->qx);
+  LAUNCHCHK();
+  TRY(heads_attention<T>(c, L, W, R, decode, len_hint, st));
+  return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
+}
+
 template <typename T>
 static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st, Slices* out) {
   HybridModel* m = c->hy;
@@ -546,23 +740,26 @@ static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int 
   return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
 }
 
-// routed mixture: expert outputs stay in copy order (slices `out`, row m->mpos[r top + j], weight m->mw[r top + j]); the norm kernel adds them up
+// routed mixture: expert outputs stay in copy order (slices `out`, row m->mpos[r moe_top + j], weight m->mw[r moe_top + j]); the norm kernel adds them up
 template <typename T>
 static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipStream_t st, Slices* out) {
   HybridModel* m = c->hy;
   const ixt_layer& l = L.c;
-  const int pairs = R * l.top;
-  if (R <= 256) hipLaunchKernelGGL((k_route<1>), dim3(R), dim3(256), sizeof(float) * l.experts, st, m->x, W.router, m->E, m->Ep, l.experts, l.top, R, m->midx, m->mw);
-  else hipLaunchKernelGGL((k_route<4>), dim3((R + 3) / 4), dim3(256), sizeof(float) * 4 * l.experts, st, m->x, W.router, m->E, m->Ep, l.experts, l.top, R, m->midx, m->mw);
+  const int pairs = R * L.moe_top, n = L.moe_n;
+  const RouteRule rule{l.experts, l.top, l.router, l.groups > 1 ? l.groups : 0, l.groups_keep, l.router_norm, L.moe_shared, l.router_scale, W.corr};
+  const float* h = (m->norm_places & IXT_NORM_BEFORE) ? m->h32 : m->x;
+  const size_t lds = sizeof(float) * (l.experts + 2 * rule.groups);
+  if (R <= 256) hipLaunchKernelGGL((k_route<1>), dim3(R), dim3(256), lds, st, h, W.router, m->E, m->Ep, rule, R, m->midx, m->mw);
+  else hipLaunchKernelGGL((k_route<4>), dim3((R + 3) / 4), dim3(256), 4 * lds, st, h, W.router, m->E, m->Ep, rule, R, m->midx, m->mw);
   LAUNCHCHK();
   const int align = (m->f32 || pairs <= 64) ? 16 : 128;
-  const int rows_g = up_to(pairs, align) + align * std::min(l.experts, pairs);     // every expert with a copy may waste up to align - 1 rows
+  const int rows_g = up_to(pairs, align) + align * std::min(n, pairs);     // every expert with a copy may waste up to align - 1 rows
   if (rows_g > m->moe_cap) return set_err(IXT_ERR_INVALID, "moe: %d copies exceed the routed workspaces", pairs);
-  hipLaunchKernelGGL(k_moe_plan_any, dim3(1), dim3(1024), 0, st, m->midx, pairs, l.experts, align, rows_g / 16, m->mpos, m->mrb);
-  if constexpr (sizeof(T) == 2) hipLaunchKernelGGL(k_moe_gather, dim3((m->Ep + 2047) / 2048, pairs), dim3(256), 0, st, (const bf16_t*)m->xb, m->mpos, l.top, m->Ep, (bf16_t*)m->xg);
-  else hipLaunchKernelGGL(k_gather32, dim3((m->Ep + 255) / 256, pairs), dim3(256), 0, st, (const float*)m->xb, m->mpos, l.top, m->Ep, (float*)m->xg);
+  hipLaunchKernelGGL(k_moe_plan_any, dim3(1), dim3(1024), 0, st, m->midx, pairs, n, align, rows_g / 16, m->mpos, m->mrb);
+  if constexpr (sizeof(T) == 2) hipLaunchKernelGGL(k_moe_gather, dim3(pairs, (m->Ep + 2047) / 2048), dim3(256), 0, st, (const bf16_t*)m->xb, m->mpos, L.moe_top, m->Ep, (bf16_t*)m->xg);
+  else hipLaunchKernelGGL(k_gather32, dim3(pairs, (m->Ep + 255) / 256), dim3(256), 0, st, (const float*)m->xb, m->mpos, L.moe_top, m->Ep, (float*)m->xg);
   LAUNCHCHK();
-  TRY(hglu<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu_limit, (T*)m->mhact, st));
+  TRY(hglu<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, l.glu_limit, (T*)m->mhact, st));
   return hdot_grouped<T>(c, (const T*)m->mhact, W.down, W.down_stride, rows_g, align, m->mrb, c->part, c->part_floats, st, out);
 }
 
@@ -573,7 +770,9 @@ static int hybrid_logits(ixt_ctx* c, int R, int lrow0, int nl, const int32_t* lr
   const int nblk = (m->V + 1023) / 1024;
   for (int i0 = 0; i0 < nl; i0 += c->NLmax) {
     const int n = std::min(c->NLmax, nl - i0);
-    hipLaunchKernelGGL((k_final_norm<T>), dim3(n), dim3(256), 0, st, m->x, lrows ? lrows + i0 : nullptr, lrow0 + i0, R, m->fnorm, m->eps, m->E, m->Ep, (T*)m->xn);
+#define HFINAL(KIND_) hipLaunchKernelGGL((k_final_norm<T, KIND_>), dim3(n), dim3(256), 0, st, m->x, lrows ? lrows + i0 : nullptr, lrow0 + i0, R, m->fnorm, m->eps, m->E, m->Ep, (T*)m->xn)
+    if (m->norm_kind == IXT_NORM_TANH) HFINAL(IXT_NORM_TANH); else HFINAL(IXT_NORM_RMS);
+#undef HFINAL
     LAUNCHCHK();
     Slices t;
     TRY(hdot<T>(c, (const T*)m->xn, m->head, n, c->part, c->part_floats, st, &t));
@@ -584,11 +783,15 @@ static int hybrid_logits(ixt_ctx* c, int R, int lrow0, int nl, const int32_t* lr
   return IXT_OK;
 }
 
+// x <- x + post(t), the next operand pre(x) (k_sub_norm); routed: its f32 copy too
 template <typename T>
-static int hybrid_norm(ixt_ctx* c, const Slices& t, const int32_t* pos, const float* wts, int top, const float* w, int R, hipStream_t st) {
+static int hybrid_norm(ixt_ctx* c, const Slices& t, const int32_t* pos, const float* wts, int top, const NormW& post, const NormW& pre, bool routed, int R, hipStream_t st) {
   HybridModel* m = c->hy;
-#define HNORM(NI_) hipLaunchKernelGGL((k_post_norm<T, NI_>), dim3(R), dim3(256), 0, st, t, pos, wts, top, w, m->eps, m->E, m->Ep, m->x, (T*)m->xb)
-  if (m->Ep <= 2048) HNORM(1); else if (m->Ep <= 4096) HNORM(2); else if (m->Ep <= 8192) HNORM(4); else HNORM(6);
+  float* h32 = routed && pre.w != nullptr ? m->h32 : nullptr;
+#define HNORM(NI_, KIND_) hipLaunchKernelGGL((k_sub_norm<T, NI_, KIND_>), dim3(R), dim3(256), 0, st, t, pos, wts, top, post, pre, m->eps, m->E, m->Ep, m->x, (T*)m->xb, h32)
+#define HNORM_K(NI_) do { if (m->norm_kind == IXT_NORM_TANH) HNORM(NI_, IXT_NORM_TANH); else HNORM(NI_, IXT_NORM_RMS); } while (0)
+  if (m->Ep <= 2048) HNORM_K(1); else if (m->Ep <= 4096) HNORM_K(2); else if (m->Ep <= 8192) HNORM_K(4); else HNORM_K(6);
+#undef HNORM_K
 #undef HNORM
   LAUNCHCHK();
   return IXT_OK;
@@ -599,29 +802,34 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
                                  int nseg_max, hipStream_t st) {
   HybridModel* m = c->hy;
   const int Rp = (sizeof(T) == 2 && R >= c->ring_min_rows) ? up_to(R, 128) : up_to(R, 16);
-  hipLaunchKernelGGL(k_segments, dim3(1), dim3(1024), 0, st, R, c->row_active, c->row_slot, c->row_pos, m->row_seg, m->row_j, m->seg, m->nseg, m->state_len, m->parity, m->claim, c->G,
+  if (m->recurrent || m->maxH > 0)
+    hipLaunchKernelGGL(k_segments, dim3(1), dim3(1024), 0, st, R, c->row_active, c->row_slot, c->row_pos, m->row_seg, m->row_j, m->seg, m->nseg, m->state_len, m->parity, m->claim, c->G,
                      m->recurrent ? 1 : 0, m->err, m->head_rb, m->maxH * (Rp / 16), Rp / 16);
-  hipLaunchKernelGGL((k_embed_scaled<T>), dim3(R), dim3(256), 0, st, (const T*)m->embed, tokens, m->emb_scale, m->E, m->Ep, m->V, m->x, (T*)m->xb);
+  const NormW none{}, first = m->layers[m->layers[0].src].n1;
+  hipLaunchKernelGGL((k_embed_scaled<T>), dim3(R), dim3(256), 0, st, (const T*)m->embed, tokens, m->emb_scale, m->E, m->Ep, m->V, m->norm_kind == IXT_NORM_TANH ? first : none, m->x, (T*)m->xb);
   LAUNCHCHK();
+  if (m->norm_kind == IXT_NORM_RMS && first.w != nullptr) TRY((hybrid_norm<T>(c, Slices{nullptr, 0, 0, 0}, nullptr, nullptr, 0, none, first, false, R, st)));
   for (size_t i = 0; i < m->layers.size(); ++i) {
     const HLayer& L = m->layers[i];
     const HLayer& W = m->layers[L.src];
     Slices t;
     if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) TRY((hybrid_mixer_latent<T>(c, L, W, R, Rp, decode, len_hint, st, &t)));
+    else if (L.c.mixer == IXT_MIX_ATTENTION) TRY((hybrid_mixer_heads<T>(c, L, W, R, decode, len_hint, st, &t)));
     else TRY((hybrid_mixer_delta<T>(c, L, W, R, nseg_max, decode, st, &t)));
-    TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n1, R, st)));
+    const NormW next = i + 1 < m->layers.size() ? m->layers[m->layers[i + 1].src].n1 : none;      // (the head's norm is taken of the wanted rows only)
+    TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n1b, L.c.ffn == IXT_FFN_NONE ? next : W.n2, L.c.ffn == IXT_FFN_MOE, R, st)));
     if (L.c.ffn == IXT_FFN_DENSE) {
-      TRY(hglu<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu_limit, (T*)m->hact, st));
+      TRY(hglu<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, L.c.glu_limit, (T*)m->hact, st));
       TRY(hdot<T>(c, (const T*)m->hact, W.down, R, c->part, c->part_floats, st, &t));
-      TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n2, R, st)));
+      TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n2b, next, false, R, st)));
     } else if (L.c.ffn == IXT_FFN_MOE) {
       TRY(hybrid_moe<T>(c, L, W, R, st, &t));
       if (t.n > 2 && R <= 64) {
-        hipLaunchKernelGGL(k_moe_sum, dim3((t.ncols + 255) / 256, R), dim3(64), 0, st, t, m->mpos, m->mw, L.c.top, m->msum);
+        hipLaunchKernelGGL(k_moe_sum, dim3((t.ncols + 255) / 256, R), dim3(64), 0, st, t, m->mpos, m->mw, L.moe_top, m->msum);
         LAUNCHCHK();
-        TRY((hybrid_norm<T>(c, Slices{m->msum, 1, 0, t.ncols}, nullptr, nullptr, 0, W.n2, R, st)));
+        TRY((hybrid_norm<T>(c, Slices{m->msum, 1, 0, t.ncols}, nullptr, nullptr, 0, W.n2b, next, false, R, st)));
       } else {
-        TRY((hybrid_norm<T>(c, t, m->mpos, m->mw, L.c.top, W.n2, R, st)));
+        TRY((hybrid_norm<T>(c, t, m->mpos, m->mw, L.moe_top, W.n2b, next, false, R, st)));
       }
     }
     if (m->tap && !c->capturing) {

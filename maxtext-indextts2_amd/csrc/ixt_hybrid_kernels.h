@@ -1,6 +1,6 @@
 // ixt_hybrid_kernels.h -- kernels of decoders whose layers are listed one by one (ixt_config.layers): each layer has a sequence mixer (latent
-// attention over a paged latent cache, or a gated delta rule with a recurrent state per page group), a feed-forward (a clamped gated unit, dense or
-// as a routed mixture) and norms on the sublayers' outputs only.
+// attention over a paged latent cache, a gated delta rule with a recurrent state per page group, or attention over keys and values per head:
+// ixt_heads_kernels.h), a feed-forward (a gated unit, dense or as a routed mixture) and norms in front of the sublayers, behind them, or both.
 //
 // Every kernel is a template over T, the storage of activations and cached keys: bf16_t (activations in the dot kernels' fragment order, xidx) or
 // float (row-major; the 32-bit mode).  The residual stream, norms, rotations, scores, routers and the recurrence are f32 in both.
@@ -116,17 +116,21 @@ static __global__ __launch_bounds__(256) void k_dot32(const float* __restrict__ 
 }
 
 // ---------------------------------------------------------------------------------------------------- weights
-// src [n][k] row-major ([out, in] linear weights) -> rows n of a dot operand of Kp k-columns, at (column n_off + n, k k_off + k).  inter: 16-column
-// tile j goes to tile 2 j + n_off (the two matrices of a gated unit side by side).  trans: src is [k][n].
+// src [n][k] row-major ([out, in] linear weights, rows `ld` apart) -> rows n of a dot operand of Kp k-columns, at (column n_off + n, k k_off + k).
+// inter: 16-column tile j goes to tile 2 j + n_off (the two matrices of a gated unit side by side).  trans: src is [k][n].  ng / kg > 0: groups of ng
+// columns (kg k) are laid ngp (kgp) apart, zeros between them.
+struct LoadMap { int n, k, ld, Kp, n_off, k_off, inter, trans, ng, ngp, kg, kgp; };
 template <typename S, typename T>
-__global__ void k_load_nk(const S* __restrict__ src, T* __restrict__ dst, int n, int k, int Kp, int n_off, int k_off, int inter, int trans) {
+__global__ void k_load_nk(const S* __restrict__ src, T* __restrict__ dst, LoadMap m) {
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= (int64_t)n * k) return;
-  const int nn = trans ? (int)(i % n) : (int)(i / k), kk = trans ? (int)(i / n) : (int)(i % k);
-  const int col = inter ? ((nn >> 4) * 2 + n_off) * 16 + (nn & 15) : n_off + nn;
-  const float v = to_f(src[i]);
-  if constexpr (sizeof(T) == 2) dst[widx(k_off + kk, col, Kp)] = f2bf(v);
-  else dst[(size_t)col * Kp + k_off + kk] = v;
+  if (i >= (int64_t)m.n * m.k) return;
+  int nn = m.trans ? (int)(i % m.n) : (int)(i / m.k), kk = m.trans ? (int)(i / m.n) : (int)(i % m.k);
+  const float v = to_f(src[m.trans ? (size_t)kk * m.ld + nn : (size_t)nn * m.ld + kk]);
+  if (m.ng > 0) nn = nn / m.ng * m.ngp + nn % m.ng;
+  if (m.kg > 0) kk = kk / m.kg * m.kgp + kk % m.kg;
+  const int col = m.inter ? ((nn >> 4) * 2 + m.n_off) * 16 + (nn & 15) : m.n_off + nn;
+  if constexpr (sizeof(T) == 2) dst[widx(m.k_off + kk, col, m.Kp)] = f2bf(v);
+  else dst[(size_t)col * m.Kp + m.k_off + kk] = v;
 }
 template <typename S, typename T>
 __global__ void k_load_vec(const S* __restrict__ src, T* __restrict__ dst, int64_t n) {
@@ -228,9 +232,31 @@ static __global__ __launch_bounds__(256) void k_latent_pages_copy(PageStateDev s
 }
 
 // ---------------------------------------------------------------------------------------------------- embedding, norms
-// x[r] = table[token] * scale (f32) and its copy as the first dot's operand.  grid R, block 256.
+// A norm's parameters (zeros behind feature E - 1); w null: no norm.  KIND IXT_NORM_RMS: t / sqrt(mean(t^2) + eps) (1 + w); IXT_NORM_TANH: feature by
+// feature tanh(alpha t) w + b.
+struct NormW { const float *w, *b, *alpha; };
+__device__ __forceinline__ void load8(const float* __restrict__ p, float* o) {       // p % 16 bytes == 0
+  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+  o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w; o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
+}
+// 8 features k0 .. k0 + 7 through a norm; s: the tanh norm's alpha, or the RMS norm's 1 / sqrt(mean + eps)
+template <int KIND>
+__device__ __forceinline__ void norm8(const NormW& n, float s, int k0, const float* t, float* o) {
+  float w[8], b[8];
+  load8(n.w + k0, w);
+  if constexpr (KIND == IXT_NORM_TANH) {
+    load8(n.b + k0, b);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = fmaf(ixt_tanh(s * t[j]), w[j], b[j]);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = t[j] * s * (1.0f + w[j]);
+  }
+}
+
+// x[r] = table[token] * scale (f32) and its copy as the first dot's operand, through a tanh norm if `pre` is one.  grid R, block 256.
 template <typename T>
-__global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ table, const int32_t* __restrict__ ids, float scale, int E, int Ep, int V, float* __restrict__ x,
+__global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ table, const int32_t* __restrict__ ids, float scale, int E, int Ep, int V, NormW pre, float* __restrict__ x,
                                                       T* __restrict__ xb) {
   const int r = blockIdx.x;
   const int id = min(max(ids[r], 0), V - 1);
@@ -241,16 +267,18 @@ __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ tabl
       v[j] = k0 + j < E ? to_f(table[(size_t)id * E + k0 + j]) * scale : 0.0f;
       if (k0 + j < E) x[(size_t)r * E + k0 + j] = v[j];
     }
+    if (pre.w != nullptr) norm8<IXT_NORM_TANH>(pre, *pre.alpha, k0, v, v);
     act_store8(xb, r, k0, Ep, v);
   }
 }
 
-// A sublayer's output t (slices, or the weighted sum of a row's expert outputs) -> RMS norm with a zero-centred weight -> residual:
-//   x <- x + t / sqrt(mean(t^2) + eps) * (1 + w);  xb = the new x as the next dot's operand.
-// pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  A thread owns 8 consecutive features of every 2048 (NI times).  grid R, block 256.
-template <typename T, int NI>
-__global__ __launch_bounds__(256) void k_post_norm(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, const float* __restrict__ w, float eps,
-                                                   int E, int Ep, float* __restrict__ x, T* __restrict__ xb) {
+// A sublayer's output t (slices, or the weighted sum of a row's expert outputs) -> norm behind the sublayer -> residual -> norm in front of the next one:
+//   x <- x + post(t);  xb = pre(x) as the next dot's operand, h32 (if given) the same in f32.
+// t.n == 0: t = 0 and x stays.  pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  A thread owns 8 consecutive features of every 2048 (NI
+// times).  grid R, block 256.
+template <typename T, int NI, int KIND>
+__global__ __launch_bounds__(256) void k_sub_norm(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, NormW post, NormW pre, float eps,
+                                                  int E, int Ep, float* __restrict__ x, T* __restrict__ xb, float* __restrict__ h32) {
   __shared__ float red[4];
   const int r = blockIdx.x;
   const bool vec = (E & 3) == 0;
@@ -265,7 +293,7 @@ __global__ __launch_bounds__(256) void k_post_norm(Slices t, const int32_t* __re
     for (int q = 0; q < 8; q += 4) {
       if (k0 + q >= E) continue;
       if (pos == nullptr) {
-        t.at4(r, k0 + q, v[i] + q);
+        if (t.n > 0) t.at4(r, k0 + q, v[i] + q);
       } else {
         for (int j = 0; j < top; ++j) {
           float u[4];
@@ -284,45 +312,77 @@ __global__ __launch_bounds__(256) void k_post_norm(Slices t, const int32_t* __re
           if (k0 + q + e < E) xv[i][q + e] = x[(size_t)r * E + k0 + q + e];
       }
     }
+    if constexpr (KIND == IXT_NORM_RMS) {
 #pragma unroll
-    for (int j = 0; j < 8; ++j)
-      if (k0 + j < E) ss = fmaf(v[i][j], v[i][j], ss);
+      for (int j = 0; j < 8; ++j)
+        if (k0 + j < E) ss = fmaf(v[i][j], v[i][j], ss);
+    }
   }
-  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+  float s_post = 0.0f, s_pre = 0.0f;
+  if constexpr (KIND == IXT_NORM_RMS) {
+    if (post.w != nullptr) s_post = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+  } else {
+    if (post.w != nullptr) s_post = *post.alpha;
+    if (pre.w != nullptr) s_pre = *pre.alpha;
+  }
+  ss = 0.0f;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int k0 = i * 2048 + threadIdx.x * 8;
     if (k0 >= Ep) continue;
-    float y[8];
+    if (t.n > 0 && post.w != nullptr) norm8<KIND>(post, s_post, k0, v[i], v[i]);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) y[j] = k0 + j < E ? xv[i][j] + v[i][j] * rs * (1.0f + w[k0 + j]) : 0.0f;
-    if (vec) {
+    for (int j = 0; j < 8; ++j) {
+      xv[i][j] = k0 + j < E ? xv[i][j] + v[i][j] : 0.0f;
+      if (KIND == IXT_NORM_RMS) ss = fmaf(xv[i][j], xv[i][j], ss);
+    }
+    if (t.n > 0) {
+      if (vec) {
 #pragma unroll
-      for (int q = 0; q < 8; q += 4)
-        if (k0 + q < E) *reinterpret_cast<float4*>(x + (size_t)r * E + k0 + q) = make_float4(y[q], y[q + 1], y[q + 2], y[q + 3]);
-    } else {
+        for (int q = 0; q < 8; q += 4)
+          if (k0 + q < E) *reinterpret_cast<float4*>(x + (size_t)r * E + k0 + q) = make_float4(xv[i][q], xv[i][q + 1], xv[i][q + 2], xv[i][q + 3]);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          if (k0 + j < E) x[(size_t)r * E + k0 + j] = xv[i][j];
+      }
+    }
+  }
+  if (KIND == IXT_NORM_RMS && pre.w != nullptr) s_pre = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int k0 = i * 2048 + threadIdx.x * 8;
+    if (k0 >= Ep) continue;
+    if (pre.w != nullptr) norm8<KIND>(pre, s_pre, k0, xv[i], xv[i]);      // (zeros behind feature E - 1: so are w and b there)
+    if (h32 != nullptr) {
 #pragma unroll
       for (int j = 0; j < 8; ++j)
-        if (k0 + j < E) x[(size_t)r * E + k0 + j] = y[j];
+        if (k0 + j < E) h32[(size_t)r * E + k0 + j] = xv[i][j];
     }
-    act_store8(xb, r, k0, Ep, y);
+    act_store8(xb, r, k0, Ep, xv[i]);
   }
 }
 
-// rows lrows[i] (or lrow0 + i) of x -> zero-centred RMS norm -> the head's operand.  grid nl, block 256.
-template <typename T>
-__global__ __launch_bounds__(256) void k_final_norm(const float* __restrict__ x, const int32_t* __restrict__ lrows, int lrow0, int nrows, const float* __restrict__ w, float eps,
-                                                    int E, int Ep, T* __restrict__ xn) {
+// rows lrows[i] (or lrow0 + i) of x -> the model's norm -> the head's operand.  grid nl, block 256.
+template <typename T, int KIND>
+__global__ __launch_bounds__(256) void k_final_norm(const float* __restrict__ x, const int32_t* __restrict__ lrows, int lrow0, int nrows, NormW w, float eps, int E, int Ep,
+                                                    T* __restrict__ xn) {
   __shared__ float red[4];
   const int i = blockIdx.x;
   const int r = min(max(lrows != nullptr ? lrows[i] : lrow0 + i, 0), nrows - 1);
-  float ss = 0.0f;
-  for (int k = threadIdx.x; k < E; k += 256) { const float v = x[(size_t)r * E + k]; ss = fmaf(v, v, ss); }
-  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+  float s;
+  if constexpr (KIND == IXT_NORM_RMS) {
+    float ss = 0.0f;
+    for (int k = threadIdx.x; k < E; k += 256) { const float v = x[(size_t)r * E + k]; ss = fmaf(v, v, ss); }
+    s = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+  } else {
+    s = *w.alpha;
+  }
   for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
     float v[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = k0 + j < E ? x[(size_t)r * E + k0 + j] * rs * (1.0f + w[k0 + j]) : 0.0f;
+    for (int j = 0; j < 8; ++j) v[j] = k0 + j < E ? x[(size_t)r * E + k0 + j] : 0.0f;
+    norm8<KIND>(w, s, k0, v, v);
     act_store8(xn, i, k0, Ep, v);
   }
 }
@@ -357,6 +417,85 @@ static __global__ __launch_bounds__(256) void k_head_post(Slices t, int V, ColRa
     amax_val[(size_t)r * gridDim.x + blockIdx.x] = best;
     amax_idx[(size_t)r * gridDim.x + blockIdx.x] = idx;
   }
+}
+
+// ---------------------------------------------------------------------------------------------------- tiles of cached rows
+// Tiles of 64 cached rows of D elements (D a multiple of 32) in LDS, for the matrix cores.  Groups of 8 pieces of 16 bytes (64 features), each [64 rows]
+// [8 pieces]; piece c of row r lies at place c ^ (r & 7), so that neither the score operand (16 rows x 16 bytes) nor the column-wise reads of the value
+// operand (ds_read_b64_tr_b16: 4 rows x 16 columns) pile up on a bank.  D an odd multiple of 32: a last group of 4 pieces, [64 rows][4 pieces], place
+// c ^ (r & 3).  A wave load (1 KiB) is 8 rows of a group (16 of the last), so all its addresses are two (three) row pointers plus constants.
+// 64 cached rows -> LDS: `off` = the row that this lane's key (key lane of the tile) occupies in the pool
+template <int D>
+__device__ __forceinline__ void tile_dma(const bf16_t* __restrict__ pages, int off, bf16_t* tile, int wave, int lane) {
+  constexpr int NG = D / 64;
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int o = __shfl(off, (wave + 4 * j) * 8 + (lane >> 3), 64);
+    const bf16_t* src = pages + (size_t)o * D + ((lane & 7) ^ (lane >> 3)) * 8;
+#pragma unroll
+    for (int gr = 0; gr < NG; ++gr)
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + gr * 64),
+                                       (__attribute__((address_space(3))) void*)(tile + gr * 4096 + (wave + 4 * j) * 512), 16, 0, 0);
+  }
+  if constexpr (D % 64 != 0) {
+    const int o = __shfl(off, wave * 16 + (lane >> 2), 64);
+    const bf16_t* src = pages + (size_t)o * D + NG * 64 + ((lane & 3) ^ ((lane >> 2) & 3)) * 8;
+    __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src, (__attribute__((address_space(3))) void*)(tile + NG * 4096 + wave * 512), 16, 0, 0);
+  }
+}
+__device__ __forceinline__ int cached_row(const int32_t* __restrict__ prow, int key, int pshift) { return (prow[key >> pshift] << pshift) + (key & ((1 << pshift) - 1)); }
+// where a lane reads in a tile (byte offsets; the rest of every address is a constant)
+struct TileLane {
+  uint32_t k0, k1, kh;      // score operand: row r_in, even / odd steps of a full group, the half group
+  uint32_t v[4];            // value operand: row 4 q + a, column tiles 0 .. 3 of a group (lane 4 a + p of a 16-lane group: columns 4 p .. 4 p + 3)
+  uint32_t vh[2];           // the same, column tiles 0 and 1 of the half group
+};
+__device__ __forceinline__ TileLane tile_lane(int r_in, int cq) {
+  TileLane L;
+  L.k0 = r_in * 128 + ((cq ^ (r_in & 7)) * 16);
+  L.k1 = r_in * 128 + (((4 + cq) ^ (r_in & 7)) * 16);
+  L.kh = r_in * 64 + ((cq ^ (r_in & 3)) * 16);
+  const int row = 4 * cq + (r_in >> 2), p = r_in & 3;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) L.v[i] = row * 128 + (((2 * i + (p >> 1)) ^ (row & 7)) * 16) + (p & 1) * 8;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) L.vh[i] = row * 64 + (((2 * i + (p >> 1)) ^ (row & 3)) * 16) + (p & 1) * 8;
+  return L;
+}
+// score operand of step ks, rows 16 n .. 16 n + 15
+template <int D>
+__device__ __forceinline__ bf16x8 tile_kf(const char* tile, const TileLane& L, int ks, int n) {
+  if (D % 64 != 0 && ks == D / 64 * 2) return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + L.kh + D / 64 * 8192 + n * 1024));
+  return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + ((ks & 1) ? L.k1 : L.k0) + (ks >> 1) * 8192 + n * 2048));
+}
+// value operand of column tiles 4 G .. 4 G + 3 (group G), keys 32 U + 4 q .. + 3 and 32 U + 16 + 4 q .. + 3 for lane group q; tb = LDS address of the tile
+#define IXT_TILE_VT(F_, TB_, L_, G_, U_)                                                                                                                    \
+  do {                                                                                                                                                        \
+    _Pragma("unroll") for (int i_ = 0; i_ < 4; ++i_) {                                                                                                        \
+      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][0]) : "v"((TB_) + (L_).v[i_]), "n"((G_) * 8192 + (U_) * 4096) : "memory");              \
+      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][1]) : "v"((TB_) + (L_).v[i_]), "n"((G_) * 8192 + (U_) * 4096 + 2048) : "memory");       \
+    }                                                                                                                                                         \
+  } while (0)
+// the two column tiles of the half group G
+#define IXT_TILE_VTH(F_, TB_, L_, G_, U_)                                                                                                                     \
+  do {                                                                                                                                                        \
+    _Pragma("unroll") for (int i_ = 0; i_ < 2; ++i_) {                                                                                                        \
+      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][0]) : "v"((TB_) + (L_).vh[i_]), "n"((G_) * 8192 + (U_) * 2048) : "memory");             \
+      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][1]) : "v"((TB_) + (L_).vh[i_]), "n"((G_) * 8192 + (U_) * 2048 + 1024) : "memory");      \
+    }                                                                                                                                                         \
+  } while (0)
+// all but the youngest N_ reads have been delivered: everything that uses the NF_ operands F_ comes behind this
+#define IXT_TILE_VWAITN(F_, NF_, N_)                                                                                                                          \
+  do {                                                                                                                                                        \
+    asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(N_) : "memory");                                                                                               \
+    __builtin_amdgcn_sched_barrier(0);                                                                                                                        \
+    _Pragma("unroll") for (int i_ = 0; i_ < (NF_); ++i_) asm volatile("" : "+v"(F_[i_][0]), "+v"(F_[i_][1]));                                                  \
+  } while (0)
+#define IXT_TILE_VWAIT(F_, N_) IXT_TILE_VWAITN(F_, 4, N_)
+__device__ __forceinline__ uint32_t lds_addr(const void* p) { return (uint32_t)(uintptr_t)((const __attribute__((address_space(3))) void*)(p)); }
+__device__ __forceinline__ bf16x8 tile_vfrag(const uint2 (&f)[2]) {
+  u32x4 v; v.x = f[0].x; v.y = f[0].y; v.z = f[1].x; v.w = f[1].y;
+  return __builtin_bit_cast(bf16x8, v);
 }
 
 // ---------------------------------------------------------------------------------------------------- latent attention
@@ -475,9 +614,7 @@ __global__ __launch_bounds__(256) void k_latent_attn_any(Slices qa, const T* __r
 }
 
 // The bf16 matrix-core forms.  All heads of a row share the cached latent, so the M side of the products is (row, head) pairs and every cached row is
-// read once for all of them.  Keys come in tiles of 64 by LDS-DMA (no registers in between); inside a group of 8 pieces of 16 bytes a row's pieces
-// are XORed with the row number, so that neither the score operand (16 rows x 16 bytes) nor the column-wise reads of the value operand
-// (ds_read_b64_tr_b16: 4 rows x 16 columns) pile up on a bank.
+// read once for all of them.  Keys come in tiles of 64 by LDS-DMA (no registers in between).
 //   scores   D[key][pair] = mfma(A = cached rows, B = queries [latent | rotated]): a lane holds 4 keys of one pair per product
 //   weights  running maximum / sum per pair in f32, exp2; P goes to bf16
 //   output   D[column][pair] = mfma(A = cached latent read column-wise, B = P)
@@ -490,34 +627,11 @@ struct LatentAttnArgs {
   bf16_t* out; int Kp;                     // act, row h Rp + r
   float *part_o, *part_ml;                 // splits > 1: [R H][splits][rankp], [R H][splits][2]
 };
-// A tile in LDS: groups of 8 pieces (64 features), each [64 rows][8 pieces]; piece c of row r lies at place c ^ (r & 7).  RS odd: a last group of 4 pieces,
-// [64 rows][4 pieces], place c ^ (r & 3).  A wave load (1 KiB) is 8 rows of a group (16 of the last), so all its addresses are two (three) row pointers
-// plus constants.
 template <int RT, int RS> struct LatentTile {
   static_assert(RT % 4 == 0 && (RS == 1 || RS == 2), "whole groups of the latent; one group or half a group of the rotated part");
-  static constexpr int DK = RT * 16 + RS * 32, NKS = RT / 2 + RS, NG = DK / 64;                 // elements per row, score steps, full groups
+  static constexpr int DK = RT * 16 + RS * 32, NKS = RT / 2 + RS;                               // elements per row, score steps
   static constexpr int BYTES = 64 * DK * 2;
 };
-// 64 cached rows -> LDS: `off` = the row that this lane's key (key lane of the tile) occupies in the pool
-template <int RT, int RS>
-__device__ __forceinline__ void latent_dma(const bf16_t* __restrict__ pages, int off, bf16_t* tile, int wave, int lane) {
-  typedef LatentTile<RT, RS> T;
-#pragma unroll
-  for (int j = 0; j < 2; ++j) {
-    const int o = __shfl(off, (wave + 4 * j) * 8 + (lane >> 3), 64);
-    const bf16_t* src = pages + (size_t)o * T::DK + ((lane & 7) ^ (lane >> 3)) * 8;
-#pragma unroll
-    for (int gr = 0; gr < T::NG; ++gr)
-      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + gr * 64),
-                                       (__attribute__((address_space(3))) void*)(tile + gr * 4096 + (wave + 4 * j) * 512), 16, 0, 0);
-  }
-  if constexpr (RS == 1) {
-    const int o = __shfl(off, wave * 16 + (lane >> 2), 64);
-    const bf16_t* src = pages + (size_t)o * T::DK + T::NG * 64 + ((lane & 3) ^ ((lane >> 2) & 3)) * 8;
-    __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src, (__attribute__((address_space(3))) void*)(tile + T::NG * 4096 + wave * 512), 16, 0, 0);
-  }
-}
-__device__ __forceinline__ int latent_row(const int32_t* __restrict__ prow, int key, int pshift) { return (prow[key >> pshift] << pshift) + (key & ((1 << pshift) - 1)); }
 __device__ __forceinline__ bf16x8 latent_q8(const LatentAttnArgs& a, int qrow, int c) {
   float v[8];
   a.qa.at4(qrow, c, v);
@@ -526,48 +640,6 @@ __device__ __forceinline__ bf16x8 latent_q8(const LatentAttnArgs& a, int qrow, i
   o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3])); o.z = pack2(f2bf(v[4]), f2bf(v[5])); o.w = pack2(f2bf(v[6]), f2bf(v[7]));
   return __builtin_bit_cast(bf16x8, o);
 }
-// where a lane reads in a tile (byte offsets; the rest of every address is a constant)
-struct LatentLane {
-  uint32_t k0, k1, kh;      // score operand: row r_in, even / odd steps of a full group, the half group
-  uint32_t v[4];            // value operand: row 4 q + a, column tiles 0 .. 3 of a group (lane 4 a + p of a 16-lane group: columns 4 p .. 4 p + 3)
-};
-__device__ __forceinline__ LatentLane latent_lane(int r_in, int cq) {
-  LatentLane L;
-  L.k0 = r_in * 128 + ((cq ^ (r_in & 7)) * 16);
-  L.k1 = r_in * 128 + (((4 + cq) ^ (r_in & 7)) * 16);
-  L.kh = r_in * 64 + ((cq ^ (r_in & 3)) * 16);
-  const int row = 4 * cq + (r_in >> 2), p = r_in & 3;
-#pragma unroll
-  for (int i = 0; i < 4; ++i) L.v[i] = row * 128 + (((2 * i + (p >> 1)) ^ (row & 7)) * 16) + (p & 1) * 8;
-  return L;
-}
-// score operand of step ks, rows 16 n .. 16 n + 15
-template <int RT, int RS>
-__device__ __forceinline__ bf16x8 latent_kf(const char* tile, const LatentLane& L, int ks, int n) {
-  if (RS == 1 && ks == RT / 2) return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + L.kh + LatentTile<RT, RS>::NG * 8192 + n * 1024));
-  return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(tile + ((ks & 1) ? L.k1 : L.k0) + (ks >> 1) * 8192 + n * 2048));
-}
-// value operand of column tiles 4 G .. 4 G + 3 (group G), keys 32 U + 4 q .. + 3 and 32 U + 16 + 4 q .. + 3 for lane group q; tb = LDS address of the tile
-#define IXT_LATENT_VT(F_, TB_, L_, G_, U_)                                                                                                                    \
-  do {                                                                                                                                                        \
-    _Pragma("unroll") for (int i_ = 0; i_ < 4; ++i_) {                                                                                                        \
-      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][0]) : "v"((TB_) + (L_).v[i_]), "n"((G_) * 8192 + (U_) * 4096) : "memory");              \
-      asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(F_[i_][1]) : "v"((TB_) + (L_).v[i_]), "n"((G_) * 8192 + (U_) * 4096 + 2048) : "memory");       \
-    }                                                                                                                                                         \
-  } while (0)
-// all but the youngest N_ reads have been delivered: everything that uses F_ comes behind this
-#define IXT_LATENT_VWAIT(F_, N_)                                                                                                                                \
-  do {                                                                                                                                                        \
-    asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(N_) : "memory");                                                                                               \
-    __builtin_amdgcn_sched_barrier(0);                                                                                                                        \
-    _Pragma("unroll") for (int i_ = 0; i_ < 4; ++i_) asm volatile("" : "+v"(F_[i_][0]), "+v"(F_[i_][1]));                                                      \
-  } while (0)
-__device__ __forceinline__ uint32_t lds_addr(const void* p) { return (uint32_t)(uintptr_t)((const __attribute__((address_space(3))) void*)(p)); }
-__device__ __forceinline__ bf16x8 latent_vfrag(const uint2 (&f)[2]) {
-  u32x4 v; v.x = f[0].x; v.y = f[0].y; v.z = f[1].x; v.w = f[1].y;
-  return __builtin_bit_cast(bf16x8, v);
-}
-
 // Prompts: a block owns 64 pairs = up to 64 / HB consecutive rows x HB heads (a wave 16 of them), all waves walk the same key tiles, the next tile
 // arriving while the current one is used.  P stays in registers: with the key order 4q .. 4q + 3, 16 + 4q .. 16 + 4q + 3 per lane group q of 32
 // keys, the lane's own scores ARE its operand of the next product.  grid (ceil(R / NQ), ceil(H / HB)), block 256, LDS two tiles.
@@ -594,7 +666,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentAttnArgs a) {
   for (int i = 0; i < RT; ++i) o[i] = f32x4(0.0f);
   float m = -INFINITY, l = 0.0f;
   const float sc = g.scale * 1.44269504088896340736f;
-  const LatentLane L = latent_lane(r_in, cq);
+  const TileLane L = tile_lane(r_in, cq);
   for (int ra = 0; ra < nr;) {                            // runs of rows that share a page group
     if (!a.row_active[r0 + ra]) { ++ra; continue; }
     const int slot = a.row_slot[r0 + ra];
@@ -607,28 +679,28 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentAttnArgs a) {
     const int32_t* prow = a.page_map + (size_t)slot * g.mpg;
     const int my_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
     __syncthreads();                                      // the previous run's last tile has been read
-    int off = latent_row(prow, min(k_lo + lane, hi), a.pshift);
-    latent_dma<RT, RS>(a.pages, off, lds, wave, lane);
-    off = latent_row(prow, min(k_lo + 64 + lane, hi), a.pshift);
+    int off = cached_row(prow, min(k_lo + lane, hi), a.pshift);
+    tile_dma<T::DK>(a.pages, off, lds, wave, lane);
+    off = cached_row(prow, min(k_lo + 64 + lane, hi), a.pshift);
     for (int t = 0; t < ntile; ++t) {
       const bf16_t* tile = lds + (size_t)(t & 1) * 64 * T::DK;
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
       __syncthreads();                                    // the tile is there; every wave is done with the other one
       if (t + 1 < ntile) {
-        latent_dma<RT, RS>(a.pages, off, lds + (size_t)((t + 1) & 1) * 64 * T::DK, wave, lane);
-        off = latent_row(prow, min(k_lo + (t + 2) * 64 + lane, hi), a.pshift);
+        tile_dma<T::DK>(a.pages, off, lds + (size_t)((t + 1) & 1) * 64 * T::DK, wave, lane);
+        off = cached_row(prow, min(k_lo + (t + 2) * 64 + lane, hi), a.pshift);
       }
       f32x4 s[4];
 #pragma unroll
       for (int n = 0; n < 4; ++n) s[n] = f32x4(0.0f);
       bf16x8 kf[2][4];                                    // operands one step ahead of the products
 #pragma unroll
-      for (int n = 0; n < 4; ++n) kf[0][n] = latent_kf<RT, RS>(reinterpret_cast<const char*>(tile), L, 0, n);
+      for (int n = 0; n < 4; ++n) kf[0][n] = tile_kf<T::DK>(reinterpret_cast<const char*>(tile), L, 0, n);
 #pragma unroll
       for (int ks = 0; ks < T::NKS; ++ks) {
         if (ks + 1 < T::NKS) {
 #pragma unroll
-          for (int n = 0; n < 4; ++n) kf[(ks + 1) & 1][n] = latent_kf<RT, RS>(reinterpret_cast<const char*>(tile), L, ks + 1, n);
+          for (int n = 0; n < 4; ++n) kf[(ks + 1) & 1][n] = tile_kf<T::DK>(reinterpret_cast<const char*>(tile), L, ks + 1, n);
         }
 #pragma unroll
         for (int n = 0; n < 4; ++n) s[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][n], qf[ks], s[n], 0, 0, 0);
@@ -669,17 +741,17 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentAttnArgs a) {
         pk.z = pack2(f2bf(s[2 * u + 1][0]), f2bf(s[2 * u + 1][1])); pk.w = pack2(f2bf(s[2 * u + 1][2]), f2bf(s[2 * u + 1][3]));
         const bf16x8 pf = __builtin_bit_cast(bf16x8, pk);
         uint2 f[2][4][2];
-        IXT_LATENT_VT(f[0], tb, L, 0, u);
+        IXT_TILE_VT(f[0], tb, L, 0, u);
 #pragma unroll
         for (int gr = 0; gr < RT / 4; ++gr) {             // the next group's reads travel under this one's products
           if (gr + 1 < RT / 4) {
-            IXT_LATENT_VT(f[(gr + 1) & 1], tb, L, gr + 1, u);
-            IXT_LATENT_VWAIT(f[gr & 1], 8);
+            IXT_TILE_VT(f[(gr + 1) & 1], tb, L, gr + 1, u);
+            IXT_TILE_VWAIT(f[gr & 1], 8);
           } else {
-            IXT_LATENT_VWAIT(f[gr & 1], 0);
+            IXT_TILE_VWAIT(f[gr & 1], 0);
           }
 #pragma unroll
-          for (int i = 0; i < 4; ++i) o[gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_vfrag(f[gr & 1][i]), pf, o[gr * 4 + i], 0, 0, 0);
+          for (int i = 0; i < 4; ++i) o[gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(f[gr & 1][i]), pf, o[gr * 4 + i], 0, 0, 0);
         }
       }
     }
@@ -715,7 +787,7 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
   const int32_t* prow = a.page_map + (size_t)slot * g.mpg;
   const int k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0, ntile = (pos - k_lo) / 64 + 1;
   int t = blockIdx.z;
-  if (t < ntile) latent_dma<RT, RS>(a.pages, latent_row(prow, min(k_lo + t * 64 + lane, pos), a.pshift), tile, wave, lane);
+  if (t < ntile) tile_dma<T::DK>(a.pages, cached_row(prow, min(k_lo + t * 64 + lane, pos), a.pshift), tile, wave, lane);
   bf16x8 qf[T::NKS];
 #pragma unroll
   for (int ks = 0; ks < RT / 2; ++ks) qf[ks] = latent_q8(a, head * a.Rp + row, ks * 32 + cq * 8);
@@ -727,18 +799,18 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
   for (int i = 0; i < OT; ++i) o[i] = f32x4(0.0f);
   float m = -INFINITY, l = 0.0f;                          // l: this lane's keys only
   const float sc = g.scale * 1.44269504088896340736f;
-  const LatentLane L = latent_lane(r_in, cq);
+  const TileLane L = tile_lane(r_in, cq);
   [[maybe_unused]] const uint32_t tb = lds_addr(tile) + wave * (OT / 4) * 8192;                              // the wave's first column group
   [[maybe_unused]] const uint32_t tg = lds_addr(tile) + (wave * OT / 4) * 8192;                              // fewer than 4 tiles per wave: the group they are in
   for (; t < ntile; t += nsplit) {
     int off = 0;
-    if (t + nsplit < ntile) off = latent_row(prow, min(k_lo + (t + nsplit) * 64 + lane, pos), a.pshift);
+    if (t + nsplit < ntile) off = cached_row(prow, min(k_lo + (t + nsplit) * 64 + lane, pos), a.pshift);
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
     f32x4 s = f32x4(0.0f);
 #pragma unroll
     for (int ks = 0; ks < T::NKS; ++ks) {
-      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_kf<RT, RS>(reinterpret_cast<const char*>(tile) + wave * (RS == 1 && ks == RT / 2 ? 1024 : 2048), L, ks, 0), qf[ks], s, 0, 0, 0);
+      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_kf<T::DK>(reinterpret_cast<const char*>(tile) + wave * (RS == 1 && ks == RT / 2 ? 1024 : 2048), L, ks, 0), qf[ks], s, 0, 0, 0);
     }
     float tm = -INFINITY;
 #pragma unroll
@@ -772,22 +844,22 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
       const bf16x8 pf = __builtin_bit_cast(bf16x8, pv);
       if constexpr (OT >= 4) {                            // whole column groups
         uint2 f[2][4][2];
-        IXT_LATENT_VT(f[0], tb, L, 0, u);
+        IXT_TILE_VT(f[0], tb, L, 0, u);
 #pragma unroll
         for (int gr = 0; gr < OT / 4; ++gr) {
           if (gr + 1 < OT / 4) {
-            IXT_LATENT_VT(f[(gr + 1) & 1], tb, L, gr + 1, u);
-            IXT_LATENT_VWAIT(f[gr & 1], 8);
+            IXT_TILE_VT(f[(gr + 1) & 1], tb, L, gr + 1, u);
+            IXT_TILE_VWAIT(f[gr & 1], 8);
           } else {
-            IXT_LATENT_VWAIT(f[gr & 1], 0);
+            IXT_TILE_VWAIT(f[gr & 1], 0);
           }
 #pragma unroll
-          for (int i = 0; i < 4; ++i) o[gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_vfrag(f[gr & 1][i]), pf, o[gr * 4 + i], 0, 0, 0);
+          for (int i = 0; i < 4; ++i) o[gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(f[gr & 1][i]), pf, o[gr * 4 + i], 0, 0, 0);
         }
       } else {                                            // OT column tiles, from place (wave OT) % 4 of one group on
         uint2 f[4][2];
-        IXT_LATENT_VT(f, tg, L, 0, u);
-        IXT_LATENT_VWAIT(f, 0);
+        IXT_TILE_VT(f, tg, L, 0, u);
+        IXT_TILE_VWAIT(f, 0);
         const int at = (wave * OT) & 3;
 #pragma unroll
         for (int i = 0; i < OT; ++i) {
@@ -798,12 +870,12 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
             x.x = take ? f[k + i][0].x : x.x; x.y = take ? f[k + i][0].y : x.y; y.x = take ? f[k + i][1].x : y.x; y.y = take ? f[k + i][1].y : y.y;
           }
           const uint2 xy[2] = {x, y};
-          o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(latent_vfrag(xy), pf, o[i], 0, 0, 0);
+          o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(xy), pf, o[i], 0, 0, 0);
         }
       }
     }
     __syncthreads();                                      // the tile has been read by every wave
-    if (t + nsplit < ntile) latent_dma<RT, RS>(a.pages, off, tile, wave, lane);
+    if (t + nsplit < ntile) tile_dma<T::DK>(a.pages, off, tile, wave, lane);
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
@@ -829,16 +901,11 @@ __global__ __launch_bounds__(256, 2) void k_latent_decode(LatentAttnArgs a) {
     if (wave == 0 && cq == 0) { a.part_ml[pi * 2] = m; a.part_ml[pi * 2 + 1] = l; }
   }
 }
-// the key splits of a row's heads put together.  grid (R, H), block 128; nsplit <= 16.
-static __global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int cols, int H, int Rp,
-                                                        const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
-  __shared__ float fac[16];
-  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
-  if (!row_active[r]) return;
-  const size_t p0 = ((size_t)r * H + h) * nsplit;
+// Key splits (<= 16) of one (row, head): ml = {maximum, sum} per split -> fac[s] = what split s's weighted sum counts for (threads 0 .. 63 work, all call)
+__device__ __forceinline__ void split_factors(const float* __restrict__ ml, int nsplit, int tid, float* fac /*[16] LDS*/) {
   if (tid < 64) {
     const int s = tid & 15;
-    const float ms = s < nsplit ? part_ml[(p0 + s) * 2] : -INFINITY, ls = s < nsplit ? part_ml[(p0 + s) * 2 + 1] : 0.0f;
+    const float ms = s < nsplit ? ml[s * 2] : -INFINITY, ls = s < nsplit ? ml[s * 2 + 1] : 0.0f;
     float mm = ms;
 #pragma unroll
     for (int off = 1; off < 16; off <<= 1) mm = fmaxf(mm, __shfl_xor(mm, off, 64));
@@ -847,20 +914,32 @@ static __global__ __launch_bounds__(128) void k_latent_combine(const float* __re
     if (tid < 16) fac[s] = f / ll;
   }
   __syncthreads();
+}
+// four columns of the weighted sums (cols apart per split) put together
+__device__ __forceinline__ void split_sum4(const float* __restrict__ o, int cols, int nsplit, const float* fac, float* v) {
+  v[0] = v[1] = v[2] = v[3] = 0.0f;
+  for (int s0 = 0; s0 < nsplit; s0 += 4) {
+    float4 u[4];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) u[s] = *reinterpret_cast<const float4*>(o + (size_t)min(s0 + s, nsplit - 1) * cols);
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      const float f = s0 + s < nsplit ? fac[s0 + s] : 0.0f;
+      if (f != 0.0f) { v[0] = fmaf(u[s].x, f, v[0]); v[1] = fmaf(u[s].y, f, v[1]); v[2] = fmaf(u[s].z, f, v[2]); v[3] = fmaf(u[s].w, f, v[3]); }
+    }
+  }
+}
+// the key splits of a row's heads put together.  grid (R, H), block 128; nsplit <= 16.
+static __global__ __launch_bounds__(128) void k_latent_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int cols, int H, int Rp,
+                                                        const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
+  __shared__ float fac[16];
+  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  if (!row_active[r]) return;
+  const size_t p0 = ((size_t)r * H + h) * nsplit;
+  split_factors(part_ml + p0 * 2, nsplit, tid, fac);
   for (int c = tid * 4; c < Kp; c += 512) {
     float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-    if (c < cols) {
-      for (int s0 = 0; s0 < nsplit; s0 += 4) {
-        float4 u[4];
-#pragma unroll
-        for (int s = 0; s < 4; ++s) u[s] = *reinterpret_cast<const float4*>(part_o + (p0 + min(s0 + s, nsplit - 1)) * cols + c);
-#pragma unroll
-        for (int s = 0; s < 4; ++s) {
-          const float f = s0 + s < nsplit ? fac[s0 + s] : 0.0f;
-          if (f != 0.0f) { v[0] = fmaf(u[s].x, f, v[0]); v[1] = fmaf(u[s].y, f, v[1]); v[2] = fmaf(u[s].z, f, v[2]); v[3] = fmaf(u[s].w, f, v[3]); }
-        }
-      }
-    }
+    if (c < cols) split_sum4(part_o + p0 * cols + c, cols, nsplit, fac, v);
     act_store4(out, h * Rp + r, c, Kp, v);
   }
 }
@@ -1211,29 +1290,76 @@ __global__ __launch_bounds__(256) void k_delta_out(const float* __restrict__ o, 
 }
 
 // ---------------------------------------------------------------------------------------------------- feed-forward
-// clamped gated unit from interleaved slices (tile 2 j gate, 2 j + 1 up): y = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up).
-// grid (ceil(Fp / 256), rows), block 256; rb_exp: rows of blocks without an expert are skipped.
+// gated unit (kind: IXT_GLU_*) from interleaved slices (tile 2 j gate, 2 j + 1 up).  grid (rows, ceil(Fp / 256)), block 256; rb_exp: rows of blocks
+// without an expert are skipped.
 template <typename T>
-__global__ __launch_bounds__(256) void k_glu_clamped(Slices t, int Fp, float limit, T* __restrict__ out, const int32_t* __restrict__ rb_exp) {
-  const int f = blockIdx.x * 256 + threadIdx.x, r = blockIdx.y;
+__global__ __launch_bounds__(256) void k_glu_slices(Slices t, int Fp, int kind, float limit, T* __restrict__ out, const int32_t* __restrict__ rb_exp) {
+  const int f = blockIdx.y * 256 + threadIdx.x, r = blockIdx.x;
   if (f >= Fp || (rb_exp != nullptr && rb_exp[r >> 4] < 0)) return;
   const int c = (f >> 4) * 32 + (f & 15);
-  act_store1(out, r, f, Fp, ixt_glu_clamped(t.at(r, c), t.at(r, c + 16), limit));
+  act_store1(out, r, f, Fp, ixt_glu(kind, t.at(r, c), t.at(r, c + 16), limit));
 }
 
-// softmax over all n logits of a row in f32, the `top` largest (first index on a tie), their scores as they are.  One wave; z in LDS or HBM.
-__device__ __forceinline__ void route_top(const float* z, int n, int top, int lane, int32_t* idx, float* wts) {
-  float v[16];
-  float mx = -INFINITY;
+// The choice of experts for a row.  IXT_ROUTE_SOFTMAX: scores s = softmax over all n logits; IXT_ROUTE_SIGMOID: s = sigmoid(z).  The `top` largest
+// s + corr (first index on a tie), inside the `keep` of `groups` equal groups of neighbours whose two largest s + corr add up to most; weights are the
+// picked s, divided by (their sum + 1e-20) if norm, times scale.  `shared` further experts n, n + 1, .. follow with weight 1.
+struct RouteRule { int n, top, kind, groups, keep, norm, shared; float scale; const float* corr; };
+// one wave; z [n] in LDS (overwritten: choice scores), gs [2 groups] in LDS; n <= 1024
+__device__ __forceinline__ void route_top(float* z, float* gs, const RouteRule& a, int lane, int32_t* idx, float* wts) {
+  const int n = a.n;
+  float v[16], mx = -INFINITY, sum = 1.0f;
 #pragma unroll
-  for (int i = 0; i < 16; ++i) { v[i] = lane + 64 * i < n ? z[lane + 64 * i] : -INFINITY; mx = fmaxf(mx, v[i]); }
+  for (int i = 0; i < 16; ++i) v[i] = lane + 64 * i < n ? z[lane + 64 * i] : -INFINITY;
+  if (a.kind == IXT_ROUTE_SOFTMAX) {
 #pragma unroll
-  for (int off = 1; off < 64; off <<= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
-  float sum = 0.0f;
+    for (int i = 0; i < 16; ++i) mx = fmaxf(mx, v[i]);
 #pragma unroll
-  for (int i = 0; i < 16; ++i) if (lane + 64 * i < n) sum += expf(v[i] - mx);
-  sum = wave_sum(sum);
-  for (int j = 0; j < top; ++j) {
+    for (int off = 1; off < 64; off <<= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
+    sum = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) if (lane + 64 * i < n) sum += expf(v[i] - mx);
+    sum = wave_sum(sum);
+  }
+  float s[16];                                             // scores; v becomes the choice scores
+#pragma unroll
+  for (int i = 0; i < 16; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = 0.0f;
+    if (e < n) {
+      s[i] = a.kind == IXT_ROUTE_SOFTMAX ? expf(v[i] - mx) / sum : f32_sigmoid(v[i]);
+      v[i] = a.corr != nullptr ? s[i] + a.corr[e] : s[i];
+    }
+  }
+  if (a.groups > 1) {                                      // closed groups: minus infinity
+    const int size = n / a.groups;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) if (lane + 64 * i < n) z[lane + 64 * i] = v[i];
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    for (int g = lane; g < a.groups; g += 64) {
+      float b1 = -INFINITY, b2 = -INFINITY;
+      for (int e = 0; e < size; ++e) {
+        const float c = z[g * size + e];
+        b2 = fmaxf(b2, fminf(b1, c));
+        b1 = fmaxf(b1, c);
+      }
+      gs[g] = size > 1 ? b1 + b2 : b1;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    for (int g = lane; g < a.groups; g += 64) {            // open if fewer than `keep` groups come before it
+      int before = 0;
+      for (int o = 0; o < a.groups; ++o) before += gs[o] > gs[g] || (gs[o] == gs[g] && o < g) ? 1 : 0;
+      gs[a.groups + g] = before < a.keep ? 1.0f : 0.0f;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < 16; ++i)
+      if (lane + 64 * i < n && gs[a.groups + (lane + 64 * i) / size] == 0.0f) v[i] = -INFINITY;
+  }
+  float total = 0.0f;
+  for (int j = 0; j < a.top; ++j) {
     float b = -INFINITY;
     int bi = 0x7fffffff;
 #pragma unroll
@@ -1245,19 +1371,27 @@ __device__ __forceinline__ void route_top(const float* z, int n, int top, int la
       const int oi = __shfl_xor(bi, off, 64);
       if (ob > b || (ob == b && oi < bi)) { b = ob; bi = oi; }
     }
-    if (bi >= n) bi = 0;                                   // only a row without finite logits gets here: any expert will do
+    if (bi >= n) bi = 0;                                   // only a row without finite scores gets here: any expert will do
+    float w = 0.0f;
 #pragma unroll
-    for (int i = 0; i < 16; ++i) if (lane + 64 * i == bi) v[i] = -INFINITY;
-    if (lane == 0) { idx[j] = bi; wts[j] = expf(b - mx) / sum; }
+    for (int i = 0; i < 16; ++i) if (lane + 64 * i == bi) { v[i] = -INFINITY; w = s[i]; }
+    w = __shfl(w, bi & 63, 64);
+    total += w;
+    if (lane == 0) { idx[j] = bi; wts[j] = w; }
   }
+  const float f = a.norm ? a.scale / (total + 1e-20f) : a.scale;
+  if (lane == 0 && (a.norm || a.scale != 1.0f))
+    for (int j = 0; j < a.top; ++j) wts[j] *= f;
+  for (int j = lane; j < a.shared; j += 64) { idx[a.top + j] = n + j; wts[a.top + j] = 1.0f; }
 }
 // router: logits (f32 residual x f32 weights) and choice of RB rows in one block, eight experts at a time: a thread takes every 256th feature of the RB
-// rows and the eight weight rows.  w [n][Ep]; grid ceil(R / RB), block 256, LDS RB n floats.
+// rows and the eight weight rows.  w [n][Ep]; grid ceil(R / RB), block 256, LDS RB (n + 2 groups) floats.
 template <int RB>
-__global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, const float* __restrict__ w, int E, int Ep, int n, int top, int R, int32_t* __restrict__ idx,
+__global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, const float* __restrict__ w, int E, int Ep, RouteRule rule, int R, int32_t* __restrict__ idx,
                                                float* __restrict__ wts) {
-  extern __shared__ __attribute__((aligned(16))) float z[];            // [RB][n]
+  extern __shared__ __attribute__((aligned(16))) float z[];            // [RB][n], [RB][2 groups]
   __shared__ float red[4][RB * 8];
+  const int n = rule.n, row = rule.top + rule.shared;
   const int r0 = blockIdx.x * RB, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const float* xr[RB];
 #pragma unroll
@@ -1295,7 +1429,7 @@ __global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, cons
     __syncthreads();
   }
   for (int i = wave; i < RB; i += 4)
-    if (r0 + i < R) route_top(z + (size_t)i * n, n, top, lane, idx + (size_t)(r0 + i) * top, wts + (size_t)(r0 + i) * top);
+    if (r0 + i < R) route_top(z + (size_t)i * n, z + (size_t)RB * n + i * 2 * rule.groups, rule, lane, idx + (size_t)(r0 + i) * row, wts + (size_t)(r0 + i) * row);
 }
 // any number of experts (<= 1024): destination row of every copy by one pass of counters; the order inside an expert is free.  One block of 1024.
 static __global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __restrict__ idx, int npairs, int n, int align, int nrb_cap, int32_t* __restrict__ pos, int32_t* __restrict__ rb_exp) {
@@ -1324,7 +1458,7 @@ static __global__ __launch_bounds__(1024) void k_moe_plan_any(const int32_t* __r
   for (int p = tid; p < npairs; p += 1024) pos[p] += off[idx[p]];
 }
 static __global__ __launch_bounds__(256) void k_gather32(const float* __restrict__ x, const int32_t* __restrict__ pos, int top, int Ep, float* __restrict__ xg) {
-  const int k = blockIdx.x * 256 + threadIdx.x, p = blockIdx.y;
+  const int k = blockIdx.y * 256 + threadIdx.x, p = blockIdx.x;
   if (k < Ep) xg[(size_t)pos[p] * Ep + k] = x[(size_t)(p / top) * Ep + k];
 }
 // few rows whose expert outputs lie in many split-K slices: the weighted sum of a row's copies as one slice.  grid (ceil(ncols / 256), R), block 64.

@@ -85,7 +85,7 @@ __host__ __device__ __forceinline__ int qk_col(int i, int half) {
 //   Routed experts (rb_exp != nullptr; NRB = 1): row block rb belongs to expert rb_exp[rb], whose kernels start wstride 16-byte units after
 //   wt; a row block of no expert (-1) leaves at once (k_moe_plan, ixt_moe_kernels.h).
 //   EPI = 1 (whole-K blocks only): the columns are interleaved (wi_0, wi_1) tiles (k_tile_w mode 2) and `out` is the bf16 activation buffer of the
-//   next dot (glu: the clamped gated unit of the f32 totals instead): the odd wave of a pair hands its totals to the even one through LDS, which writes bf16(bf16(a * bf16(sigmoid a)) * b) in the x layout
+//   next dot (glu: that gated unit of the f32 totals instead, ixt_glu): the odd wave of a pair hands its totals to the even one through LDS, which writes bf16(bf16(a * bf16(sigmoid a)) * b) in the x layout
 //   (linears.py:331-361) -- no f32 slice leaves the chip (routed experts at decode: 132 MB of slices per layer and the kernel that re-read them).
 template <int NRB, bool SPLIT, bool NT, int EPI = 0>
 __global__ __launch_bounds__(256, 2) void k_dotb(const u32x4* __restrict__ xt, const u32x4* __restrict__ wt, int K, int N, int R,
@@ -196,7 +196,7 @@ __global__ __launch_bounds__(256, 2) void k_dotb(const u32x4* __restrict__ xt, c
           const f32x4 up = ex[((wave >> 1) * NRB + b) * 64 + lane];
           bf16_t o[4];
 #pragma unroll
-          for (int j = 0; j < 4; ++j) o[j] = glu ? f2bf(ixt_glu_clamped(tot[b][j], up[j], glu_limit)) : ixt_swiglu(rbf(tot[b][j]), rbf(up[j]));
+          for (int j = 0; j < 4; ++j) o[j] = glu ? f2bf(ixt_glu(glu, tot[b][j], up[j], glu_limit)) : ixt_swiglu(rbf(tot[b][j]), rbf(up[j]));
           uint2 ov;
           ov.x = pack2(o[0], o[1]); ov.y = pack2(o[2], o[3]);
           *reinterpret_cast<uint2*>(act + xidx(row, f0, F)) = ov;

@@ -216,7 +216,7 @@ static __global__ __launch_bounds__(1024) void k_moe_plan(const int32_t* idx /*[
 
 // grid = (ceil(E / 2048), npairs), block 256: 8 consecutive features per thread.
 static __global__ __launch_bounds__(256) void k_moe_gather(const bf16_t* xn /*xidx, [R][E]*/, const int32_t* pos, int top_k, int E, bf16_t* xg /*xidx*/) {
-  const int k0 = (blockIdx.x * 256 + threadIdx.x) * 8, p = blockIdx.y;
+  const int k0 = (blockIdx.y * 256 + threadIdx.x) * 8, p = blockIdx.x;
   if (k0 >= E || pos[p] < 0) return;
   *reinterpret_cast<u32x4*>(xg + xidx(pos[p], k0, E)) = *reinterpret_cast<const u32x4*>(xn + xidx(p / top_k, k0, E));
 }

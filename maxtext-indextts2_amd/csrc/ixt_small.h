@@ -195,7 +195,7 @@ __global__ __launch_bounds__(1024) void k_sdot(SdotArgs a) {
       const int F = N >> 1, f0 = (tile >> 1) * 16 + cq * 4;
       bf16_t o[4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = a.e.glu ? f2bf(ixt_glu_clamped(tot[j], tot2[j], a.e.glu_limit)) : ixt_swiglu(rbf(tot[j]), rbf(tot2[j]));
+      for (int j = 0; j < 4; ++j) o[j] = a.e.glu ? f2bf(ixt_glu(a.e.glu, tot[j], tot2[j], a.e.glu_limit)) : ixt_swiglu(rbf(tot[j]), rbf(tot2[j]));
       uint2 ov;
       ov.x = pack2(o[0], o[1]); ov.y = pack2(o[2], o[3]);
       *reinterpret_cast<uint2*>(a.e.act + xidx(row, f0, F)) = ov;

@@ -109,6 +109,7 @@ class MaxEngine(engine_api.Engine):
           *[_lib.IxtLayer(**{n: getattr(l, n) for n in fields}) for l in config.hybrid_layers])
       c.layers, c.num_decoder_layers = self._hybrid_layers, len(config.hybrid_layers)
       c.embedding_scale, c.float32 = float(config.embedding_scale), 1 if config.dtype == "float32" else 0
+      c.norm_kind, c.norm_places = int(config.hybrid_norm_kind), int(config.hybrid_norm_places)
     elif config.dtype != "bfloat16":
       raise NotImplementedError(f"dtype {config.dtype}: only decoder_block hybrid runs in float32")
     elif config.decoder_block in ("gemma2", "gemma3"):   # layers/gemma2.py:69-236, layers/gemma3.py:35-200

@@ -200,8 +200,10 @@ def synth_weights_hybrid(cfg, seed: int = 0) -> Dict[str, np.ndarray]:
       z = z - np.float32(1.0)
     elif leaf == "conv":
       z = z * np.float32(1.0 / math.sqrt(shape[1]))
-    elif leaf in ("norm1", "norm2") or name == "final.norm":      # zero-centred
-      z = np.float32(0.1) * z
+    elif leaf in ("norm1", "norm2", "norm1b", "norm2b") or name == "final.norm":
+      z = np.float32(cfg.hybrid_norm_kind) + np.float32(0.1) * z  # zero-centred, or (tanh norms) plain
+    elif leaf in ("alpha", "b", "correction", "sink"):
+      z = np.float32(1.0 if leaf in ("alpha", "sink") else 0.0) + np.float32(0.1) * z
     elif leaf == "norm":                                          # plain
       z = np.float32(1.0) + np.float32(0.1) * z
     else:
@@ -291,7 +293,7 @@ def device_tree_spec(cfg):
   """[(tree path, shape, std or None for a norm scale)] of the configured block (llama2, gemma2, mixtral, hybrid)."""
   if getattr(cfg, "decoder_block", "llama2") == "hybrid":
     from . import architectures  # pylint: disable=import-outside-toplevel
-    std = lambda name, shape: (1 / cfg.embedding_scale if name == "embed" else 0.1 if "norm" in name else 0.5 if len(shape) == 1 else 1 / math.sqrt(shape[-1]))
+    std = lambda name, shape: (1 / cfg.embedding_scale if name == "embed" else None if name.endswith("alpha") else 0.1 if "norm" in name else 0.5 if len(shape) == 1 else 1 / math.sqrt(shape[-1]))
     return [(name, shape, std(name, shape)) for name, shape in architectures.parameter_shapes(cfg).items()]
   E, Q, KV, D, F, V = cfg.emb_dim, cfg.num_query_heads, cfg.num_kv_heads, cfg.head_dim, cfg.mlp_dim, cfg.vocab_size
   block = getattr(cfg, "decoder_block", "llama2")
