@@ -465,6 +465,7 @@ int hybrid_load_weight(ixt_ctx* c, const std::string& name, const void* src, int
   HTensor& t = it->second;
   bool same = ndim == (int)t.shape.size();
   for (int i = 0; same && i < ndim; ++i) same = shape[i] == t.shape[i];
+  if (t.shape.empty()) same = ndim == 0 || (ndim == 1 && shape[0] == 1);       // a scalar
   if (!same) {
     std::string want;
     for (int64_t v : t.shape) want += (want.empty() ? "" : " x ") + std::to_string(v);

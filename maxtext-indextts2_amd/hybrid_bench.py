@@ -1,6 +1,7 @@
-"""`bench.py --hybrid SIZES`: prefill and decode rates of Vilepel decoders (half latent attention, half gated delta rule) at layer sizes of real
-models, beside the closest model of the framework at the same width, head count, feed-forward and number of layers (the llama2 block, or Mixtral for
-the routed size).  Random weights drawn on the device, one GPU, both models in turn in one process.
+"""`bench.py --hybrid SIZES`: prefill and decode rates of hybrid decoders (Vilepel: half latent attention, half gated delta rule; Vazilorn: windowed
+attention with sinks and tanh norms) at layer sizes of real models, beside the closest model of the framework at the same width, head count,
+feed-forward and number of layers (the llama2 block, or Mixtral for the routed sizes).  Random weights drawn on the device, one GPU, both models in
+turn in one process.
 
 Per model: `prefill_packed` = 8 prompts of 256 tokens in one pass (2048 rows), `prefill_long` = one 4096-token prompt in 1024-row chunks,
 `decode_<slots>` = generate steps of that many slots at a context of about 1000 tokens.  Every figure is the best of three timed repetitions, each
@@ -39,7 +40,20 @@ def _model(width, pairs, latent, delta, mlp):
           "layers": [dict(l, mlp=mlp) for _ in range(pairs) for l in (delta, latent)]}
 
 
-# name -> (Vilepel config, keys of the closest model)
+def _heads(heads, kv_heads, window, dim=128):
+  return {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": window},
+                                         "rot": {"base": 500000.0, "dims": dim, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+
+
+def _vazilorn(width, layers, heads, mlp):
+  return {"architecture": "Vazilorn", "norm": {"eps": 1e-5}, "vocab": 32000, "width": width, "layers": [dict(heads, mlp=mlp) for _ in range(layers)]}
+
+
+def _grouped_moe(ff, experts, top, groups, keep, shared):
+  return {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": shared}, "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}, "scale": 2.5}}
+
+
+# name -> (config.json, keys of the closest model)
 SIZES = {
     "w1024": (_model(1024, 4, _latent(8, 256, 512, dim=64), _delta(8, 8), _dense(3584)),
               dict(base_emb_dim=1024, base_num_query_heads=8, base_num_kv_heads=8, base_mlp_dim=3584, base_num_decoder_layers=8)),
@@ -48,6 +62,13 @@ SIZES = {
     "w4096-moe": (_model(4096, 1, _latent(32, 512, 1024), _delta(32, 32), _moe(14336, 8, 2)),
                   dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=2, num_experts=8, num_experts_per_tok=2,
                        decoder_block="mixtral")),
+    "vazilorn-w1024": (_vazilorn(1024, 8, _heads(8, 8, 512), {"kind": "dense", "ff": 3584}),
+                       dict(base_emb_dim=1024, base_num_query_heads=8, base_num_kv_heads=8, base_mlp_dim=3584, base_num_decoder_layers=8)),
+    "vazilorn-w2048": (_vazilorn(2048, 8, _heads(16, 16, 1024), {"kind": "dense", "ff": 7168}),
+                       dict(base_emb_dim=2048, base_num_query_heads=16, base_num_kv_heads=16, base_mlp_dim=7168, base_num_decoder_layers=8)),
+    "vazilorn-w4096-moe": (_vazilorn(4096, 2, _heads(32, 8, 1024), _grouped_moe(14336, 8, 2, 4, 2, 2048)),
+                           dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=2, num_experts=8, num_experts_per_tok=2,
+                                decoder_block="mixtral")),
 }
 
 
@@ -130,16 +151,17 @@ def run(args) -> int:
   rows = {}
   for name in names:
     cfg_json, like = SIZES[name]
+    design = cfg_json["architecture"].lower()
     common = lambda slots: dict(attention="paged", scan_layers=False, per_device_batch_size=float(slots), max_prefill_predict_length=CHUNK, max_target_length=LONG + 32,
                                 pagedattn_tokens_per_page=32, pagedattn_num_pages=2 + max(slots * 34, LONG // 32 + 2 + PACK * PROMPT // 32 + 8), use_chunked_prefill=True,
                                 ixt_staging_groups=PACK, ixt_max_packed_rows=PROMPT * PACK, run_name="bench", ixt_use_hip_graph=not args.no_graph)
     with tempfile.TemporaryDirectory() as d:
       with open(os.path.join(d, "config.json"), "w", encoding="utf-8") as f:
         json.dump(cfg_json, f)
-      mine = _measure(lambda slots: pyconfig.initialize(["bench", base], ixt_model_dir=d, **common(slots)), slots_list, args.opt, lambda m: log(f"{name} vilepel {m}"))
+      mine = _measure(lambda slots: pyconfig.initialize(["bench", base], ixt_model_dir=d, **common(slots)), slots_list, args.opt, lambda m: log(f"{name} {design} {m}"))
     closest = _measure(lambda slots: pyconfig.initialize(["bench", base], vocab_size=32000, head_dim=128, **like, **common(slots)), slots_list, args.opt,
                        lambda m: log(f"{name} closest {m}"))
     time_of = lambda r: r.get("ms", r.get("ms_per_step"))
-    rows[name] = {"vilepel": mine, "closest": closest, "closest_model": like.get("decoder_block", "llama2"), "time_ratio": {k: time_of(mine[k]) / time_of(closest[k]) for k in mine}}
+    rows[name] = {design: mine, "closest": closest, "closest_model": like.get("decoder_block", "llama2"), "time_ratio": {k: time_of(mine[k]) / time_of(closest[k]) for k in mine}}
   print(json.dumps({"metric": "hybrid_decoder_rates", "data": "synthetic", "dtype": "bf16", "build_id": build.source_hash(), "rows": rows}), flush=True)
   return 0

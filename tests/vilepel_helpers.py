@@ -105,7 +105,7 @@ def write_model(path, cfg, weights):
   os.makedirs(path, exist_ok=True)
   with open(os.path.join(path, "config.json"), "w", encoding="utf-8") as f:
     json.dump(cfg, f)
-  save_file({k: torch.from_numpy(np.ascontiguousarray(v)).to(torch.bfloat16) for k, v in weights.items()}, os.path.join(path, "model.safetensors"))
+  save_file({k: torch.from_numpy(np.array(v, order="C")).to(torch.bfloat16) for k, v in weights.items()}, os.path.join(path, "model.safetensors"))
   return str(path)
 
 
