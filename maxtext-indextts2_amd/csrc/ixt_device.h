@@ -109,15 +109,24 @@ __device__ __forceinline__ bf16_t ixt_geglu(float a, float b) {
 }
 
 // gated units in f32, by kind (IXT_GLU_*).  1: g = min(a, limit), u = clamp(b, -limit, limit), g sigmoid(1.702 g) (u + 1); 2: tanh form of gelu, as
-// a sigmoid(2 sqrt(2 / pi) (a + 0.044715 a^3)) b; 3: a sigmoid(a) b
+// a sigmoid(2 sqrt(2 / pi) (a + 0.044715 a^3)) b; 3: a sigmoid(a) b (ixt_glu)
 __device__ __forceinline__ float ixt_glu_clamped(float a, float b, float limit) {
   const float g = fminf(a, limit), u = fminf(fmaxf(b, -limit), limit);
   return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
 }
+// 2^x and 1 / x of the hardware (1 ulp; results below the normal range go to zero)
+__device__ __forceinline__ float hw_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float hw_rcp(float x) { return __builtin_amdgcn_rcpf(x); }
 __device__ __forceinline__ float ixt_glu(int kind, float a, float b, float limit) {
   if (kind == 1) return ixt_glu_clamped(a, b, limit);
   const float z = kind == 2 ? 1.59576912160573071176f * fmaf(0.044715f * a * a, a, a) : a;
-  return a / (1.0f + expf(-z)) * b;
+  return a * hw_rcp(1.0f + hw_exp2(-1.44269504088896340736f * z)) * b;
+}
+// tanh in f32, error below 1e-6 of the value: (1 - e) / (1 + e), e = exp(-2 |x|); |x| < 1/16 by the odd series (next term < 2e-13 relative)
+__device__ __forceinline__ float tanh_f32(float x) {
+  const float a = fabsf(x), w = a * a, e = hw_exp2(-2.88539008177792681472f * a);
+  const float p = fmaf(fmaf(fmaf(-5.39682539682539682540e-2f, w, 1.33333333333333333333e-1f), w, -3.33333333333333333333e-1f), w, 1.0f);
+  return copysignf(a < 0.0625f ? a * p : (1.0f - e) * hw_rcp(1.0f + e), x);
 }
 
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));

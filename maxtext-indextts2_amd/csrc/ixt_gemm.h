@@ -22,12 +22,60 @@
 //   GEPI_RESID    h_out = bf16(h_in + bf16(t))                                   (llama2.py:127, :157)
 //   GEPI_SWIGLU   act = bf16(bf16(silu(bf16(t_0))) * bf16(t_1))                  (linears.py:449-464); the fused wi kernel stores
 //                 wi_0 tile j and wi_1 tile j as column tiles 2j, 2j+1, so both gates of a feature are in one wave
+//   GEPI_TANHNORM residual and norms of a decoder with tanh norms (TanhNormEpi)
 //   GEPI_QKV      bf16(t), RoPE (embeddings.py:277-315), q -> qbuf, k / v -> the row's page (paged_attention.py:446-471).  Q and K
 //                 head columns are stored pair-interleaved (qk_col): a 16-column tile holds features 8j..8j+7 and half+8j..half+8j+7,
 //                 so the two RoPE partners of a feature sit in lanes l and l ^ 32 of one accumulator register.
 #pragma once
 
-enum { GEPI_F32 = 0, GEPI_UNEMBED = 1, GEPI_RESID = 2, GEPI_SWIGLU = 3, GEPI_QKV = 4 };
+enum { GEPI_F32 = 0, GEPI_UNEMBED = 1, GEPI_RESID = 2, GEPI_SWIGLU = 3, GEPI_QKV = 4, GEPI_TANHNORM = 5 };
+
+// GEPI_TANHNORM: an f32 residual stream between tanh norms, x <- x + post(t), act = bf16(pre(x)), norm(y) = tanh(alpha y) w + b feature by feature (w
+// null: no norm).  Nothing in it looks at a row's other features, so it needs no launch of its own.
+struct TanhNormEpi {
+  const float *post_w, *post_b, *post_alpha, *pre_w, *pre_b, *pre_alpha;      // zeros behind feature E - 1
+  float *x, *h32;                                       // [R][E]; h32 (or nullptr): pre(x) in f32
+  int E, Ep;                                            // features, and the row length of `act`
+};
+// four columns of one row; col % 4 == 0, col + 3 < Ep
+__device__ __forceinline__ void tanhnorm_epi(const TanhNormEpi& n, bf16_t* act, int row, int col, const f32x4& t) {
+  float y[4] = {t[0], t[1], t[2], t[3]}, x[4];
+  const bool vec = (n.E & 3) == 0 && col < n.E;
+  float* xp = n.x + (size_t)row * n.E + col;
+  if (vec) { const float4 v = *reinterpret_cast<const float4*>(xp); x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w; }
+  else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) x[j] = col + j < n.E ? xp[j] : 0.0f;
+  }
+  if (n.post_w != nullptr) {
+    const float4 w = *reinterpret_cast<const float4*>(n.post_w + col), b = *reinterpret_cast<const float4*>(n.post_b + col);
+    const float al = *n.post_alpha;
+    y[0] = fmaf(tanh_f32(al * y[0]), w.x, b.x); y[1] = fmaf(tanh_f32(al * y[1]), w.y, b.y);
+    y[2] = fmaf(tanh_f32(al * y[2]), w.z, b.z); y[3] = fmaf(tanh_f32(al * y[3]), w.w, b.w);
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) x[j] += y[j];
+  if (vec) *reinterpret_cast<float4*>(xp) = make_float4(x[0], x[1], x[2], x[3]);
+  else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (col + j < n.E) xp[j] = x[j];
+  }
+  if (n.pre_w != nullptr) {
+    const float4 w = *reinterpret_cast<const float4*>(n.pre_w + col), b = *reinterpret_cast<const float4*>(n.pre_b + col);
+    const float al = *n.pre_alpha;
+    x[0] = fmaf(tanh_f32(al * x[0]), w.x, b.x); x[1] = fmaf(tanh_f32(al * x[1]), w.y, b.y);
+    x[2] = fmaf(tanh_f32(al * x[2]), w.z, b.z); x[3] = fmaf(tanh_f32(al * x[3]), w.w, b.w);
+  }
+  if (n.h32 != nullptr) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (col + j < n.E) n.h32[(size_t)row * n.E + col + j] = x[j];
+  }
+  uint2 o;
+  o.x = pack2(f2bf(x[0]), f2bf(x[1])); o.y = pack2(f2bf(x[2]), f2bf(x[3]));
+  *reinterpret_cast<uint2*>(act + xidx(row, col, n.Ep)) = o;
+}
 
 struct GemmEpi {
   float* out;                                           // F32: [slices][R][N]; UNEMBED: rounded logits [R][N] or nullptr
@@ -40,6 +88,7 @@ struct GemmEpi {
   AttnGeom g;
   const float* xscale; const float* wscale;             // F8: activation scales [rows][chains], column scales [N] (ixt_fp8.h)
   size_t sstride;                                       // F8 + routed experts: floats between two experts' column scales
+  TanhNormEpi tn;                                       // TANHNORM (with act)
   int glu; float glu_limit;                             // SWIGLU: glu != 0 takes that gated unit of the f32 totals instead (ixt_glu)
   const int32_t* rb_exp; size_t wstride;                // routed experts: expert of every 16-row block (-1: none), 16-byte units between experts' kernels
 };
@@ -267,6 +316,16 @@ __global__ __launch_bounds__(WR * WC * 64, 2) void k_gemm_ring(const u32x4* __re
           ov.y = pack2(f2bf(bflo(hv.y) + rbf(tot[i][b][2])), f2bf(bfhi(hv.y) + rbf(tot[i][b][3])));
           *reinterpret_cast<uint2*>(e.h_out + o) = ov;
         }
+      }
+    }
+  } else if constexpr (EPI == GEPI_TANHNORM) {
+#pragma unroll
+    for (int i = 0; i < CT; ++i) {
+      const int tile = colg * TC + wc * CT + i;
+#pragma unroll
+      for (int b = 0; b < RB; ++b) {
+        const int row = (rowg * TR + wr * RB + b) * 16 + r_in;
+        if (tile < ntile && row < R) tanhnorm_epi(e.tn, e.act, row, tile * 16 + cq * 4, tot[i][b]);
       }
     }
   } else if constexpr (EPI == GEPI_SWIGLU) {

@@ -19,44 +19,81 @@ struct HeadsGeom {
 };
 struct RowsArgs { const int32_t *slot, *pos, *active, *page_map; };      // the rows of a pass
 
-// A wave per head: queries and keys are normed (qn / kn; null: not) and rotated in f32, values copied.  rope: f32 [position][rot / 2] cos, sin.
-// grid (R, ceil((H + 2 G) / 4)), block 256.
-template <typename T>
-__global__ __launch_bounds__(256) void k_heads_prep(Slices t, HeadsGeom g, const float* __restrict__ qn, const float* __restrict__ kn, float eps, const float* __restrict__ rope_cos,
-                                                    const float* __restrict__ rope_sin, RowsArgs rows, T* __restrict__ kpages, T* __restrict__ vpages, T* __restrict__ q) {
-  const int r = blockIdx.x, j = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+// A query or key head (columns c0 .. of row r of the projection) by LP lanes, four features each at a time: norm by w (nullptr: none), rotation;
+// emit(f, o): features f .. f + 3 of the n asked for (zeros behind the head's own).  rope: f32 [position][rot / 2] cos, sin.
+struct HeadsRope { const float *cos, *sin; };
+template <int LP, typename F>
+__device__ __forceinline__ void head_norm_rotate(const Slices& t, int r, int c0, const HeadsGeom& g, const float* __restrict__ w, float eps, HeadsRope rope, int pos, int n, int sl, F emit) {
+  float v[4] = {0.0f, 0.0f, 0.0f, 0.0f}, rs = 1.0f;
+  if (sl * 4 < g.hs) t.at4(r, c0 + sl * 4, v);              // (columns d .. hs - 1 are zero)
+  if (w != nullptr) {
+    float ss = fmaf(v[0], v[0], fmaf(v[1], v[1], fmaf(v[2], v[2], v[3] * v[3])));
+    for (int f = (sl + LP) * 4; f < g.hs; f += 4 * LP) {
+      float u[4];
+      t.at4(r, c0 + f, u);
+      ss += fmaf(u[0], u[0], fmaf(u[1], u[1], fmaf(u[2], u[2], u[3] * u[3])));
+    }
+    ss = row16_sum(ss);
+#pragma unroll
+    for (int off = 16; off < LP; off <<= 1) ss += __shfl_xor(ss, off, 64);
+    rs = 1.0f / sqrtf(ss / (float)g.d + eps);
+  }
+  const int half = g.rot >> 1;
+  for (int f = sl * 4; f < n; f += 4 * LP) {
+    if (f != sl * 4) {
+      v[0] = v[1] = v[2] = v[3] = 0.0f;
+      if (f < g.hs) t.at4(r, c0 + f, v);
+    }
+    if (w != nullptr && f < g.hs) {                         // (the weight's tail is zero, too)
+      const float4 ww = *reinterpret_cast<const float4*>(w + f);
+      v[0] *= rs * ww.x; v[1] *= rs * ww.y; v[2] *= rs * ww.z; v[3] *= rs * ww.w;
+    }
+    float o[4] = {v[0], v[1], v[2], v[3]};
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int pr = f / 2 + i;
+      if (pr < half) {
+        const float c = rope.cos[(size_t)pos * half + pr], s = rope.sin[(size_t)pos * half + pr];
+        o[2 * i] = v[2 * i] * c - v[2 * i + 1] * s;
+        o[2 * i + 1] = v[2 * i + 1] * c + v[2 * i] * s;
+      }
+    }
+    emit(f, o);
+  }
+}
+__device__ __forceinline__ void store4(bf16_t* p, const float* v) {
+  uint2 o;
+  o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3]));
+  *reinterpret_cast<uint2*>(p) = o;
+}
+__device__ __forceinline__ void store4(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+
+// LP lanes per head (16, 32, 64): queries [R][H][dkp], and the row's keys and values in their pages.  grid (R, ceil((H + 2 G) LP / 256)), block 256.
+template <typename T, int LP>
+__global__ __launch_bounds__(256) void k_heads_prep(Slices t, HeadsGeom g, const float* __restrict__ qn, const float* __restrict__ kn, float eps, HeadsRope rope, RowsArgs rows,
+                                                    T* __restrict__ kpages, T* __restrict__ vpages, T* __restrict__ q) {
+  const int r = blockIdx.x, j = blockIdx.y * (256 / LP) + threadIdx.x / LP, sl = threadIdx.x % LP;
   if (j >= g.H + 2 * g.G) return;
   const bool act = rows.active[r] != 0;
   if (!act && j >= g.H) return;
   const int pos = act ? rows.pos[r] : 0;
-  const int page = act ? rows.page_map[(size_t)rows.slot[r] * g.mpg + pos / g.P] : 0;
-  const bool is_q = j < g.H;
-  const int kh = is_q ? 0 : (j - g.H) % g.G;
-  const size_t at = ((size_t)page * g.G + kh) * g.P + pos % g.P;          // row of the key / value pools
-  if (j >= g.H + g.G) {
-    T* v = vpages + at * g.dvp;
-    for (int c = lane; c < g.dv; c += 64) v[c] = from_f<T>(t.at(r, g.ov + kh * g.vs + c));
+  if (j < g.H) {
+    T* o = q + ((size_t)r * g.H + j) * g.dkp;
+    head_norm_rotate<LP>(t, r, j * g.hs, g, qn, eps, rope, pos, g.dkp, sl, [&](int f, const float* v) { store4(o + f, v); });
     return;
   }
-  const int c0 = is_q ? j * g.hs : g.ok + kh * g.hs;
-  const float* w = is_q ? qn : kn;
-  float rs = 1.0f;
-  if (w != nullptr) {
-    float ss = 0.0f;
-    for (int c = lane; c < g.d; c += 64) { const float v = t.at(r, c0 + c); ss = fmaf(v, v, ss); }
-    rs = 1.0f / sqrtf(wave_sum(ss) / (float)g.d + eps);
+  const int kh = (j - g.H) % g.G;
+  const size_t at = ((size_t)rows.page_map[(size_t)rows.slot[r] * g.mpg + pos / g.P] * g.G + kh) * g.P + pos % g.P;          // row of the key / value pools
+  if (j < g.H + g.G) {
+    T* o = kpages + at * g.dkp;
+    head_norm_rotate<LP>(t, r, g.ok + kh * g.hs, g, kn, eps, rope, pos, g.hs, sl, [&](int f, const float* v) { store4(o + f, v); });
+    return;
   }
-  T* o = is_q ? q + ((size_t)r * g.H + j) * g.dkp : kpages + at * g.dkp;
-  const int half = g.rot >> 1;
-  for (int i = lane; i < g.dkp / 2; i += 64) {
-    float u = 2 * i < g.d ? t.at(r, c0 + 2 * i) * rs : 0.0f, v = 2 * i + 1 < g.d ? t.at(r, c0 + 2 * i + 1) * rs : 0.0f;
-    if (w != nullptr) { u *= 2 * i < g.d ? w[2 * i] : 0.0f; v *= 2 * i + 1 < g.d ? w[2 * i + 1] : 0.0f; }
-    if (i < half) {
-      const float c = rope_cos[(size_t)pos * half + i], s = rope_sin[(size_t)pos * half + i], a = u;
-      u = a * c - v * s; v = v * c + a * s;
-    }
-    if constexpr (sizeof(T) == 2) *reinterpret_cast<uint32_t*>(o + 2 * i) = pack2(f2bf(u), f2bf(v));
-    else *reinterpret_cast<float2*>(o + 2 * i) = make_float2(u, v);
+  T* o = vpages + at * g.dvp;
+  for (int f = sl * 4; f < g.vs; f += 4 * LP) {
+    float v[4];
+    t.at4(r, g.ov + kh * g.vs + f, v);
+    store4(o + f, v);
   }
 }
 
@@ -125,12 +162,12 @@ __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, Hea
 struct HeadsAttnArgs {
   const bf16_t* q; HeadsGeom g; const float* sink;
   RowsArgs rows;
-  const bf16_t *kpages, *vpages;
+  bf16_t *kpages, *vpages;
   int R, NQ, HB, hchunks, pshift;           // rows per block, query heads per block, blocks of query heads per key / value head
   bf16_t* out; int Kp;                      // act, column h vs + c
   float *part_o, *part_ml;                  // splits > 1: [R H][splits][dvp], [R H][splits][2]
+  Slices t; const float *qn, *kn; float eps; HeadsRope rope;      // k_heads_decode with FUSED: the projection, and what k_heads_prep needs
 };
-__device__ __forceinline__ float heads_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
 // the pool row of a key: page (G heads) -> head -> token
 __device__ __forceinline__ int heads_row(const int32_t* __restrict__ prow, int key, int pshift, int G, int kh) {
   return ((prow[key >> pshift] * G + kh) << pshift) + (key & ((1 << pshift) - 1));
@@ -249,12 +286,12 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
         tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
         tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
         const float mn = fmaxf(m[p], tm), mz = mn == -INFINITY ? 0.0f : mn;
-        const float al = heads_exp2(m[p] - mz);           // (nothing seen so far: exp2(-inf) = 0, and l and o are 0)
+        const float al = hw_exp2(m[p] - mz);           // (nothing seen so far: exp2(-inf) = 0, and l and o are 0)
         float ls = 0.0f;
 #pragma unroll
         for (int n = 0; n < 4; ++n)
 #pragma unroll
-          for (int j = 0; j < 4; ++j) { s[p][n][j] = heads_exp2(fmaf(s[p][n][j], sc, -mz)); ls += s[p][n][j]; }
+          for (int j = 0; j < 4; ++j) { s[p][n][j] = hw_exp2(fmaf(s[p][n][j], sc, -mz)); ls += s[p][n][j]; }
         ls += __shfl_xor(ls, 16, 64);
         ls += __shfl_xor(ls, 32, 64);
         l[p] = l[p] * al + ls;
@@ -319,12 +356,15 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
 // Few rows (decode): a block owns up to 16 query heads of one key / value head of ONE row and every gridDim.z-th key tile of its window.  Scores: a wave
 // takes 16 of the 64 keys; P and the tile maxima meet in LDS; output: a wave takes every fourth column tile.  One tile of LDS: several blocks share a
 // CU and one's loads run under the other's products.  grid (R, G hchunks, splits), block 256.
-template <int DK, int DV>
+// FUSED (every row the only one of its page group): no k_heads_prep in front.  A block takes its queries from the projection while the first tile is on
+// its way; the block with the last tile also takes the row's key and value, keeps them for later passes in their pages and puts them into its tile.
+template <int DK, int DV, bool FUSED>
 __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
   constexpr int NKS = DK / 32, NGV = DV / 64, NH = DV % 64 != 0 ? 1 : 0, OT = NGV + NH;     // column tiles per wave: one of every full group, waves 0 and 1 one of the half group
   extern __shared__ __attribute__((aligned(16))) bf16_t tile[];
   __shared__ __attribute__((aligned(16))) bf16_t ps[16][72];
   __shared__ float s_m[4][16], s_l[4][16];
+  __shared__ __attribute__((aligned(16))) bf16_t s_q[FUSED ? 16 : 1][DK + 8], s_k[FUSED ? DK : 8], s_v[FUSED ? DV : 8];
   const HeadsGeom& g = a.g;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
   const int row = blockIdx.x, kh = blockIdx.y % g.G, hc = blockIdx.y / g.G, GQ = g.H / g.G, nsplit = gridDim.z;
@@ -342,8 +382,29 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     tile_dma<DV>(a.vpages, off, tile + 64 * DK, wave, lane);
   }
   bf16x8 qf[NKS];
+  [[maybe_unused]] const bool last = (ntile - 1) % nsplit == (int)blockIdx.z;       // the row's own key is in one of this block's tiles
+  if constexpr (FUSED) {
+    const size_t at = ((size_t)prow[pos >> a.pshift] * g.G + kh) * g.P + (pos & (g.P - 1));
+    for (int i = wave; i < hb + (last ? 2 : 0); i += 4) {
+      if (i < hb) {
+        head_norm_rotate<64>(a.t, row, (h0 + i) * g.hs, g, a.qn, a.eps, a.rope, pos, DK, lane, [&](int f, const float* v) { store4(&s_q[i][f], v); });
+      } else if (i == hb) {
+        head_norm_rotate<64>(a.t, row, g.ok + kh * g.hs, g, a.kn, a.eps, a.rope, pos, DK, lane, [&](int f, const float* v) {
+          store4(&s_k[f], v);
+          if (hc == 0 && f < g.hs) store4(a.kpages + at * DK + f, v);
+        });
+      } else if (lane * 4 < DV) {
+        float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+        if (lane * 4 < g.vs) a.t.at4(row, g.ov + kh * g.vs + lane * 4, v);
+        store4(&s_v[lane * 4], v);
+        if (hc == 0 && lane * 4 < g.vs) store4(a.vpages + at * DV + lane * 4, v);
+      }
+    }
+    __syncthreads();
+  }
 #pragma unroll
-  for (int ks = 0; ks < NKS; ++ks) qf[ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.q + ((size_t)row * g.H + head) * DK + ks * 32 + cq * 8));
+  for (int ks = 0; ks < NKS; ++ks)
+    qf[ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(FUSED ? &s_q[pair_ok ? r_in : 0][ks * 32 + cq * 8] : a.q + ((size_t)row * g.H + head) * DK + ks * 32 + cq * 8));
   f32x4 o[OT];
 #pragma unroll
   for (int i = 0; i < OT; ++i) o[i] = f32x4(0.0f);
@@ -359,6 +420,12 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     if (t + nsplit < ntile) off = heads_row(prow, min(k_lo + (t + nsplit) * 64 + lane, pos), a.pshift, g.G, kh);
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
+    if (FUSED && last && t == ntile - 1) {                // over what the tile's load found in the page
+      const int rr = pos - k_lo - t * 64;
+      if (tid < DK / 8) tile_put<DK>(tile, rr, tid, *reinterpret_cast<const u32x4*>(&s_k[tid * 8]));
+      else if (tid >= 64 && tid < 64 + DV / 8) tile_put<DV>(tile + 64 * DK, rr, tid - 64, *reinterpret_cast<const u32x4*>(&s_v[(tid - 64) * 8]));
+      __syncthreads();
+    }
     f32x4 s = f32x4(0.0f);
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks)
@@ -374,10 +441,10 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     if (cq == 0) s_m[wave][r_in] = tm;
     __syncthreads();
     const float mn = fmaxf(m, fmaxf(fmaxf(s_m[0][r_in], s_m[1][r_in]), fmaxf(s_m[2][r_in], s_m[3][r_in])));   // (a tile has at least one visible key: finite)
-    const float al = heads_exp2(m - mn);
+    const float al = hw_exp2(m - mn);
     float p[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) p[j] = heads_exp2(s[j] - mn);
+    for (int j = 0; j < 4; ++j) p[j] = hw_exp2(s[j] - mn);
     l = l * al + ((p[0] + p[1]) + (p[2] + p[3]));
     m = mn;
     uint2 pk;

@@ -16,7 +16,7 @@ struct HLayer {
   int d_off = 0;                                 // latent layer: column of the latent in the input projection
   size_t uk_stride = 0, uv_stride = 0, gu_stride = 0, down_stride = 0;
   NormW n1{}, n1b{}, n2{}, n2b{};                // in front of / behind the mixer, in front of / behind the feed-forward
-  int moe_n = 0, moe_top = 0, moe_shared = 0;    // experts and picks per token with the shared unit counted as moe_shared experts that are always picked
+  HMat sgu, sdown;                               // a mixture's shared unit
   float *qn = nullptr, *kn = nullptr, *sink = nullptr, *corr = nullptr;
   float *cnorm = nullptr, *cq = nullptr, *ck = nullptr, *cv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *onorm = nullptr, *router = nullptr;
   const float *rope_cos = nullptr, *rope_sin = nullptr;
@@ -106,10 +106,6 @@ static int h_load_mat(const HybridModel* m, const void* src, int dtype, void* ds
   return m->f32 ? h_load_nk(src, dtype, (float*)dst, lm, st) : h_load_nk(src, dtype, (bf16_t*)dst, lm, st);
 }
 
-// The shared unit of a mixture is the sum of units over parts of its hidden features: it runs as further experts of the common padded size.
-static int moe_shared_parts(const ixt_layer& l) { return l.shared_ff > 0 ? (l.shared_ff + up_to(l.ff, IXT_KALIGN) - 1) / up_to(l.ff, IXT_KALIGN) : 0; }
-static int moe_experts(const ixt_layer& l) { return l.experts + moe_shared_parts(l); }
-
 int hybrid_check(const ixt_config& c) {
   if (!c.layers || c.num_decoder_layers < 1) return set_err(IXT_ERR_INVALID, "hybrid decoder: no layers");
   if (c.emb_dim < 1 || c.emb_dim > 12288 || c.vocab_size < 1) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: emb_dim %d (1 .. 12288), vocab_size %d", c.emb_dim, c.vocab_size);
@@ -134,8 +130,8 @@ int hybrid_check(const ixt_config& c) {
     } else return set_err(IXT_ERR_UNSUPPORTED, "layer %d: mixer %d", i, l.mixer);
     if (l.ffn != IXT_FFN_NONE && (l.glu < IXT_GLU_CLAMPED || l.glu > IXT_GLU_SILU)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: gated unit %d", i, l.glu);
     if (l.ffn == IXT_FFN_MOE) {
-      if (l.experts < 1 || l.top < 1 || l.top > l.experts || l.ff < 1 || l.shared_ff < 0 || moe_experts(l) > 1024)
-        return set_err(IXT_ERR_UNSUPPORTED, "layer %d: experts %d (with the shared unit's share 1 .. 1024), top %d", i, l.experts, l.top);
+      if (l.experts < 1 || l.experts > 1024 || l.top < 1 || l.top > l.experts || l.ff < 1 || l.shared_ff < 0)
+        return set_err(IXT_ERR_UNSUPPORTED, "layer %d: experts %d (1 .. 1024), top %d", i, l.experts, l.top);
       if (l.router != IXT_ROUTE_SOFTMAX && l.router != IXT_ROUTE_SIGMOID) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: router %d", i, l.router);
       if (l.groups > 1 && (l.experts % l.groups || l.groups_keep < 1 || l.groups_keep > l.groups || l.top > l.experts / l.groups * l.groups_keep))
         return set_err(IXT_ERR_INVALID, "layer %d: %d of %d groups of experts, top %d", i, l.groups_keep, l.groups, l.top);
@@ -174,7 +170,7 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
   const std::string p = "l" + std::to_string(i) + ".";
   auto add = [&](const std::string& name, std::vector<int64_t> shape, std::function<int(const void*, int, hipStream_t)> f) { m->tensors[p + name] = HTensor{std::move(shape), std::move(f), false}; };
   auto vec = [&](const std::string& name, float** dst, int64_t n, std::vector<int64_t> shape) -> int {
-    TRY(h_allocf(c, dst, (size_t)n));
+    TRY(h_allocf(c, dst, (size_t)up_to((int)n, 4)));
     float* d = *dst;
     add(name, std::move(shape), [d, n](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, d, n, st); });
     return IXT_OK;
@@ -258,36 +254,24 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
   }
   TRY(norm("norm2", m->norm_places & IXT_NORM_BEFORE ? &L.n2 : &L.n2b));
   if (both) TRY(norm("norm2b", &L.n2b));
-  const int Fp = up_to(l.ff, IXT_KALIGN), n = l.ffn == IXT_FFN_MOE ? L.moe_n : 1;
-  TRY(h_mat(c, &L.gu, E, 2 * Fp, n));
-  TRY(h_mat(c, &L.down, Fp, E, n));
+  auto unit = [&](const std::string& q, const HMat& gu, const HMat& down, int ff, size_t gu_off = 0, size_t down_off = 0) {
+    LoadMap gate = load_map(ff, E, gu.Kp), up = load_map(ff, E, gu.Kp, 1);
+    gate.inter = up.inter = 1;
+    mat_as(q + "gate", gu, gate, gu_off);
+    mat_as(q + "up", gu, up, gu_off);
+    mat_as(q + "down", down, load_map(E, ff, down.Kp), down_off);
+  };
+  const bool moe = l.ffn == IXT_FFN_MOE;
+  const int n = moe ? l.experts : 1;
+  TRY(h_mat(c, &L.gu, E, 2 * up_to(l.ff, IXT_KALIGN), n));
+  TRY(h_mat(c, &L.down, l.ff, E, n));
   L.gu_stride = (size_t)L.gu.Kp * L.gu.Np; L.down_stride = (size_t)L.down.Kp * L.down.Np;
-  LoadMap gate = load_map(l.ff, E, L.gu.Kp), up = load_map(l.ff, E, L.gu.Kp, 1);
-  gate.inter = up.inter = 1;
-  for (int e = 0; e < (l.ffn == IXT_FFN_MOE ? l.experts : 1); ++e) {
-    const std::string q = l.ffn == IXT_FFN_MOE ? "mlp.e" + std::to_string(e) + "." : "mlp.";
-    mat_as(q + "gate", L.gu, gate, e * L.gu_stride);
-    mat_as(q + "up", L.gu, up, e * L.gu_stride);
-    mat_as(q + "down", L.down, load_map(E, l.ff, L.down.Kp), e * L.down_stride);
-  }
-  if (l.ffn != IXT_FFN_MOE) return IXT_OK;
-  if (L.moe_shared > 0) {                                        // Fp hidden features per part
-    const HLayer* Lp = &L;
-    auto part = [&](const char* name, bool down, int n_off) {
-      std::vector<int64_t> shape = down ? std::vector<int64_t>{E, l.shared_ff} : std::vector<int64_t>{l.shared_ff, E};
-      add(std::string("mlp.shared.") + name, shape, [=](const void* s, int dt, hipStream_t st) {
-        const int ff = Lp->c.shared_ff;
-        for (int j = 0; j < Lp->moe_shared; ++j) {
-          const int w = std::min(Fp, ff - j * Fp), e = Lp->c.experts + j;
-          LoadMap lm = down ? load_map(E, w, Lp->down.Kp) : load_map(w, E, Lp->gu.Kp, n_off);
-          if (down) lm.ld = ff; else lm.inter = 1;
-          const size_t at = (size_t)j * Fp * (down ? 1 : E) * (dt == IXT_F32 ? 4 : 2);
-          TRY(h_load_mat(m, (const char*)s + at, dt, (char*)(down ? Lp->down.w : Lp->gu.w) + e * (down ? Lp->down_stride : Lp->gu_stride) * m->esz, lm, st));
-        }
-        return (int)IXT_OK;
-      });
-    };
-    part("gate", false, 0); part("up", false, 1); part("down", true, 0);
+  for (int e = 0; e < n; ++e) unit(moe ? "mlp.e" + std::to_string(e) + "." : "mlp.", L.gu, L.down, l.ff, e * L.gu_stride, e * L.down_stride);
+  if (!moe) return IXT_OK;
+  if (l.shared_ff > 0) {
+    TRY(h_mat(c, &L.sgu, E, 2 * up_to(l.shared_ff, IXT_KALIGN)));
+    TRY(h_mat(c, &L.sdown, l.shared_ff, E));
+    unit("mlp.shared.", L.sgu, L.sdown, l.shared_ff);
   }
   TRY(h_allocf(c, &L.router, (size_t)l.experts * m->Ep));
   float* d = L.router;
@@ -405,15 +389,20 @@ int hybrid_init(ixt_ctx* c) {
       if (m->f32) upd(part, (size_t)R * 2 * Fp);
       dotsz(Fp, up_to(m->E, 16));
     } else if (l.ffn == IXT_FFN_MOE) {
-      L.moe_shared = moe_shared_parts(l); L.moe_n = moe_experts(l); L.moe_top = l.top + L.moe_shared;
       const int Fp = up_to(l.ff, IXT_KALIGN);
-      if ((int64_t)R * L.moe_top > (1 << 24)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d rows x %d experts per token: smaller max_packed_rows / max_prefill_predict_length", i, R, L.moe_top);
-      const int pairs = R * L.moe_top, cap = std::max(up_to(pairs, 128) + 128 * std::min(L.moe_n, pairs), 64 + 16 * L.moe_n);
+      if ((int64_t)R * l.top > (1 << 24)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d rows x %d experts per token: smaller max_packed_rows / max_prefill_predict_length", i, R, l.top);
+      const int pairs = R * l.top, cap = std::max(up_to(pairs, 128) + 128 * std::min(l.experts, pairs), 64 + 16 * l.experts);
       m->moe_cap = std::max(m->moe_cap, cap);
       upd(xg_e, (size_t)cap * m->Ep); upd(mh_e, (size_t)cap * Fp); upd(mi, (size_t)pairs);
       upd(part, (size_t)cap * up_to(m->E, 16));
-      upd(part, (size_t)(64 + 16 * std::min(L.moe_n, 64)) * up_to(m->E, 16) * ((Fp + IXT_CHAIN - 1) / IXT_CHAIN));
+      upd(part, (size_t)(64 + 16 * std::min(l.experts, 64)) * up_to(m->E, 16) * ((Fp + IXT_CHAIN - 1) / IXT_CHAIN));
       if (m->f32) upd(part, (size_t)cap * 2 * Fp);
+      if (l.shared_ff > 0) {
+        const int Sp = up_to(l.shared_ff, IXT_KALIGN), N = up_to(m->E, 16);
+        upd(hact_k, Sp);
+        if (m->f32) upd(part, (size_t)R * 2 * Sp);
+        upd(part2, std::max((size_t)R * N, (size_t)std::min(R, 128) * N * ((Sp + IXT_CHAIN - 1) / IXT_CHAIN)));
+      }
       if (!m->h32 && (m->norm_places & IXT_NORM_BEFORE)) TRY(h_allocf(c, &m->h32, (size_t)R * m->E));
     }
   }
@@ -626,8 +615,9 @@ static int latent_attention(ixt_ctx* c, const HLayer& L, const Slices& qa, int R
   return IXT_OK;
 }
 
+// The mixers leave the operand of the output projection in m->act.
 template <typename T>
-static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int Rp, bool decode, int len_hint, hipStream_t st, Slices* out) {
+static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int Rp, bool decode, int len_hint, hipStream_t st) {
   HybridModel* m = c->hy;
   const LatentGeom& g = L.lg;
   Slices t;
@@ -640,7 +630,7 @@ static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int
   TRY(hdot_grouped<T>(c, (const T*)m->olat, W.uv, W.uv_stride, g.H * Rp, Rp, m->head_rb, c->part, c->part_floats, st, &t));
   hipLaunchKernelGGL((k_heads_x<T>), dim3(R, (W.o.Kp + 255) / 256), dim3(256), 0, st, t, g.H, L.c.vdim, Rp, (T*)m->act, W.o.Kp);
   LAUNCHCHK();
-  return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
+  return IXT_OK;
 }
 
 template <int DK, int DV, int MP>
@@ -658,29 +648,45 @@ static int heads_prompt_launch(HeadsAttnArgs a, hipStream_t st) {
   return IXT_OK;
 }
 template <int DK, int DV>
-static int heads_launch(bool tall, int splits, HeadsAttnArgs a, hipStream_t st) {
+static int heads_launch(bool tall, bool fused, int splits, HeadsAttnArgs a, hipStream_t st) {
   if (tall) return heads_prompt_launch<DK, DV, 1>(a, st);
-  hipLaunchKernelGGL((k_heads_decode<DK, DV>), dim3(a.R, a.g.G * a.hchunks, splits), dim3(256), 64 * (DK + DV) * 2, st, a);
+  const dim3 grid(a.R, a.g.G * a.hchunks, splits);
+  if (fused) hipLaunchKernelGGL((k_heads_decode<DK, DV, true>), grid, dim3(256), 64 * (DK + DV) * 2, st, a);
+  else hipLaunchKernelGGL((k_heads_decode<DK, DV, false>), grid, dim3(256), 64 * (DK + DV) * 2, st, a);
   LAUNCHCHK();
   return IXT_OK;
 }
-// queries over the paged keys and values -> act(T) of the output projection
 template <typename T>
-static int heads_attention(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, bool decode, int len_hint, hipStream_t st) {
+static int heads_prep(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& t, const HeadsRope& rope, const RowsArgs& rows, int R, hipStream_t st) {
+  HybridModel* m = c->hy;
+  const HeadsGeom& g = L.hg;
+  const int n = g.H + 2 * g.G, widest = std::max(g.dkp, g.vs);
+#define HPREP(LP_) hipLaunchKernelGGL((k_heads_prep<T, LP_>), dim3(R, (n * LP_ + 255) / 256), dim3(256), 0, st, t, g, W.qn, W.kn, m->eps, rope, rows, (T*)L.pages, (T*)L.vpages, (T*)m->qx)
+  if (widest <= 64) HPREP(16); else if (widest <= 128) HPREP(32); else HPREP(64);
+#undef HPREP
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <typename T>
+static int hybrid_mixer_heads(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, bool decode, int len_hint, hipStream_t st) {
   HybridModel* m = c->hy;
   const HeadsGeom& g = L.hg;
   const RowsArgs rows{c->row_slot, c->row_pos, c->row_active, c->ps.page_map};
+  const HeadsRope rope{L.rope_cos, L.rope_sin};
+  Slices t;
   int dkp = 0, dvp = 0;
+  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &t));
   if constexpr (sizeof(T) == 2) {
     if (heads_mfma_sizes(g.d, g.dv, m->f32, &dkp, &dvp)) {
       const bool tall = !decode && R > 32;
       const int GQ = g.H / g.G, hchunks = (GQ + 15) / 16, blocks = R * g.G * hchunks, span = g.window > 0 ? std::min(g.window, len_hint) : len_hint;
       int splits = 1;
       if (!tall) splits = std::min(std::min(16, std::max(1, IXT_HEADS_SPLIT_BLOCKS / blocks)), std::max(1, (span + 63) / 64));     // at least a tile each
-      HeadsAttnArgs a{(const bf16_t*)m->qx, g, W.sink, rows, (const bf16_t*)L.pages, (const bf16_t*)L.vpages, R, 1, (GQ + hchunks - 1) / hchunks, hchunks, __builtin_ctz(c->P),
-                      (bf16_t*)m->act, W.o.Kp, m->po, m->pml};
+      if (!decode) TRY((heads_prep<T>(c, L, W, t, rope, rows, R, st)));
+      HeadsAttnArgs a{(const bf16_t*)m->qx, g, W.sink, rows, (bf16_t*)L.pages, (bf16_t*)L.vpages, R, 1, (GQ + hchunks - 1) / hchunks, hchunks, __builtin_ctz(c->P),
+                      (bf16_t*)m->act, W.o.Kp, m->po, m->pml, t, W.qn, W.kn, m->eps, rope};
       int rc = IXT_ERR_UNSUPPORTED;
-#define X(DK_, DV_) if (dkp == DK_ && dvp == DV_) rc = heads_launch<DK_, DV_>(tall, splits, a, st);
+#define X(DK_, DV_) if (dkp == DK_ && dvp == DV_) rc = heads_launch<DK_, DV_>(tall, decode, splits, a, st);
       IXT_HEADS_SIZES(X)
 #undef X
       TRY(rc);
@@ -691,25 +697,14 @@ static int heads_attention(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, 
       return IXT_OK;
     }
   }
+  TRY((heads_prep<T>(c, L, W, t, rope, rows, R, st)));
   hipLaunchKernelGGL((k_heads_any<T>), dim3(R, g.H), dim3(256), sizeof(float) * (g.dkp + 256), st, (const T*)m->qx, g, W.sink, rows, (const T*)L.pages, (const T*)L.vpages, (T*)m->act, W.o.Kp);
   LAUNCHCHK();
   return IXT_OK;
 }
-template <typename T>
-static int hybrid_mixer_heads(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, bool decode, int len_hint, hipStream_t st, Slices* out) {
-  HybridModel* m = c->hy;
-  const HeadsGeom& g = L.hg;
-  Slices t;
-  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &t));
-  hipLaunchKernelGGL((k_heads_prep<T>), dim3(R, (g.H + 2 * g.G + 3) / 4), dim3(256), 0, st, t, g, W.qn, W.kn, m->eps, L.rope_cos, L.rope_sin,
-                     RowsArgs{c->row_slot, c->row_pos, c->row_active, c->ps.page_map}, (T*)L.pages, (T*)L.vpages, (T*)m->qx);
-  LAUNCHCHK();
-  TRY(heads_attention<T>(c, L, W, R, decode, len_hint, st));
-  return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
-}
 
 template <typename T>
-static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st, Slices* out) {
+static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st) {
   HybridModel* m = c->hy;
   const DeltaGeom& g = L.dg;
   Slices t, t2;
@@ -725,7 +720,7 @@ static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int 
     switch (g.dp / 16) { HSTEP(1); HSTEP(2); HSTEP(4); HSTEP(8); HSTEP(16); HSTEP(32); default: return set_err(IXT_ERR_UNSUPPORTED, "delta rule: %d key dims", g.d); }
 #undef HSTEP
     LAUNCHCHK();
-    return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
+    return IXT_OK;
   }
   DeltaPrepArgs pa{t, t2, g, W.cq, W.ck, W.cv, W.a_log, W.dt_bias, m->row_seg, m->row_j, m->seg, L.tails, m->dq, m->dk, m->dkq, m->dv, m->dec, m->beta};
   hipLaunchKernelGGL(k_delta_prep, dim3(R, (g.KH + g.H + 3) / 4), dim3(256), 0, st, pa);
@@ -738,16 +733,20 @@ static int hybrid_mixer_delta(ixt_ctx* c, const HLayer& L, const HLayer& W, int 
   LAUNCHCHK();
   hipLaunchKernelGGL((k_delta_out<T>), dim3(R, (g.H + 3) / 4), dim3(256), 0, st, m->dout, t2, g, W.onorm, m->eps, m->row_seg, (T*)m->act, W.o.Kp);
   LAUNCHCHK();
-  return hdot<T>(c, (const T*)m->act, W.o, R, c->part, c->part_floats, st, out);
+  return IXT_OK;
 }
 
-// routed mixture: expert outputs stay in copy order (slices `out`, row m->mpos[r moe_top + j], weight m->mw[r moe_top + j]); the norm kernel adds them up
+// routed mixture (and its shared unit: slices `shared`): expert outputs stay in copy order (slices `out`, row m->mpos[r top + j], weight m->mw[r top + j]); the norm kernel adds them up
 template <typename T>
-static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipStream_t st, Slices* out) {
+static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipStream_t st, Slices* out, Slices* shared) {
   HybridModel* m = c->hy;
   const ixt_layer& l = L.c;
-  const int pairs = R * L.moe_top, n = L.moe_n;
-  const RouteRule rule{l.experts, l.top, l.router, l.groups > 1 ? l.groups : 0, l.groups_keep, l.router_norm, L.moe_shared, l.router_scale, W.corr};
+  const int pairs = R * l.top, n = l.experts;
+  const RouteRule rule{l.experts, l.top, l.router, l.groups > 1 ? l.groups : 0, l.groups_keep, l.router_norm, l.router_scale, W.corr};
+  if (l.shared_ff > 0) {
+    TRY(hglu<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, l.glu_limit, (T*)m->hact, st));
+    TRY(hdot<T>(c, (const T*)m->hact, W.sdown, R, m->part2, m->part2_floats, st, shared));
+  }
   const float* h = (m->norm_places & IXT_NORM_BEFORE) ? m->h32 : m->x;
   const size_t lds = sizeof(float) * (l.experts + 2 * rule.groups);
   if (R <= 256) hipLaunchKernelGGL((k_route<1>), dim3(R), dim3(256), lds, st, h, W.router, m->E, m->Ep, rule, R, m->midx, m->mw);
@@ -757,8 +756,8 @@ static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipSt
   const int rows_g = up_to(pairs, align) + align * std::min(n, pairs);     // every expert with a copy may waste up to align - 1 rows
   if (rows_g > m->moe_cap) return set_err(IXT_ERR_INVALID, "moe: %d copies exceed the routed workspaces", pairs);
   hipLaunchKernelGGL(k_moe_plan_any, dim3(1), dim3(1024), 0, st, m->midx, pairs, n, align, rows_g / 16, m->mpos, m->mrb);
-  if constexpr (sizeof(T) == 2) hipLaunchKernelGGL(k_moe_gather, dim3(pairs, (m->Ep + 2047) / 2048), dim3(256), 0, st, (const bf16_t*)m->xb, m->mpos, L.moe_top, m->Ep, (bf16_t*)m->xg);
-  else hipLaunchKernelGGL(k_gather32, dim3(pairs, (m->Ep + 255) / 256), dim3(256), 0, st, (const float*)m->xb, m->mpos, L.moe_top, m->Ep, (float*)m->xg);
+  if constexpr (sizeof(T) == 2) hipLaunchKernelGGL(k_moe_gather, dim3(pairs, (m->Ep + 2047) / 2048), dim3(256), 0, st, (const bf16_t*)m->xb, m->mpos, l.top, m->Ep, (bf16_t*)m->xg);
+  else hipLaunchKernelGGL(k_gather32, dim3(pairs, (m->Ep + 255) / 256), dim3(256), 0, st, (const float*)m->xb, m->mpos, l.top, m->Ep, (float*)m->xg);
   LAUNCHCHK();
   TRY(hglu<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, l.glu_limit, (T*)m->mhact, st));
   return hdot_grouped<T>(c, (const T*)m->mhact, W.down, W.down_stride, rows_g, align, m->mrb, c->part, c->part_floats, st, out);
@@ -786,16 +785,36 @@ static int hybrid_logits(ixt_ctx* c, int R, int lrow0, int nl, const int32_t* lr
 
 // x <- x + post(t), the next operand pre(x) (k_sub_norm); routed: its f32 copy too
 template <typename T>
-static int hybrid_norm(ixt_ctx* c, const Slices& t, const int32_t* pos, const float* wts, int top, const NormW& post, const NormW& pre, bool routed, int R, hipStream_t st) {
+static int hybrid_norm(ixt_ctx* c, const Slices& t, const Slices& add, const int32_t* pos, const float* wts, int top, const NormW& post, const NormW& pre, bool routed, int R, hipStream_t st) {
   HybridModel* m = c->hy;
   float* h32 = routed && pre.w != nullptr ? m->h32 : nullptr;
-#define HNORM(NI_, KIND_) hipLaunchKernelGGL((k_sub_norm<T, NI_, KIND_>), dim3(R), dim3(256), 0, st, t, pos, wts, top, post, pre, m->eps, m->E, m->Ep, m->x, (T*)m->xb, h32)
+#define HNORM(NI_, KIND_) hipLaunchKernelGGL((k_sub_norm<T, NI_, KIND_>), dim3(R), dim3(256), 0, st, t, add, pos, wts, top, post, pre, m->eps, m->E, m->Ep, m->x, (T*)m->xb, h32)
 #define HNORM_K(NI_) do { if (m->norm_kind == IXT_NORM_TANH) HNORM(NI_, IXT_NORM_TANH); else HNORM(NI_, IXT_NORM_RMS); } while (0)
   if (m->Ep <= 2048) HNORM_K(1); else if (m->Ep <= 4096) HNORM_K(2); else if (m->Ep <= 8192) HNORM_K(4); else HNORM_K(6);
 #undef HNORM_K
 #undef HNORM
   LAUNCHCHK();
   return IXT_OK;
+}
+
+// a sublayer's last product and what follows it: x <- x + post(W v), the next operand pre(x).  Tanh norms ride in the product's epilogue where the whole
+// sum is in one place.
+template <typename T>
+static int hybrid_dot_norm(ixt_ctx* c, const T* v, const HMat& w, const NormW& post, const NormW& pre, bool routed, int R, hipStream_t st) {
+  HybridModel* m = c->hy;
+  if constexpr (sizeof(T) == 2) {
+    const bool small = R <= c->small_rows && sdot_plan(c, GEPI_TANHNORM, false, w.Kp, w.Np, R).ok;
+    if (m->norm_kind == IXT_NORM_TANH && (small || R >= c->ring_min_rows)) {
+      GemmEpi e{};
+      e.act = (bf16_t*)m->xb;
+      e.tn = TanhNormEpi{post.w, post.b, post.alpha, pre.w, pre.b, pre.alpha, m->x, routed && pre.w != nullptr ? m->h32 : nullptr, m->E, m->Ep};
+      if (small) return launch_sdot(c, GEPI_TANHNORM, false, v, nullptr, (const bf16_t*)w.w, w.Kp, w.Np, R, e, st);
+      return launch_ring(c, GEPI_TANHNORM, v, (const bf16_t*)w.w, w.Kp, w.Np, R, e, false, st);
+    }
+  }
+  Slices t;
+  TRY(hdot<T>(c, v, w, R, c->part, c->part_floats, st, &t));
+  return hybrid_norm<T>(c, t, Slices{}, nullptr, nullptr, 0, post, pre, routed, R, st);
 }
 
 template <typename T>
@@ -809,28 +828,27 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
   const NormW none{}, first = m->layers[m->layers[0].src].n1;
   hipLaunchKernelGGL((k_embed_scaled<T>), dim3(R), dim3(256), 0, st, (const T*)m->embed, tokens, m->emb_scale, m->E, m->Ep, m->V, m->norm_kind == IXT_NORM_TANH ? first : none, m->x, (T*)m->xb);
   LAUNCHCHK();
-  if (m->norm_kind == IXT_NORM_RMS && first.w != nullptr) TRY((hybrid_norm<T>(c, Slices{nullptr, 0, 0, 0}, nullptr, nullptr, 0, none, first, false, R, st)));
+  if (m->norm_kind == IXT_NORM_RMS && first.w != nullptr) TRY((hybrid_norm<T>(c, Slices{}, Slices{}, nullptr, nullptr, 0, none, first, false, R, st)));
   for (size_t i = 0; i < m->layers.size(); ++i) {
     const HLayer& L = m->layers[i];
     const HLayer& W = m->layers[L.src];
-    Slices t;
-    if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) TRY((hybrid_mixer_latent<T>(c, L, W, R, Rp, decode, len_hint, st, &t)));
-    else if (L.c.mixer == IXT_MIX_ATTENTION) TRY((hybrid_mixer_heads<T>(c, L, W, R, decode, len_hint, st, &t)));
-    else TRY((hybrid_mixer_delta<T>(c, L, W, R, nseg_max, decode, st, &t)));
+    if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) TRY((hybrid_mixer_latent<T>(c, L, W, R, Rp, decode, len_hint, st)));
+    else if (L.c.mixer == IXT_MIX_ATTENTION) TRY((hybrid_mixer_heads<T>(c, L, W, R, decode, len_hint, st)));
+    else TRY((hybrid_mixer_delta<T>(c, L, W, R, nseg_max, decode, st)));
     const NormW next = i + 1 < m->layers.size() ? m->layers[m->layers[i + 1].src].n1 : none;      // (the head's norm is taken of the wanted rows only)
-    TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n1b, L.c.ffn == IXT_FFN_NONE ? next : W.n2, L.c.ffn == IXT_FFN_MOE, R, st)));
+    TRY((hybrid_dot_norm<T>(c, (const T*)m->act, W.o, W.n1b, L.c.ffn == IXT_FFN_NONE ? next : W.n2, L.c.ffn == IXT_FFN_MOE, R, st)));
     if (L.c.ffn == IXT_FFN_DENSE) {
       TRY(hglu<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, L.c.glu_limit, (T*)m->hact, st));
-      TRY(hdot<T>(c, (const T*)m->hact, W.down, R, c->part, c->part_floats, st, &t));
-      TRY((hybrid_norm<T>(c, t, nullptr, nullptr, 0, W.n2b, next, false, R, st)));
+      TRY((hybrid_dot_norm<T>(c, (const T*)m->hact, W.down, W.n2b, next, false, R, st)));
     } else if (L.c.ffn == IXT_FFN_MOE) {
-      TRY(hybrid_moe<T>(c, L, W, R, st, &t));
+      Slices t, shared{};
+      TRY(hybrid_moe<T>(c, L, W, R, st, &t, &shared));
       if (t.n > 2 && R <= 64) {
-        hipLaunchKernelGGL(k_moe_sum, dim3((t.ncols + 255) / 256, R), dim3(64), 0, st, t, m->mpos, m->mw, L.moe_top, m->msum);
+        hipLaunchKernelGGL(k_moe_sum, dim3((t.ncols + 255) / 256, R), dim3(64), 0, st, t, m->mpos, m->mw, L.c.top, m->msum);
         LAUNCHCHK();
-        TRY((hybrid_norm<T>(c, Slices{m->msum, 1, 0, t.ncols}, nullptr, nullptr, 0, W.n2b, next, false, R, st)));
+        TRY((hybrid_norm<T>(c, Slices{m->msum, 1, 0, t.ncols}, shared, nullptr, nullptr, 0, W.n2b, next, false, R, st)));
       } else {
-        TRY((hybrid_norm<T>(c, t, m->mpos, m->mw, L.moe_top, W.n2b, next, false, R, st)));
+        TRY((hybrid_norm<T>(c, t, shared, m->mpos, m->mw, L.c.top, W.n2b, next, false, R, st)));
       }
     }
     if (m->tap && !c->capturing) {

@@ -247,7 +247,7 @@ __device__ __forceinline__ void norm8(const NormW& n, float s, int k0, const flo
   if constexpr (KIND == IXT_NORM_TANH) {
     load8(n.b + k0, b);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) o[j] = fmaf(ixt_tanh(s * t[j]), w[j], b[j]);
+    for (int j = 0; j < 8; ++j) o[j] = fmaf(tanh_f32(s * t[j]), w[j], b[j]);
   } else {
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[j] = t[j] * s * (1.0f + w[j]);
@@ -274,10 +274,10 @@ __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ tabl
 
 // A sublayer's output t (slices, or the weighted sum of a row's expert outputs) -> norm behind the sublayer -> residual -> norm in front of the next one:
 //   x <- x + post(t);  xb = pre(x) as the next dot's operand, h32 (if given) the same in f32.
-// t.n == 0: t = 0 and x stays.  pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  A thread owns 8 consecutive features of every 2048 (NI
+// t.n == 0: t = 0 and x stays.  pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  add.n > 0: its row joins t.  A thread owns 8 consecutive features of every 2048 (NI
 // times).  grid R, block 256.
 template <typename T, int NI, int KIND>
-__global__ __launch_bounds__(256) void k_sub_norm(Slices t, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, NormW post, NormW pre, float eps,
+__global__ __launch_bounds__(256) void k_sub_norm(Slices t, Slices add, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, NormW post, NormW pre, float eps,
                                                   int E, int Ep, float* __restrict__ x, T* __restrict__ xb, float* __restrict__ h32) {
   __shared__ float red[4];
   const int r = blockIdx.x;
@@ -302,6 +302,12 @@ __global__ __launch_bounds__(256) void k_sub_norm(Slices t, const int32_t* __res
 #pragma unroll
           for (int e = 0; e < 4; ++e) v[i][q + e] = fmaf(wj, u[e], v[i][q + e]);
         }
+      }
+      if (add.n > 0) {
+        float u[4];
+        add.at4(r, k0 + q, u);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[i][q + e] += u[e];
       }
       if (vec) {
         const float4 xx = *reinterpret_cast<const float4*>(x + (size_t)r * E + k0 + q);
@@ -442,6 +448,12 @@ __device__ __forceinline__ void tile_dma(const bf16_t* __restrict__ pages, int o
     const bf16_t* src = pages + (size_t)o * D + NG * 64 + ((lane & 3) ^ ((lane >> 2) & 3)) * 8;
     __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src, (__attribute__((address_space(3))) void*)(tile + NG * 4096 + wave * 512), 16, 0, 0);
   }
+}
+// piece c (features 8 c .. 8 c + 7) of row r of a tile
+template <int D>
+__device__ __forceinline__ void tile_put(bf16_t* tile, int r, int c, u32x4 v) {
+  bf16_t* p = c < D / 64 * 8 ? tile + (c >> 3) * 4096 + r * 64 + ((c ^ r) & 7) * 8 : tile + D / 64 * 4096 + r * 32 + ((c ^ r) & 3) * 8;
+  *reinterpret_cast<u32x4*>(p) = v;
 }
 __device__ __forceinline__ int cached_row(const int32_t* __restrict__ prow, int key, int pshift) { return (prow[key >> pshift] << pshift) + (key & ((1 << pshift) - 1)); }
 // where a lane reads in a tile (byte offsets; the rest of every address is a constant)
@@ -1302,8 +1314,8 @@ __global__ __launch_bounds__(256) void k_glu_slices(Slices t, int Fp, int kind, 
 
 // The choice of experts for a row.  IXT_ROUTE_SOFTMAX: scores s = softmax over all n logits; IXT_ROUTE_SIGMOID: s = sigmoid(z).  The `top` largest
 // s + corr (first index on a tie), inside the `keep` of `groups` equal groups of neighbours whose two largest s + corr add up to most; weights are the
-// picked s, divided by (their sum + 1e-20) if norm, times scale.  `shared` further experts n, n + 1, .. follow with weight 1.
-struct RouteRule { int n, top, kind, groups, keep, norm, shared; float scale; const float* corr; };
+// picked s, divided by (their sum + 1e-20) if norm, times scale.
+struct RouteRule { int n, top, kind, groups, keep, norm; float scale; const float* corr; };
 // one wave; z [n] in LDS (overwritten: choice scores), gs [2 groups] in LDS; n <= 1024
 __device__ __forceinline__ void route_top(float* z, float* gs, const RouteRule& a, int lane, int32_t* idx, float* wts) {
   const int n = a.n;
@@ -1382,7 +1394,6 @@ __device__ __forceinline__ void route_top(float* z, float* gs, const RouteRule& 
   const float f = a.norm ? a.scale / (total + 1e-20f) : a.scale;
   if (lane == 0 && (a.norm || a.scale != 1.0f))
     for (int j = 0; j < a.top; ++j) wts[j] *= f;
-  for (int j = lane; j < a.shared; j += 64) { idx[a.top + j] = n + j; wts[a.top + j] = 1.0f; }
 }
 // router: logits (f32 residual x f32 weights) and choice of RB rows in one block, eight experts at a time: a thread takes every 256th feature of the RB
 // rows and the eight weight rows.  w [n][Ep]; grid ceil(R / RB), block 256, LDS RB (n + 2 groups) floats.
@@ -1391,7 +1402,7 @@ __global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, cons
                                                float* __restrict__ wts) {
   extern __shared__ __attribute__((aligned(16))) float z[];            // [RB][n], [RB][2 groups]
   __shared__ float red[4][RB * 8];
-  const int n = rule.n, row = rule.top + rule.shared;
+  const int n = rule.n, row = rule.top;
   const int r0 = blockIdx.x * RB, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const float* xr[RB];
 #pragma unroll
