@@ -650,9 +650,16 @@ static int heads_prompt_launch(HeadsAttnArgs a, hipStream_t st) {
 template <int DK, int DV>
 static int heads_launch(bool tall, bool fused, int splits, HeadsAttnArgs a, hipStream_t st) {
   if (tall) return heads_prompt_launch<DK, DV, 1>(a, st);
+  constexpr int lds = 64 * (DK + DV) * 2;
+  static bool attr_done = false;
+  if (!attr_done) {
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_decode<DK, DV, true>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_decode<DK, DV, false>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    attr_done = true;
+  }
   const dim3 grid(a.R, a.g.G * a.hchunks, splits);
-  if (fused) hipLaunchKernelGGL((k_heads_decode<DK, DV, true>), grid, dim3(256), 64 * (DK + DV) * 2, st, a);
-  else hipLaunchKernelGGL((k_heads_decode<DK, DV, false>), grid, dim3(256), 64 * (DK + DV) * 2, st, a);
+  if (fused) hipLaunchKernelGGL((k_heads_decode<DK, DV, true>), grid, dim3(256), lds, st, a);
+  else hipLaunchKernelGGL((k_heads_decode<DK, DV, false>), grid, dim3(256), lds, st, a);
   LAUNCHCHK();
   return IXT_OK;
 }

@@ -453,29 +453,48 @@ def test_packed_prefill_and_inserts_carry_the_pages(tmp_path):
   eng.close()
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
-def test_decode_beside_many_slots(tmp_path, dtype):
-  """Forty sequences of unequal length decoding together: the form of the decode step for many rows."""
-  cfg = ZH.mixed_model()
-  w = ZH.random_weights(cfg, 5)
-  eng, params = VH.engine(VH.write_model(tmp_path, cfg, w), dtype=dtype, slots=40, pages=200, target=40, rows=32)
-  lens = [1 + (7 * i) % 30 for i in range(40)]
+def decode_all(cfg, w, eng, params, lens, steps, seed):
+  """All slots decode together; -> (logits of every step [steps, slots, vocab], what the restatement gives for the same tokens)."""
+  B = len(lens)
   st = eng.init_decode_state(materialize_logits=True)
-  seqs = []
+  seqs, got = [], []
   for i, n in enumerate(lens):
     padded = np.zeros(eng.max_prefill_length, np.int32)
-    padded[:n] = VH.tokens(cfg, n, 200 + i)
+    padded[:n] = VH.tokens(cfg, n, seed + i)
     prefix, first = eng.prefill(params=params, padded_tokens=padded, true_length=n, slot=i)
     st = eng.insert(prefix, st, i)
     seqs.append(list(padded[:n]) + [int(first.data[0, 0])])
-  for _ in range(6):
+  for _ in range(steps):
     st, r = eng.generate(params, st)
-    lg, tok = st["logits"].cpu().numpy().reshape(40, -1), r.data.cpu().numpy()[:, 0]
-    got = lg.copy()
-    for i in range(40):
-      seqs[i].append(int(tok[i]))
-  want = np.stack([Z.forward(cfg, w, s[:-1])[-1] for s in seqs])
-  ZH.check(got, want, dtype)
+    got.append(st["logits"].cpu().numpy().reshape(B, -1).copy())
+    for i, tok in enumerate(r.data.cpu().numpy()[:, 0]):
+      seqs[i].append(int(tok))
+  return np.stack(got), np.stack([Z.forward(cfg, w, s[:-1])[-steps:] for s in seqs], axis=1)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", list(ATTENTIONS))
+def test_decode_step_alone(tmp_path, name, dtype):
+  """The decode step's own attention (queries, key and value straight from the projection) at every size: positions around page and tile borders."""
+  cfg = ZH.model([ZH.with_mlp(ATTENTIONS[name], None)])
+  w = ZH.random_weights(cfg, 2)
+  eng, params = VH.engine(VH.write_model(tmp_path, cfg, w), dtype=dtype, slots=3, pages=40, target=90, rows=80)
+  got, want = decode_all(cfg, w, eng, params, (1, 61, 36), 9, 300)
+  for i in range(3):
+    ZH.check(got[:, i], want[:, i], dtype, (name, i))
+  eng.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("slots", [40, 130])
+def test_many_slots_decode_together(tmp_path, slots, dtype):
+  """Sequences of unequal length: the decode step's forms for some tens and for more than 128 rows."""
+  cfg = ZH.mixed_model()
+  w = ZH.random_weights(cfg, 5)
+  eng, params = VH.engine(VH.write_model(tmp_path, cfg, w), dtype=dtype, slots=slots, pages=5 * slots, target=40, rows=32)
+  got, want = decode_all(cfg, w, eng, params, [1 + (7 * i) % 30 for i in range(slots)], 4, 200)
+  for k in range(4):
+    ZH.check(got[k], want[k], dtype, k)
   eng.close()
 
 
