@@ -61,13 +61,6 @@ __device__ __forceinline__ void head_norm_rotate(const Slices& t, int r, int c0,
     emit(f, o);
   }
 }
-__device__ __forceinline__ void store4(bf16_t* p, const float* v) {
-  uint2 o;
-  o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3]));
-  *reinterpret_cast<uint2*>(p) = o;
-}
-__device__ __forceinline__ void store4(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
-
 // LP lanes per head (16, 32, 64): queries [R][H][dkp], and the row's keys and values in their pages.  grid (R, ceil((H + 2 G) LP / 256)), block 256.
 template <typename T, int LP>
 __global__ __launch_bounds__(256) void k_heads_prep(Slices t, HeadsGeom g, const float* __restrict__ qn, const float* __restrict__ kn, float eps, HeadsRope rope, RowsArgs rows,

@@ -239,6 +239,16 @@ __device__ __forceinline__ void load8(const float* __restrict__ p, float* o) {  
   const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
   o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w; o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
 }
+__device__ __forceinline__ void load8(const bf16_t* __restrict__ p, float* o) {
+  const u32x4 a = *reinterpret_cast<const u32x4*>(p);
+  o[0] = bflo(a.x); o[1] = bfhi(a.x); o[2] = bflo(a.y); o[3] = bfhi(a.y); o[4] = bflo(a.z); o[5] = bfhi(a.z); o[6] = bflo(a.w); o[7] = bfhi(a.w);
+}
+__device__ __forceinline__ void store4(bf16_t* p, const float* v) {
+  uint2 o;
+  o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3]));
+  *reinterpret_cast<uint2*>(p) = o;
+}
+__device__ __forceinline__ void store4(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
 // 8 features k0 .. k0 + 7 through a norm; s: the tanh norm's alpha, or the RMS norm's 1 / sqrt(mean + eps)
 template <int KIND>
 __device__ __forceinline__ void norm8(const NormW& n, float s, int k0, const float* t, float* o) {
@@ -262,10 +272,17 @@ __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ tabl
   const int id = min(max(ids[r], 0), V - 1);
   for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
     float v[8];
+    if ((E & 7) == 0 && k0 < E) {
+      load8(table + (size_t)id * E + k0, v);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      v[j] = k0 + j < E ? to_f(table[(size_t)id * E + k0 + j]) * scale : 0.0f;
-      if (k0 + j < E) x[(size_t)r * E + k0 + j] = v[j];
+      for (int j = 0; j < 8; ++j) v[j] *= scale;
+      store4(x + (size_t)r * E + k0, v); store4(x + (size_t)r * E + k0 + 4, v + 4);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        v[j] = k0 + j < E ? to_f(table[(size_t)id * E + k0 + j]) * scale : 0.0f;
+        if (k0 + j < E) x[(size_t)r * E + k0 + j] = v[j];
+      }
     }
     if (pre.w != nullptr) norm8<IXT_NORM_TANH>(pre, *pre.alpha, k0, v, v);
     act_store8(xb, r, k0, Ep, v);
