@@ -166,11 +166,11 @@ __device__ __forceinline__ int heads_row(const int32_t* __restrict__ prow, int k
   return ((prow[key >> pshift] * G + kh) << pshift) + (key & ((1 << pshift) - 1));
 }
 
-// Prompts: a block owns 64 MP pairs = up to 64 MP / HB consecutive rows x HB query heads of one key / value head (a wave 16 MP of them); all waves walk
-// the same key tiles, the next tile arriving while the current one is used.  P stays in registers: with the key order 4q .. 4q + 3, 16 + 4q ..
+// Prompts: a block owns 64 pairs = up to 64 / HB consecutive rows x HB query heads of one key / value head (a wave 16 of them: 32 measured slower, 46
+// against 29 us for 2048 rows of 16 heads); all waves walk the same key tiles, the next tile arriving while the current one is used.  P stays in registers: with the key order 4q .. 4q + 3, 16 + 4q ..
 // 16 + 4q + 3 per lane group q of 32 keys, the lane's own scores ARE its operand of the next product.  Consecutive blocks are different heads: with
 // 8 heads or a multiple of them, a head's keys and values stay in one XCD's L2.  grid (G hchunks, ceil(R / NQ)), block 256, LDS two tiles.
-template <int DK, int DV, int MP>
+template <int DK, int DV>
 __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(HeadsAttnArgs a) {
   constexpr int NKS = DK / 32, NT = DV / 16, NGV = DV / 64, TILE = 64 * (DK + DV);
   extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
@@ -178,27 +178,18 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
   const int kh = blockIdx.x % g.G, hc = blockIdx.x / g.G, GQ = g.H / g.G;
   const int r0 = blockIdx.y * a.NQ, nr = min(a.NQ, a.R - r0), h0 = kh * GQ + hc * a.HB, hb = min(a.HB, GQ - hc * a.HB);
-  int qi[MP], head[MP], row[MP], pos[MP];
-  bool live[MP];
-  bf16x8 qf[MP][NKS];                                     // queries: lane = pair r_in, 8 consecutive features per step
-  float m[MP], l[MP];
-  f32x4 o[MP][NT];
+  const int pair = wave * 16 + r_in, qi = pair / a.HB, hh = pair % a.HB;
+  const bool pair_ok = qi < nr && hh < hb;
+  const int row = r0 + (pair_ok ? qi : 0), head = h0 + (pair_ok ? hh : 0);
+  const bool live = pair_ok && a.rows.active[row] != 0;
+  const int pos = live ? a.rows.pos[row] : -1;
+  bf16x8 qf[NKS];                                         // queries: lane = pair r_in, 8 consecutive features per step
 #pragma unroll
-  for (int p = 0; p < MP; ++p) {
-    const int pair = (wave * MP + p) * 16 + r_in, hh = pair % a.HB;
-    qi[p] = pair / a.HB;
-    const bool ok = qi[p] < nr && hh < hb;
-    row[p] = r0 + (ok ? qi[p] : 0); head[p] = h0 + (ok ? hh : 0);
-    live[p] = ok && a.rows.active[row[p]] != 0;
-    pos[p] = live[p] ? a.rows.pos[row[p]] : -1;
+  for (int ks = 0; ks < NKS; ++ks) qf[ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.q + ((size_t)row * g.H + head) * DK + ks * 32 + cq * 8));
+  float m = a.sink != nullptr ? a.sink[head] * 1.44269504088896340736f : -INFINITY, l = a.sink != nullptr ? 1.0f : 0.0f;
+  f32x4 o[NT];
 #pragma unroll
-    for (int ks = 0; ks < NKS; ++ks)
-      qf[p][ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.q + ((size_t)row[p] * g.H + head[p]) * DK + ks * 32 + cq * 8));
-    m[p] = a.sink != nullptr ? a.sink[head[p]] * 1.44269504088896340736f : -INFINITY;
-    l[p] = a.sink != nullptr ? 1.0f : 0.0f;
-#pragma unroll
-    for (int i = 0; i < NT; ++i) o[p][i] = f32x4(0.0f);
-  }
+  for (int i = 0; i < NT; ++i) o[i] = f32x4(0.0f);
   const float sc = g.scale * 1.44269504088896340736f;
   const TileLane L = tile_lane(r_in, cq);
   for (int ra = 0; ra < nr;) {                            // runs of rows that share a page group
@@ -207,13 +198,8 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
     int lo = a.rows.pos[r0 + ra], hi = lo, rb = ra + 1;
     while (rb < nr && a.rows.active[r0 + rb] && a.rows.slot[r0 + rb] == slot) { const int p = a.rows.pos[r0 + rb]; lo = min(lo, p); hi = max(hi, p); ++rb; }
     const bool whole = ra == 0 && rb == nr;               // no other run in this block: only the keys decide what is masked
-    bool mine[MP];
-    int my_lo[MP];
-#pragma unroll
-    for (int p = 0; p < MP; ++p) {
-      mine[p] = live[p] && qi[p] >= ra && qi[p] < rb;
-      my_lo[p] = g.window > 0 ? max(0, pos[p] - g.window + 1) : 0;
-    }
+    const bool mine = live && qi >= ra && qi < rb;
+    const int my_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
     ra = rb;
     const int k_lo = g.window > 0 ? max(0, lo - g.window + 1) : 0, k_all = g.window > 0 ? max(0, hi - g.window + 1) : 0;    // (k_all .. lo: seen by every row)
     const int ntile = (hi - k_lo) / 64 + 1;
@@ -233,11 +219,9 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
         tile_dma<DV>(a.vpages, off, next + 64 * DK, wave, lane);
         off = heads_row(prow, min(k_lo + (t + 2) * 64 + lane, hi), a.pshift, g.G, kh);
       }
-      f32x4 s[MP][4];
+      f32x4 s[4];
 #pragma unroll
-      for (int p = 0; p < MP; ++p)
-#pragma unroll
-        for (int n = 0; n < 4; ++n) s[p][n] = f32x4(0.0f);
+      for (int n = 0; n < 4; ++n) s[n] = f32x4(0.0f);
       bf16x8 kf[2][4];                                    // operands one step ahead of the products
 #pragma unroll
       for (int n = 0; n < 4; ++n) kf[0][n] = tile_kf<DK>(reinterpret_cast<const char*>(tile), L, 0, n);
@@ -248,58 +232,53 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
           for (int n = 0; n < 4; ++n) kf[(ks + 1) & 1][n] = tile_kf<DK>(reinterpret_cast<const char*>(tile), L, ks + 1, n);
         }
 #pragma unroll
-        for (int n = 0; n < 4; ++n)
-#pragma unroll
-          for (int p = 0; p < MP; ++p) s[p][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][n], qf[p][ks], s[p][n], 0, 0, 0);
+        for (int n = 0; n < 4; ++n) s[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][n], qf[ks], s[n], 0, 0, 0);
         __builtin_amdgcn_sched_barrier(0);
       }
       const int t0 = k_lo + t * 64;
       const bool inside = whole && t0 >= k_all && t0 + 63 <= lo;
-      bf16x8 pf[MP][2];
-#pragma unroll
-      for (int p = 0; p < MP; ++p) {
-        float tm = -INFINITY;
-        if (inside) {
-#pragma unroll
-          for (int n = 0; n < 4; ++n)
-#pragma unroll
-            for (int j = 0; j < 4; ++j) tm = fmaxf(tm, s[p][n][j]);
-        } else {
-#pragma unroll
-          for (int n = 0; n < 4; ++n)
-#pragma unroll
-            for (int j = 0; j < 4; ++j) {
-              const int key = t0 + n * 16 + cq * 4 + j;
-              const bool seen = mine[p] && key <= pos[p] && key >= my_lo[p];
-              s[p][n][j] = seen ? s[p][n][j] : -INFINITY;
-              tm = fmaxf(tm, s[p][n][j]);
-            }
-        }
-        tm *= sc;                                         // (a positive factor keeps the order)
-        tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
-        tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
-        const float mn = fmaxf(m[p], tm), mz = mn == -INFINITY ? 0.0f : mn;
-        const float al = hw_exp2(m[p] - mz);           // (nothing seen so far: exp2(-inf) = 0, and l and o are 0)
-        float ls = 0.0f;
+      bf16x8 pf[2];
+      float tm = -INFINITY;
+      if (inside) {
 #pragma unroll
         for (int n = 0; n < 4; ++n)
 #pragma unroll
-          for (int j = 0; j < 4; ++j) { s[p][n][j] = hw_exp2(fmaf(s[p][n][j], sc, -mz)); ls += s[p][n][j]; }
-        ls += __shfl_xor(ls, 16, 64);
-        ls += __shfl_xor(ls, 32, 64);
-        l[p] = l[p] * al + ls;
-        m[p] = mn;
-        if (__any(al != 1.0f)) {
+          for (int j = 0; j < 4; ++j) tm = fmaxf(tm, s[n][j]);
+      } else {
 #pragma unroll
-          for (int i = 0; i < NT; ++i) { o[p][i][0] *= al; o[p][i][1] *= al; o[p][i][2] *= al; o[p][i][3] *= al; }
-        }
+        for (int n = 0; n < 4; ++n)
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {                     // 32 keys each
-          u32x4 pk;
-          pk.x = pack2(f2bf(s[p][2 * u][0]), f2bf(s[p][2 * u][1])); pk.y = pack2(f2bf(s[p][2 * u][2]), f2bf(s[p][2 * u][3]));
-          pk.z = pack2(f2bf(s[p][2 * u + 1][0]), f2bf(s[p][2 * u + 1][1])); pk.w = pack2(f2bf(s[p][2 * u + 1][2]), f2bf(s[p][2 * u + 1][3]));
-          pf[p][u] = __builtin_bit_cast(bf16x8, pk);
-        }
+          for (int j = 0; j < 4; ++j) {
+            const int key = t0 + n * 16 + cq * 4 + j;
+            const bool seen = mine && key <= pos && key >= my_lo;
+            s[n][j] = seen ? s[n][j] : -INFINITY;
+            tm = fmaxf(tm, s[n][j]);
+          }
+      }
+      tm *= sc;                                         // (a positive factor keeps the order)
+      tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+      tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+      const float mn = fmaxf(m, tm), mz = mn == -INFINITY ? 0.0f : mn;
+      const float al = hw_exp2(m - mz);           // (nothing seen so far: exp2(-inf) = 0, and l and o are 0)
+      float ls = 0.0f;
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { s[n][j] = hw_exp2(fmaf(s[n][j], sc, -mz)); ls += s[n][j]; }
+      ls += __shfl_xor(ls, 16, 64);
+      ls += __shfl_xor(ls, 32, 64);
+      l = l * al + ls;
+      m = mn;
+      if (__any(al != 1.0f)) {
+#pragma unroll
+        for (int i = 0; i < NT; ++i) { o[i][0] *= al; o[i][1] *= al; o[i][2] *= al; o[i][3] *= al; }
+      }
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {                     // 32 keys each
+        u32x4 pk;
+        pk.x = pack2(f2bf(s[2 * u][0]), f2bf(s[2 * u][1])); pk.y = pack2(f2bf(s[2 * u][2]), f2bf(s[2 * u][3]));
+        pk.z = pack2(f2bf(s[2 * u + 1][0]), f2bf(s[2 * u + 1][1])); pk.w = pack2(f2bf(s[2 * u + 1][2]), f2bf(s[2 * u + 1][3]));
+        pf[u] = __builtin_bit_cast(bf16x8, pk);
       }
       const uint32_t tb = lds_addr(tile) + 64 * DK * 2;
 #pragma unroll
@@ -315,35 +294,28 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
             IXT_TILE_VWAIT(f[gr & 1], 0);
           }
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-#pragma unroll
-            for (int p = 0; p < MP; ++p) o[p][gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(f[gr & 1][i]), pf[p][u], o[p][gr * 4 + i], 0, 0, 0);
+          for (int i = 0; i < 4; ++i) o[gr * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(f[gr & 1][i]), pf[u], o[gr * 4 + i], 0, 0, 0);
         }
         if constexpr (DV % 64 != 0) {
           uint2 fh[2][2];
           IXT_TILE_VTH(fh, tb, L, NGV, u);
           IXT_TILE_VWAITN(fh, 2, 0);
 #pragma unroll
-          for (int i = 0; i < 2; ++i)
-#pragma unroll
-            for (int p = 0; p < MP; ++p) o[p][NGV * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(fh[i]), pf[p][u], o[p][NGV * 4 + i], 0, 0, 0);
+          for (int i = 0; i < 2; ++i) o[NGV * 4 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile_vfrag(fh[i]), pf[u], o[NGV * 4 + i], 0, 0, 0);
         }
       }
     }
   }
+  if (!live) return;
+  const float inv = 1.0f / l;
 #pragma unroll
-  for (int p = 0; p < MP; ++p) {
-    if (!live[p]) continue;
-    const float inv = 1.0f / l[p];
-#pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const float v[4] = {o[p][i][0] * inv, o[p][i][1] * inv, o[p][i][2] * inv, o[p][i][3] * inv};
-      if (i * 16 + cq * 4 < g.vs) act_store4(a.out, row[p], head[p] * g.vs + i * 16 + cq * 4, a.Kp, v);      // (columns dv .. vs - 1 are zero: so are the values there)
-    }
-    const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-    if (head[p] == g.H - 1)
-      for (int c = g.H * g.vs + cq * 4; c < a.Kp; c += 16) act_store4(a.out, row[p], c, a.Kp, z);
+  for (int i = 0; i < NT; ++i) {
+    const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+    if (i * 16 + cq * 4 < g.vs) act_store4(a.out, row, head * g.vs + i * 16 + cq * 4, a.Kp, v);      // (columns dv .. vs - 1 are zero: so are the values there)
   }
+  const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  if (head == g.H - 1)
+    for (int c = g.H * g.vs + cq * 4; c < a.Kp; c += 16) act_store4(a.out, row, c, a.Kp, z);
 }
 
 // Few rows (decode): a block owns up to 16 query heads of one key / value head of ONE row and every gridDim.z-th key tile of its window.  Scores: a wave

@@ -633,23 +633,23 @@ static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int
   return IXT_OK;
 }
 
-template <int DK, int DV, int MP>
+template <int DK, int DV>
 static int heads_prompt_launch(HeadsAttnArgs a, hipStream_t st) {
   constexpr int lds = 2 * 64 * (DK + DV) * 2;
   static bool attr_done = false;
   if (!attr_done) {
-    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_prompt<DK, DV, MP>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_prompt<DK, DV>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
     attr_done = true;
   }
   const int GQ = a.g.H / a.g.G;
-  a.HB = std::min(GQ, 64 * MP); a.NQ = 64 * MP / a.HB; a.hchunks = (GQ + a.HB - 1) / a.HB;
-  hipLaunchKernelGGL((k_heads_prompt<DK, DV, MP>), dim3(a.g.G * a.hchunks, (a.R + a.NQ - 1) / a.NQ), dim3(256), lds, st, a);
+  a.HB = std::min(GQ, 64); a.NQ = 64 / a.HB; a.hchunks = (GQ + a.HB - 1) / a.HB;
+  hipLaunchKernelGGL((k_heads_prompt<DK, DV>), dim3(a.g.G * a.hchunks, (a.R + a.NQ - 1) / a.NQ), dim3(256), lds, st, a);
   LAUNCHCHK();
   return IXT_OK;
 }
 template <int DK, int DV>
 static int heads_launch(bool tall, bool fused, int splits, HeadsAttnArgs a, hipStream_t st) {
-  if (tall) return heads_prompt_launch<DK, DV, 1>(a, st);
+  if (tall) return heads_prompt_launch<DK, DV>(a, st);
   constexpr int lds = 64 * (DK + DV) * 2;
   static bool attr_done = false;
   if (!attr_done) {
