@@ -31,7 +31,7 @@ typedef enum ixt_status {
 typedef enum ixt_dtype { IXT_BF16 = 0, IXT_F32 = 1 } ixt_dtype;
 
 /* One layer of an IXT_BLOCK_HYBRID decoder: a sequence mixer, then a feed-forward, each with a norm in front, behind, or both (ixt_config.norm_places):
- *   x <- x + after(mixer(before(x))), x <- x + after(ff(before(x))), the residual x in f32. */
+ *   x <- x + after(mixer(before(x))), x <- x + after(ff(before(x))), the residual x in f32 (or several streams: ixt_config.streams). */
 typedef struct ixt_layer {
   int32_t mixer;                   /* IXT_MIX_* */
   int32_t weights_of;              /* -1, or the layer whose parameters this one shares (it keeps a cache or state of its own) */
@@ -39,7 +39,7 @@ typedef struct ixt_layer {
   /* latent attention: keys and values are up-projections of one cached latent per token plus one rotated key part shared by all heads */
   int32_t rot_dim, kv_rank;        /* rotated dims per head (even), latent size (<= 1024) */
   int32_t window;                  /* position i sees i - window + 1 .. i; <= 0: everything up to i */
-  float rope_base, attn_scale;     /* neighbouring pairs (2 i, 2 i + 1) turn by p base^(-2 i / rot_dim); score factor */
+  float rope_base, attn_scale;     /* pair i of the rotated features (rope_pairs) turns by p base^(-2 i / rot_dim); score factor */
   /* gated delta rule with one decay per head and key channel: S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q */
   int32_t kv_heads;                /* query / key heads (heads % kv_heads == 0); IXT_MIX_ATTENTION: key / value heads */
   int32_t conv;                    /* taps of the causal convolutions in front of q, k, v */
@@ -60,15 +60,29 @@ typedef struct ixt_layer {
   int32_t groups, groups_keep;     /* > 1: equal groups of neighbours, a group scores the sum of its two best choice scores, the best groups_keep are open */
   int32_t router_norm;             /* != 0: weights divided by (their sum + 1e-20) */
   float router_scale;              /* then multiplied by this */
-  int32_t shared_ff;               /* > 0: hidden size of a gated unit of the same form that every token runs through, added to the mixture */
+  int32_t shared_ff;               /* > 0: hidden size of a unit of the same form that every token runs through, added to the mixture */
+  int32_t number;                  /* the layer's tensors are named l<number>.*; -1: its place in the list (read for layers with parameters of their own) */
+  int32_t rope_pairs;              /* IXT_ROPE_*: which two of the rotated features turn together */
+  int32_t q_rank;                  /* latent attention, > 0: queries are up-projections of an RMS-normed (plain weight) latent of this size */
+  int32_t out_gate;                /* attention mixers, != 0: the concatenated heads are multiplied by sigmoid(W_g h) in front of the output projection */
+  int32_t maps;                    /* IXT_MIX_ATTENTION: 2: every head has two softmax maps of `dim` features each over the same values, and its output is
+                                      rms(a1 - lambda a2) (1 - map_diff) with lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + map_diff; 0 or 1: one map */
+  float map_diff;
+  float softcap;                   /* IXT_MIX_ATTENTION, > 0: score <- softcap tanh(score / softcap) */
+  int32_t router_bias;             /* != 0: a per-expert number joins the router's logits */
+  int32_t shared_gate;             /* != 0: the shared unit's output is multiplied by sigmoid(w . h), one number per token */
+  const double* decay;             /* IXT_MIX_RETENTION: one decay per head (HOST array of `heads` entries, copied by ixt_create) */
 } ixt_layer;
-enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1, IXT_MIX_ATTENTION = 2 };
+/* IXT_MIX_RETENTION: S <- decay S + (k / sqrt(dim)) v^T, o = S^T q with rotated q and k, per head; o / rms(o), times silu(W_g h) */
+enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1, IXT_MIX_ATTENTION = 2, IXT_MIX_RETENTION = 3 };
+enum { IXT_ROPE_NEIGHBOURS = 0, IXT_ROPE_HALVES = 1 };      /* (2 i, 2 i + 1); (i, i + rot_dim / 2) */
 enum { IXT_FFN_NONE = 0, IXT_FFN_DENSE = 1, IXT_FFN_MOE = 2 };
-/* gated units of g = gate, u = up: min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u, -limit, limit) + 1); gelu(g) u (tanh form); silu(g) u */
-enum { IXT_GLU_CLAMPED = 1, IXT_GLU_GELU_TANH = 2, IXT_GLU_SILU = 3 };
-enum { IXT_ROUTE_SOFTMAX = 0, IXT_ROUTE_SIGMOID = 1 };
-/* norms around the sublayers and in front of the head: t / sqrt(mean(t^2) + eps) (1 + w); tanh(alpha t) w + b */
-enum { IXT_NORM_RMS = 0, IXT_NORM_TANH = 1 };
+/* gated units of g = gate, u = up: min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u, -limit, limit) + 1); gelu(g) u (tanh form); silu(g) u.
+ * From IXT_ACT_RELU2 on a unit has no gate: max(u, 0)^2 */
+enum { IXT_GLU_CLAMPED = 1, IXT_GLU_GELU_TANH = 2, IXT_GLU_SILU = 3, IXT_ACT_RELU2 = 4 };
+enum { IXT_ROUTE_SOFTMAX = 0, IXT_ROUTE_SIGMOID = 1, IXT_ROUTE_CHOSEN = 2 };      /* CHOSEN: choice by logit, weights = softmax over the chosen logits */
+/* norms around the sublayers and in front of the head: t / sqrt(mean(t^2) + eps) (1 + w); tanh(alpha t) w + b; (t - mean) / sqrt(variance + eps) w + b */
+enum { IXT_NORM_RMS = 0, IXT_NORM_TANH = 1, IXT_NORM_LAYER = 2 };
 enum { IXT_NORM_BEFORE = 1, IXT_NORM_AFTER = 2 };
 
 /* Derived hyper-parameters of MaxText/pyconfig.py:551-644 that shape the path. */
@@ -140,7 +154,11 @@ typedef struct ixt_config {
   const ixt_layer* layers;
   float embedding_scale;           /* x = embedding[token] * scale */
   int32_t float32;
-  int32_t norm_kind, norm_places;  /* IXT_NORM_RMS | IXT_NORM_TANH; sum of IXT_NORM_BEFORE, IXT_NORM_AFTER */
+  int32_t norm_kind, norm_places;  /* IXT_NORM_*; sum of IXT_NORM_BEFORE, IXT_NORM_AFTER */
+  /* > 0: hyper-connections in the place of the residual sum: that many streams x_1 .. x_s, all the embedding row at the start.  Sublayer q (1: mixer, 2:
+   * feed-forward) reads u = sum_s in[s] x_s and leaves x_t <- sum_s mix[s][t] x_s + out[t] y (tensors l<i>.hc<q>.in, .mix, .out); the head reads their sum. */
+  int32_t streams;
+  float logit_scale;               /* hybrid: factor on the logits; with logits_via_embedding the head is the embedding table (without its scale) */
 } ixt_config;
 
 enum { IXT_BLOCK_LLAMA2 = 0, IXT_BLOCK_GEMMA2 = 1, IXT_BLOCK_GEMMA3 = 2, IXT_BLOCK_MIXTRAL = 3, IXT_BLOCK_HYBRID = 4 };

@@ -27,7 +27,8 @@ class IxtLayer(ctypes.Structure):
       ("glu_limit", ctypes.c_float), ("experts", ctypes.c_int32), ("top", ctypes.c_int32), ("qk_norm", ctypes.c_int32), ("sink", ctypes.c_int32)] + [
       (n, ctypes.c_float) for n in ("rope_factor", "rope_low", "rope_high", "rope_original")] + [
       (n, ctypes.c_int32) for n in ("glu", "router", "router_correction", "groups", "groups_keep", "router_norm")] + [
-      ("router_scale", ctypes.c_float), ("shared_ff", ctypes.c_int32)]
+      ("router_scale", ctypes.c_float)] + [(n, ctypes.c_int32) for n in ("shared_ff", "number", "rope_pairs", "q_rank", "out_gate", "maps")] + [
+      ("map_diff", ctypes.c_float), ("softcap", ctypes.c_float), ("router_bias", ctypes.c_int32), ("shared_gate", ctypes.c_int32), ("decay", c_f64p)]
 
 
 class IxtConfig(ctypes.Structure):
@@ -48,7 +49,7 @@ class IxtConfig(ctypes.Structure):
       ("ep_rank", ctypes.c_int32), ("ep_size", ctypes.c_int32), ("fp8_weights", ctypes.c_int32),
       ("rope_llama31", ctypes.c_int32), ("rope_use_scale", ctypes.c_int32),
       ("layers", ctypes.POINTER(IxtLayer)), ("embedding_scale", ctypes.c_float), ("float32", ctypes.c_int32),
-      ("norm_kind", ctypes.c_int32), ("norm_places", ctypes.c_int32),
+      ("norm_kind", ctypes.c_int32), ("norm_places", ctypes.c_int32), ("streams", ctypes.c_int32), ("logit_scale", ctypes.c_float),
   ]
 
 BLOCK_LLAMA2, BLOCK_GEMMA2, BLOCK_GEMMA3, BLOCK_MIXTRAL, BLOCK_HYBRID = 0, 1, 2, 3, 4

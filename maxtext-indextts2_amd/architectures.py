@@ -9,13 +9,15 @@ import dataclasses
 import json
 import os
 import struct
-from typing import Any, Callable, Dict, Mapping, Tuple
+from typing import Any, Callable, Dict, Mapping, Sequence, Tuple
 
-MIX_LATENT_ATTENTION, MIX_GATED_DELTA, MIX_ATTENTION = 0, 1, 2
+MIX_LATENT_ATTENTION, MIX_GATED_DELTA, MIX_ATTENTION, MIX_RETENTION = 0, 1, 2, 3
+RECURRENT_MIXERS = (MIX_GATED_DELTA, MIX_RETENTION)
 FFN_NONE, FFN_DENSE, FFN_MOE = 0, 1, 2
-GLU_CLAMPED, GLU_GELU_TANH, GLU_SILU = 1, 2, 3
-ROUTE_SOFTMAX, ROUTE_SIGMOID = 0, 1
-NORM_RMS, NORM_TANH = 0, 1
+GLU_CLAMPED, GLU_GELU_TANH, GLU_SILU, ACT_RELU2 = 1, 2, 3, 4      # from ACT_RELU2 on: no gate
+ROUTE_SOFTMAX, ROUTE_SIGMOID, ROUTE_CHOSEN = 0, 1, 2
+ROPE_NEIGHBOURS, ROPE_HALVES = 0, 1
+NORM_RMS, NORM_TANH, NORM_LAYER = 0, 1, 2
 NORM_BEFORE, NORM_AFTER = 1, 2
 
 
@@ -55,6 +57,16 @@ class HybridLayer:
   router_norm: int = 0
   router_scale: float = 1.0
   shared_ff: int = 0
+  number: int = -1
+  rope_pairs: int = ROPE_NEIGHBOURS
+  q_rank: int = 0
+  out_gate: int = 0
+  maps: int = 1
+  map_diff: float = 0.0
+  softcap: float = 0.0
+  router_bias: int = 0
+  shared_gate: int = 0
+  decay: Tuple[float, ...] = ()
 
 
 Shapes = Mapping[str, Tuple[int, ...]]
@@ -167,7 +179,80 @@ def vazilorn_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
   }
 
 
+def _suzulix_latent(m: Mapping[str, Any]) -> Dict[str, Any]:
+  rot = m["rot"]
+  if int(rot["dims"]) != int(m["rot_dim"]):
+    raise ValueError(f"Suzulix: rot.dims ({rot['dims']}) must equal rot_dim ({m['rot_dim']})")
+  return {"mixer": MIX_LATENT_ATTENTION, "heads": int(m["heads"]), "dim": int(m["dim"]), "vdim": int(m["vdim"]), "rot_dim": int(m["rot_dim"]), "kv_rank": int(m["kv_rank"]),
+          "q_rank": int(m["q_rank"]), "rope_base": float(rot["base"]), "rope_pairs": ROPE_HALVES, "attn_scale": float(m["scale"]), "out_gate": 1}
+
+
+def _suzulix_attention(m: Mapping[str, Any]) -> Dict[str, Any]:
+  rot = m["rot"]
+  heads, kv_heads, dim, dims = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(rot["dims"])
+  if heads % kv_heads or dims % 2 or dims > dim:
+    raise ValueError(f"Suzulix: {heads} heads over {kv_heads} key heads, {dims} of {dim} dims rotated")
+  return {"mixer": MIX_ATTENTION, "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": int(m["vdim"]), "rot_dim": dims, "rope_base": float(rot["base"]),
+          "attn_scale": float(m["scale"]), "softcap": float(m["softcap"]), "maps": 2, "map_diff": float(m["diff"]), "out_gate": 1}
+
+
+def _suzulix_retention(m: Mapping[str, Any]) -> Dict[str, Any]:
+  rot, decay = m["rot"], tuple(float(d) for d in m["decay"])
+  heads, dim, dims = int(m["heads"]), int(m["dim"]), int(rot["dims"])
+  if len(decay) != heads or dims % 2 or dims > dim:
+    raise ValueError(f"Suzulix: {len(decay)} decays for {heads} heads, {dims} of {dim} dims rotated")
+  return {"mixer": MIX_RETENTION, "heads": heads, "dim": dim, "vdim": int(m["vdim"]), "rot_dim": dims, "rope_base": float(rot["base"]), "rope_pairs": ROPE_HALVES, "decay": decay}
+
+
+_SUZULIX_MIXERS = {"latent_attention": _suzulix_latent, "attention": _suzulix_attention, "retention": _suzulix_retention}
+
+
+def _suzulix_feed_forward(mlp: Any) -> Dict[str, Any]:
+  if mlp is None:
+    return {"ffn": FFN_NONE}
+  if mlp["kind"] != "moe":
+    raise ValueError(f"Suzulix: feed-forward kind {mlp['kind']!r}")
+  shared = mlp.get("shared") or {}
+  return {"ffn": FFN_MOE, "ff": int(mlp["expert"]["ff"]), "glu": ACT_RELU2, "experts": int(mlp["router"]["experts"]), "top": int(mlp["router"]["top"]), "router": ROUTE_CHOSEN,
+          "router_bias": 1, "shared_ff": int(shared.get("ff") or 0), "shared_gate": 1 if shared.get("ff") else 0}
+
+
+def suzulix_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
+  """Suzulix: latent attention, differential attention and retention in any order, a stretch of layers run several times; layer norms in front,
+  hyper-connections, routed squared-relu units with a gated shared one, the embedding table as the head."""
+  del shapes
+  layers = []
+  for i, entry in enumerate(cfg["layers"]):
+    if entry["type"] not in _SUZULIX_MIXERS:
+      raise ValueError(f"Suzulix: layer {i} has type {entry['type']!r}")
+    layers.append(HybridLayer(number=i, **_SUZULIX_MIXERS[entry["type"]](entry["mixer"]), **_suzulix_feed_forward(entry.get("mlp"))))
+  loop = cfg.get("loop")
+  return {
+      "decoder_block": "hybrid",
+      "vocab_size": int(cfg["vocab"]),
+      "base_emb_dim": int(cfg["width"]),
+      "normalization_layer_epsilon": float(cfg["norm"]["eps"]),
+      "embedding_scale": float(cfg["embedding"]["scale"]),
+      "logits_via_embedding": True,
+      "logit_scale": float(cfg["logit_scale"]),
+      "hybrid_norm_kind": NORM_LAYER,
+      "hybrid_norm_places": NORM_BEFORE,
+      "hybrid_streams": int(cfg["streams"]),
+      **_looped(layers, *((int(loop["start"]), int(loop["stop"]), int(loop["times"])) if loop else (0, 0, 1))),
+  }
+
+
+def _looped(layers: Sequence[HybridLayer], start: int, stop: int, times: int) -> Dict[str, Any]:
+  """Layers start .. stop - 1 `times` times in a row: every further pass is a run of its own (cache, state) on the first one's parameters."""
+  if not 0 <= start <= stop <= len(layers) or times < 1:
+    raise ValueError(f"loop {start} .. {stop}, {times} times, over {len(layers)} layers")
+  again = [dataclasses.replace(layers[i], weights_of=i) for _ in range(times - 1) for i in range(start, stop)]
+  runs = tuple(layers[:stop]) + tuple(again) + tuple(layers[stop:])
+  return {"base_num_decoder_layers": len(runs), "hybrid_layers": runs}
+
+
 ARCHITECTURES: Dict[str, Callable[[Mapping[str, Any], Shapes], Dict[str, Any]]] = {
+    "Suzulix": suzulix_keys,
     "Vazilorn": vazilorn_keys,
     "Vilepel": vilepel_keys,
 }
@@ -190,34 +275,52 @@ def read_model_dir(path: str) -> Dict[str, Any]:
 
 def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
   """{tensor name: shape} of a hybrid decoder; linear weights are [out, in]."""
-  E, V = int(config.emb_dim), int(config.vocab_size)
-  out: Dict[str, Tuple[int, ...]] = {"embed": (V, E), "head": (V, E)}
+  E, V, S = int(config.emb_dim), int(config.vocab_size), int(config.hybrid_streams)
+  out: Dict[str, Tuple[int, ...]] = {"embed": (V, E)}
+  if not config.logits_via_embedding:
+    out["head"] = (V, E)
 
   def norm(name: str) -> None:
     out[name] = (E,)
+    if config.hybrid_norm_kind != NORM_RMS:
+      out[name + ".b"] = (E,)
     if config.hybrid_norm_kind == NORM_TANH:
-      out[name + ".alpha"], out[name + ".b"] = (), (E,)
+      out[name + ".alpha"] = ()
 
-  def gated(name: str, ff: int) -> None:
-    out[name + "gate"], out[name + "up"], out[name + "down"] = (ff, E), (ff, E), (E, ff)
+  def unit(name: str, ff: int, kind: int) -> None:
+    if kind < ACT_RELU2:
+      out[name + "gate"] = (ff, E)
+    out[name + "up"], out[name + "down"] = (ff, E), (E, ff)
 
   both = config.hybrid_norm_places == NORM_BEFORE | NORM_AFTER
   norm("final.norm")
   for i, l in enumerate(config.hybrid_layers):
     if l.weights_of >= 0:
       continue
-    p = f"l{i}."
+    p = f"l{i if l.number < 0 else l.number}."
+    for q in ("hc1.", "hc2.")[:0 if S == 0 else 1 if l.ffn == FFN_NONE else 2]:
+      out.update({p + q + "in": (S,), p + q + "out": (S,), p + q + "mix": (S, S)})
     for n in ("norm1", "norm1b")[:1 + both] + (() if l.ffn == FFN_NONE else ("norm2", "norm2b")[:1 + both]):
       norm(p + n)
     if l.mixer == MIX_LATENT_ATTENTION:
-      out.update({p + "mix.q": (l.heads * (l.dim + l.rot_dim), E), p + "mix.dkv": (l.kv_rank + l.rot_dim, E), p + "mix.dkv.norm": (l.kv_rank,),
+      if l.q_rank > 0:
+        out.update({p + "mix.dq": (l.q_rank, E), p + "mix.dq.norm": (l.q_rank,), p + "mix.uq": (l.heads * (l.dim + l.rot_dim), l.q_rank)})
+      else:
+        out[p + "mix.q"] = (l.heads * (l.dim + l.rot_dim), E)
+      out.update({p + "mix.dkv": (l.kv_rank + l.rot_dim, E), p + "mix.dkv.norm": (l.kv_rank,),
                   p + "mix.uk": (l.heads * l.dim, l.kv_rank), p + "mix.uv": (l.heads * l.vdim, l.kv_rank), p + "mix.o": (E, l.heads * l.vdim)})
     elif l.mixer == MIX_ATTENTION:
-      out.update({p + "mix.q": (l.heads * l.dim, E), p + "mix.k": (l.kv_heads * l.dim, E), p + "mix.v": (l.kv_heads * l.vdim, E), p + "mix.o": (E, l.heads * l.vdim)})
+      out.update({p + "mix.q": (l.heads * l.maps * l.dim, E), p + "mix.k": (l.kv_heads * l.maps * l.dim, E), p + "mix.v": (l.kv_heads * l.vdim, E),
+                  p + "mix.o": (E, l.heads * l.vdim)})
+      if l.maps > 1:
+        out.update({p + f"mix.{n}": (l.dim,) for n in ("lq1", "lk1", "lq2", "lk2")})
       if l.qk_norm:
         out[p + "mix.q.norm"] = out[p + "mix.k.norm"] = (l.dim,)
       if l.sink:
         out[p + "mix.sink"] = (l.heads,)
+    elif l.mixer == MIX_RETENTION:
+      kq, v = l.heads * l.dim, l.heads * l.vdim
+      out.update({p + "mix.q": (kq, E), p + "mix.k": (kq, E), p + "mix.v": (v, E), p + "mix.g": (v, E), p + "mix.o": (E, v)})
     else:
       kq, v = l.kv_heads * l.dim, l.heads * l.vdim
       for t, n in (("q", kq), ("k", kq), ("v", v)):
@@ -225,14 +328,20 @@ def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
       out.update({p + "mix.b": (l.heads, E), p + "mix.A_log": (l.heads,), p + "mix.norm": (l.vdim,), p + "mix.a1": (l.decay_rank, E),
                   p + "mix.a2": (l.heads * l.dim, l.decay_rank), p + "mix.dt_bias": (l.heads * l.dim,), p + "mix.g1": (l.gate_rank, E),
                   p + "mix.g2": (v, l.gate_rank), p + "mix.o": (E, v)})
+    if l.out_gate:
+      out[p + "mix.g"] = (l.heads * l.vdim, E)
     if l.ffn == FFN_DENSE:
-      gated(p + "mlp.", l.ff)
+      unit(p + "mlp.", l.ff, l.glu)
     elif l.ffn == FFN_MOE:
       for e in range(l.experts):
-        gated(p + f"mlp.e{e}.", l.ff)
+        unit(p + f"mlp.e{e}.", l.ff, l.glu)
       out[p + "mlp.router"] = (l.experts, E)
+      if l.router_bias:
+        out[p + "mlp.router.b"] = (l.experts,)
       if l.router_correction:
         out[p + "mlp.correction"] = (l.experts,)
       if l.shared_ff > 0:
-        gated(p + "mlp.shared.", l.shared_ff)
+        unit(p + "mlp.shared.", l.shared_ff, l.glu)
+        if l.shared_gate:
+          out[p + "mlp.shared.sg"] = (1, E)
   return out

@@ -749,10 +749,12 @@ int launch_ring(ixt_ctx* c, int epi, const bf16_t* x, const bf16_t* w, int K, in
   else if (two_per_cu && epi == GEPI_SWIGLU) rc = RING_P(GEPI_SWIGLU);
   else if (two_per_cu && epi == GEPI_F32) rc = RING_P(GEPI_F32);
   else if (two_per_cu && epi == GEPI_TANHNORM) rc = RING_P(GEPI_TANHNORM);
+  else if (two_per_cu && epi == GEPI_ACT) rc = RING_P(GEPI_ACT);
   else if (epi == GEPI_F32 && split) rc = RING_A(GEPI_F32, 1);
   else if (epi == GEPI_F32) RING(GEPI_F32);
   else if (epi == GEPI_RESID) RING(GEPI_RESID);
   else if (epi == GEPI_TANHNORM) RING(GEPI_TANHNORM);
+  else if (epi == GEPI_ACT) RING(GEPI_ACT);
   else if (epi == GEPI_QKV) RING(GEPI_QKV);
   else if (two_per_cu && epi == GEPI_UNEMBED) rc = RING_P(GEPI_UNEMBED);
   else if (epi == GEPI_UNEMBED) {
@@ -1229,7 +1231,7 @@ static int sdot_set_attributes() {
   if (done) return IXT_OK;
 #define SATTR(E_, N_) HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_sdot<E_, N_>), hipFuncAttributeMaxDynamicSharedMemorySize, 156 * 1024))
   SATTR(GEPI_QKV, true); SATTR(GEPI_QKV, false); SATTR(GEPI_RESID, true); SATTR(GEPI_RESID, false);
-  SATTR(GEPI_SWIGLU, true); SATTR(GEPI_SWIGLU, false); SATTR(GEPI_F32, true); SATTR(GEPI_F32, false); SATTR(GEPI_TANHNORM, false);
+  SATTR(GEPI_SWIGLU, true); SATTR(GEPI_SWIGLU, false); SATTR(GEPI_F32, true); SATTR(GEPI_F32, false); SATTR(GEPI_TANHNORM, false); SATTR(GEPI_ACT, false);
 #undef SATTR
   done = true;
   return IXT_OK;
@@ -1255,6 +1257,7 @@ int launch_sdot(ixt_ctx* c, int epi, bool norm, const bf16_t* x, const bf16_t* s
   else if (epi == GEPI_SWIGLU) rc = norm ? sdot_t<GEPI_SWIGLU, true>(a, p, st) : sdot_t<GEPI_SWIGLU, false>(a, p, st);
   else if (epi == GEPI_F32) rc = norm ? sdot_t<GEPI_F32, true>(a, p, st) : sdot_t<GEPI_F32, false>(a, p, st);
   else if (epi == GEPI_TANHNORM && !norm) rc = sdot_t<GEPI_TANHNORM, false>(a, p, st);
+  else if (epi == GEPI_ACT && !norm) rc = sdot_t<GEPI_ACT, false>(a, p, st);
   timing_end(c, st, ti);
   return rc;
 }

@@ -122,6 +122,8 @@ __device__ __forceinline__ float ixt_glu(int kind, float a, float b, float limit
   const float z = kind == 2 ? 1.59576912160573071176f * fmaf(0.044715f * a * a, a, a) : a;
   return a * hw_rcp(1.0f + hw_exp2(-1.44269504088896340736f * z)) * b;
 }
+// units without a gate, by kind (from IXT_ACT_RELU2 = 4 on): max(u, 0)^2
+__device__ __forceinline__ float ixt_act(int /*kind*/, float u) { const float p = fmaxf(u, 0.0f); return p * p; }
 // tanh in f32, error below 1e-6 of the value: (1 - e) / (1 + e), e = exp(-2 |x|); |x| < 1/16 by the odd series (next term < 2e-13 relative)
 __device__ __forceinline__ float tanh_f32(float x) {
   const float a = fabsf(x), w = a * a, e = hw_exp2(-2.88539008177792681472f * a);

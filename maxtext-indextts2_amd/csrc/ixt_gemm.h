@@ -22,13 +22,14 @@
 //   GEPI_RESID    h_out = bf16(h_in + bf16(t))                                   (llama2.py:127, :157)
 //   GEPI_SWIGLU   act = bf16(bf16(silu(bf16(t_0))) * bf16(t_1))                  (linears.py:449-464); the fused wi kernel stores
 //                 wi_0 tile j and wi_1 tile j as column tiles 2j, 2j+1, so both gates of a feature are in one wave
+//   GEPI_ACT      act = bf16(unit(t)), a unit without a gate (ixt_act)
 //   GEPI_TANHNORM residual and norms of a decoder with tanh norms (TanhNormEpi)
 //   GEPI_QKV      bf16(t), RoPE (embeddings.py:277-315), q -> qbuf, k / v -> the row's page (paged_attention.py:446-471).  Q and K
 //                 head columns are stored pair-interleaved (qk_col): a 16-column tile holds features 8j..8j+7 and half+8j..half+8j+7,
 //                 so the two RoPE partners of a feature sit in lanes l and l ^ 32 of one accumulator register.
 #pragma once
 
-enum { GEPI_F32 = 0, GEPI_UNEMBED = 1, GEPI_RESID = 2, GEPI_SWIGLU = 3, GEPI_QKV = 4, GEPI_TANHNORM = 5 };
+enum { GEPI_F32 = 0, GEPI_UNEMBED = 1, GEPI_RESID = 2, GEPI_SWIGLU = 3, GEPI_QKV = 4, GEPI_TANHNORM = 5, GEPI_ACT = 6 };
 
 // GEPI_TANHNORM: an f32 residual stream between tanh norms, x <- x + post(t), act = bf16(pre(x)), norm(y) = tanh(alpha y) w + b feature by feature (w
 // null: no norm).  Nothing in it looks at a row's other features, so it needs no launch of its own.
@@ -81,7 +82,7 @@ struct GemmEpi {
   float* out;                                           // F32: [slices][R][N]; UNEMBED: rounded logits [R][N] or nullptr
   float* amax_val; int32_t* amax_idx; ColRanges cr;     // UNEMBED: [R][WC ncolg]
   const bf16_t* h_in; bf16_t* h_out;                    // RESID: [R][N] row-major
-  bf16_t* act;                                          // SWIGLU: [R][N/2] in xidx layout
+  bf16_t* act;                                          // SWIGLU: [R][N/2] in xidx layout; ACT: [R][N]
   const int32_t* row_slot; const int32_t* row_pos; const int32_t* row_active; const int32_t* page_map;   // QKV
   const bf16_t* rope_sin; const bf16_t* rope_cos;
   bf16_t* qbuf; bf16_t* kpages; bf16_t* vpages;
@@ -89,7 +90,7 @@ struct GemmEpi {
   const float* xscale; const float* wscale;             // F8: activation scales [rows][chains], column scales [N] (ixt_fp8.h)
   size_t sstride;                                       // F8 + routed experts: floats between two experts' column scales
   TanhNormEpi tn;                                       // TANHNORM (with act)
-  int glu; float glu_limit;                             // SWIGLU: glu != 0 takes that gated unit of the f32 totals instead (ixt_glu)
+  int glu; float glu_limit;                             // ACT: the unit's kind; SWIGLU: glu != 0 takes that gated unit of the f32 totals instead (ixt_glu)
   const int32_t* rb_exp; size_t wstride;                // routed experts: expert of every 16-row block (-1: none), 16-byte units between experts' kernels
 };
 
@@ -326,6 +327,20 @@ __global__ __launch_bounds__(WR * WC * 64, 2) void k_gemm_ring(const u32x4* __re
       for (int b = 0; b < RB; ++b) {
         const int row = (rowg * TR + wr * RB + b) * 16 + r_in;
         if (tile < ntile && row < R) tanhnorm_epi(e.tn, e.act, row, tile * 16 + cq * 4, tot[i][b]);
+      }
+    }
+  } else if constexpr (EPI == GEPI_ACT) {
+#pragma unroll
+    for (int i = 0; i < CT; ++i) {
+      const int tile = colg * TC + wc * CT + i;
+#pragma unroll
+      for (int b = 0; b < RB; ++b) {
+        const int row = (rowg * TR + wr * RB + b) * 16 + r_in;
+        if (tile < ntile && row < R) {
+          uint2 ov;
+          ov.x = pack2(f2bf(ixt_act(e.glu, tot[i][b][0])), f2bf(ixt_act(e.glu, tot[i][b][1]))); ov.y = pack2(f2bf(ixt_act(e.glu, tot[i][b][2])), f2bf(ixt_act(e.glu, tot[i][b][3])));
+          *reinterpret_cast<uint2*>(e.act + xidx(row, tile * 16 + cq * 4, N)) = ov;
+        }
       }
     }
   } else if constexpr (EPI == GEPI_SWIGLU) {

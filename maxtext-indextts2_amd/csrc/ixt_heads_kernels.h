@@ -1,29 +1,35 @@
 // ixt_heads_kernels.h -- attention of hybrid decoders over keys and values per head (IXT_MIX_ATTENTION): query heads in equal groups on one key / value
 // head each, optional norm of query and key heads, rotation of a head's first features, optional window, optional sink (a number per head that joins the
-// softmax denominator without a key or a value).  Sizes of keys and values are independent.
+// softmax denominator without a key or a value), optional soft cap of the scores, optional gate on the concatenated heads.  Sizes of keys and values are
+// independent.  With two maps a head has two queries and its key head two keys per token, both of `d` features, over the same values; the two outputs
+// become one: a1 - lambda a2, over its root mean square, times a constant (differential attention).
 //
 //   k_heads_prep     projection slices -> queries [R][H][dkp], the row's keys and values in their pages
 //   k_heads_prompt   many rows, bf16, matrix cores
 //   k_heads_decode   few rows, bf16, matrix cores, keys split over blocks (+ k_heads_combine)
 //   k_heads_any      any sizes, any T
 //
-// Pages: [page][kv head][token][dkp] and [page][kv head][token][dvp]; what lies behind the real features is zero from the pool's creation on.
+// Pages: [page][kv head][token][dkp] (the maps dmp apart in a row) and [page][kv head][token][dvp]; what lies behind the real features is zero from the
+// pool's creation on.
 #pragma once
 #include "ixt_hybrid_kernels.h"
 
 struct HeadsGeom {
   int H, G, d, dv, rot, P, mpg, window;     // query heads, key / value heads, key and value dims, rotated dims, page size, pages per group, window (<= 0: none)
   int dkp, dvp;                             // padded key / value rows
-  int hs, vs, ok, ov;                       // projection columns: a query / key head takes hs, a value head vs; keys from ok on, values from ov on
-  float scale;
+  int maps, dmp;                            // softmax maps per head (1, 2); a map's part of a key row: dkp = maps dmp
+  int hs, vs, ok, ov, og;                   // projection columns: a map of a query / key head takes hs, a value head vs; keys from ok on, values from ov on, gates
+                                            // (vs per query head) from og on (< 0: none)
+  float scale, cap;                         // cap > 0: score <- cap tanh(score / cap)
 };
+struct MapsArgs { const float* lambda; float keep, eps; };               // two maps: (a1 - *lambda a2) / rms(., eps) keep
 struct RowsArgs { const int32_t *slot, *pos, *active, *page_map; };      // the rows of a pass
 
 // A query or key head (columns c0 .. of row r of the projection) by LP lanes, four features each at a time: norm by w (nullptr: none), rotation;
 // emit(f, o): features f .. f + 3 of the n asked for (zeros behind the head's own).  rope: f32 [position][rot / 2] cos, sin.
 struct HeadsRope { const float *cos, *sin; };
-template <int LP, typename F>
-__device__ __forceinline__ void head_norm_rotate(const Slices& t, int r, int c0, const HeadsGeom& g, const float* __restrict__ w, float eps, HeadsRope rope, int pos, int n, int sl, F emit) {
+template <int LP, typename G, typename F>
+__device__ __forceinline__ void head_norm_rotate(const Slices& t, int r, int c0, const G& g, const float* __restrict__ w, float eps, HeadsRope rope, int pos, int n, int sl, F emit) {
   float v[4] = {0.0f, 0.0f, 0.0f, 0.0f}, rs = 1.0f;
   if (sl * 4 < g.hs) t.at4(r, c0 + sl * 4, v);              // (columns d .. hs - 1 are zero)
   if (w != nullptr) {
@@ -61,25 +67,43 @@ __device__ __forceinline__ void head_norm_rotate(const Slices& t, int r, int c0,
     emit(f, o);
   }
 }
-// LP lanes per head (16, 32, 64): queries [R][H][dkp], and the row's keys and values in their pages.  grid (R, ceil((H + 2 G) LP / 256)), block 256.
+// lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff.  One wave.
+static __global__ __launch_bounds__(64) void k_maps_lambda(const float* lq1, const float* lk1, const float* lq2, const float* lk2, int n, float diff, float* lambda) {
+  float a = 0.0f, b = 0.0f;
+  for (int i = threadIdx.x; i < n; i += 64) { a = fmaf(lq1[i], lk1[i], a); b = fmaf(lq2[i], lk2[i], b); }
+  a = wave_sum(a); b = wave_sum(b);
+  if (threadIdx.x == 0) *lambda = expf(a) - expf(b) + diff;
+}
+// four columns of the concatenated heads (c % 4 == 0 inside head h) times their gate
+__device__ __forceinline__ void heads_gate4(const Slices& t, int r, const HeadsGeom& g, int h, int c, float* v) {
+  float z[4];
+  t.at4(r, g.og + h * g.vs + c, z);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] *= hw_rcp(1.0f + hw_exp2(-1.44269504088896340736f * z[j]));
+}
+// log2(e) times the capped score, cap (1 - 2 / (1 + exp(2 s scale / cap))): c2 = 2 scale log2(e) / cap, k2 = cap log2(e)
+__device__ __forceinline__ float capped_log2(float s, float c2, float k2) { return fmaf(-2.0f * k2, hw_rcp(1.0f + hw_exp2(c2 * s)), k2); }
+
+// LP lanes per map of a head (16, 32, 64): queries [R][H][maps][dmp], and the row's keys and values in their pages.  grid (R, ceil((maps (H + G) + G) LP /
+// 256)), block 256.
 template <typename T, int LP>
 __global__ __launch_bounds__(256) void k_heads_prep(Slices t, HeadsGeom g, const float* __restrict__ qn, const float* __restrict__ kn, float eps, HeadsRope rope, RowsArgs rows,
                                                     T* __restrict__ kpages, T* __restrict__ vpages, T* __restrict__ q) {
-  const int r = blockIdx.x, j = blockIdx.y * (256 / LP) + threadIdx.x / LP, sl = threadIdx.x % LP;
-  if (j >= g.H + 2 * g.G) return;
+  const int r = blockIdx.x, j = blockIdx.y * (256 / LP) + threadIdx.x / LP, sl = threadIdx.x % LP, QU = g.H * g.maps, KU = g.G * g.maps;
+  if (j >= QU + KU + g.G) return;
   const bool act = rows.active[r] != 0;
-  if (!act && j >= g.H) return;
+  if (!act && j >= QU) return;
   const int pos = act ? rows.pos[r] : 0;
-  if (j < g.H) {
-    T* o = q + ((size_t)r * g.H + j) * g.dkp;
-    head_norm_rotate<LP>(t, r, j * g.hs, g, qn, eps, rope, pos, g.dkp, sl, [&](int f, const float* v) { store4(o + f, v); });
+  if (j < QU) {
+    T* o = q + ((size_t)r * QU + j) * g.dmp;
+    head_norm_rotate<LP>(t, r, j * g.hs, g, qn, eps, rope, pos, g.dmp, sl, [&](int f, const float* v) { store4(o + f, v); });
     return;
   }
-  const int kh = (j - g.H) % g.G;
+  const int ku = j - QU, kh = ku < KU ? ku / g.maps : ku - KU;
   const size_t at = ((size_t)rows.page_map[(size_t)rows.slot[r] * g.mpg + pos / g.P] * g.G + kh) * g.P + pos % g.P;          // row of the key / value pools
-  if (j < g.H + g.G) {
-    T* o = kpages + at * g.dkp;
-    head_norm_rotate<LP>(t, r, g.ok + kh * g.hs, g, kn, eps, rope, pos, g.hs, sl, [&](int f, const float* v) { store4(o + f, v); });
+  if (ku < KU) {
+    T* o = kpages + at * g.dkp + ku % g.maps * g.dmp;
+    head_norm_rotate<LP>(t, r, g.ok + ku * g.hs, g, kn, eps, rope, pos, g.hs, sl, [&](int f, const float* v) { store4(o + f, v); });
     return;
   }
   T* o = vpages + at * g.dvp;
@@ -91,10 +115,11 @@ __global__ __launch_bounds__(256) void k_heads_prep(Slices t, HeadsGeom g, const
 }
 
 // Any sizes (dv <= 1024), any T: block = (row, head); thread = key for the scores (tiles of 256 keys, running maximum and sum, the sink as their start),
-// thread = value column for the weighted sum.  out: act(T), column h vs + c.  grid (R, H), block 256, LDS = (dkp + 256) floats.
+// thread = value column for the weighted sum; two maps one after the other.  t: the projection (gates).  out: act(T), column h vs + c.  grid (R, H), block
+// 256, LDS = (dkp + 256) floats.
 template <typename T>
 __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, HeadsGeom g, const float* __restrict__ sink, RowsArgs rows, const T* __restrict__ kpages,
-                                                   const T* __restrict__ vpages, T* __restrict__ out, int Kp) {
+                                                   const T* __restrict__ vpages, MapsArgs mp, Slices t, T* __restrict__ out, int Kp) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   __shared__ float red[4];
   const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, kh = h / (g.H / g.G);
@@ -105,15 +130,19 @@ __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, Hea
   __syncthreads();
   const int pos = rows.pos[r], k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
   const int32_t* prow = rows.page_map + (size_t)rows.slot[r] * g.mpg;
+  float o[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int mi = 0; mi < g.maps; ++mi) {
+  const float* qm = q + mi * g.dmp;
   float m = sink != nullptr ? sink[h] : -INFINITY, l = sink != nullptr ? 1.0f : 0.0f, acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   for (int j0 = k_lo; j0 <= pos; j0 += 256) {
     const int j = j0 + tid;
     float s = -INFINITY;
     if (j <= pos) {
-      const T* kp = kpages + (((size_t)prow[j / g.P] * g.G + kh) * g.P + j % g.P) * g.dkp;
+      const T* kp = kpages + (((size_t)prow[j / g.P] * g.G + kh) * g.P + j % g.P) * g.dkp + mi * g.dmp;
       float a = 0.0f;
-      for (int k = 0; k < g.d; ++k) a = fmaf(q[k], to_f(kp[k]), a);
+      for (int k = 0; k < g.d; ++k) a = fmaf(qm[k], to_f(kp[k]), a);
       s = a * g.scale;
+      if (g.cap > 0.0f) s = g.cap * tanhf(s / g.cap);
     }
     float tm = s;
 #pragma unroll
@@ -140,9 +169,25 @@ __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, Hea
     }
     __syncthreads();
   }
+  const float f = mi == 0 ? 1.0f / l : -*mp.lambda / l;
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
-    if (tid + 256 * i < g.vs) act_store1(out, r, h * g.vs + tid + 256 * i, Kp, tid + 256 * i < g.dv ? acc[i] / l : 0.0f);
+  for (int i = 0; i < 4; ++i) o[i] = mi == 0 ? acc[i] / l : fmaf(acc[i], f, o[i]);
+  }
+  if (g.maps > 1) {
+    float ss = 0.0f;                                        // (columns from dv on are zero)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) ss = fmaf(o[i], o[i], ss);
+    const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)g.dv + mp.eps) * mp.keep;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] *= rs;
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = tid + 256 * i;
+    if (c >= g.vs) continue;
+    if (g.og >= 0 && c < g.dv) o[i] *= f32_sigmoid(t.at(r, g.og + h * g.vs + c));
+    act_store1(out, r, h * g.vs + c, Kp, o[i]);
+  }
   if (h == g.H - 1)
     for (int k = g.H * g.vs + tid; k < Kp; k += 256) act_store1(out, r, k, Kp, 0.0f);
 }
@@ -152,14 +197,16 @@ __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, Hea
 //   scores   D[key][pair] = mfma(A = keys, B = queries): a lane holds 4 keys of one pair per product
 //   weights  running maximum / sum per pair in f32 (they start at the sink), exp2; P goes to bf16
 //   output   D[column][pair] = mfma(A = values read column-wise, B = P)
+// Two maps: pairs become (row, head, map) triples.
 struct HeadsAttnArgs {
   const bf16_t* q; HeadsGeom g; const float* sink;
   RowsArgs rows;
   bf16_t *kpages, *vpages;
   int R, NQ, HB, hchunks, pshift;           // rows per block, query heads per block, blocks of query heads per key / value head
   bf16_t* out; int Kp;                      // act, column h vs + c
-  float *part_o, *part_ml;                  // splits > 1: [R H][splits][dvp], [R H][splits][2]
-  Slices t; const float *qn, *kn; float eps; HeadsRope rope;      // k_heads_decode with FUSED: the projection, and what k_heads_prep needs
+  float *part_o, *part_ml;                  // splits > 1: [R H maps][splits][dvp], [R H maps][splits][2]
+  Slices t; const float *qn, *kn; float eps; HeadsRope rope;      // the projection (gates); k_heads_decode with FUSED: and what k_heads_prep needs
+  MapsArgs mp;
 };
 // the pool row of a key: page (G heads) -> head -> token
 __device__ __forceinline__ int heads_row(const int32_t* __restrict__ prow, int key, int pshift, int G, int kh) {
@@ -170,28 +217,37 @@ __device__ __forceinline__ int heads_row(const int32_t* __restrict__ prow, int k
 // against 29 us for 2048 rows of 16 heads); all waves walk the same key tiles, the next tile arriving while the current one is used.  P stays in registers: with the key order 4q .. 4q + 3, 16 + 4q ..
 // 16 + 4q + 3 per lane group q of 32 keys, the lane's own scores ARE its operand of the next product.  Consecutive blocks are different heads: with
 // 8 heads or a multiple of them, a head's keys and values stay in one XCD's L2.  grid (G hchunks, ceil(R / NQ)), block 256, LDS two tiles.
-template <int DK, int DV>
+// MAPS 2: 32 (row, head) pairs; waves 0 and 1 take their first map, waves 2 and 3 the second (a wave needs one map's part of the keys), and hand its
+// outputs over through LDS at the end.
+template <int DK, int DV, int MAPS>
 __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(HeadsAttnArgs a) {
-  constexpr int NKS = DK / 32, NT = DV / 16, NGV = DV / 64, TILE = 64 * (DK + DV);
+  static_assert(DK % (32 * MAPS) == 0, "whole steps per map");
+  constexpr int NKS = DK / 32 / MAPS, NT = DV / 16, NGV = DV / 64, TILE = 64 * (DK + DV);
   extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
   const HeadsGeom& g = a.g;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
   const int kh = blockIdx.x % g.G, hc = blockIdx.x / g.G, GQ = g.H / g.G;
   const int r0 = blockIdx.y * a.NQ, nr = min(a.NQ, a.R - r0), h0 = kh * GQ + hc * a.HB, hb = min(a.HB, GQ - hc * a.HB);
-  const int pair = wave * 16 + r_in, qi = pair / a.HB, hh = pair % a.HB;
+  const int map = MAPS == 2 ? wave >> 1 : 0, pair = (MAPS == 2 ? wave & 1 : wave) * 16 + r_in, qi = pair / a.HB, hh = pair % a.HB;
   const bool pair_ok = qi < nr && hh < hb;
   const int row = r0 + (pair_ok ? qi : 0), head = h0 + (pair_ok ? hh : 0);
   const bool live = pair_ok && a.rows.active[row] != 0;
   const int pos = live ? a.rows.pos[row] : -1;
   bf16x8 qf[NKS];                                         // queries: lane = pair r_in, 8 consecutive features per step
 #pragma unroll
-  for (int ks = 0; ks < NKS; ++ks) qf[ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.q + ((size_t)row * g.H + head) * DK + ks * 32 + cq * 8));
+  for (int ks = 0; ks < NKS; ++ks)
+    qf[ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a.q + (((size_t)row * g.H + head) * MAPS + map) * (DK / MAPS) + ks * 32 + cq * 8));
   float m = a.sink != nullptr ? a.sink[head] * 1.44269504088896340736f : -INFINITY, l = a.sink != nullptr ? 1.0f : 0.0f;
   f32x4 o[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) o[i] = f32x4(0.0f);
-  const float sc = g.scale * 1.44269504088896340736f;
-  const TileLane L = tile_lane(r_in, cq);
+  const float sc = g.cap > 0.0f ? 1.0f : g.scale * 1.44269504088896340736f, c2 = g.cap > 0.0f ? 2.88539008177792681472f * g.scale / g.cap : 0.0f, k2 = g.cap * 1.44269504088896340736f;
+  TileLane L = tile_lane(r_in, cq);
+  if (map == 1) {                                         // the second map's keys lie NKS steps on in the row (NKS odd: its even steps are the odd ones of a group)
+    const uint32_t k0 = L.k0;
+    L.k0 = (NKS & 1 ? L.k1 : L.k0) + NKS / 2 * 8192;
+    L.k1 = NKS & 1 ? k0 + (NKS / 2 + 1) * 8192 : L.k1 + NKS / 2 * 8192;
+  }
   for (int ra = 0; ra < nr;) {                            // runs of rows that share a page group
     if (!a.rows.active[r0 + ra]) { ++ra; continue; }
     const int slot = a.rows.slot[r0 + ra];
@@ -234,6 +290,12 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
 #pragma unroll
         for (int n = 0; n < 4; ++n) s[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks & 1][n], qf[ks], s[n], 0, 0, 0);
         __builtin_amdgcn_sched_barrier(0);
+      }
+      if (g.cap > 0.0f) {
+#pragma unroll
+        for (int n = 0; n < 4; ++n)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) s[n][j] = capped_log2(s[n][j], c2, k2);
       }
       const int t0 = k_lo + t * 64;
       const bool inside = whole && t0 >= k_all && t0 + 63 <= lo;
@@ -306,12 +368,35 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
       }
     }
   }
+  float inv = 1.0f / l;
+  if constexpr (MAPS == 2) {
+    f32x4* hand = reinterpret_cast<f32x4*>(lds);          // [wave & 1][column tile][lane]
+    __syncthreads();                                      // the last tile has been read
+    if (map == 1) {
+#pragma unroll
+      for (int i = 0; i < NT; ++i) hand[((wave & 1) * NT + i) * 64 + lane] = o[i] * inv;
+    }
+    __syncthreads();
+    if (map == 1) return;
+    const float lambda = *a.mp.lambda;
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const f32x4 o2 = hand[(wave * NT + i) * 64 + lane];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { o[i][j] = fmaf(-lambda, o2[j], o[i][j] * inv); ss = fmaf(o[i][j], o[i][j], ss); }
+    }
+    ss += __shfl_xor(ss, 16, 64);
+    ss += __shfl_xor(ss, 32, 64);
+    inv = a.mp.keep / sqrtf(ss / (float)g.dv + a.mp.eps);
+  }
   if (!live) return;
-  const float inv = 1.0f / l;
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
-    const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
-    if (i * 16 + cq * 4 < g.vs) act_store4(a.out, row, head * g.vs + i * 16 + cq * 4, a.Kp, v);      // (columns dv .. vs - 1 are zero: so are the values there)
+    float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+    if (i * 16 + cq * 4 >= g.vs) continue;
+    if (g.og >= 0) heads_gate4(a.t, row, g, head, i * 16 + cq * 4, v);
+    act_store4(a.out, row, head * g.vs + i * 16 + cq * 4, a.Kp, v);      // (columns dv .. vs - 1 are zero: so are the values there)
   }
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   if (head == g.H - 1)
@@ -323,21 +408,23 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
 // CU and one's loads run under the other's products.  grid (R, G hchunks, splits), block 256.
 // FUSED (every row the only one of its page group): no k_heads_prep in front.  A block takes its queries from the projection while the first tile is on
 // its way; the block with the last tile also takes the row's key and value, keeps them for later passes in their pages and puts them into its tile.
-template <int DK, int DV, bool FUSED>
+// MAPS 2: neighbouring pairs are the two maps of a head; a pair's query is zero on the other map's part of the keys.
+template <int DK, int DV, bool FUSED, int MAPS>
 __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
-  constexpr int NKS = DK / 32, NGV = DV / 64, NH = DV % 64 != 0 ? 1 : 0, OT = NGV + NH;     // column tiles per wave: one of every full group, waves 0 and 1 one of the half group
+  static_assert(DK % (32 * MAPS) == 0, "whole steps per map");
+  constexpr int DM = DK / MAPS, NKM = DM / 32, NKS = DK / 32, NGV = DV / 64, NH = DV % 64 != 0 ? 1 : 0, OT = NGV + NH;     // column tiles per wave: one of every full group, waves 0 and 1 one of the half group
   extern __shared__ __attribute__((aligned(16))) bf16_t tile[];
   __shared__ __attribute__((aligned(16))) bf16_t ps[16][72];
   __shared__ float s_m[4][16], s_l[4][16];
-  __shared__ __attribute__((aligned(16))) bf16_t s_q[FUSED ? 16 : 1][DK + 8], s_k[FUSED ? DK : 8], s_v[FUSED ? DV : 8];
+  __shared__ __attribute__((aligned(16))) bf16_t s_q[FUSED ? 16 : 1][DM + 8], s_k[FUSED ? DK : 8], s_v[FUSED ? DV : 8];
   const HeadsGeom& g = a.g;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
   const int row = blockIdx.x, kh = blockIdx.y % g.G, hc = blockIdx.y / g.G, GQ = g.H / g.G, nsplit = gridDim.z;
-  const int h0 = kh * GQ + hc * a.HB, hb = min(a.HB, GQ - hc * a.HB);
+  const int h0 = kh * GQ + hc * a.HB, hb = min(a.HB, GQ - hc * a.HB), nu = hb * MAPS;
   const int active = a.rows.active[row], pos = a.rows.pos[row], slot = a.rows.slot[row];     // (requested together)
   if (!active) return;
-  const bool pair_ok = r_in < hb;
-  const int head = h0 + (pair_ok ? r_in : 0);
+  const bool pair_ok = r_in < nu;
+  const int u_in = pair_ok ? r_in : 0, map = u_in % MAPS, head = h0 + u_in / MAPS;
   const int32_t* prow = a.rows.page_map + (size_t)slot * g.mpg;
   const int k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0, ntile = (pos - k_lo) / 64 + 1;
   int t = blockIdx.z;
@@ -350,13 +437,14 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
   [[maybe_unused]] const bool last = (ntile - 1) % nsplit == (int)blockIdx.z;       // the row's own key is in one of this block's tiles
   if constexpr (FUSED) {
     const size_t at = ((size_t)prow[pos >> a.pshift] * g.G + kh) * g.P + (pos & (g.P - 1));
-    for (int i = wave; i < hb + (last ? 2 : 0); i += 4) {
-      if (i < hb) {
-        head_norm_rotate<64>(a.t, row, (h0 + i) * g.hs, g, a.qn, a.eps, a.rope, pos, DK, lane, [&](int f, const float* v) { store4(&s_q[i][f], v); });
-      } else if (i == hb) {
-        head_norm_rotate<64>(a.t, row, g.ok + kh * g.hs, g, a.kn, a.eps, a.rope, pos, DK, lane, [&](int f, const float* v) {
-          store4(&s_k[f], v);
-          if (hc == 0 && f < g.hs) store4(a.kpages + at * DK + f, v);
+    for (int i = wave; i < nu + (last ? MAPS + 1 : 0); i += 4) {
+      if (i < nu) {
+        head_norm_rotate<64>(a.t, row, (h0 * MAPS + i) * g.hs, g, a.qn, a.eps, a.rope, pos, DM, lane, [&](int f, const float* v) { store4(&s_q[i][f], v); });
+      } else if (i < nu + MAPS) {
+        const int m_ = i - nu;
+        head_norm_rotate<64>(a.t, row, g.ok + (kh * MAPS + m_) * g.hs, g, a.kn, a.eps, a.rope, pos, DM, lane, [&](int f, const float* v) {
+          store4(&s_k[m_ * DM + f], v);
+          if (hc == 0 && f < g.hs) store4(a.kpages + at * DK + m_ * DM + f, v);
         });
       } else if (lane * 4 < DV) {
         float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
@@ -368,14 +456,17 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     __syncthreads();
   }
 #pragma unroll
-  for (int ks = 0; ks < NKS; ++ks)
-    qf[ks] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(FUSED ? &s_q[pair_ok ? r_in : 0][ks * 32 + cq * 8] : a.q + ((size_t)row * g.H + head) * DK + ks * 32 + cq * 8));
+  for (int ks = 0; ks < NKS; ++ks) {
+    const int km = ks % NKM * 32 + cq * 8;
+    const u32x4 v = *reinterpret_cast<const u32x4*>(FUSED ? &s_q[u_in][km] : a.q + (((size_t)row * g.H + head) * MAPS + map) * DM + km);
+    qf[ks] = __builtin_bit_cast(bf16x8, MAPS == 1 || ks / NKM == map ? v : u32x4(0));
+  }
   f32x4 o[OT];
 #pragma unroll
   for (int i = 0; i < OT; ++i) o[i] = f32x4(0.0f);
   const bool sink = a.sink != nullptr && blockIdx.z == 0;          // counted once
   float m = sink ? a.sink[head] * 1.44269504088896340736f : -INFINITY, l = sink && wave == 0 && cq == 0 ? 1.0f : 0.0f;      // l: this lane's keys only
-  const float sc = g.scale * 1.44269504088896340736f;
+  const float sc = g.scale * 1.44269504088896340736f, c2 = g.cap > 0.0f ? 2.88539008177792681472f * g.scale / g.cap : 0.0f, k2 = g.cap * 1.44269504088896340736f;
   const TileLane L = tile_lane(r_in, cq);
   const uint32_t vl = wave == 0 ? L.v[0] : (wave == 1 ? L.v[1] : (wave == 2 ? L.v[2] : L.v[3]));
   [[maybe_unused]] const uint32_t vh = (wave & 1) ? L.vh[1] : L.vh[0];
@@ -398,7 +489,7 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     float tm = -INFINITY;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      s[j] = k_lo + t * 64 + wave * 16 + cq * 4 + j <= pos ? s[j] * sc : -INFINITY;
+      s[j] = k_lo + t * 64 + wave * 16 + cq * 4 + j <= pos ? (g.cap > 0.0f ? capped_log2(s[j], c2, k2) : s[j] * sc) : -INFINITY;
       tm = fmaxf(tm, s[j]);
     }
     tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
@@ -450,16 +541,37 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
   if (cq == 0) s_l[wave][r_in] = l;
   __syncthreads();
   l = (s_l[0][r_in] + s_l[1][r_in]) + (s_l[2][r_in] + s_l[3][r_in]);
+  float inv = nsplit == 1 ? 1.0f / l : 1.0f;
+  if (MAPS == 2 && nsplit == 1) {                         // the even pair of a head takes both
+    const float lambda = *a.mp.lambda;
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < OT; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float v = o[i][j] * inv;
+        o[i][j] = fmaf(-lambda, __shfl_xor(v, 1, 64), v);
+        if (i < NGV || wave <= 1) ss = fmaf(o[i][j], o[i][j], ss);
+      }
+    ss += __shfl_xor(ss, 16, 64);
+    ss += __shfl_xor(ss, 32, 64);
+    if (cq == 0) s_m[wave][r_in] = ss;
+    __syncthreads();
+    inv = a.mp.keep / sqrtf(((s_m[0][r_in] + s_m[1][r_in]) + (s_m[2][r_in] + s_m[3][r_in])) / (float)g.dv + a.mp.eps);
+    if (map == 1) return;
+  }
   if (!pair_ok) return;
-  const size_t pi = ((size_t)row * g.H + head) * nsplit + blockIdx.z;
-  const float inv = nsplit == 1 ? 1.0f / l : 1.0f;
+  const size_t pi = (((size_t)row * g.H + head) * MAPS + map) * nsplit + blockIdx.z;
 #pragma unroll
   for (int i = 0; i < OT; ++i) {
     if (i == NGV && wave > 1) continue;                   // the half group has two column tiles
     const int c = i * 64 + wave * 16 + cq * 4;
-    const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
-    if (nsplit == 1) { if (c < g.vs) act_store4(a.out, row, head * g.vs + c, a.Kp, v); }
-    else *reinterpret_cast<float4*>(a.part_o + pi * DV + c) = make_float4(v[0], v[1], v[2], v[3]);
+    float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+    if (nsplit == 1) {
+      if (c >= g.vs) continue;
+      if (g.og >= 0) heads_gate4(a.t, row, g, head, c, v);
+      act_store4(a.out, row, head * g.vs + c, a.Kp, v);
+    } else *reinterpret_cast<float4*>(a.part_o + pi * DV + c) = make_float4(v[0], v[1], v[2], v[3]);
   }
   if (nsplit > 1) {
     if (wave == 0 && cq == 0) { a.part_ml[pi * 2] = m; a.part_ml[pi * 2 + 1] = l; }
@@ -468,17 +580,28 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     for (int c = g.H * g.vs + cq * 4; c < a.Kp; c += 16) act_store4(a.out, row, c, a.Kp, z);
   }
 }
-// the key splits of a row's heads put together.  grid (R, H), block 64; nsplit <= 16.
-static __global__ __launch_bounds__(64) void k_heads_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int dvp, int H, int vs,
+// the key splits of a row's heads (and their maps) put together.  grid (R, H), block 64; nsplit <= 16, vs <= 256.
+static __global__ __launch_bounds__(64) void k_heads_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, HeadsGeom g, MapsArgs mp, Slices t,
                                                       const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
-  __shared__ float fac[16];
-  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  __shared__ float fac[2][16];
+  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, c = tid * 4, H = g.H, vs = g.vs, dvp = g.dvp;
   if (!row_active[r]) return;
-  const size_t p0 = ((size_t)r * H + h) * nsplit;
-  split_factors(part_ml + p0 * 2, nsplit, tid, fac);
-  for (int c = tid * 4; c < vs; c += 256) {
-    float v[4];
-    split_sum4(part_o + p0 * dvp + c, dvp, nsplit, fac, v);
+  const size_t p0 = ((size_t)r * H + h) * g.maps * nsplit;
+  for (int m = 0; m < g.maps; ++m) split_factors(part_ml + (p0 + m * nsplit) * 2, nsplit, tid, fac[m]);
+  float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  if (c < vs) split_sum4(part_o + p0 * dvp + c, dvp, nsplit, fac[0], v);
+  if (g.maps == 2) {
+    const float lambda = *mp.lambda;
+    float u[4] = {0.0f, 0.0f, 0.0f, 0.0f}, ss = 0.0f;
+    if (c < vs) split_sum4(part_o + (p0 + nsplit) * dvp + c, dvp, nsplit, fac[1], u);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) { v[j] = fmaf(-lambda, u[j], v[j]); ss = fmaf(v[j], v[j], ss); }
+    const float rs = mp.keep / sqrtf(wave_sum(ss) / (float)g.dv + mp.eps);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] *= rs;
+  }
+  if (c < vs) {
+    if (g.og >= 0) heads_gate4(t, r, g, h, c, v);
     act_store4(out, r, h * vs + c, Kp, v);
   }
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};

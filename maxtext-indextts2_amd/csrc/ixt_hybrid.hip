@@ -1,69 +1,10 @@
 // ixt_hybrid.hip -- host side of IXT_BLOCK_HYBRID: layer plans, weight loading, caches and states, and the forward pass over rows that every engine
 // entry point (prefill chunk, packed rows, decode step) ends in.
-#include "ixt_internal.h"
-#include "ixt_heads_kernels.h"
-#include "ixt_hybrid_kernels.h"
+#include "ixt_hybrid.h"
 
-struct HMat { void* w = nullptr; int K = 0, N = 0, Kp = 0, Np = 0; };       // a dot operand of the ctx's storage type, zero-padded
-struct HLayer {
-  ixt_layer c{};
-  int src = 0;                                   // the layer whose parameters are used
-  LatentGeom lg{};
-  DeltaGeom dg{};
-  HeadsGeom hg{};
-  HMat in, low, o, gu, down;                     // input projection, second low-rank product, output projection, gate | up, down
-  HMat uk, uv;                                   // per-head matrices of a latent layer (heads * wstride elements apart): d -> rank, rank -> v
-  int d_off = 0;                                 // latent layer: column of the latent in the input projection
-  size_t uk_stride = 0, uv_stride = 0, gu_stride = 0, down_stride = 0;
-  NormW n1{}, n1b{}, n2{}, n2b{};                // in front of / behind the mixer, in front of / behind the feed-forward
-  HMat sgu, sdown;                               // a mixture's shared unit
-  float *qn = nullptr, *kn = nullptr, *sink = nullptr, *corr = nullptr;
-  float *cnorm = nullptr, *cq = nullptr, *ck = nullptr, *cv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *onorm = nullptr, *router = nullptr;
-  const float *rope_cos = nullptr, *rope_sin = nullptr;
-  void* pages = nullptr;                         // latent layer: [page][token][rankp + rotp]; attention layer: keys [page][kv head][token][dkp]
-  void* vpages = nullptr;                        // attention layer: values [page][kv head][token][dvp]
-  float *state = nullptr, *tails = nullptr;      // delta layer: [group][H][dv][dp], [group][2][taps - 1][C]
-};
-struct HTensor { std::vector<int64_t> shape; std::function<int(const void*, int, hipStream_t)> load; bool done = false; };   // load empty: accepted, unused
-struct HybridModel {
-  bool f32 = false, recurrent = false;
-  size_t esz = 2;                                // bytes per activation / weight element
-  int E = 0, Ep = 0, V = 0, maxH = 0, kmax_pad = 0, norm_kind = 0, norm_places = 0;      // maxH: most heads of a latent layer
-  float emb_scale = 1.0f, eps = 1e-5f;
-  std::vector<HLayer> layers;
-  std::map<std::string, HTensor> tensors;
-  size_t missing = 0;
-  void* embed = nullptr;
-  HMat head;
-  NormW fnorm{};
-  // workspaces
-  float *x = nullptr, *part2 = nullptr, *h32 = nullptr;      // h32: a routed layer's normed input in f32
-  size_t part2_floats = 0;
-  void *xb = nullptr, *act = nullptr, *hact = nullptr, *xn = nullptr, *qx = nullptr, *qr = nullptr, *olat = nullptr, *xg = nullptr, *mhact = nullptr;
-  float *dq = nullptr, *dk = nullptr, *dkq = nullptr, *dv = nullptr, *dec = nullptr, *beta = nullptr, *dout = nullptr, *mw = nullptr, *msum = nullptr, *po = nullptr, *pml = nullptr;
-  int32_t *midx = nullptr, *mpos = nullptr, *mrb = nullptr;
-  int moe_cap = 0;
-  int32_t *row_seg = nullptr, *row_j = nullptr, *seg = nullptr, *nseg = nullptr, *state_len = nullptr, *parity = nullptr, *claim = nullptr, *err = nullptr, *head_rb = nullptr;
-  // copies of whole groups
-  float** st_bases = nullptr; int64_t* st_per = nullptr; int st_n = 0;
-  char** pg_pools = nullptr; int64_t* pg_bytes = nullptr; int pg_n = 0;
-  float* tap = nullptr; size_t tap_floats = 0;   // residual after every layer, on request
-};
-
-static int up_to(int v, int m) { return (v + m - 1) / m * m; }
 // what one latent row is padded to: the matrix-core kernel's sizes, beyond them multiples of 32 (k_latent_attn_any)
 static int latent_rankp(int rank) { return rank <= 64 ? 64 : rank <= 128 ? 128 : rank <= 256 ? 256 : rank <= 512 ? 512 : up_to(rank, 32); }
 static int latent_rotp(int rot) { return rot <= 32 ? 32 : rot <= 64 ? 64 : up_to(rot, 32); }
-// k_heads_prompt / k_heads_decode: the padded (key, value) sizes they are built for, cheapest first; none fits: k_heads_any
-#define IXT_HEADS_SIZES(X) X(32, 32) X(64, 64) X(64, 128) X(128, 64) X(96, 96) X(128, 128) X(192, 128) X(192, 192) X(256, 256)
-#define IXT_HEADS_SPLIT_BLOCKS 1024              // few rows: blocks that the keys of a launch are split into (four per CU)
-static bool heads_mfma_sizes(int d, int dv, bool f32, int* dkp, int* dvp) {
-  if (f32) return false;
-#define X(DK_, DV_) if (d <= DK_ && dv <= DV_) { *dkp = DK_; *dvp = DV_; return true; }
-  IXT_HEADS_SIZES(X)
-#undef X
-  return false;
-}
 static bool latent_mfma_fits(const HybridModel& m, const LatentGeom& g) { return !m.f32 && g.rankp <= 512 && g.rotp <= 64; }
 
 static int h_alloc(ixt_ctx* c, void** p, size_t bytes) {      // zero-filled: padding behind real columns is never written and must read as zero
@@ -82,6 +23,11 @@ static int h_mat(ixt_ctx* c, HMat* m, int K, int N, size_t copies = 1) {
 static LoadMap load_map(int n, int k, int Kp, int n_off = 0, int k_off = 0) {
   LoadMap m{};
   m.n = n; m.k = k; m.ld = k; m.Kp = Kp; m.n_off = n_off; m.k_off = k_off;
+  return m;
+}
+// of every `group` columns the `rot` from r0 on turn in pairs (ixt_layer.rope_pairs): the kernels want those side by side
+static LoadMap rotated(LoadMap m, const ixt_layer& l, int group, int r0) {
+  if (l.rope_pairs == IXT_ROPE_HALVES && l.rot_dim > 0) { m.rg = group; m.r0 = r0; m.rn = l.rot_dim; }
   return m;
 }
 template <typename T>
@@ -110,29 +56,36 @@ int hybrid_check(const ixt_config& c) {
   if (!c.layers || c.num_decoder_layers < 1) return set_err(IXT_ERR_INVALID, "hybrid decoder: no layers");
   if (c.emb_dim < 1 || c.emb_dim > 12288 || c.vocab_size < 1) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: emb_dim %d (1 .. 12288), vocab_size %d", c.emb_dim, c.vocab_size);
   if (c.fp8_weights) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: fp8 weights are not built");
-  if ((c.norm_kind != IXT_NORM_RMS && c.norm_kind != IXT_NORM_TANH) || c.norm_places < IXT_NORM_BEFORE || c.norm_places > (IXT_NORM_BEFORE | IXT_NORM_AFTER))
+  if (c.norm_kind < IXT_NORM_RMS || c.norm_kind > IXT_NORM_LAYER || c.norm_places < IXT_NORM_BEFORE || c.norm_places > (IXT_NORM_BEFORE | IXT_NORM_AFTER))
     return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: norm kind %d, places %d", c.norm_kind, c.norm_places);
+  if (c.streams < 0 || c.streams > HC_MAX) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: %d streams (at most %d)", c.streams, HC_MAX);
   for (int i = 0; i < c.num_decoder_layers; ++i) {
     const ixt_layer& l = c.layers[i];
+    if (l.rope_pairs != IXT_ROPE_NEIGHBOURS && l.rope_pairs != IXT_ROPE_HALVES) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: rope_pairs %d", i, l.rope_pairs);
     if (l.weights_of >= c.num_decoder_layers || (l.weights_of >= 0 && c.layers[l.weights_of].weights_of >= 0) || l.weights_of == i)
       return set_err(IXT_ERR_INVALID, "layer %d: weights_of %d", i, l.weights_of);
     if (l.heads < 1 || l.dim < 1 || l.vdim < 1) return set_err(IXT_ERR_INVALID, "layer %d: heads / dim / vdim", i);
     if (l.mixer == IXT_MIX_LATENT_ATTENTION) {
-      if (l.kv_rank < 1 || l.kv_rank > 1024 || l.rot_dim < 0 || l.rot_dim % 2) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: kv_rank %d (1 .. 1024), rot_dim %d (even)", i, l.kv_rank, l.rot_dim);
+      if (l.kv_rank < 1 || l.kv_rank > 1024 || l.rot_dim < 0 || l.rot_dim % 2 || l.q_rank < 0)
+        return set_err(IXT_ERR_UNSUPPORTED, "layer %d: kv_rank %d (1 .. 1024), rot_dim %d (even), q_rank %d", i, l.kv_rank, l.rot_dim, l.q_rank);
     } else if (l.mixer == IXT_MIX_GATED_DELTA) {
       if (l.kv_heads < 1 || l.heads % l.kv_heads || l.conv < 1 || l.decay_rank < 1 || l.gate_rank < 1) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / conv / ranks", i);
       if (l.dim > 512) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: delta rule key dims %d (at most 512)", i, l.dim);
     } else if (l.mixer == IXT_MIX_ATTENTION) {
       if (l.kv_heads < 1 || l.heads % l.kv_heads || l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > l.dim) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / rot_dim", i);
+      if (l.maps < 0 || l.maps > 2 || !(l.softcap >= 0.0f)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d maps (1, 2), soft cap %g", i, l.maps, l.softcap);
       if (l.dim > 4096 || l.vdim > 1024) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d key dims (at most 4096), %d value dims (at most 1024)", i, l.dim, l.vdim);
       if (!(l.attn_scale > 0.0f)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: score factor %g (positive)", i, l.attn_scale);
       if (l.rope_factor > 0.0f && !(l.rope_low > 0.0f && l.rope_high > l.rope_low && l.rope_original > 0.0f)) return set_err(IXT_ERR_INVALID, "layer %d: rotation scaling", i);
+    } else if (l.mixer == IXT_MIX_RETENTION) {
+      if (!l.decay || l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > l.dim) return set_err(IXT_ERR_INVALID, "layer %d: decays / rot_dim", i);
+      if (l.dim > 1024 || l.vdim > 1024) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d key dims, %d value dims (at most 1024)", i, l.dim, l.vdim);
     } else return set_err(IXT_ERR_UNSUPPORTED, "layer %d: mixer %d", i, l.mixer);
-    if (l.ffn != IXT_FFN_NONE && (l.glu < IXT_GLU_CLAMPED || l.glu > IXT_GLU_SILU)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: gated unit %d", i, l.glu);
+    if (l.ffn != IXT_FFN_NONE && (l.glu < IXT_GLU_CLAMPED || l.glu > IXT_ACT_RELU2)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: unit %d", i, l.glu);
     if (l.ffn == IXT_FFN_MOE) {
       if (l.experts < 1 || l.experts > 1024 || l.top < 1 || l.top > l.experts || l.ff < 1 || l.shared_ff < 0)
         return set_err(IXT_ERR_UNSUPPORTED, "layer %d: experts %d (1 .. 1024), top %d", i, l.experts, l.top);
-      if (l.router != IXT_ROUTE_SOFTMAX && l.router != IXT_ROUTE_SIGMOID) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: router %d", i, l.router);
+      if (l.router < IXT_ROUTE_SOFTMAX || l.router > IXT_ROUTE_CHOSEN) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: router %d", i, l.router);
       if (l.groups > 1 && (l.experts % l.groups || l.groups_keep < 1 || l.groups_keep > l.groups || l.top > l.experts / l.groups * l.groups_keep))
         return set_err(IXT_ERR_INVALID, "layer %d: %d of %d groups of experts, top %d", i, l.groups_keep, l.groups, l.top);
     } else if (l.ffn == IXT_FFN_DENSE) {
@@ -142,7 +95,7 @@ int hybrid_check(const ixt_config& c) {
   return IXT_OK;
 }
 
-// a norm's tensors: `name`, and for a tanh norm name.alpha (a scalar) and name.b; zeros behind the E features
+// a norm's tensors: `name`, name.b (tanh and layer norms), name.alpha (tanh norms: a scalar); zeros behind the E features
 static int hybrid_norm_params(ixt_ctx* c, const std::string& name, NormW* w) {
   HybridModel* m = c->hy;
   const int E = m->E;
@@ -154,10 +107,8 @@ static int hybrid_norm_params(ixt_ctx* c, const std::string& name, NormW* w) {
     return IXT_OK;
   };
   TRY(one(name, &w->w, E, {E}));
-  if (m->norm_kind == IXT_NORM_TANH) {
-    TRY(one(name + ".alpha", &w->alpha, 1, {}));
-    TRY(one(name + ".b", &w->b, E, {E}));
-  }
+  if (m->norm_kind == IXT_NORM_TANH) TRY(one(name + ".alpha", &w->alpha, 1, {}));
+  if (m->norm_kind != IXT_NORM_RMS) TRY(one(name + ".b", &w->b, E, {E}));
   return IXT_OK;
 }
 
@@ -167,7 +118,7 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
   HLayer& L = m->layers[i];
   const ixt_layer& l = L.c;
   const int E = m->E;
-  const std::string p = "l" + std::to_string(i) + ".";
+  const std::string p = "l" + std::to_string(l.number < 0 ? i : l.number) + ".";
   auto add = [&](const std::string& name, std::vector<int64_t> shape, std::function<int(const void*, int, hipStream_t)> f) { m->tensors[p + name] = HTensor{std::move(shape), std::move(f), false}; };
   auto vec = [&](const std::string& name, float** dst, int64_t n, std::vector<int64_t> shape) -> int {
     TRY(h_allocf(c, dst, (size_t)up_to((int)n, 4)));
@@ -181,15 +132,39 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
   };
   auto mat = [&](const std::string& name, const HMat& M, int n, int k, int n_off, int k_off = 0) { mat_as(name, M, load_map(n, k, M.Kp, n_off, k_off)); };
   auto norm = [&](const std::string& name, NormW* w) -> int { return hybrid_norm_params(c, p + name, w); };
+  auto hyper = [&](const std::string& q, float** dst, bool used) -> int {         // a sublayer's hyper-connection
+    if (m->streams == 0) return IXT_OK;
+    const int S = m->streams;
+    float* d = nullptr;
+    if (used) TRY(h_allocf(c, &d, 2 * HC_MAX + HC_MAX * HC_MAX));
+    *dst = d;
+    const std::vector<std::pair<std::string, LoadMap>> parts = {{"in", load_map(1, S, HC_MAX)}, {"out", load_map(1, S, HC_MAX)}, {"mix", load_map(S, S, HC_MAX)}};
+    for (int j = 0; j < 3; ++j) {
+      const LoadMap lm = parts[j].second;
+      float* to = d + j * HC_MAX;
+      const std::vector<int64_t> shape = j < 2 ? std::vector<int64_t>{S} : std::vector<int64_t>{S, S};
+      if (used) add(q + parts[j].first, shape, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, to, lm, st); });
+      else m->tensors[p + q + parts[j].first] = HTensor{shape, nullptr, true};
+    }
+    return IXT_OK;
+  };
+  TRY(hyper("hc1.", &L.hc1, true));
+  TRY(hyper("hc2.", &L.hc2, l.ffn != IXT_FFN_NONE));
   const bool both = m->norm_places == (IXT_NORM_BEFORE | IXT_NORM_AFTER);
   TRY(norm("norm1", m->norm_places & IXT_NORM_BEFORE ? &L.n1 : &L.n1b));
   if (both) TRY(norm("norm1b", &L.n1b));
   if (l.mixer == IXT_MIX_LATENT_ATTENTION) {
     const LatentGeom& g = L.lg;
     const int NQ = g.H * (g.dn + g.dr);
-    TRY(h_mat(c, &L.in, E, L.d_off + g.rank + g.dr));
-    mat("mix.q", L.in, NQ, E, 0);
-    mat("mix.dkv", L.in, g.rank + g.dr, E, L.d_off);
+    TRY(h_mat(c, &L.in, E, l.out_gate ? L.g_off + g.H * l.vdim : L.d_off + g.rank + g.dr));
+    if (l.q_rank > 0) {
+      mat("mix.dq", L.in, l.q_rank, E, 0);
+      TRY(vec("mix.dq.norm", &L.qnorm, l.q_rank, {l.q_rank}));
+      TRY(h_mat(c, &L.uq, l.q_rank, NQ));
+      mat_as("mix.uq", L.uq, rotated(load_map(NQ, l.q_rank, L.uq.Kp), l, g.dn + g.dr, g.dn));
+    } else mat_as("mix.q", L.in, rotated(load_map(NQ, E, L.in.Kp), l, g.dn + g.dr, g.dn));
+    mat_as("mix.dkv", L.in, rotated(load_map(g.rank + g.dr, E, L.in.Kp, L.d_off), l, g.rank + g.dr, g.rank));
+    if (l.out_gate) mat("mix.g", L.in, g.H * l.vdim, E, L.g_off);
     TRY(vec("mix.dkv.norm", &L.cnorm, g.rank, {g.rank}));
     TRY(h_mat(c, &L.uk, g.dn, g.rankp, g.H));
     TRY(h_mat(c, &L.uv, g.rankp, l.vdim, g.H));
@@ -211,14 +186,57 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     mat("mix.o", L.o, E, g.H * l.vdim, 0);
   } else if (l.mixer == IXT_MIX_ATTENTION) {
     const HeadsGeom& g = L.hg;
-    TRY(h_mat(c, &L.in, E, g.ov + g.G * g.vs));
-    LoadMap q = load_map(g.H * g.d, E, L.in.Kp), k = load_map(g.G * g.d, E, L.in.Kp, g.ok), v = load_map(g.G * g.dv, E, L.in.Kp, g.ov);
+    TRY(h_mat(c, &L.in, E, g.og >= 0 ? g.og + g.H * g.vs : g.ov + g.G * g.vs));
+    LoadMap q = load_map(g.H * g.maps * g.d, E, L.in.Kp), k = load_map(g.G * g.maps * g.d, E, L.in.Kp, g.ok), v = load_map(g.G * g.dv, E, L.in.Kp, g.ov);
     q.ng = k.ng = g.d; q.ngp = k.ngp = g.hs; v.ng = g.dv; v.ngp = g.vs;
-    mat_as("mix.q", L.in, q);
-    mat_as("mix.k", L.in, k);
+    mat_as("mix.q", L.in, rotated(q, l, g.d, 0));
+    mat_as("mix.k", L.in, rotated(k, l, g.d, 0));
     mat_as("mix.v", L.in, v);
-    if (l.qk_norm) { TRY(vec("mix.q.norm", &L.qn, g.d, {g.d})); TRY(vec("mix.k.norm", &L.kn, g.d, {g.d})); }
+    if (g.og >= 0) {
+      LoadMap gm = load_map(g.H * g.dv, E, L.in.Kp, g.og);
+      gm.ng = g.dv; gm.ngp = g.vs;
+      mat_as("mix.g", L.in, gm);
+    }
+    if (g.maps == 2) {                                            // every one of the four vectors works lambda out anew: the last to come leaves the right one
+      const int n = up_to(g.d, 4);
+      TRY(h_allocf(c, &L.maps, (size_t)4 * n)); TRY(h_allocf(c, &L.lambda, 4));
+      const char* names[4] = {"lq1", "lk1", "lq2", "lk2"};
+      float *base = L.maps, *lam = L.lambda;
+      const int d = g.d;
+      const float diff = l.map_diff;
+      for (int j = 0; j < 4; ++j) {
+        float* to = base + (size_t)j * n;
+        add(std::string("mix.") + names[j], {d}, [=](const void* s, int dt, hipStream_t st) -> int {
+          TRY(h_load_vec(s, dt, to, (int64_t)d, st));
+          hipLaunchKernelGGL(k_maps_lambda, dim3(1), dim3(64), 0, st, base, base + n, base + 2 * n, base + 3 * n, d, diff, lam);
+          LAUNCHCHK();
+          return IXT_OK;
+        });
+      }
+    }
+    if (l.qk_norm) {
+      for (int j = 0; j < 2; ++j) {
+        float** dst = j == 0 ? &L.qn : &L.kn;
+        TRY(h_allocf(c, dst, (size_t)up_to(g.d, 4)));
+        float* d = *dst;
+        const LoadMap lm = rotated(load_map(g.d, 1, 1), l, g.d, 0);
+        add(j == 0 ? "mix.q.norm" : "mix.k.norm", {g.d}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, lm, st); });
+      }
+    }
     if (l.sink) TRY(vec("mix.sink", &L.sink, g.H, {g.H}));
+    TRY(h_mat(c, &L.o, g.H * g.vs, E));
+    LoadMap o = load_map(E, g.H * g.dv, L.o.Kp);
+    o.kg = g.dv; o.kgp = g.vs;
+    mat_as("mix.o", L.o, o);
+  } else if (l.mixer == IXT_MIX_RETENTION) {
+    const RetGeom& g = L.rg;
+    TRY(h_mat(c, &L.in, E, g.og + g.H * g.vs));
+    for (const char* t : {"q", "k", "v", "g"}) {
+      const bool qk = *t == 'q' || *t == 'k';
+      LoadMap lm = load_map(g.H * (qk ? g.d : g.dv), E, L.in.Kp, *t == 'q' ? 0 : *t == 'k' ? g.ok : *t == 'v' ? g.ov : g.og);
+      lm.ng = qk ? g.d : g.dv; lm.ngp = qk ? g.hs : g.vs;
+      mat_as(std::string("mix.") + t, L.in, qk ? rotated(lm, l, g.d, 0) : lm);
+    }
     TRY(h_mat(c, &L.o, g.H * g.vs, E));
     LoadMap o = load_map(E, g.H * g.dv, L.o.Kp);
     o.kg = g.dv; o.kgp = g.vs;
@@ -248,33 +266,44 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     for (const char* n : {"norm2", "norm2b"}) {
       if (!both && std::string(n) == "norm2b") continue;
       m->tensors[p + n] = HTensor{{E}, nullptr, true};
-      if (m->norm_kind == IXT_NORM_TANH) { m->tensors[p + n + ".alpha"] = HTensor{{}, nullptr, true}; m->tensors[p + n + ".b"] = HTensor{{E}, nullptr, true}; }
+      if (m->norm_kind == IXT_NORM_TANH) m->tensors[p + n + ".alpha"] = HTensor{{}, nullptr, true};
+      if (m->norm_kind != IXT_NORM_RMS) m->tensors[p + n + ".b"] = HTensor{{E}, nullptr, true};
     }
     return IXT_OK;
   }
   TRY(norm("norm2", m->norm_places & IXT_NORM_BEFORE ? &L.n2 : &L.n2b));
   if (both) TRY(norm("norm2b", &L.n2b));
+  const bool gated = l.glu < IXT_ACT_RELU2;
   auto unit = [&](const std::string& q, const HMat& gu, const HMat& down, int ff, size_t gu_off = 0, size_t down_off = 0) {
-    LoadMap gate = load_map(ff, E, gu.Kp), up = load_map(ff, E, gu.Kp, 1);
-    gate.inter = up.inter = 1;
-    mat_as(q + "gate", gu, gate, gu_off);
-    mat_as(q + "up", gu, up, gu_off);
+    if (gated) {
+      LoadMap gate = load_map(ff, E, gu.Kp), up = load_map(ff, E, gu.Kp, 1);
+      gate.inter = up.inter = 1;
+      mat_as(q + "gate", gu, gate, gu_off);
+      mat_as(q + "up", gu, up, gu_off);
+    } else mat_as(q + "up", gu, load_map(ff, E, gu.Kp), gu_off);
     mat_as(q + "down", down, load_map(E, ff, down.Kp), down_off);
   };
   const bool moe = l.ffn == IXT_FFN_MOE;
   const int n = moe ? l.experts : 1;
-  TRY(h_mat(c, &L.gu, E, 2 * up_to(l.ff, IXT_KALIGN), n));
+  TRY(h_mat(c, &L.gu, E, (gated ? 2 : 1) * up_to(l.ff, IXT_KALIGN), n));
   TRY(h_mat(c, &L.down, l.ff, E, n));
   L.gu_stride = (size_t)L.gu.Kp * L.gu.Np; L.down_stride = (size_t)L.down.Kp * L.down.Np;
   for (int e = 0; e < n; ++e) unit(moe ? "mlp.e" + std::to_string(e) + "." : "mlp.", L.gu, L.down, l.ff, e * L.gu_stride, e * L.down_stride);
   if (!moe) return IXT_OK;
   if (l.shared_ff > 0) {
-    TRY(h_mat(c, &L.sgu, E, 2 * up_to(l.shared_ff, IXT_KALIGN)));
+    TRY(h_mat(c, &L.sgu, E, (gated ? 2 : 1) * up_to(l.shared_ff, IXT_KALIGN)));
     TRY(h_mat(c, &L.sdown, l.shared_ff, E));
     unit("mlp.shared.", L.sgu, L.sdown, l.shared_ff);
   }
-  TRY(h_allocf(c, &L.router, (size_t)l.experts * m->Ep));
+  const bool sg = l.shared_ff > 0 && l.shared_gate;
+  TRY(h_allocf(c, &L.router, (size_t)(l.experts + sg) * m->Ep));
   float* d = L.router;
+  if (sg) {                                                       // one more row behind the experts
+    float* dg = d + (size_t)l.experts * m->Ep;
+    const LoadMap lg = load_map(1, E, m->Ep);
+    add("mlp.shared.sg", {1, E}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, dg, lg, st); });
+  }
+  if (l.router_bias) TRY(vec("mlp.router.b", &L.bias, l.experts, {l.experts}));
   const LoadMap lm = load_map(l.experts, E, m->Ep);
   add("mlp.router", {l.experts, E}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, lm, st); });
   if (l.router_correction) TRY(vec("mlp.correction", &L.corr, l.experts, {l.experts}));
@@ -313,18 +342,22 @@ int hybrid_init(ixt_ctx* c) {
   HybridModel* m = c->hy;
   m->f32 = cf.float32 != 0; m->esz = m->f32 ? 4 : 2;
   m->E = cf.emb_dim; m->Ep = up_to(m->E, IXT_KALIGN); m->V = cf.vocab_size; m->emb_scale = cf.embedding_scale; m->eps = cf.normalization_layer_epsilon;
-  m->norm_kind = cf.norm_kind; m->norm_places = cf.norm_places;
+  m->norm_kind = cf.norm_kind; m->norm_places = cf.norm_places; m->streams = cf.streams; m->tied = cf.logits_via_embedding != 0; m->logit_scale = cf.logit_scale;
   const int n = cf.num_decoder_layers, R = c->Rmax, Rp = up_to(R, 128);
   m->layers.resize(n);
   TRY(h_alloc(c, &m->embed, (size_t)m->V * m->E * m->esz));
-  { void* d = m->embed; const int64_t ne = (int64_t)m->V * m->E; const bool f = m->f32;
-    m->tensors["embed"] = HTensor{{m->V, m->E}, [=](const void* s, int dt, hipStream_t st) { return f ? h_load_vec(s, dt, (float*)d, ne, st) : h_load_vec(s, dt, (bf16_t*)d, ne, st); }, false}; }
   TRY(h_mat(c, &m->head, m->E, m->V));
-  { void* d = m->head.w; const LoadMap lm = load_map(m->V, m->E, m->head.Kp);
-    m->tensors["head"] = HTensor{{m->V, m->E}, [=](const void* s, int dt, hipStream_t st) { return h_load_mat(m, s, dt, d, lm, st); }, false}; }
+  { void *d = m->embed, *dh = m->head.w; const int64_t ne = (int64_t)m->V * m->E; const bool f = m->f32, tied = m->tied; const LoadMap lm = load_map(m->V, m->E, m->head.Kp);
+    auto head = [=](const void* s, int dt, hipStream_t st) { return h_load_mat(m, s, dt, dh, lm, st); };
+    m->tensors["embed"] = HTensor{{m->V, m->E}, [=](const void* s, int dt, hipStream_t st) -> int {
+      if (tied) TRY(head(s, dt, st));                              // (twice in memory: rows for the lookup, the dot's order for the logits)
+      return f ? h_load_vec(s, dt, (float*)d, ne, st) : h_load_vec(s, dt, (bf16_t*)d, ne, st);
+    }, false};
+    if (!tied) m->tensors["head"] = HTensor{{m->V, m->E}, head, false}; }
   TRY(hybrid_norm_params(c, "final.norm", &m->fnorm));
   std::map<std::vector<float>, std::pair<float*, float*>> ropes;
-  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0;
+  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0, ret_u = 0;
+  const size_t max_chunks = (size_t)R / SEG_CHUNK + (size_t)std::min(R, c->G) + 1;      // of a pass: a group has at most one run of rows
   auto upd = [](size_t& a, size_t v) { if (v > a) a = v; };
   // f32 slices of a dot over at most R rows (split-K only below 128 rows; launch_dot keeps to one slice when the slices do not fit)
   auto dotsz = [&](int K, int N) { upd(part, std::max((size_t)R * N, (size_t)std::min(R, 128) * N * ((K + IXT_CHAIN - 1) / IXT_CHAIN))); };
@@ -337,12 +370,19 @@ int hybrid_init(ixt_ctx* c) {
       LatentGeom& g = L.lg;
       g.H = l.heads; g.dn = l.dim; g.dr = l.rot_dim; g.rank = l.kv_rank; g.P = c->P; g.mpg = c->mpg; g.window = l.window; g.scale = l.attn_scale;
       g.rankp = latent_rankp(l.kv_rank); g.rotp = latent_rotp(l.rot_dim);
-      L.d_off = up_to(g.H * (g.dn + g.dr), 16);
+      const int NQ = up_to(g.H * (g.dn + g.dr), 16);
+      L.d_off = l.q_rank > 0 ? up_to(l.q_rank, 16) : NQ;
+      L.g_off = L.d_off + up_to(g.rank + g.dr, 16);
       TRY(h_alloc(c, &L.pages, (size_t)cf.pagedattn_num_pages * c->P * (g.rankp + g.rotp) * m->esz));
       TRY(hybrid_rope(c, l, &ropes, &L));
       m->maxH = std::max(m->maxH, g.H);
       const int dnp = up_to(g.dn, IXT_KALIGN), ukn = up_to(g.rankp, 16), kp = up_to(g.rankp, IXT_KALIGN), uvn = up_to(l.vdim, 16);
-      dotsz(m->Ep, up_to(L.d_off + g.rank + g.dr, 16));
+      {                                                                     // (with a query latent or a gate it stays in use beside the dots behind it)
+        const int N = up_to(l.out_gate ? L.g_off + g.H * l.vdim : L.d_off + g.rank + g.dr, 16);
+        dotsz(m->Ep, N);
+        if (l.out_gate || l.q_rank > 0) upd(part2, std::max((size_t)R * N, (size_t)std::min(R, 128) * N * ((m->Ep + IXT_CHAIN - 1) / IXT_CHAIN)));
+        if (l.q_rank > 0) { dotsz(up_to(l.q_rank, IXT_KALIGN), NQ); upd(act_k, up_to(l.q_rank, IXT_KALIGN)); }
+      }
       upd(part, (size_t)g.H * Rp * ukn);                                    // several slices only below 128 rows
       upd(part, (size_t)g.H * up_to(std::min(R, 128), 16) * ukn * ((dnp + IXT_CHAIN - 1) / IXT_CHAIN));
       upd(part, (size_t)g.H * Rp * uvn);
@@ -354,18 +394,38 @@ int hybrid_init(ixt_ctx* c) {
     } else if (l.mixer == IXT_MIX_ATTENTION) {
       HeadsGeom& g = L.hg;
       g.H = l.heads; g.G = l.kv_heads; g.d = l.dim; g.dv = l.vdim; g.rot = l.rot_dim; g.P = c->P; g.mpg = c->mpg; g.window = l.window; g.scale = l.attn_scale;
-      if (!heads_mfma_sizes(l.dim, l.vdim, m->f32, &g.dkp, &g.dvp)) { g.dkp = up_to(l.dim, 32); g.dvp = up_to(l.vdim, 32); }
-      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4); g.ok = up_to(g.H * g.hs, 16); g.ov = g.ok + up_to(g.G * g.hs, 16);
+      g.maps = std::max(l.maps, 1); g.cap = l.softcap;
+      if (!heads_mfma_sizes(l.dim, g.maps, l.vdim, m->f32, &g.dkp, &g.dvp)) { g.dkp = g.maps * up_to(l.dim, 32); g.dvp = up_to(l.vdim, 32); }
+      g.dmp = g.dkp / g.maps;
+      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4); g.ok = up_to(g.H * g.maps * g.hs, 16); g.ov = g.ok + up_to(g.G * g.maps * g.hs, 16);
+      g.og = l.out_gate ? g.ov + up_to(g.G * g.vs, 16) : -1;
       const size_t tokens = (size_t)cf.pagedattn_num_pages * c->P * g.G;
       if (tokens > (size_t)INT32_MAX) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %zu cached heads in the page pool", i, tokens);
       TRY(h_alloc(c, &L.pages, tokens * g.dkp * m->esz));
       TRY(h_alloc(c, &L.vpages, tokens * g.dvp * m->esz));
       TRY(hybrid_rope(c, l, &ropes, &L));
-      dotsz(m->Ep, up_to(g.ov + g.G * g.vs, 16));
+      dotsz(m->Ep, up_to(g.og >= 0 ? g.og + g.H * g.vs : g.ov + g.G * g.vs, 16));
       dotsz(up_to(g.H * g.vs, IXT_KALIGN), up_to(m->E, 16));
       upd(act_k, up_to(g.H * g.vs, IXT_KALIGN));
       upd(qx_e, (size_t)R * g.H * g.dkp);
       upd(po, (size_t)IXT_HEADS_SPLIT_BLOCKS * 16 * g.dvp);
+    } else if (l.mixer == IXT_MIX_RETENTION) {
+      m->recurrent = true;
+      RetGeom& g = L.rg;
+      g.H = l.heads; g.d = l.dim; g.dv = l.vdim; g.dp = up_to(l.dim, 16); g.dvp = up_to(l.vdim, 16); g.rot = l.rot_dim;
+      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4);
+      g.ok = up_to(g.H * g.hs, 16); g.ov = 2 * g.ok; g.og = g.ov + up_to(g.H * g.vs, 16);
+      TRY(h_allocf(c, &L.state, (size_t)c->G * g.H * g.dp * g.dvp));
+      TRY(hybrid_rope(c, l, &ropes, &L));
+      std::vector<float> pw((size_t)g.H * (SEG_CHUNK + 1));
+      for (int h = 0; h < g.H; ++h)
+        for (int j = 0; j <= SEG_CHUNK; ++j) pw[(size_t)h * (SEG_CHUNK + 1) + j] = (float)pow(l.decay[h], j);
+      TRY(h_allocf(c, &L.pow, pw.size()));
+      HIPCHK(hipMemcpy(L.pow, pw.data(), pw.size() * 4, hipMemcpyHostToDevice));
+      dotsz(m->Ep, up_to(g.og + g.H * g.vs, 16));
+      dotsz(up_to(g.H * g.vs, IXT_KALIGN), up_to(m->E, 16));
+      upd(act_k, up_to(g.H * g.vs, IXT_KALIGN));
+      upd(s_q, (size_t)R * g.H * g.dp); upd(s_v, (size_t)R * g.H * g.dvp); upd(ret_u, max_chunks * g.H * g.dp * g.dvp);
     } else {
       m->recurrent = true;
       DeltaGeom& g = L.dg;
@@ -413,7 +473,8 @@ int hybrid_init(ixt_ctx* c) {
   upd(part, (size_t)c->NLmax * m->head.Np * (c->NLmax < 128 ? (m->head.Kp + IXT_CHAIN - 1) / IXT_CHAIN : 1));
   c->part_floats = part; TRY(h_allocf(c, &c->part, part));
   m->part2_floats = part2; TRY(h_allocf(c, &m->part2, part2 + 4));
-  TRY(h_allocf(c, &m->x, (size_t)R * m->E));
+  TRY(h_allocf(c, &m->x, (size_t)R * std::max(1, m->streams) * m->E));
+  TRY(h_allocf(c, &m->ret_u, ret_u + 4)); TRY(h_allocf(c, &m->chunk, max_chunks)); TRY(h_allocf(c, &m->sgate, (size_t)R + 4));
   TRY(h_alloc(c, &m->xb, (size_t)Rp * m->Ep * m->esz));
   TRY(h_alloc(c, &m->act, (size_t)Rp * act_k * m->esz));
   TRY(h_alloc(c, &m->hact, (size_t)Rp * (hact_k + 8) * m->esz));
@@ -438,6 +499,7 @@ int hybrid_init(ixt_ctx* c) {
       pp.push_back((char*)L.pages); pb.push_back((int64_t)c->P * L.hg.G * L.hg.dkp * (int64_t)m->esz);
       pp.push_back((char*)L.vpages); pb.push_back((int64_t)c->P * L.hg.G * L.hg.dvp * (int64_t)m->esz);
     } else if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) { pp.push_back((char*)L.pages); pb.push_back((int64_t)c->P * (L.lg.rankp + L.lg.rotp) * (int64_t)m->esz); }
+    else if (L.c.mixer == IXT_MIX_RETENTION) { sb.push_back(L.state); sp.push_back((int64_t)L.rg.H * L.rg.dp * L.rg.dvp); }
     else { sb.push_back(L.state); sp.push_back((int64_t)L.dg.H * L.dg.dv * L.dg.dp); sb.push_back(L.tails); sp.push_back((int64_t)2 * (L.dg.taps - 1) * L.dg.C); }
   }
   m->st_n = (int)sb.size(); m->pg_n = (int)pp.size();
@@ -521,6 +583,31 @@ template <> int hdot_grouped<float>(ixt_ctx*, const float* x, const HMat& w, siz
   hipLaunchKernelGGL(k_dot32, dim3((w.Np + 63) / 64, (rows + 15) / 16), dim3(256), 0, st, x, (const float*)w.w, w.Kp, w.Np, rows, out, rb, stride);
   LAUNCHCHK();
   *res = Slices{out, 1, (size_t)rows * w.Np, w.Np};
+  return IXT_OK;
+}
+// product with a unit without a gate (from IXT_ACT_RELU2 on) behind it -> act(T) of the down product
+template <typename T> static int hact_unit(ixt_ctx* c, const T* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, T* out, hipStream_t st);
+template <> int hact_unit<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, bf16_t* out, hipStream_t st) {
+  GemmEpi e{};
+  e.act = out; e.glu = kind; e.rb_exp = rb; e.wstride = stride / 8;
+  if (rb ? group_rows % 128 == 0 : rows >= c->ring_min_rows) return launch_ring(c, GEPI_ACT, x, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, false, st);
+  if (!rb && rows <= c->small_rows && sdot_plan(c, GEPI_ACT, false, w.Kp, w.Np, rows).ok) return launch_sdot(c, GEPI_ACT, false, x, nullptr, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, st);
+  const int rowblocks = (rows + 15) / 16, nrb = rb ? 1 : (rowblocks >= 3 ? 4 : rowblocks), zblocks = (rowblocks + nrb - 1) / nrb, ntile = w.Np / 16;
+  dim3 grid((((ntile + 3) / 4 + 7) / 8) * 8 * zblocks, 1, 1);
+#define HACT(B_, NT_) hipLaunchKernelGGL((k_dotb<B_, false, NT_, 2>), grid, dim3(256), (size_t)(B_) * 16 * 1024, st, reinterpret_cast<const u32x4*>(x), reinterpret_cast<const u32x4*>(w.w), \
+                                         w.Kp, w.Np, rows, reinterpret_cast<float*>(out), ntile, zblocks, rb, stride / 8, kind, 0.0f)
+  if (nrb == 4) { if (zblocks == 1) HACT(4, true); else HACT(4, false); }
+  else if (nrb == 2) HACT(2, true);
+  else HACT(1, true);
+#undef HACT
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <> int hact_unit<float>(ixt_ctx* c, const float* x, const HMat& w, size_t stride, int rows, int, const int32_t* rb, int kind, float* out, hipStream_t st) {
+  Slices t;
+  TRY(hdot_grouped<float>(c, x, w, stride, rows, 16, rb, c->part, c->part_floats, st, &t));
+  hipLaunchKernelGGL((k_act_slices<float>), dim3(rows, (w.Np + 255) / 256), dim3(256), 0, st, t, w.Np, kind, out, rb);
+  LAUNCHCHK();
   return IXT_OK;
 }
 // gate | up product with the gated unit (IXT_GLU_*) behind it -> act(T) of the down product
@@ -620,92 +707,67 @@ template <typename T>
 static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int Rp, bool decode, int len_hint, hipStream_t st) {
   HybridModel* m = c->hy;
   const LatentGeom& g = L.lg;
-  Slices t;
-  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &t));
-  hipLaunchKernelGGL((k_latent_prep<T>), dim3(R, 1 + (g.H + 3) / 4), dim3(256), 0, st, t, L.d_off, g, W.cnorm, m->eps, L.rope_cos, L.rope_sin, c->row_slot, c->row_pos, c->row_active,
+  Slices t, in;
+  const bool kept = L.c.out_gate || L.c.q_rank > 0;              // the input projection outlives the next dots
+  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, kept ? m->part2 : c->part, kept ? m->part2_floats : c->part_floats, st, &in));
+  t = in;
+  if (L.c.q_rank > 0) {
+    hipLaunchKernelGGL((k_rms_x<T>), dim3(R), dim3(256), 0, st, in, 0, L.c.q_rank, W.qnorm, m->eps, (T*)m->act, W.uq.Kp);
+    LAUNCHCHK();
+    TRY(hdot<T>(c, (const T*)m->act, W.uq, R, c->part, c->part_floats, st, &t));
+  }
+  hipLaunchKernelGGL((k_latent_prep<T>), dim3(R, 1 + (g.H + 3) / 4), dim3(256), 0, st, in, t, L.d_off, g, W.cnorm, m->eps, L.rope_cos, L.rope_sin, c->row_slot, c->row_pos, c->row_active,
                      c->ps.page_map, (T*)L.pages, (T*)m->qx, W.uk.Kp, Rp, (T*)m->qr);
   LAUNCHCHK();
   TRY(hdot_grouped<T>(c, (const T*)m->qx, W.uk, W.uk_stride, g.H * Rp, Rp, m->head_rb, c->part, c->part_floats, st, &t));
   TRY(latent_attention<T>(c, L, t, R, Rp, decode, len_hint, st));
   TRY(hdot_grouped<T>(c, (const T*)m->olat, W.uv, W.uv_stride, g.H * Rp, Rp, m->head_rb, c->part, c->part_floats, st, &t));
-  hipLaunchKernelGGL((k_heads_x<T>), dim3(R, (W.o.Kp + 255) / 256), dim3(256), 0, st, t, g.H, L.c.vdim, Rp, (T*)m->act, W.o.Kp);
+  hipLaunchKernelGGL((k_heads_x<T>), dim3(R, (W.o.Kp + 255) / 256), dim3(256), 0, st, t, g.H, L.c.vdim, Rp, L.c.out_gate ? in : Slices{}, L.g_off, (T*)m->act, W.o.Kp);
   LAUNCHCHK();
   return IXT_OK;
 }
 
-template <int DK, int DV>
-static int heads_prompt_launch(HeadsAttnArgs a, hipStream_t st) {
-  constexpr int lds = 2 * 64 * (DK + DV) * 2;
-  static bool attr_done = false;
-  if (!attr_done) {
-    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_prompt<DK, DV>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
-    attr_done = true;
-  }
-  const int GQ = a.g.H / a.g.G;
-  a.HB = std::min(GQ, 64); a.NQ = 64 / a.HB; a.hchunks = (GQ + a.HB - 1) / a.HB;
-  hipLaunchKernelGGL((k_heads_prompt<DK, DV>), dim3(a.g.G * a.hchunks, (a.R + a.NQ - 1) / a.NQ), dim3(256), lds, st, a);
-  LAUNCHCHK();
-  return IXT_OK;
-}
-template <int DK, int DV>
-static int heads_launch(bool tall, bool fused, int splits, HeadsAttnArgs a, hipStream_t st) {
-  if (tall) return heads_prompt_launch<DK, DV>(a, st);
-  constexpr int lds = 64 * (DK + DV) * 2;
-  static bool attr_done = false;
-  if (!attr_done) {
-    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_decode<DK, DV, true>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
-    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_heads_decode<DK, DV, false>), hipFuncAttributeMaxDynamicSharedMemorySize, lds));
-    attr_done = true;
-  }
-  const dim3 grid(a.R, a.g.G * a.hchunks, splits);
-  if (fused) hipLaunchKernelGGL((k_heads_decode<DK, DV, true>), grid, dim3(256), lds, st, a);
-  else hipLaunchKernelGGL((k_heads_decode<DK, DV, false>), grid, dim3(256), lds, st, a);
-  LAUNCHCHK();
-  return IXT_OK;
-}
-template <typename T>
-static int heads_prep(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& t, const HeadsRope& rope, const RowsArgs& rows, int R, hipStream_t st) {
-  HybridModel* m = c->hy;
-  const HeadsGeom& g = L.hg;
-  const int n = g.H + 2 * g.G, widest = std::max(g.dkp, g.vs);
-#define HPREP(LP_) hipLaunchKernelGGL((k_heads_prep<T, LP_>), dim3(R, (n * LP_ + 255) / 256), dim3(256), 0, st, t, g, W.qn, W.kn, m->eps, rope, rows, (T*)L.pages, (T*)L.vpages, (T*)m->qx)
-  if (widest <= 64) HPREP(16); else if (widest <= 128) HPREP(32); else HPREP(64);
-#undef HPREP
-  LAUNCHCHK();
-  return IXT_OK;
-}
 template <typename T>
 static int hybrid_mixer_heads(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, bool decode, int len_hint, hipStream_t st) {
+  Slices t;
+  TRY(hdot<T>(c, (const T*)c->hy->xb, W.in, R, c->part, c->part_floats, st, &t));
+  return heads_attention<T>(c, L, W, t, R, decode, len_hint, st);
+}
+
+template <int NT, bool FUSED, typename T>
+static int ret_out_launch(const RetArgs& a, int chunks, T* out, int Kp, hipStream_t st) {
+  hipLaunchKernelGGL((k_ret_out<T, NT, FUSED>), dim3(chunks, a.g.H, (a.g.dvp + 16 * NT - 1) / (16 * NT)), dim3(256), 0, st, a, out, Kp);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <typename T>
+static int hybrid_mixer_retention(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st) {
   HybridModel* m = c->hy;
-  const HeadsGeom& g = L.hg;
+  const RetGeom& g = L.rg;
+  Slices t;
+  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &t));
   const RowsArgs rows{c->row_slot, c->row_pos, c->row_active, c->ps.page_map};
   const HeadsRope rope{L.rope_cos, L.rope_sin};
-  Slices t;
-  int dkp = 0, dvp = 0;
-  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &t));
-  if constexpr (sizeof(T) == 2) {
-    if (heads_mfma_sizes(g.d, g.dv, m->f32, &dkp, &dvp)) {
-      const bool tall = !decode && R > 32;
-      const int GQ = g.H / g.G, hchunks = (GQ + 15) / 16, blocks = R * g.G * hchunks, span = g.window > 0 ? std::min(g.window, len_hint) : len_hint;
-      int splits = 1;
-      if (!tall) splits = std::min(std::min(16, std::max(1, IXT_HEADS_SPLIT_BLOCKS / blocks)), std::max(1, (span + 63) / 64));     // at least a tile each
-      if (!decode) TRY((heads_prep<T>(c, L, W, t, rope, rows, R, st)));
-      HeadsAttnArgs a{(const bf16_t*)m->qx, g, W.sink, rows, (bf16_t*)L.pages, (bf16_t*)L.vpages, R, 1, (GQ + hchunks - 1) / hchunks, hchunks, __builtin_ctz(c->P),
-                      (bf16_t*)m->act, W.o.Kp, m->po, m->pml, t, W.qn, W.kn, m->eps, rope};
-      int rc = IXT_ERR_UNSUPPORTED;
-#define X(DK_, DV_) if (dkp == DK_ && dvp == DV_) rc = heads_launch<DK_, DV_>(tall, decode, splits, a, st);
-      IXT_HEADS_SIZES(X)
-#undef X
-      TRY(rc);
-      if (splits > 1) {
-        hipLaunchKernelGGL(k_heads_combine, dim3(R, g.H), dim3(64), 0, st, m->po, m->pml, splits, g.dvp, g.H, g.vs, c->row_active, (bf16_t*)m->act, W.o.Kp);
-        LAUNCHCHK();
-      }
-      return IXT_OK;
-    }
+  const RetArgs a{g, t, L.pow, m->seg, m->chunk, m->nseg, m->dq, m->dk, m->dv, m->ret_u, L.state, m->dout, m->eps};
+  T* out = (T*)m->act;
+  if (single) {            // every row is a run of one token
+    const int ns = 256 / (g.dvp / 4);
+    hipLaunchKernelGGL((k_ret_step<T>), dim3(R, g.H), dim3(256), sizeof(float) * (2 * g.dp + g.dvp + ns * g.dvp), st, a, rope, rows, out, W.o.Kp);
+    LAUNCHCHK();
+    return IXT_OK;
   }
-  TRY((heads_prep<T>(c, L, W, t, rope, rows, R, st)));
-  hipLaunchKernelGGL((k_heads_any<T>), dim3(R, g.H), dim3(256), sizeof(float) * (g.dkp + 256), st, (const T*)m->qx, g, W.sink, rows, (const T*)L.pages, (const T*)L.vpages, (T*)m->act, W.o.Kp);
+  const int widest = std::max(g.dp, g.dvp), chunks = R / SEG_CHUNK + nseg_max;
+#define RPREP(LP_) hipLaunchKernelGGL((k_ret_prep<LP_>), dim3(R, (3 * g.H * LP_ + 255) / 256), dim3(256), 0, st, a, rope, rows)
+  if (widest <= 64) RPREP(16); else if (widest <= 128) RPREP(32); else RPREP(64);
+#undef RPREP
+  hipLaunchKernelGGL(k_ret_sums, dim3(chunks, g.H, (g.dp + 63) / 64 * ((g.dvp + 127) / 128)), dim3(256), 0, st, a);
+  hipLaunchKernelGGL(k_ret_carry, dim3(nseg_max, g.H, (g.dp * g.dvp + 1023) / 1024), dim3(256), 0, st, a);
+  LAUNCHCHK();
+  if (g.dvp <= 32) return ret_out_launch<2, true, T>(a, chunks, out, W.o.Kp, st);
+  if (g.dvp <= 64) return ret_out_launch<4, true, T>(a, chunks, out, W.o.Kp, st);
+  if (g.dvp <= 128) return ret_out_launch<8, true, T>(a, chunks, out, W.o.Kp, st);
+  TRY((ret_out_launch<8, false, T>(a, chunks, out, W.o.Kp, st)));
+  hipLaunchKernelGGL((k_ret_gate<T>), dim3(R, (g.H + 3) / 4), dim3(256), 0, st, a, c->row_active, out, W.o.Kp);
   LAUNCHCHK();
   return IXT_OK;
 }
@@ -749,9 +811,10 @@ static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipSt
   HybridModel* m = c->hy;
   const ixt_layer& l = L.c;
   const int pairs = R * l.top, n = l.experts;
-  const RouteRule rule{l.experts, l.top, l.router, l.groups > 1 ? l.groups : 0, l.groups_keep, l.router_norm, l.router_scale, W.corr};
+  const RouteRule rule{l.experts, l.top, l.router, l.groups > 1 ? l.groups : 0, l.groups_keep, l.router_norm, l.router_scale, W.corr, W.bias, l.shared_ff > 0 && l.shared_gate ? m->sgate : nullptr};
+  const bool gated = l.glu < IXT_ACT_RELU2;
   if (l.shared_ff > 0) {
-    TRY(hglu<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, l.glu_limit, (T*)m->hact, st));
+    TRY(gated ? hglu<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, l.glu_limit, (T*)m->hact, st) : hact_unit<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, (T*)m->hact, st));
     TRY(hdot<T>(c, (const T*)m->hact, W.sdown, R, m->part2, m->part2_floats, st, shared));
   }
   const float* h = (m->norm_places & IXT_NORM_BEFORE) ? m->h32 : m->x;
@@ -766,7 +829,8 @@ static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipSt
   if constexpr (sizeof(T) == 2) hipLaunchKernelGGL(k_moe_gather, dim3(pairs, (m->Ep + 2047) / 2048), dim3(256), 0, st, (const bf16_t*)m->xb, m->mpos, l.top, m->Ep, (bf16_t*)m->xg);
   else hipLaunchKernelGGL(k_gather32, dim3(pairs, (m->Ep + 255) / 256), dim3(256), 0, st, (const float*)m->xb, m->mpos, l.top, m->Ep, (float*)m->xg);
   LAUNCHCHK();
-  TRY(hglu<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, l.glu_limit, (T*)m->mhact, st));
+  TRY(gated ? hglu<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, l.glu_limit, (T*)m->mhact, st)
+            : hact_unit<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, (T*)m->mhact, st));
   return hdot_grouped<T>(c, (const T*)m->mhact, W.down, W.down_stride, rows_g, align, m->mrb, c->part, c->part_floats, st, out);
 }
 
@@ -777,41 +841,25 @@ static int hybrid_logits(ixt_ctx* c, int R, int lrow0, int nl, const int32_t* lr
   const int nblk = (m->V + 1023) / 1024;
   for (int i0 = 0; i0 < nl; i0 += c->NLmax) {
     const int n = std::min(c->NLmax, nl - i0);
-#define HFINAL(KIND_) hipLaunchKernelGGL((k_final_norm<T, KIND_>), dim3(n), dim3(256), 0, st, m->x, lrows ? lrows + i0 : nullptr, lrow0 + i0, R, m->fnorm, m->eps, m->E, m->Ep, (T*)m->xn)
-    if (m->norm_kind == IXT_NORM_TANH) HFINAL(IXT_NORM_TANH); else HFINAL(IXT_NORM_RMS);
-#undef HFINAL
-    LAUNCHCHK();
+    TRY((hybrid_final_norm<T>(c, R, n, lrows ? lrows + i0 : nullptr, lrow0 + i0, st)));
     Slices t;
     TRY(hdot<T>(c, (const T*)m->xn, m->head, n, c->part, c->part_floats, st, &t));
-    hipLaunchKernelGGL(k_head_post, dim3(nblk, n), dim3(256), 0, st, t, m->V, c->sample_cols, logits_out ? logits_out + (size_t)i0 * m->V : nullptr, c->amax_val, c->amax_idx);
+    hipLaunchKernelGGL(k_head_post, dim3(nblk, n), dim3(256), 0, st, t, m->V, m->logit_scale, c->sample_cols, logits_out ? logits_out + (size_t)i0 * m->V : nullptr, c->amax_val, c->amax_idx);
     if (argmax_out) hipLaunchKernelGGL(k_argmax_final, dim3(n), dim3(256), 0, st, c->amax_val, c->amax_idx, nblk, argmax_out + i0);
     LAUNCHCHK();
   }
   return IXT_OK;
 }
 
-// x <- x + post(t), the next operand pre(x) (k_sub_norm); routed: its f32 copy too
-template <typename T>
-static int hybrid_norm(ixt_ctx* c, const Slices& t, const Slices& add, const int32_t* pos, const float* wts, int top, const NormW& post, const NormW& pre, bool routed, int R, hipStream_t st) {
-  HybridModel* m = c->hy;
-  float* h32 = routed && pre.w != nullptr ? m->h32 : nullptr;
-#define HNORM(NI_, KIND_) hipLaunchKernelGGL((k_sub_norm<T, NI_, KIND_>), dim3(R), dim3(256), 0, st, t, add, pos, wts, top, post, pre, m->eps, m->E, m->Ep, m->x, (T*)m->xb, h32)
-#define HNORM_K(NI_) do { if (m->norm_kind == IXT_NORM_TANH) HNORM(NI_, IXT_NORM_TANH); else HNORM(NI_, IXT_NORM_RMS); } while (0)
-  if (m->Ep <= 2048) HNORM_K(1); else if (m->Ep <= 4096) HNORM_K(2); else if (m->Ep <= 8192) HNORM_K(4); else HNORM_K(6);
-#undef HNORM_K
-#undef HNORM
-  LAUNCHCHK();
-  return IXT_OK;
-}
-
 // a sublayer's last product and what follows it: x <- x + post(W v), the next operand pre(x).  Tanh norms ride in the product's epilogue where the whole
 // sum is in one place.
 template <typename T>
-static int hybrid_dot_norm(ixt_ctx* c, const T* v, const HMat& w, const NormW& post, const NormW& pre, bool routed, int R, hipStream_t st) {
+static int hybrid_dot_norm(ixt_ctx* c, const T* v, const HMat& w, const Around& ar, bool routed, int R, hipStream_t st) {
   HybridModel* m = c->hy;
+  [[maybe_unused]] const NormW &post = ar.post, &pre = ar.pre;
   if constexpr (sizeof(T) == 2) {
     const bool small = R <= c->small_rows && sdot_plan(c, GEPI_TANHNORM, false, w.Kp, w.Np, R).ok;
-    if (m->norm_kind == IXT_NORM_TANH && (small || R >= c->ring_min_rows)) {
+    if (m->norm_kind == IXT_NORM_TANH && m->streams == 0 && (small || R >= c->ring_min_rows)) {
       GemmEpi e{};
       e.act = (bf16_t*)m->xb;
       e.tn = TanhNormEpi{post.w, post.b, post.alpha, pre.w, pre.b, pre.alpha, m->x, routed && pre.w != nullptr ? m->h32 : nullptr, m->E, m->Ep};
@@ -821,7 +869,7 @@ static int hybrid_dot_norm(ixt_ctx* c, const T* v, const HMat& w, const NormW& p
   }
   Slices t;
   TRY(hdot<T>(c, v, w, R, c->part, c->part_floats, st, &t));
-  return hybrid_norm<T>(c, t, Slices{}, nullptr, nullptr, 0, post, pre, routed, R, st);
+  return hybrid_norm<T>(c, SubOut{t}, ar, routed, R, st);
 }
 
 template <typename T>
@@ -830,37 +878,48 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
   HybridModel* m = c->hy;
   const int Rp = (sizeof(T) == 2 && R >= c->ring_min_rows) ? up_to(R, 128) : up_to(R, 16);
   if (m->recurrent || m->maxH > 0)
-    hipLaunchKernelGGL(k_segments, dim3(1), dim3(1024), 0, st, R, c->row_active, c->row_slot, c->row_pos, m->row_seg, m->row_j, m->seg, m->nseg, m->state_len, m->parity, m->claim, c->G,
+    hipLaunchKernelGGL(k_segments, dim3(1), dim3(1024), 0, st, R, c->row_active, c->row_slot, c->row_pos, m->row_seg, m->row_j, m->seg, m->chunk, m->nseg, m->state_len, m->parity, m->claim, c->G,
                      m->recurrent ? 1 : 0, m->err, m->head_rb, m->maxH * (Rp / 16), Rp / 16);
-  const NormW none{}, first = m->layers[m->layers[0].src].n1;
-  hipLaunchKernelGGL((k_embed_scaled<T>), dim3(R), dim3(256), 0, st, (const T*)m->embed, tokens, m->emb_scale, m->E, m->Ep, m->V, m->norm_kind == IXT_NORM_TANH ? first : none, m->x, (T*)m->xb);
+  const HLayer& head = m->layers[m->layers[0].src];
+  const NormW none{}, first = head.n1;
+  const bool tanh_first = m->norm_kind == IXT_NORM_TANH && m->streams == 0;      // that norm rides with the lookup
+  hipLaunchKernelGGL((k_embed_scaled<T>), dim3(R), dim3(256), 0, st, (const T*)m->embed, tokens, m->emb_scale, m->E, m->Ep, m->V, std::max(1, m->streams),
+                     tanh_first ? first : none, m->x, (T*)m->xb);
   LAUNCHCHK();
-  if (m->norm_kind == IXT_NORM_RMS && first.w != nullptr) TRY((hybrid_norm<T>(c, Slices{}, Slices{}, nullptr, nullptr, 0, none, first, false, R, st)));
+  if (!tanh_first && (first.w != nullptr || m->streams > 0)) TRY((hybrid_norm<T>(c, SubOut{}, Around{none, first, nullptr, head.hc1}, false, R, st)));
   for (size_t i = 0; i < m->layers.size(); ++i) {
     const HLayer& L = m->layers[i];
     const HLayer& W = m->layers[L.src];
     if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) TRY((hybrid_mixer_latent<T>(c, L, W, R, Rp, decode, len_hint, st)));
     else if (L.c.mixer == IXT_MIX_ATTENTION) TRY((hybrid_mixer_heads<T>(c, L, W, R, decode, len_hint, st)));
+    else if (L.c.mixer == IXT_MIX_RETENTION) TRY((hybrid_mixer_retention<T>(c, L, W, R, nseg_max, decode, st)));
     else TRY((hybrid_mixer_delta<T>(c, L, W, R, nseg_max, decode, st)));
-    const NormW next = i + 1 < m->layers.size() ? m->layers[m->layers[i + 1].src].n1 : none;      // (the head's norm is taken of the wanted rows only)
-    TRY((hybrid_dot_norm<T>(c, (const T*)m->act, W.o, W.n1b, L.c.ffn == IXT_FFN_NONE ? next : W.n2, L.c.ffn == IXT_FFN_MOE, R, st)));
+    const HLayer* next = i + 1 < m->layers.size() ? &m->layers[m->layers[i + 1].src] : nullptr;      // (the head's norm is taken of the wanted rows only)
+    const NormW next_n = next ? next->n1 : none;
+    const float* next_hc = next ? next->hc1 : nullptr;
+    const bool ffn = L.c.ffn != IXT_FFN_NONE;
+    const Around ar1{W.n1b, ffn ? W.n2 : next_n, W.hc1, ffn ? W.hc2 : next_hc}, ar2{W.n2b, next_n, W.hc2, next_hc};
+    TRY((hybrid_dot_norm<T>(c, (const T*)m->act, W.o, ar1, L.c.ffn == IXT_FFN_MOE, R, st)));
     if (L.c.ffn == IXT_FFN_DENSE) {
-      TRY(hglu<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, L.c.glu_limit, (T*)m->hact, st));
-      TRY((hybrid_dot_norm<T>(c, (const T*)m->hact, W.down, W.n2b, next, false, R, st)));
+      TRY(L.c.glu < IXT_ACT_RELU2 ? hglu<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, L.c.glu_limit, (T*)m->hact, st)
+                                  : hact_unit<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, (T*)m->hact, st));
+      TRY((hybrid_dot_norm<T>(c, (const T*)m->hact, W.down, ar2, false, R, st)));
     } else if (L.c.ffn == IXT_FFN_MOE) {
       Slices t, shared{};
+      const float* addw = L.c.shared_gate ? m->sgate : nullptr;
       TRY(hybrid_moe<T>(c, L, W, R, st, &t, &shared));
       if (t.n > 2 && R <= 64) {
         hipLaunchKernelGGL(k_moe_sum, dim3((t.ncols + 255) / 256, R), dim3(64), 0, st, t, m->mpos, m->mw, L.c.top, m->msum);
         LAUNCHCHK();
-        TRY((hybrid_norm<T>(c, Slices{m->msum, 1, 0, t.ncols}, shared, nullptr, nullptr, 0, W.n2b, next, false, R, st)));
+        TRY((hybrid_norm<T>(c, SubOut{Slices{m->msum, 1, 0, t.ncols}, shared, addw}, ar2, false, R, st)));
       } else {
-        TRY((hybrid_norm<T>(c, t, shared, m->mpos, m->mw, L.c.top, W.n2b, next, false, R, st)));
+        TRY((hybrid_norm<T>(c, SubOut{t, shared, addw, m->mpos, m->mw, L.c.top}, ar2, false, R, st)));
       }
     }
     if (m->tap && !c->capturing) {
       if ((i + 1) * (size_t)R * m->E > m->tap_floats) return set_err(IXT_ERR_INVALID, "residual tap: buffer too small");
-      HIPCHK(hipMemcpyAsync(m->tap + i * (size_t)R * m->E, m->x, sizeof(float) * (size_t)R * m->E, hipMemcpyDeviceToDevice, st));
+      hipLaunchKernelGGL(k_stream_sum, dim3(R, (m->E + 255) / 256), dim3(256), 0, st, m->x, std::max(1, m->streams), m->E, m->tap + i * (size_t)R * m->E);
+      LAUNCHCHK();
     }
   }
   c->h_final_rows = R;

@@ -1,6 +1,7 @@
 // ixt_hybrid_kernels.h -- kernels of decoders whose layers are listed one by one (ixt_config.layers): each layer has a sequence mixer (latent
-// attention over a paged latent cache, a gated delta rule with a recurrent state per page group, or attention over keys and values per head:
-// ixt_heads_kernels.h), a feed-forward (a gated unit, dense or as a routed mixture) and norms in front of the sublayers, behind them, or both.
+// attention over a paged latent cache, a gated delta rule with a recurrent state per page group, attention over keys and values per head:
+// ixt_heads_kernels.h, retention: ixt_retention_kernels.h), a feed-forward (a unit, dense or as a routed mixture) and norms in front of the sublayers,
+// behind them, or both; around a sublayer stands one residual sum, or several streams that mix (hyper-connections).
 //
 // Every kernel is a template over T, the storage of activations and cached keys: bf16_t (activations in the dot kernels' fragment order, xidx) or
 // float (row-major; the 32-bit mode).  The residual stream, norms, rotations, scores, routers and the recurrence are f32 in both.
@@ -118,14 +119,19 @@ static __global__ __launch_bounds__(256) void k_dot32(const float* __restrict__ 
 // ---------------------------------------------------------------------------------------------------- weights
 // src [n][k] row-major ([out, in] linear weights, rows `ld` apart) -> rows n of a dot operand of Kp k-columns, at (column n_off + n, k k_off + k).
 // inter: 16-column tile j goes to tile 2 j + n_off (the two matrices of a gated unit side by side).  trans: src is [k][n].  ng / kg > 0: groups of ng
-// columns (kg k) are laid ngp (kgp) apart, zeros between them.
-struct LoadMap { int n, k, ld, Kp, n_off, k_off, inter, trans, ng, ngp, kg, kgp; };
+// columns (kg k) are laid ngp (kgp) apart, zeros between them.  rn > 0: of every rg columns those from r0 on are rn rotated features in halves (i turns
+// with i + rn / 2); they are laid as neighbours, which is the order the kernels turn (the order of a head's features changes no score).
+struct LoadMap { int n, k, ld, Kp, n_off, k_off, inter, trans, ng, ngp, kg, kgp, rg, r0, rn; };
 template <typename S, typename T>
 __global__ void k_load_nk(const S* __restrict__ src, T* __restrict__ dst, LoadMap m) {
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= (int64_t)m.n * m.k) return;
   int nn = m.trans ? (int)(i % m.n) : (int)(i / m.k), kk = m.trans ? (int)(i / m.n) : (int)(i % m.k);
   const float v = to_f(src[m.trans ? (size_t)kk * m.ld + nn : (size_t)nn * m.ld + kk]);
+  if (m.rn > 0) {
+    const int f = nn % m.rg - m.r0, h = m.rn / 2;
+    if (f >= 0 && f < m.rn) nn += (f < h ? 2 * f : 2 * (f - h) + 1) - f;
+  }
   if (m.ng > 0) nn = nn / m.ng * m.ngp + nn % m.ng;
   if (m.kg > 0) kk = kk / m.kg * m.kgp + kk % m.kg;
   const int col = m.inter ? ((nn >> 4) * 2 + m.n_off) * 16 + (nn & 15) : m.n_off + nn;
@@ -141,20 +147,23 @@ __global__ void k_load_vec(const S* __restrict__ src, T* __restrict__ dst, int64
 // ---------------------------------------------------------------------------------------------------- row segments
 // A segment = consecutive rows of one page group at consecutive positions: what a recurrence walks through.  One block of 1024 threads.
 //   row_seg[r], row_j[r]   segment of row r and its place in it (row_seg -1: idle)
-//   seg[s] = {first row, rows, page group, first position, parity of the convolution tail to read, 0, 0, 0}
+//   seg[s] = {first row, rows, page group, first position, parity of the convolution tail to read, first chunk, 0, 0}
+//   chunk[c] = {first row, rows (<= SEG_CHUNK), segment, place in the segment}: a segment's chunks lie side by side (what a recurrence over blocks of
+//   rows walks through), nseg_out[1] of them
 // recurrent != 0: a segment must start at position 0 (the state counts as zero) or where its group's state stands (state_len); anything else, and a
 // second segment of a group in one call, idles and is counted in err[0].  The tails of short convolutions are double-buffered: a pass reads parity
 // p and writes 1 - p, so no row waits for another one's tail.
 // head_rb: 16-row block b of a head-major activation matrix (rbh blocks per head) belongs to head b / rbh.
+#define SEG_CHUNK 64
 static __global__ __launch_bounds__(1024) void k_segments(int R, int32_t* row_active, const int32_t* row_slot, const int32_t* row_pos, int32_t* row_seg, int32_t* row_j,
-                                                   int32_t* seg /*[.][8]*/, int32_t* nseg_out, int32_t* state_len, int32_t* parity, int32_t* claim, int groups,
+                                                   int32_t* seg /*[.][8]*/, int4* chunk, int32_t* nseg_out, int32_t* state_len, int32_t* parity, int32_t* claim, int groups,
                                                    int recurrent, int32_t* err, int32_t* head_rb, int nhead_rb, int rbh) {
   __shared__ int s_last[1024];
-  __shared__ int s_cnt;
+  __shared__ int s_cnt, s_chunks;
   const int tid = threadIdx.x;
   for (int i = tid; i < groups; i += 1024) claim[i] = 0;
   for (int i = tid; i < nhead_rb; i += 1024) head_rb[i] = i / rbh;
-  if (tid == 0) s_cnt = 0;
+  if (tid == 0) s_cnt = s_chunks = 0;
   const int per = (R + 1023) / 1024, lo = min(tid * per, R), hi = min(lo + per, R);
   auto starts = [&](int r) { return r == 0 || !row_active[r - 1] || row_slot[r - 1] != row_slot[r] || row_pos[r - 1] + 1 != row_pos[r]; };
   int last = -1;
@@ -196,6 +205,11 @@ static __global__ __launch_bounds__(1024) void k_segments(int R, int32_t* row_ac
     }
     int32_t* d = seg + (size_t)s * 8;
     d[0] = cur; d[1] = ok ? n : 0; d[2] = g; d[3] = start; d[4] = par;
+    if (recurrent && ok) {
+      const int nc = (n + SEG_CHUNK - 1) / SEG_CHUNK, base = atomicAdd(&s_chunks, nc);
+      d[5] = base;
+      for (int i = 0; i < nc; ++i) chunk[base + i] = make_int4(cur + i * SEG_CHUNK, min(SEG_CHUNK, n - i * SEG_CHUNK), s, i);
+    }
   }
   __syncthreads();
   cur = cur0;
@@ -210,7 +224,7 @@ static __global__ __launch_bounds__(1024) void k_segments(int R, int32_t* row_ac
   __syncthreads();
   for (int r = lo; r < hi; ++r)
     if (row_seg[r] < 0) row_active[r] = 0;
-  if (tid == 0) *nseg_out = s_cnt;
+  if (tid == 0) { nseg_out[0] = s_cnt; nseg_out[1] = s_chunks; }
 }
 
 // state of group src -> group dst (both tail buffers, the recurrent matrices, the length).  grid (chunks), block 256; n0, n1: floats per group
@@ -233,7 +247,7 @@ static __global__ __launch_bounds__(256) void k_latent_pages_copy(PageStateDev s
 
 // ---------------------------------------------------------------------------------------------------- embedding, norms
 // A norm's parameters (zeros behind feature E - 1); w null: no norm.  KIND IXT_NORM_RMS: t / sqrt(mean(t^2) + eps) (1 + w); IXT_NORM_TANH: feature by
-// feature tanh(alpha t) w + b.
+// feature tanh(alpha t) w + b; IXT_NORM_LAYER: (t - mean) / sqrt(mean((t - mean)^2) + eps) w + b.
 struct NormW { const float *w, *b, *alpha; };
 __device__ __forceinline__ void load8(const float* __restrict__ p, float* o) {       // p % 16 bytes == 0
   const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
@@ -249,25 +263,56 @@ __device__ __forceinline__ void store4(bf16_t* p, const float* v) {
   *reinterpret_cast<uint2*>(p) = o;
 }
 __device__ __forceinline__ void store4(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
-// 8 features k0 .. k0 + 7 through a norm; s: the tanh norm's alpha, or the RMS norm's 1 / sqrt(mean + eps)
+// What a norm needs to know of a row: s = the tanh norm's alpha, or 1 / sqrt(mean + eps); mu: the layer norm's mean.
+struct NormStat { float s, mu; };
+// 8 features k0 .. k0 + 7 through a norm
 template <int KIND>
-__device__ __forceinline__ void norm8(const NormW& n, float s, int k0, const float* t, float* o) {
+__device__ __forceinline__ void norm8(const NormW& n, NormStat st, int k0, const float* t, float* o) {
+  const float s = st.s;
   float w[8], b[8];
   load8(n.w + k0, w);
   if constexpr (KIND == IXT_NORM_TANH) {
     load8(n.b + k0, b);
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[j] = fmaf(tanh_f32(s * t[j]), w[j], b[j]);
+  } else if constexpr (KIND == IXT_NORM_LAYER) {
+    load8(n.b + k0, b);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = fmaf((t[j] - st.mu) * s, w[j], b[j]);
   } else {
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[j] = t[j] * s * (1.0f + w[j]);
   }
 }
 
-// x[r] = table[token] * scale (f32) and its copy as the first dot's operand, through a tanh norm if `pre` is one.  grid R, block 256.
+// Statistics of a row that a block of 256 holds as v[NI][8] (features i 2048 + 8 tid + j, zeros behind feature E - 1)
+template <int KIND, int NI>
+__device__ __forceinline__ NormStat row_stat(const NormW& n, const float (*v)[8], int E, float eps, float* red) {
+  if constexpr (KIND == IXT_NORM_TANH) return NormStat{*n.alpha, 0.0f};
+  float mu = 0.0f, ss = 0.0f;
+  if constexpr (KIND == IXT_NORM_LAYER) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) mu += v[i][j];
+    mu = block_sum256(mu, red) / (float)E;
+  }
+#pragma unroll
+  for (int i = 0; i < NI; ++i)
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (i * 2048 + (int)threadIdx.x * 8 + j < E) ss = fmaf(v[i][j] - mu, v[i][j] - mu, ss);
+  return NormStat{1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps), mu};
+}
+// Hyper-connections.  A sublayer's numbers: HC_IN, HC_OUT [HC_MAX] each, then mix [from][to], rows HC_MAX apart.
+#define HC_MAX 16
+struct HyperW { const float *in, *out, *mix; };      // in: of the sublayer that follows (nullptr: none does); out, mix: of the one that ends
+
+// x[r] = table[token] * scale (f32; `streams` copies of it) and its copy as the first dot's operand, through a tanh norm if `pre` is one.  grid R, block 256.
 template <typename T>
-__global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ table, const int32_t* __restrict__ ids, float scale, int E, int Ep, int V, NormW pre, float* __restrict__ x,
-                                                      T* __restrict__ xb) {
+__global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ table, const int32_t* __restrict__ ids, float scale, int E, int Ep, int V, int streams, NormW pre,
+                                                      float* __restrict__ x, T* __restrict__ xb) {
+  x += (size_t)blockIdx.x * (streams - 1) * E;             // rows are `streams` E apart
   const int r = blockIdx.x;
   const int id = min(max(ids[r], 0), V - 1);
   for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
@@ -276,31 +321,41 @@ __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ tabl
       load8(table + (size_t)id * E + k0, v);
 #pragma unroll
       for (int j = 0; j < 8; ++j) v[j] *= scale;
-      store4(x + (size_t)r * E + k0, v); store4(x + (size_t)r * E + k0 + 4, v + 4);
+      for (int s = 0; s < streams; ++s) { store4(x + (size_t)(r + s) * E + k0, v); store4(x + (size_t)(r + s) * E + k0 + 4, v + 4); }
     } else {
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
         v[j] = k0 + j < E ? to_f(table[(size_t)id * E + k0 + j]) * scale : 0.0f;
-        if (k0 + j < E) x[(size_t)r * E + k0 + j] = v[j];
+        if (k0 + j < E)
+          for (int s = 0; s < streams; ++s) x[(size_t)(r + s) * E + k0 + j] = v[j];
       }
     }
-    if (pre.w != nullptr) norm8<IXT_NORM_TANH>(pre, *pre.alpha, k0, v, v);
+    if (pre.w != nullptr) norm8<IXT_NORM_TANH>(pre, NormStat{*pre.alpha, 0.0f}, k0, v, v);
     act_store8(xb, r, k0, Ep, v);
   }
 }
 
 // A sublayer's output t (slices, or the weighted sum of a row's expert outputs) -> norm behind the sublayer -> residual -> norm in front of the next one:
 //   x <- x + post(t);  xb = pre(x) as the next dot's operand, h32 (if given) the same in f32.
-// t.n == 0: t = 0 and x stays.  pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  add.n > 0: its row joins t.  A thread owns 8 consecutive features of every 2048 (NI
-// times).  grid R, block 256.
-template <typename T, int NI, int KIND>
-__global__ __launch_bounds__(256) void k_sub_norm(Slices t, Slices add, const int32_t* __restrict__ pos, const float* __restrict__ wts, int top, NormW post, NormW pre, float eps,
-                                                  int E, int Ep, float* __restrict__ x, T* __restrict__ xb, float* __restrict__ h32) {
+// t.n == 0: t = 0 and x stays.  pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  add.n > 0: its row, times addw[r] if that is given, joins t.
+// SM > 0: `streams` (<= SM) streams in the place of x ([R][streams][E]): x_t <- sum_s mix[s][t] x_s + out[t] post(t), and pre takes sum_s in[s] x_s.
+// A thread owns 8 consecutive features of every 2048 (NI times).  grid R, block 256.
+struct SubNormArgs {
+  Slices t, add; const float* addw;
+  const int32_t* pos; const float* wts; int top;
+  NormW post, pre; float eps; int E, Ep, streams; HyperW hc;
+};
+template <typename T, int NI, int KIND, int SM>
+__global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restrict__ x, T* __restrict__ xb, float* __restrict__ h32) {
   __shared__ float red[4];
-  const int r = blockIdx.x;
+  const Slices &t = a.t, &add = a.add;
+  const int32_t* __restrict__ pos = a.pos;
+  const float* __restrict__ wts = a.wts;
+  const NormW &post = a.post, &pre = a.pre;
+  const int r = blockIdx.x, top = a.top, E = a.E, Ep = a.Ep;
   const bool vec = (E & 3) == 0;
   float v[NI][8], xv[NI][8];
-  float ss = 0.0f;
+  const float fadd = a.addw != nullptr ? a.addw[r] : 1.0f;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int k0 = i * 2048 + threadIdx.x * 8;
@@ -324,8 +379,9 @@ __global__ __launch_bounds__(256) void k_sub_norm(Slices t, Slices add, const in
         float u[4];
         add.at4(r, k0 + q, u);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[i][q + e] += u[e];
+        for (int e = 0; e < 4; ++e) v[i][q + e] = fmaf(fadd, u[e], v[i][q + e]);
       }
+      if constexpr (SM > 0) continue;
       if (vec) {
         const float4 xx = *reinterpret_cast<const float4*>(x + (size_t)r * E + k0 + q);
         xv[i][q] = xx.x; xv[i][q + 1] = xx.y; xv[i][q + 2] = xx.z; xv[i][q + 3] = xx.w;
@@ -335,30 +391,72 @@ __global__ __launch_bounds__(256) void k_sub_norm(Slices t, Slices add, const in
           if (k0 + q + e < E) xv[i][q + e] = x[(size_t)r * E + k0 + q + e];
       }
     }
-    if constexpr (KIND == IXT_NORM_RMS) {
+  }
+  if (t.n > 0 && post.w != nullptr) {
+    const NormStat st = row_stat<KIND, NI>(post, v, E, a.eps, red);
 #pragma unroll
-      for (int j = 0; j < 8; ++j)
-        if (k0 + j < E) ss = fmaf(v[i][j], v[i][j], ss);
-    }
+    for (int i = 0; i < NI; ++i)
+      if (i * 2048 + (int)threadIdx.x * 8 < Ep) norm8<KIND>(post, st, i * 2048 + threadIdx.x * 8, v[i], v[i]);
   }
-  float s_post = 0.0f, s_pre = 0.0f;
-  if constexpr (KIND == IXT_NORM_RMS) {
-    if (post.w != nullptr) s_post = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
-  } else {
-    if (post.w != nullptr) s_post = *post.alpha;
-    if (pre.w != nullptr) s_pre = *pre.alpha;
-  }
-  ss = 0.0f;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int k0 = i * 2048 + threadIdx.x * 8;
     if (k0 >= Ep) continue;
-    if (t.n > 0 && post.w != nullptr) norm8<KIND>(post, s_post, k0, v[i], v[i]);
+    if constexpr (SM > 0) {                                  // (features behind E - 1 are never read; xv stays 0 there)
+      float* xr = x + (size_t)r * a.streams * E;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      xv[i][j] = k0 + j < E ? xv[i][j] + v[i][j] : 0.0f;
-      if (KIND == IXT_NORM_RMS) ss = fmaf(xv[i][j], xv[i][j], ss);
+      for (int q = 0; q < 8; q += 4) {
+        if (k0 + q >= E) continue;
+        float old[SM][4];
+#pragma unroll
+        for (int s = 0; s < SM; ++s) {
+          old[s][0] = old[s][1] = old[s][2] = old[s][3] = 0.0f;
+          if (s >= a.streams) continue;
+          const float* p = xr + (size_t)s * E + k0 + q;
+          if (vec) { const float4 u = *reinterpret_cast<const float4*>(p); old[s][0] = u.x; old[s][1] = u.y; old[s][2] = u.z; old[s][3] = u.w; }
+          else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (k0 + q + e < E) old[s][e] = p[e];
+          }
+        }
+#pragma unroll SM <= 4 ? SM : 1
+        for (int d = 0; d < (SM <= 4 ? SM : a.streams); ++d) {
+          if (d >= a.streams) continue;
+          float nw[4];
+          float* p = xr + (size_t)d * E + k0 + q;
+          if (t.n > 0) {
+            const float fo = a.hc.out[d];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) nw[e] = fo * v[i][q + e];
+#pragma unroll
+            for (int s = 0; s < SM; ++s) {
+              const float fm = a.hc.mix[s * HC_MAX + d];      // (rows behind the last stream are zero)
+#pragma unroll
+              for (int e = 0; e < 4; ++e) nw[e] = fmaf(fm, old[s][e], nw[e]);
+            }
+            if (vec) *reinterpret_cast<float4*>(p) = make_float4(nw[0], nw[1], nw[2], nw[3]);
+            else {
+#pragma unroll
+              for (int e = 0; e < 4; ++e)
+                if (k0 + q + e < E) p[e] = nw[e];
+            }
+          } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) nw[e] = k0 + q + e < E ? p[e] : 0.0f;
+          }
+          if (a.hc.in != nullptr) {
+            const float fi = a.hc.in[d];
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (k0 + q + e < E) xv[i][q + e] = fmaf(fi, nw[e], xv[i][q + e]);
+          }
+        }
+      }
+      continue;
     }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) xv[i][j] = k0 + j < E ? xv[i][j] + v[i][j] : 0.0f;
     if (t.n > 0) {
       if (vec) {
 #pragma unroll
@@ -371,12 +469,14 @@ __global__ __launch_bounds__(256) void k_sub_norm(Slices t, Slices add, const in
       }
     }
   }
-  if (KIND == IXT_NORM_RMS && pre.w != nullptr) s_pre = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
+  if (SM > 0 && a.hc.in == nullptr) return;                // the head takes the streams themselves
+  NormStat st{};
+  if (pre.w != nullptr) st = row_stat<KIND, NI>(pre, xv, E, a.eps, red);
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int k0 = i * 2048 + threadIdx.x * 8;
     if (k0 >= Ep) continue;
-    if (pre.w != nullptr) norm8<KIND>(pre, s_pre, k0, xv[i], xv[i]);      // (zeros behind feature E - 1: so are w and b there)
+    if (pre.w != nullptr) norm8<KIND>(pre, st, k0, xv[i], xv[i]);      // (w and b are zero behind feature E - 1)
     if (h32 != nullptr) {
 #pragma unroll
       for (int j = 0; j < 8; ++j)
@@ -386,32 +486,42 @@ __global__ __launch_bounds__(256) void k_sub_norm(Slices t, Slices add, const in
   }
 }
 
-// rows lrows[i] (or lrow0 + i) of x -> the model's norm -> the head's operand.  grid nl, block 256.
-template <typename T, int KIND>
-__global__ __launch_bounds__(256) void k_final_norm(const float* __restrict__ x, const int32_t* __restrict__ lrows, int lrow0, int nrows, NormW w, float eps, int E, int Ep,
-                                                    T* __restrict__ xn) {
+// rows lrows[i] (or lrow0 + i) of x (the sum of their streams) -> the model's norm -> the head's operand.  grid nl, block 256.
+template <typename T, int NI, int KIND>
+__global__ __launch_bounds__(256) void k_final_norm(const float* __restrict__ x, const int32_t* __restrict__ lrows, int lrow0, int nrows, int streams, NormW w, float eps, int E,
+                                                    int Ep, T* __restrict__ xn) {
   __shared__ float red[4];
-  const int i = blockIdx.x;
-  const int r = min(max(lrows != nullptr ? lrows[i] : lrow0 + i, 0), nrows - 1);
-  float s;
-  if constexpr (KIND == IXT_NORM_RMS) {
-    float ss = 0.0f;
-    for (int k = threadIdx.x; k < E; k += 256) { const float v = x[(size_t)r * E + k]; ss = fmaf(v, v, ss); }
-    s = 1.0f / sqrtf(block_sum256(ss, red) / (float)E + eps);
-  } else {
-    s = *w.alpha;
-  }
-  for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
-    float v[8];
+  const int r = min(max(lrows != nullptr ? lrows[blockIdx.x] : lrow0 + (int)blockIdx.x, 0), nrows - 1);
+  float v[NI][8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = k0 + j < E ? x[(size_t)r * E + k0 + j] : 0.0f;
-    norm8<KIND>(w, s, k0, v, v);
-    act_store8(xn, i, k0, Ep, v);
+  for (int i = 0; i < NI; ++i)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int k = i * 2048 + threadIdx.x * 8 + j;
+      v[i][j] = 0.0f;
+      if (k < E)
+        for (int s = 0; s < streams; ++s) v[i][j] += x[((size_t)r * streams + s) * E + k];
+    }
+  const NormStat st = row_stat<KIND, NI>(w, v, E, eps, red);
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int k0 = i * 2048 + threadIdx.x * 8;
+    if (k0 >= Ep) continue;
+    norm8<KIND>(w, st, k0, v[i], v[i]);
+    act_store8(xn, blockIdx.x, k0, Ep, v[i]);
   }
 }
+// the residual stream as one row per token: the sum of its streams.  grid (R, ceil(E / 256)), block 256.
+static __global__ __launch_bounds__(256) void k_stream_sum(const float* __restrict__ x, int streams, int E, float* __restrict__ out) {
+  const int r = blockIdx.x, k = blockIdx.y * 256 + threadIdx.x;
+  if (k >= E) return;
+  float v = 0.0f;
+  for (int s = 0; s < streams; ++s) v += x[((size_t)r * streams + s) * E + k];
+  out[(size_t)r * E + k] = v;
+}
 
-// logits = the head's slices; (max, first index) per block of 1024 columns over the allowed ones.  grid (ceil(V / 1024), nl), block 256.
-static __global__ __launch_bounds__(256) void k_head_post(Slices t, int V, ColRanges cr, float* __restrict__ logits /*[nl][V] or nullptr*/, float* __restrict__ amax_val,
+// logits = the head's slices times scale; (max, first index) per block of 1024 columns over the allowed ones.  grid (ceil(V / 1024), nl), block 256.
+static __global__ __launch_bounds__(256) void k_head_post(Slices t, int V, float scale, ColRanges cr, float* __restrict__ logits /*[nl][V] or nullptr*/, float* __restrict__ amax_val,
                                                    int32_t* __restrict__ amax_idx) {
   __shared__ float bv[4];
   __shared__ int bi[4];
@@ -422,7 +532,7 @@ static __global__ __launch_bounds__(256) void k_head_post(Slices t, int V, ColRa
   for (int i = 0; i < 4; ++i) {
     const int c = blockIdx.x * 1024 + i * 256 + threadIdx.x;
     if (c >= V) continue;
-    const float v = t.at(r, c);
+    const float v = t.at(r, c) * scale;
     if (logits != nullptr) logits[(size_t)r * V + c] = v;
     if (v > best && col_allowed(cr, c)) { best = v; idx = c; }
   }
@@ -534,11 +644,11 @@ struct LatentGeom {
   float scale;
 };
 
-// The input projection's slices ([q heads of dn + dr | d_off: latent, rotated key part]) -> the row's cache entry (normed latent, rotated key part)
-// and the queries: unrotated parts head-major as the operand of the key up-projection (row h Rp + r), rotated parts qr [R][H][rotp].
-// rope: f32 [position][dr / 2] cos, sin.  grid (R, 1 + ceil(H / 4)), block 256: y = 0 the cache entry, y > 0 four heads (a wave each).
+// The input projection's slices t (d_off: latent, rotated key part) -> the row's cache entry (normed latent, rotated key part); the queries' slices tq
+// (heads of dn + dr, columns from 0 on) -> unrotated parts head-major as the operand of the key up-projection (row h Rp + r), rotated parts qr
+// [R][H][rotp].  rope: f32 [position][dr / 2] cos, sin.  grid (R, 1 + ceil(H / 4)), block 256: y = 0 the cache entry, y > 0 four heads (a wave each).
 template <typename T>
-__global__ __launch_bounds__(256) void k_latent_prep(Slices t, int d_off, LatentGeom g, const float* __restrict__ cnorm, float eps, const float* __restrict__ rope_cos,
+__global__ __launch_bounds__(256) void k_latent_prep(Slices t, Slices tq, int d_off, LatentGeom g, const float* __restrict__ cnorm, float eps, const float* __restrict__ rope_cos,
                                                      const float* __restrict__ rope_sin, const int32_t* __restrict__ row_slot, const int32_t* __restrict__ row_pos,
                                                      const int32_t* __restrict__ row_active, const int32_t* __restrict__ page_map, T* __restrict__ pages, T* __restrict__ qx,
                                                      int dnp, int Rp, T* __restrict__ qr) {
@@ -565,17 +675,28 @@ __global__ __launch_bounds__(256) void k_latent_prep(Slices t, int d_off, Latent
   const int h = (blockIdx.y - 1) * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (h >= g.H) return;
   const int c0 = h * (g.dn + g.dr);
-  for (int k = lane; k < dnp; k += 64) act_store1(qx, h * Rp + r, k, dnp, k < g.dn ? t.at(r, c0 + k) : 0.0f);
+  for (int k = lane; k < dnp; k += 64) act_store1(qx, h * Rp + r, k, dnp, k < g.dn ? tq.at(r, c0 + k) : 0.0f);
   T* qo = qr + ((size_t)r * g.H + h) * g.rotp;
   for (int i = lane; i < g.rotp / 2; i += 64) {
     float a = 0.0f, b = 0.0f;
     if (i < half) {
-      const float u = t.at(r, c0 + g.dn + 2 * i), v = t.at(r, c0 + g.dn + 2 * i + 1);
+      const float u = tq.at(r, c0 + g.dn + 2 * i), v = tq.at(r, c0 + g.dn + 2 * i + 1);
       const float c = rope_cos[(size_t)pos * half + i], s = rope_sin[(size_t)pos * half + i];
       a = u * c - v * s; b = v * c + u * s;
     }
     qo[2 * i] = from_f<T>(a); qo[2 * i + 1] = from_f<T>(b);
   }
+}
+
+// n columns of a projection from c0 on, RMS-normed with a plain weight, as the next dot's operand.  grid R, block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_rms_x(Slices t, int c0, int n, const float* __restrict__ w, float eps, T* __restrict__ out, int Kp) {
+  __shared__ float red[4];
+  const int r = blockIdx.x;
+  float ss = 0.0f;
+  for (int k = threadIdx.x; k < n; k += 256) { const float v = t.at(r, c0 + k); ss = fmaf(v, v, ss); }
+  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)n + eps);
+  for (int k = threadIdx.x; k < Kp; k += 256) act_store1(out, r, k, Kp, k < n ? t.at(r, c0 + k) * rs * w[k] : 0.0f);
 }
 
 // Any sizes (rank <= 1024), any T: block = (row, head); thread = key for the scores (tiles of 256 keys, running maximum and sum), thread = latent
@@ -972,12 +1093,18 @@ static __global__ __launch_bounds__(128) void k_latent_combine(const float* __re
     act_store4(out, h * Rp + r, c, Kp, v);
   }
 }
-// head-major slices (row h Rp + r, n columns each) -> act of the output projection: column h n + c.  grid (R, ceil(Kp / 256)), block 256.
+// head-major slices (row h Rp + r, n columns each) -> act of the output projection: column h n + c, times sigmoid of gate column g0 + h n + c (gate.n ==
+// 0: none).  grid (R, ceil(Kp / 256)), block 256.
 template <typename T>
-__global__ __launch_bounds__(256) void k_heads_x(Slices t, int H, int n, int Rp, T* __restrict__ out, int Kp) {
+__global__ __launch_bounds__(256) void k_heads_x(Slices t, int H, int n, int Rp, Slices gate, int g0, T* __restrict__ out, int Kp) {
   const int r = blockIdx.x, k = blockIdx.y * 256 + threadIdx.x;
   if (k >= Kp) return;
-  act_store1(out, r, k, Kp, k < H * n ? t.at((k / n) * Rp + r, k % n) : 0.0f);
+  float v = 0.0f;
+  if (k < H * n) {
+    v = t.at((k / n) * Rp + r, k % n);
+    if (gate.n > 0) v *= f32_sigmoid(gate.at(r, g0 + k));
+  }
+  act_store1(out, r, k, Kp, v);
 }
 
 // ---------------------------------------------------------------------------------------------------- gated delta rule
@@ -1329,10 +1456,19 @@ __global__ __launch_bounds__(256) void k_glu_slices(Slices t, int Fp, int kind, 
   act_store1(out, r, f, Fp, ixt_glu(kind, t.at(r, c), t.at(r, c + 16), limit));
 }
 
-// The choice of experts for a row.  IXT_ROUTE_SOFTMAX: scores s = softmax over all n logits; IXT_ROUTE_SIGMOID: s = sigmoid(z).  The `top` largest
-// s + corr (first index on a tie), inside the `keep` of `groups` equal groups of neighbours whose two largest s + corr add up to most; weights are the
-// picked s, divided by (their sum + 1e-20) if norm, times scale.
-struct RouteRule { int n, top, kind, groups, keep, norm; float scale; const float* corr; };
+// the same for a unit without a gate.  grid (rows, ceil(Fp / 256)), block 256
+template <typename T>
+__global__ __launch_bounds__(256) void k_act_slices(Slices t, int Fp, int kind, T* __restrict__ out, const int32_t* __restrict__ rb_exp) {
+  const int f = blockIdx.y * 256 + threadIdx.x, r = blockIdx.x;
+  if (f >= Fp || (rb_exp != nullptr && rb_exp[r >> 4] < 0)) return;
+  act_store1(out, r, f, Fp, ixt_act(kind, t.at(r, f)));
+}
+
+// The choice of experts for a row.  IXT_ROUTE_SOFTMAX: scores s = softmax over all n logits; IXT_ROUTE_SIGMOID: s = sigmoid(z); IXT_ROUTE_CHOSEN: s = z.
+// The `top` largest s + corr (first index on a tie), inside the `keep` of `groups` equal groups of neighbours whose two largest s + corr add up to most;
+// weights are the picked s (CHOSEN: the softmax over the picked ones), divided by (their sum + 1e-20) if norm, times scale.
+// Logits are products plus bias[e] (nullptr: none).  gate: one more row of the router's matrix behind the experts, whose sigmoid goes to gate[row].
+struct RouteRule { int n, top, kind, groups, keep, norm; float scale; const float *corr, *bias; float* gate; };
 // one wave; z [n] in LDS (overwritten: choice scores), gs [2 groups] in LDS; n <= 1024
 __device__ __forceinline__ void route_top(float* z, float* gs, const RouteRule& a, int lane, int32_t* idx, float* wts) {
   const int n = a.n;
@@ -1355,7 +1491,7 @@ __device__ __forceinline__ void route_top(float* z, float* gs, const RouteRule& 
     const int e = lane + 64 * i;
     s[i] = 0.0f;
     if (e < n) {
-      s[i] = a.kind == IXT_ROUTE_SOFTMAX ? expf(v[i] - mx) / sum : f32_sigmoid(v[i]);
+      s[i] = a.kind == IXT_ROUTE_SOFTMAX ? expf(v[i] - mx) / sum : a.kind == IXT_ROUTE_SIGMOID ? f32_sigmoid(v[i]) : v[i];
       v[i] = a.corr != nullptr ? s[i] + a.corr[e] : s[i];
     }
   }
@@ -1405,26 +1541,31 @@ __device__ __forceinline__ void route_top(float* z, float* gs, const RouteRule& 
 #pragma unroll
     for (int i = 0; i < 16; ++i) if (lane + 64 * i == bi) { v[i] = -INFINITY; w = s[i]; }
     w = __shfl(w, bi & 63, 64);
+    if (a.kind == IXT_ROUTE_CHOSEN) {                      // relative to the first, the largest
+      if (j == 0) mx = w;
+      w = expf(w - mx);
+    }
     total += w;
     if (lane == 0) { idx[j] = bi; wts[j] = w; }
   }
-  const float f = a.norm ? a.scale / (total + 1e-20f) : a.scale;
-  if (lane == 0 && (a.norm || a.scale != 1.0f))
+  const bool divide = a.norm || a.kind == IXT_ROUTE_CHOSEN;
+  const float f = divide ? a.scale / (total + 1e-20f) : a.scale;
+  if (lane == 0 && (divide || a.scale != 1.0f))
     for (int j = 0; j < a.top; ++j) wts[j] *= f;
 }
 // router: logits (f32 residual x f32 weights) and choice of RB rows in one block, eight experts at a time: a thread takes every 256th feature of the RB
-// rows and the eight weight rows.  w [n][Ep]; grid ceil(R / RB), block 256, LDS RB (n + 2 groups) floats.
+// rows and the eight weight rows.  w [n (+ 1)][Ep]; grid ceil(R / RB), block 256, LDS RB (n + 2 groups) floats.
 template <int RB>
 __global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, const float* __restrict__ w, int E, int Ep, RouteRule rule, int R, int32_t* __restrict__ idx,
                                                float* __restrict__ wts) {
   extern __shared__ __attribute__((aligned(16))) float z[];            // [RB][n], [RB][2 groups]
   __shared__ float red[4][RB * 8];
-  const int n = rule.n, row = rule.top;
+  const int n = rule.n, nw = n + (rule.gate != nullptr ? 1 : 0), row = rule.top;
   const int r0 = blockIdx.x * RB, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const float* xr[RB];
 #pragma unroll
   for (int i = 0; i < RB; ++i) xr[i] = x + (size_t)min(r0 + i, R - 1) * E;
-  for (int e0 = 0; e0 < n; e0 += 8) {
+  for (int e0 = 0; e0 < nw; e0 += 8) {
     float acc[RB][8];
 #pragma unroll
     for (int i = 0; i < RB; ++i)
@@ -1432,7 +1573,7 @@ __global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, cons
       for (int e = 0; e < 8; ++e) acc[i][e] = 0.0f;
     const float* wr[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) wr[e] = w + (size_t)min(e0 + e, n - 1) * Ep;
+    for (int e = 0; e < 8; ++e) wr[e] = w + (size_t)min(e0 + e, nw - 1) * Ep;
 #pragma unroll 2
     for (int k = tid; k < E; k += 256) {
       float xv[RB], wv[8];
@@ -1453,7 +1594,12 @@ __global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, cons
         if (lane == 0) red[wave][i * 8 + e] = t;
       }
     __syncthreads();
-    if (tid < RB * 8 && e0 + (tid & 7) < n) z[(tid >> 3) * n + e0 + (tid & 7)] = (red[0][tid] + red[1][tid]) + (red[2][tid] + red[3][tid]);
+    if (tid < RB * 8 && e0 + (tid & 7) < nw) {
+      const int e = e0 + (tid & 7), i = tid >> 3;
+      const float v = (red[0][tid] + red[1][tid]) + (red[2][tid] + red[3][tid]);
+      if (e < n) z[i * n + e] = rule.bias != nullptr ? v + rule.bias[e] : v;
+      else if (r0 + i < R) rule.gate[r0 + i] = f32_sigmoid(v);
+    }
     __syncthreads();
   }
   for (int i = wave; i < RB; i += 4)

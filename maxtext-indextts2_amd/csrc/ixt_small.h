@@ -183,6 +183,12 @@ __global__ __launch_bounds__(1024) void k_sdot(SdotArgs a) {
     if (row_ok) *reinterpret_cast<float4*>(a.e.out + (size_t)row * N + tile * 16 + cq * 4) = make_float4(tot[0], tot[1], tot[2], tot[3]);
   } else if constexpr (EPI == GEPI_TANHNORM) {
     if (row_ok) tanhnorm_epi(a.e.tn, a.e.act, row, tile * 16 + cq * 4, tot);
+  } else if constexpr (EPI == GEPI_ACT) {
+    if (row_ok) {
+      uint2 ov;
+      ov.x = pack2(f2bf(ixt_act(a.e.glu, tot[0])), f2bf(ixt_act(a.e.glu, tot[1]))); ov.y = pack2(f2bf(ixt_act(a.e.glu, tot[2])), f2bf(ixt_act(a.e.glu, tot[3])));
+      *reinterpret_cast<uint2*>(a.e.act + xidx(row, tile * 16 + cq * 4, N)) = ov;
+    }
   } else if constexpr (EPI == GEPI_RESID) {
     if (row_ok) {
       const size_t o = (size_t)row * N + tile * 16 + cq * 4;

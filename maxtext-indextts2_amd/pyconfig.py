@@ -180,8 +180,8 @@ def _derive(keys: Dict[str, Any]) -> None:
   elif keys["num_experts"] != 1 or keys["num_experts_per_tok"] != 1:
     raise ValueError("num_experts > 1 is built for decoder_block mixtral only")
   if keys["decoder_block"] not in ("gemma2", "gemma3") and (keys["attn_logits_soft_cap"] or keys["final_logits_soft_cap"] or keys["sliding_window_size"] or
-                                            keys["use_post_attn_norm"] or keys["use_post_ffw_norm"] or keys["logits_via_embedding"]):
-    raise ValueError("soft caps, sliding_window_size, post norms and logits_via_embedding are built for decoder_block gemma2 / gemma3 only")
+                                            keys["use_post_attn_norm"] or keys["use_post_ffw_norm"] or (keys["logits_via_embedding"] and keys["decoder_block"] != "hybrid")):
+    raise ValueError("soft caps, sliding_window_size, post norms and logits_via_embedding are built for decoder_block gemma2 / gemma3 (the last one also hybrid) only")
   if isinstance(keys["mlp_activations"], list):
     keys["mlp_activations"] = tuple(keys["mlp_activations"])
 

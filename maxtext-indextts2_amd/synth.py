@@ -201,11 +201,15 @@ def synth_weights_hybrid(cfg, seed: int = 0) -> Dict[str, np.ndarray]:
     elif leaf == "conv":
       z = z * np.float32(1.0 / math.sqrt(shape[1]))
     elif leaf in ("norm1", "norm2", "norm1b", "norm2b") or name == "final.norm":
-      z = np.float32(cfg.hybrid_norm_kind) + np.float32(0.1) * z  # zero-centred, or (tanh norms) plain
+      z = np.float32(cfg.hybrid_norm_kind != architectures.NORM_RMS) + np.float32(0.1) * z  # zero-centred, or plain
     elif leaf in ("alpha", "b", "correction", "sink"):
       z = np.float32(1.0 if leaf in ("alpha", "sink") else 0.0) + np.float32(0.1) * z
     elif leaf == "norm":                                          # plain
       z = np.float32(1.0) + np.float32(0.1) * z
+    elif leaf in ("in", "out", "mix") and ".hc" in name:          # streams that mix a little around one residual sum
+      z = np.float32(0.05) * z + (np.eye(cfg.hybrid_streams, dtype=np.float32) if leaf == "mix" else np.float32(1.0 / cfg.hybrid_streams if leaf == "in" else 1.0))
+    elif leaf in ("lq1", "lk1", "lq2", "lk2"):
+      z = z * np.float32(0.5 / math.sqrt(shape[0]))
     else:
       z = z * np.float32(1.0 / math.sqrt(shape[-1]))
     w[name] = f32_to_bf16_bits(z).reshape(shape)
@@ -293,7 +297,7 @@ def device_tree_spec(cfg):
   """[(tree path, shape, std or None for a norm scale)] of the configured block (llama2, gemma2, mixtral, hybrid)."""
   if getattr(cfg, "decoder_block", "llama2") == "hybrid":
     from . import architectures  # pylint: disable=import-outside-toplevel
-    std = lambda name, shape: (1 / cfg.embedding_scale if name == "embed" else None if name.endswith("alpha") else 0.1 if "norm" in name else 0.5 if len(shape) == 1 else 1 / math.sqrt(shape[-1]))
+    std = lambda name, shape: (1 / cfg.embedding_scale if name == "embed" else None if name.endswith("alpha") else 0.1 if "norm" in name or name.rsplit(".", 1)[-1] in ("lq1", "lk1", "lq2", "lk2") else 0.5 if len(shape) == 1 or ".hc" in name else 1 / math.sqrt(shape[-1]))
     return [(name, shape, std(name, shape)) for name, shape in architectures.parameter_shapes(cfg).items()]
   E, Q, KV, D, F, V = cfg.emb_dim, cfg.num_query_heads, cfg.num_kv_heads, cfg.head_dim, cfg.mlp_dim, cfg.vocab_size
   block = getattr(cfg, "decoder_block", "llama2")
