@@ -1,5 +1,5 @@
 """`bench.py --hybrid SIZES`: prefill and decode rates of hybrid decoders (Vilepel: half latent attention, half gated delta rule; Vazilorn: windowed
-attention with sinks and tanh norms) at layer sizes of real models, beside the closest model of the framework at the same width, head count,
+attention with sinks and tanh norms; Suzulix: differential attention, retention and latent attention among four streams) at layer sizes of real models, beside the closest model of the framework at the same width, head count,
 feed-forward and number of layers (the llama2 block, or Mixtral for the routed sizes).  Random weights drawn on the device, one GPU, both models in
 turn in one process.
 
@@ -53,6 +53,20 @@ def _grouped_moe(ff, experts, top, groups, keep, shared):
   return {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": shared}, "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}, "scale": 2.5}}
 
 
+def _suzulix(width, mixers, heads, mlp):
+  """Layers of differential attention, retention and latent attention in turn, four streams."""
+  dim = 128
+  kinds = {"attention": {"heads": heads, "kv_heads": heads // 2, "dim": dim // 2, "vdim": dim, "scale": (dim // 2) ** -0.5, "softcap": 30.0, "diff": 0.5, "rot": {"base": 500000.0, "dims": dim // 2}},
+           "retention": {"heads": heads, "dim": dim, "vdim": dim, "decay": [1.0 - 2.0 ** -(5 + 6.0 * i / heads) for i in range(heads)], "rot": {"base": 10000.0, "dims": dim}},
+           "latent_attention": {"heads": heads, "dim": dim, "rot_dim": 64, "vdim": dim, "kv_rank": 512, "q_rank": width // 2, "scale": (dim + 64) ** -0.5, "rot": {"base": 10000.0, "dims": 64}}}
+  return {"architecture": "Suzulix", "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5}, "vocab": 32000, "width": width, "streams": 4, "logit_scale": 1.0,
+          "layers": [{"type": t, "mixer": kinds[t], "mlp": mlp} for t in mixers]}
+
+
+def _square_moe(ff, experts, top, shared):
+  return {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": shared}, "router": {"experts": experts, "top": top}}
+
+
 # name -> (config.json, keys of the closest model)
 SIZES = {
     "w1024": (_model(1024, 4, _latent(8, 256, 512, dim=64), _delta(8, 8), _dense(3584)),
@@ -69,6 +83,15 @@ SIZES = {
     "vazilorn-w4096-moe": (_vazilorn(4096, 2, _heads(32, 8, 1024), _grouped_moe(14336, 8, 2, 4, 2, 2048)),
                            dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=2, num_experts=8, num_experts_per_tok=2,
                                 decoder_block="mixtral")),
+    "suzulix-w1024": (_suzulix(1024, ("attention", "retention", "latent_attention") * 2, 8, _square_moe(3584, 8, 2, 3584)),
+                      dict(base_emb_dim=1024, base_num_query_heads=8, base_num_kv_heads=4, base_mlp_dim=3584, base_num_decoder_layers=6, num_experts=8, num_experts_per_tok=2,
+                           decoder_block="mixtral")),
+    "suzulix-w2048": (_suzulix(2048, ("attention", "retention", "latent_attention"), 16, _square_moe(7168, 8, 2, 7168)),
+                      dict(base_emb_dim=2048, base_num_query_heads=16, base_num_kv_heads=8, base_mlp_dim=7168, base_num_decoder_layers=3, num_experts=8, num_experts_per_tok=2,
+                           decoder_block="mixtral")),
+    "suzulix-w4096": (_suzulix(4096, ("attention", "retention", "latent_attention"), 32, _square_moe(14336, 8, 2, 2048)),
+                      dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=3, num_experts=8, num_experts_per_tok=2,
+                           decoder_block="mixtral")),
 }
 
 
