@@ -819,8 +819,13 @@ static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipSt
   }
   const float* h = (m->norm_places & IXT_NORM_BEFORE) ? m->h32 : m->x;
   const size_t lds = sizeof(float) * (l.experts + 2 * rule.groups);
-  if (R <= 256) hipLaunchKernelGGL((k_route<1>), dim3(R), dim3(256), lds, st, h, W.router, m->E, m->Ep, rule, R, m->midx, m->mw);
-  else hipLaunchKernelGGL((k_route<4>), dim3((R + 3) / 4), dim3(256), 4 * lds, st, h, W.router, m->E, m->Ep, rule, R, m->midx, m->mw);
+  const int nw = n + (rule.gate != nullptr ? 1 : 0);              // rows of the router's matrix; 12 at a time where that saves a pass
+#define HROUTE(NE_) do { \
+    if (R <= 256) hipLaunchKernelGGL((k_route<1, NE_>), dim3(R), dim3(256), lds, st, h, W.router, m->E, m->Ep, rule, R, m->midx, m->mw); \
+    else hipLaunchKernelGGL((k_route<4, NE_>), dim3((R + 3) / 4), dim3(256), 4 * lds, st, h, W.router, m->E, m->Ep, rule, R, m->midx, m->mw); \
+  } while (0)
+  if ((nw + 11) / 12 < (nw + 7) / 8) HROUTE(12); else HROUTE(8);
+#undef HROUTE
   LAUNCHCHK();
   const int align = (m->f32 || pairs <= 64) ? 16 : 128;
   const int rows_g = up_to(pairs, align) + align * std::min(n, pairs);     // every expert with a copy may waste up to align - 1 rows

@@ -355,6 +355,19 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
   const int r = blockIdx.x, top = a.top, E = a.E, Ep = a.Ep;
   const bool vec = (E & 3) == 0;
   float v[NI][8], xv[NI][8];
+  constexpr bool EARLY = SM > 0 && NI * SM <= 8;           // the streams are requested before anything else
+  float4 es[EARLY ? NI * SM * 2 : 1];
+  if constexpr (EARLY) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i)
+#pragma unroll
+      for (int s = 0; s < SM; ++s)
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+          const int k = i * 2048 + threadIdx.x * 8 + q * 4;
+          if (vec && k < E && s < a.streams) es[(i * SM + s) * 2 + q] = *reinterpret_cast<const float4*>(x + ((size_t)r * a.streams + s) * E + k);
+        }
+  }
   const float fadd = a.addw != nullptr ? a.addw[r] : 1.0f;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
@@ -413,7 +426,7 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
           old[s][0] = old[s][1] = old[s][2] = old[s][3] = 0.0f;
           if (s >= a.streams) continue;
           const float* p = xr + (size_t)s * E + k0 + q;
-          if (vec) { const float4 u = *reinterpret_cast<const float4*>(p); old[s][0] = u.x; old[s][1] = u.y; old[s][2] = u.z; old[s][3] = u.w; }
+          if (vec) { const float4 u = EARLY ? es[EARLY ? (i * SM + s) * 2 + q / 4 : 0] : *reinterpret_cast<const float4*>(p); old[s][0] = u.x; old[s][1] = u.y; old[s][2] = u.z; old[s][3] = u.w; }
           else {
 #pragma unroll
             for (int e = 0; e < 4; ++e)
@@ -1553,49 +1566,62 @@ __device__ __forceinline__ void route_top(float* z, float* gs, const RouteRule& 
   if (lane == 0 && (divide || a.scale != 1.0f))
     for (int j = 0; j < a.top; ++j) wts[j] *= f;
 }
-// router: logits (f32 residual x f32 weights) and choice of RB rows in one block, eight experts at a time: a thread takes every 256th feature of the RB
-// rows and the eight weight rows.  w [n (+ 1)][Ep]; grid ceil(R / RB), block 256, LDS RB (n + 2 groups) floats.
-template <int RB>
+// router: logits (f32 residual x f32 weights) and choice of RB rows in one block, NE experts at a time: a thread takes every 256th feature (every 256th group
+// of four where rows start on 16 bytes) of the RB rows and the NE weight rows.  w [n (+ 1)][Ep]; grid ceil(R / RB), block 256, LDS RB (n + 2 groups) floats.
+template <int RB, int NE>
 __global__ __launch_bounds__(256) void k_route(const float* __restrict__ x, const float* __restrict__ w, int E, int Ep, RouteRule rule, int R, int32_t* __restrict__ idx,
                                                float* __restrict__ wts) {
   extern __shared__ __attribute__((aligned(16))) float z[];            // [RB][n], [RB][2 groups]
-  __shared__ float red[4][RB * 8];
+  __shared__ float red[4][RB * NE];
   const int n = rule.n, nw = n + (rule.gate != nullptr ? 1 : 0), row = rule.top;
   const int r0 = blockIdx.x * RB, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const float* xr[RB];
 #pragma unroll
   for (int i = 0; i < RB; ++i) xr[i] = x + (size_t)min(r0 + i, R - 1) * E;
-  for (int e0 = 0; e0 < nw; e0 += 8) {
-    float acc[RB][8];
+  for (int e0 = 0; e0 < nw; e0 += NE) {
+    float acc[RB][NE];
 #pragma unroll
     for (int i = 0; i < RB; ++i)
 #pragma unroll
-      for (int e = 0; e < 8; ++e) acc[i][e] = 0.0f;
-    const float* wr[8];
+      for (int e = 0; e < NE; ++e) acc[i][e] = 0.0f;
+    const float* wr[NE];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) wr[e] = w + (size_t)min(e0 + e, nw - 1) * Ep;
-#pragma unroll 2
-    for (int k = tid; k < E; k += 256) {
-      float xv[RB], wv[8];
+    for (int e = 0; e < NE; ++e) wr[e] = w + (size_t)min(e0 + e, nw - 1) * Ep;
+    if ((E & 3) == 0) {
+      for (int k = tid * 4; k < E; k += 1024) {
+        float4 xv[RB], wv[NE];
 #pragma unroll
-      for (int i = 0; i < RB; ++i) xv[i] = xr[i][k];
+        for (int i = 0; i < RB; ++i) xv[i] = *reinterpret_cast<const float4*>(xr[i] + k);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) wv[e] = wr[e][k];
+        for (int e = 0; e < NE; ++e) wv[e] = *reinterpret_cast<const float4*>(wr[e] + k);
 #pragma unroll
-      for (int i = 0; i < RB; ++i)
+        for (int i = 0; i < RB; ++i)
 #pragma unroll
-        for (int e = 0; e < 8; ++e) acc[i][e] = fmaf(xv[i], wv[e], acc[i][e]);
+          for (int e = 0; e < NE; ++e) acc[i][e] = fmaf(xv[i].x, wv[e].x, fmaf(xv[i].y, wv[e].y, fmaf(xv[i].z, wv[e].z, fmaf(xv[i].w, wv[e].w, acc[i][e]))));
+      }
+    } else {
+      for (int k = tid; k < E; k += 256) {
+        float xv[RB], wv[NE];
+#pragma unroll
+        for (int i = 0; i < RB; ++i) xv[i] = xr[i][k];
+#pragma unroll
+        for (int e = 0; e < NE; ++e) wv[e] = wr[e][k];
+#pragma unroll
+        for (int i = 0; i < RB; ++i)
+#pragma unroll
+          for (int e = 0; e < NE; ++e) acc[i][e] = fmaf(xv[i], wv[e], acc[i][e]);
+      }
     }
 #pragma unroll
     for (int i = 0; i < RB; ++i)
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
+      for (int e = 0; e < NE; ++e) {
         const float t = wave_sum(acc[i][e]);
-        if (lane == 0) red[wave][i * 8 + e] = t;
+        if (lane == 0) red[wave][i * NE + e] = t;
       }
     __syncthreads();
-    if (tid < RB * 8 && e0 + (tid & 7) < nw) {
-      const int e = e0 + (tid & 7), i = tid >> 3;
+    if (tid < RB * NE && e0 + tid % NE < nw) {
+      const int e = e0 + tid % NE, i = tid / NE;
       const float v = (red[0][tid] + red[1][tid]) + (red[2][tid] + red[3][tid]);
       if (e < n) z[i * n + e] = rule.bias != nullptr ? v + rule.bias[e] : v;
       else if (r0 + i < R) rule.gate[r0 + i] = f32_sigmoid(v);

@@ -57,13 +57,20 @@ __global__ __launch_bounds__(256) void k_ret_prep(RetArgs a, HeadsRope rope, Row
 // n (<= SEG_CHUNK) rows of W columns (from c0 on, as far as they exist) of x [row][heads][cols], times f(row) -> LDS [SEG_CHUNK][LD], zeros elsewhere
 template <int W, int LD, typename F>
 __device__ __forceinline__ void ret_stage(const float* __restrict__ x, int row0, int n, int H, int h, int cols, int c0, float* lds, int tid, F f) {
+  constexpr int NIT = SEG_CHUNK * W / 1024;
+  float4 v[NIT];
+  float s[NIT];
 #pragma unroll
-  for (int it = 0; it < SEG_CHUNK * W / 1024; ++it) {
+  for (int it = 0; it < NIT; ++it) {                         // (everything requested before the first store)
     const int e = it * 256 + tid, j = e / (W / 4), c = e % (W / 4) * 4;
-    float4 v = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-    if (j < n && c0 + c < cols) v = *reinterpret_cast<const float4*>(x + ((size_t)(row0 + j) * H + h) * cols + c0 + c);
-    const float s = f(j);
-    *reinterpret_cast<float4*>(lds + j * LD + c) = make_float4(v.x * s, v.y * s, v.z * s, v.w * s);
+    v[it] = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    if (j < n && c0 + c < cols) v[it] = *reinterpret_cast<const float4*>(x + ((size_t)(row0 + j) * H + h) * cols + c0 + c);
+    s[it] = f(j);
+  }
+#pragma unroll
+  for (int it = 0; it < NIT; ++it) {
+    const int e = it * 256 + tid, j = e / (W / 4), c = e % (W / 4) * 4;
+    *reinterpret_cast<float4*>(lds + j * LD + c) = make_float4(v[it].x * s[it], v[it].y * s[it], v[it].z * s[it], v[it].w * s[it]);
   }
 }
 
@@ -163,12 +170,17 @@ __global__ __launch_bounds__(256, 2) void k_ret_out(RetArgs a, T* __restrict__ o
 #pragma unroll
   for (int t = 0; t < 4; ++t) p[t] = f32x4(0.0f);
   for (int d0 = 0; d0 < g.dp; d0 += 64) {
+    const int steps = min(4, (g.dp - d0) / 16);
+    f32x4 q[4];                                              // (on their way together with the keys)
+#pragma unroll
+    for (int s = 0; s < 4; ++s) q[s] = *reinterpret_cast<const f32x4*>(qp + d0 + min(s, steps - 1) * 16 + q4 * 4);
     if (d0 > 0) __syncthreads();
     ret_stage<64, LDK>(a.k, c.x, n, g.H, h, g.dp, d0, ks, tid, [](int) { return 1.0f; });
     __syncthreads();
-    const int steps = min(4, (g.dp - d0) / 16);
-    for (int s = 0; s < steps; ++s) {
-      const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + d0 + s * 16 + q4 * 4);
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      if (s >= steps) continue;
+      const f32x4 qf = q[s];
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
         if (t > wave) continue;                              // keys behind the wave's rows
@@ -184,18 +196,28 @@ __global__ __launch_bounds__(256, 2) void k_ret_out(RetArgs a, T* __restrict__ o
   if (!first) {
     const float* sp = a.u + ((size_t)ch * g.H + h) * g.dp * g.dvp;
     for (int d0 = 0; d0 < g.dp; d0 += 64) {
-      __syncthreads();
+      const int steps = min(4, (g.dp - d0) / 16);
+      f32x4 q[4];
 #pragma unroll
-      for (int it = 0; it < SEG_CHUNK * W / 1024; ++it) {    // 64 key rows of the state
+      for (int s = 0; s < 4; ++s) q[s] = *reinterpret_cast<const f32x4*>(qp + d0 + min(s, steps - 1) * 16 + q4 * 4);
+      float4 sv[SEG_CHUNK * W / 1024];                       // 64 key rows of the state, requested while the buffer is still being read
+#pragma unroll
+      for (int it = 0; it < SEG_CHUNK * W / 1024; ++it) {
         const int e = it * 256 + tid, j = e / (W / 4), cc = e % (W / 4) * 4;
-        float4 v = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-        if (d0 + j < g.dp && v0 + cc < g.dvp) v = *reinterpret_cast<const float4*>(sp + (size_t)(d0 + j) * g.dvp + v0 + cc);
-        *reinterpret_cast<float4*>(ks + j * LDV + cc) = v;
+        sv[it] = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+        if (d0 + j < g.dp && v0 + cc < g.dvp) sv[it] = *reinterpret_cast<const float4*>(sp + (size_t)(d0 + j) * g.dvp + v0 + cc);
       }
       __syncthreads();
-      const int steps = min(4, (g.dp - d0) / 16);
-      for (int s = 0; s < steps; ++s) {
-        const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + d0 + s * 16 + q4 * 4);
+#pragma unroll
+      for (int it = 0; it < SEG_CHUNK * W / 1024; ++it) {
+        const int e = it * 256 + tid, j = e / (W / 4), cc = e % (W / 4) * 4;
+        *reinterpret_cast<float4*>(ks + j * LDV + cc) = sv[it];
+      }
+      __syncthreads();
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        if (s >= steps) continue;
+        const f32x4 qf = q[s];
 #pragma unroll
         for (int e = 0; e < 4; ++e)
 #pragma unroll
