@@ -132,46 +132,46 @@ __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, Hea
   const int32_t* prow = rows.page_map + (size_t)rows.slot[r] * g.mpg;
   float o[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   for (int mi = 0; mi < g.maps; ++mi) {
-  const float* qm = q + mi * g.dmp;
-  float m = sink != nullptr ? sink[h] : -INFINITY, l = sink != nullptr ? 1.0f : 0.0f, acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-  for (int j0 = k_lo; j0 <= pos; j0 += 256) {
-    const int j = j0 + tid;
-    float s = -INFINITY;
-    if (j <= pos) {
-      const T* kp = kpages + (((size_t)prow[j / g.P] * g.G + kh) * g.P + j % g.P) * g.dkp + mi * g.dmp;
-      float a = 0.0f;
-      for (int k = 0; k < g.d; ++k) a = fmaf(qm[k], to_f(kp[k]), a);
-      s = a * g.scale;
-      if (g.cap > 0.0f) s = g.cap * tanhf(s / g.cap);
+    const float* qm = q + mi * g.dmp;
+    float m = sink != nullptr ? sink[h] : -INFINITY, l = sink != nullptr ? 1.0f : 0.0f, acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    for (int j0 = k_lo; j0 <= pos; j0 += 256) {
+      const int j = j0 + tid;
+      float s = -INFINITY;
+      if (j <= pos) {
+        const T* kp = kpages + (((size_t)prow[j / g.P] * g.G + kh) * g.P + j % g.P) * g.dkp + mi * g.dmp;
+        float a = 0.0f;
+        for (int k = 0; k < g.d; ++k) a = fmaf(qm[k], to_f(kp[k]), a);
+        s = a * g.scale;
+        if (g.cap > 0.0f) s = g.cap * tanhf(s / g.cap);
+      }
+      float tm = s;
+#pragma unroll
+      for (int off = 1; off < 64; off <<= 1) tm = fmaxf(tm, __shfl_xor(tm, off, 64));
+      __syncthreads();
+      if ((tid & 63) == 0) red[tid >> 6] = tm;
+      __syncthreads();
+      const float mn = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), m);
+      const float e = j <= pos ? expf(s - mn) : 0.0f;
+      p[tid] = e;
+      const float al = expf(m - mn);
+      const float ls = block_sum256(e, red);                  // (its barriers also publish p)
+      l = l * al + ls;
+      m = mn;
+      const int nk = min(256, pos - j0 + 1);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[i] *= al;
+      for (int kk = 0; kk < nk; ++kk) {
+        const T* vp = vpages + (((size_t)prow[(j0 + kk) / g.P] * g.G + kh) * g.P + (j0 + kk) % g.P) * g.dvp;
+        const float w = p[kk];
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (tid + 256 * i < g.dv) acc[i] = fmaf(w, to_f(vp[tid + 256 * i]), acc[i]);
+      }
+      __syncthreads();
     }
-    float tm = s;
+    const float f = mi == 0 ? 1.0f / l : -*mp.lambda / l;
 #pragma unroll
-    for (int off = 1; off < 64; off <<= 1) tm = fmaxf(tm, __shfl_xor(tm, off, 64));
-    __syncthreads();
-    if ((tid & 63) == 0) red[tid >> 6] = tm;
-    __syncthreads();
-    const float mn = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), m);
-    const float e = j <= pos ? expf(s - mn) : 0.0f;
-    p[tid] = e;
-    const float al = expf(m - mn);
-    const float ls = block_sum256(e, red);                  // (its barriers also publish p)
-    l = l * al + ls;
-    m = mn;
-    const int nk = min(256, pos - j0 + 1);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] *= al;
-    for (int kk = 0; kk < nk; ++kk) {
-      const T* vp = vpages + (((size_t)prow[(j0 + kk) / g.P] * g.G + kh) * g.P + (j0 + kk) % g.P) * g.dvp;
-      const float w = p[kk];
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        if (tid + 256 * i < g.dv) acc[i] = fmaf(w, to_f(vp[tid + 256 * i]), acc[i]);
-    }
-    __syncthreads();
-  }
-  const float f = mi == 0 ? 1.0f / l : -*mp.lambda / l;
-#pragma unroll
-  for (int i = 0; i < 4; ++i) o[i] = mi == 0 ? acc[i] / l : fmaf(acc[i], f, o[i]);
+    for (int i = 0; i < 4; ++i) o[i] = mi == 0 ? acc[i] / l : fmaf(acc[i], f, o[i]);
   }
   if (g.maps > 1) {
     float ss = 0.0f;                                        // (columns from dv on are zero)
