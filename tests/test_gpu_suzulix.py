@@ -57,7 +57,7 @@ MIXERS = {
     "attention: one pair turns": SH.attn(heads=4, kv_heads=2, dims=2),
     "attention: many heads on one": SH.attn(heads=20, kv_heads=1, dim=12, vdim=12, dims=12),
     "attention: more heads than a tile": SH.attn(heads=70, kv_heads=2, dim=8, vdim=4, dims=4),
-    "attention: 32": SH.attn(heads=4, kv_heads=2, dim=32, vdim=64, dims=16, softcap=30.0),
+    "attention: 32": SH.attn(heads=6, kv_heads=2, dim=32, vdim=56, dims=16, softcap=30.0),
     "attention: values wider": SH.attn(heads=4, kv_heads=2, dim=30, vdim=110, dims=30),
     "attention: keys wider": SH.attn(heads=4, kv_heads=4, dim=64, vdim=60, dims=64),
     "attention: 64": SH.attn(heads=6, kv_heads=2, dim=60, vdim=128, dims=32, scale=0.125, diff=0.8),
@@ -78,7 +78,7 @@ MIXERS = {
     "retention: one head": SH.retention(heads=1, dim=8, vdim=8, dims=8),
     "retention: odd sizes": SH.retention(heads=5, dim=23, vdim=17, dims=6),
     "retention: nothing turns": SH.retention(heads=2, dims=0),
-    "retention: 64": SH.retention(heads=2, dim=64, vdim=64, dims=64),
+    "retention: 64": SH.retention(heads=3, dim=64, vdim=62, dims=48),
     "retention: values wider": SH.retention(heads=2, dim=40, vdim=128, dims=40),
     "retention: keys wider": SH.retention(heads=2, dim=130, vdim=20, dims=64),
     "retention: 128 and 200": SH.retention(heads=2, dim=128, vdim=200, dims=128),
@@ -127,7 +127,7 @@ def test_router_logits_from_level_to_far_apart(tmp_path):
 def test_many_rows_take_the_prompt_kernels(tmp_path, dtype):
   """300 rows in one pass: the ring GEMMs, tall attention tiles, several chunks of the recurrence and 128-row expert groups."""
   for i, layer in enumerate((SH.with_mlp(SH.attn(), SH.moe(experts=9)), SH.with_mlp(SH.attn(heads=8, kv_heads=2, dim=60, vdim=120, dims=60, scale=0.1), None), SH.with_mlp(SH.latent(), SH.moe(shared=200)),
-                             SH.with_mlp(SH.retention(heads=2, dim=90, vdim=100, decay=[0.97, 1 - 2.0 ** -11]), None), SH.with_mlp(SH.retention(dim=20, vdim=20), SH.moe(shared=0)))):
+                             SH.with_mlp(SH.retention(heads=2, dim=90, vdim=100, decay=[0.97, 1 - 2.0 ** -10]), None), SH.with_mlp(SH.retention(dim=20, vdim=20), SH.moe(shared=0)))):
     one_layer(tmp_path / str(i), layer, dtype, n=300, portions=((150, 129, 1),), target=320, rows=320, pages=40, outliers=layer["mlp"] is not None)
 
 
