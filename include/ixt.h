@@ -50,7 +50,7 @@ typedef struct ixt_layer {
   float glu_limit;                 /* IXT_GLU_CLAMPED: the limit */
   int32_t experts, top;            /* MoE */
   /* attention over keys and values per head (heads / kv_heads query heads share one; rot_dim <= dim: the first rot_dim features of a head turn) */
-  int32_t qk_norm;                 /* != 0: every query and key head is RMS-normed with a plain weight before the rotation */
+  int32_t qk_norm;                 /* 1: every query and key head is RMS-normed with a plain weight before the rotation; 2: without a weight (before or after: a rotation keeps it) */
   int32_t sink;                    /* != 0: the softmax denominator of head h also holds exp(sink_h) */
   float rope_factor, rope_low, rope_high, rope_original;   /* rope_factor > 0: a pair of wavelength l = 2 pi / f turns at f where l < original / high, at
                                       f / factor where l > original / low, in between at the mixture linear in original / l */
@@ -64,25 +64,40 @@ typedef struct ixt_layer {
   int32_t number;                  /* the layer's tensors are named l<number>.*; -1: its place in the list (read for layers with parameters of their own) */
   int32_t rope_pairs;              /* IXT_ROPE_*: which two of the rotated features turn together */
   int32_t q_rank;                  /* latent attention, > 0: queries are up-projections of an RMS-normed (plain weight) latent of this size */
-  int32_t out_gate;                /* attention mixers, != 0: the concatenated heads are multiplied by sigmoid(W_g h) in front of the output projection */
+  int32_t out_gate;                /* attention mixers: the concatenated heads are multiplied by sigmoid(W_g h) in front of the output projection: 1 one number per
+                                      feature, 2 (IXT_MIX_ATTENTION) one per head */
   int32_t maps;                    /* IXT_MIX_ATTENTION: 2: every head has two softmax maps of `dim` features each over the same values, and its output is
                                       rms(a1 - lambda a2) (1 - map_diff) with lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + map_diff; 0 or 1: one map */
   float map_diff;
   float softcap;                   /* IXT_MIX_ATTENTION, > 0: score <- softcap tanh(score / softcap) */
   int32_t router_bias;             /* != 0: a per-expert number joins the router's logits */
   int32_t shared_gate;             /* != 0: the shared unit's output is multiplied by sigmoid(w . h), one number per token */
-  const double* decay;             /* IXT_MIX_RETENTION: one decay per head (HOST array of `heads` entries, copied by ixt_create) */
+  const double* decay;             /* IXT_MIX_RETENTION, IXT_MIX_LIGHTNING: one decay per head (HOST array of `heads` entries, copied by ixt_create) */
+  int32_t chunk;                   /* IXT_MIX_ATTENTION, > 0: position i sees only the positions j <= i with j / chunk == i / chunk (whole numbers); no window beside it */
+  int32_t key_values;              /* IXT_MIX_ATTENTION, != 0: the values are the keys as projected, before norm and rotation (vdim == dim, one map, no W_v) */
+  int32_t mix_bias;                /* IXT_MIX_ATTENTION, != 0: q, k, v and the output projection have biases (tensors *.b) */
+  int32_t inner, state, dt_rank;   /* IXT_MIX_SCAN: channels, states per channel, rank of the step-size projection; `conv` taps */
+  float mix_scale;                 /* factor on the mixer's output (its output bias included): attention over heads, retention, lightning */
+  const struct ixt_layer* beside;  /* a second mixer that reads the same input and whose output is added (HOST, copied by ixt_create; NULL: none).  Both are one of
+                                      IXT_MIX_ATTENTION, _RETENTION, _LIGHTNING; their tensors are mix.left.* and mix.right.* */
+  int32_t shift;                   /* != 0: what the mixer reads, h, is replaced by h + (h' - h) l<i>.shift, h' being the previous token's h (zeros for the first) */
+  int32_t loop_pass;               /* >= 0: in front of this layer x <- W [x; x0] + loop.step[loop_pass], W = loop.in [emb][2 emb], x0 the embedding output */
 } ixt_layer;
 /* IXT_MIX_RETENTION: S <- decay S + (k / sqrt(dim)) v^T, o = S^T q with rotated q and k, per head; o / rms(o), times silu(W_g h) */
-enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1, IXT_MIX_ATTENTION = 2, IXT_MIX_RETENTION = 3 };
+/* IXT_MIX_LIGHTNING: q, k, v = silu of their projections, S <- decay S + k v^T, o = S^T q per head; all heads normed together (RMS, plain weight mix.norm), times
+ * sigmoid(W_g h).  IXT_MIX_SCAN (selective scan): W_in h = [x | z]; x through a causal convolution with bias and silu; W_x x = [t | B | C]; dt = softplus(W_dt t +
+ * bias); per channel c and state n S <- exp(-dt_c exp(A_log[c, n])) S + dt_c x_c B_n, y_c = sum_n S C_n + D_c x_c; W_o (y silu(z)) */
+enum { IXT_MIX_LATENT_ATTENTION = 0, IXT_MIX_GATED_DELTA = 1, IXT_MIX_ATTENTION = 2, IXT_MIX_RETENTION = 3, IXT_MIX_LIGHTNING = 4, IXT_MIX_SCAN = 5 };
 enum { IXT_ROPE_NEIGHBOURS = 0, IXT_ROPE_HALVES = 1 };      /* (2 i, 2 i + 1); (i, i + rot_dim / 2) */
 enum { IXT_FFN_NONE = 0, IXT_FFN_DENSE = 1, IXT_FFN_MOE = 2 };
 /* gated units of g = gate, u = up: min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u, -limit, limit) + 1); gelu(g) u (tanh form); silu(g) u.
- * From IXT_ACT_RELU2 on a unit has no gate: max(u, 0)^2 */
-enum { IXT_GLU_CLAMPED = 1, IXT_GLU_GELU_TANH = 2, IXT_GLU_SILU = 3, IXT_ACT_RELU2 = 4 };
+ * From IXT_ACT_RELU2 on a unit has no gate: max(u, 0)^2; a u^2 + u / 2 for u > 0, b (exp(u) - 1 - u) + u / 2 for u <= 0 with a = softplus(act[0]), b = 1/2 +
+ * softplus(act[1]) (xIELU; tensor l<i>.mlp.act; dense only) */
+enum { IXT_GLU_CLAMPED = 1, IXT_GLU_GELU_TANH = 2, IXT_GLU_SILU = 3, IXT_ACT_RELU2 = 4, IXT_ACT_XIELU = 5 };
 enum { IXT_ROUTE_SOFTMAX = 0, IXT_ROUTE_SIGMOID = 1, IXT_ROUTE_CHOSEN = 2 };      /* CHOSEN: choice by logit, weights = softmax over the chosen logits */
-/* norms around the sublayers and in front of the head: t / sqrt(mean(t^2) + eps) (1 + w); tanh(alpha t) w + b; (t - mean) / sqrt(variance + eps) w + b */
-enum { IXT_NORM_RMS = 0, IXT_NORM_TANH = 1, IXT_NORM_LAYER = 2 };
+/* norms around the sublayers and in front of the head: t / sqrt(mean(t^2) + eps) (1 + w); tanh(alpha t) w + b; (t - mean) / sqrt(variance + eps) w + b;
+ * t / sqrt(mean(t^2) + eps) g with g one number for all features */
+enum { IXT_NORM_RMS = 0, IXT_NORM_TANH = 1, IXT_NORM_LAYER = 2, IXT_NORM_ONE = 3 };
 enum { IXT_NORM_BEFORE = 1, IXT_NORM_AFTER = 2 };
 
 /* Derived hyper-parameters of MaxText/pyconfig.py:551-644 that shape the path. */

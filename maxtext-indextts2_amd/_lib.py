@@ -28,7 +28,9 @@ class IxtLayer(ctypes.Structure):
       (n, ctypes.c_float) for n in ("rope_factor", "rope_low", "rope_high", "rope_original")] + [
       (n, ctypes.c_int32) for n in ("glu", "router", "router_correction", "groups", "groups_keep", "router_norm")] + [
       ("router_scale", ctypes.c_float)] + [(n, ctypes.c_int32) for n in ("shared_ff", "number", "rope_pairs", "q_rank", "out_gate", "maps")] + [
-      ("map_diff", ctypes.c_float), ("softcap", ctypes.c_float), ("router_bias", ctypes.c_int32), ("shared_gate", ctypes.c_int32), ("decay", c_f64p)]
+      ("map_diff", ctypes.c_float), ("softcap", ctypes.c_float), ("router_bias", ctypes.c_int32), ("shared_gate", ctypes.c_int32), ("decay", c_f64p)] + [
+      (n, ctypes.c_int32) for n in ("chunk", "key_values", "mix_bias", "inner", "state", "dt_rank")] + [
+      ("mix_scale", ctypes.c_float), ("beside", vp), ("shift", ctypes.c_int32), ("loop_pass", ctypes.c_int32)]      # beside: address of another IxtLayer
 
 
 class IxtConfig(ctypes.Structure):

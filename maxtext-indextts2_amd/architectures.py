@@ -9,15 +9,17 @@ import dataclasses
 import json
 import os
 import struct
-from typing import Any, Callable, Dict, Mapping, Sequence, Tuple
+from typing import Any, Callable, Dict, Mapping, Optional, Sequence, Tuple
 
-MIX_LATENT_ATTENTION, MIX_GATED_DELTA, MIX_ATTENTION, MIX_RETENTION = 0, 1, 2, 3
-RECURRENT_MIXERS = (MIX_GATED_DELTA, MIX_RETENTION)
+MIX_LATENT_ATTENTION, MIX_GATED_DELTA, MIX_ATTENTION, MIX_RETENTION, MIX_LIGHTNING, MIX_SCAN = 0, 1, 2, 3, 4, 5
+RECURRENT_MIXERS = (MIX_GATED_DELTA, MIX_RETENTION, MIX_LIGHTNING, MIX_SCAN)
 FFN_NONE, FFN_DENSE, FFN_MOE = 0, 1, 2
-GLU_CLAMPED, GLU_GELU_TANH, GLU_SILU, ACT_RELU2 = 1, 2, 3, 4      # from ACT_RELU2 on: no gate
+GLU_CLAMPED, GLU_GELU_TANH, GLU_SILU, ACT_RELU2, ACT_XIELU = 1, 2, 3, 4, 5      # from ACT_RELU2 on: no gate
 ROUTE_SOFTMAX, ROUTE_SIGMOID, ROUTE_CHOSEN = 0, 1, 2
 ROPE_NEIGHBOURS, ROPE_HALVES = 0, 1
-NORM_RMS, NORM_TANH, NORM_LAYER = 0, 1, 2
+NORM_RMS, NORM_TANH, NORM_LAYER, NORM_ONE = 0, 1, 2, 3
+GATE_FEATURES, GATE_HEADS = 1, 2
+QK_NORM_WEIGHTS, QK_NORM_PLAIN = 1, 2
 NORM_BEFORE, NORM_AFTER = 1, 2
 
 
@@ -67,6 +69,21 @@ class HybridLayer:
   router_bias: int = 0
   shared_gate: int = 0
   decay: Tuple[float, ...] = ()
+  chunk: int = 0
+  key_values: int = 0
+  mix_bias: int = 0
+  inner: int = 1
+  state: int = 1
+  dt_rank: int = 1
+  mix_scale: float = 1.0
+  beside: Optional["HybridLayer"] = None
+  shift: int = 0
+  loop_pass: int = -1
+
+
+def carries_state(l: HybridLayer) -> bool:
+  """The layer has more than a cache of keys: tokens must come in order, and a run cannot start over in the middle."""
+  return l.mixer in RECURRENT_MIXERS or bool(l.shift) or (l.beside is not None and carries_state(l.beside))
 
 
 Shapes = Mapping[str, Tuple[int, ...]]
@@ -242,6 +259,71 @@ def suzulix_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
   }
 
 
+def _lulenex_attention(m: Mapping[str, Any], factor: float) -> Dict[str, Any]:
+  rot = m["rot"]
+  heads, kv_heads, dim, dims = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(rot["dims"])
+  if heads % kv_heads or dims % 2 or dims > dim:
+    raise ValueError(f"Lulenex: {heads} heads over {kv_heads} key heads, {dims} of {dim} dims rotated")
+  if int(m["vdim"]) != dim:
+    raise ValueError(f"Lulenex: the values are the keys, vdim ({m['vdim']}) must equal dim ({dim})")
+  return {"mixer": MIX_ATTENTION, "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "rot_dim": dims, "rope_base": float(rot["base"]), "rope_pairs": ROPE_HALVES,
+          "chunk": int((m.get("mask") or {}).get("size") or 0), "attn_scale": float(m["scale"]), "qk_norm": QK_NORM_PLAIN, "sink": 1, "out_gate": GATE_HEADS, "key_values": 1, "mix_bias": 1,
+          "mix_scale": factor}
+
+
+def _lulenex_lightning(m: Mapping[str, Any], factor: float) -> HybridLayer:
+  decay = tuple(float(d) for d in m["decay"])
+  if len(decay) != int(m["heads"]):
+    raise ValueError(f"Lulenex: {len(decay)} decays for {m['heads']} heads")
+  return HybridLayer(mixer=MIX_LIGHTNING, heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), decay=decay, mix_scale=factor)
+
+
+def _lulenex_parallel(m: Mapping[str, Any]) -> Dict[str, Any]:
+  return dict(_lulenex_attention(m["left"], float(m["left_scale"])), beside=_lulenex_lightning(m["right"], float(m["right_scale"])))
+
+
+def _lulenex_scan(m: Mapping[str, Any]) -> Dict[str, Any]:
+  return {"mixer": MIX_SCAN, "inner": int(m["inner"]), "state": int(m["state"]), "dt_rank": int(m["dt_rank"]), "conv": int(m["conv"])}
+
+
+_LULENEX_MIXERS = {"parallel": _lulenex_parallel, "mamba1": _lulenex_scan}
+
+
+def _lulenex_feed_forward(mlp: Any) -> Dict[str, Any]:
+  if mlp is None:
+    return {"ffn": FFN_NONE}
+  if mlp["kind"] != "dense":
+    raise ValueError(f"Lulenex: feed-forward kind {mlp['kind']!r}")
+  return {"ffn": FFN_DENSE, "ff": int(mlp["ff"]), "glu": ACT_XIELU}
+
+
+def lulenex_keys(cfg: Mapping[str, Any], shapes: Shapes) -> Dict[str, Any]:
+  """Lulenex: chunked attention beside lightning attention, or a selective scan, in any order behind one-number norms and a token shift; xIELU units; a
+  stretch of layers run several times, the embedding output joining in front of every pass."""
+  del shapes
+  layers = []
+  for i, entry in enumerate(cfg["layers"]):
+    if entry["type"] not in _LULENEX_MIXERS:
+      raise ValueError(f"Lulenex: layer {i} has type {entry['type']!r}")
+    layers.append(HybridLayer(number=i, shift=1, **_LULENEX_MIXERS[entry["type"]](entry["mixer"]), **_lulenex_feed_forward(entry.get("mlp"))))
+  loop = cfg.get("loop")
+  keys = _looped(layers, *((int(loop["start"]), int(loop["stop"]), int(loop["times"])) if loop else (0, 0, 1)))
+  if loop and int(loop["stop"]) > int(loop["start"]):
+    runs, start, span = list(keys["hybrid_layers"]), int(loop["start"]), int(loop["stop"]) - int(loop["start"])
+    for t in range(int(loop["times"])):
+      runs[start + t * span] = dataclasses.replace(runs[start + t * span], loop_pass=t)
+    keys["hybrid_layers"] = tuple(runs)
+  return {
+      "decoder_block": "hybrid",
+      "vocab_size": int(cfg["vocab"]),
+      "base_emb_dim": int(cfg["width"]),
+      "normalization_layer_epsilon": float(cfg["norm"]["eps"]),
+      "hybrid_norm_kind": NORM_ONE,
+      "hybrid_norm_places": NORM_BEFORE,
+      **keys,
+  }
+
+
 def _looped(layers: Sequence[HybridLayer], start: int, stop: int, times: int) -> Dict[str, Any]:
   """Layers start .. stop - 1 `times` times in a row: every further pass is a run of its own (cache, state) on the first one's parameters."""
   if not 0 <= start <= stop <= len(layers) or times < 1:
@@ -252,6 +334,7 @@ def _looped(layers: Sequence[HybridLayer], start: int, stop: int, times: int) ->
 
 
 ARCHITECTURES: Dict[str, Callable[[Mapping[str, Any], Shapes], Dict[str, Any]]] = {
+    "Lulenex": lulenex_keys,
     "Suzulix": suzulix_keys,
     "Vazilorn": vazilorn_keys,
     "Vilepel": vilepel_keys,
@@ -281,8 +364,8 @@ def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
     out["head"] = (V, E)
 
   def norm(name: str) -> None:
-    out[name] = (E,)
-    if config.hybrid_norm_kind != NORM_RMS:
+    out[name] = () if config.hybrid_norm_kind == NORM_ONE else (E,)
+    if config.hybrid_norm_kind in (NORM_TANH, NORM_LAYER):
       out[name + ".b"] = (E,)
     if config.hybrid_norm_kind == NORM_TANH:
       out[name + ".alpha"] = ()
@@ -294,6 +377,33 @@ def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
 
   both = config.hybrid_norm_places == NORM_BEFORE | NORM_AFTER
   norm("final.norm")
+  passes = 1 + max(l.loop_pass for l in config.hybrid_layers)
+  if passes > 0:
+    out["loop.in"], out["loop.step"] = (E, 2 * E), (passes, E)
+
+  def attention(p: str, l: HybridLayer) -> None:
+    sizes = {"q": l.heads * l.maps * l.dim, "k": l.kv_heads * l.maps * l.dim}
+    if not l.key_values:
+      sizes["v"] = l.kv_heads * l.vdim
+    out.update({p + t: (n, E) for t, n in sizes.items()})
+    out[p + "o"] = (E, l.heads * l.vdim)
+    if l.mix_bias:
+      out.update({p + t + ".b": (n,) for t, n in dict(sizes, o=E).items()})
+    if l.maps > 1:
+      out.update({p + n: (l.dim,) for n in ("lq1", "lk1", "lq2", "lk2")})
+    if l.qk_norm == QK_NORM_WEIGHTS:
+      out[p + "q.norm"] = out[p + "k.norm"] = (l.dim,)
+    if l.sink:
+      out[p + "sink"] = (l.heads,)
+    if l.out_gate:
+      out[p + "g"] = (l.heads * (l.vdim if l.out_gate == GATE_FEATURES else 1), E)
+
+  def linear_attention(p: str, l: HybridLayer) -> None:
+    kq, v = l.heads * l.dim, l.heads * l.vdim
+    out.update({p + "q": (kq, E), p + "k": (kq, E), p + "v": (v, E), p + "g": (v, E), p + "o": (E, v)})
+    if l.mixer == MIX_LIGHTNING:
+      out[p + "norm"] = (v,)
+
   for i, l in enumerate(config.hybrid_layers):
     if l.weights_of >= 0:
       continue
@@ -309,18 +419,15 @@ def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
         out[p + "mix.q"] = (l.heads * (l.dim + l.rot_dim), E)
       out.update({p + "mix.dkv": (l.kv_rank + l.rot_dim, E), p + "mix.dkv.norm": (l.kv_rank,),
                   p + "mix.uk": (l.heads * l.dim, l.kv_rank), p + "mix.uv": (l.heads * l.vdim, l.kv_rank), p + "mix.o": (E, l.heads * l.vdim)})
-    elif l.mixer == MIX_ATTENTION:
-      out.update({p + "mix.q": (l.heads * l.maps * l.dim, E), p + "mix.k": (l.kv_heads * l.maps * l.dim, E), p + "mix.v": (l.kv_heads * l.vdim, E),
-                  p + "mix.o": (E, l.heads * l.vdim)})
-      if l.maps > 1:
-        out.update({p + f"mix.{n}": (l.dim,) for n in ("lq1", "lk1", "lq2", "lk2")})
-      if l.qk_norm:
-        out[p + "mix.q.norm"] = out[p + "mix.k.norm"] = (l.dim,)
-      if l.sink:
-        out[p + "mix.sink"] = (l.heads,)
-    elif l.mixer == MIX_RETENTION:
-      kq, v = l.heads * l.dim, l.heads * l.vdim
-      out.update({p + "mix.q": (kq, E), p + "mix.k": (kq, E), p + "mix.v": (v, E), p + "mix.g": (v, E), p + "mix.o": (E, v)})
+      if l.out_gate:
+        out[p + "mix.g"] = (l.heads * l.vdim, E)
+    elif l.mixer in (MIX_ATTENTION, MIX_RETENTION, MIX_LIGHTNING):
+      for q, x in (("mix.", l),) if l.beside is None else (("mix.left.", l), ("mix.right.", l.beside)):
+        (attention if x.mixer == MIX_ATTENTION else linear_attention)(p + q, x)
+    elif l.mixer == MIX_SCAN:
+      C, N, r = l.inner, l.state, l.dt_rank
+      out.update({p + "mix.in": (2 * C, E), p + "mix.conv": (C, l.conv), p + "mix.conv.b": (C,), p + "mix.x": (r + 2 * N, C), p + "mix.dt": (C, r), p + "mix.dt.b": (C,),
+                  p + "mix.A_log": (C, N), p + "mix.D": (C,), p + "mix.o": (E, C)})
     else:
       kq, v = l.kv_heads * l.dim, l.heads * l.vdim
       for t, n in (("q", kq), ("k", kq), ("v", v)):
@@ -328,9 +435,11 @@ def parameter_shapes(config: Any) -> Dict[str, Tuple[int, ...]]:
       out.update({p + "mix.b": (l.heads, E), p + "mix.A_log": (l.heads,), p + "mix.norm": (l.vdim,), p + "mix.a1": (l.decay_rank, E),
                   p + "mix.a2": (l.heads * l.dim, l.decay_rank), p + "mix.dt_bias": (l.heads * l.dim,), p + "mix.g1": (l.gate_rank, E),
                   p + "mix.g2": (v, l.gate_rank), p + "mix.o": (E, v)})
-    if l.out_gate:
-      out[p + "mix.g"] = (l.heads * l.vdim, E)
+    if l.shift:
+      out[p + "shift"] = (E,)
     if l.ffn == FFN_DENSE:
+      if l.glu == ACT_XIELU:
+        out[p + "mlp.act"] = (2,)
       unit(p + "mlp.", l.ff, l.glu)
     elif l.ffn == FFN_MOE:
       for e in range(l.experts):

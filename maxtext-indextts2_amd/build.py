@@ -10,8 +10,8 @@ import tempfile
 PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(PKG_DIR, "csrc")
 LIB = os.path.join(PKG_DIR, "libixt.so")
-SOURCES = ["ixt_api.hip", "ixt_hybrid.hip", "ixt_hybrid_heads.hip", "ixt_hybrid_norm.hip", "ixt_train.hip"]
-HEADERS = ["ixt_device.h", "ixt_kernels.h", "ixt_gemma_kernels.h", "ixt_moe_kernels.h", "ixt_gemm.h", "ixt_small.h", "ixt_fp8.h", "ixt_hybrid_kernels.h", "ixt_heads_kernels.h", "ixt_retention_kernels.h", "ixt_internal.h", "ixt_hybrid.h", "ixt_train_kernels.h", os.path.join("..", "..", "include", "ixt.h"),
+SOURCES = ["ixt_api.hip", "ixt_hybrid.hip", "ixt_hybrid_heads.hip", "ixt_hybrid_norm.hip", "ixt_hybrid_state.hip", "ixt_train.hip"]
+HEADERS = ["ixt_device.h", "ixt_kernels.h", "ixt_gemma_kernels.h", "ixt_moe_kernels.h", "ixt_gemm.h", "ixt_small.h", "ixt_fp8.h", "ixt_hybrid_kernels.h", "ixt_heads_kernels.h", "ixt_retention_kernels.h", "ixt_scan_kernels.h", "ixt_internal.h", "ixt_hybrid.h", "ixt_train_kernels.h", os.path.join("..", "..", "include", "ixt.h"),
            os.path.join("..", "..", "include", "ixt_train.h")]
 
 # -ffp-contract=off: the numerics contract allows fused multiply-adds only where the source

@@ -1511,7 +1511,7 @@ static int moe_experts_routed(ixt_ctx* c, const LayerW& w, const bf16_t* x, cons
       const int ti = timing_begin(c, st, (double)K * N * 2.0 * c->NEL + (double)rows_g * K * 2.0 + out_bytes);
       dim3 grid((((nwaves + 3) / 4 + 7) / 8) * 8 * zblocks, 1, 1);
       hipLaunchKernelGGL(kern, grid, dim3(256), (size_t)64 * 1024, st, reinterpret_cast<const u32x4*>(xin), reinterpret_cast<const u32x4*>(wbase), K, N, rows_g, out, nwaves, zblocks,
-                         c->moe_rbexp, wstride, 0, 0.0f);
+                         c->moe_rbexp, wstride, 0, 0.0f, (const float*)nullptr);
       timing_end(c, st, ti);
     };
     if ((size_t)rows_g * E > c->part_floats) return set_err(IXT_ERR_INVALID, "moe: output workspace too small");

@@ -122,8 +122,13 @@ __device__ __forceinline__ float ixt_glu(int kind, float a, float b, float limit
   const float z = kind == 2 ? 1.59576912160573071176f * fmaf(0.044715f * a * a, a, a) : a;
   return a * hw_rcp(1.0f + hw_exp2(-1.44269504088896340736f * z)) * b;
 }
-// units without a gate, by kind (from IXT_ACT_RELU2 = 4 on): max(u, 0)^2
-__device__ __forceinline__ float ixt_act(int /*kind*/, float u) { const float p = fmaxf(u, 0.0f); return p * p; }
+// units without a gate, by kind (from IXT_ACT_RELU2 = 4 on): max(u, 0)^2; 5: par[0] u^2 + u / 2 for u > 0, par[1] (exp(u) - 1 - u) + u / 2 for the others
+__device__ __forceinline__ float ixt_act(int kind, float u, const float* __restrict__ par) {
+  const float p = fmaxf(u, 0.0f);
+  if (kind == 4) return p * p;
+  const float n = fminf(u, 0.0f);
+  return fmaf(0.5f, u, fmaf(par[0] * p, p, par[1] * (hw_exp2(1.44269504088896340736f * n) - 1.0f - n)));
+}
 // tanh in f32, error below 1e-6 of the value: (1 - e) / (1 + e), e = exp(-2 |x|); |x| < 1/16 by the odd series (next term < 2e-13 relative)
 __device__ __forceinline__ float tanh_f32(float x) {
   const float a = fabsf(x), w = a * a, e = hw_exp2(-2.88539008177792681472f * a);

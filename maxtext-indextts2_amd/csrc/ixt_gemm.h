@@ -90,7 +90,7 @@ struct GemmEpi {
   const float* xscale; const float* wscale;             // F8: activation scales [rows][chains], column scales [N] (ixt_fp8.h)
   size_t sstride;                                       // F8 + routed experts: floats between two experts' column scales
   TanhNormEpi tn;                                       // TANHNORM (with act)
-  int glu; float glu_limit;                             // ACT: the unit's kind; SWIGLU: glu != 0 takes that gated unit of the f32 totals instead (ixt_glu)
+  int glu; float glu_limit; const float* act_par;       // ACT: the unit's kind and its numbers; SWIGLU: glu != 0 takes that gated unit of the f32 totals instead (ixt_glu)
   const int32_t* rb_exp; size_t wstride;                // routed experts: expert of every 16-row block (-1: none), 16-byte units between experts' kernels
 };
 
@@ -338,7 +338,8 @@ __global__ __launch_bounds__(WR * WC * 64, 2) void k_gemm_ring(const u32x4* __re
         const int row = (rowg * TR + wr * RB + b) * 16 + r_in;
         if (tile < ntile && row < R) {
           uint2 ov;
-          ov.x = pack2(f2bf(ixt_act(e.glu, tot[i][b][0])), f2bf(ixt_act(e.glu, tot[i][b][1]))); ov.y = pack2(f2bf(ixt_act(e.glu, tot[i][b][2])), f2bf(ixt_act(e.glu, tot[i][b][3])));
+          ov.x = pack2(f2bf(ixt_act(e.glu, tot[i][b][0], e.act_par)), f2bf(ixt_act(e.glu, tot[i][b][1], e.act_par)));
+          ov.y = pack2(f2bf(ixt_act(e.glu, tot[i][b][2], e.act_par)), f2bf(ixt_act(e.glu, tot[i][b][3], e.act_par)));
           *reinterpret_cast<uint2*>(e.act + xidx(row, tile * 16 + cq * 4, N)) = ov;
         }
       }

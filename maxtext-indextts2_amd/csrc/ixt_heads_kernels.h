@@ -1,7 +1,8 @@
 // ixt_heads_kernels.h -- attention of hybrid decoders over keys and values per head (IXT_MIX_ATTENTION): query heads in equal groups on one key / value
 // head each, optional norm of query and key heads, rotation of a head's first features, optional window, optional sink (a number per head that joins the
 // softmax denominator without a key or a value), optional soft cap of the scores, optional gate on the concatenated heads.  Sizes of keys and values are
-// independent.  With two maps a head has two queries and its key head two keys per token, both of `d` features, over the same values; the two outputs
+// independent.  Values may be the keys as projected; a chunked mask shows a position the keys of its own chunk only; the gate may be one number per head.
+// With two maps a head has two queries and its key head two keys per token, both of `d` features, over the same values; the two outputs
 // become one: a1 - lambda a2, over its root mean square, times a constant (differential attention).
 //
 //   k_heads_prep     projection slices -> queries [R][H][dkp], the row's keys and values in their pages
@@ -19,9 +20,14 @@ struct HeadsGeom {
   int dkp, dvp;                             // padded key / value rows
   int maps, dmp;                            // softmax maps per head (1, 2); a map's part of a key row: dkp = maps dmp
   int hs, vs, ok, ov, og;                   // projection columns: a map of a query / key head takes hs, a value head vs; keys from ok on, values from ov on, gates
-                                            // (vs per query head) from og on (< 0: none)
+                                            // (vs per query head, or one: head_gate) from og on (< 0: none)
   float scale, cap;                         // cap > 0: score <- cap tanh(score / cap)
+  int chunk, head_gate;                     // chunk > 0: only keys of the position's own chunk of that many positions (window unused)
+  int oc, kend;                             // act of the output projection: the heads' first column, and where the zeros behind them end
+  float of;                                 // factor on the outputs
 };
+// the first key that position p sees
+__device__ __forceinline__ int first_key(const HeadsGeom& g, int p) { return g.chunk > 0 ? p - p % g.chunk : g.window > 0 ? max(0, p - g.window + 1) : 0; }
 struct MapsArgs { const float* lambda; float keep, eps; };               // two maps: (a1 - *lambda a2) / rms(., eps) keep
 struct RowsArgs { const int32_t *slot, *pos, *active, *page_map; };      // the rows of a pass
 
@@ -74,12 +80,18 @@ static __global__ __launch_bounds__(64) void k_maps_lambda(const float* lq1, con
   a = wave_sum(a); b = wave_sum(b);
   if (threadIdx.x == 0) *lambda = expf(a) - expf(b) + diff;
 }
-// four columns of the concatenated heads (c % 4 == 0 inside head h) times their gate
-__device__ __forceinline__ void heads_gate4(const Slices& t, int r, const HeadsGeom& g, int h, int c, float* v) {
-  float z[4];
-  t.at4(r, g.og + h * g.vs + c, z);
+// four columns of the concatenated heads (c % 4 == 0 inside head h) times their gate and the layer's factor -> act
+__device__ __forceinline__ void heads_out4(const Slices& t, int r, const HeadsGeom& g, int h, int c, float* v, bf16_t* out, int Kp) {
+  if (g.og >= 0) {
+    float z[4];
+    if (g.head_gate) z[0] = z[1] = z[2] = z[3] = t.at(r, g.og + h);
+    else t.at4(r, g.og + h * g.vs + c, z);
 #pragma unroll
-  for (int j = 0; j < 4; ++j) v[j] *= hw_rcp(1.0f + hw_exp2(-1.44269504088896340736f * z[j]));
+    for (int j = 0; j < 4; ++j) v[j] *= hw_rcp(1.0f + hw_exp2(-1.44269504088896340736f * z[j]));
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] *= g.of;
+  act_store4(out, r, g.oc + h * g.vs + c, Kp, v);
 }
 // log2(e) times the capped score, cap (1 - 2 / (1 + exp(2 s scale / cap))): c2 = 2 scale log2(e) / cap, k2 = cap log2(e)
 __device__ __forceinline__ float capped_log2(float s, float c2, float k2) { return fmaf(-2.0f * k2, hw_rcp(1.0f + hw_exp2(c2 * s)), k2); }
@@ -128,7 +140,7 @@ __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, Hea
   float* p = sm + g.dkp;
   for (int k = tid; k < g.dkp; k += 256) q[k] = to_f(qb[((size_t)r * g.H + h) * g.dkp + k]);
   __syncthreads();
-  const int pos = rows.pos[r], k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
+  const int pos = rows.pos[r], k_lo = first_key(g, pos);
   const int32_t* prow = rows.page_map + (size_t)rows.slot[r] * g.mpg;
   float o[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   for (int mi = 0; mi < g.maps; ++mi) {
@@ -185,11 +197,11 @@ __global__ __launch_bounds__(256) void k_heads_any(const T* __restrict__ qb, Hea
   for (int i = 0; i < 4; ++i) {
     const int c = tid + 256 * i;
     if (c >= g.vs) continue;
-    if (g.og >= 0 && c < g.dv) o[i] *= f32_sigmoid(t.at(r, g.og + h * g.vs + c));
-    act_store1(out, r, h * g.vs + c, Kp, o[i]);
+    if (g.og >= 0 && c < g.dv) o[i] *= f32_sigmoid(t.at(r, g.og + (g.head_gate ? h : h * g.vs + c)));
+    act_store1(out, r, g.oc + h * g.vs + c, Kp, o[i] * g.of);
   }
   if (h == g.H - 1)
-    for (int k = g.H * g.vs + tid; k < Kp; k += 256) act_store1(out, r, k, Kp, 0.0f);
+    for (int k = g.oc + g.H * g.vs + tid; k < g.kend; k += 256) act_store1(out, r, k, Kp, 0.0f);
 }
 
 // ---------------------------------------------------------------------------------------------------- matrix-core forms
@@ -203,7 +215,7 @@ struct HeadsAttnArgs {
   RowsArgs rows;
   bf16_t *kpages, *vpages;
   int R, NQ, HB, hchunks, pshift;           // rows per block, query heads per block, blocks of query heads per key / value head
-  bf16_t* out; int Kp;                      // act, column h vs + c
+  bf16_t* out; int Kp;                      // act, column oc + h vs + c
   float *part_o, *part_ml;                  // splits > 1: [R H maps][splits][dvp], [R H maps][splits][2]
   Slices t; const float *qn, *kn; float eps; HeadsRope rope;      // the projection (gates); k_heads_decode with FUSED: and what k_heads_prep needs
   MapsArgs mp;
@@ -255,9 +267,9 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
     while (rb < nr && a.rows.active[r0 + rb] && a.rows.slot[r0 + rb] == slot) { const int p = a.rows.pos[r0 + rb]; lo = min(lo, p); hi = max(hi, p); ++rb; }
     const bool whole = ra == 0 && rb == nr;               // no other run in this block: only the keys decide what is masked
     const bool mine = live && qi >= ra && qi < rb;
-    const int my_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0;
+    const int my_lo = mine ? first_key(g, pos) : 0;
     ra = rb;
-    const int k_lo = g.window > 0 ? max(0, lo - g.window + 1) : 0, k_all = g.window > 0 ? max(0, hi - g.window + 1) : 0;    // (k_all .. lo: seen by every row)
+    const int k_lo = first_key(g, lo), k_all = first_key(g, hi);      // (k_all .. lo: seen by every row)
     const int ntile = (hi - k_lo) / 64 + 1;
     const int32_t* prow = a.rows.page_map + (size_t)slot * g.mpg;
     __syncthreads();                                      // the previous run's last tile has been read
@@ -395,12 +407,11 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
   for (int i = 0; i < NT; ++i) {
     float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
     if (i * 16 + cq * 4 >= g.vs) continue;
-    if (g.og >= 0) heads_gate4(a.t, row, g, head, i * 16 + cq * 4, v);
-    act_store4(a.out, row, head * g.vs + i * 16 + cq * 4, a.Kp, v);      // (columns dv .. vs - 1 are zero: so are the values there)
+    heads_out4(a.t, row, g, head, i * 16 + cq * 4, v, a.out, a.Kp);      // (columns dv .. vs - 1 are zero: so are the values there)
   }
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   if (head == g.H - 1)
-    for (int c = g.H * g.vs + cq * 4; c < a.Kp; c += 16) act_store4(a.out, row, c, a.Kp, z);
+    for (int c = g.oc + g.H * g.vs + cq * 4; c < g.kend; c += 16) act_store4(a.out, row, c, a.Kp, z);
 }
 
 // Few rows (decode): a block owns up to 16 query heads of one key / value head of ONE row and every gridDim.z-th key tile of its window.  Scores: a wave
@@ -426,7 +437,7 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
   const bool pair_ok = r_in < nu;
   const int u_in = pair_ok ? r_in : 0, map = u_in % MAPS, head = h0 + u_in / MAPS;
   const int32_t* prow = a.rows.page_map + (size_t)slot * g.mpg;
-  const int k_lo = g.window > 0 ? max(0, pos - g.window + 1) : 0, ntile = (pos - k_lo) / 64 + 1;
+  const int k_lo = first_key(g, pos), ntile = (pos - k_lo) / 64 + 1;
   int t = blockIdx.z;
   if (t < ntile) {
     const int off = heads_row(prow, min(k_lo + t * 64 + lane, pos), a.pshift, g.G, kh);
@@ -569,15 +580,14 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
     if (nsplit == 1) {
       if (c >= g.vs) continue;
-      if (g.og >= 0) heads_gate4(a.t, row, g, head, c, v);
-      act_store4(a.out, row, head * g.vs + c, a.Kp, v);
+      heads_out4(a.t, row, g, head, c, v, a.out, a.Kp);
     } else *reinterpret_cast<float4*>(a.part_o + pi * DV + c) = make_float4(v[0], v[1], v[2], v[3]);
   }
   if (nsplit > 1) {
     if (wave == 0 && cq == 0) { a.part_ml[pi * 2] = m; a.part_ml[pi * 2 + 1] = l; }
   } else if (head == g.H - 1 && wave == 0) {
     const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-    for (int c = g.H * g.vs + cq * 4; c < a.Kp; c += 16) act_store4(a.out, row, c, a.Kp, z);
+    for (int c = g.oc + g.H * g.vs + cq * 4; c < g.kend; c += 16) act_store4(a.out, row, c, a.Kp, z);
   }
 }
 // the key splits of a row's heads (and their maps) put together.  grid (R, H), block 64; nsplit <= 16, vs <= 256.
@@ -600,11 +610,8 @@ static __global__ __launch_bounds__(64) void k_heads_combine(const float* __rest
 #pragma unroll
     for (int j = 0; j < 4; ++j) v[j] *= rs;
   }
-  if (c < vs) {
-    if (g.og >= 0) heads_gate4(t, r, g, h, c, v);
-    act_store4(out, r, h * vs + c, Kp, v);
-  }
+  if (c < vs) heads_out4(t, r, g, h, c, v, out, Kp);
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   if (h == H - 1)
-    for (int c = H * vs + tid * 4; c < Kp; c += 256) act_store4(out, r, c, Kp, z);
+    for (int c = g.oc + H * vs + tid * 4; c < g.kend; c += 256) act_store4(out, r, c, Kp, z);
 }

@@ -52,36 +52,56 @@ static int h_load_mat(const HybridModel* m, const void* src, int dtype, void* ds
   return m->f32 ? h_load_nk(src, dtype, (float*)dst, lm, st) : h_load_nk(src, dtype, (bf16_t*)dst, lm, st);
 }
 
+static bool column_mixer(const ixt_layer& l) { return l.mixer == IXT_MIX_ATTENTION || l.mixer == IXT_MIX_RETENTION || l.mixer == IXT_MIX_LIGHTNING; }      // columns of one input projection, rows of one output projection
+static int check_mixer(const ixt_layer& l, int i) {
+  if (l.heads < 1 || l.dim < 1 || l.vdim < 1) return set_err(IXT_ERR_INVALID, "layer %d: heads / dim / vdim", i);
+  if (l.rope_pairs != IXT_ROPE_NEIGHBOURS && l.rope_pairs != IXT_ROPE_HALVES) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: rope_pairs %d", i, l.rope_pairs);
+  if (l.mixer == IXT_MIX_LATENT_ATTENTION) {
+    if (l.kv_rank < 1 || l.kv_rank > 1024 || l.rot_dim < 0 || l.rot_dim % 2 || l.q_rank < 0)
+      return set_err(IXT_ERR_UNSUPPORTED, "layer %d: kv_rank %d (1 .. 1024), rot_dim %d (even), q_rank %d", i, l.kv_rank, l.rot_dim, l.q_rank);
+  } else if (l.mixer == IXT_MIX_GATED_DELTA) {
+    if (l.kv_heads < 1 || l.heads % l.kv_heads || l.conv < 1 || l.decay_rank < 1 || l.gate_rank < 1) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / conv / ranks", i);
+    if (l.dim > 512) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: delta rule key dims %d (at most 512)", i, l.dim);
+  } else if (l.mixer == IXT_MIX_ATTENTION) {
+    if (l.kv_heads < 1 || l.heads % l.kv_heads || l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > l.dim) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / rot_dim", i);
+    if (l.maps < 0 || l.maps > 2 || !(l.softcap >= 0.0f)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d maps (1, 2), soft cap %g", i, l.maps, l.softcap);
+    if (l.dim > 4096 || l.vdim > 1024) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d key dims (at most 4096), %d value dims (at most 1024)", i, l.dim, l.vdim);
+    if (!(l.attn_scale > 0.0f)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: score factor %g (positive)", i, l.attn_scale);
+    if (l.rope_factor > 0.0f && !(l.rope_low > 0.0f && l.rope_high > l.rope_low && l.rope_original > 0.0f)) return set_err(IXT_ERR_INVALID, "layer %d: rotation scaling", i);
+    if (l.key_values && (l.maps > 1 || l.dim != l.vdim)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: keys as values with %d maps, %d key and %d value dims", i, l.maps, l.dim, l.vdim);
+    if (l.chunk > 0 && l.window > 0) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: chunks of %d and a window of %d", i, l.chunk, l.window);
+    if (l.qk_norm < 0 || l.qk_norm > 2 || l.out_gate < 0 || l.out_gate > 2) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: qk_norm %d, out_gate %d", i, l.qk_norm, l.out_gate);
+  } else if (l.mixer == IXT_MIX_RETENTION || l.mixer == IXT_MIX_LIGHTNING) {
+    if (!l.decay || l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > l.dim) return set_err(IXT_ERR_INVALID, "layer %d: decays / rot_dim", i);
+    if (l.dim > 1024 || l.vdim > 1024) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d key dims, %d value dims (at most 1024)", i, l.dim, l.vdim);
+  } else if (l.mixer == IXT_MIX_SCAN) {
+    if (l.inner < 1 || l.state < 1 || l.dt_rank < 1 || l.conv < 1) return set_err(IXT_ERR_INVALID, "layer %d: inner / state / dt_rank / conv", i);
+    if (l.state > 256) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d states per channel (at most 256)", i, l.state);
+  } else return set_err(IXT_ERR_UNSUPPORTED, "layer %d: mixer %d", i, l.mixer);
+  if (l.mix_scale != 1.0f && !column_mixer(l)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: a factor on mixer %d", i, l.mixer);
+  return IXT_OK;
+}
+
 int hybrid_check(const ixt_config& c) {
   if (!c.layers || c.num_decoder_layers < 1) return set_err(IXT_ERR_INVALID, "hybrid decoder: no layers");
   if (c.emb_dim < 1 || c.emb_dim > 12288 || c.vocab_size < 1) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: emb_dim %d (1 .. 12288), vocab_size %d", c.emb_dim, c.vocab_size);
   if (c.fp8_weights) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: fp8 weights are not built");
-  if (c.norm_kind < IXT_NORM_RMS || c.norm_kind > IXT_NORM_LAYER || c.norm_places < IXT_NORM_BEFORE || c.norm_places > (IXT_NORM_BEFORE | IXT_NORM_AFTER))
+  if (c.norm_kind < IXT_NORM_RMS || c.norm_kind > IXT_NORM_ONE || c.norm_places < IXT_NORM_BEFORE || c.norm_places > (IXT_NORM_BEFORE | IXT_NORM_AFTER))
     return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: norm kind %d, places %d", c.norm_kind, c.norm_places);
   if (c.streams < 0 || c.streams > HC_MAX) return set_err(IXT_ERR_UNSUPPORTED, "hybrid decoder: %d streams (at most %d)", c.streams, HC_MAX);
   for (int i = 0; i < c.num_decoder_layers; ++i) {
     const ixt_layer& l = c.layers[i];
-    if (l.rope_pairs != IXT_ROPE_NEIGHBOURS && l.rope_pairs != IXT_ROPE_HALVES) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: rope_pairs %d", i, l.rope_pairs);
     if (l.weights_of >= c.num_decoder_layers || (l.weights_of >= 0 && c.layers[l.weights_of].weights_of >= 0) || l.weights_of == i)
       return set_err(IXT_ERR_INVALID, "layer %d: weights_of %d", i, l.weights_of);
-    if (l.heads < 1 || l.dim < 1 || l.vdim < 1) return set_err(IXT_ERR_INVALID, "layer %d: heads / dim / vdim", i);
-    if (l.mixer == IXT_MIX_LATENT_ATTENTION) {
-      if (l.kv_rank < 1 || l.kv_rank > 1024 || l.rot_dim < 0 || l.rot_dim % 2 || l.q_rank < 0)
-        return set_err(IXT_ERR_UNSUPPORTED, "layer %d: kv_rank %d (1 .. 1024), rot_dim %d (even), q_rank %d", i, l.kv_rank, l.rot_dim, l.q_rank);
-    } else if (l.mixer == IXT_MIX_GATED_DELTA) {
-      if (l.kv_heads < 1 || l.heads % l.kv_heads || l.conv < 1 || l.decay_rank < 1 || l.gate_rank < 1) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / conv / ranks", i);
-      if (l.dim > 512) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: delta rule key dims %d (at most 512)", i, l.dim);
-    } else if (l.mixer == IXT_MIX_ATTENTION) {
-      if (l.kv_heads < 1 || l.heads % l.kv_heads || l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > l.dim) return set_err(IXT_ERR_INVALID, "layer %d: kv_heads / rot_dim", i);
-      if (l.maps < 0 || l.maps > 2 || !(l.softcap >= 0.0f)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d maps (1, 2), soft cap %g", i, l.maps, l.softcap);
-      if (l.dim > 4096 || l.vdim > 1024) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d key dims (at most 4096), %d value dims (at most 1024)", i, l.dim, l.vdim);
-      if (!(l.attn_scale > 0.0f)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: score factor %g (positive)", i, l.attn_scale);
-      if (l.rope_factor > 0.0f && !(l.rope_low > 0.0f && l.rope_high > l.rope_low && l.rope_original > 0.0f)) return set_err(IXT_ERR_INVALID, "layer %d: rotation scaling", i);
-    } else if (l.mixer == IXT_MIX_RETENTION) {
-      if (!l.decay || l.rot_dim < 0 || l.rot_dim % 2 || l.rot_dim > l.dim) return set_err(IXT_ERR_INVALID, "layer %d: decays / rot_dim", i);
-      if (l.dim > 1024 || l.vdim > 1024) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %d key dims, %d value dims (at most 1024)", i, l.dim, l.vdim);
-    } else return set_err(IXT_ERR_UNSUPPORTED, "layer %d: mixer %d", i, l.mixer);
-    if (l.ffn != IXT_FFN_NONE && (l.glu < IXT_GLU_CLAMPED || l.glu > IXT_ACT_RELU2)) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: unit %d", i, l.glu);
+    TRY(check_mixer(l, i));
+    if (l.beside) {
+      TRY(check_mixer(*l.beside, i));
+      if (!column_mixer(l) || !column_mixer(*l.beside) || l.beside->beside || l.beside->mix_bias)
+        return set_err(IXT_ERR_UNSUPPORTED, "layer %d: mixers %d and %d side by side (attention over heads, retention, lightning; output biases of the first one only)", i, l.mixer, l.beside->mixer);
+    }
+    if (l.loop_pass >= 0 && c.streams > 0) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: a pass with an input of its own among streams", i);
+    if (l.shift && (c.streams > 0 || !(c.norm_places & IXT_NORM_BEFORE))) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: token shift among streams or without a norm in front", i);
+    if (l.ffn != IXT_FFN_NONE && (l.glu < IXT_GLU_CLAMPED || l.glu > IXT_ACT_XIELU || (l.glu == IXT_ACT_XIELU && l.ffn != IXT_FFN_DENSE))) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: unit %d", i, l.glu);
     if (l.ffn == IXT_FFN_MOE) {
       if (l.experts < 1 || l.experts > 1024 || l.top < 1 || l.top > l.experts || l.ff < 1 || l.shared_ff < 0)
         return set_err(IXT_ERR_UNSUPPORTED, "layer %d: experts %d (1 .. 1024), top %d", i, l.experts, l.top);
@@ -95,7 +115,7 @@ int hybrid_check(const ixt_config& c) {
   return IXT_OK;
 }
 
-// a norm's tensors: `name`, name.b (tanh and layer norms), name.alpha (tanh norms: a scalar); zeros behind the E features
+// a norm's tensors: `name` (IXT_NORM_ONE: a scalar), name.b (tanh and layer norms), name.alpha (tanh norms: a scalar); zeros behind the E features
 static int hybrid_norm_params(ixt_ctx* c, const std::string& name, NormW* w) {
   HybridModel* m = c->hy;
   const int E = m->E;
@@ -106,6 +126,7 @@ static int hybrid_norm_params(ixt_ctx* c, const std::string& name, NormW* w) {
     m->tensors[t] = HTensor{std::move(shape), [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, d, n, st); }, false};
     return IXT_OK;
   };
+  if (m->norm_kind == IXT_NORM_ONE) return one(name, &w->w, 1, {});
   TRY(one(name, &w->w, E, {E}));
   if (m->norm_kind == IXT_NORM_TANH) TRY(one(name + ".alpha", &w->alpha, 1, {}));
   if (m->norm_kind != IXT_NORM_RMS) TRY(one(name + ".b", &w->b, E, {E}));
@@ -148,11 +169,102 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     }
     return IXT_OK;
   };
+  // the tensors of a mixer that owns columns c0 .. of `in` and rows oc .. of `o`
+  auto columns = [&](HLayer& X, const std::string& q) -> int {
+    const ixt_layer& x = X.c;
+    const HMat &in = L.in, &o = L.o;
+    float* ib = L.ibias;
+    auto bias = [&](const std::string& name, LoadMap lm) {
+      lm.k = lm.ld = lm.Kp = 1;
+      add(q + name, {lm.n}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, ib, lm, st); });
+    };
+    if (x.mixer == IXT_MIX_ATTENTION) {
+      const HeadsGeom& g = X.hg;
+      LoadMap lq = load_map(g.H * g.maps * g.d, E, in.Kp, X.c0), lk = load_map(g.G * g.maps * g.d, E, in.Kp, X.c0 + g.ok), lv = load_map(g.G * g.dv, E, in.Kp, X.c0 + g.ov);
+      lq.ng = lk.ng = g.d; lq.ngp = lk.ngp = g.hs; lv.ng = g.dv; lv.ngp = g.vs;
+      lq = rotated(lq, x, g.d, 0); lk = rotated(lk, x, g.d, 0);
+      mat_as(q + "q", in, lq);
+      mat_as(q + "k", in, lk);
+      if (!x.key_values) mat_as(q + "v", in, lv);
+      if (x.mix_bias) {
+        bias("q.b", lq); bias("k.b", lk);
+        if (!x.key_values) bias("v.b", lv);
+        TRY(h_allocf(c, &X.obias, (size_t)m->Ep));
+        float* ob = X.obias;
+        add(q + "o.b", {E}, [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, ob, (int64_t)E, st); });
+      }
+      if (g.og >= 0) {
+        LoadMap gm = load_map(g.head_gate ? g.H : g.H * g.dv, E, in.Kp, X.c0 + g.og);
+        if (!g.head_gate) { gm.ng = g.dv; gm.ngp = g.vs; }
+        mat_as(q + "g", in, gm);
+      }
+      if (g.maps == 2) {                                          // every one of the four vectors works lambda out anew: the last to come leaves the right one
+        const int n = up_to(g.d, 4);
+        TRY(h_allocf(c, &X.maps, (size_t)4 * n)); TRY(h_allocf(c, &X.lambda, 4));
+        const char* names[4] = {"lq1", "lk1", "lq2", "lk2"};
+        float *base = X.maps, *lam = X.lambda;
+        const int d = g.d;
+        const float diff = x.map_diff;
+        for (int j = 0; j < 4; ++j) {
+          float* to = base + (size_t)j * n;
+          add(q + names[j], {d}, [=](const void* s, int dt, hipStream_t st) -> int {
+            TRY(h_load_vec(s, dt, to, (int64_t)d, st));
+            hipLaunchKernelGGL(k_maps_lambda, dim3(1), dim3(64), 0, st, base, base + n, base + 2 * n, base + 3 * n, d, diff, lam);
+            LAUNCHCHK();
+            return IXT_OK;
+          });
+        }
+      }
+      if (x.qk_norm == 2) {                                       // (one vector of ones serves both)
+        TRY(h_allocf(c, &X.qn, (size_t)up_to(g.d, 4)));
+        const std::vector<float> ones(g.d, 1.0f);
+        HIPCHK(hipMemcpy(X.qn, ones.data(), ones.size() * 4, hipMemcpyHostToDevice));
+        X.kn = X.qn;
+      } else if (x.qk_norm) {
+        for (int j = 0; j < 2; ++j) {
+          float** dst = j == 0 ? &X.qn : &X.kn;
+          TRY(h_allocf(c, dst, (size_t)up_to(g.d, 4)));
+          float* d = *dst;
+          const LoadMap lm = rotated(load_map(g.d, 1, 1), x, g.d, 0);
+          add(q + (j == 0 ? "q.norm" : "k.norm"), {g.d}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, lm, st); });
+        }
+      }
+      if (x.sink) TRY(vec(q + "sink", &X.sink, g.H, {g.H}));
+      LoadMap lo = load_map(E, g.H * g.dv, o.Kp, 0, g.oc);
+      lo.kg = g.dv; lo.kgp = g.vs;
+      if (x.key_values && lk.rn > 0) { lo.krg = g.d; lo.krn = lk.rn; }
+      mat_as(q + "o", o, lo);
+      return IXT_OK;
+    }
+    const RetGeom& g = X.rg;
+    for (const char* t : {"q", "k", "v", "g"}) {
+      const bool qk = *t == 'q' || *t == 'k';
+      LoadMap lm = load_map(g.H * (qk ? g.d : g.dv), E, in.Kp, X.c0 + (*t == 'q' ? 0 : *t == 'k' ? g.ok : *t == 'v' ? g.ov : g.og));
+      lm.ng = qk ? g.d : g.dv; lm.ngp = qk ? g.hs : g.vs;
+      mat_as(q + t, in, qk ? rotated(lm, x, g.d, 0) : lm);
+    }
+    if (g.join_norm) {
+      TRY(h_allocf(c, &X.onorm, (size_t)g.H * g.vs));
+      float* d = X.onorm;
+      LoadMap lm = load_map(g.H * g.dv, 1, 1);
+      lm.ng = g.dv; lm.ngp = g.vs;
+      add(q + "norm", {g.H * g.dv}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, lm, st); });
+    }
+    LoadMap lo = load_map(E, g.H * g.dv, o.Kp, 0, g.oc);
+    lo.kg = g.dv; lo.kgp = g.vs;
+    mat_as(q + "o", o, lo);
+    return IXT_OK;
+  };
   TRY(hyper("hc1.", &L.hc1, true));
   TRY(hyper("hc2.", &L.hc2, l.ffn != IXT_FFN_NONE));
   const bool both = m->norm_places == (IXT_NORM_BEFORE | IXT_NORM_AFTER);
   TRY(norm("norm1", m->norm_places & IXT_NORM_BEFORE ? &L.n1 : &L.n1b));
   if (both) TRY(norm("norm1b", &L.n1b));
+  if (l.shift) {
+    TRY(h_allocf(c, &L.mu, (size_t)m->Ep));
+    float* d = L.mu;
+    add("shift", {E}, [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, d, (int64_t)E, st); });
+  }
   if (l.mixer == IXT_MIX_LATENT_ATTENTION) {
     const LatentGeom& g = L.lg;
     const int NQ = g.H * (g.dn + g.dr);
@@ -184,63 +296,57 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
     });
     TRY(h_mat(c, &L.o, g.H * l.vdim, E));
     mat("mix.o", L.o, E, g.H * l.vdim, 0);
-  } else if (l.mixer == IXT_MIX_ATTENTION) {
-    const HeadsGeom& g = L.hg;
-    TRY(h_mat(c, &L.in, E, g.og >= 0 ? g.og + g.H * g.vs : g.ov + g.G * g.vs));
-    LoadMap q = load_map(g.H * g.maps * g.d, E, L.in.Kp), k = load_map(g.G * g.maps * g.d, E, L.in.Kp, g.ok), v = load_map(g.G * g.dv, E, L.in.Kp, g.ov);
-    q.ng = k.ng = g.d; q.ngp = k.ngp = g.hs; v.ng = g.dv; v.ngp = g.vs;
-    mat_as("mix.q", L.in, rotated(q, l, g.d, 0));
-    mat_as("mix.k", L.in, rotated(k, l, g.d, 0));
-    mat_as("mix.v", L.in, v);
-    if (g.og >= 0) {
-      LoadMap gm = load_map(g.H * g.dv, E, L.in.Kp, g.og);
-      gm.ng = g.dv; gm.ngp = g.vs;
-      mat_as("mix.g", L.in, gm);
+  } else if (column_mixer(l)) {
+    TRY(h_mat(c, &L.in, E, L.in_cols));
+    TRY(h_mat(c, &L.o, L.o_rows, E));
+    if (l.mix_bias) TRY(h_allocf(c, &L.ibias, (size_t)L.in.Np));
+    TRY(columns(L, L.side ? "mix.left." : "mix."));
+    if (L.side) TRY(columns(*L.side, "mix.right."));
+  } else if (l.mixer == IXT_MIX_SCAN) {
+    const ScanGeom& g = L.sg;
+    const int64_t C = g.C, N = g.N;
+    TRY(h_mat(c, &L.in, E, g.oz + g.C));
+    {
+      HMat& M = L.in;
+      char* d = (char*)M.w;
+      const LoadMap x = load_map(g.C, E, M.Kp), z = load_map(g.C, E, M.Kp, g.oz);
+      add("mix.in", {2 * C, E}, [=](const void* s, int dt, hipStream_t st) {
+        TRY(h_load_mat(m, s, dt, d, x, st));
+        return h_load_mat(m, (const char*)s + (size_t)C * E * (dt == IXT_F32 ? 4 : 2), dt, d, z, st);
+      });
     }
-    if (g.maps == 2) {                                            // every one of the four vectors works lambda out anew: the last to come leaves the right one
-      const int n = up_to(g.d, 4);
-      TRY(h_allocf(c, &L.maps, (size_t)4 * n)); TRY(h_allocf(c, &L.lambda, 4));
-      const char* names[4] = {"lq1", "lk1", "lq2", "lk2"};
-      float *base = L.maps, *lam = L.lambda;
-      const int d = g.d;
-      const float diff = l.map_diff;
-      for (int j = 0; j < 4; ++j) {
-        float* to = base + (size_t)j * n;
-        add(std::string("mix.") + names[j], {d}, [=](const void* s, int dt, hipStream_t st) -> int {
-          TRY(h_load_vec(s, dt, to, (int64_t)d, st));
-          hipLaunchKernelGGL(k_maps_lambda, dim3(1), dim3(64), 0, st, base, base + n, base + 2 * n, base + 3 * n, d, diff, lam);
-          LAUNCHCHK();
-          return IXT_OK;
-        });
-      }
+    TRY(vec("mix.conv", &L.cw, C * g.taps, {C, g.taps}));
+    TRY(vec("mix.conv.b", &L.cb, C, {C}));
+    TRY(h_mat(c, &L.low, g.C, g.oc + g.N));
+    {
+      char* d = (char*)L.low.w;
+      const LoadMap t = load_map(g.rank, g.C, L.low.Kp), b = load_map(g.N, g.C, L.low.Kp, g.ob), y = load_map(g.N, g.C, L.low.Kp, g.oc);
+      const int rank = g.rank;
+      add("mix.x", {rank + 2 * N, C}, [=](const void* s, int dt, hipStream_t st) {
+        const size_t row = (size_t)C * (dt == IXT_F32 ? 4 : 2);
+        TRY(h_load_mat(m, s, dt, d, t, st));
+        TRY(h_load_mat(m, (const char*)s + rank * row, dt, d, b, st));
+        return h_load_mat(m, (const char*)s + (rank + N) * row, dt, d, y, st);
+      });
     }
-    if (l.qk_norm) {
-      for (int j = 0; j < 2; ++j) {
-        float** dst = j == 0 ? &L.qn : &L.kn;
-        TRY(h_allocf(c, dst, (size_t)up_to(g.d, 4)));
-        float* d = *dst;
-        const LoadMap lm = rotated(load_map(g.d, 1, 1), l, g.d, 0);
-        add(j == 0 ? "mix.q.norm" : "mix.k.norm", {g.d}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, lm, st); });
-      }
+    TRY(h_mat(c, &L.dt, g.rank, g.C));
+    mat("mix.dt", L.dt, g.C, g.rank, 0);
+    TRY(h_allocf(c, &L.dtb, (size_t)L.dt.Np)); TRY(h_allocf(c, &L.a2, (size_t)g.C * g.Np)); TRY(h_allocf(c, &L.D, (size_t)g.Cp));
+    {
+      float *b = L.dtb, *a2 = L.a2, *D = L.D;
+      const int Np = g.Np;
+      add("mix.dt.b", {C}, [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, b, C, st); });
+      add("mix.D", {C}, [=](const void* s, int dt, hipStream_t st) { return h_load_vec(s, dt, D, C, st); });
+      const LoadMap lm = load_map(g.C, g.N, Np);
+      add("mix.A_log", {C, N}, [=](const void* s, int dt, hipStream_t st) -> int {
+        TRY(h_load_nk(s, dt, a2, lm, st));
+        hipLaunchKernelGGL(k_scan_rates, dim3((unsigned)((C * Np + 255) / 256)), dim3(256), 0, st, a2, (int)C, (int)N, Np);
+        LAUNCHCHK();
+        return IXT_OK;
+      });
     }
-    if (l.sink) TRY(vec("mix.sink", &L.sink, g.H, {g.H}));
-    TRY(h_mat(c, &L.o, g.H * g.vs, E));
-    LoadMap o = load_map(E, g.H * g.dv, L.o.Kp);
-    o.kg = g.dv; o.kgp = g.vs;
-    mat_as("mix.o", L.o, o);
-  } else if (l.mixer == IXT_MIX_RETENTION) {
-    const RetGeom& g = L.rg;
-    TRY(h_mat(c, &L.in, E, g.og + g.H * g.vs));
-    for (const char* t : {"q", "k", "v", "g"}) {
-      const bool qk = *t == 'q' || *t == 'k';
-      LoadMap lm = load_map(g.H * (qk ? g.d : g.dv), E, L.in.Kp, *t == 'q' ? 0 : *t == 'k' ? g.ok : *t == 'v' ? g.ov : g.og);
-      lm.ng = qk ? g.d : g.dv; lm.ngp = qk ? g.hs : g.vs;
-      mat_as(std::string("mix.") + t, L.in, qk ? rotated(lm, l, g.d, 0) : lm);
-    }
-    TRY(h_mat(c, &L.o, g.H * g.vs, E));
-    LoadMap o = load_map(E, g.H * g.dv, L.o.Kp);
-    o.kg = g.dv; o.kgp = g.vs;
-    mat_as("mix.o", L.o, o);
+    TRY(h_mat(c, &L.o, g.C, E));
+    mat("mix.o", L.o, E, g.C, 0);
   } else {
     const DeltaGeom& g = L.dg;
     TRY(h_mat(c, &L.in, E, g.og + g.rg));
@@ -265,9 +371,9 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
   if (l.ffn == IXT_FFN_NONE) {                                   // a layer without a feed-forward has no use for its norms
     for (const char* n : {"norm2", "norm2b"}) {
       if (!both && std::string(n) == "norm2b") continue;
-      m->tensors[p + n] = HTensor{{E}, nullptr, true};
+      m->tensors[p + n] = HTensor{m->norm_kind == IXT_NORM_ONE ? std::vector<int64_t>{} : std::vector<int64_t>{E}, nullptr, true};
       if (m->norm_kind == IXT_NORM_TANH) m->tensors[p + n + ".alpha"] = HTensor{{}, nullptr, true};
-      if (m->norm_kind != IXT_NORM_RMS) m->tensors[p + n + ".b"] = HTensor{{E}, nullptr, true};
+      if (m->norm_kind == IXT_NORM_TANH || m->norm_kind == IXT_NORM_LAYER) m->tensors[p + n + ".b"] = HTensor{{E}, nullptr, true};
     }
     return IXT_OK;
   }
@@ -289,6 +395,16 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
   TRY(h_mat(c, &L.down, l.ff, E, n));
   L.gu_stride = (size_t)L.gu.Kp * L.gu.Np; L.down_stride = (size_t)L.down.Kp * L.down.Np;
   for (int e = 0; e < n; ++e) unit(moe ? "mlp.e" + std::to_string(e) + "." : "mlp.", L.gu, L.down, l.ff, e * L.gu_stride, e * L.down_stride);
+  if (l.glu == IXT_ACT_XIELU) {
+    TRY(h_allocf(c, &L.unit, 4)); TRY(h_allocf(c, &L.unit_par, 4));
+    float *d = L.unit, *par = L.unit_par;
+    add("mlp.act", {2}, [=](const void* s, int dt, hipStream_t st) -> int {
+      TRY(h_load_vec(s, dt, d, (int64_t)2, st));
+      hipLaunchKernelGGL(k_xielu_numbers, dim3(1), dim3(64), 0, st, d, par);
+      LAUNCHCHK();
+      return IXT_OK;
+    });
+  }
   if (!moe) return IXT_OK;
   if (l.shared_ff > 0) {
     TRY(h_mat(c, &L.sgu, E, (gated ? 2 : 1) * up_to(l.shared_ff, IXT_KALIGN)));
@@ -356,16 +472,63 @@ int hybrid_init(ixt_ctx* c) {
     if (!tied) m->tensors["head"] = HTensor{{m->V, m->E}, head, false}; }
   TRY(hybrid_norm_params(c, "final.norm", &m->fnorm));
   std::map<std::vector<float>, std::pair<float*, float*>> ropes;
-  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0, ret_u = 0;
+  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0, ret_u = 0, part3 = 0, scan_x = 0, scan_u = 0, scan_s = 0;
+  bool shifts = false;
   const size_t max_chunks = (size_t)R / SEG_CHUNK + (size_t)std::min(R, c->G) + 1;      // of a pass: a group has at most one run of rows
   auto upd = [](size_t& a, size_t v) { if (v > a) a = v; };
   // f32 slices of a dot over at most R rows (split-K only below 128 rows; launch_dot keeps to one slice when the slices do not fit)
-  auto dotsz = [&](int K, int N) { upd(part, std::max((size_t)R * N, (size_t)std::min(R, 128) * N * ((K + IXT_CHAIN - 1) / IXT_CHAIN))); };
+  auto dot_floats = [&](int K, int N) { return std::max((size_t)R * N, (size_t)std::min(R, 128) * N * ((K + IXT_CHAIN - 1) / IXT_CHAIN)); };
+  auto dotsz = [&](int K, int N) { upd(part, dot_floats(K, N)); };
+  // a mixer of columns c0 .. of the input projection and rows oc .. of the output projection: its geometry, caches and states
+  auto columns = [&](HLayer& L, int i, int c0, int oc) -> int {
+    const ixt_layer& l = L.c;
+    L.c0 = c0;
+    if (l.mixer == IXT_MIX_ATTENTION) {
+      HeadsGeom& g = L.hg;
+      g.H = l.heads; g.G = l.kv_heads; g.d = l.dim; g.dv = l.vdim; g.rot = l.rot_dim; g.P = c->P; g.mpg = c->mpg; g.window = l.window; g.chunk = std::max(l.chunk, 0); g.scale = l.attn_scale;
+      g.maps = std::max(l.maps, 1); g.cap = l.softcap; g.head_gate = l.out_gate == 2; g.oc = oc; g.of = l.mix_scale;
+      if (!heads_mfma_sizes(l.dim, g.maps, l.vdim, m->f32, &g.dkp, &g.dvp)) { g.dkp = g.maps * up_to(l.dim, 32); g.dvp = up_to(l.vdim, 32); }
+      g.dmp = g.dkp / g.maps;
+      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4); g.ok = up_to(g.H * g.maps * g.hs, 16);
+      g.ov = l.key_values ? g.ok : g.ok + up_to(g.G * g.maps * g.hs, 16);
+      g.og = l.out_gate ? g.ov + up_to(g.G * g.vs, 16) : -1;
+      L.in_cols = g.og >= 0 ? g.og + (g.head_gate ? g.H : g.H * g.vs) : g.ov + g.G * g.vs;
+      L.o_rows = g.H * g.vs;
+      const size_t tokens = (size_t)cf.pagedattn_num_pages * c->P * g.G;
+      if (tokens > (size_t)INT32_MAX) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %zu cached heads in the page pool", i, tokens);
+      TRY(h_alloc(c, &L.pages, tokens * g.dkp * m->esz));
+      TRY(h_alloc(c, &L.vpages, tokens * g.dvp * m->esz));
+      upd(qx_e, (size_t)R * g.H * g.dkp);
+      upd(po, (size_t)IXT_HEADS_SPLIT_BLOCKS * 16 * g.dvp);
+    } else {
+      m->recurrent = true;
+      RetGeom& g = L.rg;
+      g.H = l.heads; g.d = l.dim; g.dv = l.vdim; g.dp = up_to(l.dim, 16); g.dvp = up_to(l.vdim, 16); g.rot = l.rot_dim;
+      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4);
+      g.ok = up_to(g.H * g.hs, 16); g.ov = 2 * g.ok; g.og = g.ov + up_to(g.H * g.vs, 16);
+      g.silu = g.join_norm = l.mixer == IXT_MIX_LIGHTNING; g.kf = g.silu ? 1.0f : (float)(1.0 / sqrt((double)l.dim)); g.oc = oc; g.of = l.mix_scale;
+      L.in_cols = g.og + g.H * g.vs;
+      L.o_rows = g.H * g.vs;
+      TRY(h_allocf(c, &L.state, (size_t)c->G * g.H * g.dp * g.dvp));
+      std::vector<float> pw((size_t)g.H * (SEG_CHUNK + 1));
+      for (int h = 0; h < g.H; ++h)
+        for (int j = 0; j <= SEG_CHUNK; ++j) pw[(size_t)h * (SEG_CHUNK + 1) + j] = (float)pow(l.decay[h], j);
+      TRY(h_allocf(c, &L.pow, pw.size()));
+      HIPCHK(hipMemcpy(L.pow, pw.data(), pw.size() * 4, hipMemcpyHostToDevice));
+      upd(s_q, (size_t)R * g.H * g.dp); upd(s_v, (size_t)R * g.H * g.dvp); upd(ret_u, max_chunks * g.H * g.dp * g.dvp);
+    }
+    return hybrid_rope(c, l, &ropes, &L);
+  };
   for (int i = 0; i < n; ++i) {
     HLayer& L = m->layers[i];
     L.c = cf.layers[i];
     L.src = L.c.weights_of >= 0 ? L.c.weights_of : i;
     const ixt_layer& l = L.c;
+    if (l.shift) {
+      shifts = m->recurrent = true;
+      TRY(h_allocf(c, &L.shift, (size_t)c->G * 2 * m->Ep));
+    }
+    m->passes = std::max(m->passes, l.loop_pass + 1);
     if (l.mixer == IXT_MIX_LATENT_ATTENTION) {
       LatentGeom& g = L.lg;
       g.H = l.heads; g.dn = l.dim; g.dr = l.rot_dim; g.rank = l.kv_rank; g.P = c->P; g.mpg = c->mpg; g.window = l.window; g.scale = l.attn_scale;
@@ -391,41 +554,37 @@ int hybrid_init(ixt_ctx* c) {
       upd(act_k, up_to(g.H * l.vdim, IXT_KALIGN));
       upd(qx_e, (size_t)g.H * Rp * dnp); upd(qr_e, (size_t)R * g.H * g.rotp); upd(olat_e, (size_t)g.H * Rp * kp);
       upd(po, (size_t)(1024 + g.H) * 16 * g.rankp);
-    } else if (l.mixer == IXT_MIX_ATTENTION) {
-      HeadsGeom& g = L.hg;
-      g.H = l.heads; g.G = l.kv_heads; g.d = l.dim; g.dv = l.vdim; g.rot = l.rot_dim; g.P = c->P; g.mpg = c->mpg; g.window = l.window; g.scale = l.attn_scale;
-      g.maps = std::max(l.maps, 1); g.cap = l.softcap;
-      if (!heads_mfma_sizes(l.dim, g.maps, l.vdim, m->f32, &g.dkp, &g.dvp)) { g.dkp = g.maps * up_to(l.dim, 32); g.dvp = up_to(l.vdim, 32); }
-      g.dmp = g.dkp / g.maps;
-      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4); g.ok = up_to(g.H * g.maps * g.hs, 16); g.ov = g.ok + up_to(g.G * g.maps * g.hs, 16);
-      g.og = l.out_gate ? g.ov + up_to(g.G * g.vs, 16) : -1;
-      const size_t tokens = (size_t)cf.pagedattn_num_pages * c->P * g.G;
-      if (tokens > (size_t)INT32_MAX) return set_err(IXT_ERR_UNSUPPORTED, "layer %d: %zu cached heads in the page pool", i, tokens);
-      TRY(h_alloc(c, &L.pages, tokens * g.dkp * m->esz));
-      TRY(h_alloc(c, &L.vpages, tokens * g.dvp * m->esz));
-      TRY(hybrid_rope(c, l, &ropes, &L));
-      dotsz(m->Ep, up_to(g.og >= 0 ? g.og + g.H * g.vs : g.ov + g.G * g.vs, 16));
-      dotsz(up_to(g.H * g.vs, IXT_KALIGN), up_to(m->E, 16));
-      upd(act_k, up_to(g.H * g.vs, IXT_KALIGN));
-      upd(qx_e, (size_t)R * g.H * g.dkp);
-      upd(po, (size_t)IXT_HEADS_SPLIT_BLOCKS * 16 * g.dvp);
-    } else if (l.mixer == IXT_MIX_RETENTION) {
+    } else if (column_mixer(l)) {
+      TRY(columns(L, i, 0, 0));
+      int n_in = L.in_cols, n_o = L.o_rows;
+      if (l.beside) {
+        L.side = std::make_unique<HLayer>();
+        L.side->c = *l.beside; L.side->src = L.src;
+        TRY(columns(*L.side, i, up_to(n_in, 16), n_o));
+        n_in = up_to(n_in, 16) + L.side->in_cols; n_o += L.side->o_rows;
+      }
+      L.in_cols = n_in; L.okp = up_to(n_o, IXT_KALIGN);
+      (L.c.mixer == IXT_MIX_ATTENTION ? L.hg.kend : L.rg.kend) = L.side ? L.o_rows : L.okp;
+      if (L.side) { L.side->okp = L.okp; (L.side->c.mixer == IXT_MIX_ATTENTION ? L.side->hg.kend : L.side->rg.kend) = L.okp; }
+      L.o_rows = n_o;
+      dotsz(m->Ep, up_to(n_in, 16));
+      dotsz(L.okp, up_to(m->E, 16));
+      upd(act_k, L.okp);
+    } else if (l.mixer == IXT_MIX_SCAN) {
       m->recurrent = true;
-      RetGeom& g = L.rg;
-      g.H = l.heads; g.d = l.dim; g.dv = l.vdim; g.dp = up_to(l.dim, 16); g.dvp = up_to(l.vdim, 16); g.rot = l.rot_dim;
-      g.hs = up_to(l.dim, 4); g.vs = up_to(l.vdim, 4);
-      g.ok = up_to(g.H * g.hs, 16); g.ov = 2 * g.ok; g.og = g.ov + up_to(g.H * g.vs, 16);
-      TRY(h_allocf(c, &L.state, (size_t)c->G * g.H * g.dp * g.dvp));
-      TRY(hybrid_rope(c, l, &ropes, &L));
-      std::vector<float> pw((size_t)g.H * (SEG_CHUNK + 1));
-      for (int h = 0; h < g.H; ++h)
-        for (int j = 0; j <= SEG_CHUNK; ++j) pw[(size_t)h * (SEG_CHUNK + 1) + j] = (float)pow(l.decay[h], j);
-      TRY(h_allocf(c, &L.pow, pw.size()));
-      HIPCHK(hipMemcpy(L.pow, pw.data(), pw.size() * 4, hipMemcpyHostToDevice));
-      dotsz(m->Ep, up_to(g.og + g.H * g.vs, 16));
-      dotsz(up_to(g.H * g.vs, IXT_KALIGN), up_to(m->E, 16));
-      upd(act_k, up_to(g.H * g.vs, IXT_KALIGN));
-      upd(s_q, (size_t)R * g.H * g.dp); upd(s_v, (size_t)R * g.H * g.dvp); upd(ret_u, max_chunks * g.H * g.dp * g.dvp);
+      ScanGeom& g = L.sg;
+      g.C = l.inner; g.Cp = up_to(l.inner, 4); g.N = l.state; g.rank = l.dt_rank; g.taps = l.conv;
+      for (g.Np = 16; g.Np < g.N;) g.Np *= 2;
+      g.oz = up_to(g.C, 16); g.ob = up_to(g.rank, 16); g.oc = g.ob + up_to(g.N, 16);
+      L.okp = up_to(g.C, IXT_KALIGN);
+      TRY(h_allocf(c, &L.state, (size_t)c->G * g.C * g.Np));
+      TRY(h_allocf(c, &L.tails, (size_t)c->G * 2 * (g.taps - 1) * g.C + 4));
+      const int Nx = up_to(g.oc + g.N, 16), Nd = up_to(g.C, 16), Kd = up_to(g.rank, IXT_KALIGN);
+      dotsz(m->Ep, up_to(g.oz + g.C, 16));
+      upd(part2, dot_floats(L.okp, Nx)); upd(part3, dot_floats(Kd, Nd));
+      dotsz(L.okp, up_to(m->E, 16));
+      upd(act_k, L.okp); upd(act_k, Kd);
+      upd(scan_x, (size_t)R * g.Cp); upd(scan_u, max_chunks * g.C * g.Np); upd(scan_s, max_chunks * g.Cp);
     } else {
       m->recurrent = true;
       DeltaGeom& g = L.dg;
@@ -466,13 +625,29 @@ int hybrid_init(ixt_ctx* c) {
       if (!m->h32 && (m->norm_places & IXT_NORM_BEFORE)) TRY(h_allocf(c, &m->h32, (size_t)R * m->E));
     }
   }
-  for (int i = 0; i < n; ++i)
+  if (shifts && !m->h32) TRY(h_allocf(c, &m->h32, (size_t)R * m->E));
+  if (m->passes > 0) {
+    TRY(h_mat(c, &m->loop_in, 2 * m->Ep, m->E)); TRY(h_allocf(c, &m->loop_step, (size_t)m->passes * m->Ep)); TRY(h_alloc(c, &m->cat, (size_t)Rp * 2 * m->Ep * m->esz));
+    dotsz(2 * m->Ep, up_to(m->E, 16));
+    LoadMap lm = load_map(m->E, 2 * m->E, m->loop_in.Kp);
+    lm.kg = m->E; lm.kgp = m->Ep;
+    void* d = m->loop_in.w;
+    m->tensors["loop.in"] = HTensor{{m->E, 2 * (int64_t)m->E}, [=](const void* s, int dt, hipStream_t st) { return h_load_mat(m, s, dt, d, lm, st); }, false};
+    const LoadMap ls = load_map(m->passes, m->E, m->Ep);
+    float* step = m->loop_step;
+    m->tensors["loop.step"] = HTensor{{m->passes, m->E}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, step, ls, st); }, false};
+  }
+  for (int i = 0; i < n; ++i) {
     if (m->layers[i].src == i) TRY(hybrid_layer_params(c, i));
+    m->layers[i].c.beside = nullptr;               // (the caller's array may go)
+  }
   m->missing = 0;
   for (auto& kv : m->tensors) m->missing += kv.second.done ? 0 : 1;
   upd(part, (size_t)c->NLmax * m->head.Np * (c->NLmax < 128 ? (m->head.Kp + IXT_CHAIN - 1) / IXT_CHAIN : 1));
   c->part_floats = part; TRY(h_allocf(c, &c->part, part));
   m->part2_floats = part2; TRY(h_allocf(c, &m->part2, part2 + 4));
+  m->part3_floats = part3; TRY(h_allocf(c, &m->part3, part3 + 4));
+  TRY(h_allocf(c, &m->scan_x, scan_x + 4)); TRY(h_allocf(c, &m->scan_u, scan_u + 4)); TRY(h_allocf(c, &m->scan_sum, scan_s + 4));
   TRY(h_allocf(c, &m->x, (size_t)R * std::max(1, m->streams) * m->E));
   TRY(h_allocf(c, &m->ret_u, ret_u + 4)); TRY(h_allocf(c, &m->chunk, max_chunks)); TRY(h_allocf(c, &m->sgate, (size_t)R + 4));
   TRY(h_alloc(c, &m->xb, (size_t)Rp * m->Ep * m->esz));
@@ -494,14 +669,17 @@ int hybrid_init(ixt_ctx* c) {
   TRY(h_allocf(c, &c->amax_val, c->amax_cap)); TRY(h_allocf(c, &c->amax_idx, c->amax_cap));
   // what a copy of a whole page group moves
   std::vector<float*> sb; std::vector<int64_t> sp, pb; std::vector<char*> pp;
-  for (HLayer& L : m->layers) {
-    if (L.c.mixer == IXT_MIX_ATTENTION) {
-      pp.push_back((char*)L.pages); pb.push_back((int64_t)c->P * L.hg.G * L.hg.dkp * (int64_t)m->esz);
-      pp.push_back((char*)L.vpages); pb.push_back((int64_t)c->P * L.hg.G * L.hg.dvp * (int64_t)m->esz);
-    } else if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) { pp.push_back((char*)L.pages); pb.push_back((int64_t)c->P * (L.lg.rankp + L.lg.rotp) * (int64_t)m->esz); }
-    else if (L.c.mixer == IXT_MIX_RETENTION) { sb.push_back(L.state); sp.push_back((int64_t)L.rg.H * L.rg.dp * L.rg.dvp); }
-    else { sb.push_back(L.state); sp.push_back((int64_t)L.dg.H * L.dg.dv * L.dg.dp); sb.push_back(L.tails); sp.push_back((int64_t)2 * (L.dg.taps - 1) * L.dg.C); }
-  }
+  auto state = [&](float* p, int64_t floats) { sb.push_back(p); sp.push_back(floats); };
+  auto pool = [&](void* p, int64_t elems) { pp.push_back((char*)p); pb.push_back(elems * (int64_t)m->esz); };
+  auto group = [&](const HLayer& L) {
+    if (L.c.mixer == IXT_MIX_ATTENTION) { pool(L.pages, (int64_t)c->P * L.hg.G * L.hg.dkp); pool(L.vpages, (int64_t)c->P * L.hg.G * L.hg.dvp); }
+    else if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) pool(L.pages, (int64_t)c->P * (L.lg.rankp + L.lg.rotp));
+    else if (L.c.mixer == IXT_MIX_RETENTION || L.c.mixer == IXT_MIX_LIGHTNING) state(L.state, (int64_t)L.rg.H * L.rg.dp * L.rg.dvp);
+    else if (L.c.mixer == IXT_MIX_SCAN) { state(L.state, (int64_t)L.sg.C * L.sg.Np); state(L.tails, (int64_t)2 * (L.sg.taps - 1) * L.sg.C); }
+    else { state(L.state, (int64_t)L.dg.H * L.dg.dv * L.dg.dp); state(L.tails, (int64_t)2 * (L.dg.taps - 1) * L.dg.C); }
+    if (L.shift) state(L.shift, (int64_t)2 * m->Ep);
+  };
+  for (const HLayer& L : m->layers) { group(L); if (L.side) group(*L.side); }
   m->st_n = (int)sb.size(); m->pg_n = (int)pp.size();
   TRY(h_allocf(c, &m->st_bases, sb.size() + 1)); TRY(h_allocf(c, &m->st_per, sb.size() + 1)); TRY(h_allocf(c, &m->pg_pools, pp.size() + 1)); TRY(h_allocf(c, &m->pg_bytes, pp.size() + 1));
   if (!sb.empty()) { HIPCHK(hipMemcpy(m->st_bases, sb.data(), sb.size() * sizeof(float*), hipMemcpyHostToDevice)); HIPCHK(hipMemcpy(m->st_per, sp.data(), sp.size() * 8, hipMemcpyHostToDevice)); }
@@ -586,16 +764,16 @@ template <> int hdot_grouped<float>(ixt_ctx*, const float* x, const HMat& w, siz
   return IXT_OK;
 }
 // product with a unit without a gate (from IXT_ACT_RELU2 on) behind it -> act(T) of the down product
-template <typename T> static int hact_unit(ixt_ctx* c, const T* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, T* out, hipStream_t st);
-template <> int hact_unit<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, bf16_t* out, hipStream_t st) {
+template <typename T> static int hact_unit(ixt_ctx* c, const T* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, const float* par, T* out, hipStream_t st);
+template <> int hact_unit<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, size_t stride, int rows, int group_rows, const int32_t* rb, int kind, const float* par, bf16_t* out, hipStream_t st) {
   GemmEpi e{};
-  e.act = out; e.glu = kind; e.rb_exp = rb; e.wstride = stride / 8;
+  e.act = out; e.glu = kind; e.act_par = par; e.rb_exp = rb; e.wstride = stride / 8;
   if (rb ? group_rows % 128 == 0 : rows >= c->ring_min_rows) return launch_ring(c, GEPI_ACT, x, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, false, st);
   if (!rb && rows <= c->small_rows && sdot_plan(c, GEPI_ACT, false, w.Kp, w.Np, rows).ok) return launch_sdot(c, GEPI_ACT, false, x, nullptr, (const bf16_t*)w.w, w.Kp, w.Np, rows, e, st);
   const int rowblocks = (rows + 15) / 16, nrb = rb ? 1 : (rowblocks >= 3 ? 4 : rowblocks), zblocks = (rowblocks + nrb - 1) / nrb, ntile = w.Np / 16;
   dim3 grid((((ntile + 3) / 4 + 7) / 8) * 8 * zblocks, 1, 1);
 #define HACT(B_, NT_) hipLaunchKernelGGL((k_dotb<B_, false, NT_, 2>), grid, dim3(256), (size_t)(B_) * 16 * 1024, st, reinterpret_cast<const u32x4*>(x), reinterpret_cast<const u32x4*>(w.w), \
-                                         w.Kp, w.Np, rows, reinterpret_cast<float*>(out), ntile, zblocks, rb, stride / 8, kind, 0.0f)
+                                         w.Kp, w.Np, rows, reinterpret_cast<float*>(out), ntile, zblocks, rb, stride / 8, kind, 0.0f, par)
   if (nrb == 4) { if (zblocks == 1) HACT(4, true); else HACT(4, false); }
   else if (nrb == 2) HACT(2, true);
   else HACT(1, true);
@@ -603,10 +781,10 @@ template <> int hact_unit<bf16_t>(ixt_ctx* c, const bf16_t* x, const HMat& w, si
   LAUNCHCHK();
   return IXT_OK;
 }
-template <> int hact_unit<float>(ixt_ctx* c, const float* x, const HMat& w, size_t stride, int rows, int, const int32_t* rb, int kind, float* out, hipStream_t st) {
+template <> int hact_unit<float>(ixt_ctx* c, const float* x, const HMat& w, size_t stride, int rows, int, const int32_t* rb, int kind, const float* par, float* out, hipStream_t st) {
   Slices t;
   TRY(hdot_grouped<float>(c, x, w, stride, rows, 16, rb, c->part, c->part_floats, st, &t));
-  hipLaunchKernelGGL((k_act_slices<float>), dim3(rows, (w.Np + 255) / 256), dim3(256), 0, st, t, w.Np, kind, out, rb);
+  hipLaunchKernelGGL((k_act_slices<float>), dim3(rows, (w.Np + 255) / 256), dim3(256), 0, st, t, w.Np, kind, par, out, rb);
   LAUNCHCHK();
   return IXT_OK;
 }
@@ -727,49 +905,31 @@ static int hybrid_mixer_latent(ixt_ctx* c, const HLayer& L, const HLayer& W, int
   return IXT_OK;
 }
 
+// one mixer, or two side by side, on columns of one projection
 template <typename T>
-static int hybrid_mixer_heads(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, bool decode, int len_hint, hipStream_t st) {
+static int hybrid_mixer_columns(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool decode, int len_hint, hipStream_t st) {
   Slices t;
   TRY(hdot<T>(c, (const T*)c->hy->xb, W.in, R, c->part, c->part_floats, st, &t));
-  return heads_attention<T>(c, L, W, t, R, decode, len_hint, st);
+  t.bias = W.ibias;
+  auto one = [&](const HLayer& l, const HLayer& w, const Slices& own) -> int {
+    if (l.c.mixer == IXT_MIX_ATTENTION) return heads_attention<T>(c, l, w, own, R, decode, len_hint, st);
+    return retention_mix<T>(c, l, w, own, R, nseg_max, decode, st);
+  };
+  TRY(one(L, W, t));
+  return L.side ? one(*L.side, *W.side, t.from(L.side->c0)) : (int)IXT_OK;
 }
 
-template <int NT, bool FUSED, typename T>
-static int ret_out_launch(const RetArgs& a, int chunks, T* out, int Kp, hipStream_t st) {
-  hipLaunchKernelGGL((k_ret_out<T, NT, FUSED>), dim3(chunks, a.g.H, (a.g.dvp + 16 * NT - 1) / (16 * NT)), dim3(256), 0, st, a, out, Kp);
-  LAUNCHCHK();
-  return IXT_OK;
-}
 template <typename T>
-static int hybrid_mixer_retention(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st) {
+static int hybrid_mixer_scan(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st) {
   HybridModel* m = c->hy;
-  const RetGeom& g = L.rg;
-  Slices t;
-  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &t));
-  const RowsArgs rows{c->row_slot, c->row_pos, c->row_active, c->ps.page_map};
-  const HeadsRope rope{L.rope_cos, L.rope_sin};
-  const RetArgs a{g, t, L.pow, m->seg, m->chunk, m->nseg, m->dq, m->dk, m->dv, m->ret_u, L.state, m->dout, m->eps};
-  T* out = (T*)m->act;
-  if (single) {            // every row is a run of one token
-    const int ns = 256 / (g.dvp / 4);
-    hipLaunchKernelGGL((k_ret_step<T>), dim3(R, g.H), dim3(256), sizeof(float) * (2 * g.dp + g.dvp + ns * g.dvp), st, a, rope, rows, out, W.o.Kp);
-    LAUNCHCHK();
-    return IXT_OK;
-  }
-  const int widest = std::max(g.dp, g.dvp), chunks = R / SEG_CHUNK + nseg_max;
-#define RPREP(LP_) hipLaunchKernelGGL((k_ret_prep<LP_>), dim3(R, (3 * g.H * LP_ + 255) / 256), dim3(256), 0, st, a, rope, rows)
-  if (widest <= 64) RPREP(16); else if (widest <= 128) RPREP(32); else RPREP(64);
-#undef RPREP
-  hipLaunchKernelGGL(k_ret_sums, dim3(chunks, g.H, (g.dp + 63) / 64 * ((g.dvp + 127) / 128)), dim3(256), 0, st, a);
-  hipLaunchKernelGGL(k_ret_carry, dim3(nseg_max, g.H, (g.dp * g.dvp + 1023) / 1024), dim3(256), 0, st, a);
-  LAUNCHCHK();
-  if (g.dvp <= 32) return ret_out_launch<2, true, T>(a, chunks, out, W.o.Kp, st);
-  if (g.dvp <= 64) return ret_out_launch<4, true, T>(a, chunks, out, W.o.Kp, st);
-  if (g.dvp <= 128) return ret_out_launch<8, true, T>(a, chunks, out, W.o.Kp, st);
-  TRY((ret_out_launch<8, false, T>(a, chunks, out, W.o.Kp, st)));
-  hipLaunchKernelGGL((k_ret_gate<T>), dim3(R, (g.H + 3) / 4), dim3(256), 0, st, a, c->row_active, out, W.o.Kp);
-  LAUNCHCHK();
-  return IXT_OK;
+  Slices in, low, dt;
+  TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &in));
+  TRY(scan_conv<T>(c, L, W, in, R, st));
+  TRY(hdot<T>(c, (const T*)m->act, W.low, R, m->part2, m->part2_floats, st, &low));
+  TRY(scan_rank<T>(c, W, low, R, st));
+  TRY(hdot<T>(c, (const T*)m->act, W.dt, R, m->part3, m->part3_floats, st, &dt));
+  dt.bias = W.dtb;
+  return scan_mix<T>(c, L, W, in, low, dt, R, nseg_max, single, st);
 }
 
 template <typename T>
@@ -814,7 +974,7 @@ static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipSt
   const RouteRule rule{l.experts, l.top, l.router, l.groups > 1 ? l.groups : 0, l.groups_keep, l.router_norm, l.router_scale, W.corr, W.bias, l.shared_ff > 0 && l.shared_gate ? m->sgate : nullptr};
   const bool gated = l.glu < IXT_ACT_RELU2;
   if (l.shared_ff > 0) {
-    TRY(gated ? hglu<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, l.glu_limit, (T*)m->hact, st) : hact_unit<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, (T*)m->hact, st));
+    TRY(gated ? hglu<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, l.glu_limit, (T*)m->hact, st) : hact_unit<T>(c, (const T*)m->xb, W.sgu, 0, R, 0, nullptr, l.glu, W.unit_par, (T*)m->hact, st));
     TRY(hdot<T>(c, (const T*)m->hact, W.sdown, R, m->part2, m->part2_floats, st, shared));
   }
   const float* h = (m->norm_places & IXT_NORM_BEFORE) ? m->h32 : m->x;
@@ -835,7 +995,7 @@ static int hybrid_moe(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, hipSt
   else hipLaunchKernelGGL(k_gather32, dim3(pairs, (m->Ep + 255) / 256), dim3(256), 0, st, (const float*)m->xb, m->mpos, l.top, m->Ep, (float*)m->xg);
   LAUNCHCHK();
   TRY(gated ? hglu<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, l.glu_limit, (T*)m->mhact, st)
-            : hact_unit<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, (T*)m->mhact, st));
+            : hact_unit<T>(c, (const T*)m->xg, W.gu, W.gu_stride, rows_g, align, m->mrb, l.glu, W.unit_par, (T*)m->mhact, st));
   return hdot_grouped<T>(c, (const T*)m->mhact, W.down, W.down_stride, rows_g, align, m->mrb, c->part, c->part_floats, st, out);
 }
 
@@ -859,12 +1019,12 @@ static int hybrid_logits(ixt_ctx* c, int R, int lrow0, int nl, const int32_t* lr
 // a sublayer's last product and what follows it: x <- x + post(W v), the next operand pre(x).  Tanh norms ride in the product's epilogue where the whole
 // sum is in one place.
 template <typename T>
-static int hybrid_dot_norm(ixt_ctx* c, const T* v, const HMat& w, const Around& ar, bool routed, int R, hipStream_t st) {
+static int hybrid_dot_norm(ixt_ctx* c, const T* v, const HMat& w, const Around& ar, bool routed, int R, bool single, const float* bias, float fbias, hipStream_t st) {
   HybridModel* m = c->hy;
   [[maybe_unused]] const NormW &post = ar.post, &pre = ar.pre;
   if constexpr (sizeof(T) == 2) {
     const bool small = R <= c->small_rows && sdot_plan(c, GEPI_TANHNORM, false, w.Kp, w.Np, R).ok;
-    if (m->norm_kind == IXT_NORM_TANH && m->streams == 0 && (small || R >= c->ring_min_rows)) {
+    if (m->norm_kind == IXT_NORM_TANH && m->streams == 0 && ar.mu == nullptr && !ar.to_cat && bias == nullptr && (small || R >= c->ring_min_rows)) {
       GemmEpi e{};
       e.act = (bf16_t*)m->xb;
       e.tn = TanhNormEpi{post.w, post.b, post.alpha, pre.w, pre.b, pre.alpha, m->x, routed && pre.w != nullptr ? m->h32 : nullptr, m->E, m->Ep};
@@ -874,7 +1034,9 @@ static int hybrid_dot_norm(ixt_ctx* c, const T* v, const HMat& w, const Around& 
   }
   Slices t;
   TRY(hdot<T>(c, v, w, R, c->part, c->part_floats, st, &t));
-  return hybrid_norm<T>(c, SubOut{t}, ar, routed, R, st);
+  SubOut o{t};
+  o.bias = bias; o.fbias = fbias;
+  return hybrid_norm<T>(c, o, ar, routed, R, single, st);
 }
 
 template <typename T>
@@ -885,30 +1047,43 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
   if (m->recurrent || m->maxH > 0)
     hipLaunchKernelGGL(k_segments, dim3(1), dim3(1024), 0, st, R, c->row_active, c->row_slot, c->row_pos, m->row_seg, m->row_j, m->seg, m->chunk, m->nseg, m->state_len, m->parity, m->claim, c->G,
                      m->recurrent ? 1 : 0, m->err, m->head_rb, m->maxH * (Rp / 16), Rp / 16);
-  const HLayer& head = m->layers[m->layers[0].src];
-  const NormW none{}, first = head.n1;
-  const bool tanh_first = m->norm_kind == IXT_NORM_TANH && m->streams == 0;      // that norm rides with the lookup
+  const NormW none{};
+  auto entry = [&](size_t i) {                                     // what stands in front of the mixer of run i
+    const HLayer& W = m->layers[m->layers[i].src];
+    return Around{none, W.n1, nullptr, W.hc1, W.mu, m->layers[i].shift, false};
+  };
+  auto before = [&](size_t i) {                                    // what a sublayer in front of run i leaves (the head's norm is taken of the wanted rows only)
+    if (i >= m->layers.size()) return Around{none, none, nullptr, nullptr};
+    if (m->layers[i].c.loop_pass >= 0) return Around{none, none, nullptr, nullptr, nullptr, nullptr, true};
+    return entry(i);
+  };
+  const Around first = before(0);
+  const bool tanh_first = m->norm_kind == IXT_NORM_TANH && m->streams == 0 && first.mu == nullptr;      // that norm rides with the lookup
   hipLaunchKernelGGL((k_embed_scaled<T>), dim3(R), dim3(256), 0, st, (const T*)m->embed, tokens, m->emb_scale, m->E, m->Ep, m->V, std::max(1, m->streams),
-                     tanh_first ? first : none, m->x, (T*)m->xb);
+                     tanh_first ? first.pre : none, m->x, (T*)m->xb, (T*)m->cat);
   LAUNCHCHK();
-  if (!tanh_first && (first.w != nullptr || m->streams > 0)) TRY((hybrid_norm<T>(c, SubOut{}, Around{none, first, nullptr, head.hc1}, false, R, st)));
+  if (!tanh_first && (first.pre.w != nullptr || m->streams > 0)) TRY((hybrid_norm<T>(c, SubOut{}, first, false, R, decode, st)));
   for (size_t i = 0; i < m->layers.size(); ++i) {
     const HLayer& L = m->layers[i];
     const HLayer& W = m->layers[L.src];
+    if (L.c.loop_pass >= 0) {                                      // a pass begins: x <- W [x; x0] + its step
+      SubOut o{};
+      TRY(hdot<T>(c, (const T*)m->cat, m->loop_in, R, c->part, c->part_floats, st, &o.t));
+      o.bias = m->loop_step + (size_t)L.c.loop_pass * m->Ep; o.fresh = true;
+      TRY((hybrid_norm<T>(c, o, entry(i), false, R, decode, st)));
+    }
     if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) TRY((hybrid_mixer_latent<T>(c, L, W, R, Rp, decode, len_hint, st)));
-    else if (L.c.mixer == IXT_MIX_ATTENTION) TRY((hybrid_mixer_heads<T>(c, L, W, R, decode, len_hint, st)));
-    else if (L.c.mixer == IXT_MIX_RETENTION) TRY((hybrid_mixer_retention<T>(c, L, W, R, nseg_max, decode, st)));
+    else if (L.c.mixer == IXT_MIX_SCAN) TRY((hybrid_mixer_scan<T>(c, L, W, R, nseg_max, decode, st)));
+    else if (column_mixer(L.c)) TRY((hybrid_mixer_columns<T>(c, L, W, R, nseg_max, decode, len_hint, st)));
     else TRY((hybrid_mixer_delta<T>(c, L, W, R, nseg_max, decode, st)));
-    const HLayer* next = i + 1 < m->layers.size() ? &m->layers[m->layers[i + 1].src] : nullptr;      // (the head's norm is taken of the wanted rows only)
-    const NormW next_n = next ? next->n1 : none;
-    const float* next_hc = next ? next->hc1 : nullptr;
     const bool ffn = L.c.ffn != IXT_FFN_NONE;
-    const Around ar1{W.n1b, ffn ? W.n2 : next_n, W.hc1, ffn ? W.hc2 : next_hc}, ar2{W.n2b, next_n, W.hc2, next_hc};
-    TRY((hybrid_dot_norm<T>(c, (const T*)m->act, W.o, ar1, L.c.ffn == IXT_FFN_MOE, R, st)));
+    Around ar1 = ffn ? Around{none, W.n2, nullptr, W.hc2} : before(i + 1), ar2 = before(i + 1);
+    ar1.post = W.n1b; ar1.hc = W.hc1; ar2.post = W.n2b; ar2.hc = W.hc2;
+    TRY((hybrid_dot_norm<T>(c, (const T*)m->act, W.o, ar1, L.c.ffn == IXT_FFN_MOE, R, decode, W.obias, L.c.mix_scale, st)));
     if (L.c.ffn == IXT_FFN_DENSE) {
       TRY(L.c.glu < IXT_ACT_RELU2 ? hglu<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, L.c.glu_limit, (T*)m->hact, st)
-                                  : hact_unit<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, (T*)m->hact, st));
-      TRY((hybrid_dot_norm<T>(c, (const T*)m->hact, W.down, ar2, false, R, st)));
+                                  : hact_unit<T>(c, (const T*)m->xb, W.gu, 0, R, 0, nullptr, L.c.glu, W.unit_par, (T*)m->hact, st));
+      TRY((hybrid_dot_norm<T>(c, (const T*)m->hact, W.down, ar2, false, R, decode, nullptr, 1.0f, st)));
     } else if (L.c.ffn == IXT_FFN_MOE) {
       Slices t, shared{};
       const float* addw = L.c.shared_gate ? m->sgate : nullptr;
@@ -916,9 +1091,9 @@ static int forward_rows_hybrid_t(ixt_ctx* c, int R, const int32_t* tokens, int l
       if (t.n > 2 && R <= 64) {
         hipLaunchKernelGGL(k_moe_sum, dim3((t.ncols + 255) / 256, R), dim3(64), 0, st, t, m->mpos, m->mw, L.c.top, m->msum);
         LAUNCHCHK();
-        TRY((hybrid_norm<T>(c, SubOut{Slices{m->msum, 1, 0, t.ncols}, shared, addw}, ar2, false, R, st)));
+        TRY((hybrid_norm<T>(c, SubOut{Slices{m->msum, 1, 0, t.ncols}, shared, addw}, ar2, false, R, decode, st)));
       } else {
-        TRY((hybrid_norm<T>(c, SubOut{t, shared, addw, m->mpos, m->mw, L.c.top}, ar2, false, R, st)));
+        TRY((hybrid_norm<T>(c, SubOut{t, shared, addw, m->mpos, m->mw, L.c.top}, ar2, false, R, decode, st)));
       }
     }
     if (m->tap && !c->capturing) {

@@ -65,12 +65,12 @@ int heads_attention(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& 
   if constexpr (sizeof(T) == 2) {
     if (heads_mfma_sizes(g.d, g.maps, g.dv, m->f32, &dkp, &dvp)) {
       const bool tall = !decode && R > 32;
-      const int GQ = g.H / g.G, hchunks = (GQ * g.maps + 15) / 16, blocks = R * g.G * hchunks, span = g.window > 0 ? std::min(g.window, len_hint) : len_hint;
+      const int GQ = g.H / g.G, hchunks = (GQ * g.maps + 15) / 16, blocks = R * g.G * hchunks, most = g.chunk > 0 ? g.chunk : g.window, span = most > 0 ? std::min(most, len_hint) : len_hint;
       int splits = 1;
       if (!tall) splits = std::min(std::min(16, std::max(1, IXT_HEADS_SPLIT_BLOCKS / blocks)), std::max(1, (span + 63) / 64));     // at least a tile each
       if (!decode) TRY((heads_prep<T>(c, L, W, t, rope, rows, R, st)));
       HeadsAttnArgs a{(const bf16_t*)m->qx, g, W.sink, rows, (bf16_t*)L.pages, (bf16_t*)L.vpages, R, 1, (GQ + hchunks - 1) / hchunks, hchunks, __builtin_ctz(c->P),
-                      (bf16_t*)m->act, W.o.Kp, m->po, m->pml, t, W.qn, W.kn, m->eps, rope, mp};
+                      (bf16_t*)m->act, W.okp, m->po, m->pml, t, W.qn, W.kn, m->eps, rope, mp};
       int rc = IXT_ERR_UNSUPPORTED;
 #define X(DK_, DV_) if (dkp == DK_ && dvp == DV_) rc = heads_launch<DK_, DV_, 1>(tall, decode, splits, a, st);
 #define X2(DK_, DV_) if (dkp == DK_ && dvp == DV_) rc = heads_launch<DK_, DV_, 2>(tall, decode, splits, a, st);
@@ -79,7 +79,7 @@ int heads_attention(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& 
 #undef X
       TRY(rc);
       if (splits > 1) {
-        hipLaunchKernelGGL(k_heads_combine, dim3(R, g.H), dim3(64), 0, st, m->po, m->pml, splits, g, mp, t, c->row_active, (bf16_t*)m->act, W.o.Kp);
+        hipLaunchKernelGGL(k_heads_combine, dim3(R, g.H), dim3(64), 0, st, m->po, m->pml, splits, g, mp, t, c->row_active, (bf16_t*)m->act, W.okp);
         LAUNCHCHK();
       }
       return IXT_OK;
@@ -87,7 +87,7 @@ int heads_attention(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& 
   }
   TRY((heads_prep<T>(c, L, W, t, rope, rows, R, st)));
   hipLaunchKernelGGL((k_heads_any<T>), dim3(R, g.H), dim3(256), sizeof(float) * (g.dkp + 256), st, (const T*)m->qx, g, W.sink, rows, (const T*)L.pages, (const T*)L.vpages, mp, t, (T*)m->act,
-                     W.o.Kp);
+                     W.okp);
   LAUNCHCHK();
   return IXT_OK;
 }

@@ -37,12 +37,13 @@ template <typename T> __device__ __forceinline__ T from_f(float v);
 template <> __device__ __forceinline__ bf16_t from_f<bf16_t>(float v) { return f2bf(v); }
 template <> __device__ __forceinline__ float from_f<float>(float v) { return v; }
 
-struct Slices {             // a dot's output
-  const float* p; int n; size_t stride; int ncols;
+struct Slices {             // a dot's output; bias: one number per column joins the sum (nullptr: none)
+  const float* p; int n; size_t stride; int ncols; const float* bias = nullptr;
   __device__ __forceinline__ float at(int r, int c) const {
     const float* q = p + (size_t)r * ncols + c;
     float t = q[0];
     for (int s = 1; s < n; ++s) t += q[(size_t)s * stride];
+    if (bias != nullptr) t += bias[c];
     return t;
   }
   __device__ __forceinline__ void at4(int r, int c, float* o) const {       // c % 4 == 0
@@ -56,8 +57,14 @@ struct Slices {             // a dot's output
       for (int i = 0; i < 4; ++i)
         if (s + i < n) { t.x += u[i].x; t.y += u[i].y; t.z += u[i].z; t.w += u[i].w; }
     }
+    if (bias != nullptr) {
+      const float4 b = *reinterpret_cast<const float4*>(bias + c);
+      t.x += b.x; t.y += b.y; t.z += b.z; t.w += b.w;
+    }
     o[0] = t.x; o[1] = t.y; o[2] = t.z; o[3] = t.w;
   }
+  // the columns from c on (c % 4 == 0)
+  __host__ __device__ __forceinline__ Slices from(int c) const { Slices s = *this; s.p += c; if (bias != nullptr) s.bias += c; return s; }
 };
 
 __device__ __forceinline__ float wave_sum(float v) {
@@ -120,18 +127,21 @@ static __global__ __launch_bounds__(256) void k_dot32(const float* __restrict__ 
 // src [n][k] row-major ([out, in] linear weights, rows `ld` apart) -> rows n of a dot operand of Kp k-columns, at (column n_off + n, k k_off + k).
 // inter: 16-column tile j goes to tile 2 j + n_off (the two matrices of a gated unit side by side).  trans: src is [k][n].  ng / kg > 0: groups of ng
 // columns (kg k) are laid ngp (kgp) apart, zeros between them.  rn > 0: of every rg columns those from r0 on are rn rotated features in halves (i turns
-// with i + rn / 2); they are laid as neighbours, which is the order the kernels turn (the order of a head's features changes no score).
-struct LoadMap { int n, k, ld, Kp, n_off, k_off, inter, trans, ng, ngp, kg, kgp, rg, r0, rn; };
+// with i + rn / 2); they are laid as neighbours, which is the order the kernels turn (the order of a head's features changes no score).  krn > 0: the same for
+// the first krn of every krg inputs (values that are keys come in that order).
+struct LoadMap { int n, k, ld, Kp, n_off, k_off, inter, trans, ng, ngp, kg, kgp, rg, r0, rn, krg, krn; };
+__device__ __forceinline__ int halves_to_pairs(int i, int group, int first, int n) {
+  const int f = i % group - first, h = n / 2;
+  return f >= 0 && f < n ? i + (f < h ? 2 * f : 2 * (f - h) + 1) - f : i;
+}
 template <typename S, typename T>
 __global__ void k_load_nk(const S* __restrict__ src, T* __restrict__ dst, LoadMap m) {
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= (int64_t)m.n * m.k) return;
   int nn = m.trans ? (int)(i % m.n) : (int)(i / m.k), kk = m.trans ? (int)(i / m.n) : (int)(i % m.k);
   const float v = to_f(src[m.trans ? (size_t)kk * m.ld + nn : (size_t)nn * m.ld + kk]);
-  if (m.rn > 0) {
-    const int f = nn % m.rg - m.r0, h = m.rn / 2;
-    if (f >= 0 && f < m.rn) nn += (f < h ? 2 * f : 2 * (f - h) + 1) - f;
-  }
+  if (m.rn > 0) nn = halves_to_pairs(nn, m.rg, m.r0, m.rn);
+  if (m.krn > 0) kk = halves_to_pairs(kk, m.krg, 0, m.krn);
   if (m.ng > 0) nn = nn / m.ng * m.ngp + nn % m.ng;
   if (m.kg > 0) kk = kk / m.kg * m.kgp + kk % m.kg;
   const int col = m.inter ? ((nn >> 4) * 2 + m.n_off) * 16 + (nn & 15) : m.n_off + nn;
@@ -247,7 +257,7 @@ static __global__ __launch_bounds__(256) void k_latent_pages_copy(PageStateDev s
 
 // ---------------------------------------------------------------------------------------------------- embedding, norms
 // A norm's parameters (zeros behind feature E - 1); w null: no norm.  KIND IXT_NORM_RMS: t / sqrt(mean(t^2) + eps) (1 + w); IXT_NORM_TANH: feature by
-// feature tanh(alpha t) w + b; IXT_NORM_LAYER: (t - mean) / sqrt(mean((t - mean)^2) + eps) w + b.
+// feature tanh(alpha t) w + b; IXT_NORM_LAYER: (t - mean) / sqrt(mean((t - mean)^2) + eps) w + b; IXT_NORM_ONE: t / sqrt(mean(t^2) + eps) w[0].
 struct NormW { const float *w, *b, *alpha; };
 __device__ __forceinline__ void load8(const float* __restrict__ p, float* o) {       // p % 16 bytes == 0
   const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
@@ -270,6 +280,12 @@ template <int KIND>
 __device__ __forceinline__ void norm8(const NormW& n, NormStat st, int k0, const float* t, float* o) {
   const float s = st.s;
   float w[8], b[8];
+  if constexpr (KIND == IXT_NORM_ONE) {
+    const float g = s * n.w[0];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = t[j] * g;
+    return;
+  }
   load8(n.w + k0, w);
   if constexpr (KIND == IXT_NORM_TANH) {
     load8(n.b + k0, b);
@@ -308,10 +324,11 @@ __device__ __forceinline__ NormStat row_stat(const NormW& n, const float (*v)[8]
 #define HC_MAX 16
 struct HyperW { const float *in, *out, *mix; };      // in: of the sublayer that follows (nullptr: none does); out, mix: of the one that ends
 
-// x[r] = table[token] * scale (f32; `streams` copies of it) and its copy as the first dot's operand, through a tanh norm if `pre` is one.  grid R, block 256.
+// x[r] = table[token] * scale (f32; `streams` copies of it) and its copy as the first dot's operand, through a tanh norm if `pre` is one.  cat (nullptr: none):
+// act of two Ep columns, the row as it is in both halves.  grid R, block 256.
 template <typename T>
 __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ table, const int32_t* __restrict__ ids, float scale, int E, int Ep, int V, int streams, NormW pre,
-                                                      float* __restrict__ x, T* __restrict__ xb) {
+                                                      float* __restrict__ x, T* __restrict__ xb, T* __restrict__ cat) {
   x += (size_t)blockIdx.x * (streams - 1) * E;             // rows are `streams` E apart
   const int r = blockIdx.x;
   const int id = min(max(ids[r], 0), V - 1);
@@ -330,6 +347,7 @@ __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ tabl
           for (int s = 0; s < streams; ++s) x[(size_t)(r + s) * E + k0 + j] = v[j];
       }
     }
+    if (cat != nullptr) { act_store8(cat, r, k0, 2 * Ep, v); act_store8(cat, r, Ep + k0, 2 * Ep, v); }
     if (pre.w != nullptr) norm8<IXT_NORM_TANH>(pre, NormStat{*pre.alpha, 0.0f}, k0, v, v);
     act_store8(xb, r, k0, Ep, v);
   }
@@ -338,12 +356,17 @@ __global__ __launch_bounds__(256) void k_embed_scaled(const T* __restrict__ tabl
 // A sublayer's output t (slices, or the weighted sum of a row's expert outputs) -> norm behind the sublayer -> residual -> norm in front of the next one:
 //   x <- x + post(t);  xb = pre(x) as the next dot's operand, h32 (if given) the same in f32.
 // t.n == 0: t = 0 and x stays.  pos != nullptr: t = sum_j wts[r][j] * slices row pos[r][j].  add.n > 0: its row, times addw[r] if that is given, joins t.
+// bias, times fbias, joins t; fresh != 0: t takes the place of x instead of joining it.
+// shift.mu != nullptr (every row the only one of its page group): the operand is h + (h' - h) mu of h = pre(x), h' the group's h of one token before.
 // SM > 0: `streams` (<= SM) streams in the place of x ([R][streams][E]): x_t <- sum_s mix[s][t] x_s + out[t] post(t), and pre takes sum_s in[s] x_s.
 // A thread owns 8 consecutive features of every 2048 (NI times).  grid R, block 256.
+// Token shift: mu (zeros behind feature E - 1); the group's last h [group][2][Ep], read at one parity and written at the other (k_segments)
+struct ShiftArgs { const float* mu; float* state; const int32_t *slot, *pos, *active, *parity; };
 struct SubNormArgs {
   Slices t, add; const float* addw;
   const int32_t* pos; const float* wts; int top;
   NormW post, pre; float eps; int E, Ep, streams; HyperW hc;
+  const float* bias; float fbias; int fresh; ShiftArgs shift; int Kp;      // Kp: columns of the operand's rows
 };
 template <typename T, int NI, int KIND, int SM>
 __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restrict__ x, T* __restrict__ xb, float* __restrict__ h32) {
@@ -394,7 +417,11 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[i][q + e] = fmaf(fadd, u[e], v[i][q + e]);
       }
-      if constexpr (SM > 0) continue;
+      if (a.bias != nullptr) {
+        const float4 b = *reinterpret_cast<const float4*>(a.bias + k0 + q);
+        v[i][q] = fmaf(a.fbias, b.x, v[i][q]); v[i][q + 1] = fmaf(a.fbias, b.y, v[i][q + 1]); v[i][q + 2] = fmaf(a.fbias, b.z, v[i][q + 2]); v[i][q + 3] = fmaf(a.fbias, b.w, v[i][q + 3]);
+      }
+      if (SM > 0 || a.fresh) continue;
       if (vec) {
         const float4 xx = *reinterpret_cast<const float4*>(x + (size_t)r * E + k0 + q);
         xv[i][q] = xx.x; xv[i][q + 1] = xx.y; xv[i][q + 2] = xx.z; xv[i][q + 3] = xx.w;
@@ -485,6 +512,14 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
   if (SM > 0 && a.hc.in == nullptr) return;                // the head takes the streams themselves
   NormStat st{};
   if (pre.w != nullptr) st = row_stat<KIND, NI>(pre, xv, E, a.eps, red);
+  const float* before = nullptr;                           // the group's last h, and where this one goes
+  float* keep = nullptr;
+  if (a.shift.mu != nullptr && a.shift.active[r]) {
+    const int grp = a.shift.slot[r], par = a.shift.parity[grp] ^ 1;
+    float* base = a.shift.state + (size_t)grp * 2 * Ep;
+    if (a.shift.pos[r] > 0) before = base + (size_t)par * Ep;
+    keep = base + (size_t)(par ^ 1) * Ep;
+  }
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int k0 = i * 2048 + threadIdx.x * 8;
@@ -495,7 +530,47 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
       for (int j = 0; j < 8; ++j)
         if (k0 + j < E) h32[(size_t)r * E + k0 + j] = xv[i][j];
     }
-    act_store8(xb, r, k0, Ep, xv[i]);
+    if (a.shift.mu != nullptr) {
+      float mu[8], old[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
+      load8(a.shift.mu + k0, mu);
+      if (before != nullptr) load8(before + k0, old);
+      if (keep != nullptr) { store4(keep + k0, xv[i]); store4(keep + k0 + 4, xv[i] + 4); }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) xv[i][j] = fmaf(old[j] - xv[i][j], mu[j], xv[i][j]);
+    }
+    if (xb != nullptr) act_store8(xb, r, k0, a.Kp, xv[i]);
+  }
+}
+
+// Token shift over runs of rows: the operand is h + (h' - h) mu, h' the row before, or (first of its run) what the group has kept; the run's last row leaves
+// its own.  h [R][E], state as in ShiftArgs.  grid R, block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_token_shift(const float* __restrict__ h, const float* __restrict__ mu, float* __restrict__ state, const int32_t* __restrict__ row_seg,
+                                                     const int32_t* __restrict__ row_j, const int32_t* __restrict__ seg, int E, int Ep, T* __restrict__ xb) {
+  const int r = blockIdx.x, s = row_seg[r], j = row_j[r];
+  if (s < 0) return;
+  const int32_t* sg = seg + (size_t)s * 8;
+  const int n = sg[1], start = sg[3], par = sg[4];
+  float* base = state + (size_t)sg[2] * 2 * Ep;
+  const float *hr = h + (size_t)r * E, *before = j > 0 ? hr - E : start > 0 ? base + (size_t)par * Ep : nullptr;
+  float* keep = j == n - 1 ? base + (size_t)(par ^ 1) * Ep : nullptr;
+  for (int k0 = threadIdx.x * 8; k0 < Ep; k0 += 2048) {
+    float v[8], old[8], m[8];
+    load8(mu + k0, m);
+    if ((E & 3) == 0 && k0 + 8 <= E) {
+      load8(hr + k0, v);
+      if (before != nullptr) load8(before + k0, old);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        v[i] = k0 + i < E ? hr[k0 + i] : 0.0f;
+        if (before != nullptr) old[i] = k0 + i < E ? before[k0 + i] : 0.0f;
+      }
+    }
+    if (keep != nullptr) { store4(keep + k0, v); store4(keep + k0 + 4, v + 4); }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = fmaf((before != nullptr ? old[i] : 0.0f) - v[i], m[i], v[i]);
+    act_store8(xb, r, k0, Ep, v);
   }
 }
 
@@ -1471,10 +1546,18 @@ __global__ __launch_bounds__(256) void k_glu_slices(Slices t, int Fp, int kind, 
 
 // the same for a unit without a gate.  grid (rows, ceil(Fp / 256)), block 256
 template <typename T>
-__global__ __launch_bounds__(256) void k_act_slices(Slices t, int Fp, int kind, T* __restrict__ out, const int32_t* __restrict__ rb_exp) {
+__global__ __launch_bounds__(256) void k_act_slices(Slices t, int Fp, int kind, const float* __restrict__ par, T* __restrict__ out, const int32_t* __restrict__ rb_exp) {
   const int f = blockIdx.y * 256 + threadIdx.x, r = blockIdx.x;
   if (f >= Fp || (rb_exp != nullptr && rb_exp[r >> 4] < 0)) return;
-  act_store1(out, r, f, Fp, ixt_act(kind, t.at(r, f)));
+  const float u = t.at(r, f);
+  if (kind == IXT_ACT_XIELU) {                              // (no hardware functions here: the 32-bit mode)
+    const float n = fminf(u, 0.0f), p = fmaxf(u, 0.0f);
+    act_store1(out, r, f, Fp, fmaf(0.5f, u, fmaf(par[0] * p, p, par[1] * (expm1f(n) - n))));
+  } else act_store1(out, r, f, Fp, ixt_act(kind, u, par));
+}
+// the numbers of an xIELU unit from its tensor: par = {softplus(p), 1/2 + softplus(q)}
+static __global__ void k_xielu_numbers(const float* __restrict__ act, float* __restrict__ par) {
+  if (threadIdx.x == 0) { par[0] = f32_softplus(act[0]); par[1] = 0.5f + f32_softplus(act[1]); }
 }
 
 // The choice of experts for a row.  IXT_ROUTE_SOFTMAX: scores s = softmax over all n logits; IXT_ROUTE_SIGMOID: s = sigmoid(z); IXT_ROUTE_CHOSEN: s = z.

@@ -1,0 +1,106 @@
+// ixt_hybrid_state.hip -- launches of the mixers whose state is a recurrence over chunks of rows: retention (ixt_retention_kernels.h), selective scan
+// (ixt_scan_kernels.h)
+#include "ixt_hybrid.h"
+
+template <int NT, bool FUSED, typename T>
+static int ret_out_launch(const RetArgs& a, int chunks, T* out, int Kp, hipStream_t st) {
+  hipLaunchKernelGGL((k_ret_out<T, NT, FUSED>), dim3(chunks, a.g.H, (a.g.dvp + 16 * NT - 1) / (16 * NT)), dim3(256), 0, st, a, out, Kp);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <typename T>
+int retention_mix(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& t, int R, int nseg_max, bool single, hipStream_t st) {
+  HybridModel* m = c->hy;
+  const RetGeom& g = L.rg;
+  const RowsArgs rows{c->row_slot, c->row_pos, c->row_active, c->ps.page_map};
+  const HeadsRope rope{L.rope_cos, L.rope_sin};
+  const RetArgs a{g, t, L.pow, m->seg, m->chunk, m->nseg, m->dq, m->dk, m->dv, m->ret_u, L.state, m->dout, m->eps};
+  T* out = (T*)m->act;
+  const int Kp = W.okp;
+  if (single) {            // every row is a run of one token
+    const int ns = 256 / (g.dvp / 4);
+    hipLaunchKernelGGL((k_ret_step<T>), dim3(R, g.H), dim3(256), sizeof(float) * (2 * g.dp + g.dvp + ns * g.dvp), st, a, rope, rows, out, Kp);
+  } else {
+    const int widest = std::max(g.dp, g.dvp), chunks = R / SEG_CHUNK + nseg_max;
+#define RPREP(LP_) hipLaunchKernelGGL((k_ret_prep<LP_>), dim3(R, (3 * g.H * LP_ + 255) / 256), dim3(256), 0, st, a, rope, rows)
+    if (widest <= 64) RPREP(16); else if (widest <= 128) RPREP(32); else RPREP(64);
+#undef RPREP
+    hipLaunchKernelGGL(k_ret_sums, dim3(chunks, g.H, (g.dp + 63) / 64 * ((g.dvp + 127) / 128)), dim3(256), 0, st, a);
+    hipLaunchKernelGGL(k_ret_carry, dim3(nseg_max, g.H, (g.dp * g.dvp + 1023) / 1024), dim3(256), 0, st, a);
+    LAUNCHCHK();
+    if (g.join_norm) TRY(g.dvp <= 32 ? (ret_out_launch<2, false, T>(a, chunks, out, Kp, st)) : g.dvp <= 64 ? (ret_out_launch<4, false, T>(a, chunks, out, Kp, st)) : (ret_out_launch<8, false, T>(a, chunks, out, Kp, st)));
+    else if (g.dvp <= 32) return ret_out_launch<2, true, T>(a, chunks, out, Kp, st);
+    else if (g.dvp <= 64) return ret_out_launch<4, true, T>(a, chunks, out, Kp, st);
+    else if (g.dvp <= 128) return ret_out_launch<8, true, T>(a, chunks, out, Kp, st);
+    else {
+      TRY((ret_out_launch<8, false, T>(a, chunks, out, Kp, st)));
+      hipLaunchKernelGGL((k_ret_gate<T>), dim3(R, (g.H + 3) / 4), dim3(256), 0, st, a, c->row_active, out, Kp);
+    }
+  }
+  if (g.join_norm) hipLaunchKernelGGL((k_ret_join<T>), dim3(R), dim3(256), 0, st, a, W.onorm, c->row_active, out, Kp);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template int retention_mix<bf16_t>(ixt_ctx*, const HLayer&, const HLayer&, const Slices&, int, int, bool, hipStream_t);
+template int retention_mix<float>(ixt_ctx*, const HLayer&, const HLayer&, const Slices&, int, int, bool, hipStream_t);
+
+template <typename T>
+int scan_conv(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& in, int R, hipStream_t st) {
+  HybridModel* m = c->hy;
+  const ScanConvArgs a{in, L.sg, W.cw, W.cb, m->row_seg, m->row_j, m->seg, L.tails, m->scan_x};
+  hipLaunchKernelGGL((k_scan_conv<T>), dim3(R, (W.low.Kp + 255) / 256), dim3(256), 0, st, a, (T*)m->act, W.low.Kp);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <typename T>
+int scan_rank(ixt_ctx* c, const HLayer& W, const Slices& low, int R, hipStream_t st) {
+  hipLaunchKernelGGL((k_scan_rank<T>), dim3(R), dim3(128), 0, st, low, W.sg.rank, (T*)c->hy->act, W.dt.Kp);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <typename T, int SPL, int LPC>
+static int scan_chunks(ixt_ctx* c, const ScanArgs& a, int R, int nseg_max, int Kp, hipStream_t st) {
+  static bool attr_done = false;
+  if (!attr_done) {
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_scan_sums<SPL, LPC>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)scan_lds<SPL, LPC, false>()));
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_scan_out<T, SPL, LPC>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)scan_lds<SPL, LPC, true>()));
+    attr_done = true;
+  }
+  constexpr int CB = 256 / LPC;
+  const ScanGeom& g = a.g;
+  const int chunks = R / SEG_CHUNK + nseg_max;
+  hipLaunchKernelGGL((k_scan_sums<SPL, LPC>), dim3(chunks, (g.C + CB - 1) / CB), dim3(256), (scan_lds<SPL, LPC, false>()), st, a);
+  hipLaunchKernelGGL(k_scan_carry, dim3(nseg_max, (unsigned)(((size_t)g.C * g.Np + 1023) / 1024)), dim3(256), 0, st, a);
+  hipLaunchKernelGGL((k_scan_out<T, SPL, LPC>), dim3(chunks, (std::max(g.C, Kp) + CB - 1) / CB), dim3(256), (scan_lds<SPL, LPC, true>()), st, a, (T*)c->hy->act, Kp);
+  LAUNCHCHK();
+  return IXT_OK;
+}
+template <typename T>
+int scan_mix(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& in, const Slices& low, const Slices& dt, int R, int nseg_max, bool single, hipStream_t st) {
+  HybridModel* m = c->hy;
+  const ScanGeom& g = L.sg;
+  const ScanArgs a{g, in, low, dt, W.a2, W.D, m->seg, m->chunk, m->nseg, m->scan_x, m->scan_u, m->scan_sum, L.state};
+  const int Kp = W.okp;
+  if (single) {
+#define SSTEP(LPC_) case 4 * LPC_: hipLaunchKernelGGL((k_scan_step<T, LPC_>), dim3(R, (std::max(g.C, Kp) * LPC_ + 255) / 256), dim3(256), 0, st, a, c->row_active, c->row_slot, c->row_pos, \
+                                                      (T*)m->act, Kp); break
+    switch (g.Np) { SSTEP(4); SSTEP(8); SSTEP(16); SSTEP(32); SSTEP(64); default: return set_err(IXT_ERR_UNSUPPORTED, "selective scan: %d states", g.N); }
+#undef SSTEP
+    LAUNCHCHK();
+    return IXT_OK;
+  }
+  switch (g.Np) {
+    case 16: return scan_chunks<T, 4, 4>(c, a, R, nseg_max, Kp, st);
+    case 32: return scan_chunks<T, 8, 4>(c, a, R, nseg_max, Kp, st);
+    case 64: return scan_chunks<T, 16, 4>(c, a, R, nseg_max, Kp, st);
+    case 128: return scan_chunks<T, 16, 8>(c, a, R, nseg_max, Kp, st);
+    case 256: return scan_chunks<T, 16, 16>(c, a, R, nseg_max, Kp, st);
+    default: return set_err(IXT_ERR_UNSUPPORTED, "selective scan: %d states", g.N);
+  }
+}
+#define SCAN_T(T) \
+  template int scan_conv<T>(ixt_ctx*, const HLayer&, const HLayer&, const Slices&, int, hipStream_t); \
+  template int scan_rank<T>(ixt_ctx*, const HLayer&, const Slices&, int, hipStream_t); \
+  template int scan_mix<T>(ixt_ctx*, const HLayer&, const HLayer&, const Slices&, const Slices&, const Slices&, int, int, bool, hipStream_t);
+SCAN_T(bf16_t)
+SCAN_T(float)

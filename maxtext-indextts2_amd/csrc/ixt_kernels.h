@@ -87,11 +87,11 @@ __host__ __device__ __forceinline__ int qk_col(int i, int half) {
 //   EPI = 1 (whole-K blocks only): the columns are interleaved (wi_0, wi_1) tiles (k_tile_w mode 2) and `out` is the bf16 activation buffer of the
 //   next dot (glu: that gated unit of the f32 totals instead, ixt_glu): the odd wave of a pair hands its totals to the even one through LDS, which writes bf16(bf16(a * bf16(sigmoid a)) * b) in the x layout
 //   (linears.py:331-361) -- no f32 slice leaves the chip (routed experts at decode: 132 MB of slices per layer and the kernel that re-read them).
-//   EPI = 2: a unit without a gate instead (glu: its kind, ixt_act); every wave writes its own columns.
+//   EPI = 2: a unit without a gate instead (glu: its kind, act_par: its numbers, ixt_act); every wave writes its own columns.
 template <int NRB, bool SPLIT, bool NT, int EPI = 0>
 __global__ __launch_bounds__(256, 2) void k_dotb(const u32x4* __restrict__ xt, const u32x4* __restrict__ wt, int K, int N, int R,
                                                  float* __restrict__ out, int nwaves, int zblocks, const int32_t* __restrict__ rb_exp = nullptr,
-                                                 size_t wstride = 0, int glu = 0, float glu_limit = 0.0f) {
+                                                 size_t wstride = 0, int glu = 0, float glu_limit = 0.0f, const float* __restrict__ act_par = nullptr) {
   extern __shared__ __attribute__((aligned(16))) u32x4 xs[];   // [NRB][16 steps][64 lanes]
   const int tid = threadIdx.x, nthr = blockDim.x, wpb = nthr >> 6;
   const int wave = tid >> 6, lane = tid & 63;
@@ -211,7 +211,8 @@ __global__ __launch_bounds__(256, 2) void k_dotb(const u32x4* __restrict__ xt, c
       const int row = (rb0 + b) * 16 + r_in;
       if (tile_ok && row < R) {
         uint2 ov;
-        ov.x = pack2(f2bf(ixt_act(glu, tot[b][0])), f2bf(ixt_act(glu, tot[b][1]))); ov.y = pack2(f2bf(ixt_act(glu, tot[b][2])), f2bf(ixt_act(glu, tot[b][3])));
+        ov.x = pack2(f2bf(ixt_act(glu, tot[b][0], act_par)), f2bf(ixt_act(glu, tot[b][1], act_par)));
+        ov.y = pack2(f2bf(ixt_act(glu, tot[b][2], act_par)), f2bf(ixt_act(glu, tot[b][3], act_par)));
         *reinterpret_cast<uint2*>(act + xidx(row, tile * 16 + cq * 4, N)) = ov;
       }
     }

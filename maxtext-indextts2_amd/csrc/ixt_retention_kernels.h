@@ -2,6 +2,8 @@
 //   S_t = g S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t,
 // q and k rotated, k over sqrt(d); the head's output is o / rms(o) silu(gate).  Everything is f32, products included (v_mfma_f32_16x16x4_f32); the state
 // [group][H][dp][dvp] lives as long as its page group.
+// Lightning attention (IXT_MIX_LIGHTNING): the same recurrence on silu(q), silu(k), silu(v) without a rotation and a factor, and one norm over all heads
+// (join_norm): the outputs stay in memory until k_ret_join.
 //
 // Over a run of rows the recurrence goes by chunks of SEG_CHUNK rows (k_segments lists them).  Row i of a chunk (from 0), state S in front of it:
 //   o_i = g^(i + 1) S^T q_i + sum_(j <= i) g^(i - j) (k_j . q_i) v_j,      S <- g^n S + sum_j g^(n - 1 - j) k_j v_j^T
@@ -10,7 +12,8 @@
 //   k_ret_sums   chunk by chunk: U = sum_j g^(n - 1 - j) k_j v_j^T
 //   k_ret_carry  run by run: the state in front of every chunk, in the place of its U; the group's new state
 //   k_ret_out    chunk by chunk: the outputs (with up to 128 value dims also norm and gate; beyond: k_ret_gate)
-//   k_ret_step   one token per row (decode): all of it in one launch
+//   k_ret_step   one token per row (decode): all of it in one launch (join_norm: up to the outputs)
+//   k_ret_join   norm over all heads, weight, sigmoid gate
 //
 // Matrix products: lane (i = lane & 15, q = lane >> 4) holds element i of four terms 4 q + e of a 16-term step, e = 0 .. 3 being four instructions; the
 // order of the terms is the same for both operands.  D: lane holds rows 4 q + e of column i.
@@ -20,7 +23,15 @@
 struct RetGeom {
   int H, d, dv, dp, dvp, rot;               // heads, key / value dims and both padded to 16, rotated dims
   int hs, vs, ok, ov, og;                   // projection columns: a query / key head takes hs, a value head (and its gate) vs
+  int silu, join_norm;                      // silu on q, k, v; all heads normed together
+  float kf;                                 // factor on the keys
+  int oc, kend;                             // act of the output projection: the heads' first column, and where the zeros behind them end
+  float of;                                 // factor on the outputs
 };
+__device__ __forceinline__ void ret_act4(const RetGeom& g, float f, const float* v, float* o) {
+#pragma unroll
+  for (int j = 0; j < 4; ++j) o[j] = (g.silu ? v[j] * f32_sigmoid(v[j]) : v[j]) * f;
+}
 // pow [H][SEG_CHUNK + 1]: powers of a head's decay
 struct RetArgs {
   RetGeom g; Slices t;
@@ -40,16 +51,17 @@ __global__ __launch_bounds__(256) void k_ret_prep(RetArgs a, HeadsRope rope, Row
   const int h = j % g.H, pos = rows.pos[r];
   if (j < 2 * g.H) {
     const bool key = j >= g.H;
-    const float f = key ? 1.0f / sqrtf((float)g.d) : 1.0f;
+    const float f = key ? g.kf : 1.0f;
     float* o = (key ? a.k : a.q) + ((size_t)r * g.H + h) * g.dp;
     head_norm_rotate<LP>(a.t, r, (key ? g.ok : 0) + h * g.hs, g, nullptr, 0.0f, rope, pos, g.dp, sl,
-                         [&](int c, const float* v) { *reinterpret_cast<float4*>(o + c) = make_float4(v[0] * f, v[1] * f, v[2] * f, v[3] * f); });
+                         [&](int c, const float* v) { float u[4]; ret_act4(g, f, v, u); *reinterpret_cast<float4*>(o + c) = make_float4(u[0], u[1], u[2], u[3]); });
     return;
   }
   float* o = a.v + ((size_t)r * g.H + h) * g.dvp;
   for (int c = sl * 4; c < g.dvp; c += 4 * LP) {
     float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
     if (c < g.vs) a.t.at4(r, g.ov + h * g.vs + c, v);
+    ret_act4(g, 1.0f, v, v);
     *reinterpret_cast<float4*>(o + c) = make_float4(v[0], v[1], v[2], v[3]);
   }
 }
@@ -142,8 +154,9 @@ static __global__ __launch_bounds__(256) void k_ret_carry(RetArgs a) {
   *sp = S;
 }
 
-// four columns of a head's output, normed by rs, times silu of their gates
+// four columns of a head's output, normed by rs, times silu of their gates and the layer's factor
 __device__ __forceinline__ void ret_gate4(const Slices& t, int r, const RetGeom& g, int h, int c, float rs, float* v) {
+  rs *= g.of;
   float z[4];
   t.at4(r, g.og + h * g.vs + c, z);
 #pragma unroll
@@ -255,11 +268,11 @@ __global__ __launch_bounds__(256, 2) void k_ret_out(RetArgs a, T* __restrict__ o
       if (cc >= g.vs) continue;
       float v[4] = {o[t][0], o[t][1], o[t][2], o[t][3]};
       ret_gate4(a.t, row, g, h, cc, rs, v);
-      act_store4(out, row, h * g.vs + cc, Kp, v);
+      act_store4(out, row, g.oc + h * g.vs + cc, Kp, v);
     }
     const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
     if (h == g.H - 1)
-      for (int k = g.H * g.vs + q4 * 4; k < Kp; k += 16) act_store4(out, row, k, Kp, z);
+      for (int k = g.oc + g.H * g.vs + q4 * 4; k < g.kend; k += 16) act_store4(out, row, k, Kp, z);
   } else {
     if (!ok) return;
 #pragma unroll
@@ -281,11 +294,55 @@ __global__ __launch_bounds__(256) void k_ret_gate(RetArgs a, const int32_t* __re
     const float4 u = *reinterpret_cast<const float4*>(oh + c);
     float v[4] = {u.x, u.y, u.z, u.w};
     ret_gate4(a.t, r, g, h, c, rs, v);
-    act_store4(out, r, h * g.vs + c, Kp, v);
+    act_store4(out, r, g.oc + h * g.vs + c, Kp, v);
   }
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   if (h == g.H - 1)
-    for (int k = g.H * g.vs + lane * 4; k < Kp; k += 256) act_store4(out, r, k, Kp, z);
+    for (int k = g.oc + g.H * g.vs + lane * 4; k < g.kend; k += 256) act_store4(out, r, k, Kp, z);
+}
+// all heads of a row: o / rms(o) w sigmoid(gate); w [H][vs], zeros behind a head's dv.  grid R, block 256.
+template <typename T>
+__global__ __launch_bounds__(256) void k_ret_join(RetArgs a, const float* __restrict__ w, const int32_t* __restrict__ row_active, T* __restrict__ out, int Kp) {
+  __shared__ float red[4];
+  const RetGeom& g = a.g;
+  const int r = blockIdx.x, tid = threadIdx.x, n = g.H * g.vs;
+  if (!row_active[r]) return;
+  const float* o = a.o + (size_t)r * g.H * g.dvp;
+  constexpr int B = 4;                                       // columns of a thread that stay in registers, in fours
+  float4 v[B], z[B];
+  float ss = 0.0f;
+#pragma unroll
+  for (int i = 0; i < B; ++i) {
+    const int c = (i * 256 + tid) * 4;
+    v[i] = z[i] = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    if (c < n) {
+      v[i] = *reinterpret_cast<const float4*>(o + c / g.vs * g.dvp + c % g.vs);      // (columns from dv on are zero)
+      a.t.at4(r, g.og + c, &z[i].x);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < B; ++i) ss = fmaf(v[i].x, v[i].x, fmaf(v[i].y, v[i].y, fmaf(v[i].z, v[i].z, fmaf(v[i].w, v[i].w, ss))));
+  for (int c = (B * 256 + tid) * 4; c < n; c += 1024) {
+    const float4 u = *reinterpret_cast<const float4*>(o + c / g.vs * g.dvp + c % g.vs);
+    ss = fmaf(u.x, u.x, fmaf(u.y, u.y, fmaf(u.z, u.z, fmaf(u.w, u.w, ss))));
+  }
+  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)(g.H * g.dv) + a.eps) * g.of;
+  auto put = [&](int c, const float4& u, const float4& y) {
+    const float4 ww = *reinterpret_cast<const float4*>(w + c);
+    const float q[4] = {u.x * rs * ww.x * f32_sigmoid(y.x), u.y * rs * ww.y * f32_sigmoid(y.y), u.z * rs * ww.z * f32_sigmoid(y.z), u.w * rs * ww.w * f32_sigmoid(y.w)};
+    act_store4(out, r, g.oc + c, Kp, q);
+  };
+#pragma unroll
+  for (int i = 0; i < B; ++i)
+    if ((i * 256 + tid) * 4 < n) put((i * 256 + tid) * 4, v[i], z[i]);
+  for (int c = (B * 256 + tid) * 4; c < n; c += 1024) {
+    const float4 u = *reinterpret_cast<const float4*>(o + c / g.vs * g.dvp + c % g.vs);
+    float4 y;
+    a.t.at4(r, g.og + c, &y.x);
+    put(c, u, y);
+  }
+  const float zero[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int k = g.oc + n + tid * 4; k < g.kend; k += 1024) act_store4(out, r, k, Kp, zero);
 }
 
 // Decode: block = (row, head).  A thread owns four value columns and every `ns`-th key row; the first of them are requested before anything else.
@@ -311,14 +368,15 @@ __global__ __launch_bounds__(256) void k_ret_step(RetArgs a, HeadsRope rope, Row
     if (mine && pos > 0 && d < g.d) S[i] = *reinterpret_cast<const float4*>(sp + (size_t)d * g.dvp);
   }
   if (wave < 2) {
-    const float f = wave == 1 ? 1.0f / sqrtf((float)g.d) : 1.0f;
+    const float f = wave == 1 ? g.kf : 1.0f;
     float* o = wave == 1 ? ks : qs;
     head_norm_rotate<64>(a.t, r, (wave == 1 ? g.ok : 0) + h * g.hs, g, nullptr, 0.0f, rope, pos, g.dp, lane,
-                         [&](int c, const float* v) { *reinterpret_cast<float4*>(o + c) = make_float4(v[0] * f, v[1] * f, v[2] * f, v[3] * f); });
+                         [&](int c, const float* v) { float u[4]; ret_act4(g, f, v, u); *reinterpret_cast<float4*>(o + c) = make_float4(u[0], u[1], u[2], u[3]); });
   } else if (wave == 2) {
     for (int c = lane * 4; c < g.dvp; c += 256) {
       float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
       if (c < g.vs) a.t.at4(r, g.ov + h * g.vs + c, v);
+      ret_act4(g, 1.0f, v, v);
       *reinterpret_cast<float4*>(vs + c) = make_float4(v[0], v[1], v[2], v[3]);
     }
   }
@@ -354,14 +412,18 @@ __global__ __launch_bounds__(256) void k_ret_step(RetArgs a, HeadsRope rope, Row
       const float4 p = *reinterpret_cast<const float4*>(os + s * g.dvp + tid * 4);
       o.x += p.x; o.y += p.y; o.z += p.z; o.w += p.w;
     }
+  if (g.join_norm) {
+    if (tid < ncg) *reinterpret_cast<float4*>(a.o + ((size_t)r * g.H + h) * g.dvp + tid * 4) = o;
+    return;
+  }
   const float ss = fmaf(o.x, o.x, fmaf(o.y, o.y, fmaf(o.z, o.z, o.w * o.w)));      // (columns from dv on are zero)
   const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)g.dv + a.eps);
   if (tid * 4 < g.vs) {
     float v[4] = {o.x, o.y, o.z, o.w};
     ret_gate4(a.t, r, g, h, tid * 4, rs, v);
-    act_store4(out, r, h * g.vs + tid * 4, Kp, v);
+    act_store4(out, r, g.oc + h * g.vs + tid * 4, Kp, v);
   }
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   if (h == g.H - 1)
-    for (int k = g.H * g.vs + tid * 4; k < Kp; k += 1024) act_store4(out, r, k, Kp, z);
+    for (int k = g.oc + g.H * g.vs + tid * 4; k < g.kend; k += 1024) act_store4(out, r, k, Kp, z);
 }

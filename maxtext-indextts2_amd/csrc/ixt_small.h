@@ -186,7 +186,8 @@ __global__ __launch_bounds__(1024) void k_sdot(SdotArgs a) {
   } else if constexpr (EPI == GEPI_ACT) {
     if (row_ok) {
       uint2 ov;
-      ov.x = pack2(f2bf(ixt_act(a.e.glu, tot[0])), f2bf(ixt_act(a.e.glu, tot[1]))); ov.y = pack2(f2bf(ixt_act(a.e.glu, tot[2])), f2bf(ixt_act(a.e.glu, tot[3])));
+      ov.x = pack2(f2bf(ixt_act(a.e.glu, tot[0], a.e.act_par)), f2bf(ixt_act(a.e.glu, tot[1], a.e.act_par)));
+      ov.y = pack2(f2bf(ixt_act(a.e.glu, tot[2], a.e.act_par)), f2bf(ixt_act(a.e.glu, tot[3], a.e.act_par)));
       *reinterpret_cast<uint2*>(a.e.act + xidx(row, tile * 16 + cq * 4, N)) = ov;
     }
   } else if constexpr (EPI == GEPI_RESID) {

@@ -105,9 +105,16 @@ class MaxEngine(engine_api.Engine):
     if config.decoder_block == "hybrid":               # the layers are listed one by one (architectures.py)
       c.decoder_block = _lib.BLOCK_HYBRID
       fields = [f.name for f in dataclasses.fields(_architectures.HybridLayer)]
-      per_head = [(ctypes.c_double * max(1, len(l.decay)))(*l.decay) for l in config.hybrid_layers]      # (alive until ixt_create has copied them)
-      self._hybrid_layers = (_lib.IxtLayer * len(config.hybrid_layers))(
-          *[_lib.IxtLayer(**dict({n: getattr(l, n) for n in fields}, decay=d)) for l, d in zip(config.hybrid_layers, per_head)])
+      alive = []                                         # what the entries point at, until ixt_create has copied it
+
+      def entry(l):
+        alive.append((ctypes.c_double * max(1, len(l.decay)))(*l.decay))
+        decay = alive[-1]
+        if l.beside is not None:
+          alive.append(entry(l.beside))
+        return _lib.IxtLayer(**dict({n: getattr(l, n) for n in fields}, decay=decay, beside=None if l.beside is None else ctypes.addressof(alive[-1])))
+
+      self._hybrid_layers = (_lib.IxtLayer * len(config.hybrid_layers))(*[entry(l) for l in config.hybrid_layers])
       c.layers, c.num_decoder_layers = self._hybrid_layers, len(config.hybrid_layers)
       c.embedding_scale, c.float32 = float(config.embedding_scale), 1 if config.dtype == "float32" else 0
       c.norm_kind, c.norm_places = int(config.hybrid_norm_kind), int(config.hybrid_norm_places)
@@ -147,7 +154,7 @@ class MaxEngine(engine_api.Engine):
     self._result = torch.zeros((B, 3), dtype=torch.int32, device=self.device)
     self._first = torch.zeros((1,), dtype=torch.int32, device=self.device)
     self._page_failures = 0
-    self._recurrent = any(l.mixer in _architectures.RECURRENT_MIXERS for l in config.hybrid_layers) if config.decoder_block == "hybrid" else False
+    self._recurrent = any(_architectures.carries_state(l) for l in config.hybrid_layers) if config.decoder_block == "hybrid" else False
     self._status_host = torch.zeros((4,), dtype=torch.int32).pin_memory()   # deferred reservation check of the packed prefill
     self._status_event = None
     self._status_what = ""

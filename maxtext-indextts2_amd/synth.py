@@ -196,7 +196,9 @@ def synth_weights_hybrid(cfg, seed: int = 0) -> Dict[str, np.ndarray]:
       z = z * np.float32(1.0 / cfg.embedding_scale)
     elif leaf == "A_log":
       z = np.float32(0.5) * z
-    elif leaf == "dt_bias":
+    elif leaf in ("D", "shift", "act", "step"):                   # skips around one, shifts around a half, unit numbers, what a pass adds
+      z = np.float32({"D": 1.0, "shift": 0.5}.get(leaf, 0.0)) + np.float32(0.2) * z
+    elif leaf == "dt_bias" or name.endswith("dt.b"):
       z = z - np.float32(1.0)
     elif leaf == "conv":
       z = z * np.float32(1.0 / math.sqrt(shape[1]))
@@ -297,7 +299,7 @@ def device_tree_spec(cfg):
   """[(tree path, shape, std or None for a norm scale)] of the configured block (llama2, gemma2, mixtral, hybrid)."""
   if getattr(cfg, "decoder_block", "llama2") == "hybrid":
     from . import architectures  # pylint: disable=import-outside-toplevel
-    std = lambda name, shape: (1 / cfg.embedding_scale if name == "embed" else None if name.endswith("alpha") else 0.1 if "norm" in name or name.rsplit(".", 1)[-1] in ("lq1", "lk1", "lq2", "lk2") else 0.5 if len(shape) == 1 or ".hc" in name else 1 / math.sqrt(shape[-1]))
+    std = lambda name, shape: (1 / cfg.embedding_scale if name == "embed" else None if name.endswith("alpha") or shape == () else 0.1 if "norm" in name or name.rsplit(".", 1)[-1] in ("lq1", "lk1", "lq2", "lk2") else 0.5 if len(shape) == 1 or ".hc" in name else 1 / math.sqrt(shape[-1]))
     return [(name, shape, std(name, shape)) for name, shape in architectures.parameter_shapes(cfg).items()]
   E, Q, KV, D, F, V = cfg.emb_dim, cfg.num_query_heads, cfg.num_kv_heads, cfg.head_dim, cfg.mlp_dim, cfg.vocab_size
   block = getattr(cfg, "decoder_block", "llama2")
