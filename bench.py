@@ -70,7 +70,7 @@ def parse(argv=None):
   ap.add_argument("--sync-every", type=int, default=0, help="synchronise the stream every N engine calls (profiling runs: bounds the launch backlog)")
   ap.add_argument("--backend", default="nccl", help="torch.distributed backend (nccl = RCCL; gloo for the CPU rehearsal)")
   ap.add_argument("--opt", action="append", default=[], help="library option name=value (ixt_set_option), e.g. kv_head_major=1; experiments")
-  ap.add_argument("--hybrid", default="", help="instead of the headline workload: rates of hybrid decoders (Vilepel, Vazilorn, Suzulix) beside the closest existing model of equal size; "
+  ap.add_argument("--hybrid", default="", help="instead of the headline workload: rates of hybrid decoders (Vilepel, Vazilorn, Suzulix, Lulenex) beside the closest existing model of equal size; "
                   "comma-separated sizes of hybrid_bench.SIZES, or all")
   ap.add_argument("--stub-engine", action="store_true", help="CPU rehearsal of the multi-process plumbing (tests/test_dp_cpu.py): no GPU, no model")
   return ap.parse_args(argv)

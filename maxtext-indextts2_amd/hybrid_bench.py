@@ -1,6 +1,6 @@
 """`bench.py --hybrid SIZES`: prefill and decode rates of hybrid decoders (Vilepel: half latent attention, half gated delta rule; Vazilorn: windowed
-attention with sinks and tanh norms; Suzulix: differential attention, retention and latent attention among four streams) at layer sizes of real models, beside the closest model of the framework at the same width, head count,
-feed-forward and number of layers (the llama2 block, or Mixtral for the routed sizes).  Random weights drawn on the device, one GPU, both models in
+attention with sinks and tanh norms; Suzulix: differential attention, retention and latent attention among four streams; Lulenex: chunked attention beside lightning attention, and selective scans) at layer sizes of real models, beside the closest model of the framework at the same width, head count,
+feed-forward and number of layers (the llama2 block, or Mixtral for the routed sizes; a unit without a gate gets half as many features more).  Random weights drawn on the device, one GPU, both models in
 turn in one process.
 
 Per model: `prefill_packed` = 8 prompts of 256 tokens in one pass (2048 rows), `prefill_long` = one 4096-token prompt in 1024-row chunks,
@@ -67,6 +67,17 @@ def _square_moe(ff, experts, top, shared):
   return {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": shared}, "router": {"experts": experts, "top": top}}
 
 
+def _lulenex(width, heads, ff, chunk, layers):
+  """Attention beside lightning attention and selective scans in turn (the sizes of Mamba's own: inner 2 width, 16 states, rank width / 16)."""
+  dim = 128
+  both = {"type": "parallel", "mixer": {"left_scale": 1.0, "right_scale": 1.0,
+                                        "left": {"heads": heads, "kv_heads": heads // 4, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": chunk}, "rot": {"base": 500000.0, "dims": dim // 2}},
+                                        "right": {"heads": heads, "dim": dim, "vdim": dim, "decay": [1.0 - 2.0 ** -(3 + 6.0 * i / heads) for i in range(heads)]}}}
+  scan = {"type": "mamba1", "mixer": {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4}}
+  return {"architecture": "Lulenex", "norm": {"eps": 1e-5}, "vocab": 32000, "width": width, "loop": None,
+          "layers": [dict((both, scan)[i % 2], mlp={"kind": "dense", "ff": ff}) for i in range(layers)]}
+
+
 # name -> (config.json, keys of the closest model)
 SIZES = {
     "w1024": (_model(1024, 4, _latent(8, 256, 512, dim=64), _delta(8, 8), _dense(3584)),
@@ -92,6 +103,9 @@ SIZES = {
     "suzulix-w4096": (_suzulix(4096, ("attention", "retention", "latent_attention"), 32, _square_moe(14336, 8, 2, 2048)),
                       dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=3, num_experts=8, num_experts_per_tok=2,
                            decoder_block="mixtral")),
+    "lulenex-w1024": (_lulenex(1024, 8, 5376, 512, 8), dict(base_emb_dim=1024, base_num_query_heads=8, base_num_kv_heads=8, base_mlp_dim=3584, base_num_decoder_layers=8)),
+    "lulenex-w2048": (_lulenex(2048, 16, 10752, 1024, 8), dict(base_emb_dim=2048, base_num_query_heads=16, base_num_kv_heads=16, base_mlp_dim=7168, base_num_decoder_layers=8)),
+    "lulenex-w4096": (_lulenex(4096, 32, 21504, 1024, 2), dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=2)),
 }
 
 
