@@ -421,16 +421,15 @@ __global__ __launch_bounds__(256, DK + DV <= 320 ? 2 : 1) void k_heads_prompt(He
 // its way; the block with the last tile also takes the row's key and value, keeps them for later passes in their pages and puts them into its tile.
 // MAPS 2: neighbouring pairs are the two maps of a head; a pair's query is zero on the other map's part of the keys.
 template <int DK, int DV, bool FUSED, int MAPS>
-__global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
+__device__ __forceinline__ void heads_decode(const HeadsAttnArgs& a, const int row, const int hblock, const int split, const int nsplit, bf16_t* tile) {
   static_assert(DK % (32 * MAPS) == 0, "whole steps per map");
   constexpr int DM = DK / MAPS, NKM = DM / 32, NKS = DK / 32, NGV = DV / 64, NH = DV % 64 != 0 ? 1 : 0, OT = NGV + NH;     // column tiles per wave: one of every full group, waves 0 and 1 one of the half group
-  extern __shared__ __attribute__((aligned(16))) bf16_t tile[];
   __shared__ __attribute__((aligned(16))) bf16_t ps[16][72];
   __shared__ float s_m[4][16], s_l[4][16];
   __shared__ __attribute__((aligned(16))) bf16_t s_q[FUSED ? 16 : 1][DM + 8], s_k[FUSED ? DK : 8], s_v[FUSED ? DV : 8];
   const HeadsGeom& g = a.g;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r_in = lane & 15, cq = lane >> 4;
-  const int row = blockIdx.x, kh = blockIdx.y % g.G, hc = blockIdx.y / g.G, GQ = g.H / g.G, nsplit = gridDim.z;
+  const int kh = hblock % g.G, hc = hblock / g.G, GQ = g.H / g.G;
   const int h0 = kh * GQ + hc * a.HB, hb = min(a.HB, GQ - hc * a.HB), nu = hb * MAPS;
   const int active = a.rows.active[row], pos = a.rows.pos[row], slot = a.rows.slot[row];     // (requested together)
   if (!active) return;
@@ -438,14 +437,14 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
   const int u_in = pair_ok ? r_in : 0, map = u_in % MAPS, head = h0 + u_in / MAPS;
   const int32_t* prow = a.rows.page_map + (size_t)slot * g.mpg;
   const int k_lo = first_key(g, pos), ntile = (pos - k_lo) / 64 + 1;
-  int t = blockIdx.z;
+  int t = split;
   if (t < ntile) {
     const int off = heads_row(prow, min(k_lo + t * 64 + lane, pos), a.pshift, g.G, kh);
     tile_dma<DK>(a.kpages, off, tile, wave, lane);
     tile_dma<DV>(a.vpages, off, tile + 64 * DK, wave, lane);
   }
   bf16x8 qf[NKS];
-  [[maybe_unused]] const bool last = (ntile - 1) % nsplit == (int)blockIdx.z;       // the row's own key is in one of this block's tiles
+  [[maybe_unused]] const bool last = (ntile - 1) % nsplit == split;       // the row's own key is in one of this block's tiles
   if constexpr (FUSED) {
     const size_t at = ((size_t)prow[pos >> a.pshift] * g.G + kh) * g.P + (pos & (g.P - 1));
     for (int i = wave; i < nu + (last ? MAPS + 1 : 0); i += 4) {
@@ -475,7 +474,7 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
   f32x4 o[OT];
 #pragma unroll
   for (int i = 0; i < OT; ++i) o[i] = f32x4(0.0f);
-  const bool sink = a.sink != nullptr && blockIdx.z == 0;          // counted once
+  const bool sink = a.sink != nullptr && split == 0;          // counted once
   float m = sink ? a.sink[head] * 1.44269504088896340736f : -INFINITY, l = sink && wave == 0 && cq == 0 ? 1.0f : 0.0f;      // l: this lane's keys only
   const float sc = g.scale * 1.44269504088896340736f, c2 = g.cap > 0.0f ? 2.88539008177792681472f * g.scale / g.cap : 0.0f, k2 = g.cap * 1.44269504088896340736f;
   const TileLane L = tile_lane(r_in, cq);
@@ -572,7 +571,7 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     if (map == 1) return;
   }
   if (!pair_ok) return;
-  const size_t pi = (((size_t)row * g.H + head) * MAPS + map) * nsplit + blockIdx.z;
+  const size_t pi = (((size_t)row * g.H + head) * MAPS + map) * nsplit + split;
 #pragma unroll
   for (int i = 0; i < OT; ++i) {
     if (i == NGV && wave > 1) continue;                   // the half group has two column tiles
@@ -590,11 +589,16 @@ __global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
     for (int c = g.oc + g.H * g.vs + cq * 4; c < g.kend; c += 16) act_store4(a.out, row, c, a.Kp, z);
   }
 }
-// the key splits of a row's heads (and their maps) put together.  grid (R, H), block 64; nsplit <= 16, vs <= 256.
-static __global__ __launch_bounds__(64) void k_heads_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, HeadsGeom g, MapsArgs mp, Slices t,
-                                                      const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
+template <int DK, int DV, bool FUSED, int MAPS>
+__global__ __launch_bounds__(256, 2) void k_heads_decode(HeadsAttnArgs a) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t tile[];
+  heads_decode<DK, DV, FUSED, MAPS>(a, blockIdx.x, blockIdx.y, blockIdx.z, gridDim.z, tile);
+}
+// the key splits of one head of a row (and its maps) put together, by the first 64 threads or more of a block; nsplit <= 16, vs <= 256.
+__device__ __forceinline__ void heads_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, const HeadsGeom& g, const MapsArgs& mp, const Slices& t,
+                                              const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp, int r, int h) {
   __shared__ float fac[2][16];
-  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, c = tid * 4, H = g.H, vs = g.vs, dvp = g.dvp;
+  const int tid = threadIdx.x, c = tid * 4, H = g.H, vs = g.vs, dvp = g.dvp;
   if (!row_active[r]) return;
   const size_t p0 = ((size_t)r * H + h) * g.maps * nsplit;
   for (int m = 0; m < g.maps; ++m) split_factors(part_ml + (p0 + m * nsplit) * 2, nsplit, tid, fac[m]);
@@ -613,5 +617,10 @@ static __global__ __launch_bounds__(64) void k_heads_combine(const float* __rest
   if (c < vs) heads_out4(t, r, g, h, c, v, out, Kp);
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   if (h == H - 1)
-    for (int c = g.oc + H * vs + tid * 4; c < g.kend; c += 256) act_store4(out, r, c, Kp, z);
+    for (int c = g.oc + H * vs + tid * 4; c < g.kend; c += blockDim.x * 4) act_store4(out, r, c, Kp, z);
+}
+// grid (R, H), block 64
+static __global__ __launch_bounds__(64) void k_heads_combine(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, HeadsGeom g, MapsArgs mp, Slices t,
+                                                      const int32_t* __restrict__ row_active, bf16_t* __restrict__ out, int Kp) {
+  heads_combine(part_o, part_ml, nsplit, g, mp, t, row_active, out, Kp, blockIdx.x, blockIdx.y);
 }

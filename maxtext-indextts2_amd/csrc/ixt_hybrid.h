@@ -20,7 +20,9 @@ struct HLayer {
   RetGeom rg{};
   ScanGeom sg{};
   HMat in, low, o, gu, down;                     // input projection, second low-rank product (scan: x -> [t | B | C]), output projection, gate | up (or up), down
-  HMat dt;                                       // scan: t -> step sizes
+  HMat dt;                                       // scan: t -> step sizes, and the same row by row [channel][rankp] for few rows
+  void* dtw = nullptr;
+  int rankp = 0;
   std::unique_ptr<HLayer> side;                  // the mixer beside this one: its geometry, parameters, caches and state; columns of the same `in` and `o`
   int in_cols = 0, o_rows = 0;                   // columns of `in`, rows of `o` (a side mixer: its own)
   int c0 = 0, okp = 0;                           // first column of `in` that is this mixer's; columns of a row of the output projection's operand
@@ -63,7 +65,8 @@ struct HybridModel {
   float *x = nullptr, *part2 = nullptr, *h32 = nullptr;      // h32: a routed layer's normed input in f32
   size_t part2_floats = 0;
   void *cat = nullptr;                           // a loop: act of [x | embedding output], Ep columns each
-  float *part3 = nullptr, *scan_x = nullptr, *scan_u = nullptr, *scan_sum = nullptr;
+  void* scan_t = nullptr;                        // the operand of a scan's third projection
+  float *part3 = nullptr, *scan_u = nullptr, *scan_sum = nullptr;
   size_t part3_floats = 0;
   void *xb = nullptr, *act = nullptr, *hact = nullptr, *xn = nullptr, *qx = nullptr, *qr = nullptr, *olat = nullptr, *xg = nullptr, *mhact = nullptr;
   float *dq = nullptr, *dk = nullptr, *dkq = nullptr, *dv = nullptr, *dec = nullptr, *beta = nullptr, *dout = nullptr, *mw = nullptr, *msum = nullptr, *po = nullptr, *pml = nullptr, *ret_u = nullptr, *sgate = nullptr;
@@ -96,10 +99,18 @@ int hybrid_final_norm(ixt_ctx* c, int R, int n, const int32_t* lrows, int lrow0,
 // attention of a layer over heads: projection t -> pages, and the operand of the output projection in m->act.  L: the layer, W: the one with its parameters
 template <typename T>
 int heads_attention(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& t, int R, bool decode, int len_hint, hipStream_t st);
+// one token per row, attention beside retention or lightning attention (L.side), t: the projection of both.  Done where `done` comes back true
+template <typename T>
+int heads_beside_retention(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& t, int R, int len_hint, hipStream_t st, bool* done);
+static inline RetArgs ret_args(const HybridModel* m, const HLayer& L, const Slices& t) {
+  return RetArgs{L.rg, t, L.pow, m->seg, m->chunk, m->nseg, m->dq, m->dk, m->dv, m->ret_u, L.state, m->dout, m->eps};
+}
+static inline size_t ret_step_lds(const RetGeom& g) { return sizeof(float) * (2 * g.dp + g.dvp + 256 / (g.dvp / 4) * g.dvp); }
 // retention (or lightning attention) of a layer: projection t -> the operand of the output projection in m->act
 template <typename T>
 int retention_mix(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& t, int R, int nseg_max, bool single, hipStream_t st);
-// selective scan: the convolved inputs (m->scan_x, and the second projection's operand in m->act); the third projection's operand; everything behind it
+// selective scan: the convolved inputs (the second projection's operand, m->act); the third projection's operand (m->scan_t); everything behind it
+// (dt empty, single only: the third projection as well)
 template <typename T>
 int scan_conv(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& in, int R, hipStream_t st);
 template <typename T>

@@ -48,6 +48,17 @@ static int h_load_vec(const void* src, int dtype, T* dst, int64_t n, hipStream_t
   LAUNCHCHK();
   return IXT_OK;
 }
+// [n][k] -> rows of kp elements (zeros behind k are there already)
+static int h_load_rows(const HybridModel* m, const void* src, int dtype, void* dst, int64_t n, int64_t k, int64_t kp, hipStream_t st) {
+  const unsigned blocks = (unsigned)((n * k + 255) / 256);
+#define HROWS(S_, T_) hipLaunchKernelGGL((k_load_rows<S_, T_>), dim3(blocks), dim3(256), 0, st, (const S_*)src, (T_*)dst, n, k, kp)
+  if (dtype == IXT_BF16) { if (m->f32) HROWS(bf16_t, float); else HROWS(bf16_t, bf16_t); }
+  else if (dtype == IXT_F32) { if (m->f32) HROWS(float, float); else HROWS(float, bf16_t); }
+  else return set_err(IXT_ERR_INVALID, "dtype %d", dtype);
+#undef HROWS
+  LAUNCHCHK();
+  return IXT_OK;
+}
 static int h_load_mat(const HybridModel* m, const void* src, int dtype, void* dst, const LoadMap& lm, hipStream_t st) {
   return m->f32 ? h_load_nk(src, dtype, (float*)dst, lm, st) : h_load_nk(src, dtype, (bf16_t*)dst, lm, st);
 }
@@ -315,7 +326,13 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
         return h_load_mat(m, (const char*)s + (size_t)C * E * (dt == IXT_F32 ? 4 : 2), dt, d, z, st);
       });
     }
-    TRY(vec("mix.conv", &L.cw, C * g.taps, {C, g.taps}));
+    TRY(h_allocf(c, &L.cw, (size_t)g.taps * g.Cp));
+    {
+      float* d = L.cw;
+      LoadMap lm = load_map(g.taps, g.C, g.Cp);                   // tap by tap
+      lm.trans = 1; lm.ld = g.taps;
+      add("mix.conv", {C, g.taps}, [=](const void* s, int dt, hipStream_t st) { return h_load_nk(s, dt, d, lm, st); });
+    }
     TRY(vec("mix.conv.b", &L.cb, C, {C}));
     TRY(h_mat(c, &L.low, g.C, g.oc + g.N));
     {
@@ -330,7 +347,17 @@ static int hybrid_layer_params(ixt_ctx* c, int i) {
       });
     }
     TRY(h_mat(c, &L.dt, g.rank, g.C));
-    mat("mix.dt", L.dt, g.C, g.rank, 0);
+    L.rankp = up_to(g.rank, 8);
+    TRY(h_alloc(c, &L.dtw, (size_t)g.C * L.rankp * m->esz));
+    {
+      void *d = L.dt.w, *rows = L.dtw;
+      const LoadMap lm = load_map(g.C, g.rank, L.dt.Kp);
+      const int64_t wide = L.rankp, rank = g.rank;
+      add("mix.dt", {C, g.rank}, [=](const void* s, int dt, hipStream_t st) -> int {
+        TRY(h_load_mat(m, s, dt, d, lm, st));
+        return h_load_rows(m, s, dt, rows, C, rank, wide, st);
+      });
+    }
     TRY(h_allocf(c, &L.dtb, (size_t)L.dt.Np)); TRY(h_allocf(c, &L.a2, (size_t)g.C * g.Np)); TRY(h_allocf(c, &L.D, (size_t)g.Cp));
     {
       float *b = L.dtb, *a2 = L.a2, *D = L.D;
@@ -472,7 +499,7 @@ int hybrid_init(ixt_ctx* c) {
     if (!tied) m->tensors["head"] = HTensor{{m->V, m->E}, head, false}; }
   TRY(hybrid_norm_params(c, "final.norm", &m->fnorm));
   std::map<std::vector<float>, std::pair<float*, float*>> ropes;
-  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0, ret_u = 0, part3 = 0, scan_x = 0, scan_u = 0, scan_s = 0;
+  size_t act_k = m->Ep, hact_k = 0, qx_e = 0, qr_e = 0, olat_e = 0, part = 0, part2 = 0, s_q = 0, s_kq = 0, s_v = 0, s_dec = 0, s_b = 0, xg_e = 0, mh_e = 0, mi = 0, po = 0, ret_u = 0, part3 = 0, scan_t = 0, scan_u = 0, scan_s = 0;
   bool shifts = false;
   const size_t max_chunks = (size_t)R / SEG_CHUNK + (size_t)std::min(R, c->G) + 1;      // of a pass: a group has at most one run of rows
   auto upd = [](size_t& a, size_t v) { if (v > a) a = v; };
@@ -578,13 +605,13 @@ int hybrid_init(ixt_ctx* c) {
       g.oz = up_to(g.C, 16); g.ob = up_to(g.rank, 16); g.oc = g.ob + up_to(g.N, 16);
       L.okp = up_to(g.C, IXT_KALIGN);
       TRY(h_allocf(c, &L.state, (size_t)c->G * g.C * g.Np));
-      TRY(h_allocf(c, &L.tails, (size_t)c->G * 2 * (g.taps - 1) * g.C + 4));
+      TRY(h_allocf(c, &L.tails, (size_t)c->G * 2 * (g.taps - 1) * g.Cp + 4));
       const int Nx = up_to(g.oc + g.N, 16), Nd = up_to(g.C, 16), Kd = up_to(g.rank, IXT_KALIGN);
       dotsz(m->Ep, up_to(g.oz + g.C, 16));
       upd(part2, dot_floats(L.okp, Nx)); upd(part3, dot_floats(Kd, Nd));
       dotsz(L.okp, up_to(m->E, 16));
-      upd(act_k, L.okp); upd(act_k, Kd);
-      upd(scan_x, (size_t)R * g.Cp); upd(scan_u, max_chunks * g.C * g.Np); upd(scan_s, max_chunks * g.Cp);
+      upd(act_k, L.okp);
+      upd(scan_t, (size_t)Rp * Kd); upd(scan_u, max_chunks * g.C * g.Np); upd(scan_s, max_chunks * g.Cp);
     } else {
       m->recurrent = true;
       DeltaGeom& g = L.dg;
@@ -647,7 +674,7 @@ int hybrid_init(ixt_ctx* c) {
   c->part_floats = part; TRY(h_allocf(c, &c->part, part));
   m->part2_floats = part2; TRY(h_allocf(c, &m->part2, part2 + 4));
   m->part3_floats = part3; TRY(h_allocf(c, &m->part3, part3 + 4));
-  TRY(h_allocf(c, &m->scan_x, scan_x + 4)); TRY(h_allocf(c, &m->scan_u, scan_u + 4)); TRY(h_allocf(c, &m->scan_sum, scan_s + 4));
+  TRY(h_alloc(c, &m->scan_t, (scan_t + 8) * m->esz)); TRY(h_allocf(c, &m->scan_u, scan_u + 4)); TRY(h_allocf(c, &m->scan_sum, scan_s + 4));
   TRY(h_allocf(c, &m->x, (size_t)R * std::max(1, m->streams) * m->E));
   TRY(h_allocf(c, &m->ret_u, ret_u + 4)); TRY(h_allocf(c, &m->chunk, max_chunks)); TRY(h_allocf(c, &m->sgate, (size_t)R + 4));
   TRY(h_alloc(c, &m->xb, (size_t)Rp * m->Ep * m->esz));
@@ -675,7 +702,7 @@ int hybrid_init(ixt_ctx* c) {
     if (L.c.mixer == IXT_MIX_ATTENTION) { pool(L.pages, (int64_t)c->P * L.hg.G * L.hg.dkp); pool(L.vpages, (int64_t)c->P * L.hg.G * L.hg.dvp); }
     else if (L.c.mixer == IXT_MIX_LATENT_ATTENTION) pool(L.pages, (int64_t)c->P * (L.lg.rankp + L.lg.rotp));
     else if (L.c.mixer == IXT_MIX_RETENTION || L.c.mixer == IXT_MIX_LIGHTNING) state(L.state, (int64_t)L.rg.H * L.rg.dp * L.rg.dvp);
-    else if (L.c.mixer == IXT_MIX_SCAN) { state(L.state, (int64_t)L.sg.C * L.sg.Np); state(L.tails, (int64_t)2 * (L.sg.taps - 1) * L.sg.C); }
+    else if (L.c.mixer == IXT_MIX_SCAN) { state(L.state, (int64_t)L.sg.C * L.sg.Np); state(L.tails, (int64_t)2 * (L.sg.taps - 1) * L.sg.Cp); }
     else { state(L.state, (int64_t)L.dg.H * L.dg.dv * L.dg.dp); state(L.tails, (int64_t)2 * (L.dg.taps - 1) * L.dg.C); }
     if (L.shift) state(L.shift, (int64_t)2 * m->Ep);
   };
@@ -915,6 +942,9 @@ static int hybrid_mixer_columns(ixt_ctx* c, const HLayer& L, const HLayer& W, in
     if (l.c.mixer == IXT_MIX_ATTENTION) return heads_attention<T>(c, l, w, own, R, decode, len_hint, st);
     return retention_mix<T>(c, l, w, own, R, nseg_max, decode, st);
   };
+  bool done = false;
+  if (decode) TRY(heads_beside_retention<T>(c, L, W, t, R, len_hint, st, &done));
+  if (done) return IXT_OK;
   TRY(one(L, W, t));
   return L.side ? one(*L.side, *W.side, t.from(L.side->c0)) : (int)IXT_OK;
 }
@@ -922,13 +952,15 @@ static int hybrid_mixer_columns(ixt_ctx* c, const HLayer& L, const HLayer& W, in
 template <typename T>
 static int hybrid_mixer_scan(ixt_ctx* c, const HLayer& L, const HLayer& W, int R, int nseg_max, bool single, hipStream_t st) {
   HybridModel* m = c->hy;
-  Slices in, low, dt;
+  Slices in, low, dt{};
   TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &in));
   TRY(scan_conv<T>(c, L, W, in, R, st));
   TRY(hdot<T>(c, (const T*)m->act, W.low, R, m->part2, m->part2_floats, st, &low));
-  TRY(scan_rank<T>(c, W, low, R, st));
-  TRY(hdot<T>(c, (const T*)m->act, W.dt, R, m->part3, m->part3_floats, st, &dt));
-  dt.bias = W.dtb;
+  if (!single || R > 32) {                                         // (few rows: k_scan_step works the step sizes out itself)
+    TRY(scan_rank<T>(c, W, low, R, st));
+    TRY(hdot<T>(c, (const T*)m->scan_t, W.dt, R, m->part3, m->part3_floats, st, &dt));
+    dt.bias = W.dtb;
+  }
   return scan_mix<T>(c, L, W, in, low, dt, R, nseg_max, single, st);
 }
 

@@ -15,6 +15,7 @@
 // ---------------------------------------------------------------------------------------------------- activation storage
 __device__ __forceinline__ void act_store1(bf16_t* b, int r, int k, int Kp, float v) { b[xidx(r, k, Kp)] = f2bf(v); }
 __device__ __forceinline__ void act_store1(float* b, int r, int k, int Kp, float v) { b[(size_t)r * Kp + k] = v; }
+template <typename T> __device__ __forceinline__ size_t act_at(int r, int k, int Kp) { return sizeof(T) == 2 ? (size_t)xidx(r, k, Kp) : (size_t)r * Kp + k; }      // place of an element
 __device__ __forceinline__ void act_store4(bf16_t* b, int r, int k0, int Kp, const float* v) {      // k0 % 4 == 0
   uint2 o;
   o.x = pack2(f2bf(v[0]), f2bf(v[1])); o.y = pack2(f2bf(v[2]), f2bf(v[3]));
@@ -46,15 +47,16 @@ struct Slices {             // a dot's output; bias: one number per column joins
     if (bias != nullptr) t += bias[c];
     return t;
   }
-  __device__ __forceinline__ void at4(int r, int c, float* o) const {       // c % 4 == 0
+  template <int B = 4>
+  __device__ __forceinline__ void at4(int r, int c, float* o) const {       // c % 4 == 0; B slices in flight
     const float* q = p + (size_t)r * ncols + c;
     float4 t = *reinterpret_cast<const float4*>(q);
-    for (int s = 1; s < n; s += 4) {                                        // four slices in flight
-      float4 u[4];
+    for (int s = 1; s < n; s += B) {
+      float4 u[B];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) u[i] = *reinterpret_cast<const float4*>(q + (size_t)min(s + i, n - 1) * stride);
+      for (int i = 0; i < B; ++i) u[i] = *reinterpret_cast<const float4*>(q + (size_t)min(s + i, n - 1) * stride);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+      for (int i = 0; i < B; ++i)
         if (s + i < n) { t.x += u[i].x; t.y += u[i].y; t.z += u[i].z; t.w += u[i].w; }
     }
     if (bias != nullptr) {
@@ -89,6 +91,14 @@ __device__ __forceinline__ float block_sum256(float v, float* red /*[4] LDS*/) {
 }
 __device__ __forceinline__ float f32_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float f32_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// The same by max(z, 0) + log(1 + e), e = exp(-|z|), log(1 + e) = 2 artanh(s), s = e / (2 + e) <= 1/3, by its series (next term below 2e-8 of the sum): error
+// below 1e-6 of the value for |z| < 10, |z| 1e-7 beyond
+__device__ __forceinline__ float hw_softplus(float z) {
+  const float e = hw_exp2(-1.44269504088896340736f * fabsf(z)), s = e * hw_rcp(2.0f + e), q = s * s;
+  float p = fmaf(q, 1.0f / 15.0f, 1.0f / 13.0f);
+  p = fmaf(q, p, 1.0f / 11.0f); p = fmaf(q, p, 1.0f / 9.0f); p = fmaf(q, p, 1.0f / 7.0f); p = fmaf(q, p, 0.2f); p = fmaf(q, p, 1.0f / 3.0f);
+  return fmaxf(z, 0.0f) + fmaf(2.0f * s * q, p, 2.0f * s);
+}
 
 // ---------------------------------------------------------------------------------------------------- f32 dot
 // out[r][n] = sum_k x[r][k] w[n][k], k ascending by fma.  x [R][Kp], w [Np][Kp] row-major f32, Kp % 32 == 0, Np % 16 == 0.  Grouped: 16-row block rb
@@ -147,6 +157,11 @@ __global__ void k_load_nk(const S* __restrict__ src, T* __restrict__ dst, LoadMa
   const int col = m.inter ? ((nn >> 4) * 2 + m.n_off) * 16 + (nn & 15) : m.n_off + nn;
   if constexpr (sizeof(T) == 2) dst[widx(m.k_off + kk, col, m.Kp)] = f2bf(v);
   else dst[(size_t)col * m.Kp + m.k_off + kk] = v;
+}
+template <typename S, typename T>
+__global__ void k_load_rows(const S* __restrict__ src, T* __restrict__ dst, int64_t n, int64_t k, int64_t kp) {
+  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n * k) dst[i / k * kp + i % k] = from_f<T>(to_f(src[i]));
 }
 template <typename S, typename T>
 __global__ void k_load_vec(const S* __restrict__ src, T* __restrict__ dst, int64_t n) {
@@ -378,6 +393,28 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
   const int r = blockIdx.x, top = a.top, E = a.E, Ep = a.Ep;
   const bool vec = (E & 3) == 0;
   float v[NI][8], xv[NI][8];
+  constexpr bool AHEAD = NI <= 2 && SM == 0;               // the group's last h is requested before anything else
+  [[maybe_unused]] float old[AHEAD ? NI : 1][8];
+  const float* before = nullptr;                           // the group's last h, and where this one goes
+  float* keep = nullptr;
+  if (SM == 0 && a.shift.mu != nullptr) {
+    const int active = a.shift.active[r], grp = a.shift.slot[r], pos = a.shift.pos[r];
+    if (active) {
+      const int par = a.shift.parity[grp] ^ 1;
+      float* base = a.shift.state + (size_t)grp * 2 * Ep;
+      if (pos > 0) before = base + (size_t)par * Ep;
+      keep = base + (size_t)(par ^ 1) * Ep;
+    }
+    if constexpr (AHEAD) {
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int k0 = i * 2048 + threadIdx.x * 8;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) old[i][j] = 0.0f;
+        if (before != nullptr && k0 < Ep) load8(before + k0, old[i]);
+      }
+    }
+  }
   constexpr bool EARLY = SM > 0 && NI * SM <= 8;           // the streams are requested before anything else
   float4 es[EARLY ? NI * SM * 2 : 1];
   if constexpr (EARLY) {
@@ -401,7 +438,7 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
     for (int q = 0; q < 8; q += 4) {
       if (k0 + q >= E) continue;
       if (pos == nullptr) {
-        if (t.n > 0) t.at4(r, k0 + q, v[i] + q);
+        if (t.n > 0) t.template at4<NI == 1 ? 10 : 4>(r, k0 + q, v[i] + q);
       } else {
         for (int j = 0; j < top; ++j) {
           float u[4];
@@ -512,14 +549,6 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
   if (SM > 0 && a.hc.in == nullptr) return;                // the head takes the streams themselves
   NormStat st{};
   if (pre.w != nullptr) st = row_stat<KIND, NI>(pre, xv, E, a.eps, red);
-  const float* before = nullptr;                           // the group's last h, and where this one goes
-  float* keep = nullptr;
-  if (a.shift.mu != nullptr && a.shift.active[r]) {
-    const int grp = a.shift.slot[r], par = a.shift.parity[grp] ^ 1;
-    float* base = a.shift.state + (size_t)grp * 2 * Ep;
-    if (a.shift.pos[r] > 0) before = base + (size_t)par * Ep;
-    keep = base + (size_t)(par ^ 1) * Ep;
-  }
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int k0 = i * 2048 + threadIdx.x * 8;
@@ -530,13 +559,16 @@ __global__ __launch_bounds__(256) void k_sub_norm(SubNormArgs a, float* __restri
       for (int j = 0; j < 8; ++j)
         if (k0 + j < E) h32[(size_t)r * E + k0 + j] = xv[i][j];
     }
-    if (a.shift.mu != nullptr) {
-      float mu[8], old[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
+    if (SM == 0 && a.shift.mu != nullptr) {
+      float mu[8], od[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
       load8(a.shift.mu + k0, mu);
-      if (before != nullptr) load8(before + k0, old);
+      if constexpr (AHEAD) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) od[j] = old[i][j];
+      } else if (before != nullptr) load8(before + k0, od);
       if (keep != nullptr) { store4(keep + k0, xv[i]); store4(keep + k0 + 4, xv[i] + 4); }
 #pragma unroll
-      for (int j = 0; j < 8; ++j) xv[i][j] = fmaf(old[j] - xv[i][j], mu[j], xv[i][j]);
+      for (int j = 0; j < 8; ++j) xv[i][j] = fmaf(od[j] - xv[i][j], mu[j], xv[i][j]);
     }
     if (xb != nullptr) act_store8(xb, r, k0, a.Kp, xv[i]);
   }

@@ -14,12 +14,11 @@ int retention_mix(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& t,
   const RetGeom& g = L.rg;
   const RowsArgs rows{c->row_slot, c->row_pos, c->row_active, c->ps.page_map};
   const HeadsRope rope{L.rope_cos, L.rope_sin};
-  const RetArgs a{g, t, L.pow, m->seg, m->chunk, m->nseg, m->dq, m->dk, m->dv, m->ret_u, L.state, m->dout, m->eps};
+  const RetArgs a = ret_args(m, L, t);
   T* out = (T*)m->act;
   const int Kp = W.okp;
   if (single) {            // every row is a run of one token
-    const int ns = 256 / (g.dvp / 4);
-    hipLaunchKernelGGL((k_ret_step<T>), dim3(R, g.H), dim3(256), sizeof(float) * (2 * g.dp + g.dvp + ns * g.dvp), st, a, rope, rows, out, Kp);
+    hipLaunchKernelGGL((k_ret_step<T>), dim3(R, g.H), dim3(256), ret_step_lds(g), st, a, rope, rows, out, Kp);
   } else {
     const int widest = std::max(g.dp, g.dvp), chunks = R / SEG_CHUNK + nseg_max;
 #define RPREP(LP_) hipLaunchKernelGGL((k_ret_prep<LP_>), dim3(R, (3 * g.H * LP_ + 255) / 256), dim3(256), 0, st, a, rope, rows)
@@ -47,14 +46,14 @@ template int retention_mix<float>(ixt_ctx*, const HLayer&, const HLayer&, const 
 template <typename T>
 int scan_conv(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& in, int R, hipStream_t st) {
   HybridModel* m = c->hy;
-  const ScanConvArgs a{in, L.sg, W.cw, W.cb, m->row_seg, m->row_j, m->seg, L.tails, m->scan_x};
-  hipLaunchKernelGGL((k_scan_conv<T>), dim3(R, (W.low.Kp + 255) / 256), dim3(256), 0, st, a, (T*)m->act, W.low.Kp);
+  const ScanConvArgs a{in, L.sg, W.cw, W.cb, m->row_seg, m->row_j, m->seg, L.tails};
+  hipLaunchKernelGGL((k_scan_conv<T>), dim3(R, (W.okp + 1023) / 1024), dim3(256), 0, st, a, (T*)m->act, W.okp);
   LAUNCHCHK();
   return IXT_OK;
 }
 template <typename T>
 int scan_rank(ixt_ctx* c, const HLayer& W, const Slices& low, int R, hipStream_t st) {
-  hipLaunchKernelGGL((k_scan_rank<T>), dim3(R), dim3(128), 0, st, low, W.sg.rank, (T*)c->hy->act, W.dt.Kp);
+  hipLaunchKernelGGL((k_scan_rank<T>), dim3(R), dim3(64), 0, st, low, W.sg.rank, (T*)c->hy->scan_t, W.dt.Kp);
   LAUNCHCHK();
   return IXT_OK;
 }
@@ -62,16 +61,16 @@ template <typename T, int SPL, int LPC>
 static int scan_chunks(ixt_ctx* c, const ScanArgs& a, int R, int nseg_max, int Kp, hipStream_t st) {
   static bool attr_done = false;
   if (!attr_done) {
-    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_scan_sums<SPL, LPC>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)scan_lds<SPL, LPC, false>()));
+    HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_scan_sums<T, SPL, LPC>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)scan_lds<SPL, LPC, false>()));
     HIPCHK(hipFuncSetAttribute(reinterpret_cast<const void*>(&k_scan_out<T, SPL, LPC>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)scan_lds<SPL, LPC, true>()));
     attr_done = true;
   }
   constexpr int CB = 256 / LPC;
   const ScanGeom& g = a.g;
   const int chunks = R / SEG_CHUNK + nseg_max;
-  hipLaunchKernelGGL((k_scan_sums<SPL, LPC>), dim3(chunks, (g.C + CB - 1) / CB), dim3(256), (scan_lds<SPL, LPC, false>()), st, a);
+  hipLaunchKernelGGL((k_scan_sums<T, SPL, LPC>), dim3(chunks, (g.C + CB - 1) / CB), dim3(256), (scan_lds<SPL, LPC, false>()), st, a, (const T*)c->hy->act, Kp);
   hipLaunchKernelGGL(k_scan_carry, dim3(nseg_max, (unsigned)(((size_t)g.C * g.Np + 1023) / 1024)), dim3(256), 0, st, a);
-  hipLaunchKernelGGL((k_scan_out<T, SPL, LPC>), dim3(chunks, (std::max(g.C, Kp) + CB - 1) / CB), dim3(256), (scan_lds<SPL, LPC, true>()), st, a, (T*)c->hy->act, Kp);
+  hipLaunchKernelGGL((k_scan_out<T, SPL, LPC>), dim3(chunks, (g.C + CB - 1) / CB), dim3(256), (scan_lds<SPL, LPC, true>()), st, a, (T*)c->hy->act, Kp);
   LAUNCHCHK();
   return IXT_OK;
 }
@@ -79,18 +78,20 @@ template <typename T>
 int scan_mix(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& in, const Slices& low, const Slices& dt, int R, int nseg_max, bool single, hipStream_t st) {
   HybridModel* m = c->hy;
   const ScanGeom& g = L.sg;
-  const ScanArgs a{g, in, low, dt, W.a2, W.D, m->seg, m->chunk, m->nseg, m->scan_x, m->scan_u, m->scan_sum, L.state};
+  const ScanArgs a{g, in, low, dt, m->part3, W.a2, W.D, m->seg, m->chunk, m->nseg, m->scan_u, m->scan_sum, L.state};
   const int Kp = W.okp;
   if (single) {
-#define SSTEP(LPC_) case 4 * LPC_: hipLaunchKernelGGL((k_scan_step<T, LPC_>), dim3(R, (std::max(g.C, Kp) * LPC_ + 255) / 256), dim3(256), 0, st, a, c->row_active, c->row_slot, c->row_pos, \
-                                                      (T*)m->act, Kp); break
+#define SSTEP_C(LPC_, CH_, OWN_) hipLaunchKernelGGL((k_scan_step<T, LPC_, CH_, OWN_>), dim3(R, (g.C * LPC_ + 256 * CH_ - 1) / (256 * CH_)), dim3(256), OWN_ ? sizeof(float) * W.rankp : 0, st, a, \
+                                                    (const T*)W.dtw, W.rankp, W.dtb, c->row_active, c->row_slot, c->row_pos, (T*)m->act, Kp)
+#define SSTEP(LPC_) case 4 * LPC_: if (dt.p == nullptr) SSTEP_C(LPC_, 1, true); else if (R * (size_t)g.C * LPC_ >= 256 * 4096) SSTEP_C(LPC_, 4, false); else SSTEP_C(LPC_, 1, false); break
     switch (g.Np) { SSTEP(4); SSTEP(8); SSTEP(16); SSTEP(32); SSTEP(64); default: return set_err(IXT_ERR_UNSUPPORTED, "selective scan: %d states", g.N); }
 #undef SSTEP
+#undef SSTEP_C
     LAUNCHCHK();
     return IXT_OK;
   }
   switch (g.Np) {
-    case 16: return scan_chunks<T, 4, 4>(c, a, R, nseg_max, Kp, st);
+    case 16: return scan_chunks<T, 4, 4>(c, a, R, nseg_max, Kp, st);      // (8 states on two lanes: 44 against 28 us)
     case 32: return scan_chunks<T, 8, 4>(c, a, R, nseg_max, Kp, st);
     case 64: return scan_chunks<T, 16, 4>(c, a, R, nseg_max, Kp, st);
     case 128: return scan_chunks<T, 16, 8>(c, a, R, nseg_max, Kp, st);

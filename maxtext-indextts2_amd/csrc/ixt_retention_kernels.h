@@ -300,12 +300,12 @@ __global__ __launch_bounds__(256) void k_ret_gate(RetArgs a, const int32_t* __re
   if (h == g.H - 1)
     for (int k = g.oc + g.H * g.vs + lane * 4; k < g.kend; k += 256) act_store4(out, r, k, Kp, z);
 }
-// all heads of a row: o / rms(o) w sigmoid(gate); w [H][vs], zeros behind a head's dv.  grid R, block 256.
+// all heads of a row: o / rms(o) w sigmoid(gate); w [H][vs], zeros behind a head's dv.  A block of 256.
 template <typename T>
-__global__ __launch_bounds__(256) void k_ret_join(RetArgs a, const float* __restrict__ w, const int32_t* __restrict__ row_active, T* __restrict__ out, int Kp) {
+__device__ __forceinline__ void ret_join(const RetArgs& a, const float* __restrict__ w, const int32_t* __restrict__ row_active, T* __restrict__ out, int Kp, const int r) {
   __shared__ float red[4];
   const RetGeom& g = a.g;
-  const int r = blockIdx.x, tid = threadIdx.x, n = g.H * g.vs;
+  const int tid = threadIdx.x, n = g.H * g.vs;
   if (!row_active[r]) return;
   const float* o = a.o + (size_t)r * g.H * g.dvp;
   constexpr int B = 4;                                       // columns of a thread that stay in registers, in fours
@@ -344,15 +344,19 @@ __global__ __launch_bounds__(256) void k_ret_join(RetArgs a, const float* __rest
   const float zero[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   for (int k = g.oc + n + tid * 4; k < g.kend; k += 1024) act_store4(out, r, k, Kp, zero);
 }
+// grid R, block 256
+template <typename T>
+__global__ __launch_bounds__(256) void k_ret_join(RetArgs a, const float* __restrict__ w, const int32_t* __restrict__ row_active, T* __restrict__ out, int Kp) {
+  ret_join<T>(a, w, row_active, out, Kp, blockIdx.x);
+}
 
 // Decode: block = (row, head).  A thread owns four value columns and every `ns`-th key row; the first of them are requested before anything else.
-// grid (R, H), block 256, LDS (2 dp + dvp + ns dvp) floats, ns = 256 / (dvp / 4).
+// A block of 256, LDS (2 dp + dvp + ns dvp) floats, ns = 256 / (dvp / 4).
 template <typename T>
-__global__ __launch_bounds__(256) void k_ret_step(RetArgs a, HeadsRope rope, RowsArgs rows, T* __restrict__ out, int Kp) {
-  extern __shared__ __attribute__((aligned(16))) float sm[];
+__device__ __forceinline__ void ret_step(const RetArgs& a, const HeadsRope& rope, const RowsArgs& rows, T* __restrict__ out, int Kp, const int r, const int h, float* sm) {
   __shared__ float red[4];
   const RetGeom& g = a.g;
-  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int active = rows.active[r], pos = rows.pos[r], grp = rows.slot[r];      // (requested together)
   if (!active) return;
   float *qs = sm, *ks = sm + g.dp, *vs = ks + g.dp, *os = vs + g.dvp;
@@ -426,4 +430,27 @@ __global__ __launch_bounds__(256) void k_ret_step(RetArgs a, HeadsRope rope, Row
   const float z[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   if (h == g.H - 1)
     for (int k = g.oc + g.H * g.vs + tid * 4; k < g.kend; k += 1024) act_store4(out, r, k, Kp, z);
+}
+// grid (R, H), block 256
+template <typename T>
+__global__ __launch_bounds__(256) void k_ret_step(RetArgs a, HeadsRope rope, RowsArgs rows, T* __restrict__ out, int Kp) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  ret_step<T>(a, rope, rows, out, Kp, blockIdx.x, blockIdx.y, sm);
+}
+
+// Attention over heads and a retention side by side, one token per row: the blocks of both in one launch, which is as long as the longer of the two and not
+// as their sum.  grid R H + R G hchunks nsplit, block 256, LDS the larger of the two.
+template <int DK, int DV>
+__global__ __launch_bounds__(256, 2) void k_pair_decode(HeadsAttnArgs a, int nsplit, RetArgs b, HeadsRope rope, int Kp) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t tile[];
+  int i = blockIdx.x;
+  if (i < a.R * b.g.H) { ret_step<bf16_t>(b, rope, a.rows, a.out, Kp, i / b.g.H, i % b.g.H, reinterpret_cast<float*>(tile)); return; }
+  i -= a.R * b.g.H;
+  const int hb = a.g.G * a.hchunks;
+  heads_decode<DK, DV, true, 1>(a, i / nsplit / hb, i / nsplit % hb, i % nsplit, nsplit, tile);
+}
+// their second half: key splits put together, the retention's heads normed together.  grid (R, H + 1), block 256.
+static __global__ __launch_bounds__(256) void k_pair_join(HeadsAttnArgs a, int nsplit, RetArgs b, const float* __restrict__ w, int Kp) {
+  if ((int)blockIdx.y < a.g.H) heads_combine(a.part_o, a.part_ml, nsplit, a.g, a.mp, a.t, a.rows.active, a.out, Kp, blockIdx.x, blockIdx.y);
+  else ret_join<bf16_t>(b, w, a.rows.active, a.out, Kp, blockIdx.x);
 }

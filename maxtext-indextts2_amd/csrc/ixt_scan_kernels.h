@@ -6,9 +6,9 @@
 // Over a run of rows the recurrence goes by chunks of SEG_CHUNK rows (k_segments lists them): the state behind a chunk is exp(A sum dt) times the one in
 // front of it plus what the chunk leaves by itself.
 //
-//   k_scan_conv   projection slices -> x in f32 and as the operand of the next projection
+//   k_scan_conv   projection slices -> x, the operand of the next projection, where every later kernel reads it and the outputs take its place
 //   k_scan_rank   the step-size part of that projection as the operand of the third one
-//   k_scan_sums   chunk by chunk: U = the state a chunk leaves from zero, and its sum of dt
+//   k_scan_sums   chunk by chunk: U = the state a chunk leaves from zero, and its sum of dt; the step sizes in the place of their projection
 //   k_scan_carry  run by run: the state in front of every chunk, in the place of its U; the group's new state
 //   k_scan_out    chunk by chunk: the outputs
 //   k_scan_step   one token per row (decode)
@@ -23,9 +23,9 @@ struct ScanGeom {
 };
 struct ScanArgs {
   ScanGeom g; Slices in, low, dt;           // the three projections (dt: the third one, with its bias)
+  float* dts;                               // the first slice of dt
   const float *a2, *D;                      // [C][Np]: -exp(A_log) log2(e), zeros behind N; [Cp]
   const int32_t* seg; const int4* chunk; const int32_t* nseg;
-  const float* x;                           // [R][Cp]
   float *u, *sum, *state;                   // [chunk][C][Np], [chunk][Cp], [group][C][Np]
 };
 
@@ -35,33 +35,72 @@ static __global__ __launch_bounds__(256) void k_scan_rates(float* __restrict__ a
   if (i < C * Np && i % Np < N) a2[i] = -1.44269504088896340736f * expf(a2[i]);
 }
 
-// grid (R, ceil(Kp / 256)), block 256: a channel per thread.  tails [group][2][taps - 1][C].
+// four elements of an operand (k0 % 4 == 0)
+__device__ __forceinline__ float4 act_load4(const bf16_t* b, int r, int k0, int Kp) {
+  const uint2 v = *reinterpret_cast<const uint2*>(b + xidx(r, k0, Kp));
+  return make_float4(bflo(v.x), bfhi(v.x), bflo(v.y), bfhi(v.y));
+}
+__device__ __forceinline__ float4 act_load4(const float* b, int r, int k0, int Kp) { return *reinterpret_cast<const float4*>(b + (size_t)r * Kp + k0); }
+
+// Convolution, bias, silu.  Weights [taps][Cp], tails [group][2][taps - 1][Cp].  grid (R, ceil(Kp / 1024)), block 256: four channels per thread.
 struct ScanConvArgs {
   Slices t; ScanGeom g; const float *w, *bias; const int32_t *row_seg, *row_j, *seg;
-  float *tails, *x;
+  float* tails;
 };
 template <typename T>
 __global__ __launch_bounds__(256) void k_scan_conv(ScanConvArgs a, T* __restrict__ out, int Kp) {
   const ScanGeom& g = a.g;
-  const int r = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x, s = a.row_seg[r];
+  const int r = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 4, s = a.row_seg[r];
   if (s < 0 || c >= Kp) return;
-  float v = 0.0f;
-  if (c < g.C) {
+  float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  if (c < g.Cp) {                                            // (everything is zero in channels C .. Cp - 1)
     const int32_t* sg = a.seg + (size_t)s * 8;
-    const size_t tsz = (size_t)(g.taps - 1) * g.C;
-    float* tb = a.tails + (size_t)sg[2] * 2 * tsz;
-    const ConvCtx cc{tb + (size_t)sg[4] * tsz, tb + (size_t)(sg[4] ^ 1) * tsz, a.row_j[r], sg[1], sg[3]};
-    v = conv_channel(a.t, r, c, a.w + (size_t)c * g.taps, g.taps, c, g.C, cc) + a.bias[c];
-    v *= f32_sigmoid(v);
+    const int n = sg[1], start = sg[3], par = sg[4], j = a.row_j[r], taps = g.taps;
+    const size_t tsz = (size_t)(taps - 1) * g.Cp;
+    const float* tin = a.tails + ((size_t)sg[2] * 2 + par) * tsz + c;
+    float* tout = a.tails + ((size_t)sg[2] * 2 + (par ^ 1)) * tsz + c;
+    const float4 b = *reinterpret_cast<const float4*>(a.bias + c), w0 = *reinterpret_cast<const float4*>(a.w + (size_t)(taps - 1) * g.Cp + c);
+    float x0[4];
+    a.t.at4(r, c, x0);
+    v[0] = fmaf(x0[0], w0.x, b.x); v[1] = fmaf(x0[1], w0.y, b.y); v[2] = fmaf(x0[2], w0.z, b.z); v[3] = fmaf(x0[3], w0.w, b.w);
+    for (int b0 = 1; b0 < taps; b0 += 3) {                   // three earlier inputs in flight: rows of the run, or what is kept of those before it (oldest first)
+      float4 x[3], w[3];
+#pragma unroll
+      for (int i = 0; i < 3; ++i) {
+        const int back = min(b0 + i, taps - 1);
+        const bool mine = j - back >= 0;
+        const float* src = mine ? a.t.p + (size_t)(r - back) * a.t.ncols + c : tin + (size_t)max(taps - 1 - (back - j), 0) * g.Cp;
+        x[i] = mine || start > 0 ? *reinterpret_cast<const float4*>(src) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+        w[i] = b0 + i < taps ? *reinterpret_cast<const float4*>(a.w + (size_t)(taps - 1 - back) * g.Cp + c) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+        if (mine)
+          for (int q = 1; q < a.t.n; ++q) {
+            const float4 u = *reinterpret_cast<const float4*>(src + (size_t)q * a.t.stride);
+            x[i].x += u.x; x[i].y += u.y; x[i].z += u.z; x[i].w += u.w;
+          }
+      }
+#pragma unroll
+      for (int i = 0; i < 3; ++i) { v[0] = fmaf(x[i].x, w[i].x, v[0]); v[1] = fmaf(x[i].y, w[i].y, v[1]); v[2] = fmaf(x[i].z, w[i].z, v[2]); v[3] = fmaf(x[i].w, w[i].w, v[3]); }
+    }
+    const int dist = n - 1 - j;                              // what the next run needs: the last taps - 1 inputs
+    if (dist < taps - 1) *reinterpret_cast<float4*>(tout + (size_t)(taps - 2 - dist) * g.Cp) = make_float4(x0[0], x0[1], x0[2], x0[3]);
+    if (dist == 0)
+      for (int e = n; e < taps - 1; ++e)
+        *reinterpret_cast<float4*>(tout + (size_t)(taps - 2 - e) * g.Cp) = start > 0 ? *reinterpret_cast<const float4*>(tin + (size_t)(taps - 2 - (e - n)) * g.Cp) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= f32_sigmoid(v[e]);
   }
-  if (c < g.Cp) a.x[(size_t)r * g.Cp + c] = v;
-  act_store1(out, r, c, Kp, v);
+  act_store4(out, r, c, Kp, v);
 }
 
-// grid (R), block 128
+// grid (R), block 64: four columns per thread and round
 template <typename T>
-__global__ __launch_bounds__(128) void k_scan_rank(Slices low, int rank, T* __restrict__ out, int Kp) {
-  for (int k = threadIdx.x; k < Kp; k += 128) act_store1(out, blockIdx.x, k, Kp, k < rank ? low.at(blockIdx.x, k) : 0.0f);
+__global__ __launch_bounds__(64) void k_scan_rank(Slices low, int rank, T* __restrict__ out, int Kp) {
+  const int r = blockIdx.x;
+  for (int k = threadIdx.x * 4; k < Kp; k += 256) {
+    float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    if (k < rank) low.at4(r, k, v);                          // (columns behind the rank are zero up to the next multiple of 16)
+    act_store4(out, r, k, Kp, v);
+  }
 }
 
 // sum over the LPC (1, 2, 4, .. 64) lanes of a channel, every lane ends up with it
@@ -74,64 +113,88 @@ __device__ __forceinline__ float lanes_sum(float v) {
   return v;
 }
 
-// A chunk's operands -> LDS: step sizes and inputs [SEG_CHUNK][CB] of CB channels from c0 on, the B (and C) columns [SEG_CHUNK][Np]
-template <int SPL, int LPC, bool OUT>
-__device__ __forceinline__ void scan_stage(const ScanArgs& a, const int4& c, int c0, float* dts, float* xs, float* bs, float* cs) {
+// the value of lane i (0 .. 3, a constant) of this lane's four
+__device__ __forceinline__ float quad_lane(float v, int i) {
+  const int x = __float_as_int(v);
+  return __int_as_float(i == 0 ? __builtin_amdgcn_update_dpp(0, x, 0x00, 0xf, 0xf, false) : i == 1 ? __builtin_amdgcn_update_dpp(0, x, 0x55, 0xf, 0xf, false)
+                        : i == 2 ? __builtin_amdgcn_update_dpp(0, x, 0xAA, 0xf, 0xf, false) : __builtin_amdgcn_update_dpp(0, x, 0xFF, 0xf, 0xf, false));
+}
+
+// A chunk's operands -> LDS: {dt, dt x} [SEG_CHUNK][CB] of CB channels from c0 on, the B (and C) columns [SEG_CHUNK][Np]; zeros behind the chunk's rows: such
+// a token changes nothing.  OUT: the step sizes are in place already (k_scan_sums)
+template <typename T, int SPL, int LPC, bool OUT>
+__device__ __forceinline__ void scan_stage(const ScanArgs& a, const int4& c, int c0, const T* __restrict__ act, int Kp, float2* ds, float* bs, float* cs) {
   constexpr int CB = 256 / LPC, NP = SPL * LPC, QB = CB / 4, QN = NP / 4;
   const ScanGeom& g = a.g;
   const int tid = threadIdx.x, n = c.y;
+#pragma unroll 4
   for (int i = tid; i < SEG_CHUNK * QB; i += 256) {
     const int j = i / QB, q = i % QB * 4, ch = c0 + q;
     float d[4] = {0.0f, 0.0f, 0.0f, 0.0f};
     float4 x = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-    if (j < n && ch < g.Cp) {                                // (columns C .. Cp - 1 of both are zero projections; a2 and D are zero there)
-      a.dt.at4(c.x + j, ch, d);
-      x = *reinterpret_cast<const float4*>(a.x + (size_t)(c.x + j) * g.Cp + ch);
+    if (j < n && ch < g.Cp) {                                // (in columns C .. Cp - 1 x is zero)
+      x = act_load4(act, c.x + j, ch, Kp);
+      if (OUT) {
+        const float4 u = *reinterpret_cast<const float4*>(a.dts + (size_t)(c.x + j) * a.dt.ncols + ch);
+        d[0] = u.x; d[1] = u.y; d[2] = u.z; d[3] = u.w;
+      } else {
+        a.dt.at4(c.x + j, ch, d);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) d[e] = f32_softplus(d[e]);
+        for (int e = 0; e < 4; ++e) d[e] = hw_softplus(d[e]);
+        *reinterpret_cast<float4*>(a.dts + (size_t)(c.x + j) * a.dt.ncols + ch) = make_float4(d[0], d[1], d[2], d[3]);
+      }
     }
-    *reinterpret_cast<float4*>(dts + j * CB + q) = make_float4(d[0], d[1], d[2], d[3]);
-    *reinterpret_cast<float4*>(xs + j * CB + q) = x;
+    float4* o = reinterpret_cast<float4*>(ds + j * CB + q);
+    o[0] = make_float4(d[0], d[0] * x.x, d[1], d[1] * x.y);
+    o[1] = make_float4(d[2], d[2] * x.z, d[3], d[3] * x.w);
   }
   for (int i = tid; i < SEG_CHUNK * QN; i += 256) {
     const int j = i / QN, q = i % QN * 4;
     float b[4] = {0.0f, 0.0f, 0.0f, 0.0f}, y[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-    if (j < n)
-#pragma unroll
-      for (int e = 0; e < 4; ++e)
-        if (q + e < g.N) {
-          b[e] = a.low.at(c.x + j, g.ob + q + e);
-          if (OUT) y[e] = a.low.at(c.x + j, g.oc + q + e);
-        }
+    if (j < n && q < g.N) {                                  // (columns behind N are zero up to the next multiple of 16)
+      a.low.at4(c.x + j, g.ob + q, b);
+      if (OUT) a.low.at4(c.x + j, g.oc + q, y);
+    }
     *reinterpret_cast<float4*>(bs + j * NP + q) = make_float4(b[0], b[1], b[2], b[3]);
     if (OUT) *reinterpret_cast<float4*>(cs + j * NP + q) = make_float4(y[0], y[1], y[2], y[3]);
   }
 }
 template <int SPL, int LPC, bool OUT> constexpr size_t scan_lds() { return sizeof(float) * SEG_CHUNK * (2 * (256 / LPC) + (OUT ? 2 : 1) * SPL * LPC); }
+template <int N>
+__device__ __forceinline__ void lds_read(const float* p, float* v) {      // N a multiple of 4
+#pragma unroll
+  for (int i = 0; i < N; i += 4) { const float4 u = *reinterpret_cast<const float4*>(p + i); v[i] = u.x; v[i + 1] = u.y; v[i + 2] = u.z; v[i + 3] = u.w; }
+}
 
 // grid (chunks, ceil(C / CB)), block 256, LDS scan_lds<SPL, LPC, false>()
-template <int SPL, int LPC>
-__global__ __launch_bounds__(256) void k_scan_sums(ScanArgs a) {
+template <typename T, int SPL, int LPC>
+__global__ __launch_bounds__(256) void k_scan_sums(ScanArgs a, const T* __restrict__ act, int Kp) {
   constexpr int CB = 256 / LPC, NP = SPL * LPC;
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const ScanGeom& g = a.g;
   const int ch = blockIdx.x, tid = threadIdx.x, cl = tid / LPC, sub = tid % LPC, c0 = blockIdx.y * CB, col = c0 + cl;
   if (ch >= a.nseg[1]) return;
   const int4 c = a.chunk[ch];
-  float *dts = sm, *xs = dts + SEG_CHUNK * CB, *bs = xs + SEG_CHUNK * CB;
+  float2* ds = reinterpret_cast<float2*>(sm);
+  float* bs = sm + 2 * SEG_CHUNK * CB;
   float a2[SPL], S[SPL];
   const size_t at = (size_t)min(col, g.C - 1) * NP + sub * SPL;
 #pragma unroll
   for (int i = 0; i < SPL; ++i) { a2[i] = a.a2[at + i]; S[i] = 0.0f; }
-  scan_stage<SPL, LPC, false>(a, c, c0, dts, xs, bs, nullptr);
+  scan_stage<T, SPL, LPC, false>(a, c, c0, act, Kp, ds, bs, nullptr);
   __syncthreads();
   float sum = 0.0f;
-  for (int j = 0; j < c.y; ++j) {
-    const float dt = dts[j * CB + cl], dx = dt * xs[j * CB + cl];
-    const float* b = bs + j * NP + sub * SPL;
-    sum += dt;
+  for (int j0 = 0; j0 < c.y; j0 += 4) {                      // (tokens behind the chunk's change nothing)
+    float2 d[4];
+    float b[4][SPL];
 #pragma unroll
-    for (int i = 0; i < SPL; ++i) S[i] = fmaf(hw_exp2(dt * a2[i]), S[i], dx * b[i]);
+    for (int k = 0; k < 4; ++k) { d[k] = ds[(j0 + k) * CB + cl]; lds_read<SPL>(bs + (j0 + k) * NP + sub * SPL, b[k]); }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      sum += d[k].x;
+#pragma unroll
+      for (int i = 0; i < SPL; ++i) S[i] = fmaf(hw_exp2(d[k].x * a2[i]), S[i], d[k].y * b[k][i]);
+    }
   }
   if (col >= g.C) return;
   float* u = a.u + (size_t)ch * g.C * NP + at;
@@ -179,76 +242,139 @@ static __global__ __launch_bounds__(256) void k_scan_carry(ScanArgs a) {
   *sp = S;
 }
 
-// outputs -> act.  grid (chunks, ceil(max(C, Kp) / CB)), block 256, LDS scan_lds<SPL, LPC, true>()
+// the output of four channels: (y + D x) silu(z), in the place of x
+template <typename T>
+__device__ __forceinline__ void scan_put4(const ScanArgs& a, int r, int c, const float* y, T* act, int Kp) {
+  const float4 x = act_load4(act, r, c, Kp), D = *reinterpret_cast<const float4*>(a.D + c);
+  float z[4], v[4];
+  a.in.at4(r, a.g.oz + c, z);                                // (z is zero in channels C .. Cp - 1)
+  v[0] = fmaf(D.x, x.x, y[0]); v[1] = fmaf(D.y, x.y, y[1]); v[2] = fmaf(D.z, x.z, y[2]); v[3] = fmaf(D.w, x.w, y[3]);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] *= z[e] * f32_sigmoid(z[e]);
+  act_store4(act, r, c, Kp, v);
+}
+
+// grid (chunks, ceil(C / CB)), block 256, LDS scan_lds<SPL, LPC, true>()
 template <typename T, int SPL, int LPC>
-__global__ __launch_bounds__(256) void k_scan_out(ScanArgs a, T* __restrict__ out, int Kp) {
-  constexpr int CB = 256 / LPC, NP = SPL * LPC, QB = CB / 4;
+__global__ __launch_bounds__(256) void k_scan_out(ScanArgs a, T* __restrict__ act, int Kp) {
+  constexpr int CB = 256 / LPC, NP = SPL * LPC, QB = CB / 4, TT = SPL > 8 ? 2 : 4;      // tokens whose operands are read together
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const ScanGeom& g = a.g;
   const int ch = blockIdx.x, tid = threadIdx.x, cl = tid / LPC, sub = tid % LPC, c0 = blockIdx.y * CB, col = c0 + cl;
   if (ch >= a.nseg[1]) return;
   const int4 c = a.chunk[ch];
-  float *dts = sm, *xs = dts + SEG_CHUNK * CB, *bs = xs + SEG_CHUNK * CB, *cs = bs + SEG_CHUNK * NP;
-  if (c0 < g.C) {
-    float a2[SPL], S[SPL];
-    const size_t at = (size_t)min(col, g.C - 1) * NP + sub * SPL;
-    const float* u = a.u + (size_t)ch * g.C * NP + at;
+  float2* ds = reinterpret_cast<float2*>(sm);
+  float *bs = sm + 2 * SEG_CHUNK * CB, *cs = bs + SEG_CHUNK * NP;
+  float a2[SPL], S[SPL];
+  const size_t at = (size_t)min(col, g.C - 1) * NP + sub * SPL;
+  const float* u = a.u + (size_t)ch * g.C * NP + at;
 #pragma unroll
-    for (int i = 0; i < SPL; ++i) { a2[i] = a.a2[at + i]; S[i] = u[i]; }
-    const float D = a.D[min(col, g.C - 1)];
-    scan_stage<SPL, LPC, true>(a, c, c0, dts, xs, bs, cs);
-    __syncthreads();
-    for (int j = 0; j < c.y; ++j) {
-      const float dt = dts[j * CB + cl], x = xs[j * CB + cl], dx = dt * x;
-      const float *b = bs + j * NP + sub * SPL, *cc = cs + j * NP + sub * SPL;
-      float y = 0.0f;
+  for (int i = 0; i < SPL; ++i) { a2[i] = a.a2[at + i]; S[i] = u[i]; }
+  scan_stage<T, SPL, LPC, true>(a, c, c0, act, Kp, ds, bs, cs);
+  __syncthreads();
+  for (int j0 = 0; j0 < c.y; j0 += TT) {
+    float2 d[TT];
+    float b[TT][SPL], cc[TT][SPL], y[TT];
+#pragma unroll
+    for (int k = 0; k < TT; ++k) { d[k] = ds[(j0 + k) * CB + cl]; lds_read<SPL>(bs + (j0 + k) * NP + sub * SPL, b[k]); lds_read<SPL>(cs + (j0 + k) * NP + sub * SPL, cc[k]); }
+#pragma unroll
+    for (int k = 0; k < TT; ++k) {
+      y[k] = 0.0f;
 #pragma unroll
       for (int i = 0; i < SPL; ++i) {
-        S[i] = fmaf(hw_exp2(dt * a2[i]), S[i], dx * b[i]);
-        y = fmaf(S[i], cc[i], y);
+        S[i] = fmaf(hw_exp2(d[k].x * a2[i]), S[i], d[k].y * b[k][i]);
+        y[k] = fmaf(S[i], cc[k][i], y[k]);
       }
-      y = lanes_sum<LPC>(y);
-      if (sub == 0) dts[j * CB + cl] = fmaf(D, x, y);          // (in the place of its step size, which only this channel's lanes read)
     }
-    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < TT; ++k) {
+      const float v = lanes_sum<LPC>(y[k]);
+      if (sub == 0) ds[(j0 + k) * CB + cl].x = v;              // (in the place of the step size, which only this channel's lanes read)
+    }
   }
+  __syncthreads();
   for (int i = tid; i < c.y * QB; i += 256) {
-    const int j = i / QB, q = i % QB * 4, col4 = c0 + q;
-    if (col4 >= Kp) continue;
-    float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-    if (col4 < g.C) {
-      const float4 y = *reinterpret_cast<const float4*>(dts + j * CB + q);
-      float z[4];
-      a.in.at4(c.x + j, g.oz + col4, z);
-      v[0] = y.x * z[0] * f32_sigmoid(z[0]); v[1] = y.y * z[1] * f32_sigmoid(z[1]); v[2] = y.z * z[2] * f32_sigmoid(z[2]); v[3] = y.w * z[3] * f32_sigmoid(z[3]);
-    }
-    act_store4(out, c.x + j, col4, Kp, v);
+    const int j = i / QB, q = i % QB * 4;
+    if (c0 + q >= g.Cp) continue;
+    const float4* p = reinterpret_cast<const float4*>(ds + j * CB + q);
+    const float y[4] = {p[0].x, p[0].z, p[1].x, p[1].z};
+    scan_put4(a, c.x + j, c0 + q, y, act, Kp);
   }
 }
 
-// Decode: four states per lane, LPC = Np / 4 lanes per channel.  grid (R, ceil(max(C, Kp) / (256 / LPC))), block 256.
-template <typename T, int LPC>
-__global__ __launch_bounds__(256) void k_scan_step(ScanArgs a, const int32_t* __restrict__ row_active, const int32_t* __restrict__ row_slot, const int32_t* __restrict__ row_pos,
-                                                   T* __restrict__ out, int Kp) {
-  constexpr int NP = 4 * LPC;
+// Decode: four states per lane, LPC = Np / 4 lanes per channel; CH (1 or 4) channels per group of lanes, CB = 256 / LPC apart, their states requested together.
+// CH 4: lane i of every four takes the step size of the group's channel i.  OWN (CH 1): the third projection happens here, dtw [C][rankp] with rankp a
+// multiple of 8; t in LDS.  grid (R, ceil(C / (CH CB))), block 256, LDS OWN ? rankp floats : 0.
+template <typename T, int LPC, int CH, bool OWN>
+__global__ __launch_bounds__(256) void k_scan_step(ScanArgs a, const T* __restrict__ dtw, int rankp, const float* __restrict__ dtb, const int32_t* __restrict__ row_active,
+                                                   const int32_t* __restrict__ row_slot, const int32_t* __restrict__ row_pos, T* __restrict__ act, int Kp) {
+  static_assert(CH == 1 || (CH == 4 && !OWN), "one channel per group of lanes, or one per lane of every four");
+  constexpr int NP = 4 * LPC, CB = 256 / LPC;
+  extern __shared__ __attribute__((aligned(16))) float ts[];
+  __shared__ __attribute__((aligned(16))) float ys[CH * CB];
   const ScanGeom& g = a.g;
-  const int r = blockIdx.x, tid = threadIdx.x, sub = tid % LPC, col = blockIdx.y * (256 / LPC) + tid / LPC;
+  const int r = blockIdx.x, tid = threadIdx.x, sub = tid % LPC, cl = tid / LPC, c0 = blockIdx.y * CB * CH;
   const int active = row_active[r], grp = row_slot[r], pos = row_pos[r];      // (requested together)
   if (!active) return;
-  if (col >= g.C) {
-    if (col < Kp && sub == 0) act_store1(out, r, col, Kp, 0.0f);
-    return;
-  }
-  float4* sp = reinterpret_cast<float4*>(a.state + ((size_t)grp * g.C + col) * NP + sub * 4);
-  const float4 S0 = pos > 0 ? *sp : make_float4(0.0f, 0.0f, 0.0f, 0.0f), a2 = *reinterpret_cast<const float4*>(a.a2 + (size_t)col * NP + sub * 4);
-  const float x = a.x[(size_t)r * g.Cp + col], z = a.in.at(r, g.oz + col), D = a.D[col], dt = f32_softplus(a.dt.at(r, col)), dx = dt * x;
-  float b[4] = {0.0f, 0.0f, 0.0f, 0.0f}, c[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  float4 S[CH], a2[CH];
+  float* sp = a.state + ((size_t)grp * g.C) * NP + sub * 4;
 #pragma unroll
-  for (int e = 0; e < 4; ++e)
-    if (sub * 4 + e < g.N) { b[e] = a.low.at(r, g.ob + sub * 4 + e); c[e] = a.low.at(r, g.oc + sub * 4 + e); }
-  const float4 S = make_float4(fmaf(hw_exp2(dt * a2.x), S0.x, dx * b[0]), fmaf(hw_exp2(dt * a2.y), S0.y, dx * b[1]), fmaf(hw_exp2(dt * a2.z), S0.z, dx * b[2]),
-                               fmaf(hw_exp2(dt * a2.w), S0.w, dx * b[3]));
-  *sp = S;
-  const float y = lanes_sum<LPC>(fmaf(S.x, c[0], fmaf(S.y, c[1], fmaf(S.z, c[2], S.w * c[3]))));
-  if (sub == 0) act_store1(out, r, col, Kp, fmaf(D, x, y) * z * f32_sigmoid(z));
+  for (int i = 0; i < CH; ++i) {
+    const int col = min(c0 + i * CB + cl, g.C - 1);
+    S[i] = pos > 0 ? *reinterpret_cast<const float4*>(sp + (size_t)col * NP) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    a2[i] = *reinterpret_cast<const float4*>(a.a2 + (size_t)col * NP + sub * 4);
+  }
+  float b[4] = {0.0f, 0.0f, 0.0f, 0.0f}, c[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  if (sub * 4 < g.N) { a.low.at4(r, g.ob + sub * 4, b); a.low.at4(r, g.oc + sub * 4, c); }
+  const int mine = min(c0 + (CH == 4 ? (tid & 3) * CB : 0) + cl, g.C - 1);
+  const float x = to_f(act[act_at<T>(r, mine, Kp)]);
+  float z;
+  if constexpr (OWN) {
+    for (int k = tid * 4; k < rankp; k += 1024) {
+      float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+      if (k < g.rank) a.low.at4(r, k, v);                    // (columns behind the rank are zero up to the next multiple of 16)
+      *reinterpret_cast<float4*>(ts + k) = make_float4(v[0], v[1], v[2], v[3]);
+    }
+    const T* wp = dtw + (size_t)mine * rankp;
+    constexpr int B = 4;                                     // pieces of eight weights in flight
+    float w[B][8];
+#pragma unroll
+    for (int i = 0; i < B; ++i)
+      if ((i * LPC + sub) * 8 < rankp) load8(wp + (i * LPC + sub) * 8, w[i]);
+    __syncthreads();
+    z = 0.0f;
+    for (int k0 = 0; k0 < rankp; k0 += B * LPC * 8) {
+      if (k0 > 0) {
+#pragma unroll
+        for (int i = 0; i < B; ++i)
+          if (k0 + (i * LPC + sub) * 8 < rankp) load8(wp + k0 + (i * LPC + sub) * 8, w[i]);
+      }
+#pragma unroll
+      for (int i = 0; i < B; ++i) {
+        const int k = k0 + (i * LPC + sub) * 8;
+        if (k >= rankp) continue;
+        float t[8];
+        lds_read<8>(ts + k, t);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) z = fmaf(w[i][e], t[e], z);
+      }
+    }
+    z = lanes_sum<LPC>(z) + dtb[mine];
+  } else {
+    z = a.dt.at(r, mine);
+  }
+  const float dm = hw_softplus(z), dxm = dm * x;
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const int col = c0 + i * CB + cl;
+    float d = dm, dx = dxm;
+    if constexpr (CH == 4) { d = quad_lane(dm, i); dx = quad_lane(dxm, i); }
+    const float4 n = make_float4(fmaf(hw_exp2(d * a2[i].x), S[i].x, dx * b[0]), fmaf(hw_exp2(d * a2[i].y), S[i].y, dx * b[1]), fmaf(hw_exp2(d * a2[i].z), S[i].z, dx * b[2]),
+                                 fmaf(hw_exp2(d * a2[i].w), S[i].w, dx * b[3]));
+    if (col < g.C) *reinterpret_cast<float4*>(sp + (size_t)col * NP) = n;
+    const float y = lanes_sum<LPC>(fmaf(n.x, c[0], fmaf(n.y, c[1], fmaf(n.z, c[2], n.w * c[3]))));
+    if (sub == 0) ys[i * CB + cl] = y;
+  }
+  __syncthreads();                                           // (every lane has its x)
+  for (int q = tid * 4; q < CH * CB && c0 + q < g.Cp; q += 1024) scan_put4(a, r, c0 + q, ys + q, act, Kp);
 }

@@ -103,9 +103,9 @@ SIZES = {
     "suzulix-w4096": (_suzulix(4096, ("attention", "retention", "latent_attention"), 32, _square_moe(14336, 8, 2, 2048)),
                       dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=3, num_experts=8, num_experts_per_tok=2,
                            decoder_block="mixtral")),
-    "lulenex-w1024": (_lulenex(1024, 8, 5376, 512, 8), dict(base_emb_dim=1024, base_num_query_heads=8, base_num_kv_heads=8, base_mlp_dim=3584, base_num_decoder_layers=8)),
-    "lulenex-w2048": (_lulenex(2048, 16, 10752, 1024, 8), dict(base_emb_dim=2048, base_num_query_heads=16, base_num_kv_heads=16, base_mlp_dim=7168, base_num_decoder_layers=8)),
-    "lulenex-w4096": (_lulenex(4096, 32, 21504, 1024, 2), dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=2)),
+    "lulenex-w1024": (_lulenex(1024, 8, 5376, 2048, 8), dict(base_emb_dim=1024, base_num_query_heads=8, base_num_kv_heads=8, base_mlp_dim=3584, base_num_decoder_layers=8)),
+    "lulenex-w2048": (_lulenex(2048, 16, 10752, 2048, 8), dict(base_emb_dim=2048, base_num_query_heads=16, base_num_kv_heads=16, base_mlp_dim=7168, base_num_decoder_layers=8)),
+    "lulenex-w4096": (_lulenex(4096, 32, 21504, 2048, 2), dict(base_emb_dim=4096, base_num_query_heads=32, base_num_kv_heads=8, base_mlp_dim=14336, base_num_decoder_layers=2)),
 }
 
 
