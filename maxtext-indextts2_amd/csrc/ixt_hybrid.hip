@@ -608,7 +608,7 @@ int hybrid_init(ixt_ctx* c) {
       TRY(h_allocf(c, &L.tails, (size_t)c->G * 2 * (g.taps - 1) * g.Cp + 4));
       const int Nx = up_to(g.oc + g.N, 16), Nd = up_to(g.C, 16), Kd = up_to(g.rank, IXT_KALIGN);
       dotsz(m->Ep, up_to(g.oz + g.C, 16));
-      upd(part2, dot_floats(L.okp, Nx)); upd(part3, dot_floats(Kd, Nd));
+      upd(part2, std::max((size_t)R * Nx, (size_t)std::min(R, 256) * Nx * ((L.okp + IXT_CHAIN - 1) / IXT_CHAIN))); upd(part3, dot_floats(Kd, Nd));
       dotsz(L.okp, up_to(m->E, 16));
       upd(act_k, L.okp);
       upd(scan_t, (size_t)Rp * Kd); upd(scan_u, max_chunks * g.C * g.Np); upd(scan_s, max_chunks * g.Cp);
@@ -762,6 +762,20 @@ template <> int hdot<float>(ixt_ctx*, const float* x, const HMat& w, int R, floa
   LAUNCHCHK();
   *res = Slices{out, 1, (size_t)R * w.Np, w.Np};
   return IXT_OK;
+}
+// a product of few columns over a long K, some rows: whole-K blocks would leave most of the chip idle, so the reduction is cut into slices (128 x 160 outputs, K
+// 4096: 7 against 16 us; from 1024 rows on the whole form is as fast)
+template <typename T> static int hdot_narrow(ixt_ctx* c, const T* x, const HMat& w, int R, float* out, size_t out_floats, hipStream_t st, Slices* res) {
+  if constexpr (sizeof(T) == 2) {
+    const int chains = (w.Kp + IXT_CHAIN - 1) / IXT_CHAIN;
+    if (R >= c->ring_min_rows && R <= 256 && chains >= 4 && (w.Np + 31) / 32 * ((R + 63) / 64) <= 96 && (size_t)chains * R * w.Np <= out_floats) {
+      DotResult dr;
+      TRY(launch_dot(c, x, (const bf16_t*)w.w, w.Kp, w.Np, R, out, out_floats, false, st, &dr, true));
+      *res = Slices{out, dr.slices, dr.slice_stride, w.Np};
+      return IXT_OK;
+    }
+  }
+  return hdot<T>(c, x, w, R, out, out_floats, st, res);
 }
 // rows of several groups (heads, experts): 16-row block b uses the matrix of group rb_exp[b], `stride` elements apart.  group_rows: what every group's
 // rows are aligned to (128: the ring GEMM)
@@ -955,9 +969,10 @@ static int hybrid_mixer_scan(ixt_ctx* c, const HLayer& L, const HLayer& W, int R
   Slices in, low, dt{};
   TRY(hdot<T>(c, (const T*)m->xb, W.in, R, c->part, c->part_floats, st, &in));
   TRY(scan_conv<T>(c, L, W, in, R, st));
-  TRY(hdot<T>(c, (const T*)m->act, W.low, R, m->part2, m->part2_floats, st, &low));
+  TRY(hdot_narrow<T>(c, (const T*)m->act, W.low, R, m->part2, m->part2_floats, st, &low));
   if (!single || R > 32) {                                         // (few rows: k_scan_step works the step sizes out itself)
     TRY(scan_rank<T>(c, W, low, R, st));
+    low.n = 1;
     TRY(hdot<T>(c, (const T*)m->scan_t, W.dt, R, m->part3, m->part3_floats, st, &dt));
     dt.bias = W.dtb;
   }

@@ -46,14 +46,16 @@ template int retention_mix<float>(ixt_ctx*, const HLayer&, const HLayer&, const 
 template <typename T>
 int scan_conv(ixt_ctx* c, const HLayer& L, const HLayer& W, const Slices& in, int R, hipStream_t st) {
   HybridModel* m = c->hy;
-  const ScanConvArgs a{in, L.sg, W.cw, W.cb, m->row_seg, m->row_j, m->seg, L.tails};
-  hipLaunchKernelGGL((k_scan_conv<T>), dim3(R, (W.okp + 1023) / 1024), dim3(256), 0, st, a, (T*)m->act, W.okp);
+  const ScanConvArgs a{in, L.sg, W.cw, W.cb, m->row_seg, m->row_j, m->seg, L.tails, R};
+  const unsigned cols = (W.okp + 1023) / 1024;
+  if (R >= 256) hipLaunchKernelGGL((k_scan_conv<T, 4>), dim3((R + 3) / 4, cols), dim3(256), 0, st, a, (T*)m->act, W.okp);
+  else hipLaunchKernelGGL((k_scan_conv<T, 1>), dim3(R, cols), dim3(256), 0, st, a, (T*)m->act, W.okp);
   LAUNCHCHK();
   return IXT_OK;
 }
 template <typename T>
 int scan_rank(ixt_ctx* c, const HLayer& W, const Slices& low, int R, hipStream_t st) {
-  hipLaunchKernelGGL((k_scan_rank<T>), dim3(R), dim3(64), 0, st, low, W.sg.rank, (T*)c->hy->scan_t, W.dt.Kp);
+  hipLaunchKernelGGL((k_scan_rank<T>), dim3(R), dim3(64), 0, st, low, c->hy->part2, W.sg.rank, (T*)c->hy->scan_t, W.dt.Kp);
   LAUNCHCHK();
   return IXT_OK;
 }

@@ -42,63 +42,100 @@ __device__ __forceinline__ float4 act_load4(const bf16_t* b, int r, int k0, int 
 }
 __device__ __forceinline__ float4 act_load4(const float* b, int r, int k0, int Kp) { return *reinterpret_cast<const float4*>(b + (size_t)r * Kp + k0); }
 
-// Convolution, bias, silu.  Weights [taps][Cp], tails [group][2][taps - 1][Cp].  grid (R, ceil(Kp / 1024)), block 256: four channels per thread.
+// Convolution, bias, silu.  Weights [taps][Cp], tails [group][2][taps - 1][Cp].  grid (ceil(R / RB), ceil(Kp / 1024)), block 256: four channels of RB rows per
+// thread; rows in the middle of a run (taps 4, one slice) share their inputs.
 struct ScanConvArgs {
   Slices t; ScanGeom g; const float *w, *bias; const int32_t *row_seg, *row_j, *seg;
-  float* tails;
+  float* tails; int R;
 };
-template <typename T>
+__device__ __forceinline__ void fma4(const float4& x, const float4& w, float* v) { v[0] = fmaf(x.x, w.x, v[0]); v[1] = fmaf(x.y, w.y, v[1]); v[2] = fmaf(x.z, w.z, v[2]); v[3] = fmaf(x.w, w.w, v[3]); }
+// one row, any place in its run, any number of taps: v from the bias to the convolution; leaves what the next run needs
+__device__ __forceinline__ void scan_conv_row(const ScanConvArgs& a, int r, int s, int c, float* v) {
+  const ScanGeom& g = a.g;
+  const int32_t* sg = a.seg + (size_t)s * 8;
+  const int n = sg[1], start = sg[3], par = sg[4], j = a.row_j[r], taps = g.taps;
+  const size_t tsz = (size_t)(taps - 1) * g.Cp;
+  const float* tin = a.tails + ((size_t)sg[2] * 2 + par) * tsz + c;
+  float* tout = a.tails + ((size_t)sg[2] * 2 + (par ^ 1)) * tsz + c;
+  float x0[4];
+  a.t.at4(r, c, x0);
+  const float4 here = make_float4(x0[0], x0[1], x0[2], x0[3]);
+  fma4(here, *reinterpret_cast<const float4*>(a.w + (size_t)(taps - 1) * g.Cp + c), v);
+  for (int b0 = 1; b0 < taps; b0 += 3) {                     // three earlier inputs in flight: rows of the run, or what is kept of those before it (oldest first)
+    float4 x[3], w[3];
+#pragma unroll
+    for (int i = 0; i < 3; ++i) {
+      const int back = min(b0 + i, taps - 1);
+      const bool mine = j - back >= 0;
+      const float* src = mine ? a.t.p + (size_t)(r - back) * a.t.ncols + c : tin + (size_t)max(taps - 1 - (back - j), 0) * g.Cp;
+      x[i] = mine || start > 0 ? *reinterpret_cast<const float4*>(src) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+      w[i] = b0 + i < taps ? *reinterpret_cast<const float4*>(a.w + (size_t)(taps - 1 - back) * g.Cp + c) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+      if (mine)
+        for (int q = 1; q < a.t.n; ++q) {
+          const float4 u = *reinterpret_cast<const float4*>(src + (size_t)q * a.t.stride);
+          x[i].x += u.x; x[i].y += u.y; x[i].z += u.z; x[i].w += u.w;
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 3; ++i) fma4(x[i], w[i], v);
+  }
+  const int dist = n - 1 - j;                                // the last taps - 1 inputs stay
+  if (dist < taps - 1) *reinterpret_cast<float4*>(tout + (size_t)(taps - 2 - dist) * g.Cp) = here;
+  if (dist == 0)
+    for (int e = n; e < taps - 1; ++e)
+      *reinterpret_cast<float4*>(tout + (size_t)(taps - 2 - e) * g.Cp) = start > 0 ? *reinterpret_cast<const float4*>(tin + (size_t)(taps - 2 - (e - n)) * g.Cp) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+}
+template <typename T, int RB>
 __global__ __launch_bounds__(256) void k_scan_conv(ScanConvArgs a, T* __restrict__ out, int Kp) {
   const ScanGeom& g = a.g;
-  const int r = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 4, s = a.row_seg[r];
-  if (s < 0 || c >= Kp) return;
-  float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-  if (c < g.Cp) {                                            // (everything is zero in channels C .. Cp - 1)
-    const int32_t* sg = a.seg + (size_t)s * 8;
-    const int n = sg[1], start = sg[3], par = sg[4], j = a.row_j[r], taps = g.taps;
-    const size_t tsz = (size_t)(taps - 1) * g.Cp;
-    const float* tin = a.tails + ((size_t)sg[2] * 2 + par) * tsz + c;
-    float* tout = a.tails + ((size_t)sg[2] * 2 + (par ^ 1)) * tsz + c;
-    const float4 b = *reinterpret_cast<const float4*>(a.bias + c), w0 = *reinterpret_cast<const float4*>(a.w + (size_t)(taps - 1) * g.Cp + c);
-    float x0[4];
-    a.t.at4(r, c, x0);
-    v[0] = fmaf(x0[0], w0.x, b.x); v[1] = fmaf(x0[1], w0.y, b.y); v[2] = fmaf(x0[2], w0.z, b.z); v[3] = fmaf(x0[3], w0.w, b.w);
-    for (int b0 = 1; b0 < taps; b0 += 3) {                   // three earlier inputs in flight: rows of the run, or what is kept of those before it (oldest first)
-      float4 x[3], w[3];
-#pragma unroll
-      for (int i = 0; i < 3; ++i) {
-        const int back = min(b0 + i, taps - 1);
-        const bool mine = j - back >= 0;
-        const float* src = mine ? a.t.p + (size_t)(r - back) * a.t.ncols + c : tin + (size_t)max(taps - 1 - (back - j), 0) * g.Cp;
-        x[i] = mine || start > 0 ? *reinterpret_cast<const float4*>(src) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-        w[i] = b0 + i < taps ? *reinterpret_cast<const float4*>(a.w + (size_t)(taps - 1 - back) * g.Cp + c) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-        if (mine)
-          for (int q = 1; q < a.t.n; ++q) {
-            const float4 u = *reinterpret_cast<const float4*>(src + (size_t)q * a.t.stride);
-            x[i].x += u.x; x[i].y += u.y; x[i].z += u.z; x[i].w += u.w;
-          }
-      }
-#pragma unroll
-      for (int i = 0; i < 3; ++i) { v[0] = fmaf(x[i].x, w[i].x, v[0]); v[1] = fmaf(x[i].y, w[i].y, v[1]); v[2] = fmaf(x[i].z, w[i].z, v[2]); v[3] = fmaf(x[i].w, w[i].w, v[3]); }
-    }
-    const int dist = n - 1 - j;                              // what the next run needs: the last taps - 1 inputs
-    if (dist < taps - 1) *reinterpret_cast<float4*>(tout + (size_t)(taps - 2 - dist) * g.Cp) = make_float4(x0[0], x0[1], x0[2], x0[3]);
-    if (dist == 0)
-      for (int e = n; e < taps - 1; ++e)
-        *reinterpret_cast<float4*>(tout + (size_t)(taps - 2 - e) * g.Cp) = start > 0 ? *reinterpret_cast<const float4*>(tin + (size_t)(taps - 2 - (e - n)) * g.Cp) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+  const int r0 = blockIdx.x * RB, c = (blockIdx.y * 256 + threadIdx.x) * 4, nr = min(RB, a.R - r0);
+  if (c >= Kp) return;
+  float4 b = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+  const bool real = c < g.Cp;                                // (everything is zero in channels C .. Cp - 1, and there is nothing from Cp on)
+  if (real) b = *reinterpret_cast<const float4*>(a.bias + c);
+  auto put = [&](int r, float* v) {
 #pragma unroll
     for (int e = 0; e < 4; ++e) v[e] *= f32_sigmoid(v[e]);
+    act_store4(out, r, c, Kp, v);
+  };
+  if constexpr (RB > 1) {
+    const int s = a.row_seg[r0], j = a.row_j[r0];
+    if (nr == RB && real && g.taps == 4 && a.t.n == 1 && a.t.bias == nullptr && s >= 0 && j >= 3 && a.row_seg[r0 + RB - 1] == s && j + RB - 1 + 3 < a.seg[(size_t)s * 8 + 1]) {
+      float4 x[RB + 3], w[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) w[i] = *reinterpret_cast<const float4*>(a.w + (size_t)i * g.Cp + c);
+#pragma unroll
+      for (int i = 0; i < RB + 3; ++i) x[i] = *reinterpret_cast<const float4*>(a.t.p + (size_t)(r0 + i - 3) * a.t.ncols + c);
+#pragma unroll
+      for (int i = 0; i < RB; ++i) {
+        float v[4] = {b.x, b.y, b.z, b.w};
+        fma4(x[i + 3], w[3], v); fma4(x[i + 2], w[2], v); fma4(x[i + 1], w[1], v); fma4(x[i], w[0], v);      // (the order of scan_conv_row)
+        put(r0 + i, v);
+      }
+      return;
+    }
   }
-  act_store4(out, r, c, Kp, v);
+  for (int i = 0; i < nr; ++i) {
+    const int r = r0 + i, s = a.row_seg[r];
+    if (s < 0) continue;
+    float v[4] = {b.x, b.y, b.z, b.w};
+    if (real) scan_conv_row(a, r, s, c, v);
+    put(r, v);
+  }
 }
 
-// grid (R), block 64: four columns per thread and round
+// The second projection's slices are added up in the first one, too.  grid (R), block 64: four columns per thread and round.  first: the first slice
 template <typename T>
-__global__ __launch_bounds__(64) void k_scan_rank(Slices low, int rank, T* __restrict__ out, int Kp) {
+__global__ __launch_bounds__(64) void k_scan_rank(Slices low, float* __restrict__ first, int rank, T* __restrict__ out, int Kp) {
   const int r = blockIdx.x;
-  for (int k = threadIdx.x * 4; k < Kp; k += 256) {
+  for (int k = threadIdx.x * 4; k < max(Kp, low.n > 1 ? low.ncols : 0); k += 256) {
     float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-    if (k < rank) low.at4(r, k, v);                          // (columns behind the rank are zero up to the next multiple of 16)
+    if (k < low.ncols) low.template at4<8>(r, k, v);
+    if (k < low.ncols && low.n > 1) *reinterpret_cast<float4*>(first + (size_t)r * low.ncols + k) = make_float4(v[0], v[1], v[2], v[3]);
+    if (k >= Kp) continue;
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (k + e >= rank) v[e] = 0.0f;
     act_store4(out, r, k, Kp, v);
   }
 }
