@@ -1,7 +1,8 @@
 // ixt_hybrid_kernels.h -- kernels of decoders whose layers are listed one by one (ixt_config.layers): each layer has a sequence mixer (latent
 // attention over a paged latent cache, a gated delta rule with a recurrent state per page group, attention over keys and values per head:
-// ixt_heads_kernels.h, retention: ixt_retention_kernels.h), a feed-forward (a unit, dense or as a routed mixture) and norms in front of the sublayers,
-// behind them, or both; around a sublayer stands one residual sum, or several streams that mix (hyper-connections).
+// ixt_heads_kernels.h, retention and lightning attention: ixt_retention_kernels.h, selective scan: ixt_scan_kernels.h), a feed-forward (a unit, dense or as a routed mixture) and norms in front of the sublayers,
+// behind them, or both (in front of a mixer also a shift towards the token before); around a sublayer stands one residual sum, or several streams that mix
+// (hyper-connections).
 //
 // Every kernel is a template over T, the storage of activations and cached keys: bf16_t (activations in the dot kernels' fragment order, xidx) or
 // float (row-major; the 32-bit mode).  The residual stream, norms, rotations, scores, routers and the recurrence are f32 in both.
